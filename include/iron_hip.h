@@ -369,6 +369,75 @@ int iron_sample_advance_bf16(const uint16_t* logits, int n, const int* draws, in
  * iron/common/graph/carried.py:189-276, iron/operators/emit.py. */
 int iron_eval_words(int* words, int n_words, const int* exprs, int n, void* stream);
 
+/* ---- decoders with a float32 residual stream and layers that carry a state, over a batch of rows.
+ *
+ * `spans` is an int32 (slots, 4) table in device memory, 16-byte aligned: {row0, rows, start, unused}
+ * says that rows row0 .. row0 + rows - 1 of the batch are one sequence's tokens at positions start,
+ * start + 1, ...; an idle slot has no rows.  Spans must not overlap.  States are kept a slot; a span
+ * that starts at position 0 reads none, so a slot needs no clearing between sequences.
+ * `is_float`: void* activations are float instead of bf16 (a model that runs in 32 bits throughout). */
+
+/* x[i] = table[ids[i]] widened to float, for i < *valid (or rows); ids outside the table are skipped. */
+int iron_stream_embed(const uint16_t* table, const int* ids, float* x, int rows, int table_rows, int cols,
+                      const int* valid, void* stream);
+/* The stream's rows: with y, x += rmsnorm(y) * back_gain in place; with h, h = rmsnorm(x) * gain of the
+ * rows as they then stand.  Float throughout, h rounded once. */
+int iron_stream_rows(float* x, const void* y, const uint16_t* back_gain, const uint16_t* gain, void* h, int rows,
+                     int cols, float eps, int is_float, const int* valid, void* stream);
+/* out[slot] = the last row of the slot's span (left as it is for an idle slot). */
+int iron_span_tails(const float* x, const int* spans, float* out, int slots, int rows, int cols, void* stream);
+/* y = cap * tanh(x / cap) (cap 0: y = x) as float, and rounded to bf16 in rows of rounded_stride. */
+int iron_softcap(const void* x, float* y, uint16_t* rounded, int rows, int cols, int rounded_stride, float cap,
+                 int is_float, void* stream);
+/* y = act(gate) * up in float; activation 1 SiLU, 2 GELU (tanh form), 3 ReLU. */
+int iron_act_mul_f32(const float* gate, const float* up, float* y, int rows, int cols, int activation,
+                     const int* valid, void* stream);
+/* y = x w^T, x (rows, k), w (n, k) bf16, y (rows, n); float sums of float products, any sizes. */
+int iron_linear_any(const void* x, const uint16_t* w, void* y, int rows, int n, int k, int is_float,
+                    const int* valid, void* stream);
+
+/* mixed[m] = h + (before - h) * mu[m] for m < mixes, `before` the row ahead of h in its sequence (zeros
+ * ahead of the first; carry[slot] ahead of a span's first row).  carry (slots, cols) then holds each
+ * span's last row.  mu (mixes, cols), mixed (mixes, rows, cols). */
+int iron_token_shift(const void* h, const uint16_t* mu, void* carry, const int* spans, void* mixed, int slots,
+                     int rows, int cols, int mixes, int is_float, void* stream);
+/* out = -exp(w2 tanh(z) + w0): the logarithm of a decay per channel.  z (rows, rank), w2 (n, rank). */
+int iron_low_rank_decay(const void* z, const uint16_t* w2, const uint16_t* w0, float* out, int rows, int n,
+                        int rank, int is_float, const int* valid, void* stream);
+/* o_t = (S + diag(u) k_t v_t^T)^T r_t; S <- diag(exp(log_decay_t)) S + k_t v_t^T per head.
+ * r, k, v, log_decay, o (rows, heads * dim); u (heads, dim); state (slots, heads, dim, dim).  dim <= 256. */
+int iron_time_mix(const void* r, const void* k, const void* v, const float* log_decay, const uint16_t* u, float* state,
+                  const int* spans, float* o, int slots, int rows, int heads, int dim, int is_float, void* stream);
+/* x (rows, stride) = [q | k | v | .. b .. a ..]: a causal convolution of `taps` taps (channels, taps) a
+ * channel and SiLU on q, k (kv_heads x dim) and v (heads x vdim); q and k made unit vectors a head
+ * (eps 1e-6), q times dim^-1/2; decay = exp(-exp(a_log) softplus(a + dt_bias)), beta = sigmoid(b).
+ * out (rows, 2 kv_heads dim + heads vdim + 2 heads) = [q | k | v | decay | beta] in float.
+ * state (slots, taps - 1, channels): the inputs of the sequence's last taps - 1 tokens. */
+int iron_short_conv(const void* x, const uint16_t* taps_w, const uint16_t* a_log, const uint16_t* dt_bias, void* state,
+                    const int* spans, float* out, int slots, int rows, int stride, int heads, int kv_heads, int dim,
+                    int vdim, int taps, int b_at, int a_at, int is_float, void* stream);
+/* x as iron_short_conv leaves it.  S <- g S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q per value
+ * head (q/k head head / (heads / kv_heads)).  state (slots, heads, dim, vdim), o (rows, heads * vdim). */
+int iron_delta_rule(const float* x, float* state, const int* spans, float* o, int slots, int rows, int heads,
+                    int kv_heads, int dim, int vdim, void* stream);
+/* out = o / rms(o, one head) * gain * silu(gate) * scale; gain (dim) if gain_shared, else (heads * dim). */
+int iron_head_gate(const float* o, const void* gate, const uint16_t* gain, void* out, int rows, int heads, int dim,
+                   int gate_stride, int gate_at, int gain_shared, int out_stride, int out_at, float eps, float scale,
+                   int is_float, const int* valid, void* stream);
+/* x (rows, stride) = [q heads | k heads | v heads]; score = q . k * scale + bias[head][i - j] over
+ * 0 <= i - j < window, softmax, the values' sum times out_scale into columns out_at .. of out.
+ * bias (heads, window); keys (slots, ring, kv_heads, dim), values (.., vdim): position p in row p % ring,
+ * ring >= window; they receive the spans' last rows.  single: no span has more than one row. */
+int iron_mha_window(const void* x, void* keys, void* values, const float* bias, const int* spans, void* out, int slots,
+                    int rows, int stride, int heads, int kv_heads, int dim, int vdim, int window, int ring, float scale,
+                    int out_stride, int out_at, float out_scale, int single, int is_float, void* stream);
+/* iron_sample_bf16 for every slot that has rows: logits (slots, logits_stride), drawn at the position p
+ * of the span's last row by draw row slot * steps + p, recorded in record[slot * steps + p]; the span
+ * then becomes {slot, 1, p + 1}.  workspace: slots times iron_sample_workspace_bytes(n). */
+int iron_sample_slots_bf16(const uint16_t* logits, int n, int logits_stride, int* spans, int slots, int batch_rows,
+                           int steps, const int* draws, int k_max, void* workspace, int* token, int* record,
+                           void* stream);
+
 #ifdef __cplusplus
 }
 #endif

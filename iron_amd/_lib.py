@@ -88,6 +88,20 @@ SIGNATURES = {
     "iron_sample_bf16": (c_int, [_P, c_int, _P, c_int, _P, c_int, _P, _P, _P, c_int, _P, _P, _P]),
     "iron_sample_advance_bf16": (c_int, [_P, c_int, _P, c_int, _P, c_int, _P, _P, _P, c_int, _P, _P, _P, c_int, _P,
                                          c_int, _P]),
+    "iron_stream_embed": (c_int, [_P, _P, _P, c_int, c_int, c_int, _P, _P]),
+    "iron_stream_rows": (c_int, [_P, _P, _P, _P, _P, c_int, c_int, c_float, c_int, _P, _P]),
+    "iron_span_tails": (c_int, [_P, _P, _P, c_int, c_int, c_int, _P]),
+    "iron_softcap": (c_int, [_P, _P, _P, c_int, c_int, c_int, c_float, c_int, _P]),
+    "iron_act_mul_f32": (c_int, [_P, _P, _P, c_int, c_int, c_int, _P, _P]),
+    "iron_linear_any": (c_int, [_P, _P, _P, c_int, c_int, c_int, c_int, _P, _P]),
+    "iron_token_shift": (c_int, [_P] * 5 + [c_int] * 5 + [_P]),
+    "iron_low_rank_decay": (c_int, [_P] * 4 + [c_int] * 4 + [_P, _P]),
+    "iron_time_mix": (c_int, [_P] * 8 + [c_int] * 5 + [_P]),
+    "iron_short_conv": (c_int, [_P] * 7 + [c_int] * 11 + [_P]),
+    "iron_delta_rule": (c_int, [_P] * 4 + [c_int] * 6 + [_P]),
+    "iron_head_gate": (c_int, [_P] * 4 + [c_int] * 8 + [c_float, c_float, c_int, _P, _P]),
+    "iron_mha_window": (c_int, [_P] * 6 + [c_int] * 9 + [c_float, c_int, c_int, c_float, c_int, c_int, _P]),
+    "iron_sample_slots_bf16": (c_int, [_P, c_int, c_int, _P, c_int, c_int, c_int, _P, c_int, _P, _P, _P, _P]),
     "iron_eval_words": (c_int, [_P, c_int, _P, c_int, _P]),
 }
 

@@ -1,7 +1,10 @@
-"""The models wired from the shared decoder: Llama, Granite and Gemma 4's text decoder."""
+"""The models wired from the shared decoder: Llama, Granite, Gemma 4's text decoder and Pegilix."""
 
 from .gemma4 import Gemma4, Gemma4Config
 from .granite import Granite, GraniteConfig
 from .llama import Llama, LlamaConfig
+from .pegilix import Pegilix, PegilixConfig
+from .registry import ARCHITECTURES, load_model, model_class
 
-__all__ = ["Gemma4", "Gemma4Config", "Granite", "GraniteConfig", "Llama", "LlamaConfig"]
+__all__ = ["ARCHITECTURES", "Gemma4", "Gemma4Config", "Granite", "GraniteConfig", "Llama", "LlamaConfig", "Pegilix",
+           "PegilixConfig", "load_model", "model_class"]

@@ -76,7 +76,10 @@ def build(verbose: bool = False) -> Path:
     jobs = min(len(srcs), int(os.environ.get("MAX_JOBS", "8")))
     with ThreadPoolExecutor(max_workers=jobs) as pool:
         list(pool.map(compile_one, zip(srcs, objs)))
-    _run([hipcc, f"--offload-arch={ARCH}", "-shared", "-fPIC", "-o", str(LIB), *map(str, objs)])
+    # Linked beside its place and moved there whole: a build that is cut short leaves no half library.
+    part = objdir / LIB.name
+    _run([hipcc, f"--offload-arch={ARCH}", "-shared", "-fPIC", "-o", str(part), *map(str, objs)])
+    os.replace(part, LIB)
     return LIB
 
 

@@ -100,6 +100,11 @@ __device__ __forceinline__ float gelu_tanh_f32(float v) {
   return 0.5f * v * (1.0f + tanhf(inner));
 }
 
+// The gate of a gated feed-forward: 1 SiLU, 2 GELU (tanh form), 3 ReLU.
+__device__ __forceinline__ float gate_of(int kind, float g) {
+  return kind == 3 ? fmaxf(g, 0.f) : (kind == 2 ? gelu_tanh_f32(g) : silu_f32(g));
+}
+
 typedef unsigned int u32x4 __attribute__((ext_vector_type(4)));
 // 16-byte streaming load that does not displace reusable lines in the caches.
 __device__ __forceinline__ uint4 load_stream(const uint4* p) {

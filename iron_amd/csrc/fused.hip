@@ -105,7 +105,9 @@ __device__ __forceinline__ float dot_row(const uint4 (&w)[CH], const uint4 (&xp)
 }
 
 enum { EPI_NONE = 0, EPI_ADD = 1, EPI_SILU_MUL = 2, EPI_GELU_MUL = 3,     // 2 and 3: gate, up -> activation -> Mul
-       EPI_GELU_ROW = 4, EPI_SILU_ROW = 5 };                               // activation -> Mul by a given row
+       EPI_GELU_ROW = 4, EPI_SILU_ROW = 5,                                 // activation -> Mul by a given row
+       EPI_RELU_MUL = 6 };                                                 // as 2 and 3
+constexpr bool gated_epilogue(int e) { return e == EPI_SILU_MUL || e == EPI_GELU_MUL || e == EPI_RELU_MUL; }
 
 // y = E(W @ N(x)) for RPW rows a block; K <= CH * 2048.
 template <int RPW, int CH, bool NORM, int EPI>
@@ -116,7 +118,7 @@ __global__ __launch_bounds__(256) void gemv_fused_kernel(const bf16_t* __restric
                                                          const bf16_t* __restrict__ res,
                                                          float res_scale, bf16_t* __restrict__ y,
                                                          int M, int K) {
-  constexpr int MATS = (EPI == EPI_SILU_MUL || EPI == EPI_GELU_MUL) ? 2 : 1;
+  constexpr int MATS = gated_epilogue(EPI) ? 2 : 1;
   __shared__ float scratch4[4];
   __shared__ float part[4][MATS][RPW];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
@@ -155,10 +157,10 @@ __global__ __launch_bounds__(256) void gemv_fused_kernel(const bf16_t* __restric
       if (EPI == EPI_ADD) v = fmaf(res_scale, v, res_ahead);   // scale 1: the plain sum
       if (EPI == EPI_GELU_ROW || EPI == EPI_SILU_ROW)          // the activation's own rounding, then the product's
         v = round_bf16(EPI == EPI_SILU_ROW ? silu_f32(v) : gelu_tanh_f32(v)) * res_ahead;
-      if (EPI == EPI_SILU_MUL || EPI == EPI_GELU_MUL) {
+      if (gated_epilogue(EPI)) {
         const float u = round_bf16(part[0][MATS - 1][r] + part[1][MATS - 1][r] + part[2][MATS - 1][r] +
                                    part[3][MATS - 1][r]);
-        v = round_bf16(EPI == EPI_SILU_MUL ? silu_f32(v) : gelu_tanh_f32(v)) * u;
+        v = round_bf16(gate_of(EPI == EPI_RELU_MUL ? 3 : (EPI == EPI_GELU_MUL ? 2 : 1), v)) * u;
       }
       y[row] = f32_to_bf16(v);
     }
@@ -405,10 +407,10 @@ extern "C" int iron_gemv_fused_bf16(const uint16_t* W, const uint16_t* W2, const
                                     void* stream) {
   IRON_REQUIRE(W && x && y, "gemv_fused: null operand");
   IRON_REQUIRE(M > 0 && K > 0 && K % 8 == 0, "gemv_fused: M (%d) positive, K (%d) a positive multiple of 8", M, K);
-  IRON_REQUIRE(epilogue >= 0 && epilogue <= 5, "gemv_fused: epilogue (%d) is 0 to 5", epilogue);
+  IRON_REQUIRE(epilogue >= 0 && epilogue <= 6, "gemv_fused: epilogue (%d) is 0 to 6", epilogue);
   IRON_REQUIRE((epilogue != EPI_ADD && epilogue != EPI_GELU_ROW && epilogue != EPI_SILU_ROW) || residual,
                "gemv_fused: epilogues 1, 4 and 5 take a second row (the residual, the factor); none given");
-  IRON_REQUIRE((epilogue != EPI_SILU_MUL && epilogue != EPI_GELU_MUL) || W2, "gemv_fused: epilogues 2 and 3 take a second matrix; none given");
+  IRON_REQUIRE(!gated_epilogue(epilogue) || W2, "gemv_fused: epilogues 2, 3 and 6 take a second matrix; none given");
   IRON_REQUIRE((((uintptr_t)W | (uintptr_t)W2 | (uintptr_t)x | (uintptr_t)norm_w) & 15) == 0,
                "gemv_fused: operands must be 16-byte aligned");
   hipStream_t s = (hipStream_t)stream;
@@ -417,7 +419,7 @@ extern "C" int iron_gemv_fused_bf16(const uint16_t* W, const uint16_t* W2, const
   const int ch = K <= 2048 ? 1 : (K <= 4096 ? 2 : (K <= 8192 ? 4 : 8));
   // Rows a block takes (measured inside a decoder's step, on 256 CUs): two where the matrix is tall
   // and a row is short, and for 16 KB rows of a matrix of a few thousand; else one.
-  const bool pair_of_matrices = epilogue == EPI_SILU_MUL || epilogue == EPI_GELU_MUL;
+  const bool pair_of_matrices = gated_epilogue(epilogue);
   const bool plain_or_sum = epilogue == EPI_NONE || epilogue == EPI_ADD;
   const int rpw = pair_of_matrices ? (ch == 1 ? 2 : 1)
                   : (ch == 1 && M > 2048) ? (M >= 65536 ? 4 : 2)
@@ -436,6 +438,8 @@ extern "C" int iron_gemv_fused_bf16(const uint16_t* W, const uint16_t* W2, const
   IRON_FUSED(1, 4, false, 2) IRON_FUSED(1, 4, true, 2) IRON_FUSED(1, 8, false, 2) IRON_FUSED(1, 8, true, 2)
   IRON_FUSED(2, 1, false, 3) IRON_FUSED(2, 1, true, 3) IRON_FUSED(1, 2, false, 3) IRON_FUSED(1, 2, true, 3)
   IRON_FUSED(1, 4, false, 3) IRON_FUSED(1, 4, true, 3) IRON_FUSED(1, 8, false, 3) IRON_FUSED(1, 8, true, 3)
+  IRON_FUSED(2, 1, false, 6) IRON_FUSED(2, 1, true, 6) IRON_FUSED(1, 2, false, 6) IRON_FUSED(1, 2, true, 6)
+  IRON_FUSED(1, 4, false, 6) IRON_FUSED(1, 4, true, 6) IRON_FUSED(1, 8, false, 6) IRON_FUSED(1, 8, true, 6)
   IRON_FUSED(1, 1, false, 4) IRON_FUSED(1, 2, false, 4) IRON_FUSED(1, 4, false, 4) IRON_FUSED(1, 8, false, 4)
   IRON_FUSED(1, 1, false, 5) IRON_FUSED(1, 2, false, 5) IRON_FUSED(1, 4, false, 5) IRON_FUSED(1, 8, false, 5)
   IRON_FUSED(2, 1, false, 4) IRON_FUSED(2, 1, false, 5)

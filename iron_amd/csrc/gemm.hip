@@ -323,7 +323,6 @@ struct QkvTail {
   float* partial;
 };
 
-__device__ __forceinline__ float gate_of(int kind, float g) { return kind == 2 ? gelu_tanh_f32(g) : silu_f32(g); }
 
 // The k and v outputs moved to the chunk's rows of their caches.  The first row is held where the
 // rows under the bound still end inside the cache, whatever the word holds.
@@ -2208,7 +2207,7 @@ extern "C" int iron_gemm_residual_norm_bf16(const uint16_t* A, const uint16_t* B
 
 extern "C" int iron_gemm_gated_bf16(const uint16_t* A, const uint16_t* B, const uint16_t* G, uint16_t* C, int M,
                                     int N, int K, int activation, const int* valid, void* stream) {
-  IRON_REQUIRE(activation == 1 || activation == 2, "gemm_gated: activation (%d) is 1 (SiLU) or 2 (GELU, tanh form)",
+  IRON_REQUIRE(activation >= 1 && activation <= 3, "gemm_gated: activation (%d) is 1 (SiLU), 2 (GELU, tanh form) or 3 (ReLU)",
                activation);
   QkvTail tail{};
   tail.residual = G;
@@ -2220,7 +2219,7 @@ extern "C" int iron_gemm_gated_pair_bf16(const uint16_t* A, const uint16_t* Bg, 
                                          uint16_t* C, int M, int N, int K, int activation, const int* valid,
                                          void* stream) {
   IRON_REQUIRE(A && Bg && Bu && G && C, "gemm_gated_pair: null operand");
-  IRON_REQUIRE(activation == 1 || activation == 2, "gemm_gated_pair: activation (%d) is 1 (SiLU) or 2 (GELU, tanh form)",
+  IRON_REQUIRE(activation >= 1 && activation <= 3, "gemm_gated_pair: activation (%d) is 1 (SiLU), 2 (GELU, tanh form) or 3 (ReLU)",
                activation);
   IRON_REQUIRE(G != C, "gemm_gated_pair: the gate's product and the output are different buffers");
   IRON_REQUIRE(K <= (1 << 22) && N <= (1 << 22),

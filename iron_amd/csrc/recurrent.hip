@@ -1,0 +1,522 @@
+// Layers that carry a state from token to token, over a batch of rows whose spans say which rows are
+// which sequence's: the token shift, a low-rank decay, the time-mixing recurrence, the short causal
+// convolution, the gated delta rule, and the per-head norm and gate behind either recurrence.
+//
+// A slot's state belongs to the sequence in it.  A span that starts at position 0 reads no state (it
+// counts as zeros), so a slot needs no clearing between sequences.  States that the rows of a span
+// both read and replace are replaced by the thread that read them, after it read them.
+//
+// The recurrences run in float32 throughout.  The state of a head, (dim, columns), is split by
+// columns: a wave holds 4 columns, 16 lanes to a column, NI consecutive rows of it a lane, so that a
+// sum along dim is a sum in a lane and four steps of the DPP path.  A block (16 columns) stages 16
+// tokens of its head in LDS while the next 16 are on their way from memory.
+#include "../../include/iron_hip.h"
+#include "rows.h"
+
+namespace iron {
+
+constexpr int SCAN_TOKENS = 16;    // tokens staged at a time
+constexpr int SCAN_COLUMNS = 16;   // state columns a block holds
+
+__device__ __forceinline__ float sigmoid_exact(float z) { return 1.0f / (1.0f + expf(-z)); }
+__device__ __forceinline__ float softplus_exact(float z) { return z > 20.f ? z : log1pf(expf(z)); }
+
+// ------------------------------------------------------------- token shift
+// mixed[s] = h + (before - h) * mu[s], `before` the row ahead of h in its sequence.
+constexpr int SHIFT_TILE = 4;
+template <typename T, int VEC>
+__global__ __launch_bounds__(256) void token_shift_kernel(const T* __restrict__ h, const bf16_t* __restrict__ mu,
+                                                          T* __restrict__ carry, const int* __restrict__ spans,
+                                                          T* __restrict__ mixed, int rows, int cols, int mixes) {
+  const Span s = span_of(spans, blockIdx.y, rows);
+  const int first = blockIdx.x * SHIFT_TILE;
+  if (first >= s.rows) return;
+  const int last = min(s.rows, first + SHIFT_TILE);
+  T* held = carry + (size_t)blockIdx.y * cols;
+  for (int c = threadIdx.x * VEC; c < cols; c += 256 * VEC) {
+    float before[VEC];
+    if (first > 0) load_vec<VEC>(h + (size_t)(s.row0 + first - 1) * cols + c, before);
+    else if (s.start > 0) load_vec<VEC>(held + c, before);
+    else {
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) before[j] = 0.f;
+    }
+    if (first == 0) {   // the span's last row is what the next one starts from
+      float end[VEC];
+      load_vec<VEC>(h + (size_t)(s.row0 + s.rows - 1) * cols + c, end);
+      store_vec<VEC>(held + c, end);
+    }
+    for (int i = first; i < last; ++i) {
+      float now[VEC];
+      load_vec<VEC>(h + (size_t)(s.row0 + i) * cols + c, now);
+      for (int m = 0; m < mixes; ++m) {
+        float g[VEC];
+        load_vec<VEC>(mu + (size_t)m * cols + c, g);
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) g[j] = now[j] + (before[j] - now[j]) * g[j];
+        store_vec<VEC>(mixed + ((size_t)m * rows + s.row0 + i) * cols + c, g);
+      }
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) before[j] = now[j];
+    }
+  }
+}
+
+// --------------------------------------------------------- low-rank decay
+// log decay = -exp(W2 tanh(z) + w0), in float32: what the recurrence takes the exponential of.
+constexpr int DECAY_ROWS = 16;
+template <typename T>
+__global__ __launch_bounds__(256) void low_rank_decay_kernel(const T* __restrict__ z, const bf16_t* __restrict__ w2,
+                                                             const bf16_t* __restrict__ w0, float* __restrict__ out,
+                                                             int rows, int n, int rank, const int* __restrict__ valid) {
+  extern __shared__ float zt[];   // [rank][DECAY_ROWS]
+  const int live = bound_or(valid, rows);
+  const int r0 = blockIdx.y * DECAY_ROWS;
+  if (r0 >= live) return;
+  for (int i = threadIdx.x; i < rank * DECAY_ROWS; i += 256) {
+    const int r = i / rank, k = i - r * rank;
+    zt[k * DECAY_ROWS + r] = r0 + r < live ? tanhf(load_one(z + (size_t)(r0 + r) * rank + k)) : 0.f;
+  }
+  __syncthreads();
+  const int c = blockIdx.x * 256 + threadIdx.x;
+  if (c >= n) return;
+  float acc[DECAY_ROWS];
+  const float bias = bf16_to_f32(w0[c]);
+#pragma unroll
+  for (int r = 0; r < DECAY_ROWS; ++r) acc[r] = 0.f;
+  const bf16_t* wr = w2 + (size_t)c * rank;
+  for (int k = 0; k < rank; ++k) {
+    const float w = bf16_to_f32(wr[k]);
+#pragma unroll
+    for (int r = 0; r < DECAY_ROWS; ++r) acc[r] = fmaf(w, zt[k * DECAY_ROWS + r], acc[r]);
+  }
+#pragma unroll
+  for (int r = 0; r < DECAY_ROWS; ++r)
+    if (r0 + r < live) out[(size_t)(r0 + r) * n + c] = -expf(acc[r] + bias);
+}
+
+// -------------------------------------------------------------- time mixing
+template <int NI>
+__device__ __forceinline__ void lds_run(const float* __restrict__ p, float (&f)[NI]) {
+  if constexpr (NI % 4 == 0) {
+#pragma unroll
+    for (int e = 0; e < NI; e += 4) {
+      const float4 v = *reinterpret_cast<const float4*>(p + e);
+      f[e] = v.x; f[e + 1] = v.y; f[e + 2] = v.z; f[e + 3] = v.w;
+    }
+  } else {
+#pragma unroll
+    for (int e = 0; e < NI; ++e) f[e] = p[e];
+  }
+}
+
+// o_t = (S + diag(u) k v^T)^T r;  S <- diag(exp(log decay)) S + k v^T.  The bonus term is the scalar
+// sum(r u k) times v.
+template <typename T, int NI>
+__global__ __launch_bounds__(256) void time_mix_kernel(const T* __restrict__ r, const T* __restrict__ k, const T* __restrict__ v,
+                                                       const float* __restrict__ log_decay, const bf16_t* __restrict__ u,
+                                                       float* __restrict__ state, const int* __restrict__ spans,
+                                                       float* __restrict__ o, int rows, int heads, int dim) {
+  constexpr int WIDE = 16 * NI;
+  __shared__ __align__(16) float rs[SCAN_TOKENS][WIDE], ks[SCAN_TOKENS][WIDE], ds[SCAN_TOKENS][WIDE];
+  __shared__ float vs[SCAN_TOKENS][SCAN_COLUMNS], os[SCAN_TOKENS][SCAN_COLUMNS + 1], bonus[SCAN_TOKENS];
+  const int head = blockIdx.y, slot = blockIdx.z;
+  const Span s = span_of(spans, slot, rows);
+  if (s.rows == 0) return;
+  const int t = threadIdx.x, lane = t & 63, ig = t & 15, tok = t >> 4;   // staging: 16 threads a token
+  const int col = blockIdx.x * SCAN_COLUMNS + (t >> 4);                  // scanning: 16 lanes a column
+  const int width = heads * dim;
+  float* sp = state + ((size_t)slot * heads + head) * dim * dim;
+  float S[NI], gain[NI];
+#pragma unroll
+  for (int e = 0; e < NI; ++e) {
+    const int i = ig * NI + e;
+    S[e] = (s.start > 0 && i < dim && col < dim) ? sp[(size_t)i * dim + col] : 0.f;
+    gain[e] = i < dim ? bf16_to_f32(u[head * dim + i]) : 0.f;
+  }
+  float rn[NI], kn[NI], dn[NI], vn;
+  const int vcol = blockIdx.x * SCAN_COLUMNS + ig;
+  auto fetch = [&](int base) {
+    const bool live = base + tok < s.rows;
+    const size_t at = (size_t)(s.row0 + base + tok) * width + head * dim;
+#pragma unroll
+    for (int e = 0; e < NI; ++e) {
+      const int i = ig * NI + e;
+      const bool in = live && i < dim;
+      rn[e] = in ? load_one(r + at + i) : 0.f;
+      kn[e] = in ? load_one(k + at + i) : 0.f;
+      dn[e] = in ? log_decay[at + i] : 0.f;
+    }
+    vn = live && vcol < dim ? load_one(v + at + vcol) : 0.f;
+  };
+  fetch(0);
+  for (int base = 0; base < s.rows; base += SCAN_TOKENS) {
+    float b = 0.f;
+#pragma unroll
+    for (int e = 0; e < NI; ++e) {
+      rs[tok][ig * NI + e] = rn[e];
+      ks[tok][ig * NI + e] = kn[e];
+      ds[tok][ig * NI + e] = expf(dn[e]);
+      b = fmaf(rn[e] * gain[e], kn[e], b);
+    }
+    vs[tok][ig] = vn;
+    b = group16_sum(b);
+    if (ig == 0) bonus[tok] = b;
+    __syncthreads();
+    if (base + SCAN_TOKENS < s.rows) fetch(base + SCAN_TOKENS);
+    const int n = min(SCAN_TOKENS, (s.rows - base + 3) & ~3);   // past the last row: r, k, v 0, decay 1
+    for (int q = 0; q < n; q += 4) {
+#pragma unroll
+      for (int p = q; p < q + 4; ++p) {
+        float rr[NI], kk[NI], dd[NI];
+        lds_run<NI>(&rs[p][ig * NI], rr);
+        lds_run<NI>(&ks[p][ig * NI], kk);
+        lds_run<NI>(&ds[p][ig * NI], dd);
+        const float vv = vs[p][t >> 4];
+        float acc = 0.f;
+#pragma unroll
+        for (int e = 0; e < NI; ++e) {
+          acc = fmaf(rr[e], S[e], acc);
+          S[e] = fmaf(dd[e], S[e], kk[e] * vv);
+        }
+        acc = group16_sum(acc);
+        if (ig == 0) os[p][t >> 4] = fmaf(bonus[p], vv, acc);
+      }
+    }
+    __syncthreads();
+    if (base + tok < s.rows && vcol < dim) o[(size_t)(s.row0 + base + tok) * width + head * dim + vcol] = os[tok][ig];
+  }
+#pragma unroll
+  for (int e = 0; e < NI; ++e) {
+    const int i = ig * NI + e;
+    if (i < dim && col < dim) sp[(size_t)i * dim + col] = S[e];
+  }
+  (void)lane;
+}
+
+// ------------------------------------------------------- short convolution
+// The packed projection's rows [q | k | v | ... | b | a] -> float32 rows [unit q / sqrt(dim) | unit k |
+// v | decay | beta]: a causal convolution a channel and SiLU on q, k, v; unit q and k a head; the
+// step's decay exp(-exp(A_log) softplus(a + dt_bias)) and beta = sigmoid(b) a value head.
+struct ConvShape {
+  int rows, stride;                 // the projection's rows, and their length
+  int heads, kv_heads, dim, vdim;
+  int taps, b_at, a_at;             // columns of b and a in a projection row
+};
+constexpr int CONV_TILE = 16;
+template <typename T>
+__global__ __launch_bounds__(256) void short_conv_kernel(const T* __restrict__ x, const bf16_t* __restrict__ taps,
+                                                         const bf16_t* __restrict__ a_log, const bf16_t* __restrict__ dt_bias,
+                                                         T* __restrict__ state, const int* __restrict__ spans,
+                                                         float* __restrict__ out, ConvShape c) {
+  const int seg = blockIdx.y, slot = blockIdx.z, first = blockIdx.x * CONV_TILE;
+  const Span s = span_of(spans, slot, c.rows);
+  if (first >= s.rows) return;
+  const int last = min(s.rows, first + CONV_TILE);
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const int qk = c.kv_heads * c.dim, channels = 2 * qk + c.heads * c.vdim, wide = channels + 2 * c.heads;
+  if (seg == 2 * c.kv_heads + c.heads) {   // the heads' decays and betas
+    const int count = (last - first) * c.heads;
+    for (int i = threadIdx.x; i < count; i += 256) {
+      const int p = first + i / c.heads, h = i % c.heads;
+      const T* row = x + (size_t)(s.row0 + p) * c.stride;
+      float* to = out + (size_t)(s.row0 + p) * wide + channels;
+      const float a = load_one(row + c.a_at + h) + bf16_to_f32(dt_bias[h]);
+      to[h] = expf(-expf(bf16_to_f32(a_log[h])) * softplus_exact(a));
+      to[c.heads + h] = sigmoid_exact(load_one(row + c.b_at + h));
+    }
+    return;
+  }
+  const bool is_v = seg >= 2 * c.kv_heads;
+  const int len = is_v ? c.vdim : c.dim;
+  const int at = is_v ? 2 * qk + (seg - 2 * c.kv_heads) * c.vdim : seg * c.dim;
+  const int past = c.taps - 1;
+  T* held = state + (size_t)slot * past * channels;
+  // The input at place p of the span: a row of this call, the slot's state before it, zero before 0.
+  auto input = [&](int p, int ch) -> float {
+    if (p >= 0) return load_one(x + (size_t)(s.row0 + p) * c.stride + ch);
+    return s.start + p >= 0 ? load_one(held + (size_t)(past + p) * channels + ch) : 0.f;
+  };
+  for (int p = first + wave; p < last; p += 4) {
+    float f[4];
+    float ss = 0.f;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      const int j = lane + 64 * e;
+      f[e] = 0.f;
+      if (j < len) {
+        float acc = 0.f;
+        for (int i = 0; i < c.taps; ++i)
+          acc = fmaf(bf16_to_f32(taps[(size_t)(at + j) * c.taps + i]), input(p - past + i, at + j), acc);
+        f[e] = acc * sigmoid_exact(acc);
+        ss = fmaf(f[e], f[e], ss);
+      }
+    }
+    float scale = 1.f;
+    if (!is_v) {
+      scale = 1.0f / sqrtf(wave_sum(ss) + 1e-6f);
+      if (seg < c.kv_heads) scale *= 1.0f / sqrtf((float)c.dim);
+    }
+    float* to = out + (size_t)(s.row0 + p) * wide + at;
+#pragma unroll
+    for (int e = 0; e < 4; ++e)
+      if (lane + 64 * e < len) to[lane + 64 * e] = f[e] * scale;
+  }
+  if (first == 0) {   // no other block reads these channels' state; ascending, so a row is read before it is replaced
+    __syncthreads();
+    for (int j = threadIdx.x; j < len; j += 256)
+      for (int m = 0; m < past; ++m) store_one(held + (size_t)m * channels + at + j, input(s.rows - past + m, at + j));
+  }
+}
+
+// ----------------------------------------------------------- the delta rule
+// S <- g S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q.  Both sums along dim are taken of the old
+// state, so that they run side by side: o = g (S^T q) + (k . q) u.
+template <int NI>
+__global__ __launch_bounds__(256) void delta_rule_kernel(const float* __restrict__ x, float* __restrict__ state,
+                                                         const int* __restrict__ spans, float* __restrict__ o, int rows,
+                                                         int heads, int kv_heads, int dim, int vdim) {
+  constexpr int WIDE = 16 * NI;
+  __shared__ __align__(16) float qs[SCAN_TOKENS][WIDE], ks[SCAN_TOKENS][WIDE];
+  __shared__ float vs[SCAN_TOKENS][SCAN_COLUMNS], os[SCAN_TOKENS][SCAN_COLUMNS + 1];
+  __shared__ float gs[SCAN_TOKENS], bs[SCAN_TOKENS], kq[SCAN_TOKENS];
+  const int head = blockIdx.y, slot = blockIdx.z;
+  const Span s = span_of(spans, slot, rows);
+  if (s.rows == 0) return;
+  const int t = threadIdx.x, ig = t & 15, tok = t >> 4;
+  const int col = blockIdx.x * SCAN_COLUMNS + (t >> 4), vcol = blockIdx.x * SCAN_COLUMNS + ig;
+  const int qk = kv_heads * dim, channels = 2 * qk + heads * vdim, wide = channels + 2 * heads;
+  const int group = head / (heads / kv_heads);
+  float* sp = state + ((size_t)slot * heads + head) * dim * vdim;
+  float S[NI];
+#pragma unroll
+  for (int e = 0; e < NI; ++e) {
+    const int i = ig * NI + e;
+    S[e] = (s.start > 0 && i < dim && col < vdim) ? sp[(size_t)i * vdim + col] : 0.f;
+  }
+  float qn[NI], kn[NI], vn, gn, bn;
+  auto fetch = [&](int base) {
+    const bool live = base + tok < s.rows;
+    const float* row = x + (size_t)(s.row0 + base + tok) * wide;
+#pragma unroll
+    for (int e = 0; e < NI; ++e) {
+      const int i = ig * NI + e;
+      const bool in = live && i < dim;
+      qn[e] = in ? row[group * dim + i] : 0.f;
+      kn[e] = in ? row[qk + group * dim + i] : 0.f;
+    }
+    vn = live && vcol < vdim ? row[2 * qk + head * vdim + vcol] : 0.f;
+    gn = live ? row[channels + head] : 1.f;
+    bn = live ? row[channels + heads + head] : 0.f;
+  };
+  fetch(0);
+  for (int base = 0; base < s.rows; base += SCAN_TOKENS) {
+    float b = 0.f;
+#pragma unroll
+    for (int e = 0; e < NI; ++e) {
+      qs[tok][ig * NI + e] = qn[e];
+      ks[tok][ig * NI + e] = kn[e];
+      b = fmaf(qn[e], kn[e], b);
+    }
+    vs[tok][ig] = vn;
+    b = group16_sum(b);
+    if (ig == 0) {
+      kq[tok] = b;
+      gs[tok] = gn;
+      bs[tok] = bn;
+    }
+    __syncthreads();
+    if (base + SCAN_TOKENS < s.rows) fetch(base + SCAN_TOKENS);
+    const int n = min(SCAN_TOKENS, (s.rows - base + 3) & ~3);   // past the last row: q, k, v, beta 0, decay 1
+    for (int q = 0; q < n; q += 4) {
+#pragma unroll
+      for (int p = q; p < q + 4; ++p) {
+        float qq[NI], kk[NI];
+        lds_run<NI>(&qs[p][ig * NI], qq);
+        lds_run<NI>(&ks[p][ig * NI], kk);
+        const float g = gs[p];
+        float read = 0.f, out = 0.f;
+#pragma unroll
+        for (int e = 0; e < NI; ++e) {
+          read = fmaf(kk[e], S[e], read);
+          out = fmaf(qq[e], S[e], out);
+        }
+        read = group16_sum(read);
+        out = group16_sum(out);
+        const float u = bs[p] * fmaf(-g, read, vs[p][t >> 4]);
+#pragma unroll
+        for (int e = 0; e < NI; ++e) S[e] = fmaf(kk[e], u, g * S[e]);
+        if (ig == 0) os[p][t >> 4] = fmaf(kq[p], u, g * out);
+      }
+    }
+    __syncthreads();
+    if (base + tok < s.rows && vcol < vdim) o[(size_t)(s.row0 + base + tok) * (heads * vdim) + head * vdim + vcol] = os[tok][ig];
+  }
+#pragma unroll
+  for (int e = 0; e < NI; ++e) {
+    const int i = ig * NI + e;
+    if (i < dim && col < vdim) sp[(size_t)i * vdim + col] = S[e];
+  }
+}
+
+// ------------------------------------------------------- per-head norm, gate
+// out = (o / rms(o)) * gain * silu(gate) * scale, the mean over one head's columns: a wave a head's row.
+template <typename T>
+__global__ __launch_bounds__(256) void head_gate_kernel(const float* __restrict__ o, const T* __restrict__ gate,
+                                                        const bf16_t* __restrict__ gain, T* __restrict__ out, int rows,
+                                                        int heads, int dim, int gate_stride, int gate_at, int gain_shared,
+                                                        int out_stride, int out_at, float eps, float scale,
+                                                        const int* __restrict__ valid) {
+  const long item = (long)blockIdx.x * 4 + (threadIdx.x >> 6);
+  const int row = (int)(item / heads), head = (int)(item - (long)row * heads), lane = threadIdx.x & 63;
+  if (row >= bound_or(valid, rows)) return;
+  const float* src = o + ((size_t)row * heads + head) * dim;
+  float f[4], ss = 0.f;
+#pragma unroll
+  for (int e = 0; e < 4; ++e) {
+    f[e] = lane + 64 * e < dim ? src[lane + 64 * e] : 0.f;
+    ss = fmaf(f[e], f[e], ss);
+  }
+  const float inv = 1.0f / sqrtf(wave_sum(ss) / (float)dim + eps);
+#pragma unroll
+  for (int e = 0; e < 4; ++e) {
+    const int j = lane + 64 * e;
+    if (j >= dim) continue;
+    const float z = load_one(gate + (size_t)row * gate_stride + gate_at + head * dim + j);
+    const float g = bf16_to_f32(gain[gain_shared ? j : head * dim + j]);
+    store_one(out + (size_t)row * out_stride + out_at + head * dim + j, f[e] * inv * g * (z * sigmoid_exact(z)) * scale);
+  }
+}
+
+}  // namespace iron
+
+using namespace iron;
+
+static int per_lane(int dim) {   // state rows a lane holds: the power of two that covers dim over 16 lanes
+  int ni = 1;
+  while (16 * ni < dim) ni *= 2;
+  return ni;
+}
+
+#define IRON_SPANS_REQUIRE(name)                                                                       \
+  IRON_REQUIRE(spans && ((uintptr_t)spans & 15) == 0, name ": spans must be there and 16-byte aligned"); \
+  IRON_REQUIRE(slots > 0 && slots <= 65535 && rows > 0, name ": slots (%d) and rows (%d) must be positive", slots, rows)
+
+extern "C" int iron_token_shift(const void* h, const uint16_t* mu, void* carry, const int* spans, void* mixed, int slots,
+                                int rows, int cols, int mixes, int is_float, void* stream) {
+  IRON_REQUIRE(h && mu && carry && mixed, "token_shift: null operand");
+  IRON_SPANS_REQUIRE("token_shift");
+  IRON_REQUIRE(cols > 0 && mixes > 0, "token_shift: cols (%d) and mixes (%d) must be positive", cols, mixes);
+  const dim3 grid((rows + SHIFT_TILE - 1) / SHIFT_TILE, slots);
+  hipStream_t s = (hipStream_t)stream;
+  const bool vec = cols % 8 == 0 && (((uintptr_t)h | (uintptr_t)mu | (uintptr_t)carry | (uintptr_t)mixed) & 15) == 0;
+#define IRON_SHIFT(T, V) \
+  hipLaunchKernelGGL((token_shift_kernel<T, V>), grid, dim3(256), 0, s, (const T*)h, mu, (T*)carry, spans, (T*)mixed, rows, cols, mixes)
+  if (is_float) { if (vec) IRON_SHIFT(float, 8); else IRON_SHIFT(float, 1); }
+  else { if (vec) IRON_SHIFT(bf16_t, 8); else IRON_SHIFT(bf16_t, 1); }
+#undef IRON_SHIFT
+  IRON_LAUNCH_CHECK();
+}
+
+extern "C" int iron_low_rank_decay(const void* z, const uint16_t* w2, const uint16_t* w0, float* out, int rows, int n,
+                                   int rank, int is_float, const int* valid, void* stream) {
+  IRON_REQUIRE(z && w2 && w0 && out, "low_rank_decay: null operand");
+  IRON_REQUIRE(rows > 0 && n > 0 && rank > 0 && rank <= 512, "low_rank_decay: rows (%d), n (%d) positive, rank (%d) from 1 to 512",
+               rows, n, rank);
+  const dim3 grid((n + 255) / 256, (rows + DECAY_ROWS - 1) / DECAY_ROWS);
+  IRON_REQUIRE(grid.y <= 65535, "low_rank_decay: rows (%d) exceed the grid's y extent", rows);
+  const size_t lds = (size_t)rank * DECAY_ROWS * 4;
+  if (is_float)
+    hipLaunchKernelGGL((low_rank_decay_kernel<float>), grid, dim3(256), lds, (hipStream_t)stream, (const float*)z, w2, w0, out, rows, n, rank, valid);
+  else
+    hipLaunchKernelGGL((low_rank_decay_kernel<bf16_t>), grid, dim3(256), lds, (hipStream_t)stream, (const bf16_t*)z, w2, w0, out, rows, n, rank, valid);
+  IRON_LAUNCH_CHECK();
+}
+
+extern "C" int iron_time_mix(const void* r, const void* k, const void* v, const float* log_decay, const uint16_t* u,
+                             float* state, const int* spans, float* o, int slots, int rows, int heads, int dim, int is_float,
+                             void* stream) {
+  IRON_REQUIRE(r && k && v && log_decay && u && state && o, "time_mix: null operand");
+  IRON_SPANS_REQUIRE("time_mix");
+  IRON_REQUIRE(heads > 0 && heads <= 65535 && dim > 0 && dim <= 256, "time_mix: heads (%d) positive, dim (%d) from 1 to 256", heads, dim);
+  const dim3 grid((dim + SCAN_COLUMNS - 1) / SCAN_COLUMNS, heads, slots);
+  hipStream_t s = (hipStream_t)stream;
+#define IRON_TIME_MIX(T, NI)                                                                                              \
+  hipLaunchKernelGGL((time_mix_kernel<T, NI>), grid, dim3(256), 0, s, (const T*)r, (const T*)k, (const T*)v, log_decay, u, \
+                     state, spans, o, rows, heads, dim)
+#define IRON_TIME_MIX_NI(NI) { if (is_float) IRON_TIME_MIX(float, NI); else IRON_TIME_MIX(bf16_t, NI); break; }
+  switch (per_lane(dim)) {
+    case 1: IRON_TIME_MIX_NI(1)
+    case 2: IRON_TIME_MIX_NI(2)
+    case 4: IRON_TIME_MIX_NI(4)
+    case 8: IRON_TIME_MIX_NI(8)
+    default: IRON_TIME_MIX_NI(16)
+  }
+#undef IRON_TIME_MIX_NI
+#undef IRON_TIME_MIX
+  IRON_LAUNCH_CHECK();
+}
+
+extern "C" int iron_short_conv(const void* x, const uint16_t* taps_w, const uint16_t* a_log, const uint16_t* dt_bias,
+                               void* state, const int* spans, float* out, int slots, int rows, int stride, int heads,
+                               int kv_heads, int dim, int vdim, int taps, int b_at, int a_at, int is_float, void* stream) {
+  IRON_REQUIRE(x && taps_w && a_log && dt_bias && out && (state || taps == 1), "short_conv: null operand");
+  IRON_SPANS_REQUIRE("short_conv");
+  IRON_REQUIRE(heads > 0 && kv_heads > 0 && heads % kv_heads == 0, "short_conv: kv_heads (%d) must divide heads (%d)", kv_heads, heads);
+  IRON_REQUIRE(dim > 0 && dim <= 256 && vdim > 0 && vdim <= 256, "short_conv: dim (%d) and vdim (%d) from 1 to 256", dim, vdim);
+  IRON_REQUIRE(taps >= 1 && taps <= CONV_TILE + 1, "short_conv: taps (%d) from 1 to %d", taps, CONV_TILE + 1);
+  const int channels = 2 * kv_heads * dim + heads * vdim;
+  IRON_REQUIRE(b_at >= channels && a_at >= channels && b_at + heads <= stride && a_at + heads <= stride,
+               "short_conv: b (%d) and a (%d) lie behind q, k, v (%d) in a row of %d", b_at, a_at, channels, stride);
+  const ConvShape c{rows, stride, heads, kv_heads, dim, vdim, taps, b_at, a_at};
+  const dim3 grid((rows + CONV_TILE - 1) / CONV_TILE, 2 * kv_heads + heads + 1, slots);
+  IRON_REQUIRE(grid.y <= 65535, "short_conv: %d heads exceed the grid's y extent", heads);
+  if (is_float)
+    hipLaunchKernelGGL((short_conv_kernel<float>), grid, dim3(256), 0, (hipStream_t)stream, (const float*)x, taps_w, a_log, dt_bias, (float*)state, spans, out, c);
+  else
+    hipLaunchKernelGGL((short_conv_kernel<bf16_t>), grid, dim3(256), 0, (hipStream_t)stream, (const bf16_t*)x, taps_w, a_log, dt_bias, (bf16_t*)state, spans, out, c);
+  IRON_LAUNCH_CHECK();
+}
+
+extern "C" int iron_delta_rule(const float* x, float* state, const int* spans, float* o, int slots, int rows, int heads,
+                               int kv_heads, int dim, int vdim, void* stream) {
+  IRON_REQUIRE(x && state && o, "delta_rule: null operand");
+  IRON_SPANS_REQUIRE("delta_rule");
+  IRON_REQUIRE(heads > 0 && heads <= 65535 && kv_heads > 0 && heads % kv_heads == 0, "delta_rule: kv_heads (%d) must divide heads (%d)",
+               kv_heads, heads);
+  IRON_REQUIRE(dim > 0 && dim <= 256 && vdim > 0, "delta_rule: dim (%d) from 1 to 256, vdim (%d) positive", dim, vdim);
+  const dim3 grid((vdim + SCAN_COLUMNS - 1) / SCAN_COLUMNS, heads, slots);
+#define IRON_DELTA(NI)                                                                                                     \
+  {                                                                                                                        \
+    hipLaunchKernelGGL((delta_rule_kernel<NI>), grid, dim3(256), 0, (hipStream_t)stream, x, state, spans, o, rows, heads, \
+                       kv_heads, dim, vdim);                                                                               \
+    break;                                                                                                                 \
+  }
+  switch (per_lane(dim)) {
+    case 1: IRON_DELTA(1)
+    case 2: IRON_DELTA(2)
+    case 4: IRON_DELTA(4)
+    case 8: IRON_DELTA(8)
+    default: IRON_DELTA(16)
+  }
+#undef IRON_DELTA
+  IRON_LAUNCH_CHECK();
+}
+
+extern "C" int iron_head_gate(const float* o, const void* gate, const uint16_t* gain, void* out, int rows, int heads, int dim,
+                              int gate_stride, int gate_at, int gain_shared, int out_stride, int out_at, float eps,
+                              float scale, int is_float, const int* valid, void* stream) {
+  IRON_REQUIRE(o && gate && gain && out, "head_gate: null operand");
+  IRON_REQUIRE(rows > 0 && heads > 0 && dim > 0 && dim <= 256, "head_gate: rows (%d), heads (%d) positive, dim (%d) from 1 to 256",
+               rows, heads, dim);
+  IRON_REQUIRE(gate_at >= 0 && gate_at + heads * dim <= gate_stride && out_at >= 0 && out_at + heads * dim <= out_stride,
+               "head_gate: %d columns from %d of a gate row of %d, from %d of an output row of %d", heads * dim, gate_at,
+               gate_stride, out_at, out_stride);
+  const long items = (long)rows * heads;
+  const dim3 grid((unsigned)((items + 3) / 4));
+  if (is_float)
+    hipLaunchKernelGGL((head_gate_kernel<float>), grid, dim3(256), 0, (hipStream_t)stream, o, (const float*)gate, gain, (float*)out, rows, heads, dim, gate_stride, gate_at, gain_shared, out_stride, out_at, eps, scale, valid);
+  else
+    hipLaunchKernelGGL((head_gate_kernel<bf16_t>), grid, dim3(256), 0, (hipStream_t)stream, o, (const bf16_t*)gate, gain, (bf16_t*)out, rows, heads, dim, gate_stride, gate_at, gain_shared, out_stride, out_at, eps, scale, valid);
+  IRON_LAUNCH_CHECK();
+}

@@ -1,0 +1,64 @@
+// Rows of either activation type -- bf16, or float where a model runs in 32 bits throughout -- read
+// and written as floats, and the spans that say which rows belong to which sequence.
+#pragma once
+
+#include "common.h"
+
+namespace iron {
+
+// VEC consecutive elements: 8 at 16-byte alignment, or one.
+template <int VEC, typename T>
+__device__ __forceinline__ void load_vec(const T* __restrict__ p, float (&f)[VEC]) {
+  static_assert(VEC == 8 || VEC == 1, "eight elements or one");
+  if constexpr (VEC == 1) {
+    if constexpr (sizeof(T) == 2) f[0] = bf16_to_f32(*p);
+    else f[0] = *p;
+  } else if constexpr (sizeof(T) == 2) {
+    unpack8(*reinterpret_cast<const uint4*>(p), f);
+  } else {
+    const float4 a = reinterpret_cast<const float4*>(p)[0], b = reinterpret_cast<const float4*>(p)[1];
+    f[0] = a.x; f[1] = a.y; f[2] = a.z; f[3] = a.w;
+    f[4] = b.x; f[5] = b.y; f[6] = b.z; f[7] = b.w;
+  }
+}
+template <int VEC, typename T>
+__device__ __forceinline__ void store_vec(T* __restrict__ p, const float (&f)[VEC]) {
+  if constexpr (VEC == 1) {
+    if constexpr (sizeof(T) == 2) *p = f32_to_bf16(f[0]);
+    else *p = f[0];
+  } else if constexpr (sizeof(T) == 2) {
+    *reinterpret_cast<uint4*>(p) = pack8(f);
+  } else {
+    reinterpret_cast<float4*>(p)[0] = make_float4(f[0], f[1], f[2], f[3]);
+    reinterpret_cast<float4*>(p)[1] = make_float4(f[4], f[5], f[6], f[7]);
+  }
+}
+template <typename T>
+__device__ __forceinline__ float load_one(const T* __restrict__ p) {
+  float f[1];
+  load_vec<1>(p, f);
+  return f[0];
+}
+template <typename T>
+__device__ __forceinline__ void store_one(T* __restrict__ p, float v) {
+  const float f[1] = {v};
+  store_vec<1>(p, f);
+}
+
+// One sequence's part of a batch of rows: `rows` rows from `row0` on are its tokens at positions
+// `start`, `start + 1`, ...  The table has an entry a slot; an idle slot's has no rows.  Held inside
+// the batch here, so that no table can lead a kernel outside its buffers.
+struct Span {
+  int row0, rows, start;
+};
+__device__ __forceinline__ Span span_of(const int* __restrict__ spans, int slot, int batch_rows) {
+  const int4 v = reinterpret_cast<const int4*>(spans)[slot];
+  Span s;
+  s.row0 = v.x < 0 ? 0 : (v.x > batch_rows ? batch_rows : v.x);
+  const int left = batch_rows - s.row0;
+  s.rows = v.y < 0 ? 0 : (v.y > left ? left : v.y);
+  s.start = v.z < 0 ? 0 : v.z;
+  return s;
+}
+
+}  // namespace iron

@@ -7,7 +7,7 @@
 //   2. every entry at or over the floor goes to a list in LDS (about k of them), which is ranked.
 // Order everywhere: the larger logit first, of equals the lower index, NaN below every number.
 #include "../../include/iron_hip.h"
-#include "common.h"
+#include "rows.h"
 
 namespace iron {
 
@@ -200,19 +200,41 @@ __device__ double exp_det(double z) {
   return p * __longlong_as_double(scale);
 }
 
+// A batch's draw, where `spans` is given: a row of logits a slot (grid y), drawn at the position of the
+// slot's last row by that position's draw row, recorded there; the slot's span then becomes the one
+// row after it.  An idle slot draws nothing.
+struct SampleSlots {
+  int* spans;
+  int steps;                         // positions a slot's draw rows and record hold
+  int batch_rows;
+  int logits_stride, lists_stride;   // from a slot's logits, and its workspace (8-byte words), to the next one's
+};
+
 // lists: gridDim.x lists of SAMPLE_K_MAX entries, from each block's best, 0 past its last.
 __global__ __launch_bounds__(SAMPLE_THREADS) void sample_kernel(
     const bf16_t* __restrict__ logits, int n, const int* __restrict__ draws, int draws_words,
     const int* __restrict__ row, int k_max, uint64_t* workspace, int* __restrict__ token,
     int* __restrict__ record, int record_len, const int* __restrict__ at,
-    int* __restrict__ token_copy, int* words, int n_words, const int* __restrict__ exprs, int n_exprs) {
+    int* __restrict__ token_copy, int* words, int n_words, const int* __restrict__ exprs, int n_exprs, SampleSlots slots) {
   __shared__ SampleShared sh;
+  int place = 0;
+  Span span{0, 0, 0};
+  if (slots.spans != nullptr) {
+    span = span_of(slots.spans, blockIdx.y, slots.batch_rows);
+    if (span.rows == 0) return;
+    place = span.start + span.rows - 1;
+    if (place >= slots.steps) return;   // past the record: the host refuses such a call
+    place += blockIdx.y * slots.steps;
+    logits += (size_t)blockIdx.y * slots.logits_stride;
+    workspace += (size_t)blockIdx.y * slots.lists_stride;
+    token += blockIdx.y;
+  }
   unsigned int* ticket = reinterpret_cast<unsigned int*>(workspace);
   uint64_t* lists = workspace + SAMPLE_TICKET_BYTES / 8;
 
   // The draw row: {temperature (float32 bits), top-k, the 53-bit number's low and high word}.
   // A row outside the buffer, like a temperature that is not positive, is the greedy draw.
-  const int at_word = row ? *row : 0;
+  const int at_word = slots.spans != nullptr ? 4 * place : (row ? *row : 0);
   uint32_t w0 = 0, w1 = 0, w2 = 0, w3 = 0;
   if (draws != nullptr && at_word >= 0 && at_word + 4 <= draws_words) {
     w0 = (uint32_t)draws[at_word];
@@ -359,9 +381,12 @@ __global__ __launch_bounds__(SAMPLE_THREADS) void sample_kernel(
     *token = tok;
     if (token_copy != nullptr) *token_copy = tok;
     if (record != nullptr) {
-      const int where = at ? *at : 0;
+      const int where = slots.spans != nullptr ? place : (at ? *at : 0);
       if (where >= 0 && where < record_len) record[where] = tok;
     }
+    // (every other block of the slot has taken its ticket, so has read its span)
+    if (slots.spans != nullptr)
+      reinterpret_cast<int4*>(slots.spans)[blockIdx.y] = make_int4(blockIdx.y, 1, span.start + span.rows, 0);
     if (tail && !tail_in_lds) {   // more words or expressions than a wave holds: one by one, from memory
       for (int e = 0; e < n_exprs; ++e) {
         const int* x = exprs + 9 * e;
@@ -423,7 +448,7 @@ static int sample_launch(const uint16_t* logits, int n, const int* draws, int dr
                "sample: %d word expressions take the words (%d of them) and the table", n_exprs, n_words);
   hipLaunchKernelGGL(sample_kernel, dim3(sample_blocks(n)), dim3(SAMPLE_THREADS), 0, (hipStream_t)stream,
                      logits, n, draws, draws_words, row, k_max, (uint64_t*)workspace, token, record,
-                     record_len, at, token_copy, words, n_words, exprs, n_exprs);
+                     record_len, at, token_copy, words, n_words, exprs, n_exprs, SampleSlots{});
   IRON_LAUNCH_CHECK();
 }
 
@@ -440,4 +465,23 @@ extern "C" int iron_sample_advance_bf16(const uint16_t* logits, int n, const int
                                         const int* exprs, int n_exprs, void* stream) {
   return sample_launch(logits, n, draws, draws_words, row, k_max, workspace, token, record, record_len, at,
                        token_copy, words, n_words, exprs, n_exprs, stream);
+}
+
+extern "C" int iron_sample_slots_bf16(const uint16_t* logits, int n, int logits_stride, int* spans, int slots, int batch_rows,
+                                      int steps, const int* draws, int k_max, void* workspace, int* token, int* record,
+                                      void* stream) {
+  IRON_REQUIRE(logits && spans && draws && workspace && token && record, "sample_slots: null operand");
+  IRON_REQUIRE(n > 0 && sample_blocks(n) <= SAMPLE_BLOCKS_MAX, "sample_slots: n (%d) must be from 1 to %d", n,
+               SAMPLE_BLOCKS_MAX * SAMPLE_SHARE);
+  IRON_REQUIRE(slots > 0 && slots <= 65535 && batch_rows > 0 && steps > 0 && (long)slots * steps < (1L << 29),
+               "sample_slots: slots (%d), batch_rows (%d) and steps (%d) must be positive", slots, batch_rows, steps);
+  IRON_REQUIRE(k_max >= 1 && k_max <= SAMPLE_K_MAX, "sample_slots: k_max (%d) must be from 1 to %d", k_max, SAMPLE_K_MAX);
+  IRON_REQUIRE(logits_stride >= n && logits_stride % 8 == 0 && (((uintptr_t)logits | (uintptr_t)spans) & 15) == 0 &&
+                   ((uintptr_t)workspace & 7) == 0,
+               "sample_slots: 16-byte aligned rows of logits and spans, an 8-byte aligned workspace");
+  const SampleSlots per{spans, steps, batch_rows, logits_stride, (int)(iron_sample_workspace_bytes(n) / 8)};
+  hipLaunchKernelGGL(sample_kernel, dim3(sample_blocks(n), slots), dim3(SAMPLE_THREADS), 0, (hipStream_t)stream, logits, n,
+                     draws, slots * steps * 4, nullptr, k_max, (uint64_t*)workspace, token, record, slots * steps, nullptr,
+                     nullptr, nullptr, 0, nullptr, 0, per);
+  IRON_LAUNCH_CHECK();
 }

@@ -1,0 +1,294 @@
+// A decoder's residual stream held in float32: rows gathered from a bf16 table into it, a row's RMS
+// norm out of it, a block's normed output added to it, and the head's soft cap.  One rounding, to the
+// activation type, where a row leaves the stream; bandwidth bound, a block a row.
+#include "../../include/iron_hip.h"
+#include "rows.h"
+
+namespace iron {
+
+template <int VEC>
+__global__ __launch_bounds__(256) void stream_embed_kernel(const bf16_t* __restrict__ table, const int* __restrict__ ids,
+                                                           float* __restrict__ x, int rows, int table_rows, int cols,
+                                                           const int* __restrict__ valid) {
+  const int row = blockIdx.x;
+  if (row >= bound_or(valid, rows)) return;
+  const int id = ids[row];
+  if (id < 0 || id >= table_rows) return;
+  for (int c = threadIdx.x * VEC; c < cols; c += 256 * VEC) {
+    float f[VEC];
+    load_vec<VEC>(table + (size_t)id * cols + c, f);
+    store_vec<VEC>(x + (size_t)row * cols + c, f);
+  }
+}
+
+__device__ __forceinline__ float row_total(float v, float* part) {
+  v = wave_sum(v);
+  __syncthreads();   // the last total's readers are done
+  if ((threadIdx.x & 63) == 0) part[threadIdx.x >> 6] = v;
+  __syncthreads();
+  return part[0] + part[1] + part[2] + part[3];
+}
+
+// ADD: x += rmsnorm(y) * wb, in place.  NORM: h = rmsnorm(x) * w of the row as it then stands.
+// A thread holds its first CH pieces of the row between the passes and re-reads the rest.
+template <typename T, int VEC, int CH, bool ADD, bool NORM>
+__global__ __launch_bounds__(256) void stream_rows_kernel(float* __restrict__ x, const T* __restrict__ y,
+                                                          const bf16_t* __restrict__ wb, const bf16_t* __restrict__ w,
+                                                          T* __restrict__ h, int rows, int cols, float eps,
+                                                          const int* __restrict__ valid) {
+  __shared__ float part[4];
+  const int row = blockIdx.x, first = threadIdx.x * VEC;
+  constexpr int STEP = 256 * VEC;
+  float held[CH][VEC], gain[CH][VEC];
+  if (NORM) {
+#pragma unroll
+    for (int i = 0; i < CH; ++i)
+      if (first + i * STEP < cols) load_vec<VEC>(w + first + i * STEP, gain[i]);
+  }
+  if (row >= bound_or(valid, rows)) return;
+  float* xr = x + (size_t)row * cols;
+#pragma unroll
+  for (int i = 0; i < CH; ++i)
+    if (first + i * STEP < cols) load_vec<VEC>(xr + first + i * STEP, held[i]);
+
+  if (ADD) {
+    const T* yr = y + (size_t)row * cols;
+    float out[CH][VEC], back[CH][VEC];
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < CH; ++i)
+      if (first + i * STEP < cols) {
+        load_vec<VEC>(yr + first + i * STEP, out[i]);
+        load_vec<VEC>(wb + first + i * STEP, back[i]);
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) ss = fmaf(out[i][j], out[i][j], ss);
+      }
+    for (int c = first + CH * STEP; c < cols; c += STEP) {
+      float f[VEC];
+      load_vec<VEC>(yr + c, f);
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) ss = fmaf(f[j], f[j], ss);
+    }
+    const float inv = 1.0f / sqrtf(row_total(ss, part) / (float)cols + eps);
+#pragma unroll
+    for (int i = 0; i < CH; ++i)
+      if (first + i * STEP < cols) {
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) held[i][j] += out[i][j] * inv * back[i][j];
+        store_vec<VEC>(xr + first + i * STEP, held[i]);
+      }
+    for (int c = first + CH * STEP; c < cols; c += STEP) {
+      float f[VEC], b[VEC], s[VEC];
+      load_vec<VEC>(yr + c, f);
+      load_vec<VEC>(wb + c, b);
+      load_vec<VEC>(xr + c, s);
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) s[j] += f[j] * inv * b[j];
+      store_vec<VEC>(xr + c, s);
+    }
+  }
+  if (NORM) {
+    T* hr = h + (size_t)row * cols;
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < CH; ++i)
+      if (first + i * STEP < cols) {
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) ss = fmaf(held[i][j], held[i][j], ss);
+      }
+    for (int c = first + CH * STEP; c < cols; c += STEP) {   // this thread's own stores, if it made any
+      float f[VEC];
+      load_vec<VEC>(xr + c, f);
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) ss = fmaf(f[j], f[j], ss);
+    }
+    const float inv = 1.0f / sqrtf(row_total(ss, part) / (float)cols + eps);
+#pragma unroll
+    for (int i = 0; i < CH; ++i)
+      if (first + i * STEP < cols) {
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) held[i][j] = held[i][j] * inv * gain[i][j];
+        store_vec<VEC>(hr + first + i * STEP, held[i]);
+      }
+    for (int c = first + CH * STEP; c < cols; c += STEP) {
+      float f[VEC], g[VEC];
+      load_vec<VEC>(xr + c, f);
+      load_vec<VEC>(w + c, g);
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) f[j] = f[j] * inv * g[j];
+      store_vec<VEC>(hr + c, f);
+    }
+  }
+}
+
+// The last row of every span, gathered: out[slot] = x[row0 + rows - 1] (an idle slot's row is left).
+__global__ __launch_bounds__(256) void span_tails_kernel(const float* __restrict__ x, const int* __restrict__ spans,
+                                                         float* __restrict__ out, int rows, int cols) {
+  const Span s = span_of(spans, blockIdx.x, rows);
+  if (s.rows == 0) return;
+  const float* src = x + (size_t)(s.row0 + s.rows - 1) * cols;
+  for (int c = threadIdx.x; c < cols; c += 256) out[(size_t)blockIdx.x * cols + c] = src[c];
+}
+
+// cap * tanh(x / cap): in float32, and rounded to bf16 for the draw (rows of `stride`, whole 16-byte
+// pieces).  cap 0: no cap.
+template <typename T>
+__global__ __launch_bounds__(256) void softcap_kernel(const T* __restrict__ x, float* __restrict__ y,
+                                                      bf16_t* __restrict__ rounded, int cols, int stride, float cap) {
+  const size_t row = blockIdx.y;
+  for (int i = blockIdx.x * 256 + threadIdx.x; i < cols; i += gridDim.x * 256) {
+    float v = load_one(x + row * cols + i);
+    if (cap > 0.f) v = cap * tanhf(v / cap);
+    y[row * cols + i] = v;
+    rounded[row * stride + i] = f32_to_bf16(v);
+  }
+}
+
+// relu / silu / gelu (tanh form) of the gate, times up, in float32.
+__global__ __launch_bounds__(256) void act_mul_f32_kernel(const float* __restrict__ gate, const float* __restrict__ up,
+                                                          float* __restrict__ y, long n, int kind,
+                                                          const int* __restrict__ valid, int cols) {
+  if (valid != nullptr) n = min(n, (long)max(*valid, 0) * cols);
+  for (long i = (long)blockIdx.x * 256 + threadIdx.x; i < n; i += (long)gridDim.x * 256) {
+    const float g = gate[i];
+    const float a = kind == 3 ? fmaxf(g, 0.f) : (kind == 1 ? g / (1.f + expf(-g)) : gelu_tanh_f32(g));
+    y[i] = a * up[i];
+  }
+}
+
+// y = x W^T over float32 sums, one thread a 4 x 4 patch of a 64 x 64 tile, K through LDS: any sizes.
+// The 32-bit model's projections (T = float), and a bf16 row whose length is no whole 16-byte piece.
+template <typename T>
+__global__ __launch_bounds__(256) void linear_any_kernel(const T* __restrict__ x, const bf16_t* __restrict__ w,
+                                                         T* __restrict__ y, int rows, int n, int k,
+                                                         const int* __restrict__ valid) {
+  constexpr int BK = 16;
+  __shared__ float xs[BK][65], ws[BK][65];
+  const int live = bound_or(valid, rows);
+  const int r0 = blockIdx.y * 64, c0 = blockIdx.x * 64;
+  if (r0 >= live) return;
+  const int tr = threadIdx.x >> 4, tc = threadIdx.x & 15;
+  float acc[4][4] = {};
+  for (int k0 = 0; k0 < k; k0 += BK) {
+    for (int i = threadIdx.x; i < 64 * BK; i += 256) {
+      const int r = i / BK, kk = i % BK;
+      const bool in_k = k0 + kk < k;
+      xs[kk][r] = (in_k && r0 + r < live) ? load_one(x + (size_t)(r0 + r) * k + k0 + kk) : 0.f;
+      ws[kk][r] = (in_k && c0 + r < n) ? bf16_to_f32(w[(size_t)(c0 + r) * k + k0 + kk]) : 0.f;
+    }
+    __syncthreads();
+#pragma unroll
+    for (int kk = 0; kk < BK; ++kk) {
+      float a[4], b[4];
+#pragma unroll
+      for (int i = 0; i < 4; ++i) { a[i] = xs[kk][tr + 16 * i]; b[i] = ws[kk][tc + 16 * i]; }
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+#pragma unroll
+        for (int j = 0; j < 4; ++j) acc[i][j] = fmaf(a[i], b[j], acc[i][j]);
+    }
+    __syncthreads();
+  }
+#pragma unroll
+  for (int i = 0; i < 4; ++i)
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      const int r = r0 + tr + 16 * i, c = c0 + tc + 16 * j;
+      if (r < live && c < n) store_one(y + (size_t)r * n + c, acc[i][j]);
+    }
+}
+
+template <typename T, bool ADD, bool NORM>
+static int launch_stream_rows(float* x, const T* y, const bf16_t* wb, const bf16_t* w, T* h, int rows, int cols, float eps,
+                              const int* valid, hipStream_t s) {
+  const bool vec = cols % 8 == 0 && (((uintptr_t)x | (uintptr_t)y | (uintptr_t)wb | (uintptr_t)w | (uintptr_t)h) & 15) == 0;
+  if (vec && cols <= 2048)
+    hipLaunchKernelGGL((stream_rows_kernel<T, 8, 1, ADD, NORM>), dim3(rows), dim3(256), 0, s, x, y, wb, w, h, rows, cols, eps, valid);
+  else if (vec)
+    hipLaunchKernelGGL((stream_rows_kernel<T, 8, 2, ADD, NORM>), dim3(rows), dim3(256), 0, s, x, y, wb, w, h, rows, cols, eps, valid);
+  else
+    hipLaunchKernelGGL((stream_rows_kernel<T, 1, 4, ADD, NORM>), dim3(rows), dim3(256), 0, s, x, y, wb, w, h, rows, cols, eps, valid);
+  IRON_LAUNCH_CHECK();
+}
+
+static unsigned few_blocks(long n) {
+  const long b = (n + 255) / 256;
+  return (unsigned)(b > 4096 ? 4096 : b);
+}
+
+}  // namespace iron
+
+using namespace iron;
+
+extern "C" int iron_stream_embed(const uint16_t* table, const int* ids, float* x, int rows, int table_rows, int cols,
+                                 const int* valid, void* stream) {
+  IRON_REQUIRE(table && ids && x, "stream_embed: null operand");
+  IRON_REQUIRE(rows > 0 && table_rows > 0 && cols > 0, "stream_embed: rows (%d), table_rows (%d), cols (%d) must be positive",
+               rows, table_rows, cols);
+  if (cols % 8 == 0 && (((uintptr_t)table | (uintptr_t)x) & 15) == 0)
+    hipLaunchKernelGGL((stream_embed_kernel<8>), dim3(rows), dim3(256), 0, (hipStream_t)stream, table, ids, x, rows, table_rows, cols, valid);
+  else
+    hipLaunchKernelGGL((stream_embed_kernel<1>), dim3(rows), dim3(256), 0, (hipStream_t)stream, table, ids, x, rows, table_rows, cols, valid);
+  IRON_LAUNCH_CHECK();
+}
+
+extern "C" int iron_stream_rows(float* x, const void* y, const uint16_t* back_gain, const uint16_t* gain, void* h, int rows,
+                                int cols, float eps, int is_float, const int* valid, void* stream) {
+  IRON_REQUIRE(x && (h || y), "stream_rows: null operand");
+  IRON_REQUIRE((y == nullptr) == (back_gain == nullptr) && (h == nullptr) == (gain == nullptr),
+               "stream_rows: a gain for the row that is added, and one for the norm that is taken");
+  IRON_REQUIRE(rows > 0 && cols > 0, "stream_rows: rows (%d) and cols (%d) must be positive", rows, cols);
+  hipStream_t s = (hipStream_t)stream;
+#define IRON_STREAM_ROWS(T)                                                                                             \
+  if (y && h) return launch_stream_rows<T, true, true>(x, (const T*)y, back_gain, gain, (T*)h, rows, cols, eps, valid, s); \
+  if (y) return launch_stream_rows<T, true, false>(x, (const T*)y, back_gain, gain, (T*)h, rows, cols, eps, valid, s);     \
+  return launch_stream_rows<T, false, true>(x, (const T*)y, back_gain, gain, (T*)h, rows, cols, eps, valid, s);
+  if (is_float) { IRON_STREAM_ROWS(float) }
+  IRON_STREAM_ROWS(bf16_t)
+#undef IRON_STREAM_ROWS
+}
+
+extern "C" int iron_span_tails(const float* x, const int* spans, float* out, int slots, int rows, int cols, void* stream) {
+  IRON_REQUIRE(x && spans && out, "span_tails: null operand");
+  IRON_REQUIRE(((uintptr_t)spans & 15) == 0, "span_tails: spans must be 16-byte aligned");
+  IRON_REQUIRE(slots > 0 && rows > 0 && cols > 0, "span_tails: slots (%d), rows (%d), cols (%d) must be positive", slots, rows, cols);
+  hipLaunchKernelGGL(span_tails_kernel, dim3(slots), dim3(256), 0, (hipStream_t)stream, x, spans, out, rows, cols);
+  IRON_LAUNCH_CHECK();
+}
+
+extern "C" int iron_softcap(const void* x, float* y, uint16_t* rounded, int rows, int cols, int rounded_stride, float cap,
+                            int is_float, void* stream) {
+  IRON_REQUIRE(x && y && rounded, "softcap: null operand");
+  IRON_REQUIRE(rows > 0 && rows <= 65535 && cols > 0 && rounded_stride >= cols && cap >= 0.f,
+               "softcap: rows (%d) and cols (%d) must be positive, a rounded row (%d) no shorter, cap (%g) not negative", rows,
+               cols, rounded_stride, (double)cap);
+  const dim3 grid(few_blocks(cols), rows);
+  if (is_float)
+    hipLaunchKernelGGL((softcap_kernel<float>), grid, dim3(256), 0, (hipStream_t)stream, (const float*)x, y, rounded, cols, rounded_stride, cap);
+  else
+    hipLaunchKernelGGL((softcap_kernel<bf16_t>), grid, dim3(256), 0, (hipStream_t)stream, (const bf16_t*)x, y, rounded, cols, rounded_stride, cap);
+  IRON_LAUNCH_CHECK();
+}
+
+extern "C" int iron_act_mul_f32(const float* gate, const float* up, float* y, int rows, int cols, int activation,
+                                const int* valid, void* stream) {
+  IRON_REQUIRE(gate && up && y, "act_mul_f32: null operand");
+  IRON_REQUIRE(rows > 0 && cols > 0, "act_mul_f32: rows (%d) and cols (%d) must be positive", rows, cols);
+  IRON_REQUIRE(activation >= 1 && activation <= 3, "act_mul_f32: activation (%d) is 1 (SiLU), 2 (GELU, tanh form) or 3 (ReLU)", activation);
+  const long n = (long)rows * cols;
+  hipLaunchKernelGGL(act_mul_f32_kernel, dim3(few_blocks(n)), dim3(256), 0, (hipStream_t)stream, gate, up, y, n, activation, valid, cols);
+  IRON_LAUNCH_CHECK();
+}
+
+extern "C" int iron_linear_any(const void* x, const uint16_t* w, void* y, int rows, int n, int k, int is_float,
+                               const int* valid, void* stream) {
+  IRON_REQUIRE(x && w && y, "linear_any: null operand");
+  IRON_REQUIRE(rows > 0 && n > 0 && k > 0, "linear_any: rows (%d), n (%d), k (%d) must be positive", rows, n, k);
+  IRON_REQUIRE((rows + 63) / 64 <= 65535, "linear_any: rows (%d) exceed the grid's y extent", rows);
+  const dim3 grid((n + 63) / 64, (rows + 63) / 64);
+  if (is_float)
+    hipLaunchKernelGGL((linear_any_kernel<float>), grid, dim3(256), 0, (hipStream_t)stream, (const float*)x, w, (float*)y, rows, n, k, valid);
+  else
+    hipLaunchKernelGGL((linear_any_kernel<bf16_t>), grid, dim3(256), 0, (hipStream_t)stream, (const bf16_t*)x, w, (bf16_t*)y, rows, n, k, valid);
+  IRON_LAUNCH_CHECK();
+}

@@ -9,12 +9,15 @@ from __future__ import annotations
 
 import math
 
+from .bf16 import bfloat16
 from .common.declare import Precision
 from .operators.gemm import GEMM
 from .operators.gemv import GEMV
+from .operators.relu import ReLU
 from .operators.rms_norm import RMSNorm
 from .operators.rope import RoPE
 from .operators.silu import SiLU
+from .operators.stream import LinearAny
 
 BF16_EPS = 2.0**-7   # machine epsilon of bfloat16 (8 significand bits), the default norm epsilon
 
@@ -35,6 +38,9 @@ def linear(x, weight, bias=None, *, precision: Precision = Precision.HIGHEST, **
     if rank not in (1, 2):
         raise ValueError(f"linear(): x {tuple(x.shape)} is not (in,) or (rows, in)")
     rows = 1 if rank == 1 else x.shape[0]
+    if bias is None and rank == 2 and (x.dtype is not bfloat16 or x.shape[1] % 8):
+        # a model that runs in 32 bits throughout, or a row that is no whole number of 16-byte pieces
+        return LinearAny.step(x, weight, dtype=x.dtype)
     if rows > 1 and gemv:
         raise ValueError(f"linear(): {rows} rows take no GEMV {sorted(gemv)}")
     if rows == 1:
@@ -68,6 +74,11 @@ def rms_norm(x, normalized_shape, weight=None, eps: float | None = None):
 def silu(x):
     """``x * sigmoid(x)`` elementwise."""
     return SiLU.step(x)
+
+
+def relu(x):
+    """``max(x, 0)`` elementwise."""
+    return ReLU.step(x)
 
 
 def rope(x, angles):

@@ -14,6 +14,7 @@ import torch
 from ._lib import check, current_stream, lib, ptr
 
 BF16 = torch.bfloat16
+GATES = {"silu": 1, "gelu_tanh": 2, "relu": 3}   # a gated feed-forward's activation, by the C ABI's number
 
 
 def _dev(t, name, dtype=BF16):
@@ -106,9 +107,9 @@ def gemm_residual_norm(A, B, R, gain, C, Y, workspace, *, M, N, K, eps, residual
 def gemm_gated(A, B, G, C, *, M, N, K, activation="silu", valid=None):
     """``C = act(G) * (A @ B.T)`` over many rows, B stored ``(N, K)``; ``activation`` "silu" or
     "gelu_tanh"."""
-    kinds = {"silu": 1, "gelu_tanh": 2}
+    kinds = GATES
     if activation not in kinds:
-        raise ValueError(f"gemm_gated: activation {activation!r} is neither 'silu' nor 'gelu_tanh'")
+        raise ValueError(f"gemm_gated: activation {activation!r} is none of {sorted(kinds)}")
     _numel(_dev(A, "A"), M * K, "A")
     _numel(_dev(B, "B"), N * K, "B")
     _numel(_dev(G, "G"), M * N, "G")
@@ -119,9 +120,9 @@ def gemm_gated(A, B, G, C, *, M, N, K, activation="silu", valid=None):
 
 def gemm_gated_pair(A, Bg, Bu, G, C, *, M, N, K, activation="silu", valid=None):
     """``G = A @ Bg.T``, ``C = act(G) * (A @ Bu.T)`` over many rows in one launch (weights ``(N, K)``)."""
-    kinds = {"silu": 1, "gelu_tanh": 2}
+    kinds = GATES
     if activation not in kinds:
-        raise ValueError(f"gemm_gated_pair: activation {activation!r} is neither 'silu' nor 'gelu_tanh'")
+        raise ValueError(f"gemm_gated_pair: activation {activation!r} is none of {sorted(kinds)}")
     _numel(_dev(A, "A"), M * K, "A")
     _numel(_dev(Bg, "Bg"), N * K, "Bg")
     _numel(_dev(Bu, "Bu"), N * K, "Bu")
@@ -576,3 +577,178 @@ def eval_words(words, exprs, n=None):
     n = exprs.numel() // 9 if n is None else n  # nine words a record
     check(lib().iron_eval_words(ptr(words), words.numel(), ptr(exprs), n, current_stream()), "iron_eval_words")
 
+
+
+# ---- the float32 stream and the layers that carry a state (rows of a batch told apart by spans)
+
+
+def _act(t, n, name):
+    """An activation operand, bf16 or float32: its number of elements checked, and whether it is float."""
+    _dev(t, name, torch.float32 if t.dtype == torch.float32 else BF16)
+    _numel(t, n, name)
+    return t.dtype == torch.float32
+
+
+def _same_kind(is_float, **tensors):
+    for name, t in tensors.items():
+        if (t.dtype == torch.float32) != is_float:
+            raise TypeError(f"{name}: {t.dtype} beside {'float32' if is_float else 'bfloat16'} activations")
+
+
+def _f32(t, n, name):
+    _numel(_dev(t, name, torch.float32), n, name)
+
+
+def _bf16(t, n, name):
+    _numel(_dev(t, name), n, name)
+
+
+def _spans(t, slots):
+    _numel(_dev(t, "spans", torch.int32), 4 * slots, "spans")
+    return ptr(t)
+
+
+def stream_embed(table, ids, x, *, rows, table_rows, cols, valid=None):
+    _bf16(table, table_rows * cols, "table")
+    _numel(_dev(ids, "ids", torch.int32), rows, "ids")
+    _f32(x, rows * cols, "x")
+    check(lib().iron_stream_embed(ptr(table), ptr(ids), ptr(x), rows, table_rows, cols, ptr(_word(valid, "valid")),
+                                  current_stream()), "iron_stream_embed")
+
+
+def stream_rows(x, *, rows, cols, eps, y=None, back_gain=None, h=None, gain=None, valid=None):
+    """``x += rmsnorm(y) * back_gain`` (with ``y``) and ``h = rmsnorm(x) * gain`` (with ``h``), one launch."""
+    _f32(x, rows * cols, "x")
+    is_float = False
+    for t, g, name in ((y, back_gain, "y"), (h, gain, "h")):
+        if t is not None:
+            is_float = _act(t, rows * cols, name)
+            _bf16(g, cols, f"the gain of {name}")
+    if y is not None and h is not None:
+        _same_kind(is_float, y=y)
+    check(lib().iron_stream_rows(ptr(x), ptr(y), ptr(back_gain), ptr(gain), ptr(h), rows, cols, float(eps), int(is_float),
+                                 ptr(_word(valid, "valid")), current_stream()), "iron_stream_rows")
+
+
+def span_tails(x, spans, out, *, slots, rows, cols):
+    _f32(x, rows * cols, "x")
+    _f32(out, slots * cols, "out")
+    check(lib().iron_span_tails(ptr(x), _spans(spans, slots), ptr(out), slots, rows, cols, current_stream()),
+          "iron_span_tails")
+
+
+def softcap(x, y, rounded, *, rows, cols, stride, cap):
+    is_float = _act(x, rows * cols, "x")
+    _f32(y, rows * cols, "y")
+    _bf16(rounded, rows * stride, "rounded")
+    check(lib().iron_softcap(ptr(x), ptr(y), ptr(rounded), rows, cols, stride, float(cap), int(is_float),
+                             current_stream()), "iron_softcap")
+
+
+def act_mul_f32(gate, up, y, *, rows, cols, activation, valid=None):
+    for t, name in ((gate, "gate"), (up, "up"), (y, "y")):
+        _f32(t, rows * cols, name)
+    check(lib().iron_act_mul_f32(ptr(gate), ptr(up), ptr(y), rows, cols, GATES[activation], ptr(_word(valid, "valid")),
+                                 current_stream()), "iron_act_mul_f32")
+
+
+def linear_any(x, w, y, *, rows, n, k, valid=None):
+    is_float = _act(x, rows * k, "x")
+    _bf16(w, n * k, "w")
+    _same_kind(is_float, y=y)
+    _act(y, rows * n, "y")
+    check(lib().iron_linear_any(ptr(x), ptr(w), ptr(y), rows, n, k, int(is_float), ptr(_word(valid, "valid")),
+                                current_stream()), "iron_linear_any")
+
+
+def token_shift(h, mu, carry, spans, mixed, *, slots, rows, cols, mixes):
+    is_float = _act(h, rows * cols, "h")
+    _bf16(mu, mixes * cols, "mu")
+    _same_kind(is_float, carry=carry, mixed=mixed)
+    _act(carry, slots * cols, "carry")
+    _act(mixed, mixes * rows * cols, "mixed")
+    check(lib().iron_token_shift(ptr(h), ptr(mu), ptr(carry), _spans(spans, slots), ptr(mixed), slots, rows, cols, mixes,
+                                 int(is_float), current_stream()), "iron_token_shift")
+
+
+def low_rank_decay(z, w2, w0, out, *, rows, n, rank, valid=None):
+    is_float = _act(z, rows * rank, "z")
+    _bf16(w2, n * rank, "w2")
+    _bf16(w0, n, "w0")
+    _f32(out, rows * n, "out")
+    check(lib().iron_low_rank_decay(ptr(z), ptr(w2), ptr(w0), ptr(out), rows, n, rank, int(is_float),
+                                    ptr(_word(valid, "valid")), current_stream()), "iron_low_rank_decay")
+
+
+def time_mix(r, k, v, log_decay, u, state, spans, o, *, slots, rows, heads, dim):
+    n = rows * heads * dim
+    is_float = _act(r, n, "r")
+    _same_kind(is_float, k=k, v=v)
+    _act(k, n, "k")
+    _act(v, n, "v")
+    _f32(log_decay, n, "log_decay")
+    _bf16(u, heads * dim, "u")
+    _f32(state, slots * heads * dim * dim, "state")
+    _f32(o, n, "o")
+    check(lib().iron_time_mix(ptr(r), ptr(k), ptr(v), ptr(log_decay), ptr(u), ptr(state), _spans(spans, slots), ptr(o), slots,
+                              rows, heads, dim, int(is_float), current_stream()), "iron_time_mix")
+
+
+def short_conv(x, taps_w, a_log, dt_bias, state, spans, out, *, slots, rows, stride, heads, kv_heads, dim, vdim, taps,
+               b_at, a_at):
+    channels = 2 * kv_heads * dim + heads * vdim
+    is_float = _act(x, rows * stride, "x")
+    _bf16(taps_w, channels * taps, "taps_w")
+    _bf16(a_log, heads, "a_log")
+    _bf16(dt_bias, heads, "dt_bias")
+    _same_kind(is_float, state=state)
+    _act(state, slots * max(taps - 1, 1) * channels, "state")
+    _f32(out, rows * (channels + 2 * heads), "out")
+    check(lib().iron_short_conv(ptr(x), ptr(taps_w), ptr(a_log), ptr(dt_bias), ptr(state), _spans(spans, slots), ptr(out),
+                                slots, rows, stride, heads, kv_heads, dim, vdim, taps, b_at, a_at, int(is_float),
+                                current_stream()), "iron_short_conv")
+
+
+def delta_rule(x, state, spans, o, *, slots, rows, heads, kv_heads, dim, vdim):
+    _f32(x, rows * (2 * kv_heads * dim + heads * vdim + 2 * heads), "x")
+    _f32(state, slots * heads * dim * vdim, "state")
+    _f32(o, rows * heads * vdim, "o")
+    check(lib().iron_delta_rule(ptr(x), ptr(state), _spans(spans, slots), ptr(o), slots, rows, heads, kv_heads, dim, vdim,
+                                current_stream()), "iron_delta_rule")
+
+
+def head_gate(o, gate, gain, out, *, rows, heads, dim, gate_stride, gate_at, gain_shared, out_stride, out_at, eps, scale,
+              valid=None):
+    _f32(o, rows * heads * dim, "o")
+    is_float = _act(gate, rows * gate_stride, "gate")
+    _bf16(gain, dim if gain_shared else heads * dim, "gain")
+    _same_kind(is_float, out=out)
+    _act(out, rows * out_stride, "out")
+    check(lib().iron_head_gate(ptr(o), ptr(gate), ptr(gain), ptr(out), rows, heads, dim, gate_stride, gate_at,
+                               int(gain_shared), out_stride, out_at, float(eps), float(scale), int(is_float),
+                               ptr(_word(valid, "valid")), current_stream()), "iron_head_gate")
+
+
+def mha_window(x, keys, values, bias, spans, out, *, slots, rows, stride, heads, kv_heads, dim, vdim, window, ring, scale,
+               out_stride, out_at=0, out_scale=1.0, single=False):
+    is_float = _act(x, rows * stride, "x")
+    _same_kind(is_float, keys=keys, values=values, out=out)
+    _act(keys, slots * ring * kv_heads * dim, "keys")
+    _act(values, slots * ring * kv_heads * vdim, "values")
+    _f32(bias, heads * window, "bias")
+    _act(out, rows * out_stride, "out")
+    check(lib().iron_mha_window(ptr(x), ptr(keys), ptr(values), ptr(bias), _spans(spans, slots), ptr(out), slots, rows, stride,
+                                heads, kv_heads, dim, vdim, window, ring, float(scale), out_stride, out_at, float(out_scale),
+                                int(single), int(is_float), current_stream()), "iron_mha_window")
+
+
+def sample_slots(logits, spans, draws, token, record, workspace, *, n, stride, slots, batch_rows, steps, k_max=64):
+    _bf16(logits, slots * stride, "logits")
+    for t, count, name in ((draws, 4 * slots * steps, "draws"), (token, slots, "token"), (record, slots * steps, "record")):
+        _numel(_dev(t, name, torch.int32), count, name)
+    need = slots * int(lib().iron_sample_workspace_bytes(n))
+    if _dev(workspace, "workspace", None).numel() * workspace.element_size() < need:
+        raise ValueError(f"sample_slots: the workspace is smaller than {need} bytes")
+    check(lib().iron_sample_slots_bf16(ptr(logits), n, stride, _spans(spans, slots), slots, batch_rows, steps, ptr(draws),
+                                       k_max, ptr(workspace), ptr(token), ptr(record), current_stream()),
+          "iron_sample_slots_bf16")

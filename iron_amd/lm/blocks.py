@@ -15,20 +15,24 @@ import dataclasses
 import functools
 
 from .. import functional as F
-from ..bf16 import round_bf16
+from ..bf16 import bfloat16, round_bf16
 from ..common import graph as iron
 from ..common.declare import Precision
 from ..operators.axpy import AXPY
 from ..operators.copy import Copy
 from ..operators.gelu import GELU
 from ..operators.mha import MHA
+from ..operators.stream import GatedProduct
 
 # ``hidden_act`` as a config spells it -> what records it (iron/lm/blocks.py:246-266)
 _ACTIVATIONS = {
     "silu": lambda: F.silu,
     "gelu_pytorch_tanh": lambda: functools.partial(GELU.step, approximate="tanh"),
     "gelu": lambda: functools.partial(GELU.step, approximate="none"),
+    "relu": lambda: F.relu,
 }
+# the names a gated product in 32 bits has for them
+_FLOAT_GATES = {"silu": "silu", "gelu_pytorch_tanh": "gelu_tanh", "relu": "relu"}
 
 
 def activation(name: str):
@@ -300,10 +304,13 @@ class GatedMLP(iron.Graph):
         self.up_proj = dense(hidden, inner)
         self.down_proj = dense(inner, hidden)
         self.act = activation(c.hidden_act)
+        self.hidden_act = c.hidden_act
 
     def body(self, x):
         gate = self.gate_proj(x)
         up = self.up_proj(x)
+        if gate.dtype is not bfloat16:   # a model that runs in 32 bits throughout
+            return self.down_proj(GatedProduct.step(gate, up, activation=_FLOAT_GATES[self.hidden_act]))
         return self.down_proj(self.act(gate) * up)
 
 

@@ -79,6 +79,7 @@ class CausalLM(iron.Graph):
     decoder_class = Decoder
     layer_class = DecoderLayer
     config_class = DecoderConfig      # what from_checkpoint parses config.json into
+    session_class = Session           # how a conversation's history becomes launches
     checkpoint = None
     tokenizer = None
     k_max = 64                        # candidates a device draw can weigh; Sampler.rows refuses a larger top-k
@@ -87,13 +88,13 @@ class CausalLM(iron.Graph):
     def __init__(self, config: DecoderConfig, weights):
         self.config = config
         self.rotary_emb = Rope(config) if config.rope_theta is not None else None
-        rows = config.max_seq_len
-        self.draws = iron.state((rows, ROW_WORDS), np.int32)   # a draw row per position; all-zero = greedy
-        self.drawn = iron.state((rows,), np.int32)             # the device's record of what it drew where
+        shape = self.draw_shape(config)
+        self.draws = iron.state((*shape, ROW_WORDS), np.int32)   # a draw row per position; all-zero = greedy
+        self.drawn = iron.state(shape, np.int32)                 # the device's record of what it drew where
         self.sampled = False          # whether `draws` currently holds a sampler's rows
         self.decode_step = self.prompt_chunk = None
         self.holder = None            # the Session whose tokens the caches hold
-        self.session = Session(self)
+        self.session = self.session_class(self)
         self.stats = Stats()
         self.model = self.decoder_class(config, self.layer_class)
         self.layers = self.model.layers
@@ -103,6 +104,11 @@ class CausalLM(iron.Graph):
         if config.tie_word_embeddings:
             self.lm_head.weight = self.model.embed_tokens.weight
         self.load_state_dict(weights)
+
+    @staticmethod
+    def draw_shape(config) -> tuple[int, ...]:
+        """Hook: the positions draws and their record are kept for."""
+        return (config.max_seq_len,)
 
     @classmethod
     def from_checkpoint(cls, path, *, max_seq_len: int | None = None, **changes):

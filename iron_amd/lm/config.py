@@ -18,7 +18,7 @@ from ..common.declare import Precision
 
 RopeScaling = Callable[[np.ndarray], np.ndarray]
 
-_ACTIVATIONS = ("silu", "gelu_pytorch_tanh", "gelu")
+_ACTIVATIONS = ("silu", "gelu_pytorch_tanh", "gelu", "relu")
 
 
 def rope_angles(head_dim: int, context_length: int, rope_theta: float = 500000.0,
@@ -47,8 +47,26 @@ def _required(field: dataclasses.Field) -> bool:
     return field.default is dataclasses.MISSING and field.default_factory is dataclasses.MISSING
 
 
+class ConfigFile:
+    """A config that is read from a ``config.json`` through ``from_json``."""
+
+    @classmethod
+    def from_checkpoint(cls, path):
+        """Read ``config.json`` given that file, the checkpoint directory, or any file in it.
+
+        Raises:
+            FileNotFoundError: there is no ``config.json`` there.
+            ValueError: a field without a default is absent from it.
+        """
+        where = Path(path)
+        if where.name != "config.json":
+            where = (where if where.is_dir() else where.parent) / "config.json"
+        with open(where) as handle:
+            return cls.from_json(json.load(handle), where)
+
+
 @dataclasses.dataclass(frozen=True)
-class DecoderConfig:
+class DecoderConfig(ConfigFile):
     """Shape and options of a decoder.  ``max_seq_len`` starts as the checkpoint's native context
     and is usually lowered by the caller (it sizes the KV caches and the rotary table)."""
 
@@ -96,20 +114,6 @@ class DecoderConfig:
     @classmethod
     def _json_key(cls, name: str) -> str | None:
         return cls.JSON[name] if name in cls.JSON else name
-
-    @classmethod
-    def from_checkpoint(cls, path):
-        """Read ``config.json`` given that file, the checkpoint directory, or any file in it.
-
-        Raises:
-            FileNotFoundError: there is no ``config.json`` there.
-            ValueError: a field without a default is absent from it.
-        """
-        where = Path(path)
-        if where.name != "config.json":
-            where = (where if where.is_dir() else where.parent) / "config.json"
-        with open(where) as handle:
-            return cls.from_json(json.load(handle), where)
 
     @classmethod
     def from_json(cls, data: dict, source="config.json"):

@@ -1,0 +1,199 @@
+"""Token mixers over a batch of rows told apart by spans, and the layer that runs them around a float32
+residual stream: sliding-window attention with a learned distance bias, time mixing with a
+data-dependent decay, both side by side, and the gated delta rule.
+
+A module holds weights; what a run of it carries from token to token is a ``states()`` mapping the
+caller makes once per run, so that a layer run several times in a row has a state for each pass.
+Constants and sizes are constructor arguments.  ``call`` is a ``batched.BatchCall``.
+"""
+
+from __future__ import annotations
+
+import math
+
+import numpy as np
+
+from .. import functional as F
+from ..common import graph as iron
+from ..operators.mha_window import WindowMHA
+from ..operators.recurrent import DeltaRule, HeadGate, LowRankDecay, ShortConv, TimeMix, TokenShift
+from ..operators.stream import StreamAdd, StreamNorm
+from .blocks import Linear
+
+
+def as_rows(x, rows: int):
+    """A projection's output as ``rows`` rows (a single row's product comes flat)."""
+    return x if len(x.shape) == 2 else x.reshape(rows, x.elements // rows)
+
+
+def distance_buckets(count: int, rows: int, bias_max: float) -> np.ndarray:
+    """The row of a ``rows``-row distance-bias table that each of the distances ``0 .. count - 1`` reads:
+    its own up to half the rows, then logarithmically spaced ones up to ``bias_max`` and the last row
+    from there on.  In float32, as everything about positions."""
+    half = np.float32(rows / 2)
+    n = np.arange(count)
+    far = n >= rows / 2
+    ratio = np.maximum(n, 1).astype(np.float32) / half
+    steps = np.log(ratio, dtype=np.float32) / np.float32(math.log(bias_max / (rows / 2))) * np.float32(rows - rows / 2)
+    spaced = np.floor(half + np.floor(np.maximum(steps, 0)))
+    return np.where(far, np.minimum(rows - 1, spaced), n).astype(np.int64)
+
+
+class StreamRMSNorm(iron.Graph):
+    """An RMS norm at the stream's edge: ``body`` takes a normed row out of it, ``add`` a block's output
+    into it."""
+
+    def __init__(self, width: int, eps: float, dtype):
+        self.eps, self.dtype = eps, dtype
+        self.weight = iron.param(width)
+
+    def body(self, stream):
+        return StreamNorm.step(stream, self.weight, epsilon=self.eps, dtype=self.dtype)
+
+    def add(self, stream, y):
+        return StreamAdd.step(stream, y, self.weight, epsilon=self.eps, dtype=self.dtype)
+
+
+class WindowAttention(iron.Graph):
+    """Grouped-query sliding-window attention whose positions enter by a learned bias per distance bucket
+    and head.  ``qkv`` is one packed projection (q heads, k heads, v heads).  Fills columns ``at ..`` of
+    the mixer's row with the heads' outputs times ``out_scale``; the output projection is the mixer's."""
+
+    def __init__(self, width, *, heads, kv_heads, dim, vdim, window, bias_rows, bias_max, scale, context, dtype, precision,
+                 out_scale=1.0):
+        self.heads, self.kv_heads, self.dim, self.vdim = heads, kv_heads, dim, vdim
+        self.window = min(window, context)
+        self.bias_max, self.scale, self.out_scale, self.dtype = bias_max, scale, out_scale, dtype
+        self.qkv = Linear(width, heads * dim + kv_heads * (dim + vdim), precision=precision)
+        self.rel = iron.param(bias_rows, heads)
+        self.by_distance = None            # (heads, window) float32, spread from rel when the weights are loaded
+
+    @property
+    def out_width(self) -> int:
+        return self.heads * self.vdim
+
+    def loaded(self, as_float32) -> None:
+        table = as_float32(self.rel.array)
+        spread = table[distance_buckets(self.window, table.shape[0], self.bias_max)]
+        self.by_distance = iron.Weight((self.heads, self.window), np.float32, np.ascontiguousarray(spread.T, dtype=np.float32))
+
+    def states(self, slots: int) -> dict:
+        # The ring holds just the window: a portion's own keys are read from its projection's rows.
+        return {"keys": iron.state((slots, self.window, self.kv_heads, self.dim), self.dtype),
+                "values": iron.state((slots, self.window, self.kv_heads, self.vdim), self.dtype)}
+
+    def body(self, h, call, state, mixed, at=0):
+        x = as_rows(self.qkv(h), h.shape[0])
+        return WindowMHA.step(x, self.by_distance, call.spans, state["keys"], state["values"], mixed, scale=self.scale,
+                              out_scale=self.out_scale, at=at, single=not call.prompt, dtype=self.dtype)[2]
+
+
+class TimeMixing(iron.Graph):
+    """Time mixing: r, k, v, a gate and a decay, each projected from its own blend of a token and the one
+    before it, and a per-head outer-product state with a bonus for the current token.  Fills columns
+    ``at ..`` of a ``width``-column mixer row."""
+
+    BLENDS = "rkvgw"
+
+    def __init__(self, width, *, heads, dim, rank, eps, dtype, precision, out_scale=1.0):
+        self.width, self.heads, self.dim, self.eps, self.dtype, self.out_scale = width, heads, dim, eps, dtype, out_scale
+
+        def dense(fan_out):
+            return Linear(width, fan_out, precision=precision)
+
+        inner = heads * dim
+        self.mu = iron.param(len(self.BLENDS), width)
+        self.r, self.k, self.v, self.g, self.w1 = dense(inner), dense(inner), dense(inner), dense(inner), dense(rank)
+        self.w2 = iron.param(inner, rank)
+        self.w0 = iron.param(inner)
+        self.u = iron.param(heads, dim)
+        self.norm = iron.param(inner)
+
+    @property
+    def out_width(self) -> int:
+        return self.heads * self.dim
+
+    def states(self, slots: int) -> dict:
+        return {"before": iron.state((slots, self.width), self.dtype),
+                "memory": iron.state((slots, self.heads, self.dim, self.dim), np.float32)}
+
+    def body(self, h, call, state, width, at=0):
+        blends = TokenShift.step(h, self.mu, state["before"], call.spans, dtype=self.dtype)[1]
+        r, k, v, g, z = (proj(call.bound(blends[i])) for i, proj in enumerate((self.r, self.k, self.v, self.g, self.w1)))
+        r, k, v, g, z = (as_rows(x, h.shape[0]) for x in (r, k, v, g, z))
+        decay = LowRankDecay.step(z, self.w2, self.w0, dtype=self.dtype)
+        o = TimeMix.step(r, k, v, decay, self.u, state["memory"], call.spans, dtype=self.dtype)[1]
+        return HeadGate.step(o, g, self.norm, heads=self.heads, width=width, at=at, epsilon=self.eps, scale=self.out_scale,
+                             dtype=self.dtype)
+
+
+class ParallelMixer(iron.Graph):
+    """Attention (``left``) and time mixing (``right``) of the same input, weighed and summed.  Their
+    output projections are one product over the two outputs side by side, each scaled as it is made."""
+
+    def __init__(self, width, left: WindowAttention, right: TimeMixing, *, precision):
+        self.left, self.right = left, right
+        self.out = Linear(left.out_width + right.out_width, width, precision=precision)
+
+    def loaded(self, as_float32) -> None:
+        self.left.loaded(as_float32)
+
+    def states(self, slots: int) -> dict:
+        return {**self.left.states(slots), **self.right.states(slots)}
+
+    def body(self, h, call, state):
+        mixed = self.right(h, call, state, self.out.in_features, at=self.left.out_width)
+        return self.out(self.left(h, call, state, mixed))
+
+
+class DeltaMixer(iron.Graph):
+    """The gated delta rule: short convolutions over q, k and v, unit q and k, a write strength and a decay
+    a head, a matrix state a value head, a gated norm a head.  ``proj`` is one packed projection
+    (q, k, v, gate, b, a)."""
+
+    def __init__(self, width, *, heads, kv_heads, dim, vdim, taps, eps, dtype, precision):
+        self.heads, self.kv_heads, self.dim, self.vdim, self.taps = heads, kv_heads, dim, vdim, taps
+        self.eps, self.dtype = eps, dtype
+        self.channels = 2 * kv_heads * dim + heads * vdim
+        inner = heads * vdim
+        self.gate_at, self.b_at, self.a_at = self.channels, self.channels + inner, self.channels + inner + heads
+        self.proj = Linear(width, self.a_at + heads, precision=precision)
+        self.conv = iron.param(self.channels, taps)
+        self.a_log = iron.param(heads)
+        self.dt_bias = iron.param(heads)
+        self.norm = iron.param(vdim)
+        self.out = Linear(inner, width, precision=precision)
+
+    def loaded(self, as_float32) -> None:
+        pass
+
+    def states(self, slots: int) -> dict:
+        return {"inputs": iron.state((slots, max(self.taps - 1, 1), self.channels), self.dtype),
+                "memory": iron.state((slots, self.heads, self.dim, self.vdim), np.float32)}
+
+    def body(self, h, call, state):
+        sizes = dict(kv_heads=self.kv_heads)
+        x = as_rows(self.proj(h), h.shape[0])
+        _, y = ShortConv.step(x, self.conv, self.a_log, self.dt_bias, state["inputs"], call.spans, dim=self.dim, vdim=self.vdim,
+                              b_at=self.b_at, a_at=self.a_at, dtype=self.dtype, **sizes)
+        _, o = DeltaRule.step(y, state["memory"], call.spans, **sizes)
+        return self.out(HeadGate.step(o, x, self.norm, heads=self.heads, gate_at=self.gate_at, epsilon=self.eps,
+                                      dtype=self.dtype))
+
+
+class StreamLayer(iron.Graph):
+    """A sandwich layer around a float32 stream: the mixer, then the feed-forward (if any), each between a
+    norm out of the stream and a norm back into it."""
+
+    def __init__(self, width, mixer, mlp, *, eps, dtype):
+        self.norm1, self.norm1b = StreamRMSNorm(width, eps, dtype), StreamRMSNorm(width, eps, dtype)
+        self.mixer, self.mlp = mixer, mlp
+        if mlp is not None:
+            self.norm2, self.norm2b = StreamRMSNorm(width, eps, dtype), StreamRMSNorm(width, eps, dtype)
+        self.rope = None
+
+    def body(self, x, call, state):
+        x = self.norm1b.add(x, as_rows(self.mixer(self.norm1(x), call, state), x.shape[0]))
+        if self.mlp is not None:
+            x = self.norm2b.add(x, as_rows(self.mlp(self.norm2(x)), x.shape[0]))
+        return x

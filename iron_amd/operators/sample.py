@@ -120,3 +120,63 @@ class Sample(Operator):
                            advance=words.get("__carry_eval__"))
 
         return Built("iron_sample_bf16", launch)
+
+
+class SampleSlots(Operator):
+    """A draw a slot of a batch: slot s's row of ``logits`` (``vocab`` of its ``stride`` columns are tokens')
+    is drawn from at the position p of the slot's last row, by draw row ``draws[s, p]``, and recorded in
+    ``tokens[s, p]``.  Its token and span are then the next step's: one row at p + 1.  An idle slot draws
+    nothing.  The arithmetic is ``Sample``'s."""
+
+    slots: int = param()
+    vocab: int = param(array=True)
+    stride: int = param()
+    steps: int = param()
+    batch_rows: int = param(array=True)   # rows of the batch the spans are of
+    k_max: int = param(default=64, array=True)
+    workspace_words: int = param(derive=lambda op: op._workspace_words(), repr=False)
+
+    logits = In(slots, stride)
+    draws = In(slots, steps, ROW_WORDS, dtype=np.int32)
+    spans = InOut(slots, 4, dtype=np.int32)
+    token = InOut(slots, dtype=np.int32)
+    tokens = InOut(slots, steps, dtype=np.int32)
+    workspace = Scratch(workspace_words, dtype=np.float32, kept=True)
+
+    def _workspace_words(self) -> int:
+        from .._lib import lib
+
+        return self.slots * int(lib().iron_sample_workspace_bytes(self.vocab)) // 4
+
+    @classmethod
+    def infer(cls, shapes, **kw):
+        return dict(slots=shapes["logits"][0], stride=shapes["logits"][1], steps=shapes["draws"][1], **kw)
+
+    def validate(self) -> None:
+        if not 1 <= self.k_max <= K_MAX:
+            raise ValueError(f"SampleSlots: k_max ({self.k_max}) must be from 1 to {K_MAX}")
+        if not self.vocab <= self.stride:
+            raise ValueError(f"SampleSlots: {self.vocab} tokens in a row of {self.stride}")
+
+    def bind_views(self, inputs, outputs):
+        return {}
+
+    def output_valid(self, name, inputs):
+        return {}
+
+    def ops(self) -> int:
+        return 0
+
+    def tolerance(self) -> Tolerance:
+        return Tolerance.exact()
+
+    def build(self) -> Built:
+        from .. import kernels
+
+        kw = dict(n=self.vocab, stride=self.stride, slots=self.slots, batch_rows=self.batch_rows, steps=self.steps,
+                  k_max=self.k_max)
+
+        def launch(t, words):
+            kernels.sample_slots(t["logits"], t["spans"], t["draws"], t["token"], t["tokens"], t["workspace"], **kw)
+
+        return Built("iron_sample_slots_bf16", launch)

@@ -1,0 +1,235 @@
+"""The float32 residual stream of a decoder: rows into it, norms out of it, blocks' outputs added to it,
+and the head's soft cap.  ``dtype`` is what the rows that leave the stream are rounded to: bf16, or
+float32 in a model that runs in 32 bits throughout.  The stream is updated in place.
+"""
+
+from __future__ import annotations
+
+import math
+from typing import Any
+
+import numpy as np
+
+from ..bf16 import bfloat16
+from ..common.declare import Built, In, InOut, Operator, Out, param, per_call
+from ..common.verify import Tolerance
+
+F32 = np.float32
+
+
+class StreamEmbed(Operator):
+    """``x[i] = table[ids[i]]``, widened: a decoder's embedding rows as its stream's first values."""
+
+    rows: int = param()
+    table_rows: int = param(array=True)
+    cols: int = param()
+    table = In(table_rows, cols)
+    ids = In(rows, dtype=np.int32)
+    x = Out(rows, cols, dtype=F32)
+    valid = per_call(bounds=rows)
+
+    @classmethod
+    def infer(cls, shapes, **kw):
+        return dict(rows=math.prod(shapes["ids"]), table_rows=shapes["table"][0], cols=shapes["table"][1])
+
+    def tolerance(self):
+        return Tolerance.exact()
+
+    def build(self) -> Built:
+        from .. import kernels
+
+        rows, table_rows, cols = self.rows, self.table_rows, self.cols
+
+        def launch(t, words):
+            kernels.stream_embed(t["table"], t["ids"].reshape(-1), t["x"], rows=rows, table_rows=table_rows, cols=cols,
+                                 valid=words.get("valid"))
+
+        return Built("iron_stream_embed", launch)
+
+
+class StreamNorm(Operator):
+    """``y = dtype(x / rms(x) * weight)`` of a float32 row: one rounding, where it leaves the stream."""
+
+    rows: int = param()
+    cols: int = param()
+    epsilon: float = param(array=True)
+    dtype: Any = param(default=bfloat16, repr=False)
+    x = In(rows, cols, dtype=F32)
+    weight = In(cols)
+    y = Out(rows, cols, dtype=dtype)
+    valid = per_call(bounds=rows)
+
+    @classmethod
+    def infer(cls, shapes, **kw):
+        return dict(rows=shapes["x"][0], cols=shapes["x"][1], **kw)
+
+    def tolerance(self):
+        return Tolerance.relative(1e-2, 1e-2, note="float32, rounded once")
+
+    def build(self) -> Built:
+        from .. import kernels
+
+        rows, cols, eps = self.rows, self.cols, float(self.epsilon)
+
+        def launch(t, words):
+            kernels.stream_rows(t["x"], rows=rows, cols=cols, eps=eps, h=t["y"], gain=t["weight"], valid=words.get("valid"))
+
+        return Built("iron_stream_rows", launch)
+
+
+class StreamAdd(Operator):
+    """``x += y / rms(y) * weight`` in float32: a block's output, normed, joins the stream."""
+
+    rows: int = param()
+    cols: int = param()
+    epsilon: float = param(array=True)
+    dtype: Any = param(default=bfloat16, repr=False)
+    x = InOut(rows, cols, dtype=F32)
+    y = In(rows, cols, dtype=dtype)
+    weight = In(cols)
+    valid = per_call(bounds=rows)
+
+    @classmethod
+    def infer(cls, shapes, **kw):
+        return dict(rows=shapes["x"][0], cols=shapes["x"][1], **kw)
+
+    def tolerance(self):
+        return Tolerance.relative(1e-4, 1e-4, note="float32")
+
+    def build(self) -> Built:
+        from .. import kernels
+
+        rows, cols, eps = self.rows, self.cols, float(self.epsilon)
+
+        def launch(t, words):
+            kernels.stream_rows(t["x"], rows=rows, cols=cols, eps=eps, y=t["y"], back_gain=t["weight"],
+                                valid=words.get("valid"))
+
+        return Built("iron_stream_rows", launch)
+
+
+class SpanTails(Operator):
+    """The stream's row of every slot's last token: what a prompt's portion hands its head."""
+
+    slots: int = param()
+    rows: int = param()
+    cols: int = param()
+    x = In(rows, cols, dtype=F32)
+    spans = In(slots, 4, dtype=np.int32)
+    y = Out(slots, cols, dtype=F32)
+
+    @classmethod
+    def infer(cls, shapes, **kw):
+        return dict(slots=shapes["spans"][0], rows=shapes["x"][0], cols=shapes["x"][1])
+
+    def output_valid(self, name, inputs):
+        return {}
+
+    def tolerance(self):
+        return Tolerance.exact()
+
+    def build(self) -> Built:
+        from .. import kernels
+
+        slots, rows, cols = self.slots, self.rows, self.cols
+
+        def launch(t, words):
+            kernels.span_tails(t["x"], t["spans"], t["y"], slots=slots, rows=rows, cols=cols)
+
+        return Built("iron_span_tails", launch)
+
+
+class Softcap(Operator):
+    """``cap * tanh(x / cap)`` of the head's rows (``cap`` 0: as they are), as float32 and, in rows padded to
+    whole 16-byte pieces, as the bf16 the draw ranks."""
+
+    rows: int = param()
+    cols: int = param()
+    cap: float = param(default=0.0, array=True)
+    dtype: Any = param(default=bfloat16, repr=False)
+    stride: int = param(derive=lambda op: -(-op.cols // 8) * 8, repr=False)
+    x = In(rows, cols, dtype=dtype)
+    y = Out(rows, cols, dtype=F32)
+    rounded = Out(rows, stride)
+
+    @classmethod
+    def infer(cls, shapes, **kw):
+        return dict(rows=shapes["x"][0], cols=shapes["x"][1], **kw)
+
+    def tolerance(self):
+        return Tolerance.relative(1e-2, 1e-2, note="float32, the draw's copy rounded")
+
+    def build(self) -> Built:
+        from .. import kernels
+
+        rows, cols, stride, cap = self.rows, self.cols, self.stride, float(self.cap)
+
+        def launch(t, words):
+            kernels.softcap(t["x"], t["y"], t["rounded"], rows=rows, cols=cols, stride=stride, cap=cap)
+
+        return Built("iron_softcap", launch)
+
+
+class GatedProduct(Operator):
+    """``act(gate) * up`` in float32, the 32-bit model's step where a bf16 one records the two."""
+
+    rows: int = param()
+    cols: int = param()
+    activation: str = param()
+    gate = In(rows, cols, dtype=F32)
+    up = In(rows, cols, dtype=F32)
+    y = Out(rows, cols, dtype=F32)
+    valid = per_call(bounds=rows)
+
+    @classmethod
+    def infer(cls, shapes, **kw):
+        return dict(rows=shapes["gate"][0], cols=shapes["gate"][1], **kw)
+
+    def tolerance(self):
+        return Tolerance.relative(1e-5, 1e-6, note="float32")
+
+    def build(self) -> Built:
+        from .. import kernels
+
+        rows, cols, kind = self.rows, self.cols, self.activation
+
+        def launch(t, words):
+            kernels.act_mul_f32(t["gate"], t["up"], t["y"], rows=rows, cols=cols, activation=kind, valid=words.get("valid"))
+
+        return Built("iron_act_mul_f32", launch)
+
+
+class LinearAny(Operator):
+    """``x @ weight.T`` on float32 products and sums, rows of either type and any length: the 32-bit
+    model's projections (bf16 weights are float32 values), and a bf16 row of no whole 16-byte pieces."""
+
+    rows: int = param()
+    n: int = param()
+    k: int = param()
+    dtype: Any = param(default=bfloat16, repr=False)
+    x = In(rows, k, dtype=dtype)
+    weight = In(n, k)
+    y = Out(rows, n, dtype=dtype)
+    valid = per_call(bounds=rows)
+
+    @classmethod
+    def infer(cls, shapes, **kw):
+        if shapes["x"][1] != shapes["weight"][1]:
+            raise ValueError(f"x {shapes['x']} and the weight {shapes['weight']} disagree on their length")
+        return dict(rows=shapes["x"][0], n=shapes["weight"][0], k=shapes["x"][1], **kw)
+
+    def ops(self) -> int:
+        return 2 * self.rows * self.n * self.k
+
+    def tolerance(self):
+        return Tolerance.relative(1e-2, 1e-2, note="float32 sums, rounded once if bf16")
+
+    def build(self) -> Built:
+        from .. import kernels
+
+        rows, n, k = self.rows, self.n, self.k
+
+        def launch(t, words):
+            kernels.linear_any(t["x"], t["weight"], t["y"], rows=rows, n=n, k=k, valid=words.get("valid"))
+
+        return Built("iron_linear_any", launch)
