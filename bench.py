@@ -643,6 +643,169 @@ def cpu_decoder_baseline(torch, config, weights, prompt, gpu_prompt_logits, gpu_
                          "one of the host's logits", "prompt_logits_max_diff_share": share, "tokens_checked": checked}
 
 
+# Layers of a real model's sizes, by width: (heads, kv heads, head dim, feed-forward, layers timed, vocabulary)
+PEGILIX_SIZES = {2048: (32, 8, 64, 8192, 16, 128256), 3072: (24, 8, 128, 8192, 8, 128256), 4096: (32, 8, 128, 14336, 8, 128256)}
+PEGILIX_WINDOW = 1024
+
+
+def pegilix_config(width, slots=1, chunk=2048):
+    """A Pegilix of ``width``'s sizes: three parallel layers to each delta layer."""
+    from iron_amd.applications.pegilix import PegilixConfig
+
+    H, G, D, F, layers, vocab = PEGILIX_SIZES[width]
+    mlp = {"ff": F, "kind": "dense"}
+    parallel = {"type": "parallel", "mlp": mlp, "mixer": {
+        "left": {"heads": H, "kv_heads": G, "dim": D, "vdim": D, "scale": D**-0.5, "bias_max": 512, "mask": {"size": PEGILIX_WINDOW}},
+        "right": {"heads": width // 64, "dim": 64}, "left_scale": 1.1, "right_scale": 0.9}}
+    delta = {"type": "delta", "mlp": mlp, "mixer": {"heads": width // D, "kv_heads": width // D // 2, "dim": D, "vdim": D, "conv": 4}}
+    return PegilixConfig(vocab_size=vocab, hidden_size=width, layers=tuple([parallel, parallel, parallel, delta] * (layers // 4)),
+                         eps=1e-5, logit_softcap=30.0, max_seq_len=4096, prefill_chunk=chunk, slots=slots)
+
+
+def random_weights(torch, shapes, dev, seed=0):
+    """bf16 tensors of these shapes on the GPU: matrices N(0, 0.02), vectors N(1, 0.1)."""
+    g = torch.Generator(device=dev)
+    g.manual_seed(seed)
+    return {n: (torch.randn(s, generator=g, device=dev).mul_(0.02 if len(s) > 1 else 0.1).add_(0.0 if len(s) > 1 else 1.0)).to(torch.bfloat16)
+            for n, s in shapes.items()}
+
+
+def time_served(torch, run_prompt, decode, steps, prompts, repeats=5):
+    """Median milliseconds of a prompt of each length, and milliseconds a replayed decode step."""
+    out = {"prompt_ms": {}}
+    for n in prompts:
+        for _ in range(2):
+            run_prompt(n)
+        times = []
+        for _ in range(repeats):
+            torch.cuda.synchronize()
+            t0 = time.perf_counter()
+            run_prompt(n)
+            torch.cuda.synchronize()
+            times.append(time.perf_counter() - t0)
+        out["prompt_ms"][str(n)] = round(1e3 * float(np.median(times)), 3)
+        out.setdefault("prompt_tok_s", {})[str(n)] = round(n / float(np.median(times)), 1)
+    start, stop = torch.cuda.Event(enable_timing=True), torch.cuda.Event(enable_timing=True)
+    decode.replay(8)
+    torch.cuda.synchronize()
+    start.record()
+    decode.replay(steps)
+    stop.record()
+    stop.synchronize()
+    out["decode_ms"] = round(start.elapsed_time(stop) / steps, 4)
+    return out
+
+
+def pegilix_served(torch, config, weights, steps, prompts):
+    from iron_amd.applications.pegilix import Pegilix
+    from iron_amd.lm.batched import Entry
+
+    model = Pegilix(config, weights)
+    model.load_versions()
+    rng = np.random.default_rng(512)
+    tokens = [rng.integers(0, config.vocab_size, max(prompts)) for _ in range(config.slots)]
+
+    def run_prompt(n):   # the prompt in every slot
+        for i in range(config.slots):
+            model.batch.end(i)
+        model.batch.step([Entry(i, tokens[i][:n]) for i in range(config.slots)])
+
+    run_prompt(min(prompts))
+    first = time_served(torch, run_prompt, _Started(model, steps), steps, prompts)
+    first["launches_per_step"] = model.decode_step.launches_per_replay
+    first["launches_per_portion"] = model.prompt_chunk.launches_per_call
+    weight_bytes = 2 * sum(int(np.prod(t.shape)) for n, t in weights.items() if n != "embed")
+    c, state = config, 0
+    for i in c.order:
+        m = c.layers[i]["mixer"]
+        if c.layers[i]["type"] == "parallel":
+            left, right = m["left"], m["right"]
+            state += PEGILIX_WINDOW * left["kv_heads"] * (left["dim"] + left["vdim"]) * 2 + 8 * right["heads"] * right["dim"] ** 2
+        else:
+            state += 8 * m["heads"] * m["dim"] * m["vdim"]
+    bytes_step = weight_bytes + c.slots * state
+    first |= {"decode_tok_s": round(1e3 * c.slots / first["decode_ms"], 1), "decode_GBps": round(bytes_step / first["decode_ms"] / 1e6, 1),
+              "frac_hbm": round(bytes_step / first["decode_ms"] / 1e6 / HBM_PEAK_GBS, 4), "bytes_per_step": int(bytes_step)}
+    model.release()
+    return first
+
+
+class _Started:
+    """A batched model's captured decode step, started wherever its slots stand."""
+
+    def __init__(self, model, steps):
+        self.model, self.begun = model, False
+
+    def replay(self, n):
+        if not self.begun:   # the prompts' draws are the first tokens; the spans stand behind the prompts
+            self.model.decode_step.start()
+            self.begun, n = True, n - 1
+        self.model.decode_step.replay(n)
+
+
+def bench_pegilix(torch, dev, steps, widths, batch=8, prompts=(512, 2048)):
+    """Prompt and decode throughput of Pegilix layers at a few widths, one sequence and a batch of ``batch``,
+    beside a Llama of the same width, heads, feed-forward, layers and vocabulary; random weights, bf16."""
+    import dataclasses
+
+    from iron_amd.applications.llama import LLAMA_3_2_1B, Llama
+    from iron_amd.applications.llama import shapes as llama_shapes
+    from iron_amd.applications.pegilix import shapes
+
+    rows = []
+    for width in widths:
+        H, G, D, F, layers, vocab = PEGILIX_SIZES[width]
+        config = pegilix_config(width)
+        weights = random_weights(torch, shapes(config, bias_rows=32, rank=64), dev)
+        row = {"width": width, "layers": layers, "pegilix": pegilix_served(torch, config, weights, steps, prompts)}
+        if batch:
+            row[f"pegilix_batch_{batch}"] = pegilix_served(torch, dataclasses.replace(config, slots=batch), weights, steps, (512,))
+        params = sum(int(np.prod(t.shape)) for t in weights.values())
+        del weights
+        torch.cuda.empty_cache()
+        lc = dataclasses.replace(LLAMA_3_2_1B, vocab_size=vocab, hidden_size=width, num_hidden_layers=layers, num_attention_heads=H,
+                                 num_key_value_heads=G, head_dim=D, intermediate_size=F, max_seq_len=4096, prefill_chunk=2048)
+        lw = random_weights(torch, llama_shapes(lc), dev)
+        model = Llama(lc, lw)
+        model.load_versions()
+        tokens = np.random.default_rng(512).integers(0, vocab, max(prompts))
+
+        def run_prompt(n):
+            carry = None
+            for inputs, values in model.session.chunk_calls(tokens[:n], 0):
+                _, carry = model(*inputs, **values)
+            return carry
+
+        model.decode_step.start(**run_prompt(prompts[0]))
+        got = time_served(torch, run_prompt, _AfterPrompt(model, run_prompt, prompts[-1]), steps, prompts)
+        nbytes = 2 * sum(int(np.prod(t.shape)) for n, t in lw.items()) + layers * PEGILIX_WINDOW * 4 * G * D
+        got |= {"decode_tok_s": round(1e3 / got["decode_ms"], 1), "frac_hbm": round(nbytes / got["decode_ms"] / 1e6 / HBM_PEAK_GBS, 4),
+                "bytes_per_step": nbytes, "launches_per_step": model.decode_step.launches_per_replay,
+                "launches_per_portion": model.prompt_chunk.launches_per_call}
+        row |= {"llama": got, "pegilix_params": params, "llama_params": sum(int(np.prod(t.shape)) for t in lw.values())}
+        model.release()
+        del model, lw
+        torch.cuda.empty_cache()
+        rows.append(row)
+        print(json.dumps(row), file=sys.stderr, flush=True)
+    return {"what": f"prompt (ms, tok/s) and greedy decode steps as HIP-graph replays; Pegilix window {PEGILIX_WINDOW}, "
+                    "decode behind the longest prompt; frac_hbm: weights, window and states over the time a step takes",
+            "data": "synthetic", "dtype": "bf16", "sizes": rows}
+
+
+class _AfterPrompt:
+    """A single-sequence model's captured decode step behind a prompt of ``n`` tokens."""
+
+    def __init__(self, model, run_prompt, n):
+        self.model, self.run_prompt, self.n, self.begun = model, run_prompt, n, False
+
+    def replay(self, n):
+        if not self.begun:
+            self.model.decode_step.start(**self.run_prompt(self.n))
+            self.begun, n = True, n - 1
+        self.model.decode_step.replay(n)
+
+
 PROBE_COPY_BYTES = 512 << 20
 # HBM bytes one launch moves, by kernel, from hardware counters (FETCH_SIZE and WRITE_SIZE per
 # dispatch, each scaled by what the same counter reads for a plain copy of PROBE_COPY_BYTES): filled
@@ -745,6 +908,11 @@ def main():
     ap.add_argument("--attention-probe", action="store_true",
                     help="launch only decode attention at 1024 / 4096 / 16384 keys and a plain copy of known size "
                          "(for a rocprofv3 --pmc or --kernel-trace run) and exit")
+    ap.add_argument("--pegilix", action="store_true",
+                    help="time only Pegilix layers at a few widths beside a Llama of equal size, and exit")
+    ap.add_argument("--widths", type=int, nargs="+", default=sorted(PEGILIX_SIZES), choices=sorted(PEGILIX_SIZES),
+                    help="the widths --pegilix times")
+    ap.add_argument("--batch", type=int, default=8, help="sequences of --pegilix's batch (0: one sequence only)")
     args = ap.parse_args()
     if args.gpus != 1:
         print("bench.py: this build is a one-GPU hot path; --gpus must be 1 "
@@ -774,6 +942,9 @@ def main():
 
     if args.counter_probe:
         counter_probe(torch, K, dev, rng)
+        return 0
+    if args.pegilix:
+        print(json.dumps(bench_pegilix(torch, dev, args.steps, args.widths, args.batch)))
         return 0
     if args.prompt_probe:
         prompt_probe(torch, dev)

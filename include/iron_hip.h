@@ -397,8 +397,8 @@ int iron_linear_any(const void* x, const uint16_t* w, void* y, int rows, int n, 
                     const int* valid, void* stream);
 
 /* mixed[m] = h + (before - h) * mu[m] for m < mixes, `before` the row ahead of h in its sequence (zeros
- * ahead of the first; carry[slot] ahead of a span's first row).  carry (slots, cols) then holds each
- * span's last row.  mu (mixes, cols), mixed (mixes, rows, cols). */
+ * ahead of the first).  carry (slots, 2, cols) keeps position p's row in row p % 2: read ahead of a span's
+ * first row, and written with its last.  mu (mixes, cols), mixed (mixes, rows, cols). */
 int iron_token_shift(const void* h, const uint16_t* mu, void* carry, const int* spans, void* mixed, int slots,
                      int rows, int cols, int mixes, int is_float, void* stream);
 /* out = -exp(w2 tanh(z) + w0): the logarithm of a decay per channel.  z (rows, rank), w2 (n, rank). */
@@ -412,7 +412,7 @@ int iron_time_mix(const void* r, const void* k, const void* v, const float* log_
  * channel and SiLU on q, k (kv_heads x dim) and v (heads x vdim); q and k made unit vectors a head
  * (eps 1e-6), q times dim^-1/2; decay = exp(-exp(a_log) softplus(a + dt_bias)), beta = sigmoid(b).
  * out (rows, 2 kv_heads dim + heads vdim + 2 heads) = [q | k | v | decay | beta] in float.
- * state (slots, taps - 1, channels): the inputs of the sequence's last taps - 1 tokens. */
+ * state (slots, taps, channels): position p's inputs in row p % taps. */
 int iron_short_conv(const void* x, const uint16_t* taps_w, const uint16_t* a_log, const uint16_t* dt_bias, void* state,
                     const int* spans, float* out, int slots, int rows, int stride, int heads, int kv_heads, int dim,
                     int vdim, int taps, int b_at, int a_at, int is_float, void* stream);
@@ -431,6 +431,27 @@ int iron_head_gate(const float* o, const void* gate, const uint16_t* gain, void*
 int iron_mha_window(const void* x, void* keys, void* values, const float* bias, const int* spans, void* out, int slots,
                     int rows, int stride, int heads, int kv_heads, int dim, int vdim, int window, int ring, float scale,
                     int out_stride, int out_at, float out_scale, int single, int is_float, void* stream);
+/* One token a slot (no span of more than one row) through a mixer, bf16, in one launch; each computes what
+ * the entry points above compute in turn, on the same states.
+ * decode_mixed (one slot): iron_token_shift and `count` (up to 8) products y[i] = W[i] (rows[i], K) times
+ * the blend by mu[i], or the row itself (mu[i] NULL).  The four arrays are host memory, read at the call.
+ * decode_parallel: iron_low_rank_decay, iron_time_mix and iron_head_gate (columns mix_at ..; mix_dim a
+ * power of two from 16) beside iron_mha_window (columns win_at ..; widths multiples of 8).
+ * decode_delta: iron_short_conv, iron_delta_rule and iron_head_gate (shared gain; vdim a power of two
+ * from 16). */
+int iron_decode_mixed_bf16(const uint16_t* h, uint16_t* carry, const int* spans, int K, int count, const void* const* W,
+                           void* const* y, const void* const* mu, const int* rows, void* stream);
+int iron_decode_parallel_bf16(const uint16_t* r, const uint16_t* k, const uint16_t* v, const uint16_t* gate,
+                              const uint16_t* z, const uint16_t* w2, const uint16_t* w0, const uint16_t* u,
+                              const uint16_t* norm, float* memory, int mix_heads, int mix_dim, int rank, float eps,
+                              float mix_scale, int mix_at, const uint16_t* x, uint16_t* keys, uint16_t* values,
+                              const float* bias, int stride, int heads, int kv_heads, int dim, int vdim, int window,
+                              int ring, float scale, float out_scale, int win_at, const int* spans, uint16_t* out,
+                              int slots, int rows, int out_stride, void* stream);
+int iron_decode_delta_bf16(const uint16_t* x, const uint16_t* taps_w, const uint16_t* a_log, const uint16_t* dt_bias,
+                           const uint16_t* norm, uint16_t* inputs, float* state, const int* spans, uint16_t* out,
+                           int slots, int rows, int stride, int heads, int kv_heads, int dim, int vdim, int taps,
+                           int gate_at, int b_at, int a_at, float eps, void* stream);
 /* iron_sample_bf16 for every slot that has rows: logits (slots, logits_stride), drawn at the position p
  * of the span's last row by draw row slot * steps + p, recorded in record[slot * steps + p]; the span
  * then becomes {slot, 1, p + 1}.  workspace: slots times iron_sample_workspace_bytes(n). */

@@ -101,6 +101,13 @@ SIGNATURES = {
     "iron_delta_rule": (c_int, [_P] * 4 + [c_int] * 6 + [_P]),
     "iron_head_gate": (c_int, [_P] * 4 + [c_int] * 8 + [c_float, c_float, c_int, _P, _P]),
     "iron_mha_window": (c_int, [_P] * 6 + [c_int] * 9 + [c_float, c_int, c_int, c_float, c_int, c_int, _P]),
+    "iron_decode_mixed_bf16": (c_int, [_P, _P, _P, c_int, c_int, _P, _P, _P, _P, _P]),
+    "iron_decode_parallel_bf16": (
+        c_int,
+        [_P] * 10 + [c_int] * 3 + [c_float, c_float, c_int] + [_P] * 4 + [c_int] * 7 + [c_float, c_float, c_int, _P, _P]
+        + [c_int] * 3 + [_P],
+    ),
+    "iron_decode_delta_bf16": (c_int, [_P] * 9 + [c_int] * 11 + [c_float, _P]),
     "iron_sample_slots_bf16": (c_int, [_P, c_int, c_int, _P, c_int, c_int, c_int, _P, c_int, _P, _P, _P, _P]),
     "iron_eval_words": (c_int, [_P, c_int, _P, c_int, _P]),
 }

@@ -24,8 +24,16 @@ in a prompt chunk's version (several rows, 64-wide heads),
   GEMM, ElementwiseAdd / AXPY (the residual)             => iron_gemm_residual_bf16
   ... few rows over a long K, and the RMSNorm after them => iron_gemm_residual_norm_bf16
 
+in a batched decoder's decode step (bf16; a float32 stream, layers with a state),
+
+  [GEMV,] TokenShift, GEMV of its blends (one slot)      => iron_decode_mixed_bf16
+  LowRankDecay, TimeMix, HeadGate, WindowMHA             => iron_decode_parallel_bf16
+  ShortConv, DeltaRule, HeadGate                         => iron_decode_delta_bf16
+  GEMV gate, GEMV up, SiLU / GELU (tanh) / ReLU, Mul     => iron_gemv_fused_bf16 (epilogue 2 / 3 / 6)
+
 and in either,
 
+  StreamAdd, StreamNorm                                  => iron_stream_rows
   RMSNorm, ElementwiseAdd (a sandwich layer's residual)  => iron_rmsnorm_add_bf16
 
 A run is fused only if every intermediate it hides is read by nothing else.
@@ -38,6 +46,8 @@ from collections import Counter
 from collections.abc import Callable
 from typing import Any
 
+from ..bf16 import bfloat16
+
 
 @dataclasses.dataclass
 class Fused:
@@ -49,6 +59,18 @@ class Fused:
     launch: Callable[[], None]
     launches: int = 1      # 0: a step other launches made needless (nothing runs for it)
     scratch_bytes: int = 0  # device memory of its own the launch needs, live over the run
+
+
+# a gated feed-forward's activation steps: the C ABI's name, and gemv_fused's epilogue
+_GATES = {"SiLU": ("silu", 2), "GELU": ("gelu_tanh", 3), "ReLU": ("relu", 6)}
+
+
+def _gate(step) -> tuple[str, int] | None:
+    """The fused launches' names for an activation step they compute, or None."""
+    name = type(step.op).__name__
+    if name not in _GATES or (name == "GELU" and step.op.approximate != "tanh"):
+        return None
+    return _GATES[name]
 
 
 class _Anything:
@@ -131,7 +153,7 @@ def plan(recording, tensor: Callable[[Any], Any], word: Callable[[Any], Any],
             return None
         s, sl, ml = steps[j], steps[j + 1], steps[j + 2]
         if not (_name(s) == "GEMM"
-                and (_name(sl) == "SiLU" or (_name(sl) == "GELU" and sl.op.approximate == "tanh"))
+                and _gate(sl) is not None
                 and _name(ml) == "ElementwiseMul"
                 and s.op.b_col_maj and not s.op.c_col_maj and "valid_k" not in s.values
                 and s.op.M >= 64 and s.op.N >= 64 and s.op.K % 64 == 0):
@@ -161,8 +183,102 @@ def plan(recording, tensor: Callable[[Any], Any], word: Callable[[Any], Any],
                 return None
         args = dict(A=tensor(s.inputs["A"]), B=tensor(s.inputs["B"]), G=tensor(gate), C=tensor(ml.outputs["y"]))
         kw = dict(M=s.op.M, N=s.op.N, K=s.op.K, valid=word(gv),
-                  activation="silu" if _name(sl) == "SiLU" else "gelu_tanh")
+                  activation=_gate(sl)[0])
         return args, kw
+
+    def gated_rows_at(j):
+        """``(args, kw)`` of ``iron_gemv_fused_bf16`` where the four steps from ``j`` are one row's gate and up
+        projections (of one input), the gate's activation and the product, or None."""
+        if j + 3 >= len(steps):
+            return None
+        gg, gu, si, mu = steps[j : j + 4]
+        if not (gemv_row(gg) and gemv_row(gu, gg.inputs["B"]) and _gate(si) is not None and _name(mu) == "ElementwiseMul"):
+            return None
+        g, u = gg.outputs["C"], gu.outputs["C"]
+        if not (_same(si.inputs["x"], g) and once(g) and once(u) and once(si.outputs["y"]) and not si.values and not mu.values
+                and _same(mu.inputs["a"], si.outputs["y"]) and _same(mu.inputs["b"], u) and gg.op.M == gu.op.M
+                and gg.op.K == gu.op.K and _plain(mu.outputs["y"])):
+            return None
+        args = dict(W=tensor(gg.inputs["A"]), W2=tensor(gu.inputs["A"]), x=tensor(gg.inputs["B"]).reshape(-1),
+                    y=tensor(mu.outputs["y"]).reshape(-1))
+        return args, dict(M=gg.op.M, K=gg.op.K, epilogue=_gate(si)[1])
+
+    def mixed_at(j):
+        """The launch for a token shift of one row from step ``j`` on, with a projection of the shift's own input
+        ahead of it (if there is one) and those of its blends behind it -- or None."""
+        ahead = gemv_row(steps[j])
+        at = j + 1 if ahead else j
+        shift = steps[at] if at < len(steps) else None
+        if (shift is None or _name(shift) != "TokenShift" or shift.op.rows != 1 or shift.op.slots != 1
+                or shift.op.dtype is not bfloat16 or shift.op.cols % 8):
+            return None
+        h, blends, K = shift.inputs["h"], shift.outputs["mixed"], shift.op.cols
+        if ahead and not _same(steps[j].inputs["B"], h):
+            return None
+        behind = steps[at + 1 : at + 1 + shift.op.mixes]
+        if (len(behind) != shift.op.mixes or shift.op.mixes > 7 or not once(blends, shift.op.mixes)
+                or not all(gemv_row(g) and g.inputs["B"].buffer is blends.buffer and g.inputs["B"].elements == K
+                           and g.inputs["B"].offset % K == 0 and g.op.K == K for g in behind)):
+            return None
+        mu = tensor(shift.inputs["mu"])
+        gemvs = ([steps[j]] if ahead else []) + behind
+        products = [(tensor(g.inputs["A"]), tensor(g.outputs["C"]).reshape(-1),
+                     mu[g.inputs["B"].offset // K] if g is not steps[j] or not ahead else None) for g in gemvs]
+        args = dict(h=tensor(h).reshape(-1), carry=tensor(shift.inputs["carry"]).reshape(-1),
+                    spans=tensor(shift.inputs["spans"]), products=products)
+        return Fused("decode_mixed", j, len(gemvs) + 1, lambda a=args: kernels.decode_mixed(**a, k=K))
+
+    def gate_behind(o, gate):
+        """Whether ``gate`` is the head norm and gate of a recurrence's output, read by nothing else."""
+        return (_name(gate) == "HeadGate" and _same(gate.inputs["o"], o) and once(o) and not gate.values
+                and gate.op.dtype is bfloat16)
+
+    def parallel_at(j):
+        """The launch for a decode step's time mixing beside its windowed attention -- or None."""
+        if j + 3 >= len(steps):
+            return None
+        decay, mix, gate, win = steps[j : j + 4]
+        if [_name(t) for t in (mix, gate, win)] != ["TimeMix", "HeadGate", "WindowMHA"] or decay.values or not win.op.single:
+            return None
+        D, w = mix.op.dim, win.op
+        if not (_same(mix.inputs["log_decay"], decay.outputs["y"]) and once(decay.outputs["y"])
+                and gate_behind(mix.outputs["o"], gate) and mix.op.dtype is bfloat16 and w.dtype is bfloat16
+                and 16 <= D <= 256 and D & (D - 1) == 0 and w.dim % 8 == 0 and w.vdim % 8 == 0 and w.stride % 8 == 0
+                and gate.op.gains == gate.op.o_width and gate.op.gate_at == 0 and gate.op.gate_width == gate.op.o_width
+                and _same(win.inputs["y"], gate.outputs["y"]) and win.inputs["spans"].buffer is mix.inputs["spans"].buffer):
+            return None
+        flat = dict(r=mix.inputs["r"], k=mix.inputs["k"], v=mix.inputs["v"], gate=gate.inputs["gate"], z=decay.inputs["z"],
+                    w2=decay.inputs["up"], w0=decay.inputs["base"], u=mix.inputs["u"], norm=gate.inputs["gain"],
+                    memory=mix.inputs["state"], x=win.inputs["x"], keys=win.inputs["keys"], values=win.inputs["values"],
+                    bias=win.inputs["bias"], spans=win.inputs["spans"], out=win.inputs["y"])
+        args = {n: tensor(h) for n, h in flat.items()}
+        kw = dict(slots=w.slots, rows=w.rows, mix_heads=mix.op.heads, mix_dim=D, rank=decay.op.rank,
+                  eps=float(gate.op.epsilon), mix_scale=float(gate.op.scale), mix_at=gate.op.at, stride=w.stride, heads=w.heads,
+                  kv_heads=w.kv_heads, dim=w.dim, vdim=w.vdim, window=w.window, ring=w.ring, scale=float(w.scale),
+                  out_scale=float(w.out_scale), win_at=w.at, out_stride=w.width)
+        return Fused("decode_parallel", j, 4, lambda a=args, kw=kw: kernels.decode_parallel(**a, **kw))
+
+    def delta_at(j):
+        """The launch for a decode step's convolution, delta rule, head norm and gate -- or None.  The step is
+        told by its rows: one a slot (a prompt's portion carries a bound)."""
+        if j + 2 >= len(steps):
+            return None
+        conv, rule, gate = steps[j : j + 3]
+        c = conv.op
+        if not (_name(rule) == "DeltaRule" and not conv.values and c.rows == c.slots and c.dtype is bfloat16
+                and _same(rule.inputs["x"], conv.outputs["y"]) and once(conv.outputs["y"]) and gate_behind(rule.outputs["o"], gate)
+                and 16 <= c.vdim <= 256 and c.vdim & (c.vdim - 1) == 0 and gate.op.gains == c.vdim and gate.op.at == 0
+                and gate.op.width == gate.op.o_width and gate.op.scale == 1.0
+                and _same(gate.inputs["gate"], conv.inputs["x"])
+                and rule.inputs["spans"].buffer is conv.inputs["spans"].buffer):
+            return None
+        flat = dict(x=conv.inputs["x"], taps_w=conv.inputs["weight"], a_log=conv.inputs["a_log"], dt_bias=conv.inputs["dt_bias"],
+                    norm=gate.inputs["gain"], inputs=conv.inputs["state"], state=rule.inputs["state"],
+                    spans=conv.inputs["spans"], out=gate.outputs["y"])
+        args = {n: tensor(h) for n, h in flat.items()}
+        kw = dict(slots=c.slots, rows=c.rows, stride=c.stride, heads=c.heads, kv_heads=c.kv_heads, dim=c.dim, vdim=c.vdim,
+                  taps=c.taps, gate_at=gate.op.gate_at, b_at=c.b_at, a_at=c.a_at, eps=float(gate.op.epsilon))
+        return Fused("decode_delta", j, 3, lambda a=args, kw=kw: kernels.decode_delta(**a, **kw))
 
     def same_data(a, b) -> bool:
         return (a is not None and b is not None and a.buffer is b.buffer and a.offset == b.offset
@@ -480,6 +596,25 @@ def plan(recording, tensor: Callable[[Any], Any], word: Callable[[Any], Any],
                             residual=tensor(other).reshape(-1), y=tensor(mu.outputs["y"]).reshape(-1))
                 kw = dict(M=s.op.M, K=s.op.K, epilogue=5 if _name(ac) == "SiLU" else 4)
                 got = Fused("gemv_act_mul", i, 3, lambda a=args, kw=kw: kernels.gemv_fused(**a, **kw))
+        elif _name(s) == "StreamAdd" and i + 1 < len(steps) and _name(steps[i + 1]) == "StreamNorm":
+            # a block's output into the stream and the next block's norm out of it: one pass over the row
+            nm = steps[i + 1]
+            if (_same_view(nm.inputs["x"], s.outputs["x"]) and nm.op.dtype is s.op.dtype and nm.op.epsilon == s.op.epsilon
+                    and (nm.op.rows, nm.op.cols) == (s.op.rows, s.op.cols) and nm.values.get("valid") == s.values.get("valid")
+                    and set(nm.values) <= {"valid"} and set(s.values) <= {"valid"}):
+                args = dict(x=tensor(s.inputs["x"]), y=tensor(s.inputs["y"]), back_gain=tensor(s.inputs["weight"]),
+                            h=tensor(nm.outputs["y"]), gain=tensor(nm.inputs["weight"]))
+                kw = dict(rows=s.op.rows, cols=s.op.cols, eps=float(s.op.epsilon), valid=word(s.values.get("valid")))
+                got = Fused("stream_add_norm", i, 2, lambda a=args, kw=kw: kernels.stream_rows(**a, **kw))
+        elif _name(s) == "LowRankDecay":
+            got = parallel_at(i)
+        elif _name(s) == "ShortConv":
+            got = delta_at(i)
+        elif (_name(s) == "TokenShift" or gemv_row(s)) and (got := mixed_at(i)) is not None:
+            pass
+        elif gemv_row(s) and (gated := gated_rows_at(i)) is not None:
+            args, kw = gated
+            got = Fused("gemv_gate_up_mul", i, 4, lambda a=args, kw=kw: kernels.gemv_fused(**a, **kw))
         elif gemv_row(s) and i + 1 < len(steps) and _name(steps[i + 1]) in ("ElementwiseAdd", "AXPY"):
             ad = steps[i + 1]
             c = s.outputs["C"]

@@ -266,6 +266,74 @@ __global__ __launch_bounds__(256) void decode_qkv_kernel(
 }
 
 
+// Up to MIX_SEGMENTS projections of one row, each of its own blend of the row and the one before it,
+// h + (before - h) * mu, or (no mu) of the row itself: a token shift and its projections, and the
+// projections beside it that read the same row, in one launch.  `carry` (2, K) keeps position p's row in
+// row p % 2: the block that leaves this one's replaces no row that another reads.
+constexpr int MIX_SEGMENTS = 8;
+struct MixSegments {
+  const bf16_t* W[MIX_SEGMENTS];
+  bf16_t* y[MIX_SEGMENTS];
+  const bf16_t* mu[MIX_SEGMENTS];
+  int rows[MIX_SEGMENTS];
+  int block0[MIX_SEGMENTS + 1];   // the first block of each segment
+  int count;
+};
+
+template <int RPW, int CH>
+__global__ __launch_bounds__(256) void decode_mixed_kernel(MixSegments seg, const bf16_t* __restrict__ h, bf16_t* __restrict__ carry,
+                                                           const int* __restrict__ spans, int K) {
+  __shared__ float part[4][RPW];
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  int which = 0;
+#pragma unroll
+  for (int i = 1; i < MIX_SEGMENTS; ++i)
+    if (i < seg.count && (int)blockIdx.x >= seg.block0[i]) which = i;
+  const bf16_t *W = seg.W[which], *mu = seg.mu[which];
+  bf16_t* y = seg.y[which];
+  const int M = seg.rows[which], row0 = ((int)blockIdx.x - seg.block0[which]) * RPW;
+  const int4 span = *reinterpret_cast<const int4*>(spans);
+  uint4 w[RPW][CH], hv[CH], bv[CH], mv[CH];
+#pragma unroll
+  for (int i = 0; i < CH; ++i) {
+    const int c = threadIdx.x + 256 * i;
+    hv[i] = c < (K >> 3) ? reinterpret_cast<const uint4*>(h)[c] : make_uint4(0, 0, 0, 0);
+    mv[i] = (mu != nullptr && c < (K >> 3)) ? reinterpret_cast<const uint4*>(mu)[c] : make_uint4(0, 0, 0, 0);
+  }
+#pragma unroll
+  for (int r = 0; r < RPW; ++r) load_row<CH>(W + (size_t)min(row0 + r, M - 1) * K, K, w[r]);
+  const bool live = span.y > 0, older = live && span.z > 0;
+  if (mu != nullptr || blockIdx.x == 0) {
+    const uint4* before = reinterpret_cast<const uint4*>(carry + (size_t)((span.z - 1) & 1) * K);
+#pragma unroll
+    for (int i = 0; i < CH; ++i) {
+      const int c = threadIdx.x + 256 * i;
+      bv[i] = (older && c < (K >> 3)) ? before[c] : make_uint4(0, 0, 0, 0);
+      if (blockIdx.x == 0 && live && c < (K >> 3)) reinterpret_cast<uint4*>(carry + (size_t)(span.z & 1) * K)[c] = hv[i];
+    }
+    if (mu != nullptr) {
+#pragma unroll
+      for (int i = 0; i < CH; ++i) {
+        float a[8], b[8], m[8];
+        unpack8(hv[i], a);
+        unpack8(bv[i], b);
+        unpack8(mv[i], m);
+#pragma unroll
+        for (int j = 0; j < 8; ++j) a[j] = a[j] + (b[j] - a[j]) * m[j];
+        hv[i] = pack8(a);   // the blend's own rounding
+      }
+    }
+  }
+#pragma unroll
+  for (int r = 0; r < RPW; ++r) {
+    const float a = wave_sum(dot_row<CH>(w[r], hv));
+    if (lane == 0) part[wave][r] = a;
+  }
+  __syncthreads();
+  if (threadIdx.x < RPW && row0 + (int)threadIdx.x < M)
+    y[row0 + threadIdx.x] = f32_to_bf16(part[0][threadIdx.x] + part[1][threadIdx.x] + part[2][threadIdx.x] + part[3][threadIdx.x]);
+}
+
 // Between a token's q/k/v projections and its attention, where the heads are normed one by one (q and
 // k with learned gains, v without: Gemma's): RMSNorm per head, RoPE on q and k, and k's and v's rows
 // into their cache rows (twice where the cache is a ring: the slot and its mirror) -- up to nine
@@ -541,5 +609,32 @@ extern "C" int iron_decode_heads_bf16(const uint16_t* q, const uint16_t* k, cons
   a.cache_rows = cache_rows; a.heads = heads; a.kv_heads = kv_heads; a.d = d;
   const int blocks = heads + (k != nullptr ? 2 * kv_heads : 0);
   hipLaunchKernelGGL(decode_heads_kernel, dim3(blocks), dim3(256), 0, (hipStream_t)stream, a);
+  IRON_LAUNCH_CHECK();
+}
+
+extern "C" int iron_decode_mixed_bf16(const uint16_t* h, uint16_t* carry, const int* spans, int K, int count,
+                                      const void* const* W, void* const* y, const void* const* mu, const int* rows, void* stream) {
+  IRON_REQUIRE(h && carry && spans && W && y && mu && rows, "decode_mixed: null operand");
+  IRON_REQUIRE(count > 0 && count <= MIX_SEGMENTS, "decode_mixed: %d projections, from 1 to %d", count, MIX_SEGMENTS);
+  IRON_REQUIRE(K > 0 && K % 8 == 0 && K <= 8192, "decode_mixed: K (%d) is a multiple of 8 up to 8192", K);
+  IRON_REQUIRE((((uintptr_t)h | (uintptr_t)carry | (uintptr_t)spans) & 15) == 0, "decode_mixed: operands must be 16-byte aligned");
+  MixSegments seg{};
+  const int ch = K <= 2048 ? 1 : (K <= 4096 ? 2 : 4), rpw = ch == 1 ? 2 : 1;
+  int blocks = 0;
+  for (int i = 0; i < count; ++i) {
+    IRON_REQUIRE(W[i] && y[i] && rows[i] > 0, "decode_mixed: projection %d: null operand or no rows", i);
+    IRON_REQUIRE((((uintptr_t)W[i] | (uintptr_t)mu[i]) & 15) == 0, "decode_mixed: operands must be 16-byte aligned");
+    seg.W[i] = (const bf16_t*)W[i];
+    seg.y[i] = (bf16_t*)y[i];
+    seg.mu[i] = (const bf16_t*)mu[i];
+    seg.rows[i] = rows[i];
+    seg.block0[i] = blocks;
+    blocks += (rows[i] + rpw - 1) / rpw;
+  }
+  seg.count = count;
+  hipStream_t s = (hipStream_t)stream;
+  if (ch == 1) hipLaunchKernelGGL((decode_mixed_kernel<2, 1>), dim3(blocks), dim3(256), 0, s, seg, h, carry, spans, K);
+  else if (ch == 2) hipLaunchKernelGGL((decode_mixed_kernel<1, 2>), dim3(blocks), dim3(256), 0, s, seg, h, carry, spans, K);
+  else hipLaunchKernelGGL((decode_mixed_kernel<1, 4>), dim3(blocks), dim3(256), 0, s, seg, h, carry, spans, K);
   IRON_LAUNCH_CHECK();
 }

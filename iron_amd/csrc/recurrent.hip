@@ -32,11 +32,13 @@ __global__ __launch_bounds__(256) void token_shift_kernel(const T* __restrict__ 
   const int first = blockIdx.x * SHIFT_TILE;
   if (first >= s.rows) return;
   const int last = min(s.rows, first + SHIFT_TILE);
-  T* held = carry + (size_t)blockIdx.y * cols;
+  // Two rows a slot, by a position's parity: a decode step's launch reads one and leaves the other.
+  T* held = carry + (size_t)blockIdx.y * 2 * cols;
+  const int old_row = (s.start - 1) & 1, new_row = (s.start + s.rows - 1) & 1;
   for (int c = threadIdx.x * VEC; c < cols; c += 256 * VEC) {
     float before[VEC];
     if (first > 0) load_vec<VEC>(h + (size_t)(s.row0 + first - 1) * cols + c, before);
-    else if (s.start > 0) load_vec<VEC>(held + c, before);
+    else if (s.start > 0) load_vec<VEC>(held + old_row * cols + c, before);
     else {
 #pragma unroll
       for (int j = 0; j < VEC; ++j) before[j] = 0.f;
@@ -44,7 +46,7 @@ __global__ __launch_bounds__(256) void token_shift_kernel(const T* __restrict__ 
     if (first == 0) {   // the span's last row is what the next one starts from
       float end[VEC];
       load_vec<VEC>(h + (size_t)(s.row0 + s.rows - 1) * cols + c, end);
-      store_vec<VEC>(held + c, end);
+      store_vec<VEC>(held + new_row * cols + c, end);
     }
     for (int i = first; i < last; ++i) {
       float now[VEC];
@@ -231,11 +233,11 @@ __global__ __launch_bounds__(256) void short_conv_kernel(const T* __restrict__ x
   const int len = is_v ? c.vdim : c.dim;
   const int at = is_v ? 2 * qk + (seg - 2 * c.kv_heads) * c.vdim : seg * c.dim;
   const int past = c.taps - 1;
-  T* held = state + (size_t)slot * past * channels;
+  T* held = state + (size_t)slot * c.taps * channels;   // position p's input in row p % taps
   // The input at place p of the span: a row of this call, the slot's state before it, zero before 0.
   auto input = [&](int p, int ch) -> float {
     if (p >= 0) return load_one(x + (size_t)(s.row0 + p) * c.stride + ch);
-    return s.start + p >= 0 ? load_one(held + (size_t)(past + p) * channels + ch) : 0.f;
+    return s.start + p >= 0 ? load_one(held + (size_t)((s.start + p) % c.taps) * channels + ch) : 0.f;
   };
   for (int p = first + wave; p < last; p += 4) {
     float f[4];
@@ -262,10 +264,11 @@ __global__ __launch_bounds__(256) void short_conv_kernel(const T* __restrict__ x
     for (int e = 0; e < 4; ++e)
       if (lane + 64 * e < len) to[lane + 64 * e] = f[e] * scale;
   }
-  if (first == 0) {   // no other block reads these channels' state; ascending, so a row is read before it is replaced
+  if (first == 0) {   // no other block reads these channels' state
     __syncthreads();
     for (int j = threadIdx.x; j < len; j += 256)
-      for (int m = 0; m < past; ++m) store_one(held + (size_t)m * channels + at + j, input(s.rows - past + m, at + j));
+      for (int p = max(0, s.rows - past); p < s.rows; ++p)
+        store_one(held + (size_t)((s.start + p) % c.taps) * channels + at + j, input(p, at + j));
   }
 }
 
@@ -460,7 +463,7 @@ extern "C" int iron_time_mix(const void* r, const void* k, const void* v, const 
 extern "C" int iron_short_conv(const void* x, const uint16_t* taps_w, const uint16_t* a_log, const uint16_t* dt_bias,
                                void* state, const int* spans, float* out, int slots, int rows, int stride, int heads,
                                int kv_heads, int dim, int vdim, int taps, int b_at, int a_at, int is_float, void* stream) {
-  IRON_REQUIRE(x && taps_w && a_log && dt_bias && out && (state || taps == 1), "short_conv: null operand");
+  IRON_REQUIRE(x && taps_w && a_log && dt_bias && out && state, "short_conv: null operand");
   IRON_SPANS_REQUIRE("short_conv");
   IRON_REQUIRE(heads > 0 && kv_heads > 0 && heads % kv_heads == 0, "short_conv: kv_heads (%d) must divide heads (%d)", kv_heads, heads);
   IRON_REQUIRE(dim > 0 && dim <= 256 && vdim > 0 && vdim <= 256, "short_conv: dim (%d) and vdim (%d) from 1 to 256", dim, vdim);

@@ -7,6 +7,7 @@ raises ``IronHipError`` on refusal.  Nothing here computes.
 
 from __future__ import annotations
 
+import ctypes
 import math
 
 import torch
@@ -665,7 +666,7 @@ def token_shift(h, mu, carry, spans, mixed, *, slots, rows, cols, mixes):
     is_float = _act(h, rows * cols, "h")
     _bf16(mu, mixes * cols, "mu")
     _same_kind(is_float, carry=carry, mixed=mixed)
-    _act(carry, slots * cols, "carry")
+    _act(carry, slots * 2 * cols, "carry")
     _act(mixed, mixes * rows * cols, "mixed")
     check(lib().iron_token_shift(ptr(h), ptr(mu), ptr(carry), _spans(spans, slots), ptr(mixed), slots, rows, cols, mixes,
                                  int(is_float), current_stream()), "iron_token_shift")
@@ -702,7 +703,7 @@ def short_conv(x, taps_w, a_log, dt_bias, state, spans, out, *, slots, rows, str
     _bf16(a_log, heads, "a_log")
     _bf16(dt_bias, heads, "dt_bias")
     _same_kind(is_float, state=state)
-    _act(state, slots * max(taps - 1, 1) * channels, "state")
+    _act(state, slots * taps * channels, "state")
     _f32(out, rows * (channels + 2 * heads), "out")
     check(lib().iron_short_conv(ptr(x), ptr(taps_w), ptr(a_log), ptr(dt_bias), ptr(state), _spans(spans, slots), ptr(out),
                                 slots, rows, stride, heads, kv_heads, dim, vdim, taps, b_at, a_at, int(is_float),
@@ -740,6 +741,67 @@ def mha_window(x, keys, values, bias, spans, out, *, slots, rows, stride, heads,
     check(lib().iron_mha_window(ptr(x), ptr(keys), ptr(values), ptr(bias), _spans(spans, slots), ptr(out), slots, rows, stride,
                                 heads, kv_heads, dim, vdim, window, ring, float(scale), out_stride, out_at, float(out_scale),
                                 int(single), int(is_float), current_stream()), "iron_mha_window")
+
+
+def decode_mixed(h, carry, spans, products, *, k):
+    """A token shift and the projections of its blends, one row, one launch.  ``products``: (weight, output,
+    mu row or None) each."""
+    _bf16(h, k, "h")
+    _bf16(carry, 2 * k, "carry")
+    n = len(products)
+    for w, y, mu in products:
+        _dev(w, "weight")
+        if w.numel() != y.numel() * k:
+            raise ValueError(f"decode_mixed: a weight of {w.numel()} elements for {y.numel()} rows of {k}")
+        _dev(y, "output")
+        if mu is not None:
+            _bf16(mu, k, "mu")
+    pointers = ctypes.c_void_p * n
+    check(lib().iron_decode_mixed_bf16(ptr(h), ptr(carry), _spans(spans, 1), k, n, pointers(*(ptr(w) for w, _, _ in products)),
+                                       pointers(*(ptr(y) for _, y, _ in products)), pointers(*(ptr(m) for _, _, m in products)),
+                                       (ctypes.c_int * n)(*(y.numel() for _, y, _ in products)), current_stream()),
+          "iron_decode_mixed_bf16")
+
+
+def decode_parallel(r, k, v, gate, z, w2, w0, u, norm, memory, x, keys, values, bias, spans, out, *, slots, rows, mix_heads,
+                    mix_dim, rank, eps, mix_scale, mix_at, stride, heads, kv_heads, dim, vdim, window, ring, scale, out_scale,
+                    win_at, out_stride):
+    """A decode step's decay, time mixing, head norm and gate beside its windowed attention."""
+    inner = mix_heads * mix_dim
+    for t, name in ((r, "r"), (k, "k"), (v, "v"), (gate, "gate")):
+        _bf16(t, rows * inner, name)
+    _bf16(z, rows * rank, "z")
+    _bf16(w2, inner * rank, "w2")
+    for t, name in ((w0, "w0"), (u, "u"), (norm, "norm")):
+        _bf16(t, inner, name)
+    _f32(memory, slots * inner * mix_dim, "memory")
+    _bf16(x, rows * stride, "x")
+    _bf16(keys, slots * ring * kv_heads * dim, "keys")
+    _bf16(values, slots * ring * kv_heads * vdim, "values")
+    _f32(bias, heads * window, "bias")
+    _bf16(out, rows * out_stride, "out")
+    check(lib().iron_decode_parallel_bf16(ptr(r), ptr(k), ptr(v), ptr(gate), ptr(z), ptr(w2), ptr(w0), ptr(u), ptr(norm),
+                                          ptr(memory), mix_heads, mix_dim, rank, float(eps), float(mix_scale), mix_at, ptr(x),
+                                          ptr(keys), ptr(values), ptr(bias), stride, heads, kv_heads, dim, vdim, window, ring,
+                                          float(scale), float(out_scale), win_at, _spans(spans, slots), ptr(out), slots, rows,
+                                          out_stride, current_stream()), "iron_decode_parallel_bf16")
+
+
+def decode_delta(x, taps_w, a_log, dt_bias, norm, inputs, state, spans, out, *, slots, rows, stride, heads, kv_heads, dim, vdim,
+                 taps, gate_at, b_at, a_at, eps):
+    """A decode step's short convolution, gated delta rule, head norm and gate."""
+    channels = 2 * kv_heads * dim + heads * vdim
+    _bf16(x, rows * stride, "x")
+    _bf16(taps_w, channels * taps, "taps_w")
+    _bf16(a_log, heads, "a_log")
+    _bf16(dt_bias, heads, "dt_bias")
+    _bf16(norm, vdim, "norm")
+    _bf16(inputs, slots * taps * channels, "inputs")
+    _f32(state, slots * heads * dim * vdim, "state")
+    _bf16(out, rows * heads * vdim, "out")
+    check(lib().iron_decode_delta_bf16(ptr(x), ptr(taps_w), ptr(a_log), ptr(dt_bias), ptr(norm), ptr(inputs), ptr(state),
+                                       _spans(spans, slots), ptr(out), slots, rows, stride, heads, kv_heads, dim, vdim, taps,
+                                       gate_at, b_at, a_at, float(eps), current_stream()), "iron_decode_delta_bf16")
 
 
 def sample_slots(logits, spans, draws, token, record, workspace, *, n, stride, slots, batch_rows, steps, k_max=64):

@@ -82,8 +82,10 @@ class WindowAttention(iron.Graph):
         return {"keys": iron.state((slots, self.window, self.kv_heads, self.dim), self.dtype),
                 "values": iron.state((slots, self.window, self.kv_heads, self.vdim), self.dtype)}
 
-    def body(self, h, call, state, mixed, at=0):
-        x = as_rows(self.qkv(h), h.shape[0])
+    def project(self, h):
+        return as_rows(self.qkv(h), h.shape[0])
+
+    def body(self, x, call, state, mixed, at=0):
         return WindowMHA.step(x, self.by_distance, call.spans, state["keys"], state["values"], mixed, scale=self.scale,
                               out_scale=self.out_scale, at=at, single=not call.prompt, dtype=self.dtype)[2]
 
@@ -114,7 +116,7 @@ class TimeMixing(iron.Graph):
         return self.heads * self.dim
 
     def states(self, slots: int) -> dict:
-        return {"before": iron.state((slots, self.width), self.dtype),
+        return {"before": iron.state((slots, 2, self.width), self.dtype),
                 "memory": iron.state((slots, self.heads, self.dim, self.dim), np.float32)}
 
     def body(self, h, call, state, width, at=0):
@@ -142,8 +144,10 @@ class ParallelMixer(iron.Graph):
         return {**self.left.states(slots), **self.right.states(slots)}
 
     def body(self, h, call, state):
+        # All projections of h, then both mixers: the runs a decode step launches as one each.
+        x = self.left.project(h)
         mixed = self.right(h, call, state, self.out.in_features, at=self.left.out_width)
-        return self.out(self.left(h, call, state, mixed))
+        return self.out(self.left(x, call, state, mixed))
 
 
 class DeltaMixer(iron.Graph):
@@ -168,7 +172,7 @@ class DeltaMixer(iron.Graph):
         pass
 
     def states(self, slots: int) -> dict:
-        return {"inputs": iron.state((slots, max(self.taps - 1, 1), self.channels), self.dtype),
+        return {"inputs": iron.state((slots, self.taps, self.channels), self.dtype),
                 "memory": iron.state((slots, self.heads, self.dim, self.vdim), np.float32)}
 
     def body(self, h, call, state):

@@ -28,7 +28,8 @@ class _Spanned(Operator):
 
 class TokenShift(_Spanned):
     """``mixed[m] = h + (before - h) * mu[m]``: each of several projections reads its own blend of a token
-    and the one before it (zeros ahead of the first).  ``carry`` keeps each slot's last row."""
+    and the one before it (zeros ahead of the first).  ``carry`` keeps position
+    p's row in row ``p % 2`` of its slot."""
 
     slots: int = param()
     rows: int = param()
@@ -37,7 +38,7 @@ class TokenShift(_Spanned):
     dtype: Any = param(default=bfloat16, repr=False)
     h = In(rows, cols, dtype=dtype)
     mu = In(mixes, cols)
-    carry = InOut(slots, cols, dtype=dtype)
+    carry = InOut(slots, 2, cols, dtype=dtype)
     spans = In(slots, 4, dtype=np.int32)
     mixed = Out(mixes, rows, cols, dtype=dtype)
 
@@ -152,19 +153,18 @@ class _DeltaShape(_Spanned):
 class ShortConv(_DeltaShape):
     """From a packed projection ``[q | k | v | .. b .. | .. a ..]``: a short causal convolution per channel
     and SiLU on q, k and v, unit q (times ``dim ** -0.5``) and k per head, and the step's decay and write
-    strength.  ``state`` keeps each slot's last ``taps - 1`` inputs."""
+    strength.  ``state`` keeps position p's inputs in row ``p % taps`` of its slot."""
 
     stride: int = param()
     taps: int = param()
     b_at: int = param(array=True)
     a_at: int = param(array=True)
     dtype: Any = param(default=bfloat16, repr=False)
-    past: int = param(derive=lambda op: max(op.taps - 1, 1), repr=False)
     x = In(_DeltaShape.rows, stride, dtype=dtype)
     weight = In(_DeltaShape.channels, taps)
     a_log = In(_DeltaShape.heads)
     dt_bias = In(_DeltaShape.heads)
-    state = InOut(_DeltaShape.slots, past, _DeltaShape.channels, dtype=dtype)
+    state = InOut(_DeltaShape.slots, taps, _DeltaShape.channels, dtype=dtype)
     spans = In(_DeltaShape.slots, 4, dtype=np.int32)
     y = Out(_DeltaShape.rows, _DeltaShape.wide, dtype=F32)
     valid = per_call(bounds=_DeltaShape.rows)
