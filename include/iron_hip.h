@@ -410,8 +410,8 @@ int iron_time_mix(const void* r, const void* k, const void* v, const float* log_
                   const int* spans, float* o, int slots, int rows, int heads, int dim, int is_float, void* stream);
 /* x (rows, stride) = [q | k | v | .. b .. a ..]: a causal convolution of `taps` taps (channels, taps) a
  * channel and SiLU on q, k (kv_heads x dim) and v (heads x vdim); q and k made unit vectors a head
- * (eps 1e-6), q times dim^-1/2; decay = exp(-exp(a_log) softplus(a + dt_bias)), beta = sigmoid(b).
- * out (rows, 2 kv_heads dim + heads vdim + 2 heads) = [q | k | v | decay | beta] in float.
+ * (eps 1e-6), q times dim^-1/2; log decay = -exp(a_log) softplus(a + dt_bias), beta = sigmoid(b).
+ * out (rows, 2 kv_heads dim + heads vdim + 2 heads) = [q | k | v | log decay | beta] in float.
  * state (slots, taps, channels): position p's inputs in row p % taps. */
 int iron_short_conv(const void* x, const uint16_t* taps_w, const uint16_t* a_log, const uint16_t* dt_bias, void* state,
                     const int* spans, float* out, int slots, int rows, int stride, int heads, int kv_heads, int dim,
@@ -420,6 +420,16 @@ int iron_short_conv(const void* x, const uint16_t* taps_w, const uint16_t* a_log
  * head (q/k head head / (heads / kv_heads)).  state (slots, heads, dim, vdim), o (rows, heads * vdim). */
 int iron_delta_rule(const float* x, float* state, const int* spans, float* o, int slots, int rows, int heads,
                     int kv_heads, int dim, int vdim, void* stream);
+/* iron_time_mix and iron_delta_rule over portions of many rows, sixteen tokens at a time on float32 MFMAs:
+ * two launches, a workspace of the bytes given (any contents, 16-byte aligned).  The same sums in another
+ * order. */
+int64_t iron_time_mix_workspace_bytes(int slots, int rows, int heads, int dim);
+int iron_time_mix_chunked(const void* r, const void* k, const void* v, const float* log_decay, const uint16_t* u,
+                          float* state, const int* spans, float* o, void* workspace, int slots, int rows, int heads,
+                          int dim, int is_float, void* stream);
+int64_t iron_delta_rule_workspace_bytes(int slots, int rows, int heads);
+int iron_delta_rule_chunked(const float* x, float* state, const int* spans, float* o, void* workspace, int slots, int rows,
+                            int heads, int kv_heads, int dim, int vdim, void* stream);
 /* out = o / rms(o, one head) * gain * silu(gate) * scale; gain (dim) if gain_shared, else (heads * dim). */
 int iron_head_gate(const float* o, const void* gate, const uint16_t* gain, void* out, int rows, int heads, int dim,
                    int gate_stride, int gate_at, int gain_shared, int out_stride, int out_at, float eps, float scale,

@@ -99,6 +99,10 @@ SIGNATURES = {
     "iron_time_mix": (c_int, [_P] * 8 + [c_int] * 5 + [_P]),
     "iron_short_conv": (c_int, [_P] * 7 + [c_int] * 11 + [_P]),
     "iron_delta_rule": (c_int, [_P] * 4 + [c_int] * 6 + [_P]),
+    "iron_time_mix_workspace_bytes": (c_int64, [c_int] * 4),
+    "iron_time_mix_chunked": (c_int, [_P] * 9 + [c_int] * 5 + [_P]),
+    "iron_delta_rule_workspace_bytes": (c_int64, [c_int] * 3),
+    "iron_delta_rule_chunked": (c_int, [_P] * 5 + [c_int] * 6 + [_P]),
     "iron_head_gate": (c_int, [_P] * 4 + [c_int] * 8 + [c_float, c_float, c_int, _P, _P]),
     "iron_mha_window": (c_int, [_P] * 6 + [c_int] * 9 + [c_float, c_int, c_int, c_float, c_int, c_int, _P]),
     "iron_decode_mixed_bf16": (c_int, [_P, _P, _P, c_int, c_int, _P, _P, _P, _P, _P]),

@@ -1,0 +1,540 @@
+// The two recurrences over a prompt's portion, sixteen tokens at a time on float32 MFMAs.
+//
+// Within a chunk of 16 tokens everything that does not touch the state depends on the chunk alone, so a
+// first launch computes it for all chunks at once: what earlier tokens of the chunk leave of themselves
+// in later ones' outputs (a 16 x 16 matrix), and for the delta rule the inverse that turns the chunk's
+// 16 coupled updates into one product.  A second launch walks the chunks in order: a head's state, split
+// by columns over blocks and by rows over a block's four waves, is a few products a chunk.
+//
+// The 16x16x4 MFMA leaves lane (quad, l16) rows quad * 4 .. + 3 of column l16.  Taken as the B operand of
+// a following product, register r of such a result is its rows {r, 4 + r, 8 + r, 12 + r}: four products,
+// one a register, with the A operand's columns in the same order, need no exchange between lanes.  "Frag"
+// below is that A operand: lane (quad, l16) holds [l16][quad * 4 + r] in its r-th float.
+//
+// Decays enter as exponentials of differences of running sums of logarithms, later minus earlier: never
+// above 1, however strong the decay.
+#include "../../include/iron_hip.h"
+#include "rows.h"
+
+namespace iron {
+
+constexpr int CHUNK = 16;
+
+__device__ __forceinline__ f32x4 mfma4(float a, float b, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0); }
+__device__ __forceinline__ f32x4 product16(const f32x4& a, const f32x4& b, f32x4 c) {
+#pragma unroll
+  for (int r = 0; r < 4; ++r) c = mfma4(a[r], b[r], c);
+  return c;
+}
+// exp of a number that is not above 0: the hardware's where rows are bf16, the library's in 32 bits.
+template <typename T>
+__device__ __forceinline__ float decay_exp(float x) {
+  if constexpr (sizeof(T) == 2) return __expf(x);
+  else return expf(x);
+}
+__device__ __forceinline__ float widened(bf16_t v) { return bf16_to_f32(v); }
+__device__ __forceinline__ float widened(float v) { return v; }
+__device__ __forceinline__ float pick4(const f32x4& v, int i) { return i < 2 ? (i == 0 ? v[0] : v[1]) : (i == 2 ? v[2] : v[3]); }
+
+// A barrier for what the block exchanges through LDS: waits for its LDS traffic, not (as __syncthreads does)
+// for the loads from memory in flight.
+__device__ __forceinline__ void block_barrier_lds() {
+  __builtin_amdgcn_fence(__ATOMIC_RELEASE, "workgroup", "local");
+  __builtin_amdgcn_s_barrier();
+  __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "workgroup", "local");
+}
+
+// A span's first chunk in the workspace: spans in the order of their rows, each from a chunk of its own.
+__device__ __forceinline__ int first_chunk(const int* __restrict__ spans, int slots, int slot, int rows) {
+  const Span mine = span_of(spans, slot, rows);
+  int rank = 0;
+  for (int i = 0; i < slots; ++i) {
+    const Span s = span_of(spans, i, rows);
+    rank += s.rows > 0 && s.row0 < mine.row0;
+  }
+  return mine.row0 / CHUNK + rank;
+}
+__host__ __device__ inline long chunks_of(int rows, int slots) { return (rows + CHUNK - 1) / CHUNK + slots; }
+
+// ---------------------------------------------------------------- time mixing
+// Workspace of a chunk and head: r exp(L before it) frags, k exp(L_end - L) frags transposed (both 16 a
+// row tile), exp(L_end), and the 16 x 16 matrix's frag.
+__host__ __device__ inline int mix_words(int tiles) { return tiles * (2 * 256 + 16) + 256; }
+
+template <typename T>
+__global__ __launch_bounds__(256) void time_mix_chunks_kernel(const T* __restrict__ r, const T* __restrict__ k,
+                                                              const float* __restrict__ log_decay, const bf16_t* __restrict__ u,
+                                                              const int* __restrict__ spans, float* __restrict__ work, int rows,
+                                                              int slots, int heads, int dim) {
+  extern __shared__ __align__(16) float lds[];
+  const int head = blockIdx.y, slot = blockIdx.z, base = blockIdx.x * CHUNK;
+  const Span s = span_of(spans, slot, rows);
+  if (base >= s.rows) return;
+  const int n = min(CHUNK, s.rows - base), tiles = (dim + 15) / 16, wide = tiles * 16, pitch = wide + 4, t = threadIdx.x;
+  float* rs = lds;                       // [16][pitch]
+  float* ks = rs + CHUNK * pitch;
+  float* ls = ks + CHUNK * pitch;        // [17][pitch]: row i + 1 the sum up to token i
+  float* am = ls + (CHUNK + 1) * pitch;  // [16][17]
+  const size_t width = (size_t)heads * dim, at = (size_t)(s.row0 + base) * width + head * dim;
+  for (int e = t; e < CHUNK * wide; e += 256) {
+    const int i = e / wide, c = e - i * wide;
+    const bool in = i < n && c < dim;
+    rs[i * pitch + c] = in ? load_one(r + at + i * width + c) : 0.f;
+    ks[i * pitch + c] = in ? load_one(k + at + i * width + c) : 0.f;
+    ls[(i + 1) * pitch + c] = in ? log_decay[at + i * width + c] : 0.f;
+  }
+  for (int e = t; e < CHUNK * 17; e += 256) am[e] = 0.f;
+  __syncthreads();
+  for (int c = t; c < wide; c += 256) {
+    float v[CHUNK];
+#pragma unroll
+    for (int i = 0; i < CHUNK; ++i) v[i] = ls[(i + 1) * pitch + c];
+    float sum = 0.f;
+    ls[c] = 0.f;
+#pragma unroll
+    for (int i = 0; i < CHUNK; ++i) {
+      sum += v[i];
+      ls[(i + 1) * pitch + c] = sum;
+    }
+  }
+  __syncthreads();
+  float* out = work + ((size_t)(first_chunk(spans, slots, slot, rows) + blockIdx.x) * heads + head) * mix_words(tiles);
+  for (int e = t; e < tiles * 64; e += 256) {
+    const int tile = e >> 6, lane = e & 63, l16 = lane & 15, quad = lane >> 4;
+    float4 a, b;
+    {
+      const int c = tile * 16 + quad * 4;
+      const float4 rv = *reinterpret_cast<const float4*>(rs + l16 * pitch + c), lv = *reinterpret_cast<const float4*>(ls + l16 * pitch + c);
+      a = make_float4(rv.x * decay_exp<T>(lv.x), rv.y * decay_exp<T>(lv.y), rv.z * decay_exp<T>(lv.z), rv.w * decay_exp<T>(lv.w));
+    }
+    {
+      const int c = tile * 16 + l16;
+      const float end = ls[CHUNK * pitch + c];
+      float f[4];
+#pragma unroll
+      for (int j = 0; j < 4; ++j) f[j] = ks[(quad * 4 + j) * pitch + c] * decay_exp<T>(end - ls[(quad * 4 + j + 1) * pitch + c]);
+      b = make_float4(f[0], f[1], f[2], f[3]);
+    }
+    reinterpret_cast<float4*>(out)[e] = a;
+    reinterpret_cast<float4*>(out + tiles * 256)[e] = b;
+  }
+  for (int c = t; c < wide; c += 256) out[tiles * 512 + c] = decay_exp<T>(ls[CHUNK * pitch + c]);
+  // Pairs (i, j), j < i: 64 at a time, four threads a pair.
+  for (int p = t >> 2; p < CHUNK * (CHUNK - 1) / 2; p += 64) {
+    int i = 1, j = p;
+    while (j >= i) j -= i++;
+    float sum = 0.f;
+    for (int c = (t & 3) * 4; c < wide; c += 16) {
+      const float4 rv = *reinterpret_cast<const float4*>(rs + i * pitch + c), kv = *reinterpret_cast<const float4*>(ks + j * pitch + c);
+      const float4 a = *reinterpret_cast<const float4*>(ls + i * pitch + c), b = *reinterpret_cast<const float4*>(ls + (j + 1) * pitch + c);
+      sum = fmaf(rv.x * kv.x, decay_exp<T>(a.x - b.x), sum);
+      sum = fmaf(rv.y * kv.y, decay_exp<T>(a.y - b.y), sum);
+      sum = fmaf(rv.z * kv.z, decay_exp<T>(a.z - b.z), sum);
+      sum = fmaf(rv.w * kv.w, decay_exp<T>(a.w - b.w), sum);
+    }
+    sum += IRON_DPP(0.f, sum, 0xB1, 0xF);
+    sum += IRON_DPP(0.f, sum, 0x4E, 0xF);
+    if ((t & 3) == 0) am[i * 17 + j] = sum;
+  }
+  {   // the current token's bonus
+    const int i = t >> 4;
+    float sum = 0.f;
+    for (int c = t & 15; c < dim; c += 16) sum = fmaf(rs[i * pitch + c] * bf16_to_f32(u[head * dim + c]), ks[i * pitch + c], sum);
+    sum = group16_sum(sum);
+    if ((t & 15) == 0) am[i * 17 + i] = sum;
+  }
+  __syncthreads();
+  out[tiles * 528 + t] = am[((t >> 2) & 15) * 17 + (t >> 6) * 4 + (t & 3)];
+}
+
+// The walk asks for a chunk's operands DEPTH chunks ahead (a chunk's products take a fraction of a trip to
+// memory), into registers of their own: every chunk of the unrolled loop issues the same loads, rows and
+// tiles past the end clamped where they are read and zeroed where they are used, so that no branch stands
+// between the loads in flight.
+template <typename T, int NT>
+struct MixOperands {
+  float4 r[NT], k[NT], w[NT];
+  float a;
+  T v[4];   // as loaded: widened where it is used, not where it would be waited for
+};
+
+template <typename T, int NT, int DEPTH>
+__global__ __launch_bounds__(256) void time_mix_walk_kernel(const T* __restrict__ v, float* __restrict__ state,
+                                                            const int* __restrict__ spans, const float* __restrict__ work,
+                                                            float* __restrict__ o, int rows, int slots, int heads, int dim) {
+  __shared__ float4 os[2][4][64];
+  const int head = blockIdx.x, slot = blockIdx.z;   // heads fastest: a head's column blocks share an XCD's L2
+  const Span s = span_of(spans, slot, rows);
+  if (s.rows == 0) return;
+  const int t = threadIdx.x, lane = t & 63, wave = t >> 6, l16 = lane & 15, quad = lane >> 4;
+  const int tiles = (dim + 15) / 16, words = mix_words(tiles), col = blockIdx.y * 16 + l16;
+  const int count = (s.rows + CHUNK - 1) / CHUNK;
+  const size_t width = (size_t)heads * dim;
+  float* sp = state + ((size_t)slot * heads + head) * dim * dim;
+  const float* at = work + ((size_t)first_chunk(spans, slots, slot, rows) * heads + head) * words;
+  // The span's rows by 32-bit offsets; a store to an offset outside them is dropped.
+  constexpr int E = (int)sizeof(T);
+  const __amdgpu_buffer_rsrc_t vb = bounded_bytes(v + (size_t)s.row0 * width + head * dim, (int)(((size_t)s.rows * width - head * dim) * E));
+  const __amdgpu_buffer_rsrc_t ob = bounded_bytes(o + (size_t)s.row0 * width + head * dim, (int)(((size_t)s.rows * width - head * dim) * 4));
+  const int v_at = quad * 4 * (int)width * E + min(col, dim - 1) * E, row_v = (int)width * E;
+  const int o_at = col < dim ? ((quad * 4 + wave) * (int)width + col) * 4 : 0x7fffffff;
+  f32x4 S[NT];
+#pragma unroll
+  for (int n = 0; n < NT; ++n)
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      const int i = (wave * NT + n) * 16 + quad * 4 + j;
+      S[n][j] = (s.start > 0 && i < dim && col < dim) ? sp[(size_t)i * dim + col] : 0.f;
+    }
+  MixOperands<T, NT> ops[DEPTH];
+  auto fetch = [&](MixOperands<T, NT>& x, int c) {
+    c = min(c, count - 1);
+    const float* w = at + (size_t)c * heads * words;
+#pragma unroll
+    for (int n = 0; n < NT; ++n) {
+      const int tile = min(wave * NT + n, tiles - 1);
+      x.r[n] = reinterpret_cast<const float4*>(w)[tile * 64 + lane];
+      x.k[n] = reinterpret_cast<const float4*>(w + tiles * 256)[tile * 64 + lane];
+      x.w[n] = *reinterpret_cast<const float4*>(w + tiles * 512 + tile * 16 + quad * 4);
+    }
+    x.a = w[tiles * 528 + lane * 4 + wave];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {   // zero past the span's last row
+      if constexpr (sizeof(T) == 2) x.v[j] = (T)__builtin_amdgcn_raw_buffer_load_b16(vb, v_at + j * row_v, c * CHUNK * row_v, 0);
+      else x.v[j] = __builtin_bit_cast(float, __builtin_amdgcn_raw_buffer_load_b32(vb, v_at + j * row_v, c * CHUNK * row_v, 0));
+    }
+  };
+  auto run = [&](const MixOperands<T, NT>& x, int c) {
+    f32x4 vf, out = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int j = 0; j < 4; ++j) vf[j] = widened(x.v[j]);
+#pragma unroll
+    for (int n = 0; n < NT; ++n) {
+      out = product16(f32x4{x.r[n].x, x.r[n].y, x.r[n].z, x.r[n].w}, S[n], out);   // S of a tile past the last stays 0
+      S[n] *= f32x4{x.w[n].x, x.w[n].y, x.w[n].z, x.w[n].w};
+      const bool in = wave * NT + n < tiles;
+      S[n] = product16(f32x4{in ? x.k[n].x : 0.f, in ? x.k[n].y : 0.f, in ? x.k[n].z : 0.f, in ? x.k[n].w : 0.f}, vf, S[n]);
+    }
+    out = mfma4(x.a, pick4(vf, wave), out);
+    os[c & 1][wave][lane] = make_float4(out[0], out[1], out[2], out[3]);
+    block_barrier_lds();
+    float sum = 0.f;   // wave w finishes rows quad * 4 + w
+#pragma unroll
+    for (int w = 0; w < 4; ++w) sum += reinterpret_cast<const float*>(&os[c & 1][w][lane])[wave];
+    __builtin_amdgcn_raw_buffer_store_b32(__builtin_bit_cast(unsigned, sum), ob, o_at, c * CHUNK * (int)width * 4, 0);
+  };
+#pragma unroll
+  for (int d = 0; d < DEPTH; ++d) {
+    fetch(ops[d], d);
+    __builtin_amdgcn_sched_barrier(0);   // the loads go out, and are counted down, in the chunks' order
+  }
+  int c = 0;
+  for (; c + DEPTH <= count; c += DEPTH) {
+#pragma unroll
+    for (int d = 0; d < DEPTH; ++d) {
+      run(ops[d], c + d);
+      fetch(ops[d], c + d + DEPTH);
+      __builtin_amdgcn_sched_barrier(0);
+    }
+  }
+#pragma unroll
+  for (int d = 0; d < DEPTH; ++d)
+    if (c + d < count) run(ops[d], c + d);
+#pragma unroll
+  for (int n = 0; n < NT; ++n)
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      const int i = (wave * NT + n) * 16 + quad * 4 + j;
+      if (i < dim && col < dim) sp[(size_t)i * dim + col] = S[n][j];
+    }
+}
+
+// ------------------------------------------------------------- the delta rule
+// With G the running product of decays: u_t = beta_t (v_t - G_t S0^T k_t - sum_{s<t} (G_t/G_s) (k_t.k_s) u_s),
+// so U = T (beta V - beta G (K S0)), T the inverse of I + [beta_t (G_t/G_s) (k_t.k_s)]_{s<t};
+// o = G (Q S0) + P U, P = [(G_t/G_s) (q_t.k_s)]_{s<=t}; S <- G_end S0 + [(G_end/G_s) k_s] U.
+// Workspace of a chunk and head: T's and P's frags, the 16 G, G_end/G and beta.
+constexpr int DELTA_WORDS = 256 + 256 + 3 * 16;
+
+template <int NT>
+__global__ __launch_bounds__(256) void delta_chunks_kernel(const float* __restrict__ x, const int* __restrict__ spans,
+                                                           float* __restrict__ work, int rows, int slots, int heads, int kv_heads,
+                                                           int dim, int vdim) {
+  __shared__ float4 kk[4][64], qk[4][64];
+  __shared__ float m[CHUNK][CHUNK + 1], inv[CHUNK][CHUNK + 1], p[CHUNK][CHUNK + 1], logs[CHUNK], beta[CHUNK];
+  const int head = blockIdx.y, slot = blockIdx.z, base = blockIdx.x * CHUNK;
+  const Span s = span_of(spans, slot, rows);
+  if (base >= s.rows) return;
+  const int n = min(CHUNK, s.rows - base), t = threadIdx.x, lane = t & 63, wave = t >> 6, l16 = lane & 15, quad = lane >> 4;
+  const int group = head / (heads / kv_heads), qkw = kv_heads * dim, channels = 2 * qkw + heads * vdim, wide = channels + 2 * heads;
+  const float* row = x + (size_t)(s.row0 + base) * wide;
+  // Both products' operands are a token's row a lane, four of its columns.
+  f32x4 a = f32x4{0.f, 0.f, 0.f, 0.f}, b = a;
+#pragma unroll
+  for (int e = 0; e < NT; ++e) {
+    f32x4 q = f32x4{0.f, 0.f, 0.f, 0.f}, k = q;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      const int c = (wave * NT + e) * 16 + quad * 4 + j;
+      const bool in = l16 < n && c < dim;
+      q[j] = in ? row[(size_t)l16 * wide + group * dim + c] : 0.f;
+      k[j] = in ? row[(size_t)l16 * wide + qkw + group * dim + c] : 0.f;
+    }
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      a = mfma4(k[j], k[j], a);
+      b = mfma4(q[j], k[j], b);
+    }
+  }
+  kk[wave][lane] = make_float4(a[0], a[1], a[2], a[3]);
+  qk[wave][lane] = make_float4(b[0], b[1], b[2], b[3]);
+  if (t < CHUNK) {
+    float sum = 0.f;
+    for (int i = 0; i <= t; ++i) sum += i < n ? row[(size_t)i * wide + channels + head] : 0.f;
+    logs[t] = sum;
+    beta[t] = t < n ? row[(size_t)t * wide + channels + heads + head] : 0.f;
+  }
+  __syncthreads();
+  {
+    const int i = quad * 4 + wave, j = l16;   // this thread's element: a quarter of the result's lanes' registers
+    float k2 = 0.f, q2 = 0.f;
+#pragma unroll
+    for (int w = 0; w < 4; ++w) {
+      k2 += reinterpret_cast<const float*>(&kk[w][lane])[wave];
+      q2 += reinterpret_cast<const float*>(&qk[w][lane])[wave];
+    }
+    const float ratio = j <= i ? expf(logs[i] - logs[j]) : 0.f;
+    m[i][j] = j < i ? beta[i] * ratio * k2 : 0.f;
+    p[i][j] = ratio * q2;
+  }
+  __syncthreads();
+  if (t < CHUNK) {   // a column of the inverse a thread, by substitution
+    float c[CHUNK];
+#pragma unroll
+    for (int i = 0; i < CHUNK; ++i) {
+      float sum = i == t ? 1.f : 0.f;
+#pragma unroll
+      for (int j = 0; j < i; ++j) sum = fmaf(-m[i][j], c[j], sum);
+      c[i] = sum;
+      inv[i][t] = sum;
+    }
+  }
+  __syncthreads();
+  float* out = work + ((size_t)(first_chunk(spans, slots, slot, rows) + blockIdx.x) * heads + head) * DELTA_WORDS;
+  const int fl = t >> 2, fr = t & 3;
+  out[t] = inv[fl & 15][(fl >> 4) * 4 + fr];
+  out[256 + t] = p[fl & 15][(fl >> 4) * 4 + fr];
+  if (t < CHUNK) {
+    out[512 + t] = expf(logs[t]);
+    out[528 + t] = expf(logs[CHUNK - 1] - logs[t]);
+    out[544 + t] = beta[t];
+  }
+}
+
+template <int NT>
+struct DeltaOperands {
+  float4 q[NT], k[NT], T, G, left, beta;
+  float kt[NT][4], v[4], whole, P;
+};
+
+// VEC: q and k rows are whole 16-byte pieces.
+template <int NT, int DEPTH, bool VEC>
+__global__ __launch_bounds__(256) void delta_walk_kernel(const float* __restrict__ x, float* __restrict__ state,
+                                                         const int* __restrict__ spans, const float* __restrict__ work,
+                                                         float* __restrict__ o, int rows, int slots, int heads, int kv_heads,
+                                                         int dim, int vdim) {
+  __shared__ float4 ys[2][4][64], os[2][4][64];
+  const int head = blockIdx.x, slot = blockIdx.z;   // heads fastest: a head's column blocks share an XCD's L2
+  const Span s = span_of(spans, slot, rows);
+  if (s.rows == 0) return;
+  const int t = threadIdx.x, lane = t & 63, wave = t >> 6, l16 = lane & 15, quad = lane >> 4;
+  const int group = head / (heads / kv_heads), qkw = kv_heads * dim, channels = 2 * qkw + heads * vdim, wide = channels + 2 * heads;
+  const int col = blockIdx.y * 16 + l16, count = (s.rows + CHUNK - 1) / CHUNK;
+  float* sp = state + ((size_t)slot * heads + head) * dim * vdim;
+  const float* at = work + ((size_t)first_chunk(spans, slots, slot, rows) * heads + head) * DELTA_WORDS;
+  const __amdgpu_buffer_rsrc_t xb = bounded_bytes(x + (size_t)s.row0 * wide, (int)((size_t)s.rows * wide * 4));
+  const __amdgpu_buffer_rsrc_t ob = bounded_bytes(o + (size_t)s.row0 * heads * vdim, (int)((size_t)s.rows * heads * vdim * 4));
+  const int o_at = col < vdim ? ((quad * 4 + wave) * heads * vdim + head * vdim + col) * 4 : 0x7fffffff;
+  f32x4 S[NT];
+#pragma unroll
+  for (int n = 0; n < NT; ++n)
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      const int i = (wave * NT + n) * 16 + quad * 4 + j;
+      S[n][j] = (s.start > 0 && i < dim && col < vdim) ? sp[(size_t)i * vdim + col] : 0.f;
+    }
+  DeltaOperands<NT> ops[DEPTH];
+  auto one = [&](int at) { return __builtin_bit_cast(float, __builtin_amdgcn_raw_buffer_load_b32(xb, at, 0, 0)); };
+  auto four = [&](int row, int i) {   // columns i .. i + 3 of dim, from byte `row`, held inside them
+    if (VEC) return __builtin_bit_cast(float4, __builtin_amdgcn_raw_buffer_load_b128(xb, row + 4 * min(i, dim - 4), 0, 0));
+    return make_float4(one(row + 4 * min(i, dim - 1)), one(row + 4 * min(i + 1, dim - 1)), one(row + 4 * min(i + 2, dim - 1)),
+                       one(row + 4 * min(i + 3, dim - 1)));
+  };
+  auto fetch = [&](DeltaOperands<NT>& p, int c) {
+    c = min(c, count - 1);
+    const float* w = at + (size_t)c * heads * DELTA_WORDS;
+    // (past the span's last row that row again: its update is zero, and zero times anything finite stays so)
+    const int mine = (min(c * CHUNK + l16, s.rows - 1) * wide + group * dim) * 4;
+    int down[4];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) down[j] = min(c * CHUNK + quad * 4 + j, s.rows - 1) * wide * 4;
+#pragma unroll
+    for (int n = 0; n < NT; ++n) {
+      const int tile = wave * NT + n;
+      p.q[n] = four(mine, tile * 16 + quad * 4);
+      p.k[n] = four(mine + 4 * qkw, tile * 16 + quad * 4);
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        p.kt[n][j] = one(down[j] + 4 * (qkw + group * dim + min(tile * 16 + l16, dim - 1)));
+    }
+    p.T = reinterpret_cast<const float4*>(w)[lane];
+    p.G = reinterpret_cast<const float4*>(w + 512)[quad];
+    p.left = reinterpret_cast<const float4*>(w + 528)[quad];
+    p.beta = reinterpret_cast<const float4*>(w + 544)[quad];
+    p.whole = w[512 + CHUNK - 1];
+    p.P = w[256 + lane * 4 + wave];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) p.v[j] = one(down[j] + 4 * (2 * qkw + head * vdim + min(col, vdim - 1)));
+  };
+  auto finish = [&](int c) {   // chunk c's outputs: wave w adds up and writes rows quad * 4 + w
+    float sum = 0.f;
+#pragma unroll
+    for (int w = 0; w < 4; ++w) sum += reinterpret_cast<const float*>(&os[c & 1][w][lane])[wave];
+    __builtin_amdgcn_raw_buffer_store_b32(__builtin_bit_cast(unsigned, sum), ob, o_at, c * CHUNK * heads * vdim * 4, 0);
+  };
+  auto run = [&](const DeltaOperands<NT>& p, int c) {
+    // A row past the span's last: T's and P's columns for it are zero but for T's diagonal, its beta is zero,
+    // so its update is zero; what its q, k and v read as does not matter.
+    f32x4 y = f32x4{0.f, 0.f, 0.f, 0.f}, out = y;
+#pragma unroll
+    for (int n = 0; n < NT; ++n) y = product16(f32x4{p.k[n].x, p.k[n].y, p.k[n].z, p.k[n].w}, S[n], y);   // rows past dim: S is 0
+    ys[c & 1][wave][lane] = make_float4(y[0], y[1], y[2], y[3]);
+#pragma unroll
+    for (int n = 0; n < NT; ++n) out = product16(f32x4{p.q[n].x, p.q[n].y, p.q[n].z, p.q[n].w}, S[n], out);
+    const f32x4 G = f32x4{p.G.x, p.G.y, p.G.z, p.G.w}, left = f32x4{p.left.x, p.left.y, p.left.z, p.left.w};
+    f32x4 kept[NT];
+#pragma unroll
+    for (int n = 0; n < NT; ++n) {
+      const float in = (wave * NT + n) * 16 + l16 < dim ? 1.f : 0.f;
+      kept[n] = f32x4{p.kt[n][0], p.kt[n][1], p.kt[n][2], p.kt[n][3]} * left * in;
+    }
+    out *= G;
+    block_barrier_lds();
+    f32x4 sum = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int w = 0; w < 4; ++w) {
+      const float4 part = ys[c & 1][w][lane];
+      sum += f32x4{part.x, part.y, part.z, part.w};
+    }
+    const f32x4 X = f32x4{p.beta.x, p.beta.y, p.beta.z, p.beta.w} * (f32x4{p.v[0], p.v[1], p.v[2], p.v[3]} - G * sum);
+    const f32x4 U = product16(f32x4{p.T.x, p.T.y, p.T.z, p.T.w}, X, f32x4{0.f, 0.f, 0.f, 0.f});
+#pragma unroll
+    for (int n = 0; n < NT; ++n) {
+      S[n] *= p.whole;
+      S[n] = product16(kept[n], U, S[n]);
+    }
+    out = mfma4(p.P, pick4(U, wave), out);
+    os[c & 1][wave][lane] = make_float4(out[0], out[1], out[2], out[3]);
+    if (c > 0) finish(c - 1);   // behind this chunk's barrier
+  };
+#pragma unroll
+  for (int d = 0; d < DEPTH; ++d) {
+    fetch(ops[d], d);
+    __builtin_amdgcn_sched_barrier(0);   // the loads go out, and are counted down, in the chunks' order
+  }
+  int c = 0;
+  for (; c + DEPTH <= count; c += DEPTH) {
+#pragma unroll
+    for (int d = 0; d < DEPTH; ++d) {
+      run(ops[d], c + d);
+      fetch(ops[d], c + d + DEPTH);
+      __builtin_amdgcn_sched_barrier(0);
+    }
+  }
+#pragma unroll
+  for (int d = 0; d < DEPTH; ++d)
+    if (c + d < count) run(ops[d], c + d);
+  __syncthreads();
+  finish(count - 1);
+#pragma unroll
+  for (int n = 0; n < NT; ++n)
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      const int i = (wave * NT + n) * 16 + quad * 4 + j;
+      if (i < dim && col < vdim) sp[(size_t)i * vdim + col] = S[n][j];
+    }
+}
+
+}  // namespace iron
+
+using namespace iron;
+
+extern "C" int64_t iron_time_mix_workspace_bytes(int slots, int rows, int heads, int dim) {
+  return chunks_of(rows, slots) * heads * (int64_t)mix_words((dim + 15) / 16) * 4;
+}
+extern "C" int64_t iron_delta_rule_workspace_bytes(int slots, int rows, int heads) {
+  return chunks_of(rows, slots) * heads * (int64_t)DELTA_WORDS * 4;
+}
+
+#define IRON_CHUNKED_REQUIRE(name)                                                                        \
+  IRON_REQUIRE(spans && ((uintptr_t)spans & 15) == 0, name ": spans must be there and 16-byte aligned");    \
+  IRON_REQUIRE(slots > 0 && slots <= 65535 && rows > 0, name ": slots (%d) and rows (%d) must be positive", slots, rows)
+
+extern "C" int iron_time_mix_chunked(const void* r, const void* k, const void* v, const float* log_decay, const uint16_t* u,
+                                     float* state, const int* spans, float* o, void* workspace, int slots, int rows, int heads,
+                                     int dim, int is_float, void* stream) {
+  IRON_REQUIRE(r && k && v && log_decay && u && state && o && workspace, "time_mix_chunked: null operand");
+  IRON_CHUNKED_REQUIRE("time_mix_chunked");
+  IRON_REQUIRE(heads > 0 && heads <= 65535 && dim > 0 && dim <= 256, "time_mix_chunked: heads (%d) positive, dim (%d) from 1 to 256", heads, dim);
+  IRON_REQUIRE(((uintptr_t)workspace & 15) == 0, "time_mix_chunked: the workspace must be 16-byte aligned");
+  IRON_REQUIRE((long)rows * heads * dim < (1L << 28), "time_mix_chunked: the batch's rows are addressed with 32-bit offsets");
+  hipStream_t s = (hipStream_t)stream;
+  const int tiles = (dim + 15) / 16, pitch = tiles * 16 + 4;
+  const size_t lds = ((size_t)(3 * CHUNK + 1) * pitch + CHUNK * 17) * 4;
+  const dim3 all((rows + CHUNK - 1) / CHUNK, heads, slots), walk(heads, tiles, slots);
+  float* work = (float*)workspace;
+#define IRON_MIX_WALK(T, NT, DEPTH) \
+  hipLaunchKernelGGL((time_mix_walk_kernel<T, NT, DEPTH>), walk, dim3(256), 0, s, (const T*)v, state, spans, work, o, rows, slots, heads, dim)
+#define IRON_MIX(T)                                                                                                             \
+  hipLaunchKernelGGL((time_mix_chunks_kernel<T>), all, dim3(256), lds, s, (const T*)r, (const T*)k, log_decay, u, spans, work, rows, \
+                     slots, heads, dim);                                                                                        \
+  if (tiles <= 4) IRON_MIX_WALK(T, 1, 6);                                                                                          \
+  else if (tiles <= 8) IRON_MIX_WALK(T, 2, 4);                                                                                     \
+  else IRON_MIX_WALK(T, 4, 2);
+  if (is_float) { IRON_MIX(float) }
+  else { IRON_MIX(bf16_t) }
+#undef IRON_MIX
+#undef IRON_MIX_WALK
+  IRON_LAUNCH_CHECK();
+}
+
+extern "C" int iron_delta_rule_chunked(const float* x, float* state, const int* spans, float* o, void* workspace, int slots,
+                                       int rows, int heads, int kv_heads, int dim, int vdim, void* stream) {
+  IRON_REQUIRE(x && state && o && workspace, "delta_rule_chunked: null operand");
+  IRON_CHUNKED_REQUIRE("delta_rule_chunked");
+  IRON_REQUIRE(heads > 0 && heads <= 65535 && kv_heads > 0 && heads % kv_heads == 0,
+               "delta_rule_chunked: kv_heads (%d) must divide heads (%d)", kv_heads, heads);
+  IRON_REQUIRE(dim > 0 && dim <= 256 && vdim > 0, "delta_rule_chunked: dim (%d) from 1 to 256, vdim (%d) positive", dim, vdim);
+  IRON_REQUIRE(((uintptr_t)workspace & 15) == 0, "delta_rule_chunked: the workspace must be 16-byte aligned");
+  IRON_REQUIRE((long)rows * (2 * kv_heads * dim + heads * (vdim + 2)) < (1L << 28),
+               "delta_rule_chunked: the batch's rows are addressed with 32-bit offsets");
+  hipStream_t s = (hipStream_t)stream;
+  const dim3 all((rows + CHUNK - 1) / CHUNK, heads, slots), walk(heads, (vdim + 15) / 16, slots);
+  const bool vec = dim % 4 == 0 && (heads * vdim + 2 * heads) % 4 == 0 && ((uintptr_t)x & 15) == 0;   // (2 kv_heads dim is whole then)
+  float* work = (float*)workspace;
+#define IRON_DELTA_WALK(NT, DEPTH)                                                                                                    \
+  {                                                                                                                              \
+    hipLaunchKernelGGL((delta_chunks_kernel<NT>), all, dim3(256), 0, s, x, spans, work, rows, slots, heads, kv_heads, dim, vdim); \
+    if (vec)                                                                                                                     \
+      hipLaunchKernelGGL((delta_walk_kernel<NT, DEPTH, true>), walk, dim3(256), 0, s, x, state, spans, work, o, rows, slots, heads, \
+                         kv_heads, dim, vdim);                                                                                   \
+    else                                                                                                                         \
+      hipLaunchKernelGGL((delta_walk_kernel<NT, DEPTH, false>), walk, dim3(256), 0, s, x, state, spans, work, o, rows, slots,    \
+                         heads, kv_heads, dim, vdim);                                                                            \
+  }
+  if (dim <= 64) IRON_DELTA_WALK(1, 3)
+  else if (dim <= 128) IRON_DELTA_WALK(2, 2)
+  else IRON_DELTA_WALK(4, 2)
+#undef IRON_DELTA_WALK
+  IRON_LAUNCH_CHECK();
+}

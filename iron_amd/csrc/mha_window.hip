@@ -172,7 +172,7 @@ constexpr int WIN_KEYS = 64;
 template <int DKP, int DVP>
 struct WindowShared {
   __align__(16) bf16_t k[WIN_KEYS][DKP + 8];
-  __align__(16) bf16_t vt[DVP][WIN_KEYS + 4];
+  __align__(16) bf16_t vt[DVP][WIN_KEYS + 8];
   float by_distance[192 + 64];
 };
 
@@ -180,7 +180,7 @@ template <int DKP, int DVP, int QT>
 __device__ __forceinline__ void window_prefill_body(const bf16_t* __restrict__ x, const bf16_t* __restrict__ keys,
                                                     const bf16_t* __restrict__ values, const float* __restrict__ bias,
                                                     bf16_t* __restrict__ out, const WindowShape& a, const Span& s, int slot,
-                                                    int head, int tile, WindowShared<DKP, DVP>& sh) {
+                                                    int head, int tile, WindowShared<DKP, DVP>* pair) {
   constexpr int BQ = QT * 64, KD = DKP / 32, VD = DVP / 16;
   constexpr int KP = WIN_KEYS * DKP / 8 / 256;         // 16-byte pieces of a key tile a thread stages
   constexpr int VP = (WIN_KEYS / 4) * (DVP / 8);       // four-key pieces of a value tile
@@ -194,7 +194,12 @@ __device__ __forceinline__ void window_prefill_body(const bf16_t* __restrict__ x
   const bf16_t* own_v = x + a.heads * a.dim + nk + g * a.vdim;
   const bf16_t* ring_k = keys + (size_t)slot * a.ring * nk + g * a.dim;
   const bf16_t* ring_v = values + (size_t)slot * a.ring * nv + g * a.vdim;
-  const int from = max(0, first_pos - a.window + 1), tiles = (last_pos - from) / WIN_KEYS + 1;
+  // Tiles of the span's own keys start at its start, tiles of the ring's end there (the first may begin
+  // before the window, or before position 0): no tile has keys of both.
+  const int from = max(0, first_pos - a.window + 1);
+  const int old_tiles = from < s.start ? (s.start - from + WIN_KEYS - 1) / WIN_KEYS : 0;
+  const int first_base = from < s.start ? s.start - old_tiles * WIN_KEYS : from;
+  const int tiles = (last_pos - first_base) / WIN_KEYS + 1;
 
   bf16x8 qf[QT][KD];
 #pragma unroll
@@ -218,62 +223,83 @@ __device__ __forceinline__ void window_prefill_body(const bf16_t* __restrict__ x
     for (int d = 0; d < VD; ++d) acc[q][d] = f32x4{0.f, 0.f, 0.f, 0.f};
   }
 
-  uint4 kn[KP], vn[VT][4];
+  u32x4 kn[KP], vn[VT][4];
   float bn = 0.f;
-  // The next tile on its way from memory: positions base .. base + 63 (none past the span's last).
+  // The next tile on its way from memory: keys at positions base .. base + 63, by 32-bit offsets into bounded
+  // buffers (a row past the batch's last reads as zeros; one past the span's last, another sequence's, is
+  // masked below).  A thread's offsets into a tile of the call's own rows are the same for every tile.
+  // Columns past a head's width read its last ones: q is zero there, and those of v are not stored.
+  const __amdgpu_buffer_rsrc_t own_kb = bounded_bytes(own_k + (size_t)s.row0 * a.stride, (int)(((long)(a.rows - s.row0) * a.stride - (own_k - x)) * 2));
+  const __amdgpu_buffer_rsrc_t own_vb = bounded_bytes(own_v + (size_t)s.row0 * a.stride, (int)(((long)(a.rows - s.row0) * a.stride - (own_v - x)) * 2));
+  const __amdgpu_buffer_rsrc_t old_kb = bounded_bytes(ring_k, (a.ring * nk - g * a.dim) * 2);
+  const __amdgpu_buffer_rsrc_t old_vb = bounded_bytes(ring_v, (a.ring * nv - g * a.vdim) * 2);
+  int k_col[KP], v_col[VT], k_own[KP], v_own[VT], k_mod[KP], v_mod[VT][4];
+#pragma unroll
+  for (int i = 0; i < KP; ++i) {
+    const int e = t + 256 * i, row = e / (DKP / 8);
+    k_mod[i] = row % a.ring;
+    k_col[i] = 2 * min((e % (DKP / 8)) * 8, a.dim - 8);
+    k_own[i] = row * a.stride * 2 + k_col[i];
+  }
+#pragma unroll
+  for (int i = 0; i < VT; ++i) {
+    const int e = t + 256 * i, row = (e / (DVP / 8) * 4) % WIN_KEYS;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) v_mod[i][j] = (row + j) % a.ring;
+    v_col[i] = 2 * min((e % (DVP / 8)) * 8, a.vdim - 8);
+    v_own[i] = row * a.stride * 2 + v_col[i];
+  }
   auto fetch = [&](int base) {
-    const int wrap = base % a.ring;
+    if (base >= s.start) {
+      const int at = (base - s.start) * a.stride * 2;
 #pragma unroll
-    for (int i = 0; i < KP; ++i) {
-      const int e = t + 256 * i, r = e / (DKP / 8), c = (e % (DKP / 8)) * 8, p = base + r;
-      int at = wrap + r;
-      while (at >= a.ring) at -= a.ring;
-      const bf16_t* src = p >= s.start ? own_k + (size_t)(s.row0 + p - s.start) * a.stride : ring_k + (size_t)at * nk;
-      kn[i] = (p < end && c < a.dim) ? *reinterpret_cast<const uint4*>(src + c) : make_uint4(0, 0, 0, 0);
+      for (int i = 0; i < KP; ++i) kn[i] = __builtin_amdgcn_raw_buffer_load_b128(own_kb, k_own[i], at, 0);
+#pragma unroll
+      for (int i = 0; i < VT; ++i)
+#pragma unroll
+        for (int j = 0; j < 4; ++j) vn[i][j] = __builtin_amdgcn_raw_buffer_load_b128(own_vb, v_own[i], at + j * a.stride * 2, 0);
+    } else {
+      const int wrap = ((base % a.ring) + a.ring) % a.ring;
+      auto place = [&](int r) { return wrap + r - (a.ring & -(int)(wrap + r >= a.ring)); };   // r < ring
+#pragma unroll
+      for (int i = 0; i < KP; ++i) kn[i] = __builtin_amdgcn_raw_buffer_load_b128(old_kb, place(k_mod[i]) * nk * 2 + k_col[i], 0, 0);
+#pragma unroll
+      for (int i = 0; i < VT; ++i)
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+          vn[i][j] = __builtin_amdgcn_raw_buffer_load_b128(old_vb, place(v_mod[i][j]) * nv * 2 + v_col[i], 0, 0);
     }
-#pragma unroll
-    for (int i = 0; i < VT; ++i) {
-      const int e = t + 256 * i, r4 = e / (DVP / 8), c = (e % (DVP / 8)) * 8;
-#pragma unroll
-      for (int j = 0; j < 4; ++j) {
-        const int r = r4 * 4 + j, p = base + r;
-        int at = wrap + r;
-        while (at >= a.ring) at -= a.ring;
-        const bf16_t* src = p >= s.start ? own_v + (size_t)(s.row0 + p - s.start) * a.stride : ring_v + (size_t)at * nv;
-        vn[i][j] = (e < VP && p < end && c < a.vdim) ? *reinterpret_cast<const uint4*>(src + c) : make_uint4(0, 0, 0, 0);
-      }
-    }
-    // entry t: the distance (first_pos - base - 63) + t
-    const int dist = first_pos - base - (WIN_KEYS - 1) + t;
-    bn = (t < BQ + WIN_KEYS && dist >= 0 && dist < a.window) ? bias[(size_t)head * a.window + dist] * LOG2E : -INFINITY;
+    // entry t: the distance first_pos - base + BQ - 1 - t (masked where it is used)
+    bn = bias[(size_t)head * a.window + max(0, min(first_pos - base + BQ - 1 - t, a.window - 1))];
   };
-  fetch(from);
+  fetch(first_base);
   const float scale = a.scale * LOG2E;
   for (int n = 0; n < tiles; ++n) {
-    __syncthreads();   // the last tile's readers are done
+    const int base = first_base + n * WIN_KEYS;
+    WindowShared<DKP, DVP>& sh = pair[n & 1];   // its last readers are behind the barrier of the tile between
 #pragma unroll
     for (int i = 0; i < KP; ++i) {
       const int e = t + 256 * i;
-      *reinterpret_cast<uint4*>(&sh.k[e / (DKP / 8)][(e % (DKP / 8)) * 8]) = kn[i];
+      *reinterpret_cast<u32x4*>(&sh.k[e / (DKP / 8)][(e % (DKP / 8)) * 8]) = kn[i];
     }
 #pragma unroll
     for (int i = 0; i < VT; ++i) {
       const int e = t + 256 * i, r4 = e / (DVP / 8), c = (e % (DVP / 8)) * 8;
       if (e < VP) {
-        const uint32_t w[4][4] = {{vn[i][0].x, vn[i][0].y, vn[i][0].z, vn[i][0].w}, {vn[i][1].x, vn[i][1].y, vn[i][1].z, vn[i][1].w},
-                                  {vn[i][2].x, vn[i][2].y, vn[i][2].z, vn[i][2].w}, {vn[i][3].x, vn[i][3].y, vn[i][3].z, vn[i][3].w}};
 #pragma unroll
         for (int j = 0; j < 4; ++j) {   // two columns at a time: four keys each, 8 bytes
-          const uint2 even = make_uint2((w[0][j] & 0xffffu) | (w[1][j] << 16), (w[2][j] & 0xffffu) | (w[3][j] << 16));
-          const uint2 odd = make_uint2((w[0][j] >> 16) | (w[1][j] & 0xffff0000u), (w[2][j] >> 16) | (w[3][j] & 0xffff0000u));
+          const uint32_t w0 = vn[i][0][j], w1 = vn[i][1][j], w2 = vn[i][2][j], w3 = vn[i][3][j];
+          const uint2 even = make_uint2((w0 & 0xffffu) | (w1 << 16), (w2 & 0xffffu) | (w3 << 16));
+          const uint2 odd = make_uint2((w0 >> 16) | (w1 & 0xffff0000u), (w2 >> 16) | (w3 & 0xffff0000u));
           *reinterpret_cast<uint2*>(&sh.vt[c + 2 * j][r4 * 4]) = even;
           *reinterpret_cast<uint2*>(&sh.vt[c + 2 * j + 1][r4 * 4]) = odd;
         }
       }
     }
-    sh.by_distance[t] = bn;
+    const int dist = first_pos - base + BQ - 1 - t;
+    sh.by_distance[t] = (dist >= 0 && dist < a.window) ? bn * LOG2E : -INFINITY;
     __syncthreads();
-    if (n + 1 < tiles) fetch(from + (n + 1) * WIN_KEYS);
+    if (n + 1 < tiles) fetch(base + WIN_KEYS);
 
     f32x4 sc[QT][4];
 #pragma unroll
@@ -291,38 +317,50 @@ __device__ __forceinline__ void window_prefill_body(const bf16_t* __restrict__ x
     bf16x8 pf[QT][2];
 #pragma unroll
     for (int q = 0; q < QT; ++q) {
-      const int at = (wave * QT + q) * 16 + lo16 + (WIN_KEYS - 1) - quad * 4;   // key r of tile kt: - 16 kt - r
-      float top = m[q];
+      const float* by = sh.by_distance + BQ - 1 - ((wave * QT + q) * 16 + lo16) + quad * 4;   // key r of tile kt: + 16 kt + r
+      float top = -INFINITY;
 #pragma unroll
       for (int kt = 0; kt < 4; ++kt)
 #pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          sc[q][kt][r] = fmaf(sc[q][kt][r], scale, sh.by_distance[at - kt * 16 - r]);
-          top = fmaxf(top, sc[q][kt][r]);
-        }
-      top = fmaxf(top, __shfl_xor(top, 16, 64));
-      top = fmaxf(top, __shfl_xor(top, 32, 64));
-      const float fade = __builtin_amdgcn_exp2f(m[q] - top);
-      m[q] = top;
+        for (int r = 0; r < 4; ++r) sc[q][kt][r] = fmaf(sc[q][kt][r], scale, by[kt * 16 + r]);
+      if (base < 0) {   // keys ahead of the sequence
+#pragma unroll
+        for (int kt = 0; kt < 4; ++kt)
+#pragma unroll
+          for (int r = 0; r < 4; ++r)
+            if (base + kt * 16 + quad * 4 + r < 0) sc[q][kt][r] = -INFINITY;
+      }
+#pragma unroll
+      for (int kt = 0; kt < 4; ++kt) top = fmaxf(top, fmaxf(fmaxf(sc[q][kt][0], sc[q][kt][1]), fmaxf(sc[q][kt][2], sc[q][kt][3])));
+      // The reference the exponents are taken from moves only where a score would exceed it by more than 2^8:
+      // it cancels in the quotient, and the products need no rescaling between.
+      if (__builtin_amdgcn_ballot_w64(top > m[q] + 8.f) != 0) {
+        top = fmaxf(top, __shfl_xor(top, 16, 64));
+        top = fmaxf(top, __shfl_xor(top, 32, 64));
+        top = fmaxf(m[q], top);
+        const float fade = __builtin_amdgcn_exp2f(m[q] - top);
+        m[q] = top;
+        l[q] *= fade;
+#pragma unroll
+        for (int d = 0; d < VD; ++d)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) acc[q][d][r] *= fade;
+      }
       float sum = 0.f;
 #pragma unroll
       for (int kt = 0; kt < 4; ++kt)
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-          sc[q][kt][r] = __builtin_amdgcn_exp2f(sc[q][kt][r] - top);
+          sc[q][kt][r] = __builtin_amdgcn_exp2f(sc[q][kt][r] - m[q]);
           sum += sc[q][kt][r];
         }
-      l[q] = fmaf(l[q], fade, sum);
+      l[q] += sum;
 #pragma unroll
       for (int h = 0; h < 2; ++h) {
         const uint4 v = make_uint4(pack_bf16(sc[q][2 * h][0], sc[q][2 * h][1]), pack_bf16(sc[q][2 * h][2], sc[q][2 * h][3]),
                                    pack_bf16(sc[q][2 * h + 1][0], sc[q][2 * h + 1][1]), pack_bf16(sc[q][2 * h + 1][2], sc[q][2 * h + 1][3]));
         pf[q][h] = __builtin_bit_cast(bf16x8, v);
       }
-#pragma unroll
-      for (int d = 0; d < VD; ++d)
-#pragma unroll
-        for (int r = 0; r < 4; ++r) acc[q][d][r] *= fade;
     }
 #pragma unroll
     for (int d = 0; d < VD; ++d)
@@ -360,9 +398,13 @@ template <int DKP, int DVP>
 __global__ __launch_bounds__(256) void window_prefill_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ keys,
                                                              const bf16_t* __restrict__ values, const float* __restrict__ bias,
                                                              const int* __restrict__ spans, bf16_t* __restrict__ out, WindowShape a) {
-  __shared__ WindowShared<DKP, DVP> sh;
+  __shared__ WindowShared<DKP, DVP> sh[2];
   const Span s = span_of(spans, blockIdx.z, a.rows);
-  const int tile = blockIdx.x, head = blockIdx.y;
+  // Heads fastest, so that the blocks with work are a run of the grid (a pattern of idle blocks within it
+  // would leave the same compute units idle each time round), and, where they divide by the XCDs, the
+  // heads of a group on one XCD, whose L2 then reads their keys and values once.
+  const int tile = blockIdx.y, x8 = blockIdx.x;
+  const int head = a.heads % 8 == 0 ? (x8 & 7) * (a.heads >> 3) + (x8 >> 3) : x8;
   constexpr bool CAN_WIDE = DVP <= 128 && DKP <= 128;   // registers
   if (CAN_WIDE && (long)((s.rows + 127) / 128) * a.heads >= 256) {
     if (tile * 128 < s.rows)
@@ -375,7 +417,7 @@ __global__ __launch_bounds__(256) void window_prefill_kernel(const bf16_t* __res
 template <int DKP>
 static int launch_window_prefill(int dvp, const bf16_t* x, const bf16_t* keys, const bf16_t* values, const float* bias,
                                  const int* spans, bf16_t* out, const WindowShape& a, int slots, hipStream_t s) {
-  const dim3 grid((a.rows + 63) / 64, a.heads, slots);
+  const dim3 grid(a.heads, (a.rows + 63) / 64, slots);
 #define IRON_WINDOW(DVP) \
   hipLaunchKernelGGL((window_prefill_kernel<DKP, DVP>), grid, dim3(256), 0, s, x, keys, values, bias, spans, out, a)
   if (dvp <= 32) IRON_WINDOW(32);
@@ -403,6 +445,8 @@ extern "C" int iron_mha_window(const void* x, void* keys, void* values, const fl
   IRON_REQUIRE(stride >= heads * dim + kv_heads * (dim + vdim), "mha_window: a row of %d holds no q, k and v of %d heads", stride, heads);
   IRON_REQUIRE(out_at >= 0 && out_at + heads * vdim <= out_stride, "mha_window: %d columns from %d of an output row of %d",
                heads * vdim, out_at, out_stride);
+  IRON_REQUIRE((long)rows * stride < (1L << 30) && (long)ring * kv_heads * (dim > vdim ? dim : vdim) < (1L << 30),
+               "mha_window: the batch's rows and a slot's ring are addressed with 32-bit offsets");
   const WindowShape a{rows, stride, heads, kv_heads, dim, vdim, window, ring, out_stride, out_at, scale, out_scale};
   hipStream_t s = (hipStream_t)stream;
   const bool aligned = stride % 8 == 0 && dim % 8 == 0 && vdim % 8 == 0 && (((uintptr_t)x | (uintptr_t)keys | (uintptr_t)values) & 15) == 0;

@@ -71,7 +71,7 @@ template <typename T>
 __global__ __launch_bounds__(256) void low_rank_decay_kernel(const T* __restrict__ z, const bf16_t* __restrict__ w2,
                                                              const bf16_t* __restrict__ w0, float* __restrict__ out,
                                                              int rows, int n, int rank, const int* __restrict__ valid) {
-  extern __shared__ float zt[];   // [rank][DECAY_ROWS]
+  extern __shared__ __align__(16) float zt[];   // [rank][DECAY_ROWS]
   const int live = bound_or(valid, rows);
   const int r0 = blockIdx.y * DECAY_ROWS;
   if (r0 >= live) return;
@@ -87,7 +87,23 @@ __global__ __launch_bounds__(256) void low_rank_decay_kernel(const T* __restrict
 #pragma unroll
   for (int r = 0; r < DECAY_ROWS; ++r) acc[r] = 0.f;
   const bf16_t* wr = w2 + (size_t)c * rank;
-  for (int k = 0; k < rank; ++k) {
+  int k = 0;
+  if (rank % 8 == 0 && ((uintptr_t)w2 & 15) == 0)
+    for (; k < rank; k += 8) {
+      float w[8];
+      unpack8(*reinterpret_cast<const uint4*>(wr + k), w);
+#pragma unroll
+      for (int j = 0; j < 8; ++j)
+#pragma unroll
+        for (int r = 0; r < DECAY_ROWS; r += 4) {
+          const float4 z4 = *reinterpret_cast<const float4*>(zt + (k + j) * DECAY_ROWS + r);
+          acc[r] = fmaf(w[j], z4.x, acc[r]);
+          acc[r + 1] = fmaf(w[j], z4.y, acc[r + 1]);
+          acc[r + 2] = fmaf(w[j], z4.z, acc[r + 2]);
+          acc[r + 3] = fmaf(w[j], z4.w, acc[r + 3]);
+        }
+    }
+  for (; k < rank; ++k) {
     const float w = bf16_to_f32(wr[k]);
 #pragma unroll
     for (int r = 0; r < DECAY_ROWS; ++r) acc[r] = fmaf(w, zt[k * DECAY_ROWS + r], acc[r]);
@@ -198,15 +214,15 @@ __global__ __launch_bounds__(256) void time_mix_kernel(const T* __restrict__ r, 
 
 // ------------------------------------------------------- short convolution
 // The packed projection's rows [q | k | v | ... | b | a] -> float32 rows [unit q / sqrt(dim) | unit k |
-// v | decay | beta]: a causal convolution a channel and SiLU on q, k, v; unit q and k a head; the
-// step's decay exp(-exp(A_log) softplus(a + dt_bias)) and beta = sigmoid(b) a value head.
+// v | log decay | beta]: a causal convolution a channel and SiLU on q, k, v; unit q and k a head; the
+// step's log decay -exp(A_log) softplus(a + dt_bias) and beta = sigmoid(b) a value head.
 struct ConvShape {
   int rows, stride;                 // the projection's rows, and their length
   int heads, kv_heads, dim, vdim;
   int taps, b_at, a_at;             // columns of b and a in a projection row
 };
 constexpr int CONV_TILE = 16;
-template <typename T>
+template <typename T, int TAPS>   // TAPS: the number of taps where it is a small one, else 0
 __global__ __launch_bounds__(256) void short_conv_kernel(const T* __restrict__ x, const bf16_t* __restrict__ taps,
                                                          const bf16_t* __restrict__ a_log, const bf16_t* __restrict__ dt_bias,
                                                          T* __restrict__ state, const int* __restrict__ spans,
@@ -224,7 +240,7 @@ __global__ __launch_bounds__(256) void short_conv_kernel(const T* __restrict__ x
       const T* row = x + (size_t)(s.row0 + p) * c.stride;
       float* to = out + (size_t)(s.row0 + p) * wide + channels;
       const float a = load_one(row + c.a_at + h) + bf16_to_f32(dt_bias[h]);
-      to[h] = expf(-expf(bf16_to_f32(a_log[h])) * softplus_exact(a));
+      to[h] = -expf(bf16_to_f32(a_log[h])) * softplus_exact(a);
       to[c.heads + h] = sigmoid_exact(load_one(row + c.b_at + h));
     }
     return;
@@ -239,30 +255,54 @@ __global__ __launch_bounds__(256) void short_conv_kernel(const T* __restrict__ x
     if (p >= 0) return load_one(x + (size_t)(s.row0 + p) * c.stride + ch);
     return s.start + p >= 0 ? load_one(held + (size_t)((s.start + p) % c.taps) * channels + ch) : 0.f;
   };
-  for (int p = first + wave; p < last; p += 4) {
-    float f[4];
-    float ss = 0.f;
+  // A wave makes four rows one after the other; where the taps are few their inputs slide through
+  // registers, so that each is read once for the four.
+  const int p0 = first + wave * 4;
+  if (p0 < last) {
+    float f[4][4], ss[4] = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int e = 0; e < 4; ++e) {
       const int j = lane + 64 * e;
-      f[e] = 0.f;
-      if (j < len) {
-        float acc = 0.f;
-        for (int i = 0; i < c.taps; ++i)
-          acc = fmaf(bf16_to_f32(taps[(size_t)(at + j) * c.taps + i]), input(p - past + i, at + j), acc);
-        f[e] = acc * sigmoid_exact(acc);
-        ss = fmaf(f[e], f[e], ss);
-      }
-    }
-    float scale = 1.f;
-    if (!is_v) {
-      scale = 1.0f / sqrtf(wave_sum(ss) + 1e-6f);
-      if (seg < c.kv_heads) scale *= 1.0f / sqrtf((float)c.dim);
-    }
-    float* to = out + (size_t)(s.row0 + p) * wide + at;
+      if (64 * e >= len) continue;
+      const bool in = j < len;
+      const bf16_t* tw = taps + (size_t)(at + (in ? j : 0)) * c.taps;
+      if (TAPS > 0) {
+        float w[TAPS > 0 ? TAPS : 1], win[TAPS + 3];
 #pragma unroll
-    for (int e = 0; e < 4; ++e)
-      if (lane + 64 * e < len) to[lane + 64 * e] = f[e] * scale;
+        for (int i = 0; i < TAPS; ++i) w[i] = in ? bf16_to_f32(tw[i]) : 0.f;
+#pragma unroll
+        for (int i = 0; i < TAPS + 3; ++i) win[i] = (in && p0 - (TAPS - 1) + i < last) ? input(p0 - (TAPS - 1) + i, at + j) : 0.f;
+#pragma unroll
+        for (int q = 0; q < 4; ++q) {
+          float acc = 0.f;
+#pragma unroll
+          for (int i = 0; i < TAPS; ++i) acc = fmaf(w[i], win[q + i], acc);
+          f[q][e] = acc * sigmoid_exact(acc);
+        }
+      } else {
+        for (int q = 0; q < 4; ++q) {
+          float acc = 0.f;
+          if (in && p0 + q < last)
+            for (int i = 0; i < c.taps; ++i) acc = fmaf(bf16_to_f32(tw[i]), input(p0 + q - past + i, at + j), acc);
+          f[q][e] = acc * sigmoid_exact(acc);
+        }
+      }
+#pragma unroll
+      for (int q = 0; q < 4; ++q) ss[q] = fmaf(f[q][e], f[q][e], ss[q]);
+    }
+#pragma unroll
+    for (int q = 0; q < 4; ++q) {
+      float scale = 1.f;
+      if (!is_v) {
+        scale = 1.0f / sqrtf(wave_sum(ss[q]) + 1e-6f);
+        if (seg < c.kv_heads) scale *= 1.0f / sqrtf((float)c.dim);
+      }
+      if (p0 + q >= last) continue;
+      float* to = out + (size_t)(s.row0 + p0 + q) * wide + at;
+#pragma unroll
+      for (int e = 0; e < 4; ++e)
+        if (lane + 64 * e < len) to[lane + 64 * e] = f[q][e] * scale;
+    }
   }
   if (first == 0) {   // no other block reads these channels' state
     __syncthreads();
@@ -309,7 +349,7 @@ __global__ __launch_bounds__(256) void delta_rule_kernel(const float* __restrict
       kn[e] = in ? row[qk + group * dim + i] : 0.f;
     }
     vn = live && vcol < vdim ? row[2 * qk + head * vdim + vcol] : 0.f;
-    gn = live ? row[channels + head] : 1.f;
+    gn = live ? row[channels + head] : 0.f;
     bn = live ? row[channels + heads + head] : 0.f;
   };
   fetch(0);
@@ -325,7 +365,7 @@ __global__ __launch_bounds__(256) void delta_rule_kernel(const float* __restrict
     b = group16_sum(b);
     if (ig == 0) {
       kq[tok] = b;
-      gs[tok] = gn;
+      gs[tok] = expf(gn);
       bs[tok] = bn;
     }
     __syncthreads();
@@ -363,31 +403,59 @@ __global__ __launch_bounds__(256) void delta_rule_kernel(const float* __restrict
 }
 
 // ------------------------------------------------------- per-head norm, gate
-// out = (o / rms(o)) * gain * silu(gate) * scale, the mean over one head's columns: a wave a head's row.
-template <typename T>
+// out = (o / rms(o)) * gain * silu(gate) * scale, the mean over one head's columns.
+// LANES lanes to a head's row of up to 4 LANES columns, four a lane where VEC (else one of every LANES).
+template <typename T, int LANES, bool VEC>
 __global__ __launch_bounds__(256) void head_gate_kernel(const float* __restrict__ o, const T* __restrict__ gate,
                                                         const bf16_t* __restrict__ gain, T* __restrict__ out, int rows,
                                                         int heads, int dim, int gate_stride, int gate_at, int gain_shared,
                                                         int out_stride, int out_at, float eps, float scale,
                                                         const int* __restrict__ valid) {
-  const long item = (long)blockIdx.x * 4 + (threadIdx.x >> 6);
-  const int row = (int)(item / heads), head = (int)(item - (long)row * heads), lane = threadIdx.x & 63;
+  const long item = ((long)blockIdx.x * 256 + threadIdx.x) / LANES;
+  const int row = (int)(item / heads), head = (int)(item - (long)row * heads), lane = threadIdx.x % LANES;
   if (row >= bound_or(valid, rows)) return;
   const float* src = o + ((size_t)row * heads + head) * dim;
-  float f[4], ss = 0.f;
+  const T* gr = gate + (size_t)row * gate_stride + gate_at + head * dim;
+  const bf16_t* wr = gain + (gain_shared ? 0 : head * dim);
+  T* to = out + (size_t)row * out_stride + out_at + head * dim;
+  float f[4] = {0.f, 0.f, 0.f, 0.f}, z[4], g[4], ss = 0.f;
+  const int c0 = lane * 4;
+  if (VEC && c0 < dim) {
+    const float4 v = *reinterpret_cast<const float4*>(src + c0);
+    f[0] = v.x; f[1] = v.y; f[2] = v.z; f[3] = v.w;
+    if constexpr (sizeof(T) == 2) {
+      const uint2 w = *reinterpret_cast<const uint2*>(gr + c0);
+      z[0] = bf16_lo(w.x); z[1] = bf16_hi(w.x); z[2] = bf16_lo(w.y); z[3] = bf16_hi(w.y);
+    } else {
+      const float4 w = *reinterpret_cast<const float4*>(gr + c0);
+      z[0] = w.x; z[1] = w.y; z[2] = w.z; z[3] = w.w;
+    }
+    const uint2 w = *reinterpret_cast<const uint2*>(wr + c0);
+    g[0] = bf16_lo(w.x); g[1] = bf16_hi(w.x); g[2] = bf16_lo(w.y); g[3] = bf16_hi(w.y);
+  } else if (!VEC) {
 #pragma unroll
-  for (int e = 0; e < 4; ++e) {
-    f[e] = lane + 64 * e < dim ? src[lane + 64 * e] : 0.f;
-    ss = fmaf(f[e], f[e], ss);
+    for (int e = 0; e < 4; ++e)
+      if (lane + LANES * e < dim) {
+        f[e] = src[lane + LANES * e];
+        z[e] = load_one(gr + lane + LANES * e);
+        g[e] = bf16_to_f32(wr[lane + LANES * e]);
+      }
   }
-  const float inv = 1.0f / sqrtf(wave_sum(ss) / (float)dim + eps);
 #pragma unroll
-  for (int e = 0; e < 4; ++e) {
-    const int j = lane + 64 * e;
-    if (j >= dim) continue;
-    const float z = load_one(gate + (size_t)row * gate_stride + gate_at + head * dim + j);
-    const float g = bf16_to_f32(gain[gain_shared ? j : head * dim + j]);
-    store_one(out + (size_t)row * out_stride + out_at + head * dim + j, f[e] * inv * g * (z * sigmoid_exact(z)) * scale);
+  for (int e = 0; e < 4; ++e) ss = fmaf(f[e], f[e], ss);
+#pragma unroll
+  for (int mask = 1; mask < LANES; mask <<= 1) ss += __shfl_xor(ss, mask, 64);
+  const float inv = 1.0f / sqrtf(ss / (float)dim + eps);
+  if (VEC) {
+    if (c0 >= dim) return;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) f[e] = f[e] * inv * g[e] * (z[e] * sigmoid_exact(z[e])) * scale;
+    if constexpr (sizeof(T) == 2) *reinterpret_cast<uint2*>(to + c0) = make_uint2(pack_bf16(f[0], f[1]), pack_bf16(f[2], f[3]));
+    else *reinterpret_cast<float4*>(to + c0) = make_float4(f[0], f[1], f[2], f[3]);
+  } else {
+#pragma unroll
+    for (int e = 0; e < 4; ++e)
+      if (lane + LANES * e < dim) store_one(to + lane + LANES * e, f[e] * inv * g[e] * (z[e] * sigmoid_exact(z[e])) * scale);
   }
 }
 
@@ -474,10 +542,20 @@ extern "C" int iron_short_conv(const void* x, const uint16_t* taps_w, const uint
   const ConvShape c{rows, stride, heads, kv_heads, dim, vdim, taps, b_at, a_at};
   const dim3 grid((rows + CONV_TILE - 1) / CONV_TILE, 2 * kv_heads + heads + 1, slots);
   IRON_REQUIRE(grid.y <= 65535, "short_conv: %d heads exceed the grid's y extent", heads);
-  if (is_float)
-    hipLaunchKernelGGL((short_conv_kernel<float>), grid, dim3(256), 0, (hipStream_t)stream, (const float*)x, taps_w, a_log, dt_bias, (float*)state, spans, out, c);
-  else
-    hipLaunchKernelGGL((short_conv_kernel<bf16_t>), grid, dim3(256), 0, (hipStream_t)stream, (const bf16_t*)x, taps_w, a_log, dt_bias, (bf16_t*)state, spans, out, c);
+#define IRON_CONV(T, N)                                                                                                  \
+  hipLaunchKernelGGL((short_conv_kernel<T, N>), grid, dim3(256), 0, (hipStream_t)stream, (const T*)x, taps_w, a_log, dt_bias, \
+                     (T*)state, spans, out, c)
+#define IRON_CONVS(T)                     \
+  {                                       \
+    if (taps == 2) IRON_CONV(T, 2);       \
+    else if (taps == 3) IRON_CONV(T, 3);  \
+    else if (taps == 4) IRON_CONV(T, 4);  \
+    else IRON_CONV(T, 0);                 \
+  }
+  if (is_float) IRON_CONVS(float)
+  else IRON_CONVS(bf16_t)
+#undef IRON_CONVS
+#undef IRON_CONV
   IRON_LAUNCH_CHECK();
 }
 
@@ -516,10 +594,23 @@ extern "C" int iron_head_gate(const float* o, const void* gate, const uint16_t* 
                "head_gate: %d columns from %d of a gate row of %d, from %d of an output row of %d", heads * dim, gate_at,
                gate_stride, out_at, out_stride);
   const long items = (long)rows * heads;
-  const dim3 grid((unsigned)((items + 3) / 4));
-  if (is_float)
-    hipLaunchKernelGGL((head_gate_kernel<float>), grid, dim3(256), 0, (hipStream_t)stream, o, (const float*)gate, gain, (float*)out, rows, heads, dim, gate_stride, gate_at, gain_shared, out_stride, out_at, eps, scale, valid);
-  else
-    hipLaunchKernelGGL((head_gate_kernel<bf16_t>), grid, dim3(256), 0, (hipStream_t)stream, o, (const bf16_t*)gate, gain, (bf16_t*)out, rows, heads, dim, gate_stride, gate_at, gain_shared, out_stride, out_at, eps, scale, valid);
+  const bool vec = dim % 4 == 0 && gate_stride % 4 == 0 && gate_at % 4 == 0 && out_stride % 4 == 0 && out_at % 4 == 0 &&
+                   (((uintptr_t)o | (uintptr_t)gate | (uintptr_t)gain | (uintptr_t)out) & 15) == 0;
+  const int lanes = !vec ? 64 : (dim <= 64 ? 16 : (dim <= 128 ? 32 : 64));
+  const dim3 grid((unsigned)((items * lanes + 255) / 256));
+#define IRON_HEAD_GATE(T, L, V)                                                                                              \
+  hipLaunchKernelGGL((head_gate_kernel<T, L, V>), grid, dim3(256), 0, (hipStream_t)stream, o, (const T*)gate, gain, (T*)out, rows, \
+                     heads, dim, gate_stride, gate_at, gain_shared, out_stride, out_at, eps, scale, valid)
+#define IRON_HEAD_GATES(T)                                   \
+  {                                                          \
+    if (!vec) IRON_HEAD_GATE(T, 64, false);                  \
+    else if (lanes == 16) IRON_HEAD_GATE(T, 16, true);       \
+    else if (lanes == 32) IRON_HEAD_GATE(T, 32, true);       \
+    else IRON_HEAD_GATE(T, 64, true);                        \
+  }
+  if (is_float) IRON_HEAD_GATES(float)
+  else IRON_HEAD_GATES(bf16_t)
+#undef IRON_HEAD_GATES
+#undef IRON_HEAD_GATE
   IRON_LAUNCH_CHECK();
 }

@@ -681,7 +681,14 @@ def low_rank_decay(z, w2, w0, out, *, rows, n, rank, valid=None):
                                     ptr(_word(valid, "valid")), current_stream()), "iron_low_rank_decay")
 
 
-def time_mix(r, k, v, log_decay, u, state, spans, o, *, slots, rows, heads, dim):
+def _work(t, nbytes, name):
+    if _dev(t, name, None).numel() * t.element_size() < nbytes:
+        raise ValueError(f"{name}: {t.numel() * t.element_size()} bytes, {nbytes} needed")
+    return ptr(t)
+
+
+def time_mix(r, k, v, log_decay, u, state, spans, o, *, slots, rows, heads, dim, workspace=None):
+    """The recurrence token by token, or with ``workspace`` sixteen tokens at a time."""
     n = rows * heads * dim
     is_float = _act(r, n, "r")
     _same_kind(is_float, k=k, v=v)
@@ -691,6 +698,12 @@ def time_mix(r, k, v, log_decay, u, state, spans, o, *, slots, rows, heads, dim)
     _bf16(u, heads * dim, "u")
     _f32(state, slots * heads * dim * dim, "state")
     _f32(o, n, "o")
+    if workspace is not None:
+        work = _work(workspace, int(lib().iron_time_mix_workspace_bytes(slots, rows, heads, dim)), "time_mix: workspace")
+        check(lib().iron_time_mix_chunked(ptr(r), ptr(k), ptr(v), ptr(log_decay), ptr(u), ptr(state), _spans(spans, slots),
+                                          ptr(o), work, slots, rows, heads, dim, int(is_float), current_stream()),
+              "iron_time_mix_chunked")
+        return
     check(lib().iron_time_mix(ptr(r), ptr(k), ptr(v), ptr(log_decay), ptr(u), ptr(state), _spans(spans, slots), ptr(o), slots,
                               rows, heads, dim, int(is_float), current_stream()), "iron_time_mix")
 
@@ -710,10 +723,16 @@ def short_conv(x, taps_w, a_log, dt_bias, state, spans, out, *, slots, rows, str
                                 current_stream()), "iron_short_conv")
 
 
-def delta_rule(x, state, spans, o, *, slots, rows, heads, kv_heads, dim, vdim):
+def delta_rule(x, state, spans, o, *, slots, rows, heads, kv_heads, dim, vdim, workspace=None):
+    """The recurrence token by token, or with ``workspace`` sixteen tokens at a time."""
     _f32(x, rows * (2 * kv_heads * dim + heads * vdim + 2 * heads), "x")
     _f32(state, slots * heads * dim * vdim, "state")
     _f32(o, rows * heads * vdim, "o")
+    if workspace is not None:
+        work = _work(workspace, int(lib().iron_delta_rule_workspace_bytes(slots, rows, heads)), "delta_rule: workspace")
+        check(lib().iron_delta_rule_chunked(ptr(x), ptr(state), _spans(spans, slots), ptr(o), work, slots, rows, heads, kv_heads,
+                                            dim, vdim, current_stream()), "iron_delta_rule_chunked")
+        return
     check(lib().iron_delta_rule(ptr(x), ptr(state), _spans(spans, slots), ptr(o), slots, rows, heads, kv_heads, dim, vdim,
                                 current_stream()), "iron_delta_rule")
 

@@ -13,7 +13,7 @@ from typing import Any
 import numpy as np
 
 from ..bf16 import bfloat16
-from ..common.declare import Built, In, InOut, Operator, Out, param, per_call
+from ..common.declare import Built, In, InOut, Operator, Out, Scratch, param, per_call
 from ..common.verify import Tolerance
 
 F32 = np.float32
@@ -21,6 +21,9 @@ F32 = np.float32
 
 class _Spanned(Operator):
     """An operator over a batch's rows told apart by spans."""
+
+    # A portion of many rows runs its recurrence sixteen tokens at a time, a decode step's few token by token.
+    CHUNKED_ROWS = 4   # rows a slot from which the chunks win
 
     def tolerance(self):
         return Tolerance.relative(1e-2, 1e-2, note="float32 inside, rounded once where it leaves")
@@ -109,7 +112,15 @@ class TimeMix(_Spanned):
     state = InOut(slots, heads, dim, dim, dtype=F32)
     spans = In(slots, 4, dtype=np.int32)
     o = Out(rows, width, dtype=F32)
+    chunked: bool = param(default=lambda op: op.rows > op.CHUNKED_ROWS * op.slots, array=True, repr=False)
+    workspace_words: int = param(derive=lambda op: op._workspace_words(), repr=False)
+    workspace = Scratch(workspace_words, dtype=np.float32, when=chunked)
     valid = per_call(bounds=rows)
+
+    def _workspace_words(self) -> int:
+        from .._lib import lib
+
+        return int(lib().iron_time_mix_workspace_bytes(self.slots, self.rows, self.heads, self.dim)) // 4
 
     @classmethod
     def infer(cls, shapes, **kw):
@@ -125,14 +136,15 @@ class TimeMix(_Spanned):
         kw = dict(slots=self.slots, rows=self.rows, heads=self.heads, dim=self.dim)
 
         def launch(t, words):
-            kernels.time_mix(t["r"], t["k"], t["v"], t["log_decay"], t["u"], t["state"], t["spans"], t["o"], **kw)
+            kernels.time_mix(t["r"], t["k"], t["v"], t["log_decay"], t["u"], t["state"], t["spans"], t["o"],
+                             workspace=t.get("workspace"), **kw)
 
         return Built("iron_time_mix", launch)
 
 
 class _DeltaShape(_Spanned):
     """Sizes of a gated delta rule: ``kv_heads`` q/k heads of ``dim``, ``heads`` value heads of ``vdim``;
-    the rows between its two steps are ``[unit q | unit k | v | decay | beta]`` in float32."""
+    the rows between its two steps are ``[unit q | unit k | v | log decay | beta]`` in float32."""
 
     slots: int = param()
     rows: int = param()
@@ -152,8 +164,8 @@ class _DeltaShape(_Spanned):
 
 class ShortConv(_DeltaShape):
     """From a packed projection ``[q | k | v | .. b .. | .. a ..]``: a short causal convolution per channel
-    and SiLU on q, k and v, unit q (times ``dim ** -0.5``) and k per head, and the step's decay and write
-    strength.  ``state`` keeps position p's inputs in row ``p % taps`` of its slot."""
+    and SiLU on q, k and v, unit q (times ``dim ** -0.5``) and k per head, and the step's log decay and
+    write strength.  ``state`` keeps position p's inputs in row ``p % taps`` of its slot."""
 
     stride: int = param()
     taps: int = param()
@@ -198,7 +210,15 @@ class DeltaRule(_DeltaShape):
     state = InOut(_DeltaShape.slots, _DeltaShape.heads, _DeltaShape.dim, _DeltaShape.vdim, dtype=F32)
     spans = In(_DeltaShape.slots, 4, dtype=np.int32)
     o = Out(_DeltaShape.rows, width, dtype=F32)
+    chunked: bool = param(default=lambda op: op.rows > op.CHUNKED_ROWS * op.slots, array=True, repr=False)
+    workspace_words: int = param(derive=lambda op: op._workspace_words(), repr=False)
+    workspace = Scratch(workspace_words, dtype=np.float32, when=chunked)
     valid = per_call(bounds=_DeltaShape.rows)
+
+    def _workspace_words(self) -> int:
+        from .._lib import lib
+
+        return int(lib().iron_delta_rule_workspace_bytes(self.slots, self.rows, self.heads)) // 4
 
     @classmethod
     def infer(cls, shapes, **kw):
@@ -211,7 +231,7 @@ class DeltaRule(_DeltaShape):
         kw = {n: getattr(self, n) for n in ("slots", "rows", "heads", "kv_heads", "dim", "vdim")}
 
         def launch(t, words):
-            kernels.delta_rule(t["x"], t["state"], t["spans"], t["o"], **kw)
+            kernels.delta_rule(t["x"], t["state"], t["spans"], t["o"], workspace=t.get("workspace"), **kw)
 
         return Built("iron_delta_rule", launch)
 
