@@ -369,6 +369,13 @@ int iron_sample_advance_bf16(const uint16_t* logits, int n, const int* draws, in
  * iron/common/graph/carried.py:189-276, iron/operators/emit.py. */
 int iron_eval_words(int* words, int n_words, const int* exprs, int n, void* stream);
 
+/* C = A B^T for up to 64 rows of A, or with B2 C = act(A B^T) * (A B2^T) (activation 1 SiLU, 2 GELU by its
+ * tanh form, 3 ReLU; rounded where the separate steps round): bound by streaming B.  A (M, K), B and B2
+ * (N, K), C (M, N); K % 8 == 0.  What iron_gemm_bf16 and iron_gemm_gated_pair_bf16 launch for fewer than 64
+ * rows without a bound (the latter needs no G then). */
+int iron_gemm_few_bf16(const uint16_t* A, const uint16_t* B, const uint16_t* B2, uint16_t* C, int M, int N, int K,
+                       int activation, void* stream);
+
 /* ---- decoders with a float32 residual stream and layers that carry a state, over a batch of rows.
  *
  * `spans` is an int32 (slots, 4) table in device memory, 16-byte aligned: {row0, rows, start, unused}

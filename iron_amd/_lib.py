@@ -88,6 +88,7 @@ SIGNATURES = {
     "iron_sample_bf16": (c_int, [_P, c_int, _P, c_int, _P, c_int, _P, _P, _P, c_int, _P, _P, _P]),
     "iron_sample_advance_bf16": (c_int, [_P, c_int, _P, c_int, _P, c_int, _P, _P, _P, c_int, _P, _P, _P, c_int, _P,
                                          c_int, _P]),
+    "iron_gemm_few_bf16": (c_int, [_P, _P, _P, _P, c_int, c_int, c_int, c_int, _P]),
     "iron_stream_embed": (c_int, [_P, _P, _P, c_int, c_int, c_int, _P, _P]),
     "iron_stream_rows": (c_int, [_P, _P, _P, _P, _P, c_int, c_int, c_float, c_int, _P, _P]),
     "iron_span_tails": (c_int, [_P, _P, _P, c_int, c_int, c_int, _P]),

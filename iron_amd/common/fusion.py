@@ -156,7 +156,8 @@ def plan(recording, tensor: Callable[[Any], Any], word: Callable[[Any], Any],
                 and _gate(sl) is not None
                 and _name(ml) == "ElementwiseMul"
                 and s.op.b_col_maj and not s.op.c_col_maj and "valid_k" not in s.values
-                and s.op.M >= 64 and s.op.N >= 64 and s.op.K % 64 == 0):
+                and ((s.op.M >= 64 and s.op.N >= 64 and s.op.K % 64 == 0)
+                     or (s.op.M < 64 and before is not None and "valid" not in s.values))):   # a batch's few rows
             return None
         up, gate, act = s.outputs["C"], sl.inputs["x"], sl.outputs["y"]
         a, b = ml.inputs["a"], ml.inputs["b"]

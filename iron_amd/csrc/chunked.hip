@@ -391,7 +391,10 @@ __global__ __launch_bounds__(256) void delta_walk_kernel(const float* __restrict
     p.G = reinterpret_cast<const float4*>(w + 512)[quad];
     p.left = reinterpret_cast<const float4*>(w + 528)[quad];
     p.beta = reinterpret_cast<const float4*>(w + 544)[quad];
-    p.whole = w[512 + CHUNK - 1];
+    // (by a vector register's index: a scalar load would be waited for with the next LDS read)
+    int last = 512 + CHUNK - 1;
+    asm volatile("" : "+v"(last));
+    p.whole = w[last];
     p.P = w[256 + lane * 4 + wave];
 #pragma unroll
     for (int j = 0; j < 4; ++j) p.v[j] = one(down[j] + 4 * (2 * qkw + head * vdim + min(col, vdim - 1)));

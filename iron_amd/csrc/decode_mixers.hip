@@ -101,8 +101,25 @@ __device__ __forceinline__ void time_mix_step(const TimeMixStep& a, const Span& 
     bonus = r * k * bf16_to_f32(a.u[head * dim + t]);
   }
   for (int i = t; i < a.rank; i += DM_THREADS) sh.z[i] = tanhf(bf16_to_f32(a.z[row * a.rank + i]));
+  // The decays: a channel's row of w2 over as many lanes as it has 16-byte pieces, the first ones asked for
+  // ahead of the barrier; or, where its pieces are no power of two, over a wave.
+  const int pieces = a.rank >> 3, piece = t & (pieces - 1);
+  const bool dealt = a.rank % 8 == 0 && (pieces & (pieces - 1)) == 0 && pieces <= 64;
+  uint4 ahead = make_uint4(0, 0, 0, 0);
+  if (dealt && t / pieces < dim) ahead = reinterpret_cast<const uint4*>(a.w2 + (size_t)(head * dim + t / pieces) * a.rank)[piece];
   bonus = dm_block_sum(bonus, sh.part[0]);   // its barrier is the one the LDS rows wait for, too
-  for (int c = wave; c < dim; c += DM_WAVES) {   // the decays, a channel a wave at a time
+  if (dealt) {
+    for (int c = t / pieces; c - t / pieces < dim; c += DM_THREADS / pieces) {
+      float f[8], sum = 0.f;
+      unpack8(ahead, f);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) sum = fmaf(f[j], sh.z[piece * 8 + j], sum);
+      for (int mask = 1; mask < pieces; mask <<= 1) sum += __shfl_xor(sum, mask, 64);
+      if (piece == 0 && c < dim) sh.w[c] = expf(-expf(sum + bf16_to_f32(a.w0[head * dim + c])));
+      const int next = c + DM_THREADS / pieces;
+      if (next < dim) ahead = reinterpret_cast<const uint4*>(a.w2 + (size_t)(head * dim + next) * a.rank)[piece];
+    }
+  } else for (int c = wave; c < dim; c += DM_WAVES) {
     const bf16_t* w = a.w2 + (size_t)(head * dim + c) * a.rank;
     float sum = 0.f;
     for (int i = lane; i < a.rank; i += 64) sum = fmaf(bf16_to_f32(w[i]), sh.z[i], sum);
@@ -146,7 +163,7 @@ struct WindowStep {
 };
 struct WindowShared1 {
   float q[256], p[DM_WAVES][64], m[DM_WAVES], l[DM_WAVES];
-  float red[DM_WAVES * 512];              // [wave][keys at once][vdim], at most 512 floats a wave
+  __align__(16) float red[DM_WAVES * 512];              // [wave][keys at once][vdim], at most 512 floats a wave
 };
 
 __device__ __forceinline__ void window_step(const WindowStep& a, const Span& s, int slot, int head, WindowShared1& sh) {
@@ -233,6 +250,120 @@ __device__ __forceinline__ void window_step(const WindowStep& a, const Span& s, 
   }
 }
 
+// The same where keys and values are LANES 16-byte pieces wide: LANES lanes to a key, 64 / LANES keys at a
+// time, eight such steps' keys, values and biases asked for together.  A lane's scores are its own keys',
+// and it weighs the same keys' values, so nothing is exchanged until the waves meet.
+template <int LANES>
+__device__ __forceinline__ float lanes_sum(float v) {
+  static_assert(LANES == 4 || LANES == 8 || LANES == 16 || LANES == 32, "a power of two of lanes");
+  v += IRON_DPP(0.f, v, 0xB1, 0xF);
+  v += IRON_DPP(0.f, v, 0x4E, 0xF);
+  if (LANES >= 8) v += IRON_DPP(0.f, v, 0x141, 0xF);
+  if (LANES >= 16) v += IRON_DPP(0.f, v, 0x140, 0xF);
+  if (LANES >= 32) v += __shfl_xor(v, 16, 64);
+  return v;
+}
+template <int LANES>
+__device__ __forceinline__ void window_step_lanes(const WindowStep& a, const Span& s, int slot, int head, WindowShared1& sh) {
+  constexpr int AT_ONCE = 64 / LANES, STEPS = 8, KEYS = AT_ONCE * STEPS;
+  const int t = threadIdx.x, lane = t & 63, wave = t >> 6, group = a.heads / a.kv_heads, g = head / group;
+  const int nk = a.kv_heads * a.dim, part = lane % LANES, mine = lane / LANES;
+  const int pos = s.start, lo = max(0, pos - a.window + 1), count = pos - lo + 1, wrap = lo % a.ring;
+  const bf16_t* row = a.x + (size_t)s.row0 * a.stride;
+  const bf16_t* own_k = row + a.heads * a.dim + g * a.dim;
+  const bf16_t* own_v = own_k + nk;
+  bf16_t* ring_k = a.keys + (size_t)slot * a.ring * nk + g * a.dim;
+  bf16_t* ring_v = a.values + (size_t)slot * a.ring * nk + g * a.dim;
+  float q[8];
+  unpack8(*reinterpret_cast<const uint4*>(row + head * a.dim + part * 8), q);
+#pragma unroll
+  for (int j = 0; j < 8; ++j) q[j] *= a.scale;
+  if (head % group == 0 && t < 2 * LANES) {   // position pos - ring, whose row this replaces, is outside the window
+    const bf16_t* src = t < LANES ? own_k : own_v;
+    bf16_t* dst = (t < LANES ? ring_k : ring_v) + (size_t)(pos % a.ring) * nk;
+    reinterpret_cast<uint4*>(dst)[part] = reinterpret_cast<const uint4*>(src)[part];
+  }
+  const long own_k_from = (const char*)own_k - (const char*)ring_k, own_v_from = (const char*)own_v - (const char*)ring_v;
+  const float* by = a.bias + (size_t)head * a.window;
+  float acc[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f}, m = -INFINITY, l = 0.f;
+  for (int k0 = wave * KEYS; k0 < count; k0 += DM_WAVES * KEYS) {
+    u32x4 kv[STEPS], vv[STEPS];
+    float score[STEPS];
+#pragma unroll
+    for (int i = 0; i < STEPS; ++i) {
+      const int n = min(k0 + i * AT_ONCE + mine, count - 1);
+      const long mask = -(long)(n == count - 1);
+      const int at = wrap + n, back = at - a.ring;
+      const long old = (long)(back >= 0 ? back : at) * (2 * nk);
+      kv[i] = *reinterpret_cast<const u32x4*>((const char*)(ring_k + part * 8) + ((own_k_from & mask) | (old & ~mask)));
+      vv[i] = *reinterpret_cast<const u32x4*>((const char*)(ring_v + part * 8) + ((own_v_from & mask) | (old & ~mask)));
+      score[i] = by[count - 1 - n];
+    }
+    float top = m;
+#pragma unroll
+    for (int i = 0; i < STEPS; ++i) {
+      float f[8], dot = 0.f;
+      unpack8(make_uint4(kv[i].x, kv[i].y, kv[i].z, kv[i].w), f);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) dot = fmaf(f[j], q[j], dot);
+      score[i] = k0 + i * AT_ONCE + mine < count ? score[i] + lanes_sum<LANES>(dot) : -INFINITY;
+      top = fmaxf(top, score[i]);
+    }
+#pragma unroll
+    for (int mask = LANES; mask < 64; mask <<= 1) top = fmaxf(top, __shfl_xor(top, mask, 64));
+    const float fade = __expf(m - top);   // top is finite: the piece's first key is one
+    m = top;
+    l *= fade;
+#pragma unroll
+    for (int j = 0; j < 8; ++j) acc[j] *= fade;
+#pragma unroll
+    for (int i = 0; i < STEPS; ++i) {
+      float f[8];
+      const float p = __expf(score[i] - top);
+      l += p;
+      unpack8(make_uint4(vv[i].x, vv[i].y, vv[i].z, vv[i].w), f);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) acc[j] = fmaf(p, f[j], acc[j]);
+    }
+  }
+#pragma unroll
+  for (int mask = LANES; mask < 64; mask <<= 1) {
+    l += __shfl_xor(l, mask, 64);
+#pragma unroll
+    for (int j = 0; j < 8; ++j) acc[j] += __shfl_xor(acc[j], mask, 64);
+  }
+  if (lane == 0) {
+    sh.m[wave] = m;
+    sh.l[wave] = l;
+  }
+  if (mine == 0) {
+    float4* to = reinterpret_cast<float4*>(&sh.red[wave * a.dim + part * 8]);
+    to[0] = make_float4(acc[0], acc[1], acc[2], acc[3]);
+    to[1] = make_float4(acc[4], acc[5], acc[6], acc[7]);
+  }
+  __syncthreads();
+  if (t < a.dim) {
+    float top = sh.m[0], total = 0.f, sum = 0.f;
+#pragma unroll
+    for (int w = 1; w < DM_WAVES; ++w) top = fmaxf(top, sh.m[w]);
+#pragma unroll
+    for (int w = 0; w < DM_WAVES; ++w) {   // a wave without a key: m is -inf, the rest 0
+      const float fade = __expf(sh.m[w] - top);
+      total = fmaf(sh.l[w], fade, total);
+      sum = fmaf(sh.red[w * a.dim + t], fade, sum);
+    }
+    a.out[(size_t)s.row0 * a.out_stride + a.out_at + head * a.dim + t] = f32_to_bf16(sum / total * a.out_scale);
+  }
+}
+
+__device__ __forceinline__ void window_step_any(const WindowStep& a, const Span& s, int slot, int head, WindowShared1& sh) {
+  if (a.dim == a.vdim && a.dim == 64) window_step_lanes<8>(a, s, slot, head, sh);
+  else if (a.dim == a.vdim && a.dim == 128) window_step_lanes<16>(a, s, slot, head, sh);
+  else if (a.dim == a.vdim && a.dim == 32) window_step_lanes<4>(a, s, slot, head, sh);
+  else if (a.dim == a.vdim && a.dim == 256) window_step_lanes<32>(a, s, slot, head, sh);
+  else window_step(a, s, slot, head, sh);
+}
+
 union ParallelShared {
   TimeMixShared mix;
   WindowShared1 win;
@@ -243,7 +374,7 @@ __global__ __launch_bounds__(DM_THREADS) void decode_parallel_kernel(TimeMixStep
   const int slot = blockIdx.y;
   const Span s = span_of(spans, slot, rows);
   if (s.rows == 0) return;
-  if ((int)blockIdx.x < win.heads) window_step(win, s, slot, blockIdx.x, sh.win);
+  if ((int)blockIdx.x < win.heads) window_step_any(win, s, slot, blockIdx.x, sh.win);
   else time_mix_step<NR>(mix, s, slot, blockIdx.x - win.heads, sh.mix);
 }
 

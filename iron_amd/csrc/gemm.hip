@@ -2085,6 +2085,9 @@ extern "C" int iron_gemm_bf16(const uint16_t* A, const uint16_t* B, uint16_t* C,
   IRON_REQUIRE(b_col_maj || N % 8 == 0,
                "gemm: N (%d) must be a multiple of 8 when B is (K,N) (16-byte loads along N)", N);
   hipStream_t s = (hipStream_t)stream;
+  // Fewer rows than the smallest tile: bound by streaming B.
+  if (M < 64 && b_col_maj && !c_col_maj && valid == nullptr && valid_k == nullptr)
+    return iron_gemm_few_bf16(A, B, nullptr, C, M, N, K, 0, stream);
   if (!c_col_maj && valid_k == nullptr && K % BK == 0 && M >= 64 && N >= 64) {
     // Enough whole 256x256 tiles to fill the chip: the large-tile kernel (offsets are 32-bit).
     if (b_col_maj && M % BIG_BM == 0 && N % BIG_BN == 0 && (long)(M / BIG_BM) * (N / BIG_BN) >= 192 &&
@@ -2218,9 +2221,10 @@ extern "C" int iron_gemm_gated_bf16(const uint16_t* A, const uint16_t* B, const 
 extern "C" int iron_gemm_gated_pair_bf16(const uint16_t* A, const uint16_t* Bg, const uint16_t* Bu, uint16_t* G,
                                          uint16_t* C, int M, int N, int K, int activation, const int* valid,
                                          void* stream) {
-  IRON_REQUIRE(A && Bg && Bu && G && C, "gemm_gated_pair: null operand");
+  IRON_REQUIRE(A && Bg && Bu && C && (G || M < 64), "gemm_gated_pair: null operand");
   IRON_REQUIRE(activation >= 1 && activation <= 3, "gemm_gated_pair: activation (%d) is 1 (SiLU), 2 (GELU, tanh form) or 3 (ReLU)",
                activation);
+  if (M < 64 && valid == nullptr) return iron_gemm_few_bf16(A, Bg, Bu, C, M, N, K, activation, stream);
   IRON_REQUIRE(G != C, "gemm_gated_pair: the gate's product and the output are different buffers");
   IRON_REQUIRE(K <= (1 << 22) && N <= (1 << 22),
                "gemm_gated_pair: K (%d) and N (%d) may be at most 2^22 (a tile's rows are addressed with 32-bit offsets)", K, N);
