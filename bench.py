@@ -712,6 +712,7 @@ def pegilix_served(torch, config, weights, steps, prompts):
 
     run_prompt(min(prompts))
     first = time_served(torch, run_prompt, _Started(model, steps), steps, prompts)
+    first["prompt_tok_s"] = {n: round(v * config.slots, 1) for n, v in first["prompt_tok_s"].items()}
     first["launches_per_step"] = model.decode_step.launches_per_replay
     first["launches_per_portion"] = model.prompt_chunk.launches_per_call
     weight_bytes = 2 * sum(int(np.prod(t.shape)) for n, t in weights.items() if n != "embed")

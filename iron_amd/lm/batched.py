@@ -17,13 +17,12 @@ from typing import Any
 
 import numpy as np
 
-from ..bf16 import bfloat16
 from ..common import graph as iron
 from ..common.graph import Scratchpad
 from ..operators.copy import Copy
 from ..operators.sample import ROW_WORDS, SampleSlots
 from ..operators.stream import Softcap, SpanTails, StreamEmbed
-from .causal import CausalLM, Decoder
+from .causal import CausalLM, Decoder, OnHost, _HostOutput, _HostVersion
 from .mixers import StreamRMSNorm, as_rows
 from .session import Session
 
@@ -356,7 +355,7 @@ class BatchedLM(CausalLM):
     def __init__(self, config, weights):
         super().__init__(config, weights)
         c = config
-        self.stream = iron.state((max(c.prefill_chunk, c.slots), c.hidden_size), np.float32)
+        self.residual = iron.state((max(c.prefill_chunk, c.slots), c.hidden_size), np.float32)
         self.spans = iron.state((c.slots, 4), np.int32)
         self.token = iron.state((c.slots,), np.int32)
         self.runs = [(i, self.layers[i].mixer.states(c.slots)) for i in c.order]
@@ -371,10 +370,10 @@ class BatchedLM(CausalLM):
     def body(self, ids=None, picks=None, *, rows: Scratchpad[np.int32] = np.int32(1)):
         c = self.config
         if picks is not None:
-            return self.head(Copy.step(self.stream[picks], dtype=np.float32))[0]
+            return self.head(Copy.step(self.residual[picks], dtype=np.float32))[0]
         call = BatchCall(prompt=ids is not None, spans=self.spans, rows=rows)
         count = c.prefill_chunk if call.prompt else c.slots
-        x = call.bound(self.stream[:count])
+        x = call.bound(self.residual[:count])
         ids = call.bound(ids) if call.prompt else self.token
         StreamEmbed.step(self.model.embed_tokens.weight, ids, x)
         for index, states in self.runs:
@@ -418,6 +417,21 @@ class BatchedLM(CausalLM):
         return self.batch.generate([self._prompt_ids(p) for p in prompts], max_tokens, samplers)
 
 
-def runs_in_32_bits(config) -> bool:
-    """Whether the config's activations are float32 throughout."""
-    return getattr(config, "activations", bfloat16) is not bfloat16
+class _HostBatchVersion(_HostVersion):
+    """A batched version stood in by the graph's host reference."""
+
+    def __init__(self, graph, name: str | None = None):
+        super().__init__(graph, name is not None)
+        self.name = name
+
+    def __call__(self, *tensors, **values):
+        lead = (None,) if self.name == "picks" else ()
+        outs, _ = iron.Graph.reference(self.graph, *lead, *tensors, **values)
+        return _HostOutput(outs[0])
+
+
+class BatchedOnHost(OnHost):
+    """``OnHost`` for a batched model."""
+
+    def load_versions(self, **_):
+        self.use(_HostBatchVersion(self), _HostBatchVersion(self, "ids"), _HostBatchVersion(self, "picks"))

@@ -9,6 +9,8 @@ from __future__ import annotations
 
 import numpy as np
 
+from iron_amd.bf16 import bfloat16, round_bf16
+
 from . import ops
 
 
@@ -144,6 +146,170 @@ def sample(op, logits, draws, tokens, *, row=0, at=0):
     return tokens, np.array([token], dtype=np.int32)
 
 
+# ---- the float32 stream and the layers that carry a state.  ``_out`` rounds to the operator's dtype.
+
+
+def _out(op, x):
+    x = np.asarray(x, np.float32)
+    return round_bf16(x) if op.dtype is bfloat16 else x
+
+
+def _spans(spans):
+    """(slot, first row, rows, first position) of every slot that has rows."""
+    return [(s, int(r), int(n), int(p)) for s, (r, n, p, _) in enumerate(np.asarray(spans)) if n]
+
+
+def stream_embed(op, table, ids):
+    return np.asarray(table, np.float32)[np.clip(np.asarray(ids).reshape(-1), 0, op.table_rows - 1)]
+
+
+def _unit_rms(x, eps):
+    x = np.asarray(x, np.float64)
+    return x / np.sqrt((x * x).mean(-1, keepdims=True) + eps)
+
+
+def stream_norm(op, x, weight):
+    return _out(op, _unit_rms(x, op.epsilon) * np.asarray(weight, np.float64))
+
+
+def stream_add(op, x, y, weight):
+    return np.asarray(x + _unit_rms(y, op.epsilon) * np.asarray(weight, np.float64), np.float32)
+
+
+def span_tails(op, x, spans):
+    y = np.zeros((op.slots, op.cols), np.float32)
+    for s, row, n, _ in _spans(spans):
+        y[s] = x[row + n - 1]
+    return y
+
+
+def softcap(op, x):
+    y = np.asarray(x, np.float64)
+    y = np.asarray(op.cap * np.tanh(y / op.cap) if op.cap else y, np.float32)
+    rounded = np.zeros((op.rows, op.stride), np.float32)
+    rounded[:, : op.cols] = round_bf16(y)
+    return y, rounded
+
+
+def gated_product(op, gate, up):
+    g = np.asarray(gate, np.float64)
+    act = {"relu": lambda z: np.maximum(z, 0), "silu": lambda z: z / (1 + np.exp(-z)),
+           "gelu_tanh": lambda z: 0.5 * z * (1 + np.tanh(np.sqrt(2 / np.pi) * (z + 0.044715 * z**3)))}[op.activation]
+    return np.asarray(act(g) * up, np.float32)
+
+
+def linear_any(op, x, weight):
+    return _out(op, np.asarray(x, np.float64) @ np.asarray(weight, np.float64).T)
+
+
+def token_shift(op, h, mu, carry, spans):
+    carry, mixed = np.array(carry), np.zeros((op.mixes, op.rows, op.cols), np.float32)
+    for s, row, n, start in _spans(spans):
+        own = np.asarray(h[row : row + n], np.float64)
+        before = np.concatenate([carry[s, (start - 1) % 2][None] if start else np.zeros((1, op.cols)), own[:-1]])
+        mixed[:, row : row + n] = own + (before - own) * np.asarray(mu, np.float64)[:, None]
+        carry[s, (start + n - 1) % 2] = h[row + n - 1]
+    return carry, _out(op, mixed)
+
+
+def low_rank_decay(op, z, up, base):
+    return np.asarray(-np.exp(np.tanh(np.asarray(z, np.float64)) @ np.asarray(up, np.float64).T + base), np.float32)
+
+
+def time_mix(op, r, k, v, log_decay, u, state, spans):
+    H, D = op.heads, op.dim
+    state, o = np.array(state), np.zeros((op.rows, H, D), np.float32)
+    r, k, v, w = (np.asarray(x, np.float64).reshape(op.rows, H, D) for x in (r, k, v, log_decay))
+    for s, row, n, start in _spans(spans):
+        S = np.asarray(state[s], np.float64) if start else np.zeros((H, D, D))
+        for t in range(row, row + n):
+            kv = k[t][:, :, None] * v[t][:, None, :]
+            o[t] = np.einsum("hi,hij->hj", r[t], S + np.asarray(u, np.float64)[:, :, None] * kv)
+            S = np.exp(w[t])[:, :, None] * S + kv
+        state[s] = S
+    return state, o.reshape(op.rows, -1)
+
+
+def short_conv(op, x, weight, a_log, dt_bias, state, spans):
+    G, H, D, V, C = op.kv_heads, op.heads, op.dim, op.vdim, op.channels
+    state, y = np.array(state), np.zeros((op.rows, op.wide), np.float32)
+    for s, row, n, start in _spans(spans):
+        rows = np.asarray(x[row : row + n], np.float64)
+        past = [state[s, p % op.taps] if p >= 0 else np.zeros(C) for p in range(start - op.taps + 1, start)]
+        fed = np.concatenate([np.reshape(past, (-1, C)), rows[:, :C]])
+        conv = sum(fed[i : i + n] * np.asarray(weight, np.float64)[:, i] for i in range(op.taps))
+        conv = conv / (1 + np.exp(-conv))
+        qk = conv[:, : 2 * G * D].reshape(n, 2, G, D)
+        qk = qk / np.sqrt((qk * qk).sum(-1, keepdims=True) + 1e-6)
+        qk[:, 0] *= D**-0.5
+        decay = -np.exp(np.asarray(a_log, np.float64)) * np.logaddexp(0, rows[:, op.a_at : op.a_at + H] + dt_bias)
+        beta = 1 / (1 + np.exp(-rows[:, op.b_at : op.b_at + H]))
+        y[row : row + n] = np.concatenate([qk.reshape(n, -1), conv[:, 2 * G * D :], decay, beta], axis=1)
+        for p in range(max(start, start + n - op.taps), start + n):
+            state[s, p % op.taps] = x[row + p - start][:C]
+    return state, y
+
+
+def delta_rule(op, x, state, spans):
+    G, H, D, V, C = op.kv_heads, op.heads, op.dim, op.vdim, op.channels
+    x, state, o = np.asarray(x, np.float64), np.array(state), np.zeros((op.rows, H, V), np.float32)
+    group = np.arange(H) // (H // G)
+    q, k = x[:, : G * D].reshape(-1, G, D)[:, group], x[:, G * D : 2 * G * D].reshape(-1, G, D)[:, group]
+    v, g, beta = x[:, 2 * G * D : C].reshape(-1, H, V), np.exp(x[:, C : C + H]), x[:, C + H :]
+    for s, row, n, start in _spans(spans):
+        S = np.asarray(state[s], np.float64) if start else np.zeros((H, D, V))
+        for t in range(row, row + n):
+            S = g[t][:, None, None] * S
+            u = beta[t][:, None] * (v[t] - np.einsum("hij,hi->hj", S, k[t]))
+            S = S + k[t][:, :, None] * u[:, None, :]
+            o[t] = np.einsum("hij,hi->hj", S, q[t])
+        state[s] = S
+    return state, o.reshape(op.rows, -1)
+
+
+def head_gate(op, o, gate, gain):
+    H, D = op.heads, op.dim
+    z = np.asarray(gate, np.float64)[:, op.gate_at : op.gate_at + H * D]
+    gains = np.asarray(gain, np.float64) if op.gains == op.o_width else np.tile(np.asarray(gain, np.float64), H)
+    y = np.zeros((op.rows, op.width), np.float32)
+    y[:, op.at : op.at + H * D] = (_unit_rms(np.reshape(o, (-1, H, D)), op.epsilon).reshape(op.rows, -1) * gains
+                                   * z / (1 + np.exp(-z)) * op.scale)
+    return _out(op, y)
+
+
+def window_mha(op, x, bias, spans, keys, values, y):
+    H, G, D, V = op.heads, op.kv_heads, op.dim, op.vdim
+    keys, values, y = np.array(keys), np.array(values), np.array(y)
+    for s, row, n, start in _spans(spans):
+        rows = np.asarray(x[row : row + n], np.float64)
+        q, k, v = rows[:, : H * D].reshape(n, H, D), rows[:, H * D : (H + G) * D].reshape(n, G, D), \
+            rows[:, (H + G) * D : (H + G) * D + G * V].reshape(n, G, V)
+        first = max(0, start - op.window + 1)
+        old = [p % op.ring for p in range(first, start)]
+        allk = np.concatenate([np.asarray(keys[s][old], np.float64), k])
+        allv = np.concatenate([np.asarray(values[s][old], np.float64), v])
+        for i in range(n):
+            lo = max(0, start + i - op.window + 1)
+            a, b = lo - first, start + i + 1 - first
+            for h in range(H):
+                score = allk[a:b, h // (H // G)] @ q[i, h] * op.scale + bias[h][: b - a][::-1]
+                p = np.exp(score - score.max())
+                y[row + i, op.at + h * V : op.at + (h + 1) * V] = p / p.sum() @ allv[a:b, h // (H // G)] * op.out_scale
+        for i in range(max(0, n - op.ring), n):
+            keys[s, (start + i) % op.ring], values[s, (start + i) % op.ring] = k[i], v[i]
+    return keys, values, _out(op, y)
+
+
+def sample_slots(op, logits, draws, spans, token, tokens):
+    spans, token, tokens = np.array(spans), np.array(token), np.array(tokens)
+    for s, _, n, start in _spans(spans):
+        at = start + n - 1
+        temperature, top_k, n53 = ops.draw_words(np.asarray(draws)[s, at])
+        token[s] = tokens[s, at] = ops.sample_ref(np.asarray(logits)[s, : op.vocab], temperature, top_k, n53, op.k_max)
+        spans[s] = s, 1, at + 1, 0
+    return spans, token, tokens
+
+
 def install() -> None:
     from iron_amd.common.declare import REFERENCES
 
@@ -151,7 +317,10 @@ def install() -> None:
         GEMM=gemm, GEMV=gemv, RMSNorm=rms_norm, SiLU=silu, ElementwiseMul=mul, ElementwiseAdd=add,
         RoPE=rope, MHA=mha, Copy=copy, Gather=gather, GatherWords=gather_words, Sample=sample, RowwiseAdd=rowwise_add, RowwiseMul=rowwise_mul,
         GELU=gelu, ReLU=relu, Sigmoid=sigmoid, Tanh=tanh, Clamp=clamp, AXPY=axpy, LayerNorm=layer_norm,
-        Softmax=softmax,
+        Softmax=softmax, StreamEmbed=stream_embed, StreamNorm=stream_norm, StreamAdd=stream_add, SpanTails=span_tails,
+        Softcap=softcap, GatedProduct=gated_product, LinearAny=linear_any, TokenShift=token_shift, LowRankDecay=low_rank_decay,
+        TimeMix=time_mix, ShortConv=short_conv, DeltaRule=delta_rule, HeadGate=head_gate, WindowMHA=window_mha,
+        SampleSlots=sample_slots,
         # The host's draw, for iron_amd.lm.generation.Sampler's checks.
         sample_ref=ops.sample_ref, sample_weights=ops.sample_weights,
     )

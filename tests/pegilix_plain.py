@@ -176,5 +176,5 @@ class Plain:
             if trace is not None:
                 trace.append(x)
         logits = rms_norm(x, self.w["final.norm"], self.eps) @ self.w["head"].T
-        cap = self.c["logit_softcap"]
-        return cap * np.tanh(logits / cap)
+        cap = self.c.get("logit_softcap")
+        return logits if cap is None else cap * np.tanh(logits / cap)
