@@ -226,11 +226,10 @@ __device__ __forceinline__ void window_prefill_body(const bf16_t* __restrict__ x
   u32x4 kn[KP], vn[VT][4];
   float bn = 0.f;
   // The next tile on its way from memory: keys at positions base .. base + 63, by 32-bit offsets into bounded
-  // buffers (a row past the batch's last reads as zeros; one past the span's last, another sequence's, is
-  // masked below).  A thread's offsets into a tile of the call's own rows are the same for every tile.
+  // buffers: a row past the span's last, which may hold anything, reads as zeros.  A thread's offsets into a tile of the call's own rows are the same for every tile.
   // Columns past a head's width read its last ones: q is zero there, and those of v are not stored.
-  const __amdgpu_buffer_rsrc_t own_kb = bounded_bytes(own_k + (size_t)s.row0 * a.stride, (int)(((long)(a.rows - s.row0) * a.stride - (own_k - x)) * 2));
-  const __amdgpu_buffer_rsrc_t own_vb = bounded_bytes(own_v + (size_t)s.row0 * a.stride, (int)(((long)(a.rows - s.row0) * a.stride - (own_v - x)) * 2));
+  const __amdgpu_buffer_rsrc_t own_kb = bounded_bytes(own_k + (size_t)s.row0 * a.stride, (int)(((long)s.rows * a.stride - (own_k - x)) * 2));
+  const __amdgpu_buffer_rsrc_t own_vb = bounded_bytes(own_v + (size_t)s.row0 * a.stride, (int)(((long)s.rows * a.stride - (own_v - x)) * 2));
   const __amdgpu_buffer_rsrc_t old_kb = bounded_bytes(ring_k, (a.ring * nk - g * a.dim) * 2);
   const __amdgpu_buffer_rsrc_t old_vb = bounded_bytes(ring_v, (a.ring * nv - g * a.vdim) * 2);
   int k_col[KP], v_col[VT], k_own[KP], v_own[VT], k_mod[KP], v_mod[VT][4];

@@ -245,7 +245,7 @@ def short_conv(op, x, weight, a_log, dt_bias, state, spans):
         decay = -np.exp(np.asarray(a_log, np.float64)) * np.logaddexp(0, rows[:, op.a_at : op.a_at + H] + dt_bias)
         beta = 1 / (1 + np.exp(-rows[:, op.b_at : op.b_at + H]))
         y[row : row + n] = np.concatenate([qk.reshape(n, -1), conv[:, 2 * G * D :], decay, beta], axis=1)
-        for p in range(max(start, start + n - op.taps), start + n):
+        for p in range(max(start, start + n - op.taps + 1), start + n):
             state[s, p % op.taps] = x[row + p - start][:C]
     return state, y
 

@@ -378,7 +378,7 @@ def test_a_draw_a_slot_is_each_slot_s_draw(cuda):
 # ---------------------------------------------------------------- whole models
 
 
-LIMIT = {"f32": 3e-5, "bf16": 4e-2}
+LIMIT = {"f32": 1e-5, "bf16": 6e-2}   # of the logits' spread: rounding alone reaches 3e-6 and 5e-2
 
 
 @pytest.fixture(scope="module", params=[(n, d, f) for n in MODELS for d in ("f32", "bf16") for f in ((True, False) if d == "bf16" else (True,))],
