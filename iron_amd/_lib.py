@@ -134,6 +134,8 @@ def lib() -> ctypes.CDLL:
                 f"{LIB_PATH} is missing: build it with `python -m iron_amd.build` "
                 "(there is no CPU fallback)"
             )
+        import torch  # noqa: F401 -- its HIP runtime must be the process's first, or the library would bind another
+
         handle = ctypes.CDLL(str(LIB_PATH))
         for name, (restype, argtypes) in SIGNATURES.items():
             fn = getattr(handle, name)  # AttributeError names a missing symbol

@@ -38,9 +38,9 @@ def linear(x, weight, bias=None, *, precision: Precision = Precision.HIGHEST, **
     if rank not in (1, 2):
         raise ValueError(f"linear(): x {tuple(x.shape)} is not (in,) or (rows, in)")
     rows = 1 if rank == 1 else x.shape[0]
-    if bias is None and rank == 2 and (x.dtype is not bfloat16 or x.shape[1] % 8):
+    if bias is None and (x.dtype is not bfloat16 or x.shape[-1] % 8):
         # a model that runs in 32 bits throughout, or a row that is no whole number of 16-byte pieces
-        return LinearAny.step(x, weight, dtype=x.dtype)
+        return LinearAny.step(x.reshape(rows, x.shape[-1]), weight, dtype=x.dtype)
     if rows > 1 and gemv:
         raise ValueError(f"linear(): {rows} rows take no GEMV {sorted(gemv)}")
     if rows == 1:
