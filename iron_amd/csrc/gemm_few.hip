@@ -11,19 +11,25 @@ namespace iron {
 
 constexpr int FEW_WAVES = 8, FEW_STEP = 64;   // K columns a wave takes at a time
 
-template <int MT, bool GATED>
+// MODE: one tile of 16 rows of B a block, two of them (a tall B), or one of each of two matrices.
+enum { FEW_ONE = 0, FEW_TWO = 1, FEW_GATED = 2 };
+template <int MT, int MODE>
 __global__ __launch_bounds__(FEW_WAVES * 64) void gemm_few_kernel(const bf16_t* __restrict__ A, const bf16_t* __restrict__ B,
                                                                   const bf16_t* __restrict__ B2, bf16_t* __restrict__ C, int M,
                                                                   int N, int K, int activation) {
-  constexpr int MATS = GATED ? 2 : 1, DEPTH = MT <= 2 ? 2 : 1;
+  constexpr int MATS = MODE == FEW_ONE ? 1 : 2, DEPTH = MT == 1 ? 4 : (MT == 2 ? 2 : 1);
+  constexpr bool GATED = MODE == FEW_GATED;
   __shared__ float4 part[FEW_WAVES][MATS][MT][64];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, l16 = lane & 15, quad = lane >> 4;
-  const int n0 = blockIdx.x * 16, steps = (K + FEW_WAVES * FEW_STEP - 1) / (FEW_WAVES * FEW_STEP);
+  const int n0 = blockIdx.x * (MODE == FEW_TWO ? 32 : 16), steps = (K + FEW_WAVES * FEW_STEP - 1) / (FEW_WAVES * FEW_STEP);
   // Bounded buffers: a piece past K reads as zeros (of a row's own end, whatever follows it meets zeros of A).
   const __amdgpu_buffer_rsrc_t ab = bounded_bytes(A, M * K * 2);
   const size_t row = (size_t)min(n0 + l16, N - 1) * K;
   const bf16_t* w[MATS] = {B + row};
-  if (GATED) w[MATS - 1] = B2 + row;
+  if (MODE != FEW_ONE) w[MATS - 1] = GATED ? B2 + row : B + (size_t)min(n0 + 16 + l16, N - 1) * K;
+  int a_row[MT];
+#pragma unroll
+  for (int m = 0; m < MT; ++m) a_row[m] = min(m * 16 + l16, M - 1) * K * 2;
   f32x4 acc[MATS][MT];
 #pragma unroll
   for (int x = 0; x < MATS; ++x)
@@ -33,16 +39,18 @@ __global__ __launch_bounds__(FEW_WAVES * 64) void gemm_few_kernel(const bf16_t* 
     u32x4 b[MATS][2], a[MT][2];
   } held[DEPTH];
   auto fetch = [&](Piece& p, int step) {
-    const int k = (step * FEW_WAVES + wave) * FEW_STEP + quad * 8;
+    // (a lane takes 32 consecutive bytes of its row: which of the 64 columns meet in which product is free)
+    const int k = (step * FEW_WAVES + wave) * FEW_STEP + quad * 16;
 #pragma unroll
     for (int h = 0; h < 2; ++h) {
-      const int kh = k + h * 32, in = min(kh, K - 8);   // past K: B's last piece, against zeros of A
+      const int kh = k + h * 8, in = min(kh, K - 8);   // past K: B's last piece, against zeros of A
 #pragma unroll
-      for (int x = 0; x < MATS; ++x) p.b[x][h] = __builtin_nontemporal_load(reinterpret_cast<const u32x4*>(w[x] + in));
+      for (int x = 0; x < MATS; ++x) p.b[x][h] = *reinterpret_cast<const u32x4*>(w[x] + in);
 #pragma unroll
       for (int m = 0; m < MT; ++m) {
-        const int r = m * 16 + l16;
-        p.a[m][h] = __builtin_amdgcn_raw_buffer_load_b128(ab, (r < M && kh < K) ? (r * K + kh) * 2 : 0x7ffffff0, 0, 0);
+        // A row past the last reads the last again (its results are not stored).
+        const int past = (K - 1 - kh) >> 31 & 0x40000000;   // past K: outside the buffer
+        p.a[m][h] = __builtin_amdgcn_raw_buffer_load_b128(ab, a_row[m] + 2 * kh + past, 0, 0);
       }
     }
   };
@@ -51,21 +59,25 @@ __global__ __launch_bounds__(FEW_WAVES * 64) void gemm_few_kernel(const bf16_t* 
     fetch(held[d], d);
     __builtin_amdgcn_sched_barrier(0);
   }
-  for (int s = 0; s < steps; s += DEPTH) {
+  auto add = [&](const Piece& p) {
 #pragma unroll
-    for (int d = 0; d < DEPTH; ++d) {   // (a step past the last adds zeros)
-      const Piece p = held[d];
+    for (int h = 0; h < 2; ++h)
+#pragma unroll
+      for (int x = 0; x < MATS; ++x)
+#pragma unroll
+        for (int m = 0; m < MT; ++m)
+          acc[x][m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, p.b[x][h]), __builtin_bit_cast(bf16x8, p.a[m][h]), acc[x][m], 0, 0, 0);
+  };
+  for (int s = 0; s + DEPTH < steps; s += DEPTH) {   // (a step past the last adds zeros)
+#pragma unroll
+    for (int d = 0; d < DEPTH; ++d) {
+      add(held[d]);
       fetch(held[d], s + d + DEPTH);
       __builtin_amdgcn_sched_barrier(0);
-#pragma unroll
-      for (int h = 0; h < 2; ++h)
-#pragma unroll
-        for (int x = 0; x < MATS; ++x)
-#pragma unroll
-          for (int m = 0; m < MT; ++m)
-            acc[x][m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, p.b[x][h]), __builtin_bit_cast(bf16x8, p.a[m][h]), acc[x][m], 0, 0, 0);
     }
   }
+#pragma unroll
+  for (int d = 0; d < DEPTH; ++d) add(held[d]);
 #pragma unroll
   for (int x = 0; x < MATS; ++x)
 #pragma unroll
@@ -92,16 +104,19 @@ __global__ __launch_bounds__(FEW_WAVES * 64) void gemm_few_kernel(const bf16_t* 
     }
     bf16_t* to = C + (size_t)r * N + n;
 #pragma unroll
-    for (int j = 0; j < 4; ++j)
-      if (n + j < N) to[j] = f32_to_bf16(v[0][j]);
+    for (int x = 0; x < (MODE == FEW_TWO ? 2 : 1); ++x)
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        if (n + 16 * x + j < N) to[16 * x + j] = f32_to_bf16(v[x][j]);
   }
 }
 
-template <bool GATED>
+template <int MODE>
 static int launch_gemm_few(const bf16_t* A, const bf16_t* B, const bf16_t* B2, bf16_t* C, int M, int N, int K, int activation, hipStream_t s) {
-  const dim3 grid((N + 15) / 16);
+  const int per = MODE == FEW_TWO ? 32 : 16;
+  const dim3 grid((N + per - 1) / per);
 #define IRON_FEW(MT) \
-  hipLaunchKernelGGL((gemm_few_kernel<MT, GATED>), grid, dim3(FEW_WAVES * 64), 0, s, A, B, B2, C, M, N, K, activation)
+  hipLaunchKernelGGL((gemm_few_kernel<MT, MODE>), grid, dim3(FEW_WAVES * 64), 0, s, A, B, B2, C, M, N, K, activation)
   if (M <= 16) IRON_FEW(1);
   else if (M <= 32) IRON_FEW(2);
   else IRON_FEW(4);
@@ -121,6 +136,8 @@ extern "C" int iron_gemm_few_bf16(const uint16_t* A, const uint16_t* B, const ui
   IRON_REQUIRE((((uintptr_t)A | (uintptr_t)B | (uintptr_t)B2) & 15) == 0, "gemm_few: operands must be 16-byte aligned");
   IRON_REQUIRE(B2 == nullptr || (activation >= 1 && activation <= 3), "gemm_few: activation (%d) is 1 (SiLU), 2 (GELU, tanh form) or 3 (ReLU)",
                activation);
-  return B2 != nullptr ? launch_gemm_few<true>(A, B, B2, C, M, N, K, activation, (hipStream_t)stream)
-                       : launch_gemm_few<false>(A, B, nullptr, C, M, N, K, 0, (hipStream_t)stream);
+  hipStream_t s = (hipStream_t)stream;
+  if (B2 != nullptr) return launch_gemm_few<FEW_GATED>(A, B, B2, C, M, N, K, activation, s);
+  if (N >= 8192) return launch_gemm_few<FEW_TWO>(A, B, nullptr, C, M, N, K, 0, s);
+  return launch_gemm_few<FEW_ONE>(A, B, nullptr, C, M, N, K, 0, s);
 }
