@@ -1,5 +1,6 @@
 """A decoder-only language model wired from the hot-path operators (iron/lm/__init__.py)."""
 
+from .batched import Batch, BatchedLM, Entry, SlotSession
 from .blocks import (
     Attention,
     DecoderLayer,
@@ -18,10 +19,12 @@ from .causal import Call, CausalLM, Decoder, Stats
 from .checkpoint import Checkpoint, weights_file, write_safetensors
 from .config import DecoderConfig, rope_angles
 from .generation import Sampler
+from .mixers import DeltaMixer, ParallelMixer, StreamLayer, StreamRMSNorm, TimeMixing, WindowAttention
 from .session import Session
 
 __all__ = [
-    "Attention", "Call", "CausalLM", "Checkpoint", "Decoder", "DecoderConfig", "DecoderLayer", "Embedding", "GatedMLP",
-    "KVCache", "Linear", "PleLayer", "RMSNorm", "Rope", "Sampler", "SandwichLayer", "Session", "Stats", "activation",
-    "residual_add", "rope_angles", "weights_file", "write_safetensors",
+    "Attention", "Batch", "BatchedLM", "Call", "CausalLM", "Checkpoint", "Decoder", "DecoderConfig", "DecoderLayer",
+    "DeltaMixer", "Embedding", "Entry", "GatedMLP", "KVCache", "Linear", "ParallelMixer", "PleLayer", "RMSNorm",
+    "Rope", "Sampler", "SandwichLayer", "Session", "SlotSession", "Stats", "StreamLayer", "StreamRMSNorm",
+    "TimeMixing", "WindowAttention", "activation", "residual_add", "rope_angles", "weights_file", "write_safetensors",
 ]

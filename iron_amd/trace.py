@@ -3,7 +3,7 @@
 ``bin/trace_run --model DIR --dtype bfloat16|float32 --out DIR [--max-tokens N]`` reads steps from
 standard input, one JSON object a line::
 
-    {"step": 0, "entries": [{"id": "a", "tokens": [5, 17, 3], "want": [0, 2]}], "end": []}
+    {"step": 7, "entries": [{"id": "r1", "tokens": [210, 9, 31, 4], "want": [3]}], "end": ["r0"]}
 
 ``entries`` are the requests' next tokens, run as one batch after what each request holds; ``want`` the
 places among them whose logits are wanted; ``end`` the requests that are over after this step.  A step

@@ -95,7 +95,7 @@ def test_the_registry_picks_the_class_by_config_json(tmp_path):
     assert model_class(tmp_path).__name__ == "Llama"
 
 
-@pytest.mark.parametrize("rows,bias_max", [(12, 50), (6, 33), (32, 96), (16, 240), (16, 128), (7, 40), (2, 9), (3, 20)])
+@pytest.mark.parametrize("rows,bias_max", [(12, 50), (6, 33), (32, 96), (20, 300), (16, 128), (7, 40), (2, 9), (3, 20)])
 def test_distance_buckets(rows, bias_max):
     got = distance_buckets(400, rows, bias_max)
     want = [distance_bucket(n, rows, bias_max) for n in range(400)]

@@ -523,3 +523,23 @@ def test_a_trace_is_replayed(cuda, tmp_path):
         rows = np.fromfile(tmp_path / f"{step}.f32", "<f4").reshape(len(places), doc["vocab"])
         assert far_off(rows, want[places], want.std()) < LIMIT["f32"]
     assert not (tmp_path / "1.f32").exists()
+
+
+def test_the_command_line_generates_a_batch(cuda, tmp_path, capsys):
+    from iron_amd.__main__ import main
+    from iron_amd.applications.pegilix import PegilixConfig
+
+    doc, bias_rows, rank = MODELS["mixed"]
+    config = PegilixConfig.from_json(doc)
+    weights = weights_of(config, bias_rows, rank)
+    (tmp_path / "config.json").write_text(json.dumps(doc))
+    write_safetensors(tmp_path / "model.safetensors", weights)
+    prompts = [np.random.default_rng(n).integers(0, doc["vocab"], n).tolist() for n in (11, 4)]
+    asked = [a for p in prompts for a in ("--ids", ",".join(map(str, p)))]
+    assert main([str(tmp_path), *asked, "--count", "9", "--max-seq-len", "64"]) == 0
+    printed = [[int(t) for t in line.split(",")] for line in capsys.readouterr().out.splitlines()]
+    model = Pegilix.load(tmp_path, slots=2, max_seq_len=64)
+    try:
+        assert printed == model.generate_batch(prompts, 9)
+    finally:
+        model.release()
