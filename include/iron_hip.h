@@ -391,11 +391,20 @@ int iron_stream_embed(const uint16_t* table, const int* ids, float* x, int rows,
  * rows as they then stand.  Float throughout, h rounded once. */
 int iron_stream_rows(float* x, const void* y, const uint16_t* back_gain, const uint16_t* gain, void* h, int rows,
                      int cols, float eps, int is_float, const int* valid, void* stream);
+/* x += (y + y_bias) * sigmoid(gate + gate_bias) in place, gate columns gate_at .. of rows of gate_stride (y_bias
+ * may be NULL); with h, h = rmsnorm(x) * gain of the rows as they then stand.  Float throughout, h rounded once. */
+int iron_stream_gated_rows(float* x, const void* y, const uint16_t* y_bias, const void* gate, const uint16_t* gate_bias,
+                           int gate_stride, int gate_at, const uint16_t* gain, void* h, int rows, int cols, float eps,
+                           int is_float, const int* valid, void* stream);
+/* y = a N(z) + b N(z^2) + c N(z^3) + e, z columns at .. of x (rows, stride) plus bias (may be NULL), powers element
+ * by element, N over a row's root mean square; coefficients {a, b, c, e}.  y (rows, cols); float, rounded once. */
+int iron_poly_norm(const void* x, const uint16_t* bias, const uint16_t* coefficients, void* y, int rows, int cols,
+                   int stride, int at, float eps, int is_float, const int* valid, void* stream);
 /* out[slot] = the last row of the slot's span (left as it is for an idle slot). */
 int iron_span_tails(const float* x, const int* spans, float* out, int slots, int rows, int cols, void* stream);
-/* y = cap * tanh(x / cap) (cap 0: y = x) as float, and rounded to bf16 in rows of rounded_stride. */
+/* y = cap * tanh(scale x / cap) (cap 0: y = scale x) as float, and rounded to bf16 in rows of rounded_stride. */
 int iron_softcap(const void* x, float* y, uint16_t* rounded, int rows, int cols, int rounded_stride, float cap,
-                 int is_float, void* stream);
+                 float scale, int is_float, void* stream);
 /* y = act(gate) * up in float; activation 1 SiLU, 2 GELU (tanh form), 3 ReLU. */
 int iron_act_mul_f32(const float* gate, const float* up, float* y, int rows, int cols, int activation,
                      const int* valid, void* stream);
@@ -448,6 +457,32 @@ int iron_head_gate(const float* o, const void* gate, const uint16_t* gain, void*
 int iron_mha_window(const void* x, void* keys, void* values, const float* bias, const int* spans, void* out, int slots,
                     int rows, int stride, int heads, int kv_heads, int dim, int vdim, int window, int ring, float scale,
                     int out_stride, int out_at, float out_scale, int single, int is_float, void* stream);
+/* x (rows, stride) = [zx | ux | gx | ..] of `width` columns each.  Per channel z = sigmoid(zx + z_bias), u = ux + x_bias,
+ * c = u + 1/2 where u >= 0, else sigmoid(u); S <- (1 - z) S + z c; y = S silu(gx), y (rows, width).  state (slots, width).
+ * With a workspace (the bytes given, any contents, 16-byte aligned) chunks of a portion run side by side; without, a
+ * span's rows one after the other. */
+int64_t iron_min_gru_workspace_bytes(int slots, int rows, int width);
+int iron_min_gru(const void* x, const uint16_t* z_bias, const uint16_t* x_bias, float* state, const int* spans, void* y,
+                 void* workspace, int slots, int rows, int stride, int width, int is_float, void* stream);
+/* Latent attention.  latent_rows: x (rows, stride) = [query latent (q_rank) | latent (rank) | shared key part (rot) | ..];
+ * both latents RMS-normed (gains q_gain, c_gain), the first `turned` of the rot columns turned in neighbouring pairs
+ * by row p of angles (angle_rows, turned; cos and sin side by side); q_out (rows, q_rank), and position p's latent
+ * and key part in row p % ring of latents (slots, ring, rank) and shared_keys (slots, ring, rot; NULL if rot is 0).
+ * mha_latent: q (rows, heads * (dim + rot)), a head's rot columns turned here; up (heads * (dim + vdim), rank): U, V.
+ * score = (q . U c + turned q . shared key) * scale over 0 <= i - j < window, softmax (exp(sink[head]) in its denominator
+ * unless sink is NULL); y (rows, heads * vdim) the sum of V c.  The rows' own latents are in the caches already.
+ * single: no span has more than one row.  Else `cap` key rows are expanded at most: the spans' rows and, of the
+ * positions before them, the last window - 1 each; a span whose keys do not fit is left out.
+ * workspace: the bytes given, any contents. */
+int iron_latent_rows(const void* x, const uint16_t* q_gain, const uint16_t* c_gain, const float* angles, const int* spans,
+                     void* q_out, void* latents, void* shared_keys, int slots, int rows, int stride, int q_rank, int rank,
+                     int rot, int turned, int angle_rows, int ring, float eps, int is_float, void* stream);
+int64_t iron_mha_latent_workspace_bytes(int slots, int rows, int heads, int dim, int rot, int vdim, int rank, int window, int ring,
+                                        int cap, int single, int is_float);
+int iron_mha_latent(const void* q, const void* latents, const void* shared_keys, const uint16_t* up, const uint16_t* sink,
+                    const float* angles, const int* spans, void* y, void* workspace, int slots, int rows, int heads, int dim,
+                    int rot, int vdim, int rank, int turned, int angle_rows, int window, int ring, int cap, float scale, int single,
+                    int is_float, void* stream);
 /* One token a slot (no span of more than one row) through a mixer, bf16, in one launch; each computes what
  * the entry points above compute in turn, on the same states.
  * decode_mixed (one slot): iron_token_shift and `count` (up to 8) products y[i] = W[i] (rows[i], K) times

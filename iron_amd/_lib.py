@@ -92,7 +92,14 @@ SIGNATURES = {
     "iron_stream_embed": (c_int, [_P, _P, _P, c_int, c_int, c_int, _P, _P]),
     "iron_stream_rows": (c_int, [_P, _P, _P, _P, _P, c_int, c_int, c_float, c_int, _P, _P]),
     "iron_span_tails": (c_int, [_P, _P, _P, c_int, c_int, c_int, _P]),
-    "iron_softcap": (c_int, [_P, _P, _P, c_int, c_int, c_int, c_float, c_int, _P]),
+    "iron_softcap": (c_int, [_P, _P, _P, c_int, c_int, c_int, c_float, c_float, c_int, _P]),
+    "iron_stream_gated_rows": (c_int, [_P] * 5 + [c_int, c_int, _P, _P, c_int, c_int, c_float, c_int, _P, _P]),
+    "iron_poly_norm": (c_int, [_P] * 4 + [c_int] * 4 + [c_float, c_int, _P, _P]),
+    "iron_min_gru_workspace_bytes": (c_int64, [c_int] * 3),
+    "iron_min_gru": (c_int, [_P] * 7 + [c_int] * 5 + [_P]),
+    "iron_latent_rows": (c_int, [_P] * 8 + [c_int] * 9 + [c_float, c_int, _P]),
+    "iron_mha_latent_workspace_bytes": (c_int64, [c_int] * 12),
+    "iron_mha_latent": (c_int, [_P] * 9 + [c_int] * 12 + [c_float, c_int, c_int, _P]),
     "iron_act_mul_f32": (c_int, [_P, _P, _P, c_int, c_int, c_int, _P, _P]),
     "iron_linear_any": (c_int, [_P, _P, _P, c_int, c_int, c_int, c_int, _P, _P]),
     "iron_token_shift": (c_int, [_P] * 5 + [c_int] * 5 + [_P]),

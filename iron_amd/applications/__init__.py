@@ -1,10 +1,11 @@
-"""The models wired from the shared decoder: Llama, Granite, Gemma 4's text decoder and Pegilix."""
+"""The models wired from the shared decoder: Llama, Granite, Gemma 4's text decoder, Pegilix and Pufuzen."""
 
 from .gemma4 import Gemma4, Gemma4Config
 from .granite import Granite, GraniteConfig
 from .llama import Llama, LlamaConfig
 from .pegilix import Pegilix, PegilixConfig
+from .pufuzen import Pufuzen, PufuzenConfig
 from .registry import ARCHITECTURES, load_model, model_class
 
 __all__ = ["ARCHITECTURES", "Gemma4", "Gemma4Config", "Granite", "GraniteConfig", "Llama", "LlamaConfig", "Pegilix",
-           "PegilixConfig", "load_model", "model_class"]
+           "PegilixConfig", "Pufuzen", "PufuzenConfig", "load_model", "model_class"]

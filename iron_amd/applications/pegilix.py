@@ -19,14 +19,15 @@ from ..bf16 import bfloat16, from_torch
 from ..common.declare import Precision
 from ..lm.batched import BatchedLM
 from ..lm.blocks import GatedMLP
-from ..lm.config import ConfigFile
+from ..lm.checkpoint import Renaming, joined
+from ..lm.config import LayerListConfig
 from ..lm.mixers import DeltaMixer, ParallelMixer, StreamLayer, TimeMixing, WindowAttention
 
 _MIXERS = ("parallel", "delta")
 
 
 @dataclasses.dataclass(frozen=True)
-class PegilixConfig(ConfigFile):
+class PegilixConfig(LayerListConfig):
     """A Pegilix ``config.json``, and this package's own choices behind it.  ``layers`` keeps the file's
     entries.  The design bounds no positions; ``max_seq_len`` is how many a slot is served."""
 
@@ -42,60 +43,15 @@ class PegilixConfig(ConfigFile):
     activations: Any = bfloat16
     precision: Precision = Precision.HIGHEST
 
-    tie_word_embeddings = False
-    rope_theta = None
-
-    # field -> where config.json keeps it
+    ARCHITECTURE = "Pegilix"
     KEYS = {"vocab_size": ("vocab",), "hidden_size": ("width",), "layers": ("layers",), "eps": ("norm", "eps"),
             "loop": ("loop",), "logit_softcap": ("logit_softcap",)}
 
     def __post_init__(self):
-        fix = object.__setattr__
-        if self.prefill_chunk > self.max_seq_len * self.slots:
-            fix(self, "prefill_chunk", self.max_seq_len * self.slots)
-        for i, spec in enumerate(self.layers):
-            if spec["type"] not in _MIXERS:
-                raise ValueError(f"PegilixConfig: layer {i} is {spec['type']!r}, not one of {_MIXERS}")
-            mlp = spec.get("mlp")
-            if mlp is not None and mlp.get("kind") != "dense":
-                raise ValueError(f"PegilixConfig: layer {i}'s feed-forward is {mlp.get('kind')!r}, not 'dense'")
+        self.check_serving()
+        self.check_layers(_MIXERS)
         if self.loop is not None and not 0 <= self.loop["start"] <= self.loop["stop"] <= len(self.layers):
             raise ValueError(f"PegilixConfig: loop {self.loop} of {len(self.layers)} layers")
-        if self.slots < 1:
-            raise ValueError(f"PegilixConfig: slots ({self.slots}) must be at least 1")
-
-    @classmethod
-    def from_json(cls, data: dict, source="config.json") -> "PegilixConfig":
-        """Raises ValueError where a size or constant without a default is absent."""
-        given, absent = {}, []
-        for field in dataclasses.fields(cls):
-            if field.name not in cls.KEYS:
-                continue
-            value = data
-            for key in cls.KEYS[field.name]:
-                value = value.get(key) if isinstance(value, dict) else None
-            if value is not None:
-                given[field.name] = tuple(value) if field.name == "layers" else value
-            elif field.default is dataclasses.MISSING:
-                absent.append(".".join(cls.KEYS[field.name]))
-        if absent:
-            raise ValueError(f"{source} lacks {absent}")
-        return cls(**given)
-
-    def to_json(self) -> dict:
-        out: dict = {"architecture": "Pegilix"}
-        for name, keys in self.KEYS.items():
-            value, scope = getattr(self, name), out
-            if value is None:
-                continue
-            for key in keys[:-1]:
-                scope = scope.setdefault(key, {})
-            scope[keys[-1]] = list(value) if isinstance(value, tuple) else value
-        return out
-
-    @property
-    def num_hidden_layers(self) -> int:
-        return len(self.layers)
 
     @property
     def order(self) -> list[int]:
@@ -136,15 +92,6 @@ class PegilixLayer(StreamLayer):
         super().__init__(c.hidden_size, mixer, mlp, eps=c.eps, dtype=c.activations)
 
 
-def _joined(tensors, axis: int):
-    """The tensors side by side along ``axis``, torch or numpy as they come."""
-    if type(tensors[0]).__module__.split(".")[0] == "torch":
-        import torch
-
-        return torch.cat(tensors, dim=axis)
-    return np.concatenate(tensors, axis=axis)
-
-
 def _as_float32(weight) -> np.ndarray:
     is_torch = type(weight).__module__.split(".")[0] == "torch"
     return from_torch(weight) if is_torch else np.asarray(weight, dtype=np.float32)
@@ -152,18 +99,8 @@ def _as_float32(weight) -> np.ndarray:
 
 def module_weights(config: PegilixConfig, weights) -> dict:
     """A checkpoint's tensors under the modules' names, those that are read together joined."""
-    left_over = dict(weights)
-    out = {}
-
-    def take(name):
-        if name not in left_over:
-            raise ValueError(f"Pegilix: the checkpoint lacks {name}")
-        return left_over.pop(name)
-
-    def put(target, *names, axis=0):
-        found = [take(n) for n in names]
-        out[target] = found[0] if len(found) == 1 else _joined(found, axis)
-
+    names = Renaming(weights, "Pegilix")
+    put, take = names.put, names.take
     put("model.embed_tokens.weight", "embed")
     put("model.norm.weight", "final.norm")
     put("lm_head.weight", "head")
@@ -174,7 +111,7 @@ def module_weights(config: PegilixConfig, weights) -> dict:
             put(f"{dst}{norm}.weight", src + norm)
         if spec.get("mlp") is None:
             for norm in ("norm2", "norm2b"):
-                left_over.pop(src + norm, None)    # a layer without a feed-forward reads none
+                names.drop(src + norm)    # a layer without a feed-forward reads none
         else:
             for part in ("gate", "up", "down"):
                 put(f"{dst}mlp.{part}_proj.weight", f"{src}mlp.{part}")
@@ -184,7 +121,7 @@ def module_weights(config: PegilixConfig, weights) -> dict:
             put(dst + "left.rel", src + "left.rel")
             put(dst + "out.weight", src + "left.o", src + "right.o", axis=1)
             mus = [take(f"{src}right.mu.{n}") for n in TimeMixing.BLENDS]
-            out[dst + "right.mu"] = _joined([mu.reshape(1, -1) for mu in mus], 0)
+            names.named[dst + "right.mu"] = joined([mu.reshape(1, -1) for mu in mus], 0)
             for n in ("r", "k", "v", "g", "w1"):
                 put(f"{dst}right.{n}.weight", f"{src}right.{n}")
             for n in ("w2", "w0", "u", "norm"):
@@ -196,9 +133,7 @@ def module_weights(config: PegilixConfig, weights) -> dict:
             put(dst + "dt_bias", src + "dt_bias")
             put(dst + "norm", src + "norm")
             put(dst + "out.weight", src + "o")
-    if left_over:
-        raise ValueError(f"Pegilix: the checkpoint holds {sorted(left_over)}, which no layer reads")
-    return out
+    return names.done()
 
 
 class Pegilix(BatchedLM):

@@ -9,6 +9,7 @@ from .gemma4 import Gemma4
 from .granite import Granite
 from .llama import Llama
 from .pegilix import Pegilix
+from .pufuzen import Pufuzen
 
 # ``architecture`` (or an entry of ``architectures``) -> the class that serves it
 ARCHITECTURES = {
@@ -17,6 +18,7 @@ ARCHITECTURES = {
     "Gemma4ForCausalLM": Gemma4,
     "Gemma4ForConditionalGeneration": Gemma4,
     "Pegilix": Pegilix,
+    "Pufuzen": Pufuzen,
 }
 
 

@@ -44,18 +44,6 @@ __device__ __forceinline__ void block_barrier_lds() {
   __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "workgroup", "local");
 }
 
-// A span's first chunk in the workspace: spans in the order of their rows, each from a chunk of its own.
-__device__ __forceinline__ int first_chunk(const int* __restrict__ spans, int slots, int slot, int rows) {
-  const Span mine = span_of(spans, slot, rows);
-  int rank = 0;
-  for (int i = 0; i < slots; ++i) {
-    const Span s = span_of(spans, i, rows);
-    rank += s.rows > 0 && s.row0 < mine.row0;
-  }
-  return mine.row0 / CHUNK + rank;
-}
-__host__ __device__ inline long chunks_of(int rows, int slots) { return (rows + CHUNK - 1) / CHUNK + slots; }
-
 // ---------------------------------------------------------------- time mixing
 // Workspace of a chunk and head: r exp(L before it) frags, k exp(L_end - L) frags transposed (both 16 a
 // row tile), exp(L_end), and the 16 x 16 matrix's frag.
@@ -98,7 +86,7 @@ __global__ __launch_bounds__(256) void time_mix_chunks_kernel(const T* __restric
     }
   }
   __syncthreads();
-  float* out = work + ((size_t)(first_chunk(spans, slots, slot, rows) + blockIdx.x) * heads + head) * mix_words(tiles);
+  float* out = work + ((size_t)(first_chunk(spans, slots, slot, rows, CHUNK) + blockIdx.x) * heads + head) * mix_words(tiles);
   for (int e = t; e < tiles * 64; e += 256) {
     const int tile = e >> 6, lane = e & 63, l16 = lane & 15, quad = lane >> 4;
     float4 a, b;
@@ -171,7 +159,7 @@ __global__ __launch_bounds__(256) void time_mix_walk_kernel(const T* __restrict_
   const int count = (s.rows + CHUNK - 1) / CHUNK;
   const size_t width = (size_t)heads * dim;
   float* sp = state + ((size_t)slot * heads + head) * dim * dim;
-  const float* at = work + ((size_t)first_chunk(spans, slots, slot, rows) * heads + head) * words;
+  const float* at = work + ((size_t)first_chunk(spans, slots, slot, rows, CHUNK) * heads + head) * words;
   // The span's rows by 32-bit offsets; a store to an offset outside them is dropped.
   constexpr int E = (int)sizeof(T);
   const __amdgpu_buffer_rsrc_t vb = bounded_bytes(v + (size_t)s.row0 * width + head * dim, (int)(((size_t)s.rows * width - head * dim) * E));
@@ -320,7 +308,7 @@ __global__ __launch_bounds__(256) void delta_chunks_kernel(const float* __restri
     }
   }
   __syncthreads();
-  float* out = work + ((size_t)(first_chunk(spans, slots, slot, rows) + blockIdx.x) * heads + head) * DELTA_WORDS;
+  float* out = work + ((size_t)(first_chunk(spans, slots, slot, rows, CHUNK) + blockIdx.x) * heads + head) * DELTA_WORDS;
   const int fl = t >> 2, fr = t & 3;
   out[t] = inv[fl & 15][(fl >> 4) * 4 + fr];
   out[256 + t] = p[fl & 15][(fl >> 4) * 4 + fr];
@@ -351,7 +339,7 @@ __global__ __launch_bounds__(256) void delta_walk_kernel(const float* __restrict
   const int group = head / (heads / kv_heads), qkw = kv_heads * dim, channels = 2 * qkw + heads * vdim, wide = channels + 2 * heads;
   const int col = blockIdx.y * 16 + l16, count = (s.rows + CHUNK - 1) / CHUNK;
   float* sp = state + ((size_t)slot * heads + head) * dim * vdim;
-  const float* at = work + ((size_t)first_chunk(spans, slots, slot, rows) * heads + head) * DELTA_WORDS;
+  const float* at = work + ((size_t)first_chunk(spans, slots, slot, rows, CHUNK) * heads + head) * DELTA_WORDS;
   const __amdgpu_buffer_rsrc_t xb = bounded_bytes(x + (size_t)s.row0 * wide, (int)((size_t)s.rows * wide * 4));
   const __amdgpu_buffer_rsrc_t ob = bounded_bytes(o + (size_t)s.row0 * heads * vdim, (int)((size_t)s.rows * heads * vdim * 4));
   const int o_at = col < vdim ? ((quad * 4 + wave) * heads * vdim + head * vdim + col) * 4 : 0x7fffffff;
@@ -473,10 +461,10 @@ __global__ __launch_bounds__(256) void delta_walk_kernel(const float* __restrict
 using namespace iron;
 
 extern "C" int64_t iron_time_mix_workspace_bytes(int slots, int rows, int heads, int dim) {
-  return chunks_of(rows, slots) * heads * (int64_t)mix_words((dim + 15) / 16) * 4;
+  return chunks_of(rows, slots, CHUNK) * heads * (int64_t)mix_words((dim + 15) / 16) * 4;
 }
 extern "C" int64_t iron_delta_rule_workspace_bytes(int slots, int rows, int heads) {
-  return chunks_of(rows, slots) * heads * (int64_t)DELTA_WORDS * 4;
+  return chunks_of(rows, slots, CHUNK) * heads * (int64_t)DELTA_WORDS * 4;
 }
 
 #define IRON_CHUNKED_REQUIRE(name)                                                                        \

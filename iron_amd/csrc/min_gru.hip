@@ -1,0 +1,202 @@
+// A gated recurrence whose gates read the current token alone, element by element over `width` channels:
+//
+//   S_t = (1 - z) S_(t-1) + z c,   z = sigmoid(zx + zb),   c = u + 1/2 where u = ux + ub >= 0, else sigmoid(u)
+//   y_t = S_t silu(gx)
+//
+// zx, ux and gx are columns 0, width and 2 width of a packed projection's row.  Everything in float32.
+//
+// The step from one state to the next is affine, S -> a S + b, and so is any run of steps: over a prompt's
+// portion a first launch folds every chunk of GRU_CHUNK tokens to its (a, b), and a second walks each chunk
+// from the state that the chunks before it leave.  A portion's first state is put ahead of its chunks, since
+// the block of its last chunk replaces it.
+#include "../../include/iron_hip.h"
+#include "rows.h"
+
+namespace iron {
+
+constexpr int GRU_CHUNK = 32, GRU_AHEAD = 8;   // tokens a chunk, and tokens asked for at a time
+
+// Two neighbouring elements, or one.
+template <int VEC, typename T>
+__device__ __forceinline__ void load_few(const T* __restrict__ p, float (&f)[VEC]) {
+  if constexpr (VEC == 1) {
+    f[0] = load_one(p);
+  } else if constexpr (sizeof(T) == 2) {
+    const uint32_t w = *reinterpret_cast<const uint32_t*>(p);
+    f[0] = bf16_lo(w);
+    f[1] = bf16_hi(w);
+  } else {
+    const float2 w = *reinterpret_cast<const float2*>(p);
+    f[0] = w.x;
+    f[1] = w.y;
+  }
+}
+template <int VEC, typename T>
+__device__ __forceinline__ void store_few(T* __restrict__ p, const float (&f)[VEC]) {
+  if constexpr (VEC == 1) store_one(p, f[0]);
+  else if constexpr (sizeof(T) == 2) *reinterpret_cast<uint32_t*>(p) = pack_bf16(f[0], f[1]);
+  else *reinterpret_cast<float2*>(p) = make_float2(f[0], f[1]);
+}
+// The logistic function: by the hardware's exponential and reciprocal (an ulp or two) where rows are bf16.
+template <typename T>
+__device__ __forceinline__ float logistic(float z) {
+  if constexpr (sizeof(T) == 2) return __builtin_amdgcn_rcpf(1.0f + __expf(-z));
+  else return 1.0f / (1.0f + expf(-z));
+}
+// One token's step: the state's factor a, and b.
+template <typename T>
+__device__ __forceinline__ void gru_step(float zx, float ux, float& a, float& b) {
+  const float z = logistic<T>(zx), c = ux >= 0.f ? ux + 0.5f : logistic<T>(ux);
+  a = 1.0f - z;
+  b = z * c;
+}
+
+struct GruShape {
+  int slots, rows, stride, width;
+};
+
+// Workspace: a (a, b) pair a chunk and channel, each span's chunks behind one more that holds its first state.
+__device__ __forceinline__ float2* gru_chunk(float2* work, const int* spans, const GruShape& g, int slot, int chunk) {
+  return work + (size_t)(first_chunk(spans, g.slots, slot, g.rows, GRU_CHUNK) * 2 + chunk) * g.width;
+}
+
+template <typename T, int VEC>
+__global__ __launch_bounds__(256) void min_gru_fold_kernel(const T* __restrict__ x, const bf16_t* __restrict__ zb,
+                                                           const bf16_t* __restrict__ xb, const float* __restrict__ state,
+                                                           const int* __restrict__ spans, float2* __restrict__ work, GruShape g) {
+  const int slot = blockIdx.z, chunk = blockIdx.y, c = (blockIdx.x * 256 + threadIdx.x) * VEC;
+  const Span s = span_of(spans, slot, g.rows);
+  const int first = chunk * GRU_CHUNK;
+  if (first >= s.rows || c >= g.width) return;
+  float2* to = gru_chunk(work, spans, g, slot, 0) + c;
+  if (chunk == 0)
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) to[j] = make_float2(0.f, s.start > 0 ? state[(size_t)slot * g.width + c + j] : 0.f);
+  if (first + GRU_CHUNK >= s.rows) return;   // nobody starts from what the last chunk leaves
+  float zbias[VEC], xbias[VEC], a[VEC], b[VEC];
+  load_few<VEC>(zb + c, zbias);
+  load_few<VEC>(xb + c, xbias);
+#pragma unroll
+  for (int j = 0; j < VEC; ++j) a[j] = 1.f, b[j] = 0.f;
+  const T* row = x + (size_t)(s.row0 + first) * g.stride + c;
+  for (int t0 = 0; t0 < GRU_CHUNK; t0 += GRU_AHEAD) {
+    float z[GRU_AHEAD][VEC], u[GRU_AHEAD][VEC];
+#pragma unroll
+    for (int i = 0; i < GRU_AHEAD; ++i) {
+      load_few<VEC>(row + (size_t)(t0 + i) * g.stride, z[i]);
+      load_few<VEC>(row + (size_t)(t0 + i) * g.stride + g.width, u[i]);
+    }
+#pragma unroll
+    for (int i = 0; i < GRU_AHEAD; ++i)
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) {
+        float p, q;
+        gru_step<T>(z[i][j] + zbias[j], u[i][j] + xbias[j], p, q);
+        a[j] *= p;
+        b[j] = fmaf(p, b[j], q);
+      }
+  }
+#pragma unroll
+  for (int j = 0; j < VEC; ++j) to[(size_t)(chunk + 1) * g.width + j] = make_float2(a[j], b[j]);
+}
+
+// CHUNKED: a block's chunk, from what the chunks before it leave in the workspace; else all of a span's rows.
+template <typename T, int VEC, bool CHUNKED>
+__global__ __launch_bounds__(256) void min_gru_kernel(const T* __restrict__ x, const bf16_t* __restrict__ zb,
+                                                      const bf16_t* __restrict__ xb, float* __restrict__ state,
+                                                      const int* __restrict__ spans, float2* __restrict__ work,
+                                                      T* __restrict__ y, GruShape g) {
+  const int slot = blockIdx.z, chunk = blockIdx.y, c = (blockIdx.x * 256 + threadIdx.x) * VEC;
+  const Span s = span_of(spans, slot, g.rows);
+  const int first = chunk * GRU_CHUNK;
+  if (first >= s.rows || c >= g.width) return;
+  const int last = CHUNKED ? min(s.rows, first + GRU_CHUNK) : s.rows;
+  float zbias[VEC], xbias[VEC], S[VEC];
+  load_few<VEC>(zb + c, zbias);
+  load_few<VEC>(xb + c, xbias);
+  float* held = state + (size_t)slot * g.width + c;
+  if (CHUNKED) {
+    const float2* from = gru_chunk(work, spans, g, slot, 0) + c;
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) S[j] = from[j].y;
+#pragma unroll 8
+    for (int k = 1; k <= chunk; ++k)
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) {
+        const float2 ab = from[(size_t)k * g.width + j];
+        S[j] = fmaf(ab.x, S[j], ab.y);
+      }
+  } else {
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) S[j] = s.start > 0 ? held[j] : 0.f;
+  }
+  const T* row = x + (size_t)s.row0 * g.stride + c;
+  T* out = y + (size_t)s.row0 * g.width + c;
+  for (int t0 = first; t0 < last; t0 += GRU_AHEAD) {
+    float z[GRU_AHEAD][VEC], u[GRU_AHEAD][VEC], o[GRU_AHEAD][VEC];
+#pragma unroll
+    for (int i = 0; i < GRU_AHEAD; ++i) {
+      const T* at = row + (size_t)min(t0 + i, last - 1) * g.stride;
+      load_few<VEC>(at, z[i]);
+      load_few<VEC>(at + g.width, u[i]);
+      load_few<VEC>(at + 2 * g.width, o[i]);
+    }
+#pragma unroll
+    for (int i = 0; i < GRU_AHEAD; ++i) {
+      if (t0 + i >= last) break;
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) {
+        float p, q;
+        gru_step<T>(z[i][j] + zbias[j], u[i][j] + xbias[j], p, q);
+        S[j] = fmaf(p, S[j], q);
+        o[i][j] = S[j] * (o[i][j] * logistic<T>(o[i][j]));
+      }
+      store_few<VEC>(out + (size_t)(t0 + i) * g.width, o[i]);
+    }
+  }
+  if (last == s.rows)
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) held[j] = S[j];
+}
+
+template <typename T>
+static int launch_min_gru(const T* x, const bf16_t* zb, const bf16_t* xb, float* state, const int* spans, T* y, float2* work,
+                          const GruShape& g, hipStream_t s) {
+  const bool pairs = g.width % 2 == 0 && g.stride % 2 == 0 &&
+                     ((((uintptr_t)x | (uintptr_t)y) & (2 * sizeof(T) - 1)) | (((uintptr_t)zb | (uintptr_t)xb) & 3)) == 0;
+  const int chunks = work != nullptr ? (g.rows + GRU_CHUNK - 1) / GRU_CHUNK : 1;
+  const dim3 grid((g.width + (pairs ? 511 : 255)) / (pairs ? 512 : 256), chunks, g.slots);
+#define IRON_GRU(VEC)                                                                                                             \
+  if (work != nullptr) {                                                                                                          \
+    hipLaunchKernelGGL((min_gru_fold_kernel<T, VEC>), grid, dim3(256), 0, s, x, zb, xb, state, spans, work, g);                   \
+    hipLaunchKernelGGL((min_gru_kernel<T, VEC, true>), grid, dim3(256), 0, s, x, zb, xb, state, spans, work, y, g);               \
+  } else {                                                                                                                        \
+    hipLaunchKernelGGL((min_gru_kernel<T, VEC, false>), grid, dim3(256), 0, s, x, zb, xb, state, spans, work, y, g);              \
+  }
+  if (pairs) { IRON_GRU(2) }
+  else { IRON_GRU(1) }
+#undef IRON_GRU
+  IRON_LAUNCH_CHECK();
+}
+
+}  // namespace iron
+
+using namespace iron;
+
+extern "C" int64_t iron_min_gru_workspace_bytes(int slots, int rows, int width) {
+  return slots > 0 && rows > 0 && width > 0 ? (int64_t)chunks_of(rows, slots, GRU_CHUNK) * 2 * width * (int64_t)sizeof(float2) : 0;
+}
+
+extern "C" int iron_min_gru(const void* x, const uint16_t* z_bias, const uint16_t* x_bias, float* state, const int* spans, void* y,
+                            void* workspace, int slots, int rows, int stride, int width, int is_float, void* stream) {
+  IRON_REQUIRE(x && z_bias && x_bias && state && spans && y, "min_gru: null operand");
+  IRON_REQUIRE(((uintptr_t)spans & 15) == 0 && ((uintptr_t)workspace & 15) == 0, "min_gru: spans and workspace must be 16-byte aligned");
+  IRON_REQUIRE(slots > 0 && slots <= 65535 && rows > 0 && rows <= GRU_CHUNK * 65535L, "min_gru: slots (%d) and rows (%d) must be positive",
+               slots, rows);
+  IRON_REQUIRE(width > 0 && 3L * width <= stride, "min_gru: a row of %d holds no three projections of %d", stride, width);
+  const GruShape g{slots, rows, stride, width};
+  hipStream_t s = (hipStream_t)stream;
+  if (is_float)
+    return launch_min_gru<float>((const float*)x, z_bias, x_bias, state, spans, (float*)y, (float2*)workspace, g, s);
+  return launch_min_gru<bf16_t>((const bf16_t*)x, z_bias, x_bias, state, spans, (bf16_t*)y, (float2*)workspace, g, s);
+}

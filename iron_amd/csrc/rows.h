@@ -61,4 +61,17 @@ __device__ __forceinline__ Span span_of(const int* __restrict__ spans, int slot,
   return s;
 }
 
+// A batch's spans cut into chunks of `chunk` rows, one after the other in the order of their rows, each span
+// from a chunk of its own: a span's first chunk, and how many there can be.
+__device__ __forceinline__ int first_chunk(const int* __restrict__ spans, int slots, int slot, int rows, int chunk) {
+  const Span mine = span_of(spans, slot, rows);
+  int rank = 0;
+  for (int i = 0; i < slots; ++i) {
+    const Span s = span_of(spans, i, rows);
+    rank += s.rows > 0 && s.row0 < mine.row0;
+  }
+  return mine.row0 / chunk + rank;
+}
+__host__ __device__ inline long chunks_of(int rows, int slots, int chunk) { return (rows + chunk - 1) / chunk + slots; }
+
 }  // namespace iron

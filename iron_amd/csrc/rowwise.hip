@@ -2,7 +2,7 @@
 // elementwise SiLU / mul / add / SiLU*mul.  All HBM-bandwidth bound: 16-byte
 // loads and stores, f32 math, one rounding to bf16 per reference step.
 #include "../../include/iron_hip.h"
-#include "common.h"
+#include "rows.h"
 
 namespace iron {
 
@@ -88,6 +88,94 @@ __global__ __launch_bounds__(256) void rmsnorm_kernel(const bf16_t* __restrict__
   }
   for (int c = threadIdx.x + CHUNKS * 256; c < nchunk; c += 256)
     emit(c, xr[c], w != nullptr ? wr[c] : make_uint4(0, 0, 0, 0), residual != nullptr ? rr[c] : make_uint4(0, 0, 0, 0));
+}
+
+// ------------------------------------------------- polynomial of normed powers
+// y = a N(z) + b N(z^2) + c N(z^3) + e with z = x + bias (columns `at` .. of a row of `stride`), powers
+// element by element and N over a row's root mean square; in float, rounded once.  A block a row; a thread
+// holds its first CH pieces and re-reads the rest.
+template <typename T, int VEC, int CH>
+__global__ __launch_bounds__(256) void poly_norm_kernel(const T* __restrict__ x, const bf16_t* __restrict__ bias,
+                                                        const bf16_t* __restrict__ coef, T* __restrict__ y, int rows, int cols,
+                                                        int stride, int at, float eps, const int* __restrict__ valid) {
+  __shared__ float part[3][4];
+  const int row = blockIdx.x, first = threadIdx.x * VEC;
+  constexpr int STEP = 256 * VEC;
+  float held[CH][VEC];
+  if (bias != nullptr) {
+#pragma unroll
+    for (int i = 0; i < CH; ++i)
+      if (first + i * STEP < cols) load_vec<VEC>(bias + first + i * STEP, held[i]);
+  } else {
+#pragma unroll
+    for (int i = 0; i < CH; ++i)
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) held[i][j] = 0.f;
+  }
+  const float a = bf16_to_f32(coef[0]), b = bf16_to_f32(coef[1]), c = bf16_to_f32(coef[2]), e = bf16_to_f32(coef[3]);
+  if (row >= bound_or(valid, rows)) return;
+  const T* xr = x + (size_t)row * stride + at;
+  T* yr = y + (size_t)row * cols;
+  float s1 = 0.f, s2 = 0.f, s3 = 0.f;
+  auto add = [&](float z) {
+    const float p = z * z, q = p * z;
+    s1 += p;
+    s2 = fmaf(p, p, s2);
+    s3 = fmaf(q, q, s3);
+  };
+  auto rest = [&](int at_col, float (&f)[VEC]) {
+    load_vec<VEC>(xr + at_col, f);
+    if (bias != nullptr) {
+      float g[VEC];
+      load_vec<VEC>(bias + at_col, g);
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) f[j] += g[j];
+    }
+  };
+#pragma unroll
+  for (int i = 0; i < CH; ++i)
+    if (first + i * STEP < cols) {
+      float f[VEC];
+      load_vec<VEC>(xr + first + i * STEP, f);
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) {
+        held[i][j] += f[j];
+        add(held[i][j]);
+      }
+    }
+  for (int at_col = first + CH * STEP; at_col < cols; at_col += STEP) {
+    float f[VEC];
+    rest(at_col, f);
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) add(f[j]);
+  }
+  s1 = wave_sum(s1);
+  s2 = wave_sum(s2);
+  s3 = wave_sum(s3);
+  if ((threadIdx.x & 63) == 0) {
+    const int w = threadIdx.x >> 6;
+    part[0][w] = s1;
+    part[1][w] = s2;
+    part[2][w] = s3;
+  }
+  __syncthreads();
+  auto over = [&](int k, float by) { return by / sqrtf((part[k][0] + part[k][1] + part[k][2] + part[k][3]) / (float)cols + eps); };
+  const float f1 = over(0, a), f2 = over(1, b), f3 = over(2, c);
+  auto value = [&](float z) { return fmaf(z, fmaf(z, fmaf(z, f3, f2), f1), e); };
+#pragma unroll
+  for (int i = 0; i < CH; ++i)
+    if (first + i * STEP < cols) {
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) held[i][j] = value(held[i][j]);
+      store_vec<VEC>(yr + first + i * STEP, held[i]);
+    }
+  for (int at_col = first + CH * STEP; at_col < cols; at_col += STEP) {
+    float f[VEC];
+    rest(at_col, f);
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) f[j] = value(f[j]);
+    store_vec<VEC>(yr + at_col, f);
+  }
 }
 
 // ------------------------------------------------------------------- RoPE
@@ -253,6 +341,27 @@ static int rmsnorm(const uint16_t* x, const uint16_t* w, const uint16_t* residua
     hipLaunchKernelGGL((rmsnorm_kernel<2>), dim3(rows), dim3(256), 0, s, x, w, y, rows, cols, eps, valid, residual);
   else
     hipLaunchKernelGGL((rmsnorm_kernel<4>), dim3(rows), dim3(256), 0, s, x, w, y, rows, cols, eps, valid, residual);
+  IRON_LAUNCH_CHECK();
+}
+
+extern "C" int iron_poly_norm(const void* x, const uint16_t* bias, const uint16_t* coefficients, void* y, int rows, int cols,
+                              int stride, int at, float eps, int is_float, const int* valid, void* stream) {
+  IRON_REQUIRE(x && coefficients && y, "poly_norm: null operand");
+  IRON_REQUIRE(rows > 0 && cols > 0, "poly_norm: rows (%d) and cols (%d) must be positive", rows, cols);
+  IRON_REQUIRE(at >= 0 && at + cols <= stride, "poly_norm: columns %d .. + %d of a row of %d", at, cols, stride);
+  const bool vec = cols % 8 == 0 && stride % 8 == 0 && at % 8 == 0 && (((uintptr_t)x | (uintptr_t)bias | (uintptr_t)y) & 15) == 0;
+#define IRON_POLY(T, VEC, CH)                                                                                                     \
+  hipLaunchKernelGGL((poly_norm_kernel<T, VEC, CH>), dim3(rows), dim3(256), 0, (hipStream_t)stream, (const T*)x, bias, coefficients, \
+                     (T*)y, rows, cols, stride, at, eps, valid)
+#define IRON_POLY_OF(T)                       \
+  if (vec && cols <= 2048) IRON_POLY(T, 8, 1); \
+  else if (vec && cols <= 4096) IRON_POLY(T, 8, 2); \
+  else if (vec) IRON_POLY(T, 8, 4);           \
+  else IRON_POLY(T, 1, 8);
+  if (is_float) { IRON_POLY_OF(float) }
+  else { IRON_POLY_OF(bf16_t) }
+#undef IRON_POLY_OF
+#undef IRON_POLY
   IRON_LAUNCH_CHECK();
 }
 

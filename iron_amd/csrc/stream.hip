@@ -1,5 +1,5 @@
 // A decoder's residual stream held in float32: rows gathered from a bf16 table into it, a row's RMS
-// norm out of it, a block's normed output added to it, and the head's soft cap.  One rounding, to the
+// norm out of it, a block's normed or gated output added to it, and the head's scale and soft cap.  One rounding, to the
 // activation type, where a row leaves the stream; bandwidth bound, a block a row.
 #include "../../include/iron_hip.h"
 #include "rows.h"
@@ -29,13 +29,21 @@ __device__ __forceinline__ float row_total(float v, float* part) {
   return part[0] + part[1] + part[2] + part[3];
 }
 
-// ADD: x += rmsnorm(y) * wb, in place.  NORM: h = rmsnorm(x) * w of the row as it then stands.
+// What joins the stream: nothing, a block's row normed (rmsnorm(y) * wb), or a block's row gated
+// ((y + yb) * sigmoid(gate + gb), the gate columns `at` .. of rows of `stride`).
+enum { ADD_NONE = 0, ADD_NORMED = 1, ADD_GATED = 2 };
+struct StreamGate {
+  const void* gate;          // rows of the activation type
+  const bf16_t *bias, *y_bias;   // gb, yb (yb may be null)
+  int stride, at;
+};
+// x += what ADD says, in place.  NORM: h = rmsnorm(x) * w of the row as it then stands.
 // A thread holds its first CH pieces of the row between the passes and re-reads the rest.
-template <typename T, int VEC, int CH, bool ADD, bool NORM>
+template <typename T, int VEC, int CH, int ADD, bool NORM>
 __global__ __launch_bounds__(256) void stream_rows_kernel(float* __restrict__ x, const T* __restrict__ y,
                                                           const bf16_t* __restrict__ wb, const bf16_t* __restrict__ w,
                                                           T* __restrict__ h, int rows, int cols, float eps,
-                                                          const int* __restrict__ valid) {
+                                                          const int* __restrict__ valid, StreamGate g) {
   __shared__ float part[4];
   const int row = blockIdx.x, first = threadIdx.x * VEC;
   constexpr int STEP = 256 * VEC;
@@ -51,7 +59,41 @@ __global__ __launch_bounds__(256) void stream_rows_kernel(float* __restrict__ x,
   for (int i = 0; i < CH; ++i)
     if (first + i * STEP < cols) load_vec<VEC>(xr + first + i * STEP, held[i]);
 
-  if (ADD) {
+  if (ADD == ADD_GATED) {
+    const T* yr = y + (size_t)row * cols;
+    const T* gr = reinterpret_cast<const T*>(g.gate) + (size_t)row * g.stride + g.at;
+    auto gated = [&](int c, float (&f)[VEC]) {
+      float z[VEC], b[VEC], yb[VEC];
+      load_vec<VEC>(yr + c, f);
+      load_vec<VEC>(gr + c, z);
+      load_vec<VEC>(g.bias + c, b);
+      if (g.y_bias != nullptr) {
+        load_vec<VEC>(g.y_bias + c, yb);
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) f[j] += yb[j];
+      }
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) f[j] *= 1.0f / (1.0f + expf(-(z[j] + b[j])));
+    };
+#pragma unroll
+    for (int i = 0; i < CH; ++i)
+      if (first + i * STEP < cols) {
+        float f[VEC];
+        gated(first + i * STEP, f);
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) held[i][j] += f[j];
+        store_vec<VEC>(xr + first + i * STEP, held[i]);
+      }
+    for (int c = first + CH * STEP; c < cols; c += STEP) {
+      float f[VEC], s[VEC];
+      gated(c, f);
+      load_vec<VEC>(xr + c, s);
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) s[j] += f[j];
+      store_vec<VEC>(xr + c, s);
+    }
+  }
+  if (ADD == ADD_NORMED) {
     const T* yr = y + (size_t)row * cols;
     float out[CH][VEC], back[CH][VEC];
     float ss = 0.f;
@@ -130,14 +172,14 @@ __global__ __launch_bounds__(256) void span_tails_kernel(const float* __restrict
   for (int c = threadIdx.x; c < cols; c += 256) out[(size_t)blockIdx.x * cols + c] = src[c];
 }
 
-// cap * tanh(x / cap): in float32, and rounded to bf16 for the draw (rows of `stride`, whole 16-byte
-// pieces).  cap 0: no cap.
+// scale * x, then cap * tanh(x / cap): in float32, and rounded to bf16 for the draw (rows of `stride`,
+// whole 16-byte pieces).  cap 0: no cap.
 template <typename T>
 __global__ __launch_bounds__(256) void softcap_kernel(const T* __restrict__ x, float* __restrict__ y,
-                                                      bf16_t* __restrict__ rounded, int cols, int stride, float cap) {
+                                                      bf16_t* __restrict__ rounded, int cols, int stride, float cap, float scale) {
   const size_t row = blockIdx.y;
   for (int i = blockIdx.x * 256 + threadIdx.x; i < cols; i += gridDim.x * 256) {
-    float v = load_one(x + row * cols + i);
+    float v = load_one(x + row * cols + i) * scale;
     if (cap > 0.f) v = cap * tanhf(v / cap);
     y[row * cols + i] = v;
     rounded[row * stride + i] = f32_to_bf16(v);
@@ -198,16 +240,18 @@ __global__ __launch_bounds__(256) void linear_any_kernel(const T* __restrict__ x
     }
 }
 
-template <typename T, bool ADD, bool NORM>
+template <typename T, int ADD, bool NORM>
 static int launch_stream_rows(float* x, const T* y, const bf16_t* wb, const bf16_t* w, T* h, int rows, int cols, float eps,
-                              const int* valid, hipStream_t s) {
-  const bool vec = cols % 8 == 0 && (((uintptr_t)x | (uintptr_t)y | (uintptr_t)wb | (uintptr_t)w | (uintptr_t)h) & 15) == 0;
+                              const int* valid, hipStream_t s, const StreamGate& g = StreamGate{nullptr, nullptr, nullptr, 8, 8}) {
+  const bool vec = cols % 8 == 0 && g.stride % 8 == 0 && g.at % 8 == 0 &&
+                   (((uintptr_t)x | (uintptr_t)y | (uintptr_t)wb | (uintptr_t)w | (uintptr_t)h | (uintptr_t)g.gate | (uintptr_t)g.bias |
+                     (uintptr_t)g.y_bias) & 15) == 0;
   if (vec && cols <= 2048)
-    hipLaunchKernelGGL((stream_rows_kernel<T, 8, 1, ADD, NORM>), dim3(rows), dim3(256), 0, s, x, y, wb, w, h, rows, cols, eps, valid);
+    hipLaunchKernelGGL((stream_rows_kernel<T, 8, 1, ADD, NORM>), dim3(rows), dim3(256), 0, s, x, y, wb, w, h, rows, cols, eps, valid, g);
   else if (vec)
-    hipLaunchKernelGGL((stream_rows_kernel<T, 8, 2, ADD, NORM>), dim3(rows), dim3(256), 0, s, x, y, wb, w, h, rows, cols, eps, valid);
+    hipLaunchKernelGGL((stream_rows_kernel<T, 8, 2, ADD, NORM>), dim3(rows), dim3(256), 0, s, x, y, wb, w, h, rows, cols, eps, valid, g);
   else
-    hipLaunchKernelGGL((stream_rows_kernel<T, 1, 4, ADD, NORM>), dim3(rows), dim3(256), 0, s, x, y, wb, w, h, rows, cols, eps, valid);
+    hipLaunchKernelGGL((stream_rows_kernel<T, 1, 4, ADD, NORM>), dim3(rows), dim3(256), 0, s, x, y, wb, w, h, rows, cols, eps, valid, g);
   IRON_LAUNCH_CHECK();
 }
 
@@ -240,12 +284,30 @@ extern "C" int iron_stream_rows(float* x, const void* y, const uint16_t* back_ga
   IRON_REQUIRE(rows > 0 && cols > 0, "stream_rows: rows (%d) and cols (%d) must be positive", rows, cols);
   hipStream_t s = (hipStream_t)stream;
 #define IRON_STREAM_ROWS(T)                                                                                             \
-  if (y && h) return launch_stream_rows<T, true, true>(x, (const T*)y, back_gain, gain, (T*)h, rows, cols, eps, valid, s); \
-  if (y) return launch_stream_rows<T, true, false>(x, (const T*)y, back_gain, gain, (T*)h, rows, cols, eps, valid, s);     \
-  return launch_stream_rows<T, false, true>(x, (const T*)y, back_gain, gain, (T*)h, rows, cols, eps, valid, s);
+  if (y && h) return launch_stream_rows<T, ADD_NORMED, true>(x, (const T*)y, back_gain, gain, (T*)h, rows, cols, eps, valid, s); \
+  if (y) return launch_stream_rows<T, ADD_NORMED, false>(x, (const T*)y, back_gain, gain, (T*)h, rows, cols, eps, valid, s);     \
+  return launch_stream_rows<T, ADD_NONE, true>(x, (const T*)y, back_gain, gain, (T*)h, rows, cols, eps, valid, s);
   if (is_float) { IRON_STREAM_ROWS(float) }
   IRON_STREAM_ROWS(bf16_t)
 #undef IRON_STREAM_ROWS
+}
+
+extern "C" int iron_stream_gated_rows(float* x, const void* y, const uint16_t* y_bias, const void* gate, const uint16_t* gate_bias,
+                                      int gate_stride, int gate_at, const uint16_t* gain, void* h, int rows, int cols, float eps,
+                                      int is_float, const int* valid, void* stream) {
+  IRON_REQUIRE(x && y && gate && gate_bias, "stream_gated_rows: null operand");
+  IRON_REQUIRE((h == nullptr) == (gain == nullptr), "stream_gated_rows: a gain for the norm that is taken");
+  IRON_REQUIRE(rows > 0 && cols > 0, "stream_gated_rows: rows (%d) and cols (%d) must be positive", rows, cols);
+  IRON_REQUIRE(gate_at >= 0 && gate_at + cols <= gate_stride, "stream_gated_rows: columns %d .. + %d of a gate's row of %d", gate_at, cols,
+               gate_stride);
+  hipStream_t s = (hipStream_t)stream;
+  const StreamGate g{gate, gate_bias, y_bias, gate_stride, gate_at};
+#define IRON_STREAM_GATED(T)                                                                                                    \
+  if (h) return launch_stream_rows<T, ADD_GATED, true>(x, (const T*)y, nullptr, gain, (T*)h, rows, cols, eps, valid, s, g); \
+  return launch_stream_rows<T, ADD_GATED, false>(x, (const T*)y, nullptr, gain, (T*)h, rows, cols, eps, valid, s, g);
+  if (is_float) { IRON_STREAM_GATED(float) }
+  IRON_STREAM_GATED(bf16_t)
+#undef IRON_STREAM_GATED
 }
 
 extern "C" int iron_span_tails(const float* x, const int* spans, float* out, int slots, int rows, int cols, void* stream) {
@@ -257,16 +319,16 @@ extern "C" int iron_span_tails(const float* x, const int* spans, float* out, int
 }
 
 extern "C" int iron_softcap(const void* x, float* y, uint16_t* rounded, int rows, int cols, int rounded_stride, float cap,
-                            int is_float, void* stream) {
+                            float scale, int is_float, void* stream) {
   IRON_REQUIRE(x && y && rounded, "softcap: null operand");
   IRON_REQUIRE(rows > 0 && rows <= 65535 && cols > 0 && rounded_stride >= cols && cap >= 0.f,
                "softcap: rows (%d) and cols (%d) must be positive, a rounded row (%d) no shorter, cap (%g) not negative", rows,
                cols, rounded_stride, (double)cap);
   const dim3 grid(few_blocks(cols), rows);
   if (is_float)
-    hipLaunchKernelGGL((softcap_kernel<float>), grid, dim3(256), 0, (hipStream_t)stream, (const float*)x, y, rounded, cols, rounded_stride, cap);
+    hipLaunchKernelGGL((softcap_kernel<float>), grid, dim3(256), 0, (hipStream_t)stream, (const float*)x, y, rounded, cols, rounded_stride, cap, scale);
   else
-    hipLaunchKernelGGL((softcap_kernel<bf16_t>), grid, dim3(256), 0, (hipStream_t)stream, (const bf16_t*)x, y, rounded, cols, rounded_stride, cap);
+    hipLaunchKernelGGL((softcap_kernel<bf16_t>), grid, dim3(256), 0, (hipStream_t)stream, (const bf16_t*)x, y, rounded, cols, rounded_stride, cap, scale);
   IRON_LAUNCH_CHECK();
 }
 

@@ -631,6 +631,35 @@ def stream_rows(x, *, rows, cols, eps, y=None, back_gain=None, h=None, gain=None
                                  ptr(_word(valid, "valid")), current_stream()), "iron_stream_rows")
 
 
+def stream_gated_rows(x, y, gate, gate_bias, *, rows, cols, eps=0.0, gate_stride, gate_at, y_bias=None, h=None, gain=None, valid=None):
+    """``x += (y + y_bias) * sigmoid(gate + gate_bias)`` and, with ``h``, ``h = rmsnorm(x) * gain``, one launch."""
+    _f32(x, rows * cols, "x")
+    is_float = _act(y, rows * cols, "y")
+    _same_kind(is_float, gate=gate)
+    _act(gate, rows * gate_stride, "gate")
+    _bf16(gate_bias, cols, "gate_bias")
+    if y_bias is not None:
+        _bf16(y_bias, cols, "y_bias")
+    if h is not None:
+        _same_kind(is_float, h=h)
+        _act(h, rows * cols, "h")
+        _bf16(gain, cols, "gain")
+    check(lib().iron_stream_gated_rows(ptr(x), ptr(y), ptr(y_bias), ptr(gate), ptr(gate_bias), gate_stride, gate_at, ptr(gain), ptr(h),
+                                       rows, cols, float(eps), int(is_float), ptr(_word(valid, "valid")), current_stream()),
+          "iron_stream_gated_rows")
+
+
+def poly_norm(x, coefficients, y, *, rows, cols, stride, at, eps, bias=None, valid=None):
+    is_float = _act(x, rows * stride, "x")
+    _bf16(coefficients, 4, "coefficients")
+    if bias is not None:
+        _bf16(bias, cols, "bias")
+    _same_kind(is_float, y=y)
+    _act(y, rows * cols, "y")
+    check(lib().iron_poly_norm(ptr(x), ptr(bias), ptr(coefficients), ptr(y), rows, cols, stride, at, float(eps), int(is_float),
+                               ptr(_word(valid, "valid")), current_stream()), "iron_poly_norm")
+
+
 def span_tails(x, spans, out, *, slots, rows, cols):
     _f32(x, rows * cols, "x")
     _f32(out, slots * cols, "out")
@@ -638,11 +667,11 @@ def span_tails(x, spans, out, *, slots, rows, cols):
           "iron_span_tails")
 
 
-def softcap(x, y, rounded, *, rows, cols, stride, cap):
+def softcap(x, y, rounded, *, rows, cols, stride, cap, scale=1.0):
     is_float = _act(x, rows * cols, "x")
     _f32(y, rows * cols, "y")
     _bf16(rounded, rows * stride, "rounded")
-    check(lib().iron_softcap(ptr(x), ptr(y), ptr(rounded), rows, cols, stride, float(cap), int(is_float),
+    check(lib().iron_softcap(ptr(x), ptr(y), ptr(rounded), rows, cols, stride, float(cap), float(scale), int(is_float),
                              current_stream()), "iron_softcap")
 
 
@@ -760,6 +789,60 @@ def mha_window(x, keys, values, bias, spans, out, *, slots, rows, stride, heads,
     check(lib().iron_mha_window(ptr(x), ptr(keys), ptr(values), ptr(bias), _spans(spans, slots), ptr(out), slots, rows, stride,
                                 heads, kv_heads, dim, vdim, window, ring, float(scale), out_stride, out_at, float(out_scale),
                                 int(single), int(is_float), current_stream()), "iron_mha_window")
+
+
+def min_gru(x, z_bias, x_bias, state, spans, y, *, slots, rows, stride, width, workspace=None):
+    """The gated recurrence a span's rows in turn, or with ``workspace`` its chunks side by side."""
+    is_float = _act(x, rows * stride, "x")
+    _bf16(z_bias, width, "z_bias")
+    _bf16(x_bias, width, "x_bias")
+    _f32(state, slots * width, "state")
+    _same_kind(is_float, y=y)
+    _act(y, rows * width, "y")
+    work = None if workspace is None else _work(workspace, int(lib().iron_min_gru_workspace_bytes(slots, rows, width)), "min_gru: workspace")
+    check(lib().iron_min_gru(ptr(x), ptr(z_bias), ptr(x_bias), ptr(state), _spans(spans, slots), ptr(y), work, slots, rows, stride,
+                             width, int(is_float), current_stream()), "iron_min_gru")
+
+
+def _turned(angles, angle_rows, turned):
+    if turned:
+        _f32(angles, angle_rows * turned, "angles")
+    return ptr(angles)
+
+
+def latent_rows(x, q_gain, c_gain, spans, q_out, latents, *, slots, rows, stride, q_rank, rank, ring, eps, rot=0, turned=0,
+                angle_rows=0, angles=None, shared_keys=None):
+    is_float = _act(x, rows * stride, "x")
+    _bf16(q_gain, q_rank, "q_gain")
+    _bf16(c_gain, rank, "c_gain")
+    _same_kind(is_float, q_out=q_out, latents=latents)
+    _act(q_out, rows * q_rank, "q_out")
+    _act(latents, slots * ring * rank, "latents")
+    if rot:
+        _same_kind(is_float, shared_keys=shared_keys)
+        _act(shared_keys, slots * ring * rot, "shared_keys")
+    check(lib().iron_latent_rows(ptr(x), ptr(q_gain), ptr(c_gain), _turned(angles, angle_rows, turned), _spans(spans, slots), ptr(q_out),
+                                 ptr(latents), ptr(shared_keys), slots, rows, stride, q_rank, rank, rot, turned, angle_rows, ring,
+                                 float(eps), int(is_float), current_stream()), "iron_latent_rows")
+
+
+def mha_latent(q, latents, up, spans, y, workspace, *, slots, rows, heads, dim, vdim, rank, window, ring, cap, scale, rot=0, turned=0,
+               angle_rows=0, angles=None, shared_keys=None, sink=None, single=False):
+    is_float = _act(q, rows * heads * (dim + rot), "q")
+    _same_kind(is_float, latents=latents, y=y)
+    _act(latents, slots * ring * rank, "latents")
+    if rot:
+        _same_kind(is_float, shared_keys=shared_keys)
+        _act(shared_keys, slots * ring * rot, "shared_keys")
+    _bf16(up, heads * (dim + vdim) * rank, "up")
+    if sink is not None:
+        _bf16(sink, heads, "sink")
+    _act(y, rows * heads * vdim, "y")
+    need = int(lib().iron_mha_latent_workspace_bytes(slots, rows, heads, dim, rot, vdim, rank, window, ring, cap, int(single), int(is_float)))
+    check(lib().iron_mha_latent(ptr(q), ptr(latents), ptr(shared_keys), ptr(up), ptr(sink), _turned(angles, angle_rows, turned),
+                                _spans(spans, slots), ptr(y), _work(workspace, need, "mha_latent: workspace"), slots, rows, heads, dim,
+                                rot, vdim, rank, turned, angle_rows, window, ring, cap, float(scale), int(single), int(is_float),
+                                current_stream()), "iron_mha_latent")
 
 
 def decode_mixed(h, carry, spans, products, *, k):

@@ -17,14 +17,26 @@ from .blocks import (
 )
 from .causal import Call, CausalLM, Decoder, Stats
 from .checkpoint import Checkpoint, weights_file, write_safetensors
-from .config import DecoderConfig, rope_angles
+from .config import DecoderConfig, LayerListConfig, rope_angles
 from .generation import Sampler
-from .mixers import DeltaMixer, ParallelMixer, StreamLayer, StreamRMSNorm, TimeMixing, WindowAttention
+from .mixers import (
+    DeltaMixer,
+    GatedRecurrence,
+    GatedStreamLayer,
+    LatentAttention,
+    ParallelMixer,
+    PolyNormMLP,
+    StreamLayer,
+    StreamRMSNorm,
+    TimeMixing,
+    WindowAttention,
+)
 from .session import Session
 
 __all__ = [
     "Attention", "Batch", "BatchedLM", "Call", "CausalLM", "Checkpoint", "Decoder", "DecoderConfig", "DecoderLayer",
-    "DeltaMixer", "Embedding", "Entry", "GatedMLP", "KVCache", "Linear", "ParallelMixer", "PleLayer", "RMSNorm",
-    "Rope", "Sampler", "SandwichLayer", "Session", "SlotSession", "Stats", "StreamLayer", "StreamRMSNorm",
-    "TimeMixing", "WindowAttention", "activation", "residual_add", "rope_angles", "weights_file", "write_safetensors",
+    "DeltaMixer", "Embedding", "Entry", "GatedMLP", "GatedRecurrence", "GatedStreamLayer", "KVCache", "LatentAttention",
+    "LayerListConfig", "Linear", "ParallelMixer", "PleLayer", "PolyNormMLP", "RMSNorm", "Rope", "Sampler", "SandwichLayer",
+    "Session", "SlotSession", "Stats", "StreamLayer", "StreamRMSNorm", "TimeMixing", "WindowAttention", "activation",
+    "residual_add", "rope_angles", "weights_file", "write_safetensors",
 ]

@@ -151,13 +151,17 @@ class Batch:
     def _portions(self, entries, ids) -> list[np.ndarray]:
         model, c = self.lm, self.lm.config
         done = [0] * len(entries)
+        room = c.key_room
         out = [np.empty((len(e.want), c.vocab_size), np.float32) for e in entries]
         while True:
-            row, spans, portion, asked = 0, np.zeros((c.slots, 4), np.int32), np.zeros(c.prefill_chunk, np.int32), []
+            row, keys, spans, portion, asked = 0, 0, np.zeros((c.slots, 4), np.int32), np.zeros(c.prefill_chunk, np.int32), []
             for i, (e, t) in enumerate(zip(entries, ids)):
                 n = min(t.size - done[i], c.prefill_chunk - row)
+                if n > 0 and room is not None:   # (a request alone always fits: it has no more keys than positions)
+                    n = min(n, room - keys - self.held[e.key])
                 if n <= 0:
                     continue
+                keys += self.held[e.key] + n
                 spans[self.slots[e.key], :3] = row, n, self.held[e.key]
                 portion[row : row + n] = t[done[i] : done[i] + n]
                 asked += [(i, k, row + w - done[i]) for k, w in enumerate(e.want) if done[i] <= w < done[i] + n]
@@ -346,8 +350,9 @@ class BatchedLM(CausalLM):
     """A ``CausalLM`` whose graph runs a batch of spans over a float32 residual stream.  ``runs`` lists the
     layer runs in order, each the index of its layer and the states of that run alone.
 
-    The config adds to a decoder's ``slots`` (sequences served at once), ``activations`` (bf16, or float32
-    for a model in 32 bits throughout), ``order`` (layer indices in running order) and ``logit_softcap``."""
+    The config is a ``LayerListConfig``: it adds to a decoder's ``slots`` (sequences served at once),
+    ``activations`` (bf16, or float32 for a model in 32 bits throughout), ``order`` (layer indices in running
+    order), ``logit_scale``, ``logit_softcap`` and ``key_room`` (keys a portion's layers may attend in all)."""
 
     decoder_class = StreamDecoder
     session_class = SlotSession
@@ -385,9 +390,10 @@ class BatchedLM(CausalLM):
         return logits
 
     def head(self, x):
-        """Final norm, output projection and soft cap: float32 logits, and the draw's rounded ones."""
+        """Final norm, output projection, scale and soft cap: float32 logits, and the draw's rounded ones."""
         logits = as_rows(self.lm_head(self.model.norm(x)), x.shape[0])
-        return Softcap.step(logits, cap=self.config.logit_softcap or 0.0, dtype=self.config.activations)
+        return Softcap.step(logits, cap=self.config.logit_softcap or 0.0, scale=self.config.logit_scale,
+                            dtype=self.config.activations)
 
     # ------------------------------------------------------------------ versions
     def shapes(self) -> list[dict]:

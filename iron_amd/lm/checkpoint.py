@@ -285,6 +285,41 @@ class Checkpoint:
         return nest({name: self.tensors[name] for name in self._stored}, file=self.path)
 
 
+class Renaming:
+    """A checkpoint's tensors under the names of a model's modules; tensors that are read together joined.
+    ``who`` labels the errors."""
+
+    def __init__(self, weights: Mapping[str, Any], who: str):
+        self.left, self.who, self.named = dict(weights), who, {}
+
+    def take(self, name: str):
+        if name not in self.left:
+            raise ValueError(f"{self.who}: the checkpoint lacks {name}")
+        return self.left.pop(name)
+
+    def drop(self, name: str) -> None:
+        """Leave ``name`` aside if it is there."""
+        self.left.pop(name, None)
+
+    def put(self, target: str, *names: str, axis: int = 0) -> None:
+        found = [self.take(n) for n in names]
+        self.named[target] = found[0] if len(found) == 1 else joined(found, axis)
+
+    def done(self) -> dict[str, Any]:
+        if self.left:
+            raise ValueError(f"{self.who}: the checkpoint holds {sorted(self.left)}, which no layer reads")
+        return self.named
+
+
+def joined(tensors, axis: int):
+    """The tensors side by side along ``axis``, torch or numpy as they come."""
+    if type(tensors[0]).__module__.split(".")[0] == "torch":
+        import torch
+
+        return torch.cat(tensors, dim=axis)
+    return np.concatenate(tensors, axis=axis)
+
+
 # ---- dotted names <-> nested objects
 
 

@@ -176,3 +176,73 @@ class DecoderConfig(ConfigFile):
         if self.rope_theta is None:
             return None
         return rope_angles(self.rope_width, self.max_seq_len, self.rope_theta, self.rope_scaling)
+
+
+class LayerListConfig(ConfigFile):
+    """A decoder served by spans whose ``config.json`` lists its layers, each with its sizes.  A subclass is a
+    frozen dataclass with this package's own choices among its fields (``max_seq_len``: positions a slot is
+    served, ``prefill_chunk``, ``slots``, ``activations``: bf16, or float32 for a model in 32 bits throughout,
+    ``precision``) and says in KEYS where the file keeps the others."""
+
+    ARCHITECTURE = ""
+    KEYS: dict[str, tuple[str, ...]] = {}   # field -> where config.json keeps it
+
+    tie_word_embeddings = False
+    rope_theta = None
+    logit_softcap = None
+    logit_scale = 1.0
+    key_room = None        # keys, of all requests together, that a portion may attend; None: any number
+
+    def check_serving(self) -> None:
+        """Bound this package's own choices by each other."""
+        if self.prefill_chunk > self.max_seq_len * self.slots:
+            object.__setattr__(self, "prefill_chunk", self.max_seq_len * self.slots)   # the dataclass is frozen
+        if self.slots < 1:
+            raise ValueError(f"{type(self).__name__}: slots ({self.slots}) must be at least 1")
+
+    def check_layers(self, mixers) -> None:
+        """Refuse a layer whose mixer or feed-forward is none of this design's."""
+        for i, spec in enumerate(self.layers):
+            if spec["type"] not in mixers:
+                raise ValueError(f"{type(self).__name__}: layer {i} is {spec['type']!r}, not one of {tuple(mixers)}")
+            mlp = spec.get("mlp")
+            if mlp is not None and mlp.get("kind") != "dense":
+                raise ValueError(f"{type(self).__name__}: layer {i}'s feed-forward is {mlp.get('kind')!r}, not 'dense'")
+
+    @classmethod
+    def from_json(cls, data: dict, source="config.json"):
+        """Raises ValueError where a size or constant without a default is absent."""
+        given, absent = {}, []
+        for field in dataclasses.fields(cls):
+            if field.name not in cls.KEYS:
+                continue
+            value = data
+            for key in cls.KEYS[field.name]:
+                value = value.get(key) if isinstance(value, dict) else None
+            if value is not None:
+                given[field.name] = tuple(value) if isinstance(value, list) else value
+            elif _required(field):
+                absent.append(".".join(cls.KEYS[field.name]))
+        if absent:
+            raise ValueError(f"{source} lacks {absent}")
+        return cls(**given)
+
+    def to_json(self) -> dict:
+        out: dict = {"architecture": self.ARCHITECTURE}
+        for name, keys in self.KEYS.items():
+            value, scope = getattr(self, name), out
+            if value is None:
+                continue
+            for key in keys[:-1]:
+                scope = scope.setdefault(key, {})
+            scope[keys[-1]] = list(value) if isinstance(value, tuple) else value
+        return out
+
+    @property
+    def num_hidden_layers(self) -> int:
+        return len(self.layers)
+
+    @property
+    def order(self) -> list[int]:
+        """Layer indices in the order they run."""
+        return list(range(len(self.layers)))

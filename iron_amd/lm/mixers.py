@@ -1,6 +1,7 @@
 """Token mixers over a batch of rows told apart by spans, and the layer that runs them around a float32
 residual stream: sliding-window attention with a learned distance bias, time mixing with a
-data-dependent decay, both side by side, and the gated delta rule.
+data-dependent decay, both side by side, the gated delta rule, a gated recurrence element by element, and
+latent attention.
 
 A module holds weights; what a run of it carries from token to token is a ``states()`` mapping the
 caller makes once per run, so that a layer run several times in a row has a state for each pass.
@@ -15,9 +16,10 @@ import numpy as np
 
 from .. import functional as F
 from ..common import graph as iron
+from ..operators.mha_latent import EVERYTHING, LatentMHA, LatentRows
 from ..operators.mha_window import WindowMHA
-from ..operators.recurrent import DeltaRule, HeadGate, LowRankDecay, ShortConv, TimeMix, TokenShift
-from ..operators.stream import StreamAdd, StreamNorm
+from ..operators.recurrent import DeltaRule, HeadGate, LowRankDecay, MinGRU, ShortConv, TimeMix, TokenShift
+from ..operators.stream import PolyNorm, StreamAdd, StreamGatedAdd, StreamNorm
 from .blocks import Linear
 
 
@@ -200,4 +202,109 @@ class StreamLayer(iron.Graph):
         x = self.norm1b.add(x, as_rows(self.mixer(self.norm1(x), call, state), x.shape[0]))
         if self.mlp is not None:
             x = self.norm2b.add(x, as_rows(self.mlp(self.norm2(x)), x.shape[0]))
+        return x
+
+
+# ---- blocks whose packed projection carries, behind its own columns, a gate of ``gate`` columns for the layer
+
+
+class GatedRecurrence(iron.Graph):
+    """minGRU: a state a channel, moved towards a candidate by a gate, both of the current token alone, and read
+    through a SiLU gate.  ``proj`` is one packed projection (z, x, g and the layer's gate)."""
+
+    def __init__(self, width, *, inner, gate, dtype, precision):
+        self.inner, self.dtype, self.own = inner, dtype, 3 * inner
+        self.proj = Linear(width, self.own + gate, precision=precision)
+        self.z_bias = iron.param(inner)
+        self.x_bias = iron.param(inner)
+        self.out = Linear(inner, width, precision=precision)
+
+    def states(self, slots: int) -> dict:
+        return {"memory": iron.state((slots, self.inner), np.float32)}
+
+    def body(self, x, call, state):
+        return self.out(MinGRU.step(x, self.z_bias, self.x_bias, state["memory"], call.spans, dtype=self.dtype)[1])
+
+
+class LatentAttention(iron.Graph):
+    """Latent attention: queries through a normed latent of ``q_rank``; keys and values of every head from one
+    of ``rank``, the only thing kept of a position beside ``rot`` key columns that all heads share, which turn with
+    the position by ``angles``.  ``window`` None: everything before.  ``sink``: a learned term a head in the softmax's
+    denominator.  ``proj`` is one packed projection (query latent, latent, shared key part and the layer's gate);
+    ``room`` how many keys a prompt's portion may attend in all, ``portion`` its rows."""
+
+    def __init__(self, width, *, heads, dim, vdim, q_rank, rank, scale, eps, gate, context, portion, room, dtype, precision, rot=0,
+                 angles=None, window=None, sink=False):
+        self.heads, self.rot, self.rank, self.scale, self.eps, self.dtype = heads, rot, rank, scale, eps, dtype
+        self.own = q_rank + rank + rot
+        self.window = EVERYTHING if window is None or window >= context else window
+        self.context, self.portion, self.room = context, portion, room
+        self.angles = angles
+        self.proj = Linear(width, self.own + gate, precision=precision)
+        self.q_norm = iron.param(q_rank)
+        self.c_norm = iron.param(rank)
+        self.query = Linear(q_rank, heads * (dim + rot), precision=precision)
+        self.up = iron.param(heads * (dim + vdim), rank)
+        self.sink = iron.param(heads) if sink else None
+        self.out = Linear(heads * vdim, width, precision=precision)
+
+    def states(self, slots: int) -> dict:
+        # A portion's own rows are in the ring before they are attended: room for them beside the window.
+        ring = min(self.context, self.window + self.portion)
+        held = {"latents": iron.state((slots, ring, self.rank), self.dtype)}
+        if self.rot:
+            held["shared_keys"] = iron.state((slots, ring, self.rot), self.dtype)
+        return held
+
+    def keys(self, slots: int) -> int:
+        """Keys a portion can attend here."""
+        return min(self.room, slots * self.context, self.portion + slots * (self.window - 1))
+
+    def body(self, x, call, state):
+        beside = {"shared_keys": state.get("shared_keys"), "angles": self.angles}
+        q = LatentRows.step(x, self.q_norm, self.c_norm, call.spans, state["latents"], epsilon=self.eps, dtype=self.dtype, **beside)[-1]
+        q = as_rows(self.query(q), x.shape[0])
+        y = LatentMHA.step(q, state["latents"], self.up, call.spans, heads=self.heads, scale=self.scale, window=self.window,
+                           cap=self.keys(call.spans.shape[0]) if call.prompt else 0, single=not call.prompt, sink=self.sink,
+                           dtype=self.dtype, **beside)
+        return self.out(y)
+
+
+class PolyNormMLP(iron.Graph):
+    """A feed-forward of two biased projections around ``PolyNorm``.  ``proj`` is one packed projection (up and the
+    layer's gate); the down projection's bias, ``out_bias``, is added where its product joins the stream."""
+
+    def __init__(self, width, *, inner, gate, eps, dtype, precision):
+        self.own, self.eps, self.dtype = inner, eps, dtype
+        self.proj = Linear(width, inner + gate, precision=precision)
+        self.bias = iron.param(inner)
+        self.act = iron.param(4)
+        self.out = Linear(inner, width, precision=precision)
+        self.out_bias = iron.param(width)
+
+    def body(self, x):
+        return self.out(PolyNorm.step(x, self.act, bias=self.bias, cols=self.own, epsilon=self.eps, dtype=self.dtype))
+
+
+class GatedStreamLayer(iron.Graph):
+    """A pre-norm layer around a float32 stream: the mixer, then the feed-forward (if any), each joining the
+    stream element by element through a sigmoid gate of what it was given."""
+
+    def __init__(self, width, mixer, mlp, *, eps, dtype):
+        self.dtype = dtype
+        self.norm1, self.gate1_bias, self.mixer, self.mlp = StreamRMSNorm(width, eps, dtype), iron.param(width), mixer, mlp
+        if mlp is not None:
+            self.norm2, self.gate2_bias = StreamRMSNorm(width, eps, dtype), iron.param(width)
+        self.rope = None
+
+    def add(self, x, y, packed, block, bias):
+        return StreamGatedAdd.step(x, as_rows(y, x.shape[0]), packed, bias, gate_at=block.own, dtype=self.dtype,
+                                   y_bias=getattr(block, "out_bias", None))
+
+    def body(self, x, call, state):
+        packed = as_rows(self.mixer.proj(self.norm1(x)), x.shape[0])
+        x = self.add(x, self.mixer(packed, call, state), packed, self.mixer, self.gate1_bias)
+        if self.mlp is not None:
+            packed = as_rows(self.mlp.proj(self.norm2(x)), x.shape[0])
+            x = self.add(x, self.mlp(packed), packed, self.mlp, self.gate2_bias)
         return x

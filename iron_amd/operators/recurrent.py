@@ -142,6 +142,50 @@ class TimeMix(_Spanned):
         return Built("iron_time_mix", launch)
 
 
+class MinGRU(_Spanned):
+    """Per channel ``S <- (1 - z) S + z c; y = S silu(g)`` with ``z = sigmoid(zx + z_bias)`` and the candidate c,
+    of ``u = ux + x_bias``, ``u + 1/2`` from 0 up and ``sigmoid(u)`` below; rows ``[zx | ux | g | ..]``."""
+
+    slots: int = param()
+    rows: int = param()
+    stride: int = param()
+    width: int = param()
+    dtype: Any = param(default=bfloat16, repr=False)
+    x = In(rows, stride, dtype=dtype)
+    z_bias = In(width)
+    x_bias = In(width)
+    state = InOut(slots, width, dtype=F32)
+    spans = In(slots, 4, dtype=np.int32)
+    y = Out(rows, width, dtype=dtype)
+    chunked: bool = param(default=lambda op: op.rows > op.CHUNKED_ROWS * op.slots, array=True, repr=False)
+    workspace_words: int = param(derive=lambda op: op._workspace_words(), repr=False)
+    workspace = Scratch(workspace_words, dtype=np.float32, when=chunked)
+    valid = per_call(bounds=rows)
+
+    def _workspace_words(self) -> int:
+        from .._lib import lib
+
+        return int(lib().iron_min_gru_workspace_bytes(self.slots, self.rows, self.width)) // 4
+
+    @classmethod
+    def infer(cls, shapes, **kw):
+        return dict(slots=shapes["spans"][0], rows=shapes["x"][0], stride=shapes["x"][1], width=shapes["z_bias"][0], **kw)
+
+    def validate(self):
+        if 3 * self.width > self.stride:
+            raise ValueError(f"MinGRU: a row of {self.stride} holds no three projections of {self.width}")
+
+    def build(self) -> Built:
+        from .. import kernels
+
+        kw = dict(slots=self.slots, rows=self.rows, stride=self.stride, width=self.width)
+
+        def launch(t, words):
+            kernels.min_gru(t["x"], t["z_bias"], t["x_bias"], t["state"], t["spans"], t["y"], workspace=t.get("workspace"), **kw)
+
+        return Built("iron_min_gru", launch)
+
+
 class _DeltaShape(_Spanned):
     """Sizes of a gated delta rule: ``kv_heads`` q/k heads of ``dim``, ``heads`` value heads of ``vdim``;
     the rows between its two steps are ``[unit q | unit k | v | log decay | beta]`` in float32."""

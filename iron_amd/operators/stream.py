@@ -1,5 +1,5 @@
 """The float32 residual stream of a decoder: rows into it, norms out of it, blocks' outputs added to it,
-and the head's soft cap.  ``dtype`` is what the rows that leave the stream are rounded to: bf16, or
+and the head's scale and soft cap.  ``dtype`` is what the rows that leave the stream are rounded to: bf16, or
 float32 in a model that runs in 32 bits throughout.  The stream is updated in place.
 """
 
@@ -108,6 +108,85 @@ class StreamAdd(Operator):
         return Built("iron_stream_rows", launch)
 
 
+class StreamGatedAdd(Operator):
+    """``x += (y + y_bias) * sigmoid(gate + gate_bias)`` in float32: a block's output joins the stream through
+    a gate, columns ``gate_at ..`` of a projection's row."""
+
+    rows: int = param()
+    cols: int = param()
+    gate_width: int = param()
+    gate_at: int = param(default=0, array=True)
+    biased: bool = param(default=False, repr=False)
+    dtype: Any = param(default=bfloat16, repr=False)
+    x = InOut(rows, cols, dtype=F32)
+    y = In(rows, cols, dtype=dtype)
+    gate = In(rows, gate_width, dtype=dtype)
+    gate_bias = In(cols)
+    y_bias = In(cols, when=biased)
+    valid = per_call(bounds=rows)
+
+    @classmethod
+    def infer(cls, shapes, **kw):
+        return dict(rows=shapes["x"][0], cols=shapes["x"][1], gate_width=shapes["gate"][1], biased="y_bias" in shapes, **kw)
+
+    def validate(self):
+        if not 0 <= self.gate_at <= self.gate_width - self.cols:
+            raise ValueError(f"StreamGatedAdd: columns {self.gate_at} .. + {self.cols} of a row of {self.gate_width}")
+
+    def tolerance(self):
+        return Tolerance.relative(1e-4, 1e-4, note="float32")
+
+    def build(self) -> Built:
+        from .. import kernels
+
+        kw = dict(rows=self.rows, cols=self.cols, gate_stride=self.gate_width, gate_at=self.gate_at)
+
+        def launch(t, words):
+            kernels.stream_gated_rows(t["x"], t["y"], t["gate"], t["gate_bias"], y_bias=t.get("y_bias"), valid=words.get("valid"), **kw)
+
+        return Built("iron_stream_gated_rows", launch)
+
+
+class PolyNorm(Operator):
+    """``a N(z) + b N(z^2) + c N(z^3) + e``: an activation over the normed powers of a row, ``z`` columns
+    ``at ..`` of a projection's row plus a bias, N a row over its root mean square; ``coefficients`` a, b, c, e."""
+
+    rows: int = param()
+    cols: int = param()
+    stride: int = param()
+    at: int = param(default=0, array=True)
+    epsilon: float = param(array=True)
+    biased: bool = param(default=False, repr=False)
+    dtype: Any = param(default=bfloat16, repr=False)
+    x = In(rows, stride, dtype=dtype)
+    coefficients = In(4)
+    bias = In(cols, when=biased)
+    y = Out(rows, cols, dtype=dtype)
+    valid = per_call(bounds=rows)
+
+    @classmethod
+    def infer(cls, shapes, **kw):
+        given = {"cols": shapes["x"][1]} | ({"cols": shapes["bias"][0]} if "bias" in shapes else {})
+        return {"rows": shapes["x"][0], "stride": shapes["x"][1], "biased": "bias" in shapes, **given, **kw}
+
+    def validate(self):
+        if not 0 <= self.at <= self.stride - self.cols:
+            raise ValueError(f"PolyNorm: columns {self.at} .. + {self.cols} of a row of {self.stride}")
+
+    def tolerance(self):
+        return Tolerance.relative(1e-2, 1e-2, note="float32, rounded once")
+
+    def build(self) -> Built:
+        from .. import kernels
+
+        kw = dict(rows=self.rows, cols=self.cols, stride=self.stride, at=self.at, eps=float(self.epsilon))
+
+        def launch(t, words):
+            kernels.poly_norm(t["x"], t["coefficients"], t["y"], bias=t.get("bias"), valid=words.get("valid"), **kw)
+
+        return Built("iron_poly_norm", launch)
+
+
 class SpanTails(Operator):
     """The stream's row of every slot's last token: what a prompt's portion hands its head."""
 
@@ -140,12 +219,13 @@ class SpanTails(Operator):
 
 
 class Softcap(Operator):
-    """``cap * tanh(x / cap)`` of the head's rows (``cap`` 0: as they are), as float32 and, in rows padded to
-    whole 16-byte pieces, as the bf16 the draw ranks."""
+    """``cap * tanh(scale * x / cap)`` of the head's rows (``cap`` 0: ``scale * x``), as float32 and, in rows
+    padded to whole 16-byte pieces, as the bf16 the draw ranks."""
 
     rows: int = param()
     cols: int = param()
     cap: float = param(default=0.0, array=True)
+    scale: float = param(default=1.0, array=True)
     dtype: Any = param(default=bfloat16, repr=False)
     stride: int = param(derive=lambda op: -(-op.cols // 8) * 8, repr=False)
     x = In(rows, cols, dtype=dtype)
@@ -162,10 +242,10 @@ class Softcap(Operator):
     def build(self) -> Built:
         from .. import kernels
 
-        rows, cols, stride, cap = self.rows, self.cols, self.stride, float(self.cap)
+        rows, cols, stride, cap, scale = self.rows, self.cols, self.stride, float(self.cap), float(self.scale)
 
         def launch(t, words):
-            kernels.softcap(t["x"], t["y"], t["rounded"], rows=rows, cols=cols, stride=stride, cap=cap)
+            kernels.softcap(t["x"], t["y"], t["rounded"], rows=rows, cols=cols, stride=stride, cap=cap, scale=scale)
 
         return Built("iron_softcap", launch)
 

@@ -176,6 +176,82 @@ def stream_add(op, x, y, weight):
     return np.asarray(x + _unit_rms(y, op.epsilon) * np.asarray(weight, np.float64), np.float32)
 
 
+def _sigmoid(z):
+    return 1 / (1 + np.exp(-np.asarray(z, np.float64)))
+
+
+def stream_gated_add(op, x, y, gate, gate_bias, *, y_bias=None):
+    y = np.asarray(y, np.float64) + (0 if y_bias is None else y_bias)
+    z = np.asarray(gate, np.float64)[:, op.gate_at : op.gate_at + op.cols] + gate_bias
+    return np.asarray(x + y * _sigmoid(z), np.float32)
+
+
+def poly_norm(op, x, coefficients, *, bias=None):
+    z = np.asarray(x, np.float64)[:, op.at : op.at + op.cols] + (0 if bias is None else bias)
+    a, b, c, e = np.asarray(coefficients, np.float64)
+    return _out(op, a * _unit_rms(z, op.epsilon) + b * _unit_rms(z**2, op.epsilon) + c * _unit_rms(z**3, op.epsilon) + e)
+
+
+def min_gru(op, x, z_bias, x_bias, state, spans):
+    W, state, y = op.width, np.array(state), np.zeros((op.rows, op.width), np.float32)
+    x = np.asarray(x, np.float64)
+    z, u, g = _sigmoid(x[:, :W] + z_bias), x[:, W : 2 * W] + x_bias, x[:, 2 * W : 3 * W]
+    c = np.where(u >= 0, u + 0.5, _sigmoid(u))
+    for s, row, n, start in _spans(spans):
+        S = np.asarray(state[s], np.float64) if start else np.zeros(W)
+        for t in range(row, row + n):
+            S = (1 - z[t]) * S + z[t] * c[t]
+            y[t] = S * g[t] * _sigmoid(g[t])
+        state[s] = S
+    return state, _out(op, y)
+
+
+def _turn(x, angles, turned):
+    """The first ``turned`` of x's trailing columns turned, pair by pair, by rows of (cos, sin)."""
+    x = np.array(x, np.float64)
+    c, s = np.asarray(angles, np.float64)[..., 0::2], np.asarray(angles, np.float64)[..., 1::2]
+    u, v = x[..., 0:turned:2].copy(), x[..., 1:turned:2].copy()
+    x[..., 0:turned:2], x[..., 1:turned:2] = u * c - v * s, v * c + u * s
+    return x
+
+
+def latent_rows(op, x, q_gain, c_gain, spans, latents, *, shared_keys=None, angles=None):
+    x, latents, q = np.asarray(x, np.float64), np.array(latents), np.zeros((op.rows, op.q_rank), np.float32)
+    keys = None if shared_keys is None else np.array(shared_keys)
+    for s, row, n, start in _spans(spans):
+        own, at = x[row : row + n], np.arange(start, start + n)
+        q[row : row + n] = _unit_rms(own[:, : op.q_rank], op.epsilon) * q_gain
+        latents[s, at % op.ring] = _out(op, _unit_rms(own[:, op.q_rank : op.q_rank + op.rank], op.epsilon) * c_gain)
+        if keys is not None:
+            rest = own[:, op.q_rank + op.rank : op.q_rank + op.rank + op.rot]
+            keys[s, at % op.ring] = _out(op, rest if angles is None else _turn(rest, angles[at], op.turned))
+    return (latents, _out(op, q)) if keys is None else (latents, keys, _out(op, q))
+
+
+def latent_mha(op, q, latents, up, spans, *, shared_keys=None, angles=None, sink=None):
+    H, D, V, R = op.heads, op.dim, op.vdim, op.rank
+    y = np.zeros((op.rows, H, V), np.float32)
+    q, up = np.asarray(q, np.float64).reshape(op.rows, H, D + op.rot), np.asarray(up, np.float64)
+    for s, row, n, start in _spans(spans):
+        first = max(0, start - op.window + 1)
+        at = np.arange(first, start + n) % op.ring
+        c = np.asarray(latents[s, at], np.float64)
+        k, v = (c @ up[: H * D].T).reshape(-1, H, D), (c @ up[H * D :].T).reshape(-1, H, V)
+        for i in range(n):
+            lo, hi, query = max(0, start + i - op.window + 1) - first, start + i + 1 - first, q[row + i]
+            if op.turned:
+                query = np.concatenate([query[:, :D], _turn(query[:, D:], angles[start + i], op.turned)], axis=1)
+            score = np.einsum("jhd,hd->hj", k[lo:hi], query[:, :D])
+            if shared_keys is not None:
+                score = score + query[:, D:] @ np.asarray(shared_keys[s, at[lo:hi]], np.float64).T
+            score = score * op.scale
+            top = score.max(1) if sink is None else np.maximum(score.max(1), sink)
+            p = np.exp(score - top[:, None])
+            total = p.sum(1) + (0 if sink is None else np.exp(sink - top))
+            y[row + i] = np.einsum("hj,jhv->hv", p / total[:, None], v[lo:hi])
+    return _out(op, y.reshape(op.rows, -1))
+
+
 def span_tails(op, x, spans):
     y = np.zeros((op.slots, op.cols), np.float32)
     for s, row, n, _ in _spans(spans):
@@ -185,6 +261,7 @@ def span_tails(op, x, spans):
 
 def softcap(op, x):
     y = np.asarray(x, np.float64)
+    y = y * op.scale
     y = np.asarray(op.cap * np.tanh(y / op.cap) if op.cap else y, np.float32)
     rounded = np.zeros((op.rows, op.stride), np.float32)
     rounded[:, : op.cols] = round_bf16(y)
@@ -320,7 +397,8 @@ def install() -> None:
         Softmax=softmax, StreamEmbed=stream_embed, StreamNorm=stream_norm, StreamAdd=stream_add, SpanTails=span_tails,
         Softcap=softcap, GatedProduct=gated_product, LinearAny=linear_any, TokenShift=token_shift, LowRankDecay=low_rank_decay,
         TimeMix=time_mix, ShortConv=short_conv, DeltaRule=delta_rule, HeadGate=head_gate, WindowMHA=window_mha,
-        SampleSlots=sample_slots,
+        SampleSlots=sample_slots, StreamGatedAdd=stream_gated_add, PolyNorm=poly_norm, MinGRU=min_gru, LatentRows=latent_rows,
+        LatentMHA=latent_mha,
         # The host's draw, for iron_amd.lm.generation.Sampler's checks.
         sample_ref=ops.sample_ref, sample_weights=ops.sample_weights,
     )
