@@ -273,42 +273,38 @@ __device__ __forceinline__ void latent_prefill_body(const bf16_t* __restrict__ q
     for (int d = 0; d < VD; ++d) acc[n][d] = f32x4{0.f, 0.f, 0.f, 0.f};
   }
 
-  // The next tile on its way from memory, by 32-bit offsets into the tile's own bounded buffers: what lies past
-  // the last key reads as zeros.  A key's pieces past its head's width read other columns, against zeros of q.
+  // The next tile on its way from memory.  A row past the last key reads the last again (its scores are masked),
+  // and a key's pieces past its head's width other columns, against zeros of q: no load is behind a branch.
   u32x4 kn[KP], vn[VT][4];
-  int k_at[KP], v_at[VT];
+  int k_row[KP], k_col[KP], v_row[VT], v_col[VT];
   bool k_shared[KP];
 #pragma unroll
   for (int i = 0; i < KP; ++i) {
-    const int e = t + 256 * i, row = e / (DKP / 8), c = (e % (DKP / 8)) * 8;
+    const int e = t + 256 * i, c = (e % (DKP / 8)) * 8;
+    k_row[i] = e / (DKP / 8);
     k_shared[i] = c >= a.dim && c < wide;
-    k_at[i] = k_shared[i] ? row * 65536 + (c - a.dim) * 2 : (row * width + head * a.dim + (c < a.dim ? c : 0)) * 2;
+    k_col[i] = k_shared[i] ? c - a.dim : head * a.dim + (c < a.dim ? c : 0);
   }
 #pragma unroll
   for (int i = 0; i < VT; ++i) {
-    const int e = t + 256 * i, row = (e / (DVP / 8) * 4) % LATENT_KEYS, c = min((e % (DVP / 8)) * 8, a.vdim - 8);
-    v_at[i] = (row * width + a.heads * a.dim + head * a.vdim + c) * 2;
+    const int e = t + 256 * i;
+    v_row[i] = (e / (DVP / 8) * 4) % LATENT_KEYS;
+    v_col[i] = a.heads * a.dim + head * a.vdim + min((e % (DVP / 8)) * 8, a.vdim - 8);
   }
-  const bf16_t* ring = shared_keys + (size_t)slot * a.ring * a.rot;
-  const __amdgpu_buffer_rsrc_t ring_b = bounded_bytes(ring, a.ring * a.rot * 2);
+  const bf16_t* ring = a.rot > 0 ? shared_keys + (size_t)slot * a.ring * a.rot : kv;
   auto fetch = [&](int base) {
-    const int left = min(LATENT_KEYS, end - base);
-    const __amdgpu_buffer_rsrc_t b = bounded_bytes(kv + (size_t)(run.row0 + base - run.first) * width, left * width * 2);
-    const int wrap = base % a.ring;
+    const int last = end - 1 - base, wrap = base % a.ring;
+    const bf16_t* rows = kv + (size_t)(run.row0 + base - run.first) * width;
 #pragma unroll
     for (int i = 0; i < KP; ++i) {
-      if (k_shared[i]) {
-        int at = wrap + (k_at[i] >> 16);
-        at -= at >= a.ring ? a.ring : 0;
-        kn[i] = __builtin_amdgcn_raw_buffer_load_b128(ring_b, at * a.rot * 2 + (k_at[i] & 65535), 0, 0);
-      } else {
-        kn[i] = __builtin_amdgcn_raw_buffer_load_b128(b, k_at[i], 0, 0);
-      }
+      const int row = min(k_row[i], last), at = wrap + row - (wrap + row >= a.ring ? a.ring : 0);
+      const bf16_t* from_row = k_shared[i] ? ring + (size_t)(at * a.rot) : rows + (size_t)(row * width);
+      kn[i] = *reinterpret_cast<const u32x4*>(from_row + k_col[i]);
     }
 #pragma unroll
     for (int i = 0; i < VT; ++i)
 #pragma unroll
-      for (int j = 0; j < 4; ++j) vn[i][j] = __builtin_amdgcn_raw_buffer_load_b128(b, v_at[i], j * width * 2, 0);
+      for (int j = 0; j < 4; ++j) vn[i][j] = *reinterpret_cast<const u32x4*>(rows + (size_t)(min(v_row[i] + j, last) * width) + v_col[i]);
   };
   fetch(from);
   const float scale = a.scale * LATENT_LOG2E;
@@ -350,21 +346,24 @@ __device__ __forceinline__ void latent_prefill_body(const bf16_t* __restrict__ q
         for (int d = 0; d < KD; ++d) sc[u][kt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[d], qf[u][d], sc[u][kt], 0, 0, 0);
       }
     }
-    // A tile all of whose keys all of the block's queries see needs no mask.
+    // A tile all of whose keys all of the block's queries see needs no mask.  (One branch around selects: a branch
+    // a score, right behind the products, has read scores of a tile that was not done.)
     const bool edge = base + LATENT_KEYS - 1 > first_pos || first_pos + BQ - 1 - base >= a.window;
     bf16x8 pf[QT][2];
 #pragma unroll
     for (int u = 0; u < QT; ++u) {
-      const int ahead = first_pos + wave * QT * 16 + u * 16 + lo16 - base - quad * 4;   // i - j of the lane's first key
+#pragma unroll
+      for (int kt = 0; kt < 4; ++kt) sc[u][kt] *= scale;
+      if (edge) {
+        const int ahead = first_pos + wave * QT * 16 + u * 16 + lo16 - base - quad * 4;   // i - j of the lane's first key
+#pragma unroll
+        for (int kt = 0; kt < 4; ++kt)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) sc[u][kt][r] = (unsigned)(ahead - kt * 16 - r) < (unsigned)a.window ? sc[u][kt][r] : -INFINITY;
+      }
       float top = -INFINITY;
 #pragma unroll
-      for (int kt = 0; kt < 4; ++kt)
-#pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          sc[u][kt][r] *= scale;
-          if (edge && (unsigned)(ahead - kt * 16 - r) >= (unsigned)a.window) sc[u][kt][r] = -INFINITY;
-          top = fmaxf(top, sc[u][kt][r]);
-        }
+      for (int kt = 0; kt < 4; ++kt) top = fmaxf(top, fmaxf(fmaxf(sc[u][kt][0], sc[u][kt][1]), fmaxf(sc[u][kt][2], sc[u][kt][3])));
       // The reference the exponents are taken from moves only where a score would exceed it by more than 2^8:
       // it cancels in the quotient, and the products need no rescaling between.
       if (__builtin_amdgcn_ballot_w64(top > m[u] + 8.f) != 0) {
