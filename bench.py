@@ -696,11 +696,24 @@ def time_served(torch, run_prompt, decode, steps, prompts, repeats=5):
     return out
 
 
-def pegilix_served(torch, config, weights, steps, prompts):
-    from iron_amd.applications.pegilix import Pegilix
+def pegilix_state_bytes(config) -> int:
+    """Bytes of states a decode step reads and writes a slot, behind a full window."""
+    state = 0
+    for i in config.order:
+        m = config.layers[i]["mixer"]
+        if config.layers[i]["type"] == "parallel":
+            left, right = m["left"], m["right"]
+            state += PEGILIX_WINDOW * left["kv_heads"] * (left["dim"] + left["vdim"]) * 2 + 8 * right["heads"] * right["dim"] ** 2
+        else:
+            state += 8 * m["heads"] * m["dim"] * m["vdim"]
+    return state
+
+
+def batched_served(torch, model_class, config, weights, steps, prompts, state_bytes):
+    """A batched model's prompts and replayed decode steps, every slot busy."""
     from iron_amd.lm.batched import Entry
 
-    model = Pegilix(config, weights)
+    model = model_class(config, weights)
     model.load_versions()
     rng = np.random.default_rng(512)
     tokens = [rng.integers(0, config.vocab_size, max(prompts)) for _ in range(config.slots)]
@@ -716,16 +729,8 @@ def pegilix_served(torch, config, weights, steps, prompts):
     first["launches_per_step"] = model.decode_step.launches_per_replay
     first["launches_per_portion"] = model.prompt_chunk.launches_per_call
     weight_bytes = 2 * sum(int(np.prod(t.shape)) for n, t in weights.items() if n != "embed")
-    c, state = config, 0
-    for i in c.order:
-        m = c.layers[i]["mixer"]
-        if c.layers[i]["type"] == "parallel":
-            left, right = m["left"], m["right"]
-            state += PEGILIX_WINDOW * left["kv_heads"] * (left["dim"] + left["vdim"]) * 2 + 8 * right["heads"] * right["dim"] ** 2
-        else:
-            state += 8 * m["heads"] * m["dim"] * m["vdim"]
-    bytes_step = weight_bytes + c.slots * state
-    first |= {"decode_tok_s": round(1e3 * c.slots / first["decode_ms"], 1), "decode_GBps": round(bytes_step / first["decode_ms"] / 1e6, 1),
+    bytes_step = weight_bytes + config.slots * state_bytes
+    first |= {"decode_tok_s": round(1e3 * config.slots / first["decode_ms"], 1), "decode_GBps": round(bytes_step / first["decode_ms"] / 1e6, 1),
               "frac_hbm": round(bytes_step / first["decode_ms"] / 1e6 / HBM_PEAK_GBS, 4), "bytes_per_step": int(bytes_step)}
     model.release()
     return first
@@ -751,16 +756,18 @@ def bench_pegilix(torch, dev, steps, widths, batch=8, prompts=(512, 2048)):
 
     from iron_amd.applications.llama import LLAMA_3_2_1B, Llama
     from iron_amd.applications.llama import shapes as llama_shapes
-    from iron_amd.applications.pegilix import shapes
+    from iron_amd.applications.pegilix import Pegilix, shapes
 
     rows = []
     for width in widths:
         H, G, D, F, layers, vocab = PEGILIX_SIZES[width]
         config = pegilix_config(width)
         weights = random_weights(torch, shapes(config, bias_rows=32, rank=64), dev)
-        row = {"width": width, "layers": layers, "pegilix": pegilix_served(torch, config, weights, steps, prompts)}
+        row = {"width": width, "layers": layers, "pegilix": batched_served(torch, Pegilix, config, weights, steps, prompts,
+                                                                                 pegilix_state_bytes(config))}
         if batch:
-            row[f"pegilix_batch_{batch}"] = pegilix_served(torch, dataclasses.replace(config, slots=batch), weights, steps, (512,))
+            row[f"pegilix_batch_{batch}"] = batched_served(torch, Pegilix, dataclasses.replace(config, slots=batch), weights, steps, (512,),
+                                                            pegilix_state_bytes(config))
         params = sum(int(np.prod(t.shape)) for t in weights.values())
         del weights
         torch.cuda.empty_cache()
@@ -791,6 +798,69 @@ def bench_pegilix(torch, dev, steps, widths, batch=8, prompts=(512, 2048)):
         print(json.dumps(row), file=sys.stderr, flush=True)
     return {"what": f"prompt (ms, tok/s) and greedy decode steps as HIP-graph replays; Pegilix window {PEGILIX_WINDOW}, "
                     "decode behind the longest prompt; frac_hbm: weights, window and states over the time a step takes",
+            "data": "synthetic", "dtype": "bf16", "sizes": rows}
+
+
+# The latent attention of PUFUZEN layers at PEGILIX_SIZES' widths: (query latent, latent, rotated part)
+PUFUZEN_LATENTS = {2048: (1536, 512, 64), 3072: (1536, 512, 64), 4096: (1536, 512, 64)}
+
+
+def pufuzen_config(width, slots=1, chunk=2048):
+    """A Pufuzen of ``width``'s sizes: two recurrent layers, then windowed and causal latent attention, each with a
+    feed-forward; heads of 128."""
+    from iron_amd.applications.pufuzen import PufuzenConfig
+
+    _, _, _, F, layers, vocab = PEGILIX_SIZES[width]
+    q_rank, rank, rot = PUFUZEN_LATENTS[width]
+    mlp, heads = {"ff": F, "kind": "dense"}, width // 128
+    shared = {"heads": heads, "dim": 128, "vdim": 128, "q_rank": q_rank, "kv_rank": rank}
+    recurrent = {"type": "mingru", "mixer": {"width": width}, "mlp": None}
+    windowed = {"type": "latent_attention", "mlp": mlp, "mixer": {**shared, "scale": 128**-0.5, "mask": {"size": PEGILIX_WINDOW}}}
+    causal = {"type": "latent_attention_2", "mlp": mlp, "mixer": {**shared, "rot_dim": rot, "rot": {"base": 10000.0, "dims": rot},
+                                                                   "scale": (128 + rot) ** -0.5}}
+    return PufuzenConfig(vocab_size=vocab, hidden_size=width, layers=tuple([recurrent, recurrent, windowed, causal] * (layers // 4)),
+                         eps=1e-5, logit_scale=1.0, max_seq_len=4096, prefill_chunk=chunk, slots=slots)
+
+
+def pufuzen_state_bytes(config, keys) -> int:
+    """Bytes of states and latents a decode step behind ``keys`` tokens reads and writes a slot."""
+    state = 0
+    for spec in config.layers:
+        m = spec["mixer"]
+        if spec["type"] == "mingru":
+            state += 8 * m["width"]
+        else:
+            state += min(keys, m["mask"]["size"] if "mask" in m else keys) * (m["kv_rank"] + m.get("rot_dim", 0)) * 2
+    return state
+
+
+def bench_pufuzen(torch, dev, steps, widths, batch=8, prompts=(512, 2048)):
+    """Prompt and decode throughput of Pufuzen layers at a few widths, one sequence and a batch of ``batch``, beside
+    a Pegilix of the same width, feed-forward, layers and vocabulary; random weights, bf16."""
+    import dataclasses
+
+    from iron_amd.applications import pegilix, pufuzen
+
+    rows = []
+    for width in widths:
+        row = {"width": width, "layers": PEGILIX_SIZES[width][4]}
+        for name, module, cls, config, kw in (("pufuzen", pufuzen, pufuzen.Pufuzen, pufuzen_config(width), {}),
+                                              ("pegilix", pegilix, pegilix.Pegilix, pegilix_config(width), dict(bias_rows=32, rank=64))):
+            weights = random_weights(torch, module.shapes(config, **kw), dev)
+            row[f"{name}_params"] = sum(int(np.prod(t.shape)) for t in weights.values())
+
+            def state(keys, config=config, name=name):
+                return pufuzen_state_bytes(config, keys) if name == "pufuzen" else pegilix_state_bytes(config)
+
+            row[name] = batched_served(torch, cls, config, weights, steps, prompts, state(max(prompts)))
+            if batch:
+                row[f"{name}_batch_{batch}"] = batched_served(torch, cls, dataclasses.replace(config, slots=batch), weights, steps, (512,), state(512))
+            del weights
+            torch.cuda.empty_cache()
+        rows.append(row)
+        print(json.dumps(row), file=sys.stderr, flush=True)
+    return {"what": f"prompt (ms, tok/s) and greedy decode steps as HIP-graph replays; windows of {PEGILIX_WINDOW}, decode behind the longest "
+                    "prompt; frac_hbm: weights, states and keys over the time a step takes",
             "data": "synthetic", "dtype": "bf16", "sizes": rows}
 
 
@@ -911,9 +981,11 @@ def main():
                          "(for a rocprofv3 --pmc or --kernel-trace run) and exit")
     ap.add_argument("--pegilix", action="store_true",
                     help="time only Pegilix layers at a few widths beside a Llama of equal size, and exit")
+    ap.add_argument("--pufuzen", action="store_true",
+                    help="time only Pufuzen layers at a few widths beside a Pegilix of equal size, and exit")
     ap.add_argument("--widths", type=int, nargs="+", default=sorted(PEGILIX_SIZES), choices=sorted(PEGILIX_SIZES),
-                    help="the widths --pegilix times")
-    ap.add_argument("--batch", type=int, default=8, help="sequences of --pegilix's batch (0: one sequence only)")
+                    help="the widths --pegilix and --pufuzen time")
+    ap.add_argument("--batch", type=int, default=8, help="sequences of --pegilix's and --pufuzen's batch (0: one sequence only)")
     args = ap.parse_args()
     if args.gpus != 1:
         print("bench.py: this build is a one-GPU hot path; --gpus must be 1 "
@@ -946,6 +1018,9 @@ def main():
         return 0
     if args.pegilix:
         print(json.dumps(bench_pegilix(torch, dev, args.steps, args.widths, args.batch)))
+        return 0
+    if args.pufuzen:
+        print(json.dumps(bench_pufuzen(torch, dev, args.steps, args.widths, args.batch)))
         return 0
     if args.prompt_probe:
         prompt_probe(torch, dev)

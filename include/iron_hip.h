@@ -458,7 +458,8 @@ int iron_mha_window(const void* x, void* keys, void* values, const float* bias, 
                     int rows, int stride, int heads, int kv_heads, int dim, int vdim, int window, int ring, float scale,
                     int out_stride, int out_at, float out_scale, int single, int is_float, void* stream);
 /* x (rows, stride) = [zx | ux | gx | ..] of `width` columns each.  Per channel z = sigmoid(zx + z_bias), u = ux + x_bias,
- * c = u + 1/2 where u >= 0, else sigmoid(u); S <- (1 - z) S + z c; y = S silu(gx), y (rows, width).  state (slots, width).
+ * c = u + 1/2 where u >= 0, else sigmoid(u); S <- (1 - z) S + z c; y = S silu(gx), y (rows, width).  state (slots, 2, width): the
+ * state behind position p in row p % 2.
  * With a workspace (the bytes given, any contents, 16-byte aligned) chunks of a portion run side by side; without, a
  * span's rows one after the other. */
 int64_t iron_min_gru_workspace_bytes(int slots, int rows, int width);
@@ -504,6 +505,21 @@ int iron_decode_delta_bf16(const uint16_t* x, const uint16_t* taps_w, const uint
                            const uint16_t* norm, uint16_t* inputs, float* state, const int* spans, uint16_t* out,
                            int slots, int rows, int stride, int heads, int kv_heads, int dim, int vdim, int taps,
                            int gate_at, int b_at, int a_at, float eps, void* stream);
+/* One row's product with its input made and its output taken in the same launch, bf16; each computes what the entry
+ * points above and iron_gemv_bf16 compute in turn.
+ * stream_product: input 0 the bf16 row x (K); 1 the float row x, 2 the bf16 row x, RMS-normed with gain; 3 slot 0's
+ * iron_min_gru over the row x = [zx | ux | gx] (width K, biases b0 and b1); 4 iron_poly_norm (bias b0, coefficients
+ * gain).  Output: the row y (M), inputs 0 to 2; or iron_stream_gated_rows on stream_row (M), inputs 0, 3 and 4.
+ * latent_query: iron_latent_rows of slot 0's one row x (whole 16-byte pieces), and q = W (M, q_rank) times the
+ * query's latent. */
+int iron_stream_product_bf16(int input, const void* x, const uint16_t* gain, const uint16_t* b0, const uint16_t* b1,
+                             float* state, const int* spans, float eps, const uint16_t* W, int M, int K, uint16_t* y,
+                             float* stream_row, const uint16_t* y_bias, const uint16_t* gate, const uint16_t* gate_bias,
+                             void* stream);
+int iron_latent_query_bf16(const uint16_t* x, const uint16_t* q_gain, const uint16_t* c_gain, const float* angles,
+                           const int* spans, const uint16_t* W, uint16_t* q, uint16_t* latents, uint16_t* shared_keys,
+                           int M, int stride, int q_rank, int rank, int rot, int turned, int angle_rows, int ring,
+                           float eps, void* stream);
 /* iron_sample_bf16 for every slot that has rows: logits (slots, logits_stride), drawn at the position p
  * of the span's last row by draw row slot * steps + p, recorded in record[slot * steps + p]; the span
  * then becomes {slot, 1, p + 1}.  workspace: slots times iron_sample_workspace_bytes(n). */

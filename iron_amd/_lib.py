@@ -120,6 +120,8 @@ SIGNATURES = {
         + [c_int] * 3 + [_P],
     ),
     "iron_decode_delta_bf16": (c_int, [_P] * 9 + [c_int] * 11 + [c_float, _P]),
+    "iron_stream_product_bf16": (c_int, [c_int] + [_P] * 6 + [c_float, _P, c_int, c_int] + [_P] * 6),
+    "iron_latent_query_bf16": (c_int, [_P] * 9 + [c_int] * 8 + [c_float, _P]),
     "iron_sample_slots_bf16": (c_int, [_P, c_int, c_int, _P, c_int, c_int, c_int, _P, c_int, _P, _P, _P, _P]),
     "iron_eval_words": (c_int, [_P, c_int, _P, c_int, _P]),
 }

@@ -30,10 +30,14 @@ in a batched decoder's decode step (bf16; a float32 stream, layers with a state)
   LowRankDecay, TimeMix, HeadGate, WindowMHA             => iron_decode_parallel_bf16
   ShortConv, DeltaRule, HeadGate                         => iron_decode_delta_bf16
   GEMV gate, GEMV up, SiLU / GELU (tanh) / ReLU, Mul     => iron_gemv_fused_bf16 (epilogue 2 / 3 / 6)
+  StreamNorm, GEMV (one slot, as the rest here)          => iron_stream_product_bf16 (input 1)
+  [MinGRU / PolyNorm,] GEMV, StreamGatedAdd              => iron_stream_product_bf16 (input 0 / 3 / 4)
+  LatentRows, GEMV (the queries)                         => iron_latent_query_bf16
 
 and in either,
 
   StreamAdd, StreamNorm                                  => iron_stream_rows
+  StreamGatedAdd, StreamNorm                             => iron_stream_gated_rows
   RMSNorm, ElementwiseAdd (a sandwich layer's residual)  => iron_rmsnorm_add_bf16
 
 A run is fused only if every intermediate it hides is read by nothing else.
@@ -280,6 +284,88 @@ def plan(recording, tensor: Callable[[Any], Any], word: Callable[[Any], Any],
         kw = dict(slots=c.slots, rows=c.rows, stride=c.stride, heads=c.heads, kv_heads=c.kv_heads, dim=c.dim, vdim=c.vdim,
                   taps=c.taps, gate_at=gate.op.gate_at, b_at=c.b_at, a_at=c.a_at, eps=float(gate.op.epsilon))
         return Fused("decode_delta", j, 3, lambda a=args, kw=kw: kernels.decode_delta(**a, **kw))
+
+    def bare(s) -> bool:
+        return not s.values and all(_plain(h) for h in (*s.inputs.values(), *s.outputs.values()))
+
+    def gated_end(j, x):
+        """``(product, add)`` where step ``j`` is one row's product of ``x`` and the next adds it, gated, to the
+        stream -- or None."""
+        if j + 1 >= len(steps):
+            return None
+        g, add = steps[j], steps[j + 1]
+        if not (gemv_row(g) and (x is None or _same(g.inputs["B"], x)) and g.op.K % 8 == 0 and g.op.K <= 16384 and _name(add) == "StreamGatedAdd"
+                and add.op.rows == 1 and add.op.dtype is bfloat16 and bare(add) and _same(add.inputs["y"], g.outputs["C"])
+                and once(g.outputs["C"])):
+            return None
+        return g, add
+
+    def into_stream(g, add):
+        at = add.op.gate_at
+        args = dict(W=tensor(g.inputs["A"]), stream=tensor(add.inputs["x"]).reshape(-1),
+                    gate=tensor(add.inputs["gate"]).reshape(-1)[at : at + add.op.cols], gate_bias=tensor(add.inputs["gate_bias"]))
+        if "y_bias" in add.inputs:
+            args["y_bias"] = tensor(add.inputs["y_bias"])
+        return args, dict(M=g.op.M, K=g.op.K)
+
+    def stream_product_at(j):
+        """The launch for a single row's product with what makes its input ahead of it (a norm of the stream, a
+        gated recurrence's step, an activation over normed powers) or what takes its output behind it (the stream,
+        through a gate) -- or None."""
+        s = steps[j]
+        if _name(s) == "StreamNorm":
+            g = steps[j + 1] if j + 1 < len(steps) else None
+            h = s.outputs["y"]
+            if not (g is not None and s.op.rows == 1 and s.op.dtype is bfloat16 and s.op.cols % 8 == 0 and s.op.cols <= 16384 and bare(s)
+                    and gemv_row(g, h) and once(h)):
+                return None
+            args = dict(W=tensor(g.inputs["A"]), x=tensor(s.inputs["x"]).reshape(-1), gain=tensor(s.inputs["weight"]),
+                        y=tensor(g.outputs["C"]).reshape(-1))
+            kw = dict(input="stream_norm", M=g.op.M, K=g.op.K, eps=float(s.op.epsilon))
+            return Fused("stream_norm_gemv", j, 2, lambda a=args, kw=kw: kernels.stream_product(**a, **kw))
+        if _name(s) == "MinGRU":
+            y = s.outputs["y"]
+            end = gated_end(j + 1, y)
+            if not (end and s.op.rows == 1 and s.op.slots == 1 and s.op.dtype is bfloat16 and s.op.width % 8 == 0 and bare(s) and once(y)):
+                return None
+            args, kw = into_stream(*end)
+            args |= dict(x=tensor(s.inputs["x"]).reshape(-1), b0=tensor(s.inputs["z_bias"]), b1=tensor(s.inputs["x_bias"]),
+                         state=tensor(s.inputs["state"]).reshape(-1), spans=tensor(s.inputs["spans"]))
+            kw["input"] = "min_gru"
+            return Fused("min_gru_gated_product", j, 3, lambda a=args, kw=kw: kernels.stream_product(**a, **kw))
+        if _name(s) == "PolyNorm":
+            y = s.outputs["y"]
+            end = gated_end(j + 1, y)
+            if not (end and s.op.rows == 1 and s.op.biased and s.op.dtype is bfloat16 and s.op.cols % 8 == 0 and s.op.at % 8 == 0 and bare(s)
+                    and once(y)):
+                return None
+            args, kw = into_stream(*end)
+            args |= dict(x=tensor(s.inputs["x"]).reshape(-1)[s.op.at : s.op.at + s.op.cols], b0=tensor(s.inputs["bias"]),
+                         gain=tensor(s.inputs["coefficients"]))
+            kw |= dict(input="poly_norm", eps=float(s.op.epsilon))
+            return Fused("poly_norm_gated_product", j, 3, lambda a=args, kw=kw: kernels.stream_product(**a, **kw))
+        if (end := gated_end(j, None)) is not None:
+            args, kw = into_stream(*end)
+            args["x"] = tensor(s.inputs["B"]).reshape(-1)
+            return Fused("gated_product", j, 2, lambda a=args, kw=kw: kernels.stream_product(input="row", **a, **kw))
+        return None
+
+    def latent_query_at(j):
+        """The launch for a single slot's latents and the product of its queries -- or None."""
+        s = steps[j]
+        g = steps[j + 1] if j + 1 < len(steps) else None
+        o, q = s.op, s.outputs["q"]
+        if not (g is not None and o.rows == 1 and o.slots == 1 and o.dtype is bfloat16 and bare(s) and gemv_row(g, q) and once(q)
+                and not any(n % 8 for n in (o.stride, o.q_rank, o.rank, o.rot, o.turned)) and o.rank + o.rot <= 4096
+                and o.q_rank + o.rank + o.rot <= 8192):
+            return None
+        args = dict(x=tensor(s.inputs["x"]).reshape(-1), q_gain=tensor(s.inputs["q_gain"]), c_gain=tensor(s.inputs["c_gain"]),
+                    spans=tensor(s.inputs["spans"]), W=tensor(g.inputs["A"]), q=tensor(g.outputs["C"]).reshape(-1),
+                    latents=tensor(s.inputs["latents"]))
+        args |= {n: tensor(s.inputs[n]) for n in ("shared_keys", "angles") if n in s.inputs}
+        kw = {n: getattr(o, n) for n in ("stride", "q_rank", "rank", "rot", "turned", "angle_rows", "ring")}
+        kw |= dict(M=g.op.M, eps=float(o.epsilon))
+        return Fused("latent_query", j, 2, lambda a=args, kw=kw: kernels.latent_query(**a, **kw))
 
     def same_data(a, b) -> bool:
         return (a is not None and b is not None and a.buffer is b.buffer and a.offset == b.offset
@@ -607,6 +693,22 @@ def plan(recording, tensor: Callable[[Any], Any], word: Callable[[Any], Any],
                             h=tensor(nm.outputs["y"]), gain=tensor(nm.inputs["weight"]))
                 kw = dict(rows=s.op.rows, cols=s.op.cols, eps=float(s.op.epsilon), valid=word(s.values.get("valid")))
                 got = Fused("stream_add_norm", i, 2, lambda a=args, kw=kw: kernels.stream_rows(**a, **kw))
+        elif (_name(s) in ("StreamNorm", "MinGRU", "PolyNorm") or gemv_row(s)) and (got := stream_product_at(i)) is not None:
+            pass
+        elif _name(s) == "LatentRows" and (got := latent_query_at(i)) is not None:
+            pass
+        elif _name(s) == "StreamGatedAdd" and i + 1 < len(steps) and _name(steps[i + 1]) == "StreamNorm":
+            # a block's gated output into the stream and the next block's norm out of it: one pass over the row
+            nm = steps[i + 1]
+            if (_same_view(nm.inputs["x"], s.outputs["x"]) and nm.op.dtype is s.op.dtype and (nm.op.rows, nm.op.cols) == (s.op.rows, s.op.cols)
+                    and nm.values.get("valid") == s.values.get("valid") and set(nm.values) <= {"valid"} and set(s.values) <= {"valid"}):
+                args = dict(x=tensor(s.inputs["x"]), y=tensor(s.inputs["y"]), gate=tensor(s.inputs["gate"]), gate_bias=tensor(s.inputs["gate_bias"]),
+                            h=tensor(nm.outputs["y"]), gain=tensor(nm.inputs["weight"]))
+                if "y_bias" in s.inputs:
+                    args["y_bias"] = tensor(s.inputs["y_bias"])
+                kw = dict(rows=s.op.rows, cols=s.op.cols, eps=float(nm.op.epsilon), gate_stride=s.op.gate_width, gate_at=s.op.gate_at,
+                          valid=word(s.values.get("valid")))
+                got = Fused("stream_gated_add_norm", i, 2, lambda a=args, kw=kw: kernels.stream_gated_rows(**a, **kw))
         elif _name(s) == "LowRankDecay":
             got = parallel_at(i)
         elif _name(s) == "ShortConv":

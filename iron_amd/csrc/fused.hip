@@ -7,7 +7,7 @@
 //                [RMSNorm ->] GEMV(gate), GEMV(up) -> SiLU -> Mul          (the gated MLP's first half)
 //   decode_qkv:  RMSNorm -> GEMV q,k,v -> RoPE(q), RoPE(k) -> cache writes (attention's first half)
 #include "../../include/iron_hip.h"
-#include "common.h"
+#include "row_products.h"
 
 namespace iron {
 
@@ -16,14 +16,6 @@ namespace iron {
 // split K in 16-byte chunks (thread t takes chunks t, t+256, ...), so the weight loads of a row
 // are one contiguous stream per block, every lane has all its loads in flight before it needs
 // any of them, and the activation chunk a thread normalises is the one it multiplies by.
-
-// Block-wide sum through LDS (one barrier); every thread gets the total.
-__device__ __forceinline__ float block_sum(float v, float* scratch4) {
-  v = wave_sum(v);
-  if ((threadIdx.x & 63) == 0) scratch4[threadIdx.x >> 6] = v;
-  __syncthreads();
-  return scratch4[0] + scratch4[1] + scratch4[2] + scratch4[3];
-}
 
 // This thread's CH chunks of the activation as the GEMV sees them: x itself, or
 // RMSNorm(x) * w rounded as the RMSNorm step rounds (the normed row to bf16, then the
@@ -77,32 +69,6 @@ struct Activation {
     }
   }
 };
-
-// A weight row's chunks of this thread (zeros past the row's end), streamed past the caches.
-template <int CH>
-__device__ __forceinline__ void load_row(const bf16_t* __restrict__ row, int K, uint4 (&w)[CH]) {
-  const __amdgpu_buffer_rsrc_t run = bounded_bytes(row, 2 * K);
-#pragma unroll
-  for (int i = 0; i < CH; ++i) w[i] = load_bounded_stream(run, 16 * ((int)threadIdx.x + 256 * i));
-}
-
-// A row's chunks times the activation's: two-element dot products of the bf16 pairs as they were
-// loaded (v_dot2c_f32_bf16: exact products, float32 sums) -- a quarter of the instructions of
-// widening both sides and a multiply-add an element, and what a resident block does after its
-// loads have landed is time its CU's share of the memory system idles.
-typedef __bf16 bf16x2_t __attribute__((ext_vector_type(2)));
-template <int CH>
-__device__ __forceinline__ float dot_row(const uint4 (&w)[CH], const uint4 (&xp)[CH]) {
-  float acc = 0.f;
-#pragma unroll
-  for (int i = 0; i < CH; ++i) {
-    acc = __builtin_amdgcn_fdot2_f32_bf16(__builtin_bit_cast(bf16x2_t, w[i].x), __builtin_bit_cast(bf16x2_t, xp[i].x), acc, false);
-    acc = __builtin_amdgcn_fdot2_f32_bf16(__builtin_bit_cast(bf16x2_t, w[i].y), __builtin_bit_cast(bf16x2_t, xp[i].y), acc, false);
-    acc = __builtin_amdgcn_fdot2_f32_bf16(__builtin_bit_cast(bf16x2_t, w[i].z), __builtin_bit_cast(bf16x2_t, xp[i].z), acc, false);
-    acc = __builtin_amdgcn_fdot2_f32_bf16(__builtin_bit_cast(bf16x2_t, w[i].w), __builtin_bit_cast(bf16x2_t, xp[i].w), acc, false);
-  }
-  return acc;
-}
 
 enum { EPI_NONE = 0, EPI_ADD = 1, EPI_SILU_MUL = 2, EPI_GELU_MUL = 3,     // 2 and 3: gate, up -> activation -> Mul
        EPI_GELU_ROW = 4, EPI_SILU_ROW = 5,                                 // activation -> Mul by a given row

@@ -12,20 +12,11 @@
 // Caches are rings: position p's rows in row p % ring of its slot.  A call's own rows are stored before they
 // are attended, so a ring holds at least the window and a portion.
 #include "../../include/iron_hip.h"
-#include "rows.h"
+#include "latent.h"
 
 namespace iron {
 
 constexpr float LATENT_LOG2E = 1.4426950408889634f;
-
-struct LatentShape {
-  int slots, rows;                       // the batch's
-  int heads, dim, rot, vdim, rank;
-  int turned, angle_rows;                // columns of the rot ones that turn, and rows of the table of angles
-  int window, ring;
-  int cap;                               // expanded key rows there is room for
-  float scale;
-};
 
 // The key rows a slot's span attends: positions first .. first + count - 1, expanded in rows row0 ..
 struct KeyRun {
@@ -107,6 +98,21 @@ __global__ __launch_bounds__(256) void latent_rows_kernel(const T* __restrict__ 
   }
 }
 
+// The same in 16-byte pieces.
+template <typename T, int CH>
+__global__ __launch_bounds__(256) void latent_rows_wide_kernel(const T* __restrict__ x, LatentRow g, const int* __restrict__ spans,
+                                                               T* __restrict__ q_out, T* __restrict__ latents,
+                                                               T* __restrict__ shared_keys, LatentShape a, int stride) {
+  __shared__ float part[2][4];
+  const int row = blockIdx.x;
+  for (int slot = 0; slot < a.slots; ++slot) {
+    const Span s = span_of(spans, slot, a.rows);
+    if (row >= s.row0 && row < s.row0 + s.rows) {
+      latent_row<T, CH, true>(x + (size_t)row * stride, g, a, slot, s.start + row - s.row0, q_out + (size_t)row * g.q_rank, latents, shared_keys, part);
+      return;
+    }
+  }
+}
 // --------------------------------------------------------------- expansion
 // The latents a portion attends, slot after slot, and how many they are.
 constexpr int GATHER_ROWS = 16;
@@ -424,22 +430,23 @@ __device__ __forceinline__ void latent_prefill_body(const bf16_t* __restrict__ q
   }
 }
 
-// The spans' lengths are known on the device only: a block takes 128 queries where that still gives the chip a
-// block a CU, 64 otherwise (the grid is sized for 64; the blocks left over return).
+// The spans' lengths are known on the device only: a block takes 128 queries where narrow heads leave it the
+// registers and that still gives the chip a block a CU, 64 otherwise (the grid is sized for 64; the blocks left
+// over return).  The tiles with the most keys go first and those with the fewest last but in rising order, so that
+// two blocks that share a CU have about the same number of keys together, whichever CU it is.
 template <int DKP, int DVP>
-__global__ __launch_bounds__(256) void latent_prefill_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ kv,
-                                                             const bf16_t* __restrict__ shared_keys, const float* __restrict__ angles,
-                                                             const bf16_t* __restrict__ sink, const int* __restrict__ spans,
-                                                             bf16_t* __restrict__ y, LatentShape a) {
+__global__ __launch_bounds__(256, DKP + DVP <= 384 ? 2 : 1) void latent_prefill_kernel(
+    const bf16_t* __restrict__ q, const bf16_t* __restrict__ kv, const bf16_t* __restrict__ shared_keys, const float* __restrict__ angles,
+    const bf16_t* __restrict__ sink, const int* __restrict__ spans, bf16_t* __restrict__ y, LatentShape a) {
   constexpr int BUFFERS = DKP + DVP <= 192 ? 2 : 1;   // LDS: several blocks a CU
+  constexpr bool CAN_WIDE = DKP + DVP <= 192;
   __shared__ LatentShared<DKP, DVP> sh[BUFFERS];
   const Span s = span_of(spans, blockIdx.z, a.rows);
-  const int head = blockIdx.x;
-  // The last queries have the most keys: they go first.
-  constexpr bool CAN_WIDE = DVP <= 128 && DKP <= 192;   // registers
+  const int head = blockIdx.x, y_at = blockIdx.y;
   const bool wide = CAN_WIDE && (long)((s.rows + 127) / 128) * a.heads >= 256;
-  const int count = wide ? (s.rows + 127) / 128 : (s.rows + 63) / 64, tile = count - 1 - (int)blockIdx.y;
-  if (tile < 0) return;
+  const int count = wide ? (s.rows + 127) / 128 : (s.rows + 63) / 64;
+  if (y_at >= count) return;
+  const int half = (count + 1) / 2, tile = y_at < half ? count - 1 - y_at : y_at - half;
   const KeyRun run = key_run(spans, blockIdx.z, a);
   if (run.count < s.rows) return;   // no room was made for these keys
   if (wide) latent_prefill_body<DKP, DVP, CAN_WIDE ? 2 : 1, BUFFERS>(q, kv, shared_keys, angles, sink, y, a, s, run, blockIdx.z, head, tile, sh);
@@ -460,8 +467,8 @@ static void launch_latent_prefill(const bf16_t* q, const bf16_t* kv, const bf16_
 }
 
 // -------------------------------------------------------------- a decode step
-// The keys of a slot's one row, dealt to `splits` blocks in runs of whole 32-key tiles.
-constexpr int STEP_KEYS = 32;
+// The keys of a slot's one row, dealt to `splits` blocks in runs of whole 64-key tiles.
+constexpr int STEP_KEYS = 64;
 struct StepKeys {
   int first, count, per, live;   // first position, keys; keys a split, splits that have any
 };
@@ -587,26 +594,28 @@ __global__ __launch_bounds__(256) void latent_step_kernel(const float* __restric
   }
 }
 
-// bf16, rank and rot multiples of 8: sixteen heads a block on the MFMAs.  A tile of 32 keys lies in LDS as
-// [latent, padded to 64s | shared part, padded to 32s]; the waves deal the columns of the scores' product, add
-// their parts up in LDS, and deal the columns of the weighted sum.  Heads are an MFMA's columns throughout.
-// NG: groups of 64 latent columns a wave sums.
+// bf16, rank and rot multiples of 8: sixteen heads a block on the MFMAs, two teams of four waves with 32 keys at a
+// time each.  A team's keys lie in LDS as [latent, padded to 64s | shared part, padded to 32s]; its waves deal the
+// columns of the scores' product, add their parts up in LDS, and deal the columns of the weighted sum.  Heads are
+// an MFMA's columns throughout.  NG: groups of 64 latent columns a wave sums.
+constexpr int TEAM_KEYS = 32, TEAM_PARTS = 4 * 2 * 64 * 16;   // keys, and bytes of scores in parts
 template <int NG>
-__global__ __launch_bounds__(256) void latent_step_mfma_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ latents,
+__global__ __launch_bounds__(512) void latent_step_mfma_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ latents,
                                                                const bf16_t* __restrict__ shared_keys, const int* __restrict__ spans,
                                                                StepParts to, LatentShape a, int splits) {
   constexpr int PIECES = 5 * NG;              // 16-byte pieces of a tile a thread stages
   constexpr int STEPS = (10 * NG + 3) / 4;    // 32-column steps of the scores' product a wave takes
   extern __shared__ __align__(16) unsigned char dyn[];
   const int head0 = blockIdx.x * 16, split = blockIdx.y, slot = blockIdx.z;
-  const int t = threadIdx.x, lane = t & 63, wave = t >> 6, lo16 = lane & 15, quad = lane >> 4;
+  const int team = threadIdx.x >> 8, t = threadIdx.x & 255, lane = t & 63, wave = t >> 6, lo16 = lane & 15, quad = lane >> 4;
   const Span s = span_of(spans, slot, a.rows);
   if (s.rows == 0) return;
   const StepKeys k = step_keys(s, a, splits);
   if (split >= k.live) return;
   const int rank_pad = (a.rank + 63) & ~63, rot_pad = (a.rot + 31) & ~31, pitch = rank_pad + rot_pad + 8, wide = a.rank + a.rot;
-  f32x4* parts = reinterpret_cast<f32x4*>(dyn);               // [wave][key tile][lane]
-  bf16_t* tile = reinterpret_cast<bf16_t*>(dyn + 4 * 2 * 64 * 16);   // [32][pitch]
+  unsigned char* mine = dyn + team * (TEAM_PARTS + TEAM_KEYS * pitch * 2);
+  f32x4* parts = reinterpret_cast<f32x4*>(mine);                  // [wave][key tile][lane]
+  bf16_t* tile = reinterpret_cast<bf16_t*>(mine + TEAM_PARTS);    // [32][pitch]
 
   bf16x8 qf[STEPS];
   const int steps = (rank_pad + rot_pad) / 32;
@@ -619,7 +628,7 @@ __global__ __launch_bounds__(256) void latent_step_mfma_kernel(const bf16_t* __r
   }
   // The padding's zeros, which no tile replaces.
   const int pad_pieces = (pitch - 8 - wide) / 8;
-  for (int e = t; e < STEP_KEYS * pad_pieces; e += 256) {
+  for (int e = t; e < TEAM_KEYS * pad_pieces; e += 256) {
     const int row = e / pad_pieces, i = (e - row * pad_pieces) * 8, gap = rank_pad - a.rank;
     *reinterpret_cast<uint4*>(tile + row * pitch + (i < gap ? a.rank + i : rank_pad + a.rot + i - gap)) = make_uint4(0, 0, 0, 0);
   }
@@ -628,8 +637,8 @@ __global__ __launch_bounds__(256) void latent_step_mfma_kernel(const bf16_t* __r
 #pragma unroll
   for (int i = 0; i < PIECES; ++i) {
     const int e = t + 256 * i;
-    p_row[i] = e < STEP_KEYS * each ? e / each : -1;
-    p_col[i] = e < STEP_KEYS * each ? (e - e / each * each) * 8 : 0;
+    p_row[i] = e < TEAM_KEYS * each ? e / each : -1;
+    p_col[i] = e < TEAM_KEYS * each ? (e - e / each * each) * 8 : 0;
   }
   u32x4 held[PIECES];
   auto fetch = [&](int base) {
@@ -648,16 +657,16 @@ __global__ __launch_bounds__(256) void latent_step_mfma_kernel(const bf16_t* __r
     for (int e = 0; e < 4; ++e) acc[g][e] = f32x4{0.f, 0.f, 0.f, 0.f};
   float m = -1e30f, l = 0.f;
   const float scale = a.scale * LATENT_LOG2E;
-  int base = split * k.per;
+  int base = split * k.per + team * TEAM_KEYS;
   fetch(base);
-  for (; base < hi; base += STEP_KEYS) {
+  for (; base - team * TEAM_KEYS < hi; base += STEP_KEYS) {   // (a team past the last key: weights of zero)
     __syncthreads();   // the last tile's readers are done
 #pragma unroll
     for (int i = 0; i < PIECES; ++i)
       if (p_row[i] >= 0)
         *reinterpret_cast<u32x4*>(tile + p_row[i] * pitch + (p_col[i] < a.rank ? p_col[i] : rank_pad + p_col[i] - a.rank)) = held[i];
     __syncthreads();
-    if (base + STEP_KEYS < hi) fetch(base + STEP_KEYS);
+    if (base - team * TEAM_KEYS + STEP_KEYS < hi) fetch(base + STEP_KEYS);
     f32x4 sc[2] = {f32x4{0.f, 0.f, 0.f, 0.f}, f32x4{0.f, 0.f, 0.f, 0.f}};
 #pragma unroll
     for (int i = 0; i < STEPS; ++i) {
@@ -723,19 +732,42 @@ __global__ __launch_bounds__(256) void latent_step_mfma_kernel(const bf16_t* __r
   }
   l += __shfl_xor(l, 16, 64);
   l += __shfl_xor(l, 32, 64);
+  // The second team's sums join the first's, through the LDS its keys lay in.
+  __syncthreads();
+  float* other = reinterpret_cast<float*>(dyn + 2 * TEAM_PARTS + TEAM_KEYS * pitch * 2);   // [16][rank_pad]
+  float* other_stats = reinterpret_cast<float*>(dyn + TEAM_PARTS + TEAM_KEYS * pitch * 2);
+  if (team == 1) {
+#pragma unroll
+    for (int g = 0; g < NG; ++g)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int c = (wave + 4 * g) * 64 + (quad * 4 + r) * 4;
+        if (c < rank_pad) *reinterpret_cast<float4*>(other + lo16 * rank_pad + c) = make_float4(acc[g][0][r], acc[g][1][r], acc[g][2][r], acc[g][3][r]);
+      }
+    if (wave == 0 && quad == 0) {
+      other_stats[2 * lo16] = m;
+      other_stats[2 * lo16 + 1] = l;
+    }
+  }
+  __syncthreads();
   const int head = head0 + lo16;
-  if (head >= a.heads) return;
+  if (team == 1 || head >= a.heads) return;
+  const float om = other_stats[2 * lo16], top = fmaxf(m, om), f0 = __builtin_amdgcn_exp2f(m - top), f1 = __builtin_amdgcn_exp2f(om - top);
   const size_t part = ((size_t)slot * splits + split) * a.heads + head;
 #pragma unroll
   for (int g = 0; g < NG; ++g)
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const int c = (wave + 4 * g) * 64 + (quad * 4 + r) * 4;
-      if (c < a.rank) *reinterpret_cast<float4*>(to.sums + part * a.rank + c) = make_float4(acc[g][0][r], acc[g][1][r], acc[g][2][r], acc[g][3][r]);
+      if (c < a.rank) {
+        const float4 o = *reinterpret_cast<const float4*>(other + lo16 * rank_pad + c);
+        *reinterpret_cast<float4*>(to.sums + part * a.rank + c) =
+            make_float4(fmaf(acc[g][0][r], f0, o.x * f1), fmaf(acc[g][1][r], f0, o.y * f1), fmaf(acc[g][2][r], f0, o.z * f1), fmaf(acc[g][3][r], f0, o.w * f1));
+      }
     }
   if (wave == 0 && quad == 0) {
-    to.stats[2 * part] = m;
-    to.stats[2 * part + 1] = l;
+    to.stats[2 * part] = top;
+    to.stats[2 * part + 1] = fmaf(l, f0, other_stats[2 * lo16 + 1] * f1);
   }
 }
 
@@ -792,13 +824,13 @@ static bool latent_aligned(const LatentShape& a) { return a.rank % 8 == 0 && a.r
 static size_t step_mfma_lds(const LatentShape& a) {
   const int ng = a.rank <= 256 ? 1 : (a.rank <= 512 ? 2 : 4);
   if (!latent_aligned(a) || a.rank > 1024 || a.rot > 64 * ng) return 0;
-  const size_t bytes = 8192 + (size_t)STEP_KEYS * (((a.rank + 63) & ~63) + ((a.rot + 31) & ~31) + 8) * 2;
-  return bytes <= 65536 ? bytes : 0;
+  const size_t bytes = 2 * (TEAM_PARTS + (size_t)TEAM_KEYS * (((a.rank + 63) & ~63) + ((a.rot + 31) & ~31) + 8) * 2);
+  return bytes <= 163840 ? bytes : 0;
 }
 static int step_splits(const LatentShape& a) {
   const int most = a.window < a.ring ? a.window : a.ring, tiles = (most + STEP_KEYS - 1) / STEP_KEYS;
   int splits = 512 / (a.slots * ((a.heads + 15) / 16));
-  splits = splits < 8 ? 8 : (splits > 128 ? 128 : splits);
+  splits = splits < 8 ? 8 : (splits > 64 ? 64 : splits);
   return tiles < splits ? tiles : splits;
 }
 static size_t rounded16(size_t n) { return (n + 15) & ~(size_t)15; }
@@ -827,7 +859,17 @@ extern "C" int iron_latent_rows(const void* x, const uint16_t* q_gain, const uin
   const LatentShape a{slots, rows, 1, 1, rot, 1, rank, turned, angle_rows, 1, ring, 0, 1.f};
   if (const int e = check_latent("latent_rows", a, spans, shared_keys, angles)) return e;
   IRON_REQUIRE(q_rank > 0 && q_rank + rank + rot <= stride, "latent_rows: a row of %d holds no latents of %d and %d + %d", stride, q_rank, rank, rot);
-  if (is_float)
+  const LatentRow g{q_gain, c_gain, angles, q_rank, eps};
+  const bool wide = latent_row_wide(a, stride, q_rank) && (((uintptr_t)x | (uintptr_t)q_gain | (uintptr_t)c_gain | (uintptr_t)q_out | (uintptr_t)latents |
+                                                            (uintptr_t)shared_keys) & 15) == 0;
+#define IRON_LATENT_ROWS(T, CH)                                                                                                   \
+  hipLaunchKernelGGL((latent_rows_wide_kernel<T, CH>), dim3(rows), dim3(256), 0, (hipStream_t)stream, (const T*)x, g, spans, (T*)q_out, \
+                     (T*)latents, (T*)shared_keys, a, stride)
+  const bool two = q_rank + rank + rot <= 2 * 2048;
+  if (wide && is_float) { if (two) IRON_LATENT_ROWS(float, 2); else IRON_LATENT_ROWS(float, 4); }
+  else if (wide) { if (two) IRON_LATENT_ROWS(bf16_t, 2); else IRON_LATENT_ROWS(bf16_t, 4); }
+#undef IRON_LATENT_ROWS
+  else if (is_float)
     hipLaunchKernelGGL((latent_rows_kernel<float>), dim3(rows), dim3(256), 0, (hipStream_t)stream, (const float*)x, q_gain, c_gain, angles, spans,
                        (float*)q_out, (float*)latents, (float*)shared_keys, a, stride, q_rank, eps);
   else
@@ -880,11 +922,16 @@ extern "C" int iron_mha_latent(const void* q, const void* latents, const void* s
     if (mfma_lds) {
       const dim3 grid((heads + 15) / 16, splits, slots);
 #define IRON_STEP(NG)                                                                                                        \
-  hipLaunchKernelGGL((latent_step_mfma_kernel<NG>), grid, dim3(256), mfma_lds, s, (const bf16_t*)absorbed, (const bf16_t*)latents, \
+  static LdsOptIn opted##NG;                                                                                                 \
+  if (const hipError_t e = opted##NG.ensure((const void*)latent_step_mfma_kernel<NG>, 163840)) {                             \
+    set_error("mha_latent: %s", hipGetErrorString(e));                                                                       \
+    return (int)e;                                                                                                           \
+  }                                                                                                                          \
+  hipLaunchKernelGGL((latent_step_mfma_kernel<NG>), grid, dim3(512), mfma_lds, s, (const bf16_t*)absorbed, (const bf16_t*)latents, \
                      (const bf16_t*)shared_keys, spans, parts, a, splits)
-      if (rank <= 256) IRON_STEP(1);
-      else if (rank <= 512) IRON_STEP(2);
-      else IRON_STEP(4);
+      if (rank <= 256) { IRON_STEP(1); }
+      else if (rank <= 512) { IRON_STEP(2); }
+      else { IRON_STEP(4); }
 #undef IRON_STEP
     } else {
       const dim3 grid(heads, splits, slots);

@@ -8,7 +8,8 @@
 // The step from one state to the next is affine, S -> a S + b, and so is any run of steps: over a prompt's
 // portion a first launch folds every chunk of GRU_CHUNK tokens to its (a, b), and a second walks each chunk
 // from the state that the chunks before it leave.  A portion's first state is put ahead of its chunks, since
-// the block of its last chunk replaces it.
+// the block of its last chunk may replace it: a slot has two states, position p's in row p % 2, so that a
+// decode step's blocks leave the one they all read.
 #include "../../include/iron_hip.h"
 #include "rows.h"
 
@@ -71,7 +72,7 @@ __global__ __launch_bounds__(256) void min_gru_fold_kernel(const T* __restrict__
   float2* to = gru_chunk(work, spans, g, slot, 0) + c;
   if (chunk == 0)
 #pragma unroll
-    for (int j = 0; j < VEC; ++j) to[j] = make_float2(0.f, s.start > 0 ? state[(size_t)slot * g.width + c + j] : 0.f);
+    for (int j = 0; j < VEC; ++j) to[j] = make_float2(0.f, s.start > 0 ? state[(size_t)(2 * slot + ((s.start - 1) & 1)) * g.width + c + j] : 0.f);
   if (first + GRU_CHUNK >= s.rows) return;   // nobody starts from what the last chunk leaves
   float zbias[VEC], xbias[VEC], a[VEC], b[VEC];
   load_few<VEC>(zb + c, zbias);
@@ -114,7 +115,7 @@ __global__ __launch_bounds__(256) void min_gru_kernel(const T* __restrict__ x, c
   float zbias[VEC], xbias[VEC], S[VEC];
   load_few<VEC>(zb + c, zbias);
   load_few<VEC>(xb + c, xbias);
-  float* held = state + (size_t)slot * g.width + c;
+  const float* held = state + (size_t)(2 * slot + ((s.start - 1) & 1)) * g.width + c;
   if (CHUNKED) {
     const float2* from = gru_chunk(work, spans, g, slot, 0) + c;
 #pragma unroll
@@ -156,7 +157,7 @@ __global__ __launch_bounds__(256) void min_gru_kernel(const T* __restrict__ x, c
   }
   if (last == s.rows)
 #pragma unroll
-    for (int j = 0; j < VEC; ++j) held[j] = S[j];
+    for (int j = 0; j < VEC; ++j) state[(size_t)(2 * slot + ((s.start + s.rows - 1) & 1)) * g.width + c + j] = S[j];
 }
 
 template <typename T>

@@ -796,7 +796,7 @@ def min_gru(x, z_bias, x_bias, state, spans, y, *, slots, rows, stride, width, w
     is_float = _act(x, rows * stride, "x")
     _bf16(z_bias, width, "z_bias")
     _bf16(x_bias, width, "x_bias")
-    _f32(state, slots * width, "state")
+    _f32(state, slots * 2 * width, "state")
     _same_kind(is_float, y=y)
     _act(y, rows * width, "y")
     work = None if workspace is None else _work(workspace, int(lib().iron_min_gru_workspace_bytes(slots, rows, width)), "min_gru: workspace")
@@ -843,6 +843,49 @@ def mha_latent(q, latents, up, spans, y, workspace, *, slots, rows, heads, dim, 
                                 _spans(spans, slots), ptr(y), _work(workspace, need, "mha_latent: workspace"), slots, rows, heads, dim,
                                 rot, vdim, rank, turned, angle_rows, window, ring, cap, float(scale), int(single), int(is_float),
                                 current_stream()), "iron_mha_latent")
+
+
+STREAM_INPUTS = {"row": 0, "stream_norm": 1, "row_norm": 2, "min_gru": 3, "poly_norm": 4}   # by the C ABI's number
+
+
+def stream_product(W, x, *, input, M, K, y=None, stream=None, y_bias=None, gate=None, gate_bias=None, gain=None, b0=None, b1=None,
+                   state=None, spans=None, eps=0.0):
+    """One row's product: ``input`` says how its input is made of ``x``; the output is the row ``y``, or joins the
+    stream's row ``stream`` through ``gate`` (its first M elements)."""
+    _bf16(W, M * K, "W")
+    if input == "stream_norm":
+        _f32(x, K, "x")
+    elif _dev(x, "x").numel() < (3 * K if input == "min_gru" else K):
+        raise ValueError(f"stream_product: x holds {x.numel()} elements")
+    for t, n, name in ((y, M, "y"), (y_bias, M, "y_bias"), (gate_bias, M, "gate_bias"), (gain, 4 if input == "poly_norm" else K, "gain"),
+                       (b0, K, "b0"), (b1, K, "b1")):
+        if t is not None:
+            _bf16(t, n, name)
+    if state is not None:
+        _f32(state, 2 * K, "state")
+    if stream is not None:
+        _f32(stream, M, "stream")
+        if _dev(gate, "gate").numel() < M:
+            raise ValueError(f"stream_product: a gate of {gate.numel()} elements for {M}")
+    check(lib().iron_stream_product_bf16(STREAM_INPUTS[input], ptr(x), ptr(gain), ptr(b0), ptr(b1), ptr(state),
+                                         None if spans is None else _spans(spans, 1), float(eps), ptr(W), M, K, ptr(y), ptr(stream), ptr(y_bias),
+                                         ptr(gate), ptr(gate_bias), current_stream()), "iron_stream_product_bf16")
+
+
+def latent_query(x, q_gain, c_gain, spans, W, q, latents, *, M, stride, q_rank, rank, ring, eps, rot=0, turned=0, angle_rows=0,
+                 angles=None, shared_keys=None):
+    """A single slot's row: its latents normed, stored and turned, and the queries' product."""
+    _bf16(x, stride, "x")
+    _bf16(q_gain, q_rank, "q_gain")
+    _bf16(c_gain, rank, "c_gain")
+    _bf16(W, M * q_rank, "W")
+    _bf16(q, M, "q")
+    _bf16(latents, ring * rank, "latents")
+    if rot:
+        _bf16(shared_keys, ring * rot, "shared_keys")
+    check(lib().iron_latent_query_bf16(ptr(x), ptr(q_gain), ptr(c_gain), _turned(angles, angle_rows, turned), _spans(spans, 1), ptr(W), ptr(q),
+                                       ptr(latents), ptr(shared_keys), M, stride, q_rank, rank, rot, turned, angle_rows, ring, float(eps),
+                                       current_stream()), "iron_latent_query_bf16")
 
 
 def decode_mixed(h, carry, spans, products, *, k):

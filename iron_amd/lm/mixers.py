@@ -220,7 +220,7 @@ class GatedRecurrence(iron.Graph):
         self.out = Linear(inner, width, precision=precision)
 
     def states(self, slots: int) -> dict:
-        return {"memory": iron.state((slots, self.inner), np.float32)}
+        return {"memory": iron.state((slots, 2, self.inner), np.float32)}
 
     def body(self, x, call, state):
         return self.out(MinGRU.step(x, self.z_bias, self.x_bias, state["memory"], call.spans, dtype=self.dtype)[1])

@@ -144,7 +144,8 @@ class TimeMix(_Spanned):
 
 class MinGRU(_Spanned):
     """Per channel ``S <- (1 - z) S + z c; y = S silu(g)`` with ``z = sigmoid(zx + z_bias)`` and the candidate c,
-    of ``u = ux + x_bias``, ``u + 1/2`` from 0 up and ``sigmoid(u)`` below; rows ``[zx | ux | g | ..]``."""
+    of ``u = ux + x_bias``, ``u + 1/2`` from 0 up and ``sigmoid(u)`` below; rows ``[zx | ux | g | ..]``.  The
+    state behind position p is row ``p % 2`` of its slot."""
 
     slots: int = param()
     rows: int = param()
@@ -154,7 +155,7 @@ class MinGRU(_Spanned):
     x = In(rows, stride, dtype=dtype)
     z_bias = In(width)
     x_bias = In(width)
-    state = InOut(slots, width, dtype=F32)
+    state = InOut(slots, 2, width, dtype=F32)
     spans = In(slots, 4, dtype=np.int32)
     y = Out(rows, width, dtype=dtype)
     chunked: bool = param(default=lambda op: op.rows > op.CHUNKED_ROWS * op.slots, array=True, repr=False)

@@ -198,11 +198,11 @@ def min_gru(op, x, z_bias, x_bias, state, spans):
     z, u, g = _sigmoid(x[:, :W] + z_bias), x[:, W : 2 * W] + x_bias, x[:, 2 * W : 3 * W]
     c = np.where(u >= 0, u + 0.5, _sigmoid(u))
     for s, row, n, start in _spans(spans):
-        S = np.asarray(state[s], np.float64) if start else np.zeros(W)
+        S = np.asarray(state[s, (start - 1) % 2], np.float64) if start else np.zeros(W)
         for t in range(row, row + n):
             S = (1 - z[t]) * S + z[t] * c[t]
             y[t] = S * g[t] * _sigmoid(g[t])
-        state[s] = S
+        state[s, (start + n - 1) % 2] = S
     return state, _out(op, y)
 
 

@@ -79,7 +79,7 @@ def test_a_scaled_head(cuda, dtype):
 def gru_inputs(rng, op, spans):
     x = bf(rng, op.rows, op.stride, scale=1.5)
     return dict(x=x, z_bias=round_bf16(rng.uniform(-6, 2, op.width).astype(F32)), x_bias=bf(rng, op.width),
-                state=rng.standard_normal((op.slots, op.width)).astype(F32), spans=spans)
+                state=rng.standard_normal((op.slots, 2, op.width)).astype(F32), spans=spans)
 
 
 @BOTH
@@ -251,6 +251,58 @@ def test_a_long_step_over_many_splits(cuda):
                    3e-5 if dtype is F32 else 1.5e-2, workspace=True)
 
 
+# ---------------------------------------------------------------- a row's product in one launch
+
+
+def row_product(rng, M, K_):
+    return bf(rng, M, K_, scale=1 / np.sqrt(K_)), bf(rng, M), bf(rng, M + 8, scale=2), bf(rng, M), rng.standard_normal(M).astype(F32)
+
+
+@pytest.mark.parametrize("M,K_", [(70, 64), (2100, 512), (33, 2056), (40, 5000), (12, 14336)])
+def test_a_normed_row_s_product(cuda, M, K_):
+    rng = np.random.default_rng(M)
+    W, *_ = row_product(rng, M, K_)
+    gain = bf(rng, K_)
+    for kind, x in (("stream_norm", rng.standard_normal(K_).astype(F32) * 3), ("row_norm", bf(rng, K_)), ("row", bf(rng, K_))):
+        y = torch.empty(M, dtype=torch.bfloat16, device="cuda")
+        K.stream_product(device(W, BF16), device(x, F32 if kind == "stream_norm" else BF16), input=kind, M=M, K=K_, y=y, eps=1e-3,
+                         gain=None if kind == "row" else device(gain, BF16))
+        h = x if kind == "row" else round_bf16((x / np.sqrt((x.astype(np.float64) ** 2).mean() + 1e-3) * gain).astype(F32))
+        want = W.astype(np.float64) @ h
+        assert np.abs(from_torch(y) - want).max() <= 6e-3 * np.abs(want).max(), kind
+
+
+@pytest.mark.parametrize("M,K_", [(70, 64), (2100, 512), (33, 2056), (40, 5000), (12, 14336)])
+def test_a_row_s_product_joins_the_stream(cuda, M, K_):
+    rng = np.random.default_rng(M + 1)
+    W, y_bias, gate, gate_bias, stream = row_product(rng, M, K_)
+    x, b0, b1, coefficients = bf(rng, 3 * K_, scale=1.5), bf(rng, K_), bf(rng, K_), round_bf16(np.array([0.5, -1.25, 0.75, 0.25], F32))
+    opened = 1 / (1 + np.exp(-(gate[:M].astype(np.float64) + gate_bias)))
+    z = x[:K_].astype(np.float64) + b0
+    for start in (0, 5, 6):
+        state = rng.standard_normal((2, K_)).astype(F32)
+        held = None if start == 0 else state[(start - 1) % 2][None]
+        S = min_gru(x[None, :K_].astype(np.float64) + b0, x[None, K_ : 2 * K_].astype(np.float64) + b1, None if held is None else held[0])[0]
+        g = x[2 * K_ :].astype(np.float64)
+        made = {"row": x[:K_], "min_gru": S * g / (1 + np.exp(-g)),
+                "poly_norm": sum(c * z**n / np.sqrt((z ** (2 * n)).mean() + 1e-2) for c, n in zip(coefficients.astype(np.float64), (1, 2, 3))) + coefficients[3]}
+        for kind, h in made.items():
+            given = {} if kind == "row" else dict(b0=device(b0, BF16))
+            if kind == "min_gru":
+                given |= dict(b1=device(b1, BF16), state=device(state, F32), spans=device(table((0, 0, 1, start)), np.int32))
+            if kind == "poly_norm":
+                given |= dict(gain=device(coefficients, BF16), eps=1e-2)
+            for bias in (None, y_bias):
+                row = device(stream, F32)
+                K.stream_product(device(W, BF16), device(x if kind == "min_gru" else x[:K_], BF16), input=kind, M=M, K=K_, stream=row,
+                                 gate=device(gate, BF16), gate_bias=device(gate_bias, BF16), y_bias=None if bias is None else device(bias, BF16), **given)
+                want = stream + (W.astype(np.float64) @ h + (0 if bias is None else bias)) * opened
+                assert np.abs(from_torch(row) - want).max() <= 8e-3 * np.abs(want).max(), (kind, start)
+            if kind == "min_gru":   # the new state beside the old one, which is left
+                new = from_torch(given["state"]).reshape(2, K_)
+                assert np.array_equal(new[(start - 1) % 2], state[(start - 1) % 2]) and np.abs(new[start % 2] - S).max() <= 1e-5 * np.abs(S).max()
+
+
 # ---------------------------------------------------------------- whole models
 
 
@@ -337,10 +389,15 @@ def test_long_decoding(cuda):
 
 @pytest.mark.parametrize("name", MODELS)
 def test_a_single_slot_s_steps(cuda, name):
-    """One slot: a decode step's projections are single-row products."""
+    """One slot: a decode step's projections are single-row products, with what makes their inputs and takes their
+    outputs in the same launches where the sizes allow it."""
     model, plain = built(name, Pufuzen, slots=1, max_seq_len=300, prefill_chunk=96)
     model.load_versions()
     try:
+        kinds = {f.kind for f in model.decode_step._fused.values()}
+        if name != "odd":
+            assert {"stream_norm_gemv", "min_gru_gated_product", "poly_norm_gated_product", "gated_product", "latent_query"} <= kinds
+            assert "stream_gated_add_norm" in {f.kind for f in model.prompt_chunk._fused.values()}
         tokens = tokens_of(model, 200)
         want = plain(tokens)
         rows = [model.batch.step([Entry("x", tokens[:60], range(60))])[0]]
