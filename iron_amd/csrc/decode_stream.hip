@@ -234,13 +234,16 @@ static int launch_stream_product(const bf16_t* W, const StreamIn& in, const Stre
     hipLaunchKernelGGL((stream_product_kernel<RPW, CH, IN, OUT>), dim3(blocks), dim3(256), 0, s, W, in, out, M, K);               \
     IRON_LAUNCH_CHECK();                                                                                                          \
   }
-  // Rows a block takes: a few where its input is long in the making.
-  if (ch == 1 && (IN == IN_GRU || (M > 2048 && M >= 65536))) IRON_PRODUCT(4, 1)
+  // Rows a block takes (measured): more where the input is long in the making and the matrix is tall.
+  constexpr bool MADE = IN == IN_STREAM_NORM || IN == IN_GRU;
+  if (ch == 1 && IN == IN_STREAM_NORM && M >= 8192) IRON_PRODUCT(8, 1)
+  if (ch == 1 && IN == IN_GRU) IRON_PRODUCT(4, 1)
   if (ch == 1 && M > 2048) IRON_PRODUCT(2, 1)
   if (ch == 1) IRON_PRODUCT(1, 1)
+  if (ch == 2 && MADE) IRON_PRODUCT(4, 2)
   if (ch == 2) IRON_PRODUCT(2, 2)
-  if (ch == 4) IRON_PRODUCT(2, 4)
-  IRON_PRODUCT(1, 8)
+  if (ch == 4) IRON_PRODUCT(4, 4)
+  IRON_PRODUCT(2, 8)
 #undef IRON_PRODUCT
 }
 

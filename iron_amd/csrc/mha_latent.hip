@@ -114,28 +114,47 @@ __global__ __launch_bounds__(256) void latent_rows_wide_kernel(const T* __restri
   }
 }
 // --------------------------------------------------------------- expansion
-// The latents a portion attends, slot after slot, and how many they are.
+// The latents a portion attends, slot after slot, with their shared key parts, and behind the last a tile's rows of
+// zeros, so that a tile may be read whole wherever it starts; and how many rows that is.
+constexpr int LATENT_KEYS = 64;   // keys a tile
 constexpr int GATHER_ROWS = 16;
+__host__ __device__ inline long expanded_rows(long cap) { return (cap + LATENT_KEYS + 255) / 256 * 256; }   // (whole tiles of the product)
 template <typename T, int VEC>
-__global__ __launch_bounds__(256) void latent_gather_kernel(const T* __restrict__ latents, const int* __restrict__ spans,
-                                                            T* __restrict__ out, int* __restrict__ count, LatentShape a) {
-  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+__device__ __forceinline__ void copy_or_zero(const T* from, T* to, int n, int lane) {
+  for (int c = lane * VEC; c < n; c += 64 * VEC) {
+    float f[VEC];
+    if (from != nullptr) {
+      load_vec<VEC>(from + c, f);
+    } else {
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) f[j] = 0.f;
+    }
+    store_vec<VEC>(to + c, f);
+  }
+}
+template <typename T, int VEC>
+__global__ __launch_bounds__(256) void latent_gather_kernel(const T* __restrict__ latents, const T* __restrict__ shared_keys,
+                                                            const int* __restrict__ spans, T* __restrict__ out, T* __restrict__ shared_out,
+                                                            int* __restrict__ count, LatentShape a) {
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, first_row = blockIdx.x * GATHER_ROWS;
   int total = 0;
   for (int slot = 0; slot < a.slots; ++slot) {
     const Span s = span_of(spans, slot, a.rows);
     const int n = keys_of(s, a.window), first = s.start - min(s.start, a.window - 1);
-    const int lo = max((int)blockIdx.x * GATHER_ROWS, total), hi = min(min(((int)blockIdx.x + 1) * GATHER_ROWS, total + n), a.cap);
+    const int lo = max(first_row, total), hi = min(min(first_row + GATHER_ROWS, total + n), a.cap);
     for (int r = lo + wave; r < hi; r += 4) {
-      const T* from = latents + ((size_t)slot * a.ring + (first + r - total) % a.ring) * a.rank;
-      for (int c = lane * VEC; c < a.rank; c += 64 * VEC) {
-        float f[VEC];
-        load_vec<VEC>(from + c, f);
-        store_vec<VEC>(out + (size_t)r * a.rank + c, f);
-      }
+      const size_t at = (size_t)slot * a.ring + (first + r - total) % a.ring;
+      copy_or_zero<T, VEC>(latents + at * a.rank, out + (size_t)r * a.rank, a.rank, lane);
+      copy_or_zero<T, VEC>(shared_keys + at * a.rot, shared_out + (size_t)r * a.rot, a.rot, lane);
     }
     total += n;
   }
-  if (blockIdx.x == 0 && threadIdx.x == 0) *count = min(total, a.cap);
+  total = min(total, a.cap);
+  for (int r = max(first_row, total) + wave; r < min(first_row + GATHER_ROWS, total + LATENT_KEYS); r += 4) {
+    copy_or_zero<T, VEC>(nullptr, out + (size_t)r * a.rank, a.rank, lane);
+    copy_or_zero<T, VEC>(nullptr, shared_out + (size_t)r * a.rot, a.rot, lane);
+  }
+  if (blockIdx.x == 0 && threadIdx.x == 0) *count = total + LATENT_KEYS;
 }
 
 // ------------------------------------------------------- a portion, row by row
@@ -178,7 +197,7 @@ __global__ __launch_bounds__(64) void latent_rows_attention_kernel(const T* __re
     if (p0 + lane < hi) {
       const int p = p0 + lane;
       const T* kr = keys + (size_t)(k.row0 + p - k.first) * width;
-      const T* rr = shared_keys + ((size_t)slot * a.ring + p % a.ring) * a.rot;
+      const T* rr = shared_keys + (size_t)(k.row0 + p - k.first) * a.rot;
       float dot = 0.f;
       for (int c = 0; c < a.dim; ++c) dot = fmaf(load_one(kr + c), qs[c], dot);
       for (int c = 0; c < a.rot; ++c) dot = fmaf(load_one(rr + c), qs[a.dim + c], dot);
@@ -213,8 +232,6 @@ __global__ __launch_bounds__(64) void latent_rows_attention_kernel(const T* __re
 // computed transposed (keys down the MFMA's rows, queries across its columns): a lane holds one query's
 // scores, so the row statistics are a lane's own, and the weights are the second product's B operand as they
 // stand.  A sink is where a query's statistics start: a maximum, and one term of the sum.
-constexpr int LATENT_KEYS = 64;
-
 template <int DKP, int DVP>
 struct LatentShared {
   __align__(16) bf16_t k[LATENT_KEYS][DKP + 8];
@@ -225,7 +242,7 @@ template <int DKP, int DVP, int QT, int BUFFERS>
 __device__ __forceinline__ void latent_prefill_body(const bf16_t* __restrict__ q, const bf16_t* __restrict__ kv,
                                                     const bf16_t* __restrict__ shared_keys, const float* __restrict__ angles,
                                                     const bf16_t* __restrict__ sink, bf16_t* __restrict__ y, const LatentShape& a,
-                                                    const Span& s, const KeyRun& run, int slot, int head, int tile,
+                                                    const Span& s, const KeyRun& run, int head, int tile,
                                                     LatentShared<DKP, DVP>* tiles_lds) {
   constexpr int BQ = QT * 64, KD = DKP / 32, VD = DVP / 16;
   constexpr int KP = LATENT_KEYS * DKP / 8 / 256;      // 16-byte pieces of a key tile a thread stages
@@ -279,40 +296,43 @@ __device__ __forceinline__ void latent_prefill_body(const bf16_t* __restrict__ q
     for (int d = 0; d < VD; ++d) acc[n][d] = f32x4{0.f, 0.f, 0.f, 0.f};
   }
 
-  // The next tile on its way from memory.  A row past the last key reads the last again (its scores are masked),
-  // and a key's pieces past its head's width other columns, against zeros of q: no load is behind a branch.
+  // The next tile on its way from memory: a pointer a piece, moved on by a tile, and no load behind a branch.  A key's
+  // pieces past its head's width read other columns, against zeros of q.  A value piece is four keys of eight columns;
+  // a wave takes four such pieces side by side, so that its rows are read in 64-byte runs and written to LDS without
+  // conflicts.
   u32x4 kn[KP], vn[VT][4];
-  int k_row[KP], k_col[KP], v_row[VT], v_col[VT];
-  bool k_shared[KP];
+  const bf16_t *k_at[KP], *v_at[VT];
+  int k_step[KP];
+  const size_t row0 = (size_t)(run.row0 + from - run.first);
 #pragma unroll
   for (int i = 0; i < KP; ++i) {
-    const int e = t + 256 * i, c = (e % (DKP / 8)) * 8;
-    k_row[i] = e / (DKP / 8);
-    k_shared[i] = c >= a.dim && c < wide;
-    k_col[i] = k_shared[i] ? c - a.dim : head * a.dim + (c < a.dim ? c : 0);
+    const int e = t + 256 * i, c = (e % (DKP / 8)) * 8, row = e / (DKP / 8);
+    const bool part = c >= a.dim && c < wide;
+    k_step[i] = part ? a.rot : width;
+    k_at[i] = part ? shared_keys + (row0 + row) * a.rot + c - a.dim : kv + (row0 + row) * width + head * a.dim + (c < a.dim ? c : 0);
+    k_step[i] *= LATENT_KEYS;
   }
+  auto v_row = [&](int e) { return (e >> 2) & 15; };                      // a piece's keys, in fours
+  auto v_col = [&](int e) { return ((e >> 6) * 4 + (e & 3)) * 8; };       // ... and its columns
 #pragma unroll
   for (int i = 0; i < VT; ++i) {
     const int e = t + 256 * i;
-    v_row[i] = (e / (DVP / 8) * 4) % LATENT_KEYS;
-    v_col[i] = a.heads * a.dim + head * a.vdim + min((e % (DVP / 8)) * 8, a.vdim - 8);
+    v_at[i] = kv + (row0 + v_row(e) * 4) * width + a.heads * a.dim + head * a.vdim + min(v_col(e), a.vdim - 8);
   }
-  const bf16_t* ring = a.rot > 0 ? shared_keys + (size_t)slot * a.ring * a.rot : kv;
-  auto fetch = [&](int base) {
-    const int last = end - 1 - base, wrap = base % a.ring;
-    const bf16_t* rows = kv + (size_t)(run.row0 + base - run.first) * width;
+  auto fetch = [&]() {
 #pragma unroll
     for (int i = 0; i < KP; ++i) {
-      const int row = min(k_row[i], last), at = wrap + row - (wrap + row >= a.ring ? a.ring : 0);
-      const bf16_t* from_row = k_shared[i] ? ring + (size_t)(at * a.rot) : rows + (size_t)(row * width);
-      kn[i] = *reinterpret_cast<const u32x4*>(from_row + k_col[i]);
+      kn[i] = *reinterpret_cast<const u32x4*>(k_at[i]);
+      k_at[i] += k_step[i];
     }
 #pragma unroll
-    for (int i = 0; i < VT; ++i)
+    for (int i = 0; i < VT; ++i) {
 #pragma unroll
-      for (int j = 0; j < 4; ++j) vn[i][j] = *reinterpret_cast<const u32x4*>(rows + (size_t)(min(v_row[i] + j, last) * width) + v_col[i]);
+      for (int j = 0; j < 4; ++j) vn[i][j] = *reinterpret_cast<const u32x4*>(v_at[i] + (size_t)j * width);
+      v_at[i] += (size_t)LATENT_KEYS * width;
+    }
   };
-  fetch(from);
+  fetch();
   const float scale = a.scale * LATENT_LOG2E;
   for (int n = 0; n < tiles; ++n) {
     const int base = from + n * LATENT_KEYS;
@@ -325,7 +345,7 @@ __device__ __forceinline__ void latent_prefill_body(const bf16_t* __restrict__ q
     }
 #pragma unroll
     for (int i = 0; i < VT; ++i) {
-      const int e = t + 256 * i, r4 = e / (DVP / 8), c = (e % (DVP / 8)) * 8;
+      const int e = t + 256 * i, r4 = v_row(e), c = v_col(e);
       if (e < VP) {
 #pragma unroll
         for (int j = 0; j < 4; ++j) {   // two columns at a time: four keys each, 8 bytes
@@ -337,7 +357,7 @@ __device__ __forceinline__ void latent_prefill_body(const bf16_t* __restrict__ q
       }
     }
     __syncthreads();
-    if (n + 1 < tiles) fetch(base + LATENT_KEYS);
+    if (n + 1 < tiles) fetch();
 
     f32x4 sc[QT][4];
 #pragma unroll
@@ -449,8 +469,8 @@ __global__ __launch_bounds__(256, DKP + DVP <= 384 ? 2 : 1) void latent_prefill_
   const int half = (count + 1) / 2, tile = y_at < half ? count - 1 - y_at : y_at - half;
   const KeyRun run = key_run(spans, blockIdx.z, a);
   if (run.count < s.rows) return;   // no room was made for these keys
-  if (wide) latent_prefill_body<DKP, DVP, CAN_WIDE ? 2 : 1, BUFFERS>(q, kv, shared_keys, angles, sink, y, a, s, run, blockIdx.z, head, tile, sh);
-  else latent_prefill_body<DKP, DVP, 1, BUFFERS>(q, kv, shared_keys, angles, sink, y, a, s, run, blockIdx.z, head, tile, sh);
+  if (wide) latent_prefill_body<DKP, DVP, CAN_WIDE ? 2 : 1, BUFFERS>(q, kv, shared_keys, angles, sink, y, a, s, run, head, tile, sh);
+  else latent_prefill_body<DKP, DVP, 1, BUFFERS>(q, kv, shared_keys, angles, sink, y, a, s, run, head, tile, sh);
 }
 
 template <int DKP>
@@ -602,7 +622,7 @@ constexpr int TEAM_KEYS = 32, TEAM_PARTS = 4 * 2 * 64 * 16;   // keys, and bytes
 template <int NG>
 __global__ __launch_bounds__(512) void latent_step_mfma_kernel(const bf16_t* __restrict__ q, const bf16_t* __restrict__ latents,
                                                                const bf16_t* __restrict__ shared_keys, const int* __restrict__ spans,
-                                                               StepParts to, LatentShape a, int splits) {
+                                                               StepParts to, LatentShape a, int splits, unsigned each_inverse) {
   constexpr int PIECES = 5 * NG;              // 16-byte pieces of a tile a thread stages
   constexpr int STEPS = (10 * NG + 3) / 4;    // 32-column steps of the scores' product a wave takes
   extern __shared__ __align__(16) unsigned char dyn[];
@@ -617,6 +637,29 @@ __global__ __launch_bounds__(512) void latent_step_mfma_kernel(const bf16_t* __r
   f32x4* parts = reinterpret_cast<f32x4*>(mine);                  // [wave][key tile][lane]
   bf16_t* tile = reinterpret_cast<bf16_t*>(mine + TEAM_PARTS);    // [32][pitch]
 
+  const int hi = min(k.count, (split + 1) * k.per), each = wide / 8;
+  int p_row[PIECES], p_col[PIECES];
+#pragma unroll
+  for (int i = 0; i < PIECES; ++i) {
+    const int e = t + 256 * i;
+    const int row = (int)__umulhi((unsigned)e, each_inverse);   // e / each
+    p_row[i] = e < TEAM_KEYS * each ? row : -1;
+    p_col[i] = (e - row * each) * 8;
+  }
+  u32x4 held[PIECES];
+  const int wrap = k.first % a.ring;
+  auto fetch = [&](int base) {
+#pragma unroll
+    for (int i = 0; i < PIECES; ++i)
+      if (p_row[i] >= 0) {
+        const int in_ring = wrap + min(base + p_row[i], hi - 1);   // past the last: the last again
+        const size_t at = (size_t)slot * a.ring + (in_ring < a.ring ? in_ring : in_ring - a.ring);
+        const bf16_t* from = p_col[i] < a.rank ? latents + at * a.rank + p_col[i] : shared_keys + at * a.rot + p_col[i] - a.rank;
+        held[i] = *reinterpret_cast<const u32x4*>(from);
+      }
+  };
+  int base = split * k.per + team * TEAM_KEYS;
+  fetch(base);
   bf16x8 qf[STEPS];
   const int steps = (rank_pad + rot_pad) / 32;
 #pragma unroll
@@ -632,24 +675,6 @@ __global__ __launch_bounds__(512) void latent_step_mfma_kernel(const bf16_t* __r
     const int row = e / pad_pieces, i = (e - row * pad_pieces) * 8, gap = rank_pad - a.rank;
     *reinterpret_cast<uint4*>(tile + row * pitch + (i < gap ? a.rank + i : rank_pad + a.rot + i - gap)) = make_uint4(0, 0, 0, 0);
   }
-  const int hi = min(k.count, (split + 1) * k.per), each = wide / 8;
-  int p_row[PIECES], p_col[PIECES];
-#pragma unroll
-  for (int i = 0; i < PIECES; ++i) {
-    const int e = t + 256 * i;
-    p_row[i] = e < TEAM_KEYS * each ? e / each : -1;
-    p_col[i] = e < TEAM_KEYS * each ? (e - e / each * each) * 8 : 0;
-  }
-  u32x4 held[PIECES];
-  auto fetch = [&](int base) {
-#pragma unroll
-    for (int i = 0; i < PIECES; ++i)
-      if (p_row[i] >= 0) {
-        const size_t at = (size_t)slot * a.ring + (k.first + min(base + p_row[i], hi - 1)) % a.ring;   // past the last: the last again
-        const bf16_t* from = p_col[i] < a.rank ? latents + at * a.rank + p_col[i] : shared_keys + at * a.rot + p_col[i] - a.rank;
-        held[i] = *reinterpret_cast<const u32x4*>(from);
-      }
-  };
   f32x4 acc[NG][4];
 #pragma unroll
   for (int g = 0; g < NG; ++g)
@@ -657,8 +682,6 @@ __global__ __launch_bounds__(512) void latent_step_mfma_kernel(const bf16_t* __r
     for (int e = 0; e < 4; ++e) acc[g][e] = f32x4{0.f, 0.f, 0.f, 0.f};
   float m = -1e30f, l = 0.f;
   const float scale = a.scale * LATENT_LOG2E;
-  int base = split * k.per + team * TEAM_KEYS;
-  fetch(base);
   for (; base - team * TEAM_KEYS < hi; base += STEP_KEYS) {   // (a team past the last key: weights of zero)
     __syncthreads();   // the last tile's readers are done
 #pragma unroll
@@ -771,50 +794,70 @@ __global__ __launch_bounds__(512) void latent_step_mfma_kernel(const bf16_t* __r
   }
 }
 
-// The splits' sums become a head's latent, and V_h makes its values of it: a wave a value column.
-template <typename T, int VEC>
+// The splits' sums become a head's latent, and V_h makes its values of it: a wave VALUE_ROWS value columns, whose
+// weights (CH 16-byte pieces a lane; 0: any rank, read where they are needed) are on their way from the start.
+constexpr int VALUE_ROWS = 8;
+template <typename T, int CH>
 __global__ __launch_bounds__(256) void latent_values_kernel(StepParts from, const bf16_t* __restrict__ up, const bf16_t* __restrict__ sink,
-                                                            const int* __restrict__ spans, T* __restrict__ y, LatentShape a, int splits,
-                                                            int columns) {
-  extern __shared__ float lds[];   // a weight a split, then the latent
+                                                            const int* __restrict__ spans, T* __restrict__ y, LatentShape a, int splits) {
+  constexpr int HELD = CH > 0 ? CH : 1;
+  extern __shared__ __align__(16) float lds[];   // the latent, then a weight a split
   const int head = blockIdx.x, slot = blockIdx.z, t = threadIdx.x, lane = t & 63, wave = t >> 6;
+  const int v0 = (blockIdx.y * 4 + wave) * VALUE_ROWS;
+  const bf16_t* rows = up + ((size_t)a.heads * a.dim + (size_t)head * a.vdim) * a.rank;
+  uint4 w[VALUE_ROWS][HELD];
+  if (CH > 0) {
+#pragma unroll
+    for (int r = 0; r < VALUE_ROWS; ++r) {
+      const __amdgpu_buffer_rsrc_t run = bounded_bytes(rows + (size_t)min(v0 + r, a.vdim - 1) * a.rank, a.rank * 2);
+#pragma unroll
+      for (int i = 0; i < CH; ++i) w[r][i] = load_bounded(run, 16 * (lane + 64 * i));
+    }
+  }
   const Span s = span_of(spans, slot, a.rows);
   if (s.rows == 0) return;
   const StepKeys k = step_keys(s, a, splits);
-  float* latent = lds + splits;
+  float* latent = lds;
+  float* shares = lds + ((a.rank + 511) & ~511);
   const size_t part = (size_t)slot * splits * a.heads + head;
-  float top = sink != nullptr ? bf16_to_f32(sink[head]) * LATENT_LOG2E : -1e30f;
-  const float sunk = top;
+  const float sunk = sink != nullptr ? bf16_to_f32(sink[head]) * LATENT_LOG2E : -1e30f;
+  float top = sunk, total = 0.f;
   for (int i = lane; i < k.live; i += 64) top = fmaxf(top, from.stats[2 * (part + (size_t)i * a.heads)]);
   top = wave_max(top);
-  float total = 0.f;
   for (int i = lane; i < k.live; i += 64) {
-    const float w = latent_exp2<T>(from.stats[2 * (part + (size_t)i * a.heads)] - top);
-    if (wave == 0) lds[i] = w;
-    total = fmaf(w, from.stats[2 * (part + (size_t)i * a.heads) + 1], total);
+    const float share = latent_exp2<T>(from.stats[2 * (part + (size_t)i * a.heads)] - top);
+    if (wave == 0) shares[i] = share;
+    total = fmaf(share, from.stats[2 * (part + (size_t)i * a.heads) + 1], total);
   }
   total = wave_sum(total) + (sink != nullptr ? latent_exp2<T>(sunk - top) : 0.f);
   __syncthreads();
   const float inv = 1.0f / total;
-  for (int c = t; c < a.rank; c += 256) {
+  for (int c = t; c < ((a.rank + 511) & ~511); c += 256) {
     float sum = 0.f;
-#pragma unroll 8
-    for (int i = 0; i < k.live; ++i) sum = fmaf(from.sums[(part + (size_t)i * a.heads) * a.rank + c], lds[i], sum);
+    if (c < a.rank)
+#pragma unroll 16
+      for (int i = 0; i < k.live; ++i) sum = fmaf(from.sums[(part + (size_t)i * a.heads) * a.rank + c], shares[i], sum);
     latent[c] = sum * inv;
   }
   __syncthreads();
-  const int hi = min(a.vdim, (int)(blockIdx.y + 1) * columns);
-  for (int v = blockIdx.y * columns + wave; v < hi; v += 4) {
-    const bf16_t* w = up + ((size_t)a.heads * a.dim + (size_t)head * a.vdim + v) * a.rank;
-    float sum = 0.f;
-    for (int c = lane * VEC; c < a.rank; c += 64 * VEC) {
-      float f[VEC];
-      load_vec<VEC>(w + c, f);
 #pragma unroll
-      for (int j = 0; j < VEC; ++j) sum = fmaf(f[j], latent[c + j], sum);
+  for (int r = 0; r < VALUE_ROWS; ++r) {
+    if (v0 + r >= a.vdim) break;
+    float sum = 0.f;
+    if (CH > 0) {
+#pragma unroll
+      for (int i = 0; i < CH; ++i) {
+        float f[8];
+        unpack8(w[r][i], f);
+        const float4 lo = *reinterpret_cast<const float4*>(latent + (lane + 64 * i) * 8), hi = *reinterpret_cast<const float4*>(latent + (lane + 64 * i) * 8 + 4);
+        sum = fmaf(f[0], lo.x, sum); sum = fmaf(f[1], lo.y, sum); sum = fmaf(f[2], lo.z, sum); sum = fmaf(f[3], lo.w, sum);
+        sum = fmaf(f[4], hi.x, sum); sum = fmaf(f[5], hi.y, sum); sum = fmaf(f[6], hi.z, sum); sum = fmaf(f[7], hi.w, sum);
+      }
+    } else {
+      for (int c = lane; c < a.rank; c += 64) sum = fmaf(bf16_to_f32(rows[(size_t)(v0 + r) * a.rank + c]), latent[c], sum);
     }
     sum = wave_sum(sum);
-    if (lane == 0) store_one(y + ((size_t)s.row0 * a.heads + head) * a.vdim + v, sum);
+    if (lane == 0) store_one(y + ((size_t)s.row0 * a.heads + head) * a.vdim + v0 + r, sum);
   }
 }
 
@@ -883,7 +926,10 @@ extern "C" int64_t iron_mha_latent_workspace_bytes(int slots, int rows, int head
   const LatentShape a{slots, rows, heads, dim, rot, vdim, rank, 0, 0, window, ring, cap, 1.f};
   if (slots <= 0 || heads <= 0 || rank <= 0 || window <= 0 || ring <= 0) return 0;
   const size_t each = is_float ? 4 : 2;
-  if (!single) return (int64_t)(16 + rounded16((size_t)cap * rank * each) + rounded16((size_t)cap * heads * (dim + vdim) * each));
+  if (!single) {
+    const size_t n = (size_t)expanded_rows(cap);
+    return (int64_t)(16 + rounded16(n * rank * each) + rounded16(n * rot * each) + n * heads * (dim + vdim) * each);
+  }
   return (int64_t)(rounded16((size_t)slots * heads * (rank + rot) * 4) + rounded16((size_t)slots * step_splits(a) * heads * rank * 4) +
                    (size_t)slots * step_splits(a) * heads * 8);
 }
@@ -928,7 +974,7 @@ extern "C" int iron_mha_latent(const void* q, const void* latents, const void* s
     return (int)e;                                                                                                           \
   }                                                                                                                          \
   hipLaunchKernelGGL((latent_step_mfma_kernel<NG>), grid, dim3(512), mfma_lds, s, (const bf16_t*)absorbed, (const bf16_t*)latents, \
-                     (const bf16_t*)shared_keys, spans, parts, a, splits)
+                     (const bf16_t*)shared_keys, spans, parts, a, splits, (unsigned)((1ull << 32) / (unsigned)((rank + rot) / 8) + 1))
       if (rank <= 256) { IRON_STEP(1); }
       else if (rank <= 512) { IRON_STEP(2); }
       else { IRON_STEP(4); }
@@ -944,41 +990,47 @@ extern "C" int iron_mha_latent(const void* q, const void* latents, const void* s
         hipLaunchKernelGGL((latent_step_kernel<bf16_t>), grid, dim3(256), lds, s, (const float*)absorbed, (const bf16_t*)latents,
                            (const bf16_t*)shared_keys, spans, parts, a, splits);
     }
-    const int columns = 32;
-    const dim3 vg(heads, (vdim + columns - 1) / columns, slots);
-    const size_t vlds = (size_t)(splits + rank) * 4;
-#define IRON_VALUES(T)                                                                                                                 \
-  {                                                                                                                                    \
-    if (vec) hipLaunchKernelGGL((latent_values_kernel<T, 8>), vg, dim3(256), vlds, s, parts, up, sink, spans, (T*)y, a, splits, columns); \
-    else hipLaunchKernelGGL((latent_values_kernel<T, 1>), vg, dim3(256), vlds, s, parts, up, sink, spans, (T*)y, a, splits, columns);     \
+    const dim3 vg(heads, (vdim + 4 * VALUE_ROWS - 1) / (4 * VALUE_ROWS), slots);
+    const size_t vlds = (size_t)(splits + ((rank + 511) & ~511)) * 4;
+#define IRON_VALUES_CH(T, CH) hipLaunchKernelGGL((latent_values_kernel<T, CH>), vg, dim3(256), vlds, s, parts, up, sink, spans, (T*)y, a, splits)
+#define IRON_VALUES(T)                                  \
+  {                                                     \
+    if (vec && rank <= 512) IRON_VALUES_CH(T, 1);       \
+    else if (vec && rank <= 1024) IRON_VALUES_CH(T, 2); \
+    else IRON_VALUES_CH(T, 0);                          \
   }
     if (is_float) IRON_VALUES(float)
     else IRON_VALUES(bf16_t)
 #undef IRON_VALUES
+#undef IRON_VALUES_CH
     IRON_LAUNCH_CHECK();
   }
 
   IRON_REQUIRE(cap > 0 && rows <= 65535, "mha_latent: room for keys (%d), and rows (%d) within the grid's extent", cap, rows);
-  IRON_REQUIRE((long)64 * width * 2 < (1L << 31) && (long)ring * rot * 2 < (1L << 31), "mha_latent: a tile's rows are addressed with 32-bit offsets");
+  IRON_REQUIRE((long)LATENT_KEYS * width < (1L << 31) && expanded_rows(cap) < (1L << 31), "mha_latent: a tile's rows are addressed with 32-bit offsets");
+  const size_t n = (size_t)expanded_rows(cap), each = is_float ? 4 : 2;
   int* count = (int*)work;
   void* gathered = work + 16;
-  void* kv = work + 16 + rounded16((size_t)cap * rank * (is_float ? 4 : 2));
-  const dim3 gg((cap + GATHER_ROWS - 1) / GATHER_ROWS);
+  void* shared = work + 16 + rounded16(n * rank * each);
+  void* kv = work + 16 + rounded16(n * rank * each) + rounded16(n * rot * each);
+  const dim3 gg((cap + LATENT_KEYS + GATHER_ROWS - 1) / GATHER_ROWS);
   const bool vec = rank % 8 == 0;
-#define IRON_GATHER(T)                                                                                                                  \
-  {                                                                                                                                     \
-    if (vec) hipLaunchKernelGGL((latent_gather_kernel<T, 8>), gg, dim3(256), 0, s, (const T*)latents, spans, (T*)gathered, count, a);    \
-    else hipLaunchKernelGGL((latent_gather_kernel<T, 1>), gg, dim3(256), 0, s, (const T*)latents, spans, (T*)gathered, count, a);        \
+#define IRON_GATHER(T)                                                                                                                      \
+  {                                                                                                                                         \
+    if (vec && rot % 8 == 0)                                                                                                                \
+      hipLaunchKernelGGL((latent_gather_kernel<T, 8>), gg, dim3(256), 0, s, (const T*)latents, (const T*)shared_keys, spans, (T*)gathered, (T*)shared, count, a); \
+    else                                                                                                                                    \
+      hipLaunchKernelGGL((latent_gather_kernel<T, 1>), gg, dim3(256), 0, s, (const T*)latents, (const T*)shared_keys, spans, (T*)gathered, (T*)shared, count, a); \
   }
   if (is_float) IRON_GATHER(float)
   else IRON_GATHER(bf16_t)
 #undef IRON_GATHER
-  const int e = is_float || !vec ? iron_linear_any(gathered, up, kv, cap, width, rank, is_float, count, stream)
-                                 : iron_gemm_bf16((const uint16_t*)gathered, up, (uint16_t*)kv, cap, width, rank, 1, 0, count, nullptr, stream);
+  const int e = is_float || !vec ? iron_linear_any(gathered, up, kv, (int)n, width, rank, is_float, count, stream)
+                                 : iron_gemm_bf16((const uint16_t*)gathered, up, (uint16_t*)kv, (int)n, width, rank, 1, 0, count, nullptr, stream);
   if (e != IRON_OK) return e;
   const bool tiles = !is_float && dim % 8 == 0 && rot % 8 == 0 && turned % 8 == 0 && vdim % 8 == 0 && dim + rot <= 256 && vdim <= 256;
   if (tiles) {
-    const bf16_t *qb = (const bf16_t*)q, *kvb = (const bf16_t*)kv, *rb = (const bf16_t*)shared_keys;
+    const bf16_t *qb = (const bf16_t*)q, *kvb = (const bf16_t*)kv, *rb = (const bf16_t*)shared;
     if (dim + rot <= 32) launch_latent_prefill<32>(qb, kvb, rb, angles, sink, spans, (bf16_t*)y, a, s);
     else if (dim + rot <= 64) launch_latent_prefill<64>(qb, kvb, rb, angles, sink, spans, (bf16_t*)y, a, s);
     else if (dim + rot <= 128) launch_latent_prefill<128>(qb, kvb, rb, angles, sink, spans, (bf16_t*)y, a, s);
@@ -988,10 +1040,10 @@ extern "C" int iron_mha_latent(const void* q, const void* latents, const void* s
     const dim3 grid(heads, rows, slots);
     const size_t lds = (size_t)(dim + rot + 64) * 4;
     if (is_float)
-      hipLaunchKernelGGL((latent_rows_attention_kernel<float>), grid, dim3(64), lds, s, (const float*)q, (const float*)kv, (const float*)shared_keys,
+      hipLaunchKernelGGL((latent_rows_attention_kernel<float>), grid, dim3(64), lds, s, (const float*)q, (const float*)kv, (const float*)shared,
                          angles, sink, spans, (float*)y, a);
     else
-      hipLaunchKernelGGL((latent_rows_attention_kernel<bf16_t>), grid, dim3(64), lds, s, (const bf16_t*)q, (const bf16_t*)kv, (const bf16_t*)shared_keys,
+      hipLaunchKernelGGL((latent_rows_attention_kernel<bf16_t>), grid, dim3(64), lds, s, (const bf16_t*)q, (const bf16_t*)kv, (const bf16_t*)shared,
                          angles, sink, spans, (bf16_t*)y, a);
   }
   IRON_LAUNCH_CHECK();

@@ -5,17 +5,18 @@
 //
 // zx, ux and gx are columns 0, width and 2 width of a packed projection's row.  Everything in float32.
 //
-// The step from one state to the next is affine, S -> a S + b, and so is any run of steps: over a prompt's
-// portion a first launch folds every chunk of GRU_CHUNK tokens to its (a, b), and a second walks each chunk
-// from the state that the chunks before it leave.  A portion's first state is put ahead of its chunks, since
-// the block of its last chunk may replace it: a slot has two states, position p's in row p % 2, so that a
-// decode step's blocks leave the one they all read.
+// The step from one state to the next is affine, S -> a S + b, and so is any run of steps.  Over a prompt's portion
+// a block takes GRU_CHUNK tokens of 64 or 128 channels, GRU_TOKENS a wave: the waves fold their tokens to an (a, b)
+// each, and those to one a chunk.  A first launch does this for every chunk; in a second a block starts from the
+// state the chunks before its own leave, a wave from the one the waves before it leave, and walks.  A portion's
+// first state is put ahead of its chunks, since the block of its last chunk may replace it: a slot has two states,
+// position p's in row p % 2, so that a decode step's blocks leave the one they all read.
 #include "../../include/iron_hip.h"
 #include "rows.h"
 
 namespace iron {
 
-constexpr int GRU_CHUNK = 32, GRU_AHEAD = 8;   // tokens a chunk, and tokens asked for at a time
+constexpr int GRU_WAVES = 8, GRU_TOKENS = 16, GRU_CHUNK = GRU_WAVES * GRU_TOKENS;
 
 // Two neighbouring elements, or one.
 template <int VEC, typename T>
@@ -61,103 +62,131 @@ __device__ __forceinline__ float2* gru_chunk(float2* work, const int* spans, con
   return work + (size_t)(first_chunk(spans, g.slots, slot, g.rows, GRU_CHUNK) * 2 + chunk) * g.width;
 }
 
+// A wave's tokens of the columns `at ..` of the projection (its last again past the span's end).
 template <typename T, int VEC>
-__global__ __launch_bounds__(256) void min_gru_fold_kernel(const T* __restrict__ x, const bf16_t* __restrict__ zb,
-                                                           const bf16_t* __restrict__ xb, const float* __restrict__ state,
-                                                           const int* __restrict__ spans, float2* __restrict__ work, GruShape g) {
-  const int slot = blockIdx.z, chunk = blockIdx.y, c = (blockIdx.x * 256 + threadIdx.x) * VEC;
-  const Span s = span_of(spans, slot, g.rows);
-  const int first = chunk * GRU_CHUNK;
-  if (first >= s.rows || c >= g.width) return;
-  float2* to = gru_chunk(work, spans, g, slot, 0) + c;
-  if (chunk == 0)
+__device__ __forceinline__ void gru_load(const T* __restrict__ x, const GruShape& g, const Span& s, int t0, int at, float (&f)[GRU_TOKENS][VEC]) {
 #pragma unroll
-    for (int j = 0; j < VEC; ++j) to[j] = make_float2(0.f, s.start > 0 ? state[(size_t)(2 * slot + ((s.start - 1) & 1)) * g.width + c + j] : 0.f);
-  if (first + GRU_CHUNK >= s.rows) return;   // nobody starts from what the last chunk leaves
-  float zbias[VEC], xbias[VEC], a[VEC], b[VEC];
-  load_few<VEC>(zb + c, zbias);
-  load_few<VEC>(xb + c, xbias);
-#pragma unroll
-  for (int j = 0; j < VEC; ++j) a[j] = 1.f, b[j] = 0.f;
-  const T* row = x + (size_t)(s.row0 + first) * g.stride + c;
-  for (int t0 = 0; t0 < GRU_CHUNK; t0 += GRU_AHEAD) {
-    float z[GRU_AHEAD][VEC], u[GRU_AHEAD][VEC];
-#pragma unroll
-    for (int i = 0; i < GRU_AHEAD; ++i) {
-      load_few<VEC>(row + (size_t)(t0 + i) * g.stride, z[i]);
-      load_few<VEC>(row + (size_t)(t0 + i) * g.stride + g.width, u[i]);
-    }
-#pragma unroll
-    for (int i = 0; i < GRU_AHEAD; ++i)
-#pragma unroll
-      for (int j = 0; j < VEC; ++j) {
-        float p, q;
-        gru_step<T>(z[i][j] + zbias[j], u[i][j] + xbias[j], p, q);
-        a[j] *= p;
-        b[j] = fmaf(p, b[j], q);
-      }
-  }
-#pragma unroll
-  for (int j = 0; j < VEC; ++j) to[(size_t)(chunk + 1) * g.width + j] = make_float2(a[j], b[j]);
+  for (int i = 0; i < GRU_TOKENS; ++i) load_few<VEC>(x + (size_t)(s.row0 + min(t0 + i, s.rows - 1)) * g.stride + at, f[i]);
 }
 
-// CHUNKED: a block's chunk, from what the chunks before it leave in the workspace; else all of a span's rows.
-template <typename T, int VEC, bool CHUNKED>
-__global__ __launch_bounds__(256) void min_gru_kernel(const T* __restrict__ x, const bf16_t* __restrict__ zb,
-                                                      const bf16_t* __restrict__ xb, float* __restrict__ state,
-                                                      const int* __restrict__ spans, float2* __restrict__ work,
-                                                      T* __restrict__ y, GruShape g) {
-  const int slot = blockIdx.z, chunk = blockIdx.y, c = (blockIdx.x * 256 + threadIdx.x) * VEC;
+// WALK false: every chunk's (a, b) into the workspace, but the last's, which nobody starts from.
+template <typename T, int VEC, bool WALK>
+__global__ __launch_bounds__(GRU_WAVES * 64) void min_gru_chunks_kernel(const T* __restrict__ x, const bf16_t* __restrict__ zb,
+                                                                        const bf16_t* __restrict__ xb, float* __restrict__ state,
+                                                                        const int* __restrict__ spans, float2* __restrict__ work,
+                                                                        T* __restrict__ y, GruShape g) {
+  __shared__ float2 folded[GRU_WAVES][64 * VEC];
+  const int slot = blockIdx.z, chunk = blockIdx.y, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const Span s = span_of(spans, slot, g.rows);
-  const int first = chunk * GRU_CHUNK;
-  if (first >= s.rows || c >= g.width) return;
-  const int last = CHUNKED ? min(s.rows, first + GRU_CHUNK) : s.rows;
-  float zbias[VEC], xbias[VEC], S[VEC];
-  load_few<VEC>(zb + c, zbias);
-  load_few<VEC>(xb + c, xbias);
-  const float* held = state + (size_t)(2 * slot + ((s.start - 1) & 1)) * g.width + c;
-  if (CHUNKED) {
-    const float2* from = gru_chunk(work, spans, g, slot, 0) + c;
+  const int first = chunk * GRU_CHUNK, t0 = first + wave * GRU_TOKENS;
+  if (first >= s.rows) return;
+  const bool last = first + GRU_CHUNK >= s.rows;
+  const int c = (blockIdx.x * 64 + lane) * VEC, at = min(c, g.width - VEC);   // (a lane past the width: the last channels, not stored)
+  const bool in = c < g.width;
+  float2* chunks = gru_chunk(work, spans, g, slot, 0) + at;
+  if (!WALK && chunk == 0 && wave == 0 && in)
 #pragma unroll
-    for (int j = 0; j < VEC; ++j) S[j] = from[j].y;
-#pragma unroll 8
+    for (int j = 0; j < VEC; ++j) chunks[j] = make_float2(0.f, s.start > 0 ? state[(size_t)(2 * slot + ((s.start - 1) & 1)) * g.width + at + j] : 0.f);
+  if (!WALK && last) return;
+  float z[GRU_TOKENS][VEC], u[GRU_TOKENS][VEC], o[GRU_TOKENS][VEC], zbias[VEC], xbias[VEC];
+  gru_load<T, VEC>(x, g, s, t0, at, z);
+  gru_load<T, VEC>(x, g, s, t0, at + g.width, u);
+  if (WALK) gru_load<T, VEC>(x, g, s, t0, at + 2 * g.width, o);
+  load_few<VEC>(zb + at, zbias);
+  load_few<VEC>(xb + at, xbias);
+  float a[VEC], b[VEC], S[VEC];
+#pragma unroll
+  for (int j = 0; j < VEC; ++j) a[j] = 1.f, b[j] = 0.f;
+#pragma unroll
+  for (int i = 0; i < GRU_TOKENS; ++i)
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) {   // the step's own (a, b) where its two inputs were
+      float p, q;
+      gru_step<T>(z[i][j] + zbias[j], u[i][j] + xbias[j], p, q);
+      z[i][j] = p;
+      u[i][j] = q;
+      a[j] *= p;
+      b[j] = fmaf(p, b[j], q);
+    }
+#pragma unroll
+  for (int j = 0; j < VEC; ++j) folded[wave][lane * VEC + j] = make_float2(a[j], b[j]);
+  if (WALK) {
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) S[j] = chunks[j].y;
+#pragma unroll 16
     for (int k = 1; k <= chunk; ++k)
 #pragma unroll
       for (int j = 0; j < VEC; ++j) {
-        const float2 ab = from[(size_t)k * g.width + j];
+        const float2 ab = chunks[(size_t)k * g.width + j];
         S[j] = fmaf(ab.x, S[j], ab.y);
       }
-  } else {
-#pragma unroll
-    for (int j = 0; j < VEC; ++j) S[j] = s.start > 0 ? held[j] : 0.f;
   }
-  const T* row = x + (size_t)s.row0 * g.stride + c;
-  T* out = y + (size_t)s.row0 * g.width + c;
-  for (int t0 = first; t0 < last; t0 += GRU_AHEAD) {
-    float z[GRU_AHEAD][VEC], u[GRU_AHEAD][VEC], o[GRU_AHEAD][VEC];
-#pragma unroll
-    for (int i = 0; i < GRU_AHEAD; ++i) {
-      const T* at = row + (size_t)min(t0 + i, last - 1) * g.stride;
-      load_few<VEC>(at, z[i]);
-      load_few<VEC>(at + g.width, u[i]);
-      load_few<VEC>(at + 2 * g.width, o[i]);
-    }
-#pragma unroll
-    for (int i = 0; i < GRU_AHEAD; ++i) {
-      if (t0 + i >= last) break;
+  __syncthreads();
+  if (!WALK) {
+    if (wave > 0 || !in) return;
+    for (int w = 1; w < GRU_WAVES; ++w)
 #pragma unroll
       for (int j = 0; j < VEC; ++j) {
-        float p, q;
-        gru_step<T>(z[i][j] + zbias[j], u[i][j] + xbias[j], p, q);
-        S[j] = fmaf(p, S[j], q);
-        o[i][j] = S[j] * (o[i][j] * logistic<T>(o[i][j]));
+        const float2 ab = folded[w][lane * VEC + j];
+        a[j] *= ab.x;
+        b[j] = fmaf(ab.x, b[j], ab.y);
       }
-      store_few<VEC>(out + (size_t)(t0 + i) * g.width, o[i]);
-    }
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) chunks[(size_t)(chunk + 1) * g.width + j] = make_float2(a[j], b[j]);
+    return;
   }
-  if (last == s.rows)
+  for (int w = 0; w < wave; ++w)
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) {
+      const float2 ab = folded[w][lane * VEC + j];
+      S[j] = fmaf(ab.x, S[j], ab.y);
+    }
+  T* out = y + (size_t)(s.row0 + t0) * g.width + c;
+#pragma unroll
+  for (int i = 0; i < GRU_TOKENS; ++i) {
+    const bool live = t0 + i < s.rows;
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) {
+      S[j] = live ? fmaf(z[i][j], S[j], u[i][j]) : S[j];
+      o[i][j] = S[j] * (o[i][j] * logistic<T>(o[i][j]));
+    }
+    if (live && in) store_few<VEC>(out + (size_t)i * g.width, o[i]);
+  }
+  if (in && t0 < s.rows && t0 + GRU_TOKENS >= s.rows)   // the wave of the span's last row
 #pragma unroll
     for (int j = 0; j < VEC; ++j) state[(size_t)(2 * slot + ((s.start + s.rows - 1) & 1)) * g.width + c + j] = S[j];
+}
+
+// A span's rows one after the other.
+template <typename T, int VEC>
+__global__ __launch_bounds__(256) void min_gru_rows_kernel(const T* __restrict__ x, const bf16_t* __restrict__ zb, const bf16_t* __restrict__ xb,
+                                                           float* __restrict__ state, const int* __restrict__ spans, T* __restrict__ y, GruShape g) {
+  const int slot = blockIdx.y, c = (blockIdx.x * 256 + threadIdx.x) * VEC;
+  const Span s = span_of(spans, slot, g.rows);
+  if (s.rows == 0 || c >= g.width) return;
+  float zbias[VEC], xbias[VEC], S[VEC];
+  load_few<VEC>(zb + c, zbias);
+  load_few<VEC>(xb + c, xbias);
+#pragma unroll
+  for (int j = 0; j < VEC; ++j) S[j] = s.start > 0 ? state[(size_t)(2 * slot + ((s.start - 1) & 1)) * g.width + c + j] : 0.f;
+  const T* row = x + (size_t)s.row0 * g.stride + c;
+  T* out = y + (size_t)s.row0 * g.width + c;
+  for (int t = 0; t < s.rows; ++t, row += g.stride, out += g.width) {
+    float z[VEC], u[VEC], o[VEC];
+    load_few<VEC>(row, z);
+    load_few<VEC>(row + g.width, u);
+    load_few<VEC>(row + 2 * g.width, o);
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) {
+      float p, q;
+      gru_step<T>(z[j] + zbias[j], u[j] + xbias[j], p, q);
+      S[j] = fmaf(p, S[j], q);
+      o[j] = S[j] * (o[j] * logistic<T>(o[j]));
+    }
+    store_few<VEC>(out, o);
+  }
+#pragma unroll
+  for (int j = 0; j < VEC; ++j) state[(size_t)(2 * slot + ((s.start + s.rows - 1) & 1)) * g.width + c + j] = S[j];
 }
 
 template <typename T>
@@ -165,14 +194,15 @@ static int launch_min_gru(const T* x, const bf16_t* zb, const bf16_t* xb, float*
                           const GruShape& g, hipStream_t s) {
   const bool pairs = g.width % 2 == 0 && g.stride % 2 == 0 &&
                      ((((uintptr_t)x | (uintptr_t)y) & (2 * sizeof(T) - 1)) | (((uintptr_t)zb | (uintptr_t)xb) & 3)) == 0;
-  const int chunks = work != nullptr ? (g.rows + GRU_CHUNK - 1) / GRU_CHUNK : 1;
-  const dim3 grid((g.width + (pairs ? 511 : 255)) / (pairs ? 512 : 256), chunks, g.slots);
-#define IRON_GRU(VEC)                                                                                                             \
-  if (work != nullptr) {                                                                                                          \
-    hipLaunchKernelGGL((min_gru_fold_kernel<T, VEC>), grid, dim3(256), 0, s, x, zb, xb, state, spans, work, g);                   \
-    hipLaunchKernelGGL((min_gru_kernel<T, VEC, true>), grid, dim3(256), 0, s, x, zb, xb, state, spans, work, y, g);               \
-  } else {                                                                                                                        \
-    hipLaunchKernelGGL((min_gru_kernel<T, VEC, false>), grid, dim3(256), 0, s, x, zb, xb, state, spans, work, y, g);              \
+  const int vec = pairs ? 2 : 1;
+  const dim3 chunks((g.width + 64 * vec - 1) / (64 * vec), (g.rows + GRU_CHUNK - 1) / GRU_CHUNK, g.slots);
+  const dim3 rows((g.width + 256 * vec - 1) / (256 * vec), g.slots);
+#define IRON_GRU(VEC)                                                                                                                \
+  if (work != nullptr) {                                                                                                             \
+    hipLaunchKernelGGL((min_gru_chunks_kernel<T, VEC, false>), chunks, dim3(GRU_WAVES * 64), 0, s, x, zb, xb, state, spans, work, y, g); \
+    hipLaunchKernelGGL((min_gru_chunks_kernel<T, VEC, true>), chunks, dim3(GRU_WAVES * 64), 0, s, x, zb, xb, state, spans, work, y, g);  \
+  } else {                                                                                                                           \
+    hipLaunchKernelGGL((min_gru_rows_kernel<T, VEC>), rows, dim3(256), 0, s, x, zb, xb, state, spans, y, g);                         \
   }
   if (pairs) { IRON_GRU(2) }
   else { IRON_GRU(1) }
