@@ -757,7 +757,8 @@ __global__ __launch_bounds__(512) void latent_step_mfma_kernel(const bf16_t* __r
   l += __shfl_xor(l, 32, 64);
   // The second team's sums join the first's, through the LDS its keys lay in.
   __syncthreads();
-  float* other = reinterpret_cast<float*>(dyn + 2 * TEAM_PARTS + TEAM_KEYS * pitch * 2);   // [16][rank_pad]
+  const int other_pitch = rank_pad + 4;   // (sixteen heads side by side over all banks)
+  float* other = reinterpret_cast<float*>(dyn + 2 * TEAM_PARTS + TEAM_KEYS * pitch * 2);   // [16][other_pitch]
   float* other_stats = reinterpret_cast<float*>(dyn + TEAM_PARTS + TEAM_KEYS * pitch * 2);
   if (team == 1) {
 #pragma unroll
@@ -765,7 +766,7 @@ __global__ __launch_bounds__(512) void latent_step_mfma_kernel(const bf16_t* __r
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         const int c = (wave + 4 * g) * 64 + (quad * 4 + r) * 4;
-        if (c < rank_pad) *reinterpret_cast<float4*>(other + lo16 * rank_pad + c) = make_float4(acc[g][0][r], acc[g][1][r], acc[g][2][r], acc[g][3][r]);
+        if (c < rank_pad) *reinterpret_cast<float4*>(other + lo16 * other_pitch + c) = make_float4(acc[g][0][r], acc[g][1][r], acc[g][2][r], acc[g][3][r]);
       }
     if (wave == 0 && quad == 0) {
       other_stats[2 * lo16] = m;
@@ -783,7 +784,7 @@ __global__ __launch_bounds__(512) void latent_step_mfma_kernel(const bf16_t* __r
     for (int r = 0; r < 4; ++r) {
       const int c = (wave + 4 * g) * 64 + (quad * 4 + r) * 4;
       if (c < a.rank) {
-        const float4 o = *reinterpret_cast<const float4*>(other + lo16 * rank_pad + c);
+        const float4 o = *reinterpret_cast<const float4*>(other + lo16 * other_pitch + c);
         *reinterpret_cast<float4*>(to.sums + part * a.rank + c) =
             make_float4(fmaf(acc[g][0][r], f0, o.x * f1), fmaf(acc[g][1][r], f0, o.y * f1), fmaf(acc[g][2][r], f0, o.z * f1), fmaf(acc[g][3][r], f0, o.w * f1));
       }
@@ -796,7 +797,7 @@ __global__ __launch_bounds__(512) void latent_step_mfma_kernel(const bf16_t* __r
 
 // The splits' sums become a head's latent, and V_h makes its values of it: a wave VALUE_ROWS value columns, whose
 // weights (CH 16-byte pieces a lane; 0: any rank, read where they are needed) are on their way from the start.
-constexpr int VALUE_ROWS = 8;
+constexpr int VALUE_ROWS = 8, VALUE_AHEAD = 16;   // ... and the splits whose sums are asked for together
 template <typename T, int CH>
 __global__ __launch_bounds__(256) void latent_values_kernel(StepParts from, const bf16_t* __restrict__ up, const bf16_t* __restrict__ sink,
                                                             const int* __restrict__ spans, T* __restrict__ y, LatentShape a, int splits) {
@@ -824,20 +825,27 @@ __global__ __launch_bounds__(256) void latent_values_kernel(StepParts from, cons
   float top = sunk, total = 0.f;
   for (int i = lane; i < k.live; i += 64) top = fmaxf(top, from.stats[2 * (part + (size_t)i * a.heads)]);
   top = wave_max(top);
-  for (int i = lane; i < k.live; i += 64) {
-    const float share = latent_exp2<T>(from.stats[2 * (part + (size_t)i * a.heads)] - top);
+  const int padded = (k.live + VALUE_AHEAD - 1) & ~(VALUE_AHEAD - 1);   // (past the last: no share of the last)
+  for (int i = lane; i < padded; i += 64) {
+    const size_t at = 2 * (part + (size_t)min(i, k.live - 1) * a.heads);
+    const float share = i < k.live ? latent_exp2<T>(from.stats[at] - top) : 0.f;
     if (wave == 0) shares[i] = share;
-    total = fmaf(share, from.stats[2 * (part + (size_t)i * a.heads) + 1], total);
+    total = fmaf(share, from.stats[at + 1], total);
   }
   total = wave_sum(total) + (sink != nullptr ? latent_exp2<T>(sunk - top) : 0.f);
   __syncthreads();
   const float inv = 1.0f / total;
   for (int c = t; c < ((a.rank + 511) & ~511); c += 256) {
     float sum = 0.f;
-    if (c < a.rank)
-#pragma unroll 16
-      for (int i = 0; i < k.live; ++i) sum = fmaf(from.sums[(part + (size_t)i * a.heads) * a.rank + c], shares[i], sum);
-    latent[c] = sum * inv;
+    const int col = min(c, a.rank - 1);
+    for (int i = 0; i < padded; i += VALUE_AHEAD) {
+      float v[VALUE_AHEAD];
+#pragma unroll
+      for (int j = 0; j < VALUE_AHEAD; ++j) v[j] = from.sums[(part + (size_t)min(i + j, k.live - 1) * a.heads) * a.rank + col];
+#pragma unroll
+      for (int j = 0; j < VALUE_AHEAD; ++j) sum = fmaf(v[j], shares[i + j], sum);
+    }
+    latent[c] = c < a.rank ? sum * inv : 0.f;
   }
   __syncthreads();
 #pragma unroll
@@ -991,7 +999,7 @@ extern "C" int iron_mha_latent(const void* q, const void* latents, const void* s
                            (const bf16_t*)shared_keys, spans, parts, a, splits);
     }
     const dim3 vg(heads, (vdim + 4 * VALUE_ROWS - 1) / (4 * VALUE_ROWS), slots);
-    const size_t vlds = (size_t)(splits + ((rank + 511) & ~511)) * 4;
+    const size_t vlds = (size_t)(splits + VALUE_AHEAD + ((rank + 511) & ~511)) * 4;
 #define IRON_VALUES_CH(T, CH) hipLaunchKernelGGL((latent_values_kernel<T, CH>), vg, dim3(256), vlds, s, parts, up, sink, spans, (T*)y, a, splits)
 #define IRON_VALUES(T)                                  \
   {                                                     \

@@ -1,4 +1,4 @@
-// A gated recurrence whose gates read the current token alone, element by element over `width` channels:
+// minGRU over `width` channels, each a state of its own that a gate z moves towards a candidate c:
 //
 //   S_t = (1 - z) S_(t-1) + z c,   z = sigmoid(zx + zb),   c = u + 1/2 where u = ux + ub >= 0, else sigmoid(u)
 //   y_t = S_t silu(gx)

@@ -209,8 +209,7 @@ class StreamLayer(iron.Graph):
 
 
 class GatedRecurrence(iron.Graph):
-    """minGRU: a state a channel, moved towards a candidate by a gate, both of the current token alone, and read
-    through a SiLU gate.  ``proj`` is one packed projection (z, x, g and the layer's gate)."""
+    """minGRU: a state a channel that a gate moves towards a candidate, read through a SiLU gate.  ``proj`` is one packed projection (z, x, g and the layer's gate)."""
 
     def __init__(self, width, *, inner, gate, dtype, precision):
         self.inner, self.dtype, self.own = inner, dtype, 3 * inner

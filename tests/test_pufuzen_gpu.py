@@ -114,7 +114,7 @@ def test_the_recurrence_goes_on_where_a_portion_ends(cuda, chunked):
 # ---------------------------------------------------------------- latent attention
 
 # heads, dim, rot, vdim, rank, window (None: everything), a sink
-SIZES = [(4, 32, 32, 48, 64, None, True), (3, 24, 0, 80, 40, 37, False), (17, 16, 32, 24, 128, None, True), (1, 64, 64, 64, 512, None, False),
+SIZES = [(4, 40, 32, 56, 72, None, True), (3, 24, 0, 80, 40, 37, False), (17, 16, 32, 24, 128, None, True), (1, 64, 64, 64, 512, None, False),
          (2, 128, 64, 128, 320, 130, True), (2, 200, 0, 160, 96, 65, False), (5, 11, 6, 7, 19, None, True), (3, 12, 0, 20, 9, 1, False),
          (2, 128, 64, 128, 320, None, True), (3, 128, 0, 128, 64, None, False),
          (6, 8, 40, 256, 24, 9, True), (16, 96, 32, 64, 256, 64, False)]
