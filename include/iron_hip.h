@@ -384,13 +384,20 @@ int iron_gemm_few_bf16(const uint16_t* A, const uint16_t* B, const uint16_t* B2,
  * that starts at position 0 reads none, so a slot needs no clearing between sequences.
  * `is_float`: void* activations are float instead of bf16 (a model that runs in 32 bits throughout). */
 
-/* x[i] = table[ids[i]] widened to float, for i < *valid (or rows); ids outside the table are skipped. */
-int iron_stream_embed(const uint16_t* table, const int* ids, float* x, int rows, int table_rows, int cols,
+/* x[i] = table[ids[i]] widened to float, for i < *valid (or rows); ids outside the table are skipped.  also (may be
+ * NULL): the same rows once more. */
+int iron_stream_embed(const uint16_t* table, const int* ids, float* x, float* also, int rows, int table_rows, int cols,
                       const int* valid, void* stream);
-/* The stream's rows: with y, x += rmsnorm(y) * back_gain in place; with h, h = rmsnorm(x) * gain of the
- * rows as they then stand.  Float throughout, h rounded once. */
-int iron_stream_rows(float* x, const void* y, const uint16_t* back_gain, const uint16_t* gain, void* h, int rows,
-                     int cols, float eps, int is_float, const int* valid, void* stream);
+/* The stream's rows: with y, x += rmsnorm(y + y_bias) * (unit + back_gain) in place (y_bias may be NULL); with h,
+ * h = rmsnorm(x) * (unit + gain) of the rows as they then stand.  Float throughout, h rounded once. */
+int iron_stream_rows(float* x, const void* y, const uint16_t* y_bias, const uint16_t* back_gain, const uint16_t* gain, void* h,
+                     int rows, int cols, float eps, float unit, int is_float, const int* valid, void* stream);
+/* The stream's rows: with y, as above; with planes (index + 1 or more planes of plane_rows rows), the rows as they then
+ * stand become plane `index`, and the sum of weights[j] times plane j over j <= index takes their place; with h, h is
+ * the rows as they then stand, rounded once. */
+int iron_stream_depth_rows(float* x, const void* y, const uint16_t* y_bias, const uint16_t* back_gain, float* planes,
+                           const uint16_t* weights, int plane_rows, int index, void* h, int rows, int cols, float eps,
+                           float unit, int is_float, const int* valid, void* stream);
 /* x += (y + y_bias) * sigmoid(gate + gate_bias) in place, gate columns gate_at .. of rows of gate_stride (y_bias
  * may be NULL); with h, h = rmsnorm(x) * gain of the rows as they then stand.  Float throughout, h rounded once. */
 int iron_stream_gated_rows(float* x, const void* y, const uint16_t* y_bias, const void* gate, const uint16_t* gate_bias,
@@ -408,6 +415,9 @@ int iron_softcap(const void* x, float* y, uint16_t* rounded, int rows, int cols,
 /* y = act(gate) * up in float; activation 1 SiLU, 2 GELU (tanh form), 3 ReLU. */
 int iron_act_mul_f32(const float* gate, const float* up, float* y, int rows, int cols, int activation,
                      const int* valid, void* stream);
+/* y = act(x), rounded once; activation as above. */
+int iron_activation(const void* x, void* y, int rows, int cols, int activation, int is_float, const int* valid,
+                    void* stream);
 /* y = x w^T, x (rows, k), w (n, k) bf16, y (rows, n); float sums of float products, any sizes. */
 int iron_linear_any(const void* x, const uint16_t* w, void* y, int rows, int n, int k, int is_float,
                     const int* valid, void* stream);
@@ -505,16 +515,51 @@ int iron_decode_delta_bf16(const uint16_t* x, const uint16_t* taps_w, const uint
                            const uint16_t* norm, uint16_t* inputs, float* state, const int* spans, uint16_t* out,
                            int slots, int rows, int stride, int heads, int kv_heads, int dim, int vdim, int taps,
                            int gate_at, int b_at, int a_at, float eps, void* stream);
+/* Rows [q heads | k heads | v heads] of a packed projection made ready to be attended: q and k (+ bias) RMS-normed a head
+ * with q_gain / k_gain (dim), their first `turned` columns turned in neighbouring pairs by their position's row of angles
+ * (cos and sin side by side; positions behind the table's last row read that), q times scale * temp[head]; v (+ bias), with
+ * first (rows of first_stride, columns first_at ..) blended to (1 - share) v + share first. */
+int iron_turned_heads(const void* x, void* y, const uint16_t* bias, const uint16_t* q_gain, const uint16_t* k_gain,
+                      const uint16_t* temp, const float* angles, const uint16_t* share, const void* first,
+                      int first_stride, int first_at, const int* spans, int slots, int rows, int stride, int heads,
+                      int kv_heads, int dim, int vdim, int turned, int angle_rows, float scale, float eps,
+                      int is_float, const int* valid, void* stream);
+/* Attention of such rows within chunks of `chunk` positions: softmax a head over the chunk's positions up to the row's own,
+ * the heads' weights mixed by talk (heads, heads), each head's mixed weights applied to its own values.  Position p's key
+ * and value live in row p % ring of the slot's ring, ring = chunk.  single: every span is one row at most. */
+int iron_mha_talking(const void* x, void* keys, void* values, const uint16_t* talk, const int* spans, void* out, int slots,
+                     int rows, int stride, int heads, int kv_heads, int dim, int vdim, int chunk, int ring, int single,
+                     int is_float, void* stream);
+/* mLSTM: per head S <- keep S + write k v^T, n <- keep n + write k with m' = max(f + m, i), keep = exp(f + m - m'), write =
+ * exp(i - m'); i = cap tanh((gate + i_bias) / cap), f = log sigmoid of the same of its gate.  x: rows [q | k | v | ..],
+ * gates at columns i_at and f_at.  state: (slots, heads, dim, vdim + 1), n the last column; tops: (slots, 2, heads), m behind
+ * position p in row p % 2.  o: rows [S^T q dim^-1/2 (heads * vdim) | n . q dim^-1/2 (heads) | m (heads)], float. */
+int iron_matrix_memory(const void* x, const uint16_t* i_bias, const uint16_t* f_bias, float* state, float* tops,
+                       const int* spans, float* o, int slots, int rows, int stride, int heads, int dim, int vdim,
+                       int i_at, int f_at, float cap, int is_float, void* stream);
+/* y = o / (max(|n . q|, exp(-m)) + floor), RMS-normed a head, times gain (heads * dim) and sigmoid(gate). */
+int iron_memory_gate(const float* o, const void* gate, const uint16_t* gain, void* y, int rows, int heads, int dim,
+                     int gate_stride, int gate_at, float floor, float eps, int is_float, const int* valid, void* stream);
+/* A row's `top` experts by the largest of its logits w h + bias (float), and their shares, a softmax over the chosen logits. */
+int iron_router(const void* h, const uint16_t* w, const uint16_t* bias, int* ids, float* shares, int rows, int cols,
+                int experts, int top, int is_float, const int* valid, void* stream);
+/* y = sum over a row's experts e of share * down_e (act(gate_e h) * (up_e h)); gate and up (experts, ff, cols), down
+ * (experts, cols, ff).  activation: 1 SiLU, 2 GELU (tanh form), 3 ReLU. */
+int64_t iron_experts_workspace_bytes(int rows, int cols, int ff, int experts, int top, int is_float);
+int iron_experts(const void* h, const uint16_t* gate, const uint16_t* up, const uint16_t* down, const int* ids,
+                 const float* shares, void* y, void* workspace, int rows, int cols, int ff, int experts, int top,
+                 int activation, int is_float, const int* valid, void* stream);
+
 /* One row's product with its input made and its output taken in the same launch, bf16; each computes what the entry
  * points above and iron_gemv_bf16 compute in turn.
- * stream_product: input 0 the bf16 row x (K); 1 the float row x, 2 the bf16 row x, RMS-normed with gain; 3 slot 0's
+ * stream_product: input 0 the bf16 row x (K); 1 the float row x, 2 the bf16 row x, RMS-normed with unit + gain; 3 slot 0's
  * iron_min_gru over the row x = [zx | ux | gx] (width K, biases b0 and b1); 4 iron_poly_norm (bias b0, coefficients
  * gain).  Output: the row y (M), inputs 0 to 2; or iron_stream_gated_rows on stream_row (M), inputs 0, 3 and 4.
  * latent_query: iron_latent_rows of slot 0's one row x (whole 16-byte pieces), and q = W (M, q_rank) times the
  * query's latent. */
 int iron_stream_product_bf16(int input, const void* x, const uint16_t* gain, const uint16_t* b0, const uint16_t* b1,
-                             float* state, const int* spans, float eps, const uint16_t* W, int M, int K, uint16_t* y,
-                             float* stream_row, const uint16_t* y_bias, const uint16_t* gate, const uint16_t* gate_bias,
+                             float* state, const int* spans, float eps, float unit, const uint16_t* W, int M,
+                             int K, uint16_t* y, float* stream_row, const uint16_t* y_bias, const uint16_t* gate, const uint16_t* gate_bias,
                              void* stream);
 int iron_latent_query_bf16(const uint16_t* x, const uint16_t* q_gain, const uint16_t* c_gain, const float* angles,
                            const int* spans, const uint16_t* W, uint16_t* q, uint16_t* latents, uint16_t* shared_keys,

@@ -89,8 +89,17 @@ SIGNATURES = {
     "iron_sample_advance_bf16": (c_int, [_P, c_int, _P, c_int, _P, c_int, _P, _P, _P, c_int, _P, _P, _P, c_int, _P,
                                          c_int, _P]),
     "iron_gemm_few_bf16": (c_int, [_P, _P, _P, _P, c_int, c_int, c_int, c_int, _P]),
-    "iron_stream_embed": (c_int, [_P, _P, _P, c_int, c_int, c_int, _P, _P]),
-    "iron_stream_rows": (c_int, [_P, _P, _P, _P, _P, c_int, c_int, c_float, c_int, _P, _P]),
+    "iron_stream_embed": (c_int, [_P, _P, _P, _P, c_int, c_int, c_int, _P, _P]),
+    "iron_stream_rows": (c_int, [_P] * 6 + [c_int, c_int, c_float, c_float, c_int, _P, _P]),
+    "iron_stream_depth_rows": (c_int, [_P] * 6 + [c_int, c_int, _P, c_int, c_int, c_float, c_float, c_int, _P, _P]),
+    "iron_activation": (c_int, [_P, _P, c_int, c_int, c_int, c_int, _P, _P]),
+    "iron_turned_heads": (c_int, [_P] * 9 + [c_int, c_int, _P] + [c_int] * 9 + [c_float, c_float, c_int, _P, _P]),
+    "iron_mha_talking": (c_int, [_P] * 6 + [c_int] * 11 + [_P]),
+    "iron_matrix_memory": (c_int, [_P] * 7 + [c_int] * 8 + [c_float, c_int, _P]),
+    "iron_memory_gate": (c_int, [_P] * 4 + [c_int] * 5 + [c_float, c_float, c_int, _P, _P]),
+    "iron_router": (c_int, [_P] * 5 + [c_int] * 5 + [_P, _P]),
+    "iron_experts_workspace_bytes": (c_int64, [c_int] * 6),
+    "iron_experts": (c_int, [_P] * 8 + [c_int] * 7 + [_P, _P]),
     "iron_span_tails": (c_int, [_P, _P, _P, c_int, c_int, c_int, _P]),
     "iron_softcap": (c_int, [_P, _P, _P, c_int, c_int, c_int, c_float, c_float, c_int, _P]),
     "iron_stream_gated_rows": (c_int, [_P] * 5 + [c_int, c_int, _P, _P, c_int, c_int, c_float, c_int, _P, _P]),
@@ -120,7 +129,7 @@ SIGNATURES = {
         + [c_int] * 3 + [_P],
     ),
     "iron_decode_delta_bf16": (c_int, [_P] * 9 + [c_int] * 11 + [c_float, _P]),
-    "iron_stream_product_bf16": (c_int, [c_int] + [_P] * 6 + [c_float, _P, c_int, c_int] + [_P] * 6),
+    "iron_stream_product_bf16": (c_int, [c_int] + [_P] * 6 + [c_float, c_float, _P, c_int, c_int] + [_P] * 6),
     "iron_latent_query_bf16": (c_int, [_P] * 9 + [c_int] * 8 + [c_float, _P]),
     "iron_sample_slots_bf16": (c_int, [_P, c_int, c_int, _P, c_int, c_int, c_int, _P, c_int, _P, _P, _P, _P]),
     "iron_eval_words": (c_int, [_P, c_int, _P, c_int, _P]),

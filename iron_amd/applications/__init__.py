@@ -1,4 +1,5 @@
-"""The models wired from the shared decoder: Llama, Granite, Gemma 4's text decoder, Pegilix and Pufuzen."""
+"""The models wired from the shared decoder: Llama, Granite, Gemma 4's text decoder, Pegilix, Pufuzen and
+Tilarax."""
 
 from .gemma4 import Gemma4, Gemma4Config
 from .granite import Granite, GraniteConfig
@@ -6,6 +7,7 @@ from .llama import Llama, LlamaConfig
 from .pegilix import Pegilix, PegilixConfig
 from .pufuzen import Pufuzen, PufuzenConfig
 from .registry import ARCHITECTURES, load_model, model_class
+from .tilarax import Tilarax, TilaraxConfig
 
 __all__ = ["ARCHITECTURES", "Gemma4", "Gemma4Config", "Granite", "GraniteConfig", "Llama", "LlamaConfig", "Pegilix",
-           "PegilixConfig", "Pufuzen", "PufuzenConfig", "load_model", "model_class"]
+           "PegilixConfig", "Pufuzen", "PufuzenConfig", "Tilarax", "TilaraxConfig", "load_model", "model_class"]

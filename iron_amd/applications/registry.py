@@ -10,6 +10,7 @@ from .granite import Granite
 from .llama import Llama
 from .pegilix import Pegilix
 from .pufuzen import Pufuzen
+from .tilarax import Tilarax
 
 # ``architecture`` (or an entry of ``architectures``) -> the class that serves it
 ARCHITECTURES = {
@@ -19,6 +20,7 @@ ARCHITECTURES = {
     "Gemma4ForConditionalGeneration": Gemma4,
     "Pegilix": Pegilix,
     "Pufuzen": Pufuzen,
+    "Tilarax": Tilarax,
 }
 
 

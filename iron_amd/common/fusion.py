@@ -37,6 +37,7 @@ in a batched decoder's decode step (bf16; a float32 stream, layers with a state)
 and in either,
 
   StreamAdd, StreamNorm                                  => iron_stream_rows
+  [StreamAdd,] [DepthAverage,] [StreamCast] (two of them) => iron_stream_depth_rows
   StreamGatedAdd, StreamNorm                             => iron_stream_gated_rows
   RMSNorm, ElementwiseAdd (a sandwich layer's residual)  => iron_rmsnorm_add_bf16
 
@@ -321,7 +322,7 @@ def plan(recording, tensor: Callable[[Any], Any], word: Callable[[Any], Any],
                 return None
             args = dict(W=tensor(g.inputs["A"]), x=tensor(s.inputs["x"]).reshape(-1), gain=tensor(s.inputs["weight"]),
                         y=tensor(g.outputs["C"]).reshape(-1))
-            kw = dict(input="stream_norm", M=g.op.M, K=g.op.K, eps=float(s.op.epsilon))
+            kw = dict(input="stream_norm", M=g.op.M, K=g.op.K, eps=float(s.op.epsilon), unit=float(s.op.unit))
             return Fused("stream_norm_gemv", j, 2, lambda a=args, kw=kw: kernels.stream_product(**a, **kw))
         if _name(s) == "MinGRU":
             y = s.outputs["y"]
@@ -349,6 +350,39 @@ def plan(recording, tensor: Callable[[Any], Any], word: Callable[[Any], Any],
             args["x"] = tensor(s.inputs["B"]).reshape(-1)
             return Fused("gated_product", j, 2, lambda a=args, kw=kw: kernels.stream_product(input="row", **a, **kw))
         return None
+
+    def depth_rows_at(j):
+        """The launch for a block's output into the stream, the average over what it was behind every layer and the row a
+        block reads of it, where two or three of them follow each other on the same rows -- or None."""
+        found, at = {}, j
+        for name in ("StreamAdd", "DepthAverage", "StreamCast"):
+            st = steps[at] if at < len(steps) else None
+            if st is None or _name(st) != name or set(st.values) - {"valid"}:
+                continue
+            if found:
+                ahead = next(iter(found.values()))
+                if not (_same_view(st.inputs["x"], ahead.outputs["x"]) and st.values.get("valid") == ahead.values.get("valid")
+                        and (st.op.rows, st.op.cols) == (ahead.op.rows, ahead.op.cols)):
+                    break
+            found[name] = st
+            at += 1
+        add, depth, cast = (found.get(n) for n in ("StreamAdd", "DepthAverage", "StreamCast"))
+        if len(found) < 2 or (add is not None and cast is not None and add.op.dtype is not cast.op.dtype):
+            return None
+        first = next(iter(found.values()))
+        args = dict(x=tensor(first.inputs["x"]))
+        kw = dict(rows=first.op.rows, cols=first.op.cols, valid=word(first.values.get("valid")))
+        if add is not None:
+            args |= dict(y=tensor(add.inputs["y"]), back_gain=tensor(add.inputs["weight"]))
+            if "y_bias" in add.inputs:
+                args["y_bias"] = tensor(add.inputs["y_bias"])
+            kw |= dict(eps=float(add.op.epsilon), unit=float(add.op.unit))
+        if depth is not None:
+            args |= dict(planes=tensor(depth.inputs["planes"]), weights=tensor(depth.inputs["weights"]))
+            kw |= dict(plane_rows=depth.op.plane_rows, index=depth.op.count - 1)
+        if cast is not None:
+            args["h"] = tensor(cast.outputs["y"])
+        return Fused("stream_depth_rows", j, at - j, lambda a=args, kw=kw: kernels.stream_depth_rows(**a, **kw))
 
     def latent_query_at(j):
         """The launch for a single slot's latents and the product of its queries -- or None."""
@@ -683,15 +717,20 @@ def plan(recording, tensor: Callable[[Any], Any], word: Callable[[Any], Any],
                             residual=tensor(other).reshape(-1), y=tensor(mu.outputs["y"]).reshape(-1))
                 kw = dict(M=s.op.M, K=s.op.K, epilogue=5 if _name(ac) == "SiLU" else 4)
                 got = Fused("gemv_act_mul", i, 3, lambda a=args, kw=kw: kernels.gemv_fused(**a, **kw))
+        elif _name(s) in ("StreamAdd", "DepthAverage") and (got := depth_rows_at(i)) is not None:
+            pass
         elif _name(s) == "StreamAdd" and i + 1 < len(steps) and _name(steps[i + 1]) == "StreamNorm":
             # a block's output into the stream and the next block's norm out of it: one pass over the row
             nm = steps[i + 1]
-            if (_same_view(nm.inputs["x"], s.outputs["x"]) and nm.op.dtype is s.op.dtype and nm.op.epsilon == s.op.epsilon
+            if (_same_view(nm.inputs["x"], s.outputs["x"]) and nm.op.dtype is s.op.dtype
+                    and (nm.op.epsilon, nm.op.unit) == (s.op.epsilon, s.op.unit)
                     and (nm.op.rows, nm.op.cols) == (s.op.rows, s.op.cols) and nm.values.get("valid") == s.values.get("valid")
                     and set(nm.values) <= {"valid"} and set(s.values) <= {"valid"}):
                 args = dict(x=tensor(s.inputs["x"]), y=tensor(s.inputs["y"]), back_gain=tensor(s.inputs["weight"]),
                             h=tensor(nm.outputs["y"]), gain=tensor(nm.inputs["weight"]))
-                kw = dict(rows=s.op.rows, cols=s.op.cols, eps=float(s.op.epsilon), valid=word(s.values.get("valid")))
+                if "y_bias" in s.inputs:
+                    args["y_bias"] = tensor(s.inputs["y_bias"])
+                kw = dict(rows=s.op.rows, cols=s.op.cols, eps=float(s.op.epsilon), unit=float(s.op.unit), valid=word(s.values.get("valid")))
                 got = Fused("stream_add_norm", i, 2, lambda a=args, kw=kw: kernels.stream_rows(**a, **kw))
         elif (_name(s) in ("StreamNorm", "MinGRU", "PolyNorm") or gemv_row(s)) and (got := stream_product_at(i)) is not None:
             pass

@@ -25,6 +25,7 @@ struct StreamIn {
   float* state;               // IN_GRU
   const int* spans;           // IN_GRU, OUT_LATENT
   float eps;
+  float unit;                 // added to a norm's gains
 };
 struct StreamOut {
   bf16_t* y;
@@ -112,7 +113,7 @@ struct Made {
         float g[8];
         unpack8(v[IN == IN_ROW_NORM ? ROWS - 1 : 0][i], g);
 #pragma unroll
-        for (int j = 0; j < 8; ++j) x[i][j] = x[i][j] * inv * g[j];
+        for (int j = 0; j < 8; ++j) x[i][j] = x[i][j] * inv * (in.unit + g[j]);
         out[i] = pack8(x[i]);
       }
       return;
@@ -252,7 +253,7 @@ static int launch_stream_product(const bf16_t* W, const StreamIn& in, const Stre
 using namespace iron;
 
 extern "C" int iron_stream_product_bf16(int input, const void* x, const uint16_t* gain, const uint16_t* b0, const uint16_t* b1, float* state,
-                                        const int* spans, float eps, const uint16_t* W, int M, int K, uint16_t* y, float* stream_row,
+                                        const int* spans, float eps, float unit, const uint16_t* W, int M, int K, uint16_t* y, float* stream_row,
                                         const uint16_t* y_bias, const uint16_t* gate, const uint16_t* gate_bias, void* stream) {
   IRON_REQUIRE(input >= IN_ROW && input <= IN_POLY, "stream_product: input (%d) is 0 to 4", input);
   IRON_REQUIRE(x && W && ((y != nullptr) != (stream_row != nullptr)), "stream_product: null operand, or not one output");
@@ -264,7 +265,7 @@ extern "C" int iron_stream_product_bf16(int input, const void* x, const uint16_t
   IRON_REQUIRE(stream_row == nullptr || input != IN_STREAM_NORM, "stream_product: the stream is an input or the output");
   IRON_REQUIRE((((uintptr_t)x | (uintptr_t)W | (uintptr_t)b0 | (uintptr_t)b1 | (uintptr_t)state | (uintptr_t)spans |
                  (input == IN_POLY ? 0 : (uintptr_t)gain)) & 15) == 0, "stream_product: operands must be 16-byte aligned");
-  const StreamIn in{x, gain, b0, b1, state, spans, eps};
+  const StreamIn in{x, gain, b0, b1, state, spans, eps, unit};
   StreamOut out{};
   out.y = y;
   out.stream = stream_row;
@@ -296,7 +297,7 @@ extern "C" int iron_latent_query_bf16(const uint16_t* x, const uint16_t* q_gain,
   IRON_REQUIRE(turned <= rot && (turned == 0 || (angles && angle_rows > 0)), "latent_query: %d of %d columns turn, by a table of %d rows", turned, rot, angle_rows);
   IRON_REQUIRE((((uintptr_t)x | (uintptr_t)q_gain | (uintptr_t)c_gain | (uintptr_t)spans | (uintptr_t)W | (uintptr_t)latents | (uintptr_t)shared_keys) & 15) == 0,
                "latent_query: operands must be 16-byte aligned");
-  const StreamIn in{x, q_gain, nullptr, nullptr, nullptr, spans, eps};
+  const StreamIn in{x, q_gain, nullptr, nullptr, nullptr, spans, eps, 0.f};
   StreamOut out{};
   out.y = q;
   out.row = x;

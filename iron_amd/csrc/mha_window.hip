@@ -9,7 +9,7 @@
 //   rows kernel:    a block a query row and head, waves splitting the keys (decode; either type)
 //   prefill kernel: bf16 MFMA flash attention, 64 or 128 queries a block
 #include "../../include/iron_hip.h"
-#include "rows.h"
+#include "window.h"
 
 namespace iron {
 
@@ -22,21 +22,6 @@ struct WindowShape {
 };
 
 constexpr float LOG2E = 1.4426950408889634f;
-
-// ------------------------------------------------------------------ the ring
-template <typename T>
-__global__ __launch_bounds__(256) void window_store_kernel(const T* __restrict__ x, T* __restrict__ keys, T* __restrict__ values,
-                                                           const int* __restrict__ spans, WindowShape a) {
-  const Span s = span_of(spans, blockIdx.y, a.rows);
-  const int i = s.rows - 1 - (int)blockIdx.x;   // from the span's last row back
-  if (i < 0 || (int)blockIdx.x >= a.ring) return;
-  const int at = (s.start + i) % a.ring, nk = a.kv_heads * a.dim, nv = a.kv_heads * a.vdim;
-  const T* row = x + (size_t)(s.row0 + i) * a.stride + a.heads * a.dim;
-  T* kd = keys + ((size_t)blockIdx.y * a.ring + at) * nk;
-  T* vd = values + ((size_t)blockIdx.y * a.ring + at) * nv;
-  for (int c = threadIdx.x; c < nk; c += 256) kd[c] = row[c];
-  for (int c = threadIdx.x; c < nv; c += 256) vd[c] = row[nk + c];
-}
 
 // --------------------------------------------------------------- row by row
 // NW waves to a query row and head.  A wave takes 64 keys at a time: a key a lane for the scores, then
@@ -478,10 +463,8 @@ extern "C" int iron_mha_window(const void* x, void* keys, void* values, const fl
   }
 #undef IRON_WINDOW_ROWS
   // Attended: the span's last rows go into the ring.
-  const dim3 grid(rows < ring ? rows : ring, slots);
-  if (is_float)
-    hipLaunchKernelGGL((window_store_kernel<float>), grid, dim3(256), 0, s, (const float*)x, (float*)keys, (float*)values, spans, a);
-  else
-    hipLaunchKernelGGL((window_store_kernel<bf16_t>), grid, dim3(256), 0, s, (const bf16_t*)x, (bf16_t*)keys, (bf16_t*)values, spans, a);
+  const PackedHeads packed{rows, stride, heads, kv_heads, dim, vdim, ring};
+  if (is_float) launch_ring_store<float>(x, keys, values, spans, packed, slots, s);
+  else launch_ring_store<bf16_t>(x, keys, values, spans, packed, slots, s);
   IRON_LAUNCH_CHECK();
 }

@@ -1,6 +1,7 @@
-// A decoder's residual stream held in float32: rows gathered from a bf16 table into it, a row's RMS
-// norm out of it, a block's normed or gated output added to it, and the head's scale and soft cap.  One rounding, to the
-// activation type, where a row leaves the stream; bandwidth bound, a block a row.
+// A decoder's residual stream held in float32: rows gathered from a bf16 table into it, a row or its RMS
+// norm out of it, a block's normed or gated output added to it, a weighted sum of what it was after every layer in its
+// place, and the head's scale and soft cap.  One rounding, to the activation type, where a row leaves the stream;
+// bandwidth bound, a block a row.
 #include "../../include/iron_hip.h"
 #include "rows.h"
 
@@ -8,8 +9,8 @@ namespace iron {
 
 template <int VEC>
 __global__ __launch_bounds__(256) void stream_embed_kernel(const bf16_t* __restrict__ table, const int* __restrict__ ids,
-                                                           float* __restrict__ x, int rows, int table_rows, int cols,
-                                                           const int* __restrict__ valid) {
+                                                           float* __restrict__ x, float* __restrict__ also, int rows,
+                                                           int table_rows, int cols, const int* __restrict__ valid) {
   const int row = blockIdx.x;
   if (row >= bound_or(valid, rows)) return;
   const int id = ids[row];
@@ -18,6 +19,7 @@ __global__ __launch_bounds__(256) void stream_embed_kernel(const bf16_t* __restr
     float f[VEC];
     load_vec<VEC>(table + (size_t)id * cols + c, f);
     store_vec<VEC>(x + (size_t)row * cols + c, f);
+    if (also != nullptr) store_vec<VEC>(also + (size_t)row * cols + c, f);
   }
 }
 
@@ -29,7 +31,7 @@ __device__ __forceinline__ float row_total(float v, float* part) {
   return part[0] + part[1] + part[2] + part[3];
 }
 
-// What joins the stream: nothing, a block's row normed (rmsnorm(y) * wb), or a block's row gated
+// What joins the stream: nothing, a block's row normed (rmsnorm(y + yb) * (unit + wb)), or a block's row gated
 // ((y + yb) * sigmoid(gate + gb), the gate columns `at` .. of rows of `stride`).
 enum { ADD_NONE = 0, ADD_NORMED = 1, ADD_GATED = 2 };
 struct StreamGate {
@@ -37,16 +39,28 @@ struct StreamGate {
   const bf16_t *bias, *y_bias;   // gb, yb (yb may be null)
   int stride, at;
 };
-// x += what ADD says, in place.  NORM: h = rmsnorm(x) * w of the row as it then stands.
+// What leaves it: nothing, its norm (rmsnorm(x) * (unit + w)), or the row itself.
+enum { OUT_NONE = 0, OUT_NORM = 1, OUT_CAST = 2 };
+// What it was: plane j of `planes` is the stream behind layer j, `plane` floats each; the row as it stands becomes
+// plane `index`, and the sum over j <= index of weights[j] times plane j takes its place.
+struct StreamDepth {
+  float* planes;
+  const bf16_t* weights;
+  size_t plane;
+  int index;
+};
+
+// x += what ADD says, in place; then (DEPTH) the weighted sum; then what OUT says.
 // A thread holds its first CH pieces of the row between the passes and re-reads the rest.
-template <typename T, int VEC, int CH, int ADD, bool NORM>
+template <typename T, int VEC, int CH, int ADD, int OUT, bool DEPTH>
 __global__ __launch_bounds__(256) void stream_rows_kernel(float* __restrict__ x, const T* __restrict__ y,
                                                           const bf16_t* __restrict__ wb, const bf16_t* __restrict__ w,
-                                                          T* __restrict__ h, int rows, int cols, float eps,
-                                                          const int* __restrict__ valid, StreamGate g) {
+                                                          T* __restrict__ h, int rows, int cols, float eps, float unit,
+                                                          const int* __restrict__ valid, StreamGate g, StreamDepth d) {
   __shared__ float part[4];
   const int row = blockIdx.x, first = threadIdx.x * VEC;
   constexpr int STEP = 256 * VEC;
+  constexpr bool NORM = OUT == OUT_NORM;
   float held[CH][VEC], gain[CH][VEC];
   if (NORM) {
 #pragma unroll
@@ -82,7 +96,7 @@ __global__ __launch_bounds__(256) void stream_rows_kernel(float* __restrict__ x,
         gated(first + i * STEP, f);
 #pragma unroll
         for (int j = 0; j < VEC; ++j) held[i][j] += f[j];
-        store_vec<VEC>(xr + first + i * STEP, held[i]);
+        if (!DEPTH) store_vec<VEC>(xr + first + i * STEP, held[i]);
       }
     for (int c = first + CH * STEP; c < cols; c += STEP) {
       float f[VEC], s[VEC];
@@ -95,19 +109,28 @@ __global__ __launch_bounds__(256) void stream_rows_kernel(float* __restrict__ x,
   }
   if (ADD == ADD_NORMED) {
     const T* yr = y + (size_t)row * cols;
+    auto biased = [&](int c, float (&f)[VEC]) {
+      load_vec<VEC>(yr + c, f);
+      if (g.y_bias != nullptr) {
+        float yb[VEC];
+        load_vec<VEC>(g.y_bias + c, yb);
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) f[j] += yb[j];
+      }
+    };
     float out[CH][VEC], back[CH][VEC];
     float ss = 0.f;
 #pragma unroll
     for (int i = 0; i < CH; ++i)
       if (first + i * STEP < cols) {
-        load_vec<VEC>(yr + first + i * STEP, out[i]);
+        biased(first + i * STEP, out[i]);
         load_vec<VEC>(wb + first + i * STEP, back[i]);
 #pragma unroll
         for (int j = 0; j < VEC; ++j) ss = fmaf(out[i][j], out[i][j], ss);
       }
     for (int c = first + CH * STEP; c < cols; c += STEP) {
       float f[VEC];
-      load_vec<VEC>(yr + c, f);
+      biased(c, f);
 #pragma unroll
       for (int j = 0; j < VEC; ++j) ss = fmaf(f[j], f[j], ss);
     }
@@ -116,17 +139,68 @@ __global__ __launch_bounds__(256) void stream_rows_kernel(float* __restrict__ x,
     for (int i = 0; i < CH; ++i)
       if (first + i * STEP < cols) {
 #pragma unroll
-        for (int j = 0; j < VEC; ++j) held[i][j] += out[i][j] * inv * back[i][j];
-        store_vec<VEC>(xr + first + i * STEP, held[i]);
+        for (int j = 0; j < VEC; ++j) held[i][j] += out[i][j] * inv * (unit + back[i][j]);
+        if (!DEPTH) store_vec<VEC>(xr + first + i * STEP, held[i]);
       }
     for (int c = first + CH * STEP; c < cols; c += STEP) {
       float f[VEC], b[VEC], s[VEC];
-      load_vec<VEC>(yr + c, f);
+      biased(c, f);
       load_vec<VEC>(wb + c, b);
       load_vec<VEC>(xr + c, s);
 #pragma unroll
-      for (int j = 0; j < VEC; ++j) s[j] += f[j] * inv * b[j];
+      for (int j = 0; j < VEC; ++j) s[j] += f[j] * inv * (unit + b[j]);
       store_vec<VEC>(xr + c, s);
+    }
+  }
+  if (DEPTH) {
+    auto averaged = [&](int c, float (&s)[VEC]) {
+      float* at = d.planes + (size_t)row * cols + c;
+      store_vec<VEC>(at + d.index * d.plane, s);
+      const float own = bf16_to_f32(d.weights[d.index]);
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) s[j] *= own;
+      int n = 0;
+      for (; n + 4 <= d.index; n += 4) {   // four planes' loads in flight
+        float f[4][VEC];
+#pragma unroll
+        for (int q = 0; q < 4; ++q) load_vec<VEC>(at + (n + q) * d.plane, f[q]);
+#pragma unroll
+        for (int q = 0; q < 4; ++q) {
+          const float by = bf16_to_f32(d.weights[n + q]);
+#pragma unroll
+          for (int j = 0; j < VEC; ++j) s[j] = fmaf(by, f[q][j], s[j]);
+        }
+      }
+      for (; n < d.index; ++n) {
+        float f[VEC];
+        load_vec<VEC>(at + n * d.plane, f);
+        const float by = bf16_to_f32(d.weights[n]);
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) s[j] = fmaf(by, f[j], s[j]);
+      }
+    };
+#pragma unroll
+    for (int i = 0; i < CH; ++i)
+      if (first + i * STEP < cols) {
+        averaged(first + i * STEP, held[i]);
+        store_vec<VEC>(xr + first + i * STEP, held[i]);
+      }
+    for (int c = first + CH * STEP; c < cols; c += STEP) {
+      float s[VEC];
+      load_vec<VEC>(xr + c, s);
+      averaged(c, s);
+      store_vec<VEC>(xr + c, s);
+    }
+  }
+  if (OUT == OUT_CAST) {
+    T* hr = h + (size_t)row * cols;
+#pragma unroll
+    for (int i = 0; i < CH; ++i)
+      if (first + i * STEP < cols) store_vec<VEC>(hr + first + i * STEP, held[i]);
+    for (int c = first + CH * STEP; c < cols; c += STEP) {
+      float f[VEC];
+      load_vec<VEC>(xr + c, f);
+      store_vec<VEC>(hr + c, f);
     }
   }
   if (NORM) {
@@ -149,15 +223,15 @@ __global__ __launch_bounds__(256) void stream_rows_kernel(float* __restrict__ x,
     for (int i = 0; i < CH; ++i)
       if (first + i * STEP < cols) {
 #pragma unroll
-        for (int j = 0; j < VEC; ++j) held[i][j] = held[i][j] * inv * gain[i][j];
+        for (int j = 0; j < VEC; ++j) held[i][j] = held[i][j] * inv * (unit + gain[i][j]);
         store_vec<VEC>(hr + first + i * STEP, held[i]);
       }
     for (int c = first + CH * STEP; c < cols; c += STEP) {
-      float f[VEC], g[VEC];
+      float f[VEC], gn[VEC];
       load_vec<VEC>(xr + c, f);
-      load_vec<VEC>(w + c, g);
+      load_vec<VEC>(w + c, gn);
 #pragma unroll
-      for (int j = 0; j < VEC; ++j) f[j] = f[j] * inv * g[j];
+      for (int j = 0; j < VEC; ++j) f[j] = f[j] * inv * (unit + gn[j]);
       store_vec<VEC>(hr + c, f);
     }
   }
@@ -195,6 +269,20 @@ __global__ __launch_bounds__(256) void act_mul_f32_kernel(const float* __restric
     const float g = gate[i];
     const float a = kind == 3 ? fmaxf(g, 0.f) : (kind == 1 ? g / (1.f + expf(-g)) : gelu_tanh_f32(g));
     y[i] = a * up[i];
+  }
+}
+
+// silu / gelu (tanh form) / relu, rounded once.
+template <typename T, int VEC>
+__global__ __launch_bounds__(256) void activation_kernel(const T* __restrict__ x, T* __restrict__ y, long n, int kind,
+                                                         const int* __restrict__ valid, int cols) {
+  if (valid != nullptr) n = min(n, (long)max(*valid, 0) * cols);
+  for (long i = ((long)blockIdx.x * 256 + threadIdx.x) * VEC; i < n; i += (long)gridDim.x * 256 * VEC) {
+    float f[VEC];
+    load_vec<VEC>(x + i, f);
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) f[j] = kind == 3 ? fmaxf(f[j], 0.f) : (kind == 1 ? f[j] / (1.f + expf(-f[j])) : gelu_tanh_f32(f[j]));
+    store_vec<VEC>(y + i, f);
   }
 }
 
@@ -240,18 +328,19 @@ __global__ __launch_bounds__(256) void linear_any_kernel(const T* __restrict__ x
     }
 }
 
-template <typename T, int ADD, bool NORM>
-static int launch_stream_rows(float* x, const T* y, const bf16_t* wb, const bf16_t* w, T* h, int rows, int cols, float eps,
-                              const int* valid, hipStream_t s, const StreamGate& g = StreamGate{nullptr, nullptr, nullptr, 8, 8}) {
-  const bool vec = cols % 8 == 0 && g.stride % 8 == 0 && g.at % 8 == 0 &&
+template <typename T, int ADD, int OUT, bool DEPTH = false>
+static int launch_stream_rows(float* x, const T* y, const bf16_t* wb, const bf16_t* w, T* h, int rows, int cols, float eps, float unit,
+                              const int* valid, hipStream_t s, const StreamGate& g = StreamGate{nullptr, nullptr, nullptr, 8, 8},
+                              const StreamDepth& d = StreamDepth{nullptr, nullptr, 0, 0}) {
+  const bool vec = cols % 8 == 0 && g.stride % 8 == 0 && g.at % 8 == 0 && d.plane % 4 == 0 &&
                    (((uintptr_t)x | (uintptr_t)y | (uintptr_t)wb | (uintptr_t)w | (uintptr_t)h | (uintptr_t)g.gate | (uintptr_t)g.bias |
-                     (uintptr_t)g.y_bias) & 15) == 0;
-  if (vec && cols <= 2048)
-    hipLaunchKernelGGL((stream_rows_kernel<T, 8, 1, ADD, NORM>), dim3(rows), dim3(256), 0, s, x, y, wb, w, h, rows, cols, eps, valid, g);
-  else if (vec)
-    hipLaunchKernelGGL((stream_rows_kernel<T, 8, 2, ADD, NORM>), dim3(rows), dim3(256), 0, s, x, y, wb, w, h, rows, cols, eps, valid, g);
-  else
-    hipLaunchKernelGGL((stream_rows_kernel<T, 1, 4, ADD, NORM>), dim3(rows), dim3(256), 0, s, x, y, wb, w, h, rows, cols, eps, valid, g);
+                     (uintptr_t)g.y_bias | (uintptr_t)d.planes) & 15) == 0;
+#define IRON_ROWS(VEC, CH) \
+  hipLaunchKernelGGL((stream_rows_kernel<T, VEC, CH, ADD, OUT, DEPTH>), dim3(rows), dim3(256), 0, s, x, y, wb, w, h, rows, cols, eps, unit, valid, g, d)
+  if (vec && cols <= 2048) IRON_ROWS(8, 1);
+  else if (vec) IRON_ROWS(8, 2);
+  else IRON_ROWS(1, 4);
+#undef IRON_ROWS
   IRON_LAUNCH_CHECK();
 }
 
@@ -264,32 +353,59 @@ static unsigned few_blocks(long n) {
 
 using namespace iron;
 
-extern "C" int iron_stream_embed(const uint16_t* table, const int* ids, float* x, int rows, int table_rows, int cols,
+extern "C" int iron_stream_embed(const uint16_t* table, const int* ids, float* x, float* also, int rows, int table_rows, int cols,
                                  const int* valid, void* stream) {
   IRON_REQUIRE(table && ids && x, "stream_embed: null operand");
   IRON_REQUIRE(rows > 0 && table_rows > 0 && cols > 0, "stream_embed: rows (%d), table_rows (%d), cols (%d) must be positive",
                rows, table_rows, cols);
-  if (cols % 8 == 0 && (((uintptr_t)table | (uintptr_t)x) & 15) == 0)
-    hipLaunchKernelGGL((stream_embed_kernel<8>), dim3(rows), dim3(256), 0, (hipStream_t)stream, table, ids, x, rows, table_rows, cols, valid);
+  if (cols % 8 == 0 && (((uintptr_t)table | (uintptr_t)x | (uintptr_t)also) & 15) == 0)
+    hipLaunchKernelGGL((stream_embed_kernel<8>), dim3(rows), dim3(256), 0, (hipStream_t)stream, table, ids, x, also, rows, table_rows, cols, valid);
   else
-    hipLaunchKernelGGL((stream_embed_kernel<1>), dim3(rows), dim3(256), 0, (hipStream_t)stream, table, ids, x, rows, table_rows, cols, valid);
+    hipLaunchKernelGGL((stream_embed_kernel<1>), dim3(rows), dim3(256), 0, (hipStream_t)stream, table, ids, x, also, rows, table_rows, cols, valid);
   IRON_LAUNCH_CHECK();
 }
 
-extern "C" int iron_stream_rows(float* x, const void* y, const uint16_t* back_gain, const uint16_t* gain, void* h, int rows,
-                                int cols, float eps, int is_float, const int* valid, void* stream) {
+extern "C" int iron_stream_rows(float* x, const void* y, const uint16_t* y_bias, const uint16_t* back_gain, const uint16_t* gain, void* h,
+                                int rows, int cols, float eps, float unit, int is_float, const int* valid, void* stream) {
   IRON_REQUIRE(x && (h || y), "stream_rows: null operand");
   IRON_REQUIRE((y == nullptr) == (back_gain == nullptr) && (h == nullptr) == (gain == nullptr),
                "stream_rows: a gain for the row that is added, and one for the norm that is taken");
   IRON_REQUIRE(rows > 0 && cols > 0, "stream_rows: rows (%d) and cols (%d) must be positive", rows, cols);
   hipStream_t s = (hipStream_t)stream;
-#define IRON_STREAM_ROWS(T)                                                                                             \
-  if (y && h) return launch_stream_rows<T, ADD_NORMED, true>(x, (const T*)y, back_gain, gain, (T*)h, rows, cols, eps, valid, s); \
-  if (y) return launch_stream_rows<T, ADD_NORMED, false>(x, (const T*)y, back_gain, gain, (T*)h, rows, cols, eps, valid, s);     \
-  return launch_stream_rows<T, ADD_NONE, true>(x, (const T*)y, back_gain, gain, (T*)h, rows, cols, eps, valid, s);
+  const StreamGate g{nullptr, nullptr, y_bias, 8, 8};
+#define IRON_STREAM_ROWS(T)                                                                                                             \
+  if (y && h) return launch_stream_rows<T, ADD_NORMED, OUT_NORM>(x, (const T*)y, back_gain, gain, (T*)h, rows, cols, eps, unit, valid, s, g); \
+  if (y) return launch_stream_rows<T, ADD_NORMED, OUT_NONE>(x, (const T*)y, back_gain, gain, (T*)h, rows, cols, eps, unit, valid, s, g);     \
+  return launch_stream_rows<T, ADD_NONE, OUT_NORM>(x, (const T*)y, back_gain, gain, (T*)h, rows, cols, eps, unit, valid, s, g);
   if (is_float) { IRON_STREAM_ROWS(float) }
   IRON_STREAM_ROWS(bf16_t)
 #undef IRON_STREAM_ROWS
+}
+
+extern "C" int iron_stream_depth_rows(float* x, const void* y, const uint16_t* y_bias, const uint16_t* back_gain, float* planes,
+                                      const uint16_t* weights, int plane_rows, int index, void* h, int rows, int cols, float eps, float unit,
+                                      int is_float, const int* valid, void* stream) {
+  IRON_REQUIRE(x && (h || planes), "stream_depth_rows: null operand");
+  IRON_REQUIRE((y == nullptr) == (back_gain == nullptr) && (planes == nullptr) == (weights == nullptr),
+               "stream_depth_rows: a gain for the row that is added, and weights for the planes");
+  IRON_REQUIRE(rows > 0 && cols > 0, "stream_depth_rows: rows (%d) and cols (%d) must be positive", rows, cols);
+  IRON_REQUIRE(planes == nullptr || (index >= 0 && plane_rows >= rows), "stream_depth_rows: plane %d of %d rows for %d", index, plane_rows, rows);
+  hipStream_t s = (hipStream_t)stream;
+  const StreamGate g{nullptr, nullptr, y_bias, 8, 8};
+  const StreamDepth d{planes, weights, (size_t)plane_rows * cols, index};
+#define IRON_DEPTH(T, ADD, OUT, DEPTH) \
+  return launch_stream_rows<T, ADD, OUT, DEPTH>(x, (const T*)y, back_gain, nullptr, (T*)h, rows, cols, eps, unit, valid, s, g, d)
+#define IRON_DEPTHS(T)                                        \
+  if (y && planes && h) IRON_DEPTH(T, ADD_NORMED, OUT_CAST, true); \
+  if (y && planes) IRON_DEPTH(T, ADD_NORMED, OUT_NONE, true);      \
+  if (y) IRON_DEPTH(T, ADD_NORMED, OUT_CAST, false);               \
+  if (planes && h) IRON_DEPTH(T, ADD_NONE, OUT_CAST, true);        \
+  if (planes) IRON_DEPTH(T, ADD_NONE, OUT_NONE, true);             \
+  IRON_DEPTH(T, ADD_NONE, OUT_CAST, false);
+  if (is_float) { IRON_DEPTHS(float) }
+  IRON_DEPTHS(bf16_t)
+#undef IRON_DEPTHS
+#undef IRON_DEPTH
 }
 
 extern "C" int iron_stream_gated_rows(float* x, const void* y, const uint16_t* y_bias, const void* gate, const uint16_t* gate_bias,
@@ -303,8 +419,8 @@ extern "C" int iron_stream_gated_rows(float* x, const void* y, const uint16_t* y
   hipStream_t s = (hipStream_t)stream;
   const StreamGate g{gate, gate_bias, y_bias, gate_stride, gate_at};
 #define IRON_STREAM_GATED(T)                                                                                                    \
-  if (h) return launch_stream_rows<T, ADD_GATED, true>(x, (const T*)y, nullptr, gain, (T*)h, rows, cols, eps, valid, s, g); \
-  return launch_stream_rows<T, ADD_GATED, false>(x, (const T*)y, nullptr, gain, (T*)h, rows, cols, eps, valid, s, g);
+  if (h) return launch_stream_rows<T, ADD_GATED, OUT_NORM>(x, (const T*)y, nullptr, gain, (T*)h, rows, cols, eps, 0.f, valid, s, g); \
+  return launch_stream_rows<T, ADD_GATED, OUT_NONE>(x, (const T*)y, nullptr, gain, (T*)h, rows, cols, eps, 0.f, valid, s, g);
   if (is_float) { IRON_STREAM_GATED(float) }
   IRON_STREAM_GATED(bf16_t)
 #undef IRON_STREAM_GATED
@@ -339,6 +455,21 @@ extern "C" int iron_act_mul_f32(const float* gate, const float* up, float* y, in
   IRON_REQUIRE(activation >= 1 && activation <= 3, "act_mul_f32: activation (%d) is 1 (SiLU), 2 (GELU, tanh form) or 3 (ReLU)", activation);
   const long n = (long)rows * cols;
   hipLaunchKernelGGL(act_mul_f32_kernel, dim3(few_blocks(n)), dim3(256), 0, (hipStream_t)stream, gate, up, y, n, activation, valid, cols);
+  IRON_LAUNCH_CHECK();
+}
+
+extern "C" int iron_activation(const void* x, void* y, int rows, int cols, int activation, int is_float, const int* valid, void* stream) {
+  IRON_REQUIRE(x && y, "activation: null operand");
+  IRON_REQUIRE(rows > 0 && cols > 0, "activation: rows (%d) and cols (%d) must be positive", rows, cols);
+  IRON_REQUIRE(activation >= 1 && activation <= 3, "activation: kind (%d) is 1 (SiLU), 2 (GELU, tanh form) or 3 (ReLU)", activation);
+  const long n = (long)rows * cols;
+  const bool vec = cols % 8 == 0 && (((uintptr_t)x | (uintptr_t)y) & 15) == 0;
+  const dim3 grid(few_blocks(vec ? n / 8 : n));
+#define IRON_ACTIVATION(T, VEC) \
+  hipLaunchKernelGGL((activation_kernel<T, VEC>), grid, dim3(256), 0, (hipStream_t)stream, (const T*)x, (T*)y, n, activation, valid, cols)
+  if (is_float) { if (vec) IRON_ACTIVATION(float, 8); else IRON_ACTIVATION(float, 1); }
+  else { if (vec) IRON_ACTIVATION(bf16_t, 8); else IRON_ACTIVATION(bf16_t, 1); }
+#undef IRON_ACTIVATION
   IRON_LAUNCH_CHECK();
 }
 

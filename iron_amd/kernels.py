@@ -609,26 +609,135 @@ def _spans(t, slots):
     return ptr(t)
 
 
-def stream_embed(table, ids, x, *, rows, table_rows, cols, valid=None):
+def stream_embed(table, ids, x, *, rows, table_rows, cols, also=None, valid=None):
     _bf16(table, table_rows * cols, "table")
     _numel(_dev(ids, "ids", torch.int32), rows, "ids")
     _f32(x, rows * cols, "x")
-    check(lib().iron_stream_embed(ptr(table), ptr(ids), ptr(x), rows, table_rows, cols, ptr(_word(valid, "valid")),
+    if also is not None:
+        _f32(also, rows * cols, "also")
+    check(lib().iron_stream_embed(ptr(table), ptr(ids), ptr(x), ptr(also), rows, table_rows, cols, ptr(_word(valid, "valid")),
                                   current_stream()), "iron_stream_embed")
 
 
-def stream_rows(x, *, rows, cols, eps, y=None, back_gain=None, h=None, gain=None, valid=None):
-    """``x += rmsnorm(y) * back_gain`` (with ``y``) and ``h = rmsnorm(x) * gain`` (with ``h``), one launch."""
+def _added(x, y, y_bias, back_gain, h, rows, cols):
+    """The operands of a row that joins the stream and of one that leaves it; whether activations are float."""
     _f32(x, rows * cols, "x")
     is_float = False
-    for t, g, name in ((y, back_gain, "y"), (h, gain, "h")):
+    for t, name in ((y, "y"), (h, "h")):
         if t is not None:
             is_float = _act(t, rows * cols, name)
-            _bf16(g, cols, f"the gain of {name}")
+    for t, name in ((y_bias, "y_bias"), (back_gain, "the gain of y")):
+        if t is not None:
+            _bf16(t, cols, name)
     if y is not None and h is not None:
         _same_kind(is_float, y=y)
-    check(lib().iron_stream_rows(ptr(x), ptr(y), ptr(back_gain), ptr(gain), ptr(h), rows, cols, float(eps), int(is_float),
-                                 ptr(_word(valid, "valid")), current_stream()), "iron_stream_rows")
+    return is_float
+
+
+def stream_rows(x, *, rows, cols, eps, unit=0.0, y=None, y_bias=None, back_gain=None, h=None, gain=None, valid=None):
+    """``x += rmsnorm(y + y_bias) * (unit + back_gain)`` (with ``y``) and ``h = rmsnorm(x) * (unit + gain)`` (with ``h``), one
+    launch."""
+    is_float = _added(x, y, y_bias, back_gain, h, rows, cols)
+    if h is not None:
+        _bf16(gain, cols, "the gain of h")
+    check(lib().iron_stream_rows(ptr(x), ptr(y), ptr(y_bias), ptr(back_gain), ptr(gain), ptr(h), rows, cols, float(eps), float(unit),
+                                 int(is_float), ptr(_word(valid, "valid")), current_stream()), "iron_stream_rows")
+
+
+def stream_depth_rows(x, *, rows, cols, eps=0.0, unit=0.0, y=None, y_bias=None, back_gain=None, planes=None, weights=None, plane_rows=0,
+                      index=0, h=None, valid=None):
+    """``x += rmsnorm(y + y_bias) * (unit + back_gain)`` (with ``y``); with ``planes``, ``planes[index] = x`` and ``x`` the sum of
+    ``weights[j] * planes[j]``; ``h = x`` (with ``h``), one launch."""
+    is_float = _added(x, y, y_bias, back_gain, h, rows, cols)
+    if planes is not None:
+        _bf16(weights, index + 1, "weights")
+        if _dev(planes, "planes", torch.float32).numel() < (index + 1) * plane_rows * cols:
+            raise ValueError(f"planes: {planes.numel()} elements hold no {index + 1} planes of {plane_rows} rows of {cols}")
+    check(lib().iron_stream_depth_rows(ptr(x), ptr(y), ptr(y_bias), ptr(back_gain), ptr(planes), ptr(weights), plane_rows, index, ptr(h),
+                                       rows, cols, float(eps), float(unit), int(is_float), ptr(_word(valid, "valid")), current_stream()),
+          "iron_stream_depth_rows")
+
+
+def activation(x, y, *, rows, cols, kind, valid=None):
+    is_float = _act(x, rows * cols, "x")
+    _same_kind(is_float, y=y)
+    _act(y, rows * cols, "y")
+    check(lib().iron_activation(ptr(x), ptr(y), rows, cols, GATES[kind], int(is_float), ptr(_word(valid, "valid")), current_stream()),
+          "iron_activation")
+
+
+def turned_heads(x, y, bias, q_gain, k_gain, temp, spans, *, slots, rows, stride, heads, kv_heads, dim, vdim, scale, eps, turned=0,
+                 angle_rows=1, angles=None, share=None, first=None, first_stride=0, first_at=0, valid=None):
+    is_float = _act(x, rows * stride, "x")
+    _same_kind(is_float, y=y)
+    _act(y, rows * stride, "y")
+    _bf16(bias, heads * dim + kv_heads * (dim + vdim), "bias")
+    for t, n, name in ((q_gain, dim, "q_gain"), (k_gain, dim, "k_gain"), (temp, heads, "temp")):
+        _bf16(t, n, name)
+    if first is not None:
+        _same_kind(is_float, first=first)
+        _act(first, rows * first_stride, "first")
+        _bf16(share, 1, "share")
+    check(lib().iron_turned_heads(ptr(x), ptr(y), ptr(bias), ptr(q_gain), ptr(k_gain), ptr(temp), _turned(angles, angle_rows, turned),
+                                  ptr(share), ptr(first), first_stride, first_at, _spans(spans, slots), slots, rows, stride, heads, kv_heads,
+                                  dim, vdim, turned, angle_rows, float(scale), float(eps), int(is_float), ptr(_word(valid, "valid")),
+                                  current_stream()), "iron_turned_heads")
+
+
+def mha_talking(x, keys, values, talk, spans, y, *, slots, rows, stride, heads, kv_heads, dim, vdim, chunk, ring, single=False):
+    is_float = _act(x, rows * stride, "x")
+    _same_kind(is_float, keys=keys, values=values, y=y)
+    _act(keys, slots * ring * kv_heads * dim, "keys")
+    _act(values, slots * ring * kv_heads * vdim, "values")
+    _bf16(talk, heads * heads, "talk")
+    _act(y, rows * heads * vdim, "y")
+    check(lib().iron_mha_talking(ptr(x), ptr(keys), ptr(values), ptr(talk), _spans(spans, slots), ptr(y), slots, rows, stride, heads, kv_heads,
+                                 dim, vdim, chunk, ring, int(single), int(is_float), current_stream()), "iron_mha_talking")
+
+
+def matrix_memory(x, i_bias, f_bias, state, tops, spans, o, *, slots, rows, stride, heads, dim, vdim, i_at, f_at, cap):
+    is_float = _act(x, rows * stride, "x")
+    _bf16(i_bias, heads, "i_bias")
+    _bf16(f_bias, heads, "f_bias")
+    _f32(state, slots * heads * dim * (vdim + 1), "state")
+    _f32(tops, slots * 2 * heads, "tops")
+    _f32(o, rows * heads * (vdim + 2), "o")
+    check(lib().iron_matrix_memory(ptr(x), ptr(i_bias), ptr(f_bias), ptr(state), ptr(tops), _spans(spans, slots), ptr(o), slots, rows, stride,
+                                   heads, dim, vdim, i_at, f_at, float(cap), int(is_float), current_stream()), "iron_matrix_memory")
+
+
+def memory_gate(o, gate, gain, y, *, rows, heads, dim, gate_stride, gate_at, floor, eps, valid=None):
+    _f32(o, rows * heads * (dim + 2), "o")
+    is_float = _act(gate, rows * gate_stride, "gate")
+    _bf16(gain, heads * dim, "gain")
+    _same_kind(is_float, y=y)
+    _act(y, rows * heads * dim, "y")
+    check(lib().iron_memory_gate(ptr(o), ptr(gate), ptr(gain), ptr(y), rows, heads, dim, gate_stride, gate_at, float(floor), float(eps),
+                                 int(is_float), ptr(_word(valid, "valid")), current_stream()), "iron_memory_gate")
+
+
+def router(h, w, bias, ids, shares, *, rows, cols, experts, top, valid=None):
+    is_float = _act(h, rows * cols, "h")
+    _bf16(w, experts * cols, "w")
+    _bf16(bias, experts, "bias")
+    _numel(_dev(ids, "ids", torch.int32), rows * top, "ids")
+    _f32(shares, rows * top, "shares")
+    check(lib().iron_router(ptr(h), ptr(w), ptr(bias), ptr(ids), ptr(shares), rows, cols, experts, top, int(is_float),
+                            ptr(_word(valid, "valid")), current_stream()), "iron_router")
+
+
+def experts(h, gate, up, down, ids, shares, y, workspace, *, rows, cols, ff, experts, top, activation, valid=None):
+    is_float = _act(h, rows * cols, "h")
+    for t, name in ((gate, "gate"), (up, "up"), (down, "down")):
+        _bf16(t, experts * ff * cols, name)
+    _numel(_dev(ids, "ids", torch.int32), rows * top, "ids")
+    _f32(shares, rows * top, "shares")
+    _same_kind(is_float, y=y)
+    _act(y, rows * cols, "y")
+    need = int(lib().iron_experts_workspace_bytes(rows, cols, ff, experts, top, int(is_float)))
+    check(lib().iron_experts(ptr(h), ptr(gate), ptr(up), ptr(down), ptr(ids), ptr(shares), ptr(y), _work(workspace, need, "experts: workspace"),
+                             rows, cols, ff, experts, top, GATES[activation], int(is_float), ptr(_word(valid, "valid")), current_stream()),
+          "iron_experts")
 
 
 def stream_gated_rows(x, y, gate, gate_bias, *, rows, cols, eps=0.0, gate_stride, gate_at, y_bias=None, h=None, gain=None, valid=None):
@@ -849,7 +958,7 @@ STREAM_INPUTS = {"row": 0, "stream_norm": 1, "row_norm": 2, "min_gru": 3, "poly_
 
 
 def stream_product(W, x, *, input, M, K, y=None, stream=None, y_bias=None, gate=None, gate_bias=None, gain=None, b0=None, b1=None,
-                   state=None, spans=None, eps=0.0):
+                   state=None, spans=None, eps=0.0, unit=0.0):
     """One row's product: ``input`` says how its input is made of ``x``; the output is the row ``y``, or joins the
     stream's row ``stream`` through ``gate`` (its first M elements)."""
     _bf16(W, M * K, "W")
@@ -868,7 +977,7 @@ def stream_product(W, x, *, input, M, K, y=None, stream=None, y_bias=None, gate=
         if _dev(gate, "gate").numel() < M:
             raise ValueError(f"stream_product: a gate of {gate.numel()} elements for {M}")
     check(lib().iron_stream_product_bf16(STREAM_INPUTS[input], ptr(x), ptr(gain), ptr(b0), ptr(b1), ptr(state),
-                                         None if spans is None else _spans(spans, 1), float(eps), ptr(W), M, K, ptr(y), ptr(stream), ptr(y_bias),
+                                         None if spans is None else _spans(spans, 1), float(eps), float(unit), ptr(W), M, K, ptr(y), ptr(stream), ptr(y_bias),
                                          ptr(gate), ptr(gate_bias), current_stream()), "iron_stream_product_bf16")
 
 

@@ -31,12 +31,14 @@ READOUT_ROWS = 64   # rows whose logits one launch of the readout gives
 
 @dataclasses.dataclass(kw_only=True)
 class BatchCall:
-    """What one recording of a batched body gives its layers: the spans, and in a prompt's portion the
-    bound on its rows."""
+    """What one recording of a batched body gives its layers: the spans, in a prompt's portion the bound on its
+    rows, and what they hand on to each other."""
 
     prompt: bool
     spans: Any
     rows: Any = None
+    planes: Any = None                                   # what the stream was behind every layer, where layers look back
+    kept: dict = dataclasses.field(default_factory=dict)   # what a layer leaves for later ones of the same call
 
     def bound(self, x):
         """``x`` as far as this call's rows go."""
@@ -343,7 +345,7 @@ class StreamDecoder(Decoder):
 
     def __init__(self, c, layer):
         super().__init__(c, layer)
-        self.norm = StreamRMSNorm(c.hidden_size, c.eps, c.activations)
+        self.norm = StreamRMSNorm(c.hidden_size, c.eps, c.activations, c.norm_unit)
 
 
 class BatchedLM(CausalLM):
@@ -352,7 +354,8 @@ class BatchedLM(CausalLM):
 
     The config is a ``LayerListConfig``: it adds to a decoder's ``slots`` (sequences served at once),
     ``activations`` (bf16, or float32 for a model in 32 bits throughout), ``order`` (layer indices in running
-    order), ``logit_scale``, ``logit_softcap`` and ``key_room`` (keys a portion's layers may attend in all)."""
+    order), ``norm_unit`` (what the final norm's gains are stored around), ``looks_back`` (layers read the stream behind every
+    earlier one), ``logit_scale``, ``logit_softcap`` and ``key_room`` (keys a portion's layers may attend in all)."""
 
     decoder_class = StreamDecoder
     session_class = SlotSession
@@ -361,6 +364,7 @@ class BatchedLM(CausalLM):
         super().__init__(config, weights)
         c = config
         self.residual = iron.state((max(c.prefill_chunk, c.slots), c.hidden_size), np.float32)
+        self.planes = iron.state((len(c.order) + 1, *self.residual.shape), np.float32) if c.looks_back else None
         self.spans = iron.state((c.slots, 4), np.int32)
         self.token = iron.state((c.slots,), np.int32)
         self.runs = [(i, self.layers[i].mixer.states(c.slots)) for i in c.order]
@@ -376,11 +380,12 @@ class BatchedLM(CausalLM):
         c = self.config
         if picks is not None:
             return self.head(Copy.step(self.residual[picks], dtype=np.float32))[0]
-        call = BatchCall(prompt=ids is not None, spans=self.spans, rows=rows)
+        call = BatchCall(prompt=ids is not None, spans=self.spans, rows=rows, planes=self.planes)
         count = c.prefill_chunk if call.prompt else c.slots
         x = call.bound(self.residual[:count])
         ids = call.bound(ids) if call.prompt else self.token
-        StreamEmbed.step(self.model.embed_tokens.weight, ids, x)
+        first = [] if self.planes is None else [call.bound(self.planes[0][:count])]
+        StreamEmbed.step(self.model.embed_tokens.weight, ids, x, *first, twice=bool(first))
         for index, states in self.runs:
             x = self.layers[index](x, call, states)
         last = SpanTails.step(x, self.spans) if call.prompt else x

@@ -191,6 +191,8 @@ class LayerListConfig(ConfigFile):
     rope_theta = None
     logit_softcap = None
     logit_scale = 1.0
+    norm_unit = 0.0        # what the norms' weights are stored around: 1 where a gain is 1 + its weight
+    looks_back = False     # whether layers read the stream behind every earlier one
     key_room = None        # keys, of all requests together, that a portion may attend; None: any number
 
     def check_serving(self) -> None:
@@ -200,14 +202,14 @@ class LayerListConfig(ConfigFile):
         if self.slots < 1:
             raise ValueError(f"{type(self).__name__}: slots ({self.slots}) must be at least 1")
 
-    def check_layers(self, mixers) -> None:
+    def check_layers(self, mixers, feed_forwards=("dense",)) -> None:
         """Refuse a layer whose mixer or feed-forward is none of this design's."""
         for i, spec in enumerate(self.layers):
             if spec["type"] not in mixers:
                 raise ValueError(f"{type(self).__name__}: layer {i} is {spec['type']!r}, not one of {tuple(mixers)}")
             mlp = spec.get("mlp")
-            if mlp is not None and mlp.get("kind") != "dense":
-                raise ValueError(f"{type(self).__name__}: layer {i}'s feed-forward is {mlp.get('kind')!r}, not 'dense'")
+            if mlp is not None and mlp.get("kind") not in feed_forwards:
+                raise ValueError(f"{type(self).__name__}: layer {i}'s feed-forward is {mlp.get('kind')!r}, not one of {tuple(feed_forwards)}")
 
     @classmethod
     def from_json(cls, data: dict, source="config.json"):

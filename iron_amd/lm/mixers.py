@@ -1,7 +1,8 @@
 """Token mixers over a batch of rows told apart by spans, and the layer that runs them around a float32
 residual stream: sliding-window attention with a learned distance bias, time mixing with a
-data-dependent decay, both side by side, the gated delta rule, a gated recurrence element by element, and
-latent attention.
+data-dependent decay, both side by side, the gated delta rule, a gated recurrence element by element,
+latent attention, attention within chunks whose heads mix their weights, and a matrix memory; feed-forwards that go
+with them.
 
 A module holds weights; what a run of it carries from token to token is a ``states()`` mapping the
 caller makes once per run, so that a layer run several times in a row has a state for each pass.
@@ -16,10 +17,22 @@ import numpy as np
 
 from .. import functional as F
 from ..common import graph as iron
+from ..operators.experts import Experts, Router
 from ..operators.mha_latent import EVERYTHING, LatentMHA, LatentRows
+from ..operators.mha_talking import TalkingMHA, TurnedHeads
 from ..operators.mha_window import WindowMHA
-from ..operators.recurrent import DeltaRule, HeadGate, LowRankDecay, MinGRU, ShortConv, TimeMix, TokenShift
-from ..operators.stream import PolyNorm, StreamAdd, StreamGatedAdd, StreamNorm
+from ..operators.recurrent import (
+    DeltaRule,
+    HeadGate,
+    LowRankDecay,
+    MatrixMemory,
+    MemoryGate,
+    MinGRU,
+    ShortConv,
+    TimeMix,
+    TokenShift,
+)
+from ..operators.stream import Activation, DepthAverage, PolyNorm, StreamAdd, StreamCast, StreamGatedAdd, StreamNorm
 from .blocks import Linear
 
 
@@ -43,17 +56,17 @@ def distance_buckets(count: int, rows: int, bias_max: float) -> np.ndarray:
 
 class StreamRMSNorm(iron.Graph):
     """An RMS norm at the stream's edge: ``body`` takes a normed row out of it, ``add`` a block's output
-    into it."""
+    into it.  Gains are ``unit`` (0, or 1 where they are stored around zero) plus the weight."""
 
-    def __init__(self, width: int, eps: float, dtype):
-        self.eps, self.dtype = eps, dtype
+    def __init__(self, width: int, eps: float, dtype, unit: float = 0.0):
+        self.constants = dict(epsilon=eps, unit=unit, dtype=dtype)
         self.weight = iron.param(width)
 
     def body(self, stream):
-        return StreamNorm.step(stream, self.weight, epsilon=self.eps, dtype=self.dtype)
+        return StreamNorm.step(stream, self.weight, **self.constants)
 
-    def add(self, stream, y):
-        return StreamAdd.step(stream, y, self.weight, epsilon=self.eps, dtype=self.dtype)
+    def add(self, stream, y, y_bias=None):
+        return StreamAdd.step(stream, y, self.weight, y_bias=y_bias, **self.constants)
 
 
 class WindowAttention(iron.Graph):
@@ -307,3 +320,119 @@ class GatedStreamLayer(iron.Graph):
             packed = as_rows(self.mlp.proj(self.norm2(x)), x.shape[0])
             x = self.add(x, self.mlp(packed), packed, self.mlp, self.gate2_bias)
         return x
+
+
+# ---- post-normed layers that read the stream itself, and average over what it was
+
+
+class TalkingAttention(iron.Graph):
+    """Grouped-query attention within chunks of ``chunk`` positions: biased projections, q and k normed a head and turned by
+    ``angles``, scores times ``scale`` and the head's ``temp``, the heads' softmax weights mixed by ``talk``.  ``proj`` is one
+    packed projection (q, k, v); ``out_bias`` is added where the output joins the stream.  ``mixes``: the values are blended
+    with those of the call's first such layer by ``share``."""
+
+    def __init__(self, width, *, heads, kv_heads, dim, vdim, chunk, scale, eps, context, dtype, precision, angles=None, mixes=False):
+        self.heads, self.kv_heads, self.dim, self.vdim = heads, kv_heads, dim, vdim
+        self.chunk = min(chunk, context)
+        self.scale, self.eps, self.dtype, self.angles, self.mixes = scale, eps, dtype, angles, mixes
+        packed = heads * dim + kv_heads * (dim + vdim)
+        self.proj = Linear(width, packed, precision=precision)
+        self.bias = iron.param(packed)
+        self.q_norm = iron.param(dim)
+        self.k_norm = iron.param(dim)
+        self.temp = iron.param(heads)
+        self.talk = iron.param(heads, heads)
+        self.share = iron.param(1) if mixes else None
+        self.out = Linear(heads * vdim, width, precision=precision)
+        self.out_bias = iron.param(width)
+
+    def states(self, slots: int) -> dict:
+        # A position sees its own chunk only, so a ring of a chunk holds it in its first rows.
+        return {"keys": iron.state((slots, self.chunk, self.kv_heads, self.dim), self.dtype),
+                "values": iron.state((slots, self.chunk, self.kv_heads, self.vdim), self.dtype)}
+
+    def body(self, h, call, state):
+        beside, held = {"angles": self.angles}, call.kept.get("values") if self.mixes else None
+        if held is not None:
+            beside |= {"first": held[0], "share": self.share, "first_at": held[1]}
+        x = TurnedHeads.step(as_rows(self.proj(h), h.shape[0]), self.bias, self.q_norm, self.k_norm, self.temp, call.spans,
+                             kv_heads=self.kv_heads, scale=self.scale, epsilon=self.eps, dtype=self.dtype, **beside)
+        if self.mixes and held is None:
+            call.kept["values"] = x, (self.heads + self.kv_heads) * self.dim
+        y = TalkingMHA.step(x, self.talk, call.spans, state["keys"], state["values"], single=not call.prompt, dtype=self.dtype)[2]
+        return self.out(y)
+
+
+class MatrixMemoryMixer(iron.Graph):
+    """mLSTM: a matrix a head that keys and values are written into under exponential gates, read by queries, each head normed
+    and gated.  ``proj`` is one packed projection (q, k, v, gate, input gate, forget gate)."""
+
+    out_bias = None
+
+    def __init__(self, width, *, heads, dim, vdim, cap, eps, dtype, precision):
+        self.heads, self.dim, self.vdim, self.cap, self.eps, self.dtype = heads, dim, vdim, cap, eps, dtype
+        self.gate_at = heads * (2 * dim + vdim)
+        self.i_at = self.gate_at + heads * vdim
+        self.proj = Linear(width, self.i_at + 2 * heads, precision=precision)
+        self.i_bias = iron.param(heads)
+        self.f_bias = iron.param(heads)
+        self.norm = iron.param(heads * vdim)
+        self.out = Linear(heads * vdim, width, precision=precision)
+
+    def states(self, slots: int) -> dict:
+        return {"memory": iron.state((slots, self.heads, self.dim, self.vdim + 1), np.float32),
+                "tops": iron.state((slots, 2, self.heads), np.float32)}
+
+    def body(self, h, call, state):
+        x = as_rows(self.proj(h), h.shape[0])
+        o = MatrixMemory.step(x, self.i_bias, self.f_bias, state["memory"], state["tops"], call.spans, i_at=self.i_at,
+                              f_at=self.i_at + self.heads, cap=self.cap, dtype=self.dtype)[2]
+        return self.out(MemoryGate.step(o, x, self.norm, heads=self.heads, gate_at=self.gate_at, epsilon=self.eps, dtype=self.dtype))
+
+
+class ActivatedMLP(iron.Graph):
+    """``down(act(up h))``."""
+
+    def __init__(self, width, *, inner, activation, dtype, precision):
+        self.kind, self.dtype = activation, dtype
+        self.up = Linear(width, inner, precision=precision)
+        self.down = Linear(inner, width, precision=precision)
+
+    def body(self, h):
+        return self.down(Activation.step(as_rows(self.up(h), h.shape[0]), kind=self.kind, dtype=self.dtype))
+
+
+class ExpertsMLP(iron.Graph):
+    """Gated feed-forwards of which a router chooses ``top`` a row.  The experts' matrices are stacked."""
+
+    def __init__(self, width, *, inner, experts, top, activation, dtype):
+        self.top, self.kind, self.dtype = top, activation, dtype
+        self.router = iron.param(experts, width)
+        self.router_bias = iron.param(experts)
+        self.gate = iron.param(experts * inner, width)
+        self.up = iron.param(experts * inner, width)
+        self.down = iron.param(experts * width, inner)
+
+    def body(self, h):
+        ids, shares = Router.step(h, self.router, self.router_bias, top=self.top, dtype=self.dtype)
+        return Experts.step(h, self.gate, self.up, self.down, ids, shares, activation=self.kind, dtype=self.dtype)
+
+
+class PostNormLayer(iron.Graph):
+    """A layer around a float32 stream whose blocks read the stream itself and are normed where they join it.  Layer ``index``'s
+    result is kept with those of the layers before it, and what goes on is the sum of all by ``depth``."""
+
+    def __init__(self, width, mixer, mlp, *, index, eps, dtype, unit=0.0):
+        self.dtype, self.mixer, self.mlp = dtype, mixer, mlp
+        self.norm1 = StreamRMSNorm(width, eps, dtype, unit)
+        if mlp is not None:
+            self.norm2 = StreamRMSNorm(width, eps, dtype, unit)
+        self.depth = iron.param(index + 2)
+        self.rope = None
+
+    def body(self, x, call, state):
+        h = StreamCast.step(x, dtype=self.dtype)
+        x = self.norm1.add(x, as_rows(self.mixer(h, call, state), x.shape[0]), self.mixer.out_bias)
+        if self.mlp is not None:
+            x = self.norm2.add(x, as_rows(self.mlp(StreamCast.step(x, dtype=self.dtype)), x.shape[0]))
+        return DepthAverage.step(x, call.planes, self.depth)[0]

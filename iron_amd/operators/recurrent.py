@@ -327,3 +327,95 @@ class HeadGate(Operator):
             kernels.head_gate(t["o"], t["gate"], t["gain"], t["y"], valid=words.get("valid"), **kw)
 
         return Built("iron_head_gate", launch)
+
+
+class MatrixMemory(_Spanned):
+    """mLSTM: per head ``S <- keep S + write k v^T``, ``n <- keep n + write k`` with log gates i (capped) and f (the logarithm of a
+    capped one's sigmoid), ``m' = max(f + m, i)``, ``keep = exp(f + m - m')``, ``write = exp(i - m')``.  Rows ``[q | k | v | ..]``,
+    the gates at columns ``i_at`` and ``f_at``.  ``state`` is S with n behind its last column; ``tops`` holds m, position p's in row
+    ``p % 2`` of its slot.  Output rows ``[S^T q | n . q | m]``, q times ``dim ** -0.5``."""
+
+    slots: int = param()
+    rows: int = param()
+    stride: int = param()
+    heads: int = param()
+    dim: int = param()
+    vdim: int = param()
+    i_at: int = param(array=True)
+    f_at: int = param(array=True)
+    cap: float = param(array=True)
+    columns: int = param(derive=lambda op: op.vdim + 1, repr=False)
+    width: int = param(derive=lambda op: op.heads * (op.vdim + 2), repr=False)
+    dtype: Any = param(default=bfloat16, repr=False)
+    x = In(rows, stride, dtype=dtype)
+    i_bias = In(heads)
+    f_bias = In(heads)
+    state = InOut(slots, heads, dim, columns, dtype=F32)
+    tops = InOut(slots, 2, heads, dtype=F32)
+    spans = In(slots, 4, dtype=np.int32)
+    o = Out(rows, width, dtype=F32)
+    valid = per_call(bounds=rows)
+
+    @classmethod
+    def infer(cls, shapes, **kw):
+        slots, heads, dim, columns = shapes["state"]
+        return dict(slots=slots, rows=shapes["x"][0], stride=shapes["x"][1], heads=heads, dim=dim, vdim=columns - 1, **kw)
+
+    def validate(self):
+        packed = self.heads * (2 * self.dim + self.vdim)
+        if not (1 <= self.dim <= 512 and packed <= min(self.i_at, self.f_at) and max(self.i_at, self.f_at) + self.heads <= self.stride):
+            raise ValueError(f"MatrixMemory: dim ({self.dim}) from 1 to 512; gates at {self.i_at}, {self.f_at} behind {packed} of {self.stride}")
+
+    def build(self) -> Built:
+        from .. import kernels
+
+        kw = {n: getattr(self, n) for n in ("slots", "rows", "stride", "heads", "dim", "vdim", "i_at", "f_at")}
+        kw["cap"] = float(self.cap)
+
+        def launch(t, words):
+            kernels.matrix_memory(t["x"], t["i_bias"], t["f_bias"], t["state"], t["tops"], t["spans"], t["o"], **kw)
+
+        return Built("iron_matrix_memory", launch)
+
+
+class MemoryGate(Operator):
+    """``o / (max(|n . q|, exp(-m)) + floor)`` of MatrixMemory's rows, RMS-normed a head, times ``gain`` and ``sigmoid(gate)``;
+    the gate is columns ``gate_at ..`` of its row."""
+
+    rows: int = param()
+    heads: int = param()
+    dim: int = param()
+    inner: int = param(derive=lambda op: op.heads * op.dim, repr=False)
+    wide: int = param(derive=lambda op: op.heads * (op.dim + 2), repr=False)
+    gate_width: int = param()
+    gate_at: int = param(default=0, array=True)
+    floor: float = param(default=1e-6, array=True)
+    epsilon: float = param(array=True)
+    dtype: Any = param(default=bfloat16, repr=False)
+    o = In(rows, wide, dtype=F32)
+    gate = In(rows, gate_width, dtype=dtype)
+    gain = In(inner)
+    y = Out(rows, inner, dtype=dtype)
+    valid = per_call(bounds=rows)
+
+    @classmethod
+    def infer(cls, shapes, **kw):
+        return dict(rows=shapes["o"][0], dim=shapes["gain"][0] // kw["heads"], gate_width=shapes["gate"][1], **kw)
+
+    def validate(self):
+        if not 0 <= self.gate_at <= self.gate_width - self.inner:
+            raise ValueError(f"MemoryGate: {self.inner} columns from {self.gate_at} of a row of {self.gate_width}")
+
+    def tolerance(self):
+        return Tolerance.relative(1e-2, 1e-2, note="float32, rounded once")
+
+    def build(self) -> Built:
+        from .. import kernels
+
+        kw = dict(rows=self.rows, heads=self.heads, dim=self.dim, gate_stride=self.gate_width, gate_at=self.gate_at, floor=float(self.floor),
+                  eps=float(self.epsilon))
+
+        def launch(t, words):
+            kernels.memory_gate(t["o"], t["gate"], t["gain"], t["y"], valid=words.get("valid"), **kw)
+
+        return Built("iron_memory_gate", launch)

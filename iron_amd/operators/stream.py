@@ -1,5 +1,5 @@
-"""The float32 residual stream of a decoder: rows into it, norms out of it, blocks' outputs added to it,
-and the head's scale and soft cap.  ``dtype`` is what the rows that leave the stream are rounded to: bf16, or
+"""The float32 residual stream of a decoder: rows into it, rows or their norms out of it, blocks' outputs added to it,
+averages over what it was behind earlier layers, and the head's scale and soft cap.  ``dtype`` is what the rows that leave the stream are rounded to: bf16, or
 float32 in a model that runs in 32 bits throughout.  The stream is updated in place.
 """
 
@@ -18,19 +18,22 @@ F32 = np.float32
 
 
 class StreamEmbed(Operator):
-    """``x[i] = table[ids[i]]``, widened: a decoder's embedding rows as its stream's first values."""
+    """``x[i] = table[ids[i]]``, widened: a decoder's embedding rows as its stream's first values.  ``twice``: into a second
+    place as well."""
 
     rows: int = param()
     table_rows: int = param(array=True)
     cols: int = param()
+    twice: bool = param(default=False, repr=False)
     table = In(table_rows, cols)
     ids = In(rows, dtype=np.int32)
     x = Out(rows, cols, dtype=F32)
+    also = Out(rows, cols, dtype=F32, when=twice)
     valid = per_call(bounds=rows)
 
     @classmethod
     def infer(cls, shapes, **kw):
-        return dict(rows=math.prod(shapes["ids"]), table_rows=shapes["table"][0], cols=shapes["table"][1])
+        return dict(rows=math.prod(shapes["ids"]), table_rows=shapes["table"][0], cols=shapes["table"][1], **kw)
 
     def tolerance(self):
         return Tolerance.exact()
@@ -42,17 +45,18 @@ class StreamEmbed(Operator):
 
         def launch(t, words):
             kernels.stream_embed(t["table"], t["ids"].reshape(-1), t["x"], rows=rows, table_rows=table_rows, cols=cols,
-                                 valid=words.get("valid"))
+                                 also=t.get("also"), valid=words.get("valid"))
 
         return Built("iron_stream_embed", launch)
 
 
 class StreamNorm(Operator):
-    """``y = dtype(x / rms(x) * weight)`` of a float32 row: one rounding, where it leaves the stream."""
+    """``y = dtype(x / rms(x) * (unit + weight))`` of a float32 row: one rounding, where it leaves the stream."""
 
     rows: int = param()
     cols: int = param()
     epsilon: float = param(array=True)
+    unit: float = param(default=0.0, array=True)
     dtype: Any = param(default=bfloat16, repr=False)
     x = In(rows, cols, dtype=F32)
     weight = In(cols)
@@ -69,29 +73,32 @@ class StreamNorm(Operator):
     def build(self) -> Built:
         from .. import kernels
 
-        rows, cols, eps = self.rows, self.cols, float(self.epsilon)
+        kw = dict(rows=self.rows, cols=self.cols, eps=float(self.epsilon), unit=float(self.unit))
 
         def launch(t, words):
-            kernels.stream_rows(t["x"], rows=rows, cols=cols, eps=eps, h=t["y"], gain=t["weight"], valid=words.get("valid"))
+            kernels.stream_rows(t["x"], h=t["y"], gain=t["weight"], valid=words.get("valid"), **kw)
 
         return Built("iron_stream_rows", launch)
 
 
 class StreamAdd(Operator):
-    """``x += y / rms(y) * weight`` in float32: a block's output, normed, joins the stream."""
+    """``x += z / rms(z) * (unit + weight)`` in float32, ``z = y (+ y_bias)``: a block's output, normed, joins the stream."""
 
     rows: int = param()
     cols: int = param()
     epsilon: float = param(array=True)
+    unit: float = param(default=0.0, array=True)
+    biased: bool = param(default=False, repr=False)
     dtype: Any = param(default=bfloat16, repr=False)
     x = InOut(rows, cols, dtype=F32)
     y = In(rows, cols, dtype=dtype)
     weight = In(cols)
+    y_bias = In(cols, when=biased)
     valid = per_call(bounds=rows)
 
     @classmethod
     def infer(cls, shapes, **kw):
-        return dict(rows=shapes["x"][0], cols=shapes["x"][1], **kw)
+        return dict(rows=shapes["x"][0], cols=shapes["x"][1], biased="y_bias" in shapes, **kw)
 
     def tolerance(self):
         return Tolerance.relative(1e-4, 1e-4, note="float32")
@@ -99,13 +106,77 @@ class StreamAdd(Operator):
     def build(self) -> Built:
         from .. import kernels
 
-        rows, cols, eps = self.rows, self.cols, float(self.epsilon)
+        kw = dict(rows=self.rows, cols=self.cols, eps=float(self.epsilon), unit=float(self.unit))
 
         def launch(t, words):
-            kernels.stream_rows(t["x"], rows=rows, cols=cols, eps=eps, y=t["y"], back_gain=t["weight"],
-                                valid=words.get("valid"))
+            kernels.stream_rows(t["x"], y=t["y"], y_bias=t.get("y_bias"), back_gain=t["weight"], valid=words.get("valid"), **kw)
 
         return Built("iron_stream_rows", launch)
+
+
+class DepthAverage(Operator):
+    """``planes[index] = x``, then ``x = sum over j <= index of weights[j] * planes[j]``: a layer's result is kept, and a weighted
+    sum of all there are so far takes its place.  ``planes`` may have more rows than ``x``."""
+
+    rows: int = param()
+    cols: int = param()
+    depth: int = param()
+    plane_rows: int = param()
+    count: int = param()
+    x = InOut(rows, cols, dtype=F32)
+    planes = InOut(depth, plane_rows, cols, dtype=F32)
+    weights = In(count)
+    valid = per_call(bounds=rows)
+
+    @classmethod
+    def infer(cls, shapes, **kw):
+        depth, plane_rows, cols = shapes["planes"]
+        return dict(rows=shapes["x"][0], cols=cols, depth=depth, plane_rows=plane_rows, count=shapes["weights"][0], **kw)
+
+    def validate(self):
+        if not 1 <= self.count <= self.depth or self.rows > self.plane_rows:
+            raise ValueError(f"DepthAverage: {self.count} weights, {self.rows} rows for {self.depth} planes of {self.plane_rows}")
+
+    def tolerance(self):
+        return Tolerance.relative(1e-4, 1e-4, note="float32")
+
+    def build(self) -> Built:
+        from .. import kernels
+
+        kw = dict(rows=self.rows, cols=self.cols, plane_rows=self.plane_rows, index=self.count - 1)
+
+        def launch(t, words):
+            kernels.stream_depth_rows(t["x"], planes=t["planes"], weights=t["weights"], valid=words.get("valid"), **kw)
+
+        return Built("iron_stream_depth_rows", launch)
+
+
+class StreamCast(Operator):
+    """``y = dtype(x)``: the stream's row as a block without a norm ahead of it reads it."""
+
+    rows: int = param()
+    cols: int = param()
+    dtype: Any = param(default=bfloat16, repr=False)
+    x = In(rows, cols, dtype=F32)
+    y = Out(rows, cols, dtype=dtype)
+    valid = per_call(bounds=rows)
+
+    @classmethod
+    def infer(cls, shapes, **kw):
+        return dict(rows=shapes["x"][0], cols=shapes["x"][1], **kw)
+
+    def tolerance(self):
+        return Tolerance.relative(1e-2, 1e-2, note="rounded once")
+
+    def build(self) -> Built:
+        from .. import kernels
+
+        rows, cols = self.rows, self.cols
+
+        def launch(t, words):
+            kernels.stream_depth_rows(t["x"], h=t["y"], rows=rows, cols=cols, valid=words.get("valid"))
+
+        return Built("iron_stream_depth_rows", launch)
 
 
 class StreamGatedAdd(Operator):
@@ -277,6 +348,35 @@ class GatedProduct(Operator):
             kernels.act_mul_f32(t["gate"], t["up"], t["y"], rows=rows, cols=cols, activation=kind, valid=words.get("valid"))
 
         return Built("iron_act_mul_f32", launch)
+
+
+class Activation(Operator):
+    """``act(x)`` of rows of either type, rounded once."""
+
+    rows: int = param()
+    cols: int = param()
+    kind: str = param()
+    dtype: Any = param(default=bfloat16, repr=False)
+    x = In(rows, cols, dtype=dtype)
+    y = Out(rows, cols, dtype=dtype)
+    valid = per_call(bounds=rows)
+
+    @classmethod
+    def infer(cls, shapes, **kw):
+        return dict(rows=shapes["x"][0], cols=shapes["x"][1], **kw)
+
+    def tolerance(self):
+        return Tolerance.relative(1e-2, 1e-2, note="float32, rounded once")
+
+    def build(self) -> Built:
+        from .. import kernels
+
+        rows, cols, kind = self.rows, self.cols, self.kind
+
+        def launch(t, words):
+            kernels.activation(t["x"], t["y"], rows=rows, cols=cols, kind=kind, valid=words.get("valid"))
+
+        return Built("iron_activation", launch)
 
 
 class LinearAny(Operator):

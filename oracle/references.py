@@ -160,7 +160,8 @@ def _spans(spans):
 
 
 def stream_embed(op, table, ids):
-    return np.asarray(table, np.float32)[np.clip(np.asarray(ids).reshape(-1), 0, op.table_rows - 1)]
+    rows = np.asarray(table, np.float32)[np.clip(np.asarray(ids).reshape(-1), 0, op.table_rows - 1)]
+    return (rows, rows) if op.twice else rows
 
 
 def _unit_rms(x, eps):
@@ -169,11 +170,22 @@ def _unit_rms(x, eps):
 
 
 def stream_norm(op, x, weight):
-    return _out(op, _unit_rms(x, op.epsilon) * np.asarray(weight, np.float64))
+    return _out(op, _unit_rms(x, op.epsilon) * (op.unit + np.asarray(weight, np.float64)))
 
 
-def stream_add(op, x, y, weight):
-    return np.asarray(x + _unit_rms(y, op.epsilon) * np.asarray(weight, np.float64), np.float32)
+def stream_add(op, x, y, weight, *, y_bias=None):
+    z = np.asarray(y, np.float64) + (0 if y_bias is None else y_bias)
+    return np.asarray(x + _unit_rms(z, op.epsilon) * (op.unit + np.asarray(weight, np.float64)), np.float32)
+
+
+def depth_average(op, x, planes, weights):
+    planes = np.array(planes)
+    planes[op.count - 1, : op.rows] = np.reshape(x, (op.rows, op.cols))
+    return np.einsum("j,jrc->rc", np.asarray(weights, np.float64), planes[: op.count, : op.rows].astype(np.float64)).astype(np.float32), planes
+
+
+def stream_cast(op, x):
+    return _out(op, x)
 
 
 def _sigmoid(z):
@@ -252,6 +264,96 @@ def latent_mha(op, q, latents, up, spans, *, shared_keys=None, angles=None, sink
     return _out(op, y.reshape(op.rows, -1))
 
 
+def turned_heads(op, x, bias, q_gain, k_gain, temp, spans, *, angles=None, first=None, share=None):
+    H, G, D = op.heads, op.kv_heads, op.dim
+    y = np.zeros((op.rows, op.stride), np.float32)
+    for s, row, n, start in _spans(spans):
+        own = np.asarray(x, np.float64)[row : row + n] + bias
+        parts = []
+        for heads, gain in ((own[:, : H * D].reshape(n, H, D), q_gain), (own[:, H * D : (H + G) * D].reshape(n, G, D), k_gain)):
+            heads = _unit_rms(heads, op.epsilon) * gain
+            if op.turned:
+                heads = _turn(heads, np.asarray(angles)[start : start + n, None], op.turned)
+            parts.append(heads)
+        parts[0] = parts[0] * (op.scale * np.asarray(temp, np.float64))[:, None]
+        v = own[:, (H + G) * D :]
+        if op.mixed:
+            share = float(np.reshape(share, -1)[0])
+            v = (1 - share) * v + share * np.asarray(first, np.float64)[row : row + n, op.first_at : op.first_at + v.shape[1]]
+        y[row : row + n] = np.concatenate([parts[0].reshape(n, -1), parts[1].reshape(n, -1), v], axis=1)
+    return _out(op, y)
+
+
+def talking_mha(op, x, talk, spans, keys, values):
+    H, G, D, V, C = op.heads, op.kv_heads, op.dim, op.vdim, op.chunk
+    keys, values, y = np.array(keys), np.array(values), np.zeros((op.rows, H, V), np.float32)
+    group, talk = np.arange(H) // (H // G), np.asarray(talk, np.float64)
+    for s, row, n, start in _spans(spans):
+        own = np.asarray(x, np.float64)[row : row + n]
+        q, k, v = own[:, : H * D].reshape(n, H, D), own[:, H * D : (H + G) * D].reshape(n, G, D), own[:, (H + G) * D :].reshape(n, G, V)
+        for i in range(n):
+            p = start + i
+            keys[s, p % C], values[s, p % C] = k[i], v[i]
+            seen = p % C + 1
+            score = np.einsum("hd,jhd->hj", q[i], np.asarray(keys[s, :seen], np.float64)[:, group])
+            w = np.exp(score - score.max(1, keepdims=True))
+            w = talk @ (w / w.sum(1, keepdims=True))
+            y[row + i] = np.einsum("hj,jhv->hv", w, np.asarray(values[s, :seen], np.float64)[:, group])
+    return keys, values, _out(op, y.reshape(op.rows, -1))
+
+
+def matrix_memory(op, x, i_bias, f_bias, state, tops, spans):
+    H, D, V = op.heads, op.dim, op.vdim
+    state, tops, o = np.array(state), np.array(tops), np.zeros((op.rows, op.width), np.float32)
+    x = np.asarray(x, np.float64)
+    q, k, v = x[:, : H * D].reshape(-1, H, D) * D**-0.5, x[:, H * D : 2 * H * D].reshape(-1, H, D), x[:, 2 * H * D : H * (2 * D + V)].reshape(-1, H, V)
+    v = np.concatenate([v, np.ones((len(v), H, 1))], axis=2)
+    i = op.cap * np.tanh((x[:, op.i_at : op.i_at + H] + i_bias) / op.cap)
+    f = -np.logaddexp(0, -op.cap * np.tanh((x[:, op.f_at : op.f_at + H] + f_bias) / op.cap))
+    for s, row, n, start in _spans(spans):
+        S = np.asarray(state[s], np.float64) if start else np.zeros((H, D, V + 1))
+        m = np.asarray(tops[s, (start - 1) % 2], np.float64) if start else np.zeros(H)
+        for t in range(row, row + n):
+            top = np.maximum(f[t] + m, i[t])
+            S = np.exp(f[t] + m - top)[:, None, None] * S + np.exp(i[t] - top)[:, None, None] * k[t][:, :, None] * v[t][:, None]
+            m = top
+            read = np.einsum("hdv,hd->hv", S, q[t])
+            o[t] = np.concatenate([read[:, :V].reshape(-1), read[:, V], m])
+        state[s], tops[s, (start + n - 1) % 2] = S, m
+    return state, tops, o
+
+
+def memory_gate(op, o, gate, gain):
+    H, D = op.heads, op.dim
+    o = np.asarray(o, np.float64)
+    under = np.maximum(np.abs(o[:, H * D : H * D + H]), np.exp(-o[:, H * D + H :])) + op.floor
+    y = _unit_rms(o[:, : H * D].reshape(-1, H, D) / under[:, :, None], op.epsilon).reshape(op.rows, -1)
+    return _out(op, y * gain * _sigmoid(np.asarray(gate, np.float64)[:, op.gate_at : op.gate_at + H * D]))
+
+
+def activation(op, x):
+    return _out(op, _act_of(op.kind, np.asarray(x, np.float64)))
+
+
+def router(op, h, weight, bias):
+    z = np.asarray(h, np.float64) @ np.asarray(weight, np.float64).T + bias
+    ids = np.argsort(-z, axis=1, kind="stable")[:, : op.top]
+    chosen = np.take_along_axis(z, ids, 1)
+    e = np.exp(chosen - chosen.max(1, keepdims=True))
+    return ids.astype(np.int32), (e / e.sum(1, keepdims=True)).astype(np.float32)
+
+
+def experts(op, h, gate, up, down, ids, shares):
+    h, y = np.asarray(h, np.float64), np.zeros((op.rows, op.cols))
+    gate, up = (np.reshape(np.asarray(w, np.float64), (op.experts, op.ff, op.cols)) for w in (gate, up))
+    down = np.reshape(np.asarray(down, np.float64), (op.experts, op.cols, op.ff))
+    for r in range(op.rows):
+        for e, share in zip(np.asarray(ids)[r], np.asarray(shares, np.float64)[r]):
+            a = _out(op, _act_of(op.activation, gate[e] @ h[r]) * (up[e] @ h[r]))
+            y[r] += share * (down[e] @ np.asarray(a, np.float64))
+    return _out(op, y)
+
+
 def span_tails(op, x, spans):
     y = np.zeros((op.slots, op.cols), np.float32)
     for s, row, n, _ in _spans(spans):
@@ -268,11 +370,13 @@ def softcap(op, x):
     return y, rounded
 
 
+def _act_of(kind, z):
+    return {"relu": lambda z: np.maximum(z, 0), "silu": lambda z: z / (1 + np.exp(-z)),
+            "gelu_tanh": lambda z: 0.5 * z * (1 + np.tanh(np.sqrt(2 / np.pi) * (z + 0.044715 * z**3)))}[kind](z)
+
+
 def gated_product(op, gate, up):
-    g = np.asarray(gate, np.float64)
-    act = {"relu": lambda z: np.maximum(z, 0), "silu": lambda z: z / (1 + np.exp(-z)),
-           "gelu_tanh": lambda z: 0.5 * z * (1 + np.tanh(np.sqrt(2 / np.pi) * (z + 0.044715 * z**3)))}[op.activation]
-    return np.asarray(act(g) * up, np.float32)
+    return np.asarray(_act_of(op.activation, np.asarray(gate, np.float64)) * up, np.float32)
 
 
 def linear_any(op, x, weight):
@@ -398,7 +502,8 @@ def install() -> None:
         Softcap=softcap, GatedProduct=gated_product, LinearAny=linear_any, TokenShift=token_shift, LowRankDecay=low_rank_decay,
         TimeMix=time_mix, ShortConv=short_conv, DeltaRule=delta_rule, HeadGate=head_gate, WindowMHA=window_mha,
         SampleSlots=sample_slots, StreamGatedAdd=stream_gated_add, PolyNorm=poly_norm, MinGRU=min_gru, LatentRows=latent_rows,
-        LatentMHA=latent_mha,
+        LatentMHA=latent_mha, DepthAverage=depth_average, StreamCast=stream_cast, TurnedHeads=turned_heads, TalkingMHA=talking_mha,
+        MatrixMemory=matrix_memory, MemoryGate=memory_gate, Activation=activation, Router=router, Experts=experts,
         # The host's draw, for iron_amd.lm.generation.Sampler's checks.
         sample_ref=ops.sample_ref, sample_weights=ops.sample_weights,
     )
