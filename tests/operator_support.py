@@ -30,7 +30,7 @@ def ran(op, workspace=None, **inputs):
 
 
 # outputs a slot each, whatever the batch's rows
-STATES = ("state", "carry", "keys", "values", "latents", "shared_keys")
+STATES = ("state", "carry", "keys", "values", "latents", "shared_keys", "tops", "planes")
 
 
 def agrees(op, inputs, tol, rows=None, **kw):
