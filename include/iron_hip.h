@@ -537,6 +537,11 @@ int iron_mha_talking(const void* x, void* keys, void* values, const uint16_t* ta
 int iron_matrix_memory(const void* x, const uint16_t* i_bias, const uint16_t* f_bias, float* state, float* tops,
                        const int* spans, float* o, int slots, int rows, int stride, int heads, int dim, int vdim,
                        int i_at, int f_at, float cap, int is_float, void* stream);
+/* The same sixteen tokens at a time (dim up to 256), with a workspace of that many bytes, 16-byte aligned. */
+int64_t iron_matrix_memory_workspace_bytes(int slots, int rows, int heads, int dim);
+int iron_matrix_memory_chunked(const void* x, const uint16_t* i_bias, const uint16_t* f_bias, float* state, float* tops,
+                               const int* spans, float* o, void* workspace, int slots, int rows, int stride, int heads,
+                               int dim, int vdim, int i_at, int f_at, float cap, int is_float, void* stream);
 /* y = o / (max(|n . q|, exp(-m)) + floor), RMS-normed a head, times gain (heads * dim) and sigmoid(gate). */
 int iron_memory_gate(const float* o, const void* gate, const uint16_t* gain, void* y, int rows, int heads, int dim,
                      int gate_stride, int gate_at, float floor, float eps, int is_float, const int* valid, void* stream);

@@ -1,4 +1,4 @@
-// The two recurrences over a prompt's portion, sixteen tokens at a time on float32 MFMAs.
+// Time mixing, the delta rule and the matrix memory over a prompt's portion, sixteen tokens at a time on float32 MFMAs.
 //
 // Within a chunk of 16 tokens everything that does not touch the state depends on the chunk alone, so a
 // first launch computes it for all chunks at once: what earlier tokens of the chunk leave of themselves
@@ -14,6 +14,7 @@
 // Decays enter as exponentials of differences of running sums of logarithms, later minus earlier: never
 // above 1, however strong the decay.
 #include "../../include/iron_hip.h"
+#include "matrix_memory.h"
 #include "rows.h"
 
 namespace iron {
@@ -146,33 +147,39 @@ struct MixOperands {
   T v[4];   // as loaded: widened where it is used, not where it would be waited for
 };
 
-template <typename T, int NT, int DEPTH>
+// COUNTED: the state has a column behind v's last, of a v that is 1; its reading goes behind all heads' own.
+struct WalkShape {
+  int rows, slots, heads, dim, vdim;
+  int v_stride, o_stride;                // lengths of the rows v lies in (vdim columns a head) and of the readings' rows
+};
+template <typename T, int NT, int DEPTH, bool COUNTED = false>
 __global__ __launch_bounds__(256) void time_mix_walk_kernel(const T* __restrict__ v, float* __restrict__ state,
                                                             const int* __restrict__ spans, const float* __restrict__ work,
-                                                            float* __restrict__ o, int rows, int slots, int heads, int dim) {
+                                                            float* __restrict__ o, WalkShape a) {
   __shared__ float4 os[2][4][64];
   const int head = blockIdx.x, slot = blockIdx.z;   // heads fastest: a head's column blocks share an XCD's L2
+  const int rows = a.rows, slots = a.slots, heads = a.heads, dim = a.dim, vdim = a.vdim, cols = COUNTED ? vdim + 1 : vdim;
   const Span s = span_of(spans, slot, rows);
   if (s.rows == 0) return;
   const int t = threadIdx.x, lane = t & 63, wave = t >> 6, l16 = lane & 15, quad = lane >> 4;
   const int tiles = (dim + 15) / 16, words = mix_words(tiles), col = blockIdx.y * 16 + l16;
   const int count = (s.rows + CHUNK - 1) / CHUNK;
-  const size_t width = (size_t)heads * dim;
-  float* sp = state + ((size_t)slot * heads + head) * dim * dim;
+  float* sp = state + ((size_t)slot * heads + head) * dim * cols;
   const float* at = work + ((size_t)first_chunk(spans, slots, slot, rows, CHUNK) * heads + head) * words;
   // The span's rows by 32-bit offsets; a store to an offset outside them is dropped.
   constexpr int E = (int)sizeof(T);
-  const __amdgpu_buffer_rsrc_t vb = bounded_bytes(v + (size_t)s.row0 * width + head * dim, (int)(((size_t)s.rows * width - head * dim) * E));
-  const __amdgpu_buffer_rsrc_t ob = bounded_bytes(o + (size_t)s.row0 * width + head * dim, (int)(((size_t)s.rows * width - head * dim) * 4));
-  const int v_at = quad * 4 * (int)width * E + min(col, dim - 1) * E, row_v = (int)width * E;
-  const int o_at = col < dim ? ((quad * 4 + wave) * (int)width + col) * 4 : 0x7fffffff;
+  const __amdgpu_buffer_rsrc_t vb = bounded_bytes(v + (size_t)s.row0 * a.v_stride + head * vdim, (int)(((size_t)(s.rows - 1) * a.v_stride + vdim) * E));
+  const __amdgpu_buffer_rsrc_t ob = bounded_bytes(o + (size_t)s.row0 * a.o_stride, (int)((size_t)s.rows * a.o_stride * 4));
+  const int v_at = quad * 4 * a.v_stride * E + min(col, vdim - 1) * E, row_v = a.v_stride * E;
+  const int o_col = COUNTED && col == vdim ? heads * vdim + head : head * vdim + col;
+  const int o_at = col < cols ? ((quad * 4 + wave) * a.o_stride + o_col) * 4 : 0x7fffffff;
   f32x4 S[NT];
 #pragma unroll
   for (int n = 0; n < NT; ++n)
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
       const int i = (wave * NT + n) * 16 + quad * 4 + j;
-      S[n][j] = (s.start > 0 && i < dim && col < dim) ? sp[(size_t)i * dim + col] : 0.f;
+      S[n][j] = (s.start > 0 && i < dim && col < cols) ? sp[(size_t)i * cols + col] : 0.f;
     }
   MixOperands<T, NT> ops[DEPTH];
   auto fetch = [&](MixOperands<T, NT>& x, int c) {
@@ -195,7 +202,7 @@ __global__ __launch_bounds__(256) void time_mix_walk_kernel(const T* __restrict_
   auto run = [&](const MixOperands<T, NT>& x, int c) {
     f32x4 vf, out = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-    for (int j = 0; j < 4; ++j) vf[j] = widened(x.v[j]);
+    for (int j = 0; j < 4; ++j) vf[j] = COUNTED && col == vdim ? 1.f : widened(x.v[j]);
 #pragma unroll
     for (int n = 0; n < NT; ++n) {
       out = product16(f32x4{x.r[n].x, x.r[n].y, x.r[n].z, x.r[n].w}, S[n], out);   // S of a tile past the last stays 0
@@ -209,7 +216,7 @@ __global__ __launch_bounds__(256) void time_mix_walk_kernel(const T* __restrict_
     float sum = 0.f;   // wave w finishes rows quad * 4 + w
 #pragma unroll
     for (int w = 0; w < 4; ++w) sum += reinterpret_cast<const float*>(&os[c & 1][w][lane])[wave];
-    __builtin_amdgcn_raw_buffer_store_b32(__builtin_bit_cast(unsigned, sum), ob, o_at, c * CHUNK * (int)width * 4, 0);
+    __builtin_amdgcn_raw_buffer_store_b32(__builtin_bit_cast(unsigned, sum), ob, o_at, c * CHUNK * a.o_stride * 4, 0);
   };
 #pragma unroll
   for (int d = 0; d < DEPTH; ++d) {
@@ -233,8 +240,137 @@ __global__ __launch_bounds__(256) void time_mix_walk_kernel(const T* __restrict_
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
       const int i = (wave * NT + n) * 16 + quad * 4 + j;
-      if (i < dim && col < dim) sp[(size_t)i * dim + col] = S[n][j];
+      if (i < dim && col < cols) sp[(size_t)i * cols + col] = S[n][j];
     }
+}
+
+// ----------------------------------------------------------- the matrix memory
+// The same walk: with F the chunk's running sum of log forget gates and m0 the largest exponent ahead of it, m_t =
+// max(F_t + m0, max over s <= t of F_t - F_s + i_s); queries enter as q exp(F_t + m0 - m_t), keys leave as k exp(F_end - F_s +
+// i_s - m_end), the state shrinks by exp(F_end + m0 - m_end), and the 16 x 16 matrix is (q_t . k_s) exp(F_t - F_s + i_s - m_t).
+// The m0 of all chunks come first, by a launch that composes the chunks' (F_end, max over s of F_end - F_s + i_s).
+constexpr int TOPS_THREADS = 1024;
+
+template <typename T>
+__device__ __forceinline__ void log_gates(const T* __restrict__ row, const MemoryGates& g, int head, float& i, float& f) {
+  i = capped(load_one(row + g.i_at + head) + bf16_to_f32(g.i_bias[head]), g.cap);
+  f = log_sigmoid(capped(load_one(row + g.f_at + head) + bf16_to_f32(g.f_bias[head]), g.cap));
+}
+
+template <typename T>
+__global__ __launch_bounds__(TOPS_THREADS) void memory_tops_kernel(const T* __restrict__ x, MemoryGates g, float* __restrict__ tops,
+                                                                   const int* __restrict__ spans, float* __restrict__ starts, int rows,
+                                                                   int slots, int stride, int heads) {
+  constexpr int AT_ONCE = TOPS_THREADS / CHUNK;
+  __shared__ float sums[2][AT_ONCE], most[2][AT_ONCE];
+  const int head = blockIdx.x, slot = blockIdx.y, t = threadIdx.x, l16 = t & 15;
+  const Span s = span_of(spans, slot, rows);
+  if (s.rows == 0) return;
+  float* mp = tops + (size_t)slot * 2 * heads + head;
+  float m = s.start > 0 ? mp[((s.start - 1) & 1) * heads] : 0.f;
+  const int first = first_chunk(spans, slots, slot, rows, CHUNK), count = (s.rows + CHUNK - 1) / CHUNK;
+  for (int base = 0, turn = 0; base < s.rows; base += TOPS_THREADS, turn ^= 1) {
+    float i = -INFINITY, f = 0.f;
+    if (base + t < s.rows) log_gates(x + (size_t)(s.row0 + base + t) * stride, g, head, i, f);
+#pragma unroll
+    for (int d = 1; d < CHUNK; d <<= 1) {
+      const float before = __shfl_up(f, d, CHUNK);
+      if (l16 >= d) f += before;
+    }
+    const float end = __shfl(f, CHUNK - 1, CHUNK);
+    float top = end - f + i;
+#pragma unroll
+    for (int d = 1; d < CHUNK; d <<= 1) top = fmaxf(top, __shfl_xor(top, d, CHUNK));
+    if (l16 == 0) {
+      sums[turn][t / CHUNK] = end;
+      most[turn][t / CHUNK] = top;
+    }
+    __syncthreads();   // (two sets: the next turn's writers do not meet this one's readers)
+    const int n = min(AT_ONCE, count - base / CHUNK);
+    for (int c = 0; c < n; ++c) {
+      if (t == 0) starts[(size_t)(first + base / CHUNK + c) * heads + head] = m;
+      m = fmaxf(sums[turn][c] + m, most[turn][c]);
+    }
+  }
+  if (t == 0) mp[((s.start + s.rows - 1) & 1) * heads] = m;
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void memory_chunks_kernel(const T* __restrict__ x, MemoryGates g, const int* __restrict__ spans,
+                                                            const float* __restrict__ starts, float* __restrict__ work,
+                                                            float* __restrict__ o, int rows, int slots, int stride, int heads, int dim,
+                                                            int vdim) {
+  extern __shared__ __align__(16) float lds[];
+  __shared__ float4 qk[4][64];
+  __shared__ float gates[2][CHUNK], into[CHUNK], outof[CHUNK], run[CHUNK], top[CHUNK];
+  const int head = blockIdx.y, slot = blockIdx.z, base = blockIdx.x * CHUNK;
+  const Span s = span_of(spans, slot, rows);
+  if (base >= s.rows) return;
+  const int n = min(CHUNK, s.rows - base), tiles = (dim + 15) / 16, wide = tiles * 16, pitch = wide + 4, t = threadIdx.x;
+  const int lane = t & 63, wave = t >> 6, l16 = lane & 15, quad = lane >> 4, chunk = first_chunk(spans, slots, slot, rows, CHUNK) + blockIdx.x;
+  float* qs = lds;                       // [16][pitch]
+  float* ks = qs + CHUNK * pitch;
+  const T* row = x + (size_t)(s.row0 + base) * stride;
+  const float m0 = starts[(size_t)chunk * heads + head], scale = 1.0f / sqrtf((float)dim);
+  if (t < CHUNK) {
+    float i = -INFINITY, f = 0.f;
+    if (t < n) log_gates(row + (size_t)t * stride, g, head, i, f);
+    gates[0][t] = i;
+    gates[1][t] = f;
+  }
+  for (int e = t; e < CHUNK * wide; e += 256) {
+    const int i = e / wide, c = e - i * wide;
+    const bool in = i < n && c < dim;
+    const T* at = row + (size_t)i * stride + head * dim + c;
+    qs[i * pitch + c] = in ? load_one(at) * scale : 0.f;
+    ks[i * pitch + c] = in ? load_one(at + heads * dim) : 0.f;
+  }
+  __syncthreads();
+  if (t == 0) {
+    float sum = 0.f, m = m0;
+    for (int i = 0; i < CHUNK; ++i) {
+      m = fmaxf(gates[1][i] + m, gates[0][i]);   // (of a token past the last: as it was)
+      sum += gates[1][i];
+      run[i] = sum;
+      top[i] = m;
+    }
+  }
+  __syncthreads();
+  const float end = run[CHUNK - 1], m_end = top[CHUNK - 1];
+  if (t < CHUNK) {
+    into[t] = expf(run[t] + m0 - top[t]);
+    outof[t] = expf(end - run[t] + gates[0][t] - m_end);   // 0 past the last token
+    if (t < n) o[(size_t)(s.row0 + base + t) * (heads * vdim + 2 * heads) + heads * vdim + heads + head] = top[t];
+  }
+  f32x4 acc = f32x4{0.f, 0.f, 0.f, 0.f};
+  for (int tile = wave; tile < tiles; tile += 4) {
+    const int c = tile * 16 + quad * 4;
+    const float4 q = *reinterpret_cast<const float4*>(qs + l16 * pitch + c), k = *reinterpret_cast<const float4*>(ks + l16 * pitch + c);
+    acc = product16(f32x4{q.x, q.y, q.z, q.w}, f32x4{k.x, k.y, k.z, k.w}, acc);
+  }
+  qk[wave][lane] = make_float4(acc[0], acc[1], acc[2], acc[3]);
+  __syncthreads();
+  float* out = work + ((size_t)chunk * heads + head) * mix_words(tiles);
+  for (int e = t; e < tiles * 64; e += 256) {
+    const int tile = e >> 6;
+    const float by = into[l16];
+    const float4 q = *reinterpret_cast<const float4*>(qs + l16 * pitch + tile * 16 + quad * 4);
+    float f[4];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) f[j] = ks[(quad * 4 + j) * pitch + tile * 16 + l16] * outof[quad * 4 + j];
+    reinterpret_cast<float4*>(out)[e] = make_float4(q.x * by, q.y * by, q.z * by, q.w * by);
+    reinterpret_cast<float4*>(out + tiles * 256)[e] = make_float4(f[0], f[1], f[2], f[3]);
+  }
+  const float keep = expf(end + m0 - m_end);
+  for (int c = t; c < wide; c += 256) out[tiles * 512 + c] = keep;
+  {
+    const int i = quad * 4 + wave, j = l16;
+    float sum = 0.f;
+#pragma unroll
+    for (int w = 0; w < 4; ++w) sum += reinterpret_cast<const float*>(&qk[w][lane])[wave];
+    // the frag's place of element (i, j): lane (j / 4) * 16 + i, float j % 4
+    out[tiles * 528 + ((j >> 2) * 16 + i) * 4 + (j & 3)] = j <= i && j < n ? sum * expf(run[i] - run[j] + gates[0][j] - top[i]) : 0.f;
+  }
 }
 
 // ------------------------------------------------------------- the delta rule
@@ -484,8 +620,9 @@ extern "C" int iron_time_mix_chunked(const void* r, const void* k, const void* v
   const size_t lds = ((size_t)(3 * CHUNK + 1) * pitch + CHUNK * 17) * 4;
   const dim3 all((rows + CHUNK - 1) / CHUNK, heads, slots), walk(heads, tiles, slots);
   float* work = (float*)workspace;
+  const WalkShape shape{rows, slots, heads, dim, dim, heads * dim, heads * dim};
 #define IRON_MIX_WALK(T, NT, DEPTH) \
-  hipLaunchKernelGGL((time_mix_walk_kernel<T, NT, DEPTH>), walk, dim3(256), 0, s, (const T*)v, state, spans, work, o, rows, slots, heads, dim)
+  hipLaunchKernelGGL((time_mix_walk_kernel<T, NT, DEPTH>), walk, dim3(256), 0, s, (const T*)v, state, spans, work, o, shape)
 #define IRON_MIX(T)                                                                                                             \
   hipLaunchKernelGGL((time_mix_chunks_kernel<T>), all, dim3(256), lds, s, (const T*)r, (const T*)k, log_decay, u, spans, work, rows, \
                      slots, heads, dim);                                                                                        \
@@ -496,6 +633,48 @@ extern "C" int iron_time_mix_chunked(const void* r, const void* k, const void* v
   else { IRON_MIX(bf16_t) }
 #undef IRON_MIX
 #undef IRON_MIX_WALK
+  IRON_LAUNCH_CHECK();
+}
+
+extern "C" int64_t iron_matrix_memory_workspace_bytes(int slots, int rows, int heads, int dim) {
+  return chunks_of(rows, slots, CHUNK) * heads * (int64_t)(mix_words((dim + 15) / 16) * 4 + 4);
+}
+
+extern "C" int iron_matrix_memory_chunked(const void* x, const uint16_t* i_bias, const uint16_t* f_bias, float* state, float* tops,
+                                          const int* spans, float* o, void* workspace, int slots, int rows, int stride, int heads, int dim,
+                                          int vdim, int i_at, int f_at, float cap, int is_float, void* stream) {
+  IRON_REQUIRE(x && i_bias && f_bias && state && tops && o && workspace, "matrix_memory_chunked: null operand");
+  IRON_CHUNKED_REQUIRE("matrix_memory_chunked");
+  IRON_REQUIRE(heads > 0 && heads <= 65535 && dim > 0 && dim <= 256 && vdim > 0,
+               "matrix_memory_chunked: heads (%d) and vdim (%d) positive, dim (%d) from 1 to 256", heads, vdim, dim);
+  const int packed = heads * (2 * dim + vdim);
+  IRON_REQUIRE(i_at >= packed && f_at >= packed && i_at + heads <= stride && f_at + heads <= stride,
+               "matrix_memory_chunked: the gates (%d, %d) lie behind q, k, v (%d) in a row of %d", i_at, f_at, packed, stride);
+  IRON_REQUIRE(cap > 0.f, "matrix_memory_chunked: a cap (%g) above 0", (double)cap);
+  IRON_REQUIRE(((uintptr_t)workspace & 15) == 0, "matrix_memory_chunked: the workspace must be 16-byte aligned");
+  IRON_REQUIRE((long)rows * stride < (1L << 28) && (long)rows * heads * (vdim + 2) < (1L << 28),
+               "matrix_memory_chunked: the batch's rows are addressed with 32-bit offsets");
+  hipStream_t s = (hipStream_t)stream;
+  const int tiles = (dim + 15) / 16;
+  const size_t lds = (size_t)2 * CHUNK * (tiles * 16 + 4) * 4;
+  const dim3 all((rows + CHUNK - 1) / CHUNK, heads, slots), walk(heads, (vdim + 1 + 15) / 16, slots);
+  float *work = (float*)workspace, *starts = work + chunks_of(rows, slots, CHUNK) * heads * (size_t)mix_words(tiles);
+  const MemoryGates g{i_bias, f_bias, i_at, f_at, cap};
+  const WalkShape shape{rows, slots, heads, dim, vdim, stride, heads * vdim + 2 * heads};
+#define IRON_MEMORY_WALK(T, NT, DEPTH) \
+  hipLaunchKernelGGL((time_mix_walk_kernel<T, NT, DEPTH, true>), walk, dim3(256), 0, s, (const T*)x + 2 * heads * dim, state, spans, work, o, shape)
+#define IRON_MEMORY(T)                                                                                                                  \
+  hipLaunchKernelGGL((memory_tops_kernel<T>), dim3(heads, slots), dim3(TOPS_THREADS), 0, s, (const T*)x, g, tops, spans, starts, rows,  \
+                     slots, stride, heads);                                                                                             \
+  hipLaunchKernelGGL((memory_chunks_kernel<T>), all, dim3(256), lds, s, (const T*)x, g, spans, starts, work, o, rows, slots, stride,    \
+                     heads, dim, vdim);                                                                                                 \
+  if (tiles <= 4) IRON_MEMORY_WALK(T, 1, 6);                                                                                            \
+  else if (tiles <= 8) IRON_MEMORY_WALK(T, 2, 4);                                                                                       \
+  else IRON_MEMORY_WALK(T, 4, 2);
+  if (is_float) { IRON_MEMORY(float) }
+  else { IRON_MEMORY(bf16_t) }
+#undef IRON_MEMORY
+#undef IRON_MEMORY_WALK
   IRON_LAUNCH_CHECK();
 }
 

@@ -3,7 +3,9 @@
 //
 //   router:   float32 logits, a row a block
 //   pairs:    a (row, chosen expert) at a time, the weights' rows dealt to waves (few rows; either type)
+//   grouped:  pairs dealt to their experts, each expert's padded to whole row tiles, two grouped products and a row's sum (bf16)
 #include "../../include/iron_hip.h"
+#include "grouped.h"
 #include "rows.h"
 
 namespace iron {
@@ -152,6 +154,78 @@ __global__ __launch_bounds__(256) void expert_sums_kernel(const T* __restrict__ 
   }
 }
 
+// ------------------------------------------------------------- many rows
+// A call's workspace behind these offsets (in bytes): what the plan leaves, the activated rows, the experts' rows.
+struct GroupedPlan {
+  int most;                    // row tiles there can be
+  size_t which, place, rows, acts, outs, bytes;
+  GroupedPlan(int pairs, int experts, int cols, int ff) {
+    auto up = [](size_t n) { return (n + 255) & ~(size_t)255; };
+    most = pairs / 128 + (pairs < experts ? pairs : experts);
+    which = 256;                                     // (the count stands first)
+    place = which + up((size_t)most * 4);            // a pair's place among the sorted
+    rows = place + up((size_t)pairs * 4);            // a place's row
+    acts = rows + up((size_t)most * 128 * 4);
+    outs = acts + up((size_t)most * 128 * ff * 2);
+    bytes = outs + up((size_t)most * 128 * cols * 2);
+  }
+};
+
+// One block: how many pairs each expert has, where its tiles begin, and every pair's place.
+__global__ __launch_bounds__(1024) void expert_plan_kernel(const int* __restrict__ ids, int* __restrict__ count, int* __restrict__ which,
+                                                           int* __restrict__ place, int* __restrict__ rows_of, int rows, int experts, int top,
+                                                           int most, const int* __restrict__ valid) {
+  __shared__ int held[ROUTER_MAX], first[ROUTER_MAX], scan[2][ROUTER_MAX];
+  const int t = threadIdx.x, pairs = bound_or(valid, rows) * top;
+  held[t] = 0;
+  for (int i = t; i < most * 128; i += 1024) rows_of[i] = 0;   // a tile's places past its expert's pairs
+  __syncthreads();
+  for (int p = t; p < pairs; p += 1024) atomicAdd(&held[min(max(ids[p], 0), experts - 1)], 1);
+  __syncthreads();
+  const int tiles = (held[t] + 127) / 128;
+  scan[0][t] = tiles;
+  __syncthreads();
+  int at = 0;
+  for (int d = 1; d < ROUTER_MAX; d <<= 1, at ^= 1) {
+    scan[at ^ 1][t] = scan[at][t] + (t >= d ? scan[at][t - d] : 0);
+    __syncthreads();
+  }
+  const int begin = scan[at][t] - tiles;
+  first[t] = begin * 128;
+  for (int i = 0; i < tiles; ++i)
+    if (begin + i < most) which[begin + i] = t;
+  if (t == 0) *count = min(scan[at][ROUTER_MAX - 1], most);
+  __syncthreads();
+  for (int p = t; p < pairs; p += 1024) {
+    const int to = min(atomicAdd(&first[min(max(ids[p], 0), experts - 1)], 1), most * 128 - 1);
+    place[p] = to;
+    rows_of[to] = p / top;
+  }
+}
+
+// y[row] = sum over its pairs of share * what the pair's expert left.
+__global__ __launch_bounds__(256) void expert_gather_kernel(const bf16_t* __restrict__ outs, const int* __restrict__ place,
+                                                            const float* __restrict__ shares, bf16_t* __restrict__ y, int rows, int cols,
+                                                            int top, const int* __restrict__ valid) {
+  const int row = blockIdx.y, c = (blockIdx.x * 256 + threadIdx.x) * 8;
+  if (row >= bound_or(valid, rows) || c >= cols) return;
+  float sum[8];
+#pragma unroll
+  for (int j = 0; j < 8; ++j) sum[j] = 0.f;
+#pragma unroll 4
+  for (int k = 0; k < top; ++k) {
+    float f[8];
+    load_vec<8>(outs + (size_t)place[row * top + k] * cols + c, f);
+    const float share = shares[row * top + k];
+#pragma unroll
+    for (int j = 0; j < 8; ++j) sum[j] = fmaf(share, f[j], sum[j]);
+  }
+  store_vec<8>(y + (size_t)row * cols + c, sum);
+}
+
+// Rows from which a portion's pairs are grouped.
+static bool grouped_pays(int rows, int cols, int ff, int is_float) { return !is_float && rows >= 64 && cols % 64 == 0 && ff % 64 == 0; }
+
 }  // namespace iron
 
 using namespace iron;
@@ -172,7 +246,7 @@ extern "C" int iron_router(const void* h, const uint16_t* w, const uint16_t* bia
 }
 
 extern "C" int64_t iron_experts_workspace_bytes(int rows, int cols, int ff, int experts, int top, int is_float) {
-  (void)cols; (void)experts;
+  if (grouped_pays(rows, cols, ff, is_float)) return (int64_t)GroupedPlan(rows * top, experts, cols, ff).bytes;
   return (int64_t)rows * top * ff * (is_float ? 4 : 2);
 }
 
@@ -183,8 +257,24 @@ extern "C" int iron_experts(const void* h, const uint16_t* gate, const uint16_t*
   IRON_REQUIRE(rows > 0 && cols > 0 && ff > 0 && experts > 0 && top > 0 && top <= experts, "experts: sizes must be positive, top (%d) of %d experts",
                top, experts);
   IRON_REQUIRE(activation >= 1 && activation <= 3, "experts: activation (%d) is 1 (SiLU), 2 (GELU, tanh form) or 3 (ReLU)", activation);
-  IRON_REQUIRE((long)rows * top <= 65535, "experts: %d rows of %d experts exceed the grid's y extent", rows, top);
   hipStream_t s = (hipStream_t)stream;
+  if (grouped_pays(rows, cols, ff, is_float)) {
+    IRON_REQUIRE(experts <= ROUTER_MAX && rows <= 65535 && (long)rows * top <= (1 << 24) && (long)rows * cols < (1L << 30),
+                 "experts: %d rows, %d of %d experts", rows, top, experts);
+    IRON_REQUIRE((((uintptr_t)h | (uintptr_t)gate | (uintptr_t)up | (uintptr_t)down | (uintptr_t)workspace | (uintptr_t)y) & 15) == 0,
+                 "experts: operands must be 16-byte aligned");
+    const GroupedPlan p(rows * top, experts, cols, ff);
+    char* w = (char*)workspace;
+    int *count = (int*)w, *which = (int*)(w + p.which), *place = (int*)(w + p.place), *rows_of = (int*)(w + p.rows);
+    const GroupedTiles g{count, which, p.most};
+    bf16_t *acts = (bf16_t*)(w + p.acts), *outs = (bf16_t*)(w + p.outs);
+    hipLaunchKernelGGL(expert_plan_kernel, dim3(1), dim3(1024), 0, s, ids, count, which, place, rows_of, rows, experts, top, p.most, valid);
+    if (int e = launch_grouped_pair((const bf16_t*)h, gate, up, acts, ff, cols, g, rows_of, activation, s)) return e;
+    if (int e = launch_grouped(acts, down, outs, cols, ff, g, s)) return e;
+    hipLaunchKernelGGL(expert_gather_kernel, dim3((cols + 2047) / 2048, rows), dim3(256), 0, s, outs, place, shares, (bf16_t*)y, rows, cols, top, valid);
+    IRON_LAUNCH_CHECK();
+  }
+  IRON_REQUIRE((long)rows * top <= 65535, "experts: %d rows of %d experts exceed the grid's y extent", rows, top);
   const bool vec = cols % 8 == 0 && ff % 8 == 0 &&
                    (((uintptr_t)h | (uintptr_t)gate | (uintptr_t)up | (uintptr_t)down | (uintptr_t)workspace | (uintptr_t)y) & 15) == 0;
 #define IRON_PAIRS(T, VEC)                                                                                                                    \

@@ -14,6 +14,7 @@
 // lane ends up holding 4 consecutive columns of one row of C and stores them as 8 bytes.
 #include "../../include/iron_hip.h"
 #include "common.h"
+#include "grouped.h"
 
 #include <type_traits>
 
@@ -1808,11 +1809,14 @@ __global__ __launch_bounds__(256) void gemm_finish_rows_kernel(const float* __re
 // Against the same body run twice this fetches A once instead of twice (a quarter of the bytes a
 // CU draws from L2 and a quarter of its LDS fragment reads).  Each product's MFMAs run in the order
 // of the single-product body, so G and C are the separate launches' bit for bit.
+// GROUPED: the caller has chosen the tile (tiles_m, tiles_n stand for its place), A's rows are those `a_rows` lists, and the
+// gate's product is not stored.
+template <bool GROUPED = false>
 __device__ __forceinline__ void gemm_nt16_pair_body(const bf16_t* __restrict__ A, const bf16_t* __restrict__ Bg,
                                                     const bf16_t* __restrict__ Bu, bf16_t* __restrict__ G,
                                                     bf16_t* __restrict__ C, int M, int N, int K,
                                                     const int* __restrict__ valid, int tiles_m, int tiles_n,
-                                                    int patched, int activation) {
+                                                    int patched, int activation, const int* __restrict__ a_rows = nullptr) {
   constexpr int NT_BM = 128, NT_BN = 128;
   constexpr int PART = NT_BM * BK * 2;             // a 128 x 64 tile's 16 KB: A, then the gate's, then the up projection's
   constexpr int STAGE = 3 * PART, STAGES = PAIR_STAGES;
@@ -1822,8 +1826,8 @@ __device__ __forceinline__ void gemm_nt16_pair_body(const bf16_t* __restrict__ A
   extern __shared__ __align__(16) char smem_nt[];
   const int Mv = bound_or(valid, M);
 
-  int tm, tn;
-  tile_of_block(blockIdx.x, tiles_m, tiles_n, patched, tm, tn);
+  int tm = tiles_m, tn = tiles_n;
+  if constexpr (!GROUPED) tile_of_block(blockIdx.x, tiles_m, tiles_n, patched, tm, tn);
   const int m0 = tm * NT_BM;
   if (m0 >= Mv) return;
   const int n0 = tn * NT_BN;
@@ -1837,10 +1841,11 @@ __device__ __forceinline__ void gemm_nt16_pair_body(const bf16_t* __restrict__ A
     const int r = (wave * INST + i) * 8 + lrow;
     const int lch = pch ^ ((r >> 1) & 7);
     // Rows past the end re-read the last row; what they produce is never stored.
-    a_voff[i] = (int)(((size_t)(min(m0 + r, M - 1) - m0) * K + lch * 8) * 2);
+    if constexpr (GROUPED) a_voff[i] = (int)(((size_t)a_rows[m0 + r] * K + lch * 8) * 2);
+    else a_voff[i] = (int)(((size_t)(min(m0 + r, M - 1) - m0) * K + lch * 8) * 2);
     b_voff[i] = (int)(((size_t)(min(n0 + r, N - 1) - n0) * K + lch * 8) * 2);
   }
-  const bf16_t* a_tile = A + (size_t)m0 * K;
+  const bf16_t* a_tile = GROUPED ? A : A + (size_t)m0 * K;
   const bf16_t* g_tile = Bg + (size_t)n0 * K;
   const bf16_t* u_tile = Bu + (size_t)n0 * K;
   auto issue_one = [&](char* st, int kt, int idx) {   // idx: 0..3 A, 4..7 the gate's weights, 8..11 the up projection's
@@ -1968,13 +1973,15 @@ __device__ __forceinline__ void gemm_nt16_pair_body(const bf16_t* __restrict__ A
     __builtin_amdgcn_wave_barrier();   // the rows are read before the next product overwrites them
     __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
   };
+  if constexpr (!GROUPED) {
 #pragma unroll
-  for (int i = 0; i < 4; ++i)
+    for (int i = 0; i < 4; ++i)
 #pragma unroll
-    for (int j = 0; j < 4; ++j)
-      *reinterpret_cast<uint2*>(ot + (i * 16 + fr) * OROWB + (j * 16 + 4 * kq) * 2) =
-          make_uint2(pack_bf16(accg[i][j][0], accg[i][j][1]), pack_bf16(accg[i][j][2], accg[i][j][3]));
-  leave(G);
+      for (int j = 0; j < 4; ++j)
+        *reinterpret_cast<uint2*>(ot + (i * 16 + fr) * OROWB + (j * 16 + 4 * kq) * 2) =
+            make_uint2(pack_bf16(accg[i][j][0], accg[i][j][1]), pack_bf16(accg[i][j][2], accg[i][j][3]));
+    leave(G);
+  }
 #pragma unroll
   for (int i = 0; i < 4; ++i)
 #pragma unroll
@@ -2039,6 +2046,61 @@ static int launch_gemm_gated_pair(const bf16_t* A, const bf16_t* Bg, const bf16_
   if (t64.tiles_m * t64.tiles_n > blocks) blocks = t64.tiles_m * t64.tiles_n;
   hipLaunchKernelGGL(gemm_gated_pair_kernel, dim3(blocks), dim3(256), lds, s, A, Bg, Bu, G, C, M, N, K, valid, t128, t64,
                      few128, activation);
+  IRON_LAUNCH_CHECK();
+}
+
+// Products of rows dealt to several weights of one shape, stacked: the rows lie (or are listed) weight by weight, each
+// weight's padded to whole 128-row tiles, and GroupedTiles says which weight a row tile belongs to.  Blocks of an XCD share
+// columns of tiles, and go down them weight by weight: a weight's tile crosses HBM once.
+__device__ __forceinline__ bool grouped_tile(const GroupedTiles& g, int tiles_n, int& tm, int& tn, int& which) {
+  if (tiles_n % 8 == 0) {
+    const int loc = blockIdx.x >> 3;
+    tm = loc % g.most;
+    tn = (loc / g.most) * 8 + ((int)blockIdx.x & 7);
+  } else {
+    tm = (int)blockIdx.x % g.most;
+    tn = (int)blockIdx.x / g.most;
+  }
+  if (tm >= *g.count) return false;
+  which = g.which[tm];
+  return true;
+}
+__global__ __launch_bounds__(256) void gemm_grouped_pair_kernel(const bf16_t* __restrict__ A, const bf16_t* __restrict__ Bg,
+                                                                const bf16_t* __restrict__ Bu, bf16_t* __restrict__ C, int N, int K,
+                                                                GroupedTiles g, const int* __restrict__ a_rows, int activation) {
+  int tm, tn, e;
+  if (!grouped_tile(g, (N + 127) / 128, tm, tn, e)) return;
+  gemm_nt16_pair_body<true>(A, Bg + (size_t)e * N * K, Bu + (size_t)e * N * K, nullptr, C, g.most * 128, N, K, nullptr, tm, tn, 0, activation, a_rows);
+}
+__global__ __launch_bounds__(256) void gemm_grouped_kernel(const bf16_t* __restrict__ A, const bf16_t* __restrict__ B, bf16_t* __restrict__ C,
+                                                           int N, int K, GroupedTiles g) {
+  int tm, tn, e;
+  const int tiles_n = (N + 127) / 128;
+  if (!grouped_tile(g, tiles_n, tm, tn, e)) return;
+  QkvTail tail{};
+  tail.tile_plus1 = tm * tiles_n + tn + 1;
+  gemm_nt16_body<false>(A, B + (size_t)e * N * K, C, g.most * 128, N, K, nullptr, g.most, tiles_n, 0, tail);
+}
+
+int launch_grouped_pair(const bf16_t* A, const bf16_t* Bg, const bf16_t* Bu, bf16_t* C, int N, int K, const GroupedTiles& g,
+                        const int* a_rows, int activation, hipStream_t s) {
+  constexpr size_t lds = (size_t)PAIR_STAGES * 3 * 128 * BK * 2;
+  static LdsOptIn opt_in;
+  if (hipError_t e = opt_in.ensure(reinterpret_cast<const void*>(&gemm_grouped_pair_kernel), lds); e != hipSuccess) {
+    set_error("gemm_grouped_pair: %s", hipGetErrorString(e));
+    return (int)e;
+  }
+  hipLaunchKernelGGL(gemm_grouped_pair_kernel, dim3(g.most * ((N + 127) / 128)), dim3(256), lds, s, A, Bg, Bu, C, N, K, g, a_rows, activation);
+  IRON_LAUNCH_CHECK();
+}
+int launch_grouped(const bf16_t* A, const bf16_t* B, bf16_t* C, int N, int K, const GroupedTiles& g, hipStream_t s) {
+  constexpr size_t lds = (size_t)NT_STAGES * 256 * BK * 2;
+  static LdsOptIn opt_in;
+  if (hipError_t e = opt_in.ensure(reinterpret_cast<const void*>(&gemm_grouped_kernel), lds); e != hipSuccess) {
+    set_error("gemm_grouped: %s", hipGetErrorString(e));
+    return (int)e;
+  }
+  hipLaunchKernelGGL(gemm_grouped_kernel, dim3(g.most * ((N + 127) / 128)), dim3(256), lds, s, A, B, C, N, K, g);
   IRON_LAUNCH_CHECK();
 }
 

@@ -10,7 +10,7 @@
 // Float32 throughout.  A block holds 16 columns of a head's state: a wave 4 columns, 16 lanes a column, NI consecutive rows
 // of it a lane.
 #include "../../include/iron_hip.h"
-#include "rows.h"
+#include "matrix_memory.h"
 
 namespace iron {
 
@@ -27,10 +27,6 @@ struct MemoryIn {
   const int* spans;
   float* o;                              // [rows][heads * vdim | heads n . q | heads m]
 };
-
-// log(sigmoid(z)) without a difference of large numbers.
-__device__ __forceinline__ float log_sigmoid(float z) { return fminf(z, 0.f) - log1pf(expf(-fabsf(z))); }
-__device__ __forceinline__ float capped(float z, float cap) { return cap * tanhf(z / cap); }
 
 constexpr int MEM_TOKENS = 16, MEM_COLUMNS = 16;
 

@@ -695,13 +695,20 @@ def mha_talking(x, keys, values, talk, spans, y, *, slots, rows, stride, heads, 
                                  dim, vdim, chunk, ring, int(single), int(is_float), current_stream()), "iron_mha_talking")
 
 
-def matrix_memory(x, i_bias, f_bias, state, tops, spans, o, *, slots, rows, stride, heads, dim, vdim, i_at, f_at, cap):
+def matrix_memory(x, i_bias, f_bias, state, tops, spans, o, *, slots, rows, stride, heads, dim, vdim, i_at, f_at, cap, workspace=None):
+    """The recurrence token by token, or with ``workspace`` sixteen tokens at a time."""
     is_float = _act(x, rows * stride, "x")
     _bf16(i_bias, heads, "i_bias")
     _bf16(f_bias, heads, "f_bias")
     _f32(state, slots * heads * dim * (vdim + 1), "state")
     _f32(tops, slots * 2 * heads, "tops")
     _f32(o, rows * heads * (vdim + 2), "o")
+    if workspace is not None:
+        work = _work(workspace, int(lib().iron_matrix_memory_workspace_bytes(slots, rows, heads, dim)), "matrix_memory: workspace")
+        check(lib().iron_matrix_memory_chunked(ptr(x), ptr(i_bias), ptr(f_bias), ptr(state), ptr(tops), _spans(spans, slots), ptr(o), work,
+                                               slots, rows, stride, heads, dim, vdim, i_at, f_at, float(cap), int(is_float), current_stream()),
+              "iron_matrix_memory_chunked")
+        return
     check(lib().iron_matrix_memory(ptr(x), ptr(i_bias), ptr(f_bias), ptr(state), ptr(tops), _spans(spans, slots), ptr(o), slots, rows, stride,
                                    heads, dim, vdim, i_at, f_at, float(cap), int(is_float), current_stream()), "iron_matrix_memory")
 

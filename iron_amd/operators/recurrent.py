@@ -354,7 +354,15 @@ class MatrixMemory(_Spanned):
     tops = InOut(slots, 2, heads, dtype=F32)
     spans = In(slots, 4, dtype=np.int32)
     o = Out(rows, width, dtype=F32)
+    chunked: bool = param(default=lambda op: op.rows > op.CHUNKED_ROWS * op.slots and op.dim <= 256, array=True, repr=False)
+    workspace_words: int = param(derive=lambda op: op._workspace_words(), repr=False)
+    workspace = Scratch(workspace_words, dtype=F32, when=chunked)
     valid = per_call(bounds=rows)
+
+    def _workspace_words(self) -> int:
+        from .._lib import lib
+
+        return int(lib().iron_matrix_memory_workspace_bytes(self.slots, self.rows, self.heads, self.dim)) // 4
 
     @classmethod
     def infer(cls, shapes, **kw):
@@ -373,7 +381,8 @@ class MatrixMemory(_Spanned):
         kw["cap"] = float(self.cap)
 
         def launch(t, words):
-            kernels.matrix_memory(t["x"], t["i_bias"], t["f_bias"], t["state"], t["tops"], t["spans"], t["o"], **kw)
+            kernels.matrix_memory(t["x"], t["i_bias"], t["f_bias"], t["state"], t["tops"], t["spans"], t["o"],
+                                  workspace=t.get("workspace"), **kw)
 
         return Built("iron_matrix_memory", launch)
 

@@ -202,17 +202,24 @@ def memory_op(slots, rows, H, D, V, dtype, more=0, cap=9.0):
                         cap=cap, dtype=dtype)
 
 
+TOKENS = pytest.mark.parametrize("chunked", [False, True], ids=["tokens", "chunks"])
+
+
 @BOTH
+@TOKENS
 @pytest.mark.parametrize("H,D,V", [(2, 24, 40), (3, 5, 9), (1, 33, 3), (4, 16, 16), (2, 64, 128), (2, 128, 64), (2, 128, 256), (1, 256, 160), (1, 300, 33)])
-def test_a_matrix_memory(cuda, dtype, H, D, V):
+def test_a_matrix_memory(cuda, dtype, chunked, H, D, V):
+    if chunked and D > 256:
+        pytest.skip("longer keys go token by token")
     rng = np.random.default_rng(D)
     # lengths around a chunk's, rows out of slot order, slots that go on and ones that start over
     spans = table((0, 130, 33, 9), (1, 0, 32, 0), (2, 32, 1, 3), (4, 33, 97, 0), (5, 163, 2, 40), slots=6)
     op = memory_op(6, 170, H, D, V, dtype, more=H * V)
-    agrees(op, memory_inputs(rng, op, spans), 2e-5, rows_of(spans))
+    agrees(op, memory_inputs(rng, op, spans), 2e-5, rows_of(spans), workspace=chunked)
 
 
-def test_the_memory_goes_on_where_a_portion_ends(cuda):
+@TOKENS
+def test_the_memory_goes_on_where_a_portion_ends(cuda, chunked):
     rng = np.random.default_rng(7)
     H, D, V, T = 2, 32, 48, 200
     op = memory_op(1, T, H, D, V, F32)
@@ -224,12 +231,21 @@ def test_the_memory_goes_on_where_a_portion_ends(cuda):
     for sizes in ([T], [2, 31, 1, 70, 33, 2, 61], [16] * 12 + [8], [1] * 40):
         state, tops, at = whole["state"], whole["tops"], 0
         for n in sizes:
-            got = ran(memory_op(1, n, H, D, V, F32), **{**whole, "x": whole["x"][at : at + n], "state": state, "tops": tops, "spans": table((0, 0, n, at))})
+            got = ran(memory_op(1, n, H, D, V, F32), workspace=chunked, **{**whole, "x": whole["x"][at : at + n], "state": state, "tops": tops, "spans": table((0, 0, n, at))})
             o = got["o"].astype(np.float64)
             under = np.maximum(np.abs(o[:, H * V : H * V + H]), np.exp(-o[:, H * V + H :])) + 1e-6
             y = o[:, : H * V].reshape(n, H, V) / under[:, :, None]
             assert np.abs(y - want[at : at + n]).max() <= 2e-4 * np.abs(want).max(), (sizes[:3], at)   # (a quotient by what may be small)
             state, tops, at = got["state"], got["tops"], at + n
+
+
+@TOKENS
+def test_a_memory_over_many_chunks(cuda, chunked):
+    """More chunks than a launch composes at once, requests of several portions' length side by side."""
+    rng = np.random.default_rng(9)
+    spans = table((0, 5, 1500, 0), (2, 1505, 1100, 33), slots=3)
+    op = memory_op(3, 2700, 1, 20, 24, F32)
+    agrees(op, memory_inputs(rng, op, spans), 1e-4, rows_of(spans), workspace=chunked)
 
 
 @BOTH
@@ -280,13 +296,14 @@ def test_routed_feed_forwards(cuda, dtype, rows, cols, ff, experts, top):
 # ---------------------------------------------------------------- whole models
 
 
-LIMIT = {"f32": 2e-4, "bf16": 0.15}   # of the logits' spread
+LIMIT = {"f32": 2e-4, "bf16": 0.1}   # of the logits' spread
 
 
 def off_by(got, want, limit):
-    """The largest difference of a row, or, where rounding may turn a router's close call, that of all but a tenth of the rows."""
+    """The largest difference of a row; the middle one where rounding may turn a router's close call, which moves a row and what
+    a state carries of it by itself."""
     each = np.array([far_off(g[None], w[None], want.std()) for g, w in zip(got, want)])
-    return float(each.max() if limit < 1e-2 else np.quantile(each, 0.9))
+    return float(each.max() if limit < 1e-2 else np.median(each))
 
 
 @pytest.fixture(scope="module", params=[(n, d, f) for n in MODELS for d in ("f32", "bf16") for f in ((True, False) if d == "bf16" else (True,))],
@@ -332,7 +349,9 @@ def test_batches_and_slots_used_again(cuda, served):
                 for k, r in zip(live, model.batch.step([Entry(k, [prompts[k][first[k] + i]], [0]) for k in live])):
                     rows[k].append(r)
         for k in order:
-            assert off_by(np.concatenate(rows[k]), want[k], limit) < limit, (order, k)
+            off = off_by(np.concatenate(rows[k]), want[k], limit)
+            print(order, k, off)
+            assert off < limit, (order, k)
             model.batch.end(k)
 
 
