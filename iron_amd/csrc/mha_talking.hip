@@ -11,6 +11,8 @@
 // ring is written after they have been attended.
 //
 //   rows kernel:    a block a query row with all its heads, twice over the keys (either type)
+//   step kernels:   one row a slot: all scores first, then a block some columns of a key/value head's values
+//   prompt kernels: bf16 MFMAs; the rows' softmax statistics a head first, then 16 queries with all their heads a block
 #include "../../include/iron_hip.h"
 #include "window.h"
 
@@ -134,14 +136,14 @@ __host__ __device__ inline int talk_row_words(int heads, int dim, int vdim) {
   return heads * dim + heads * vdim + 2 * heads * TALK_KEYS + 2 * heads;
 }
 
-template <typename T, int VEC, bool STORE>
-__global__ __launch_bounds__(256) void talking_rows_kernel(const T* __restrict__ x, T* __restrict__ keys, T* __restrict__ values,
+template <typename T, int VEC>
+__global__ __launch_bounds__(256) void talking_rows_kernel(const T* __restrict__ x, const T* __restrict__ keys, const T* __restrict__ values,
                                                            const bf16_t* __restrict__ talk, const int* __restrict__ spans,
                                                            T* __restrict__ out, TalkShape a) {
   extern __shared__ __align__(16) float lds[];
   const int slot = blockIdx.y, i = blockIdx.x;
   const Span s = span_of(spans, slot, a.p.rows);
-  if (i >= s.rows || (STORE && i > 0)) return;
+  if (i >= s.rows) return;
   const int H = a.p.heads, G = a.p.kv_heads, D = a.p.dim, V = a.p.vdim, each = H / G, nk = G * D, nv = G * V;
   float* qs = lds;                        // [H][D]
   float* acc = qs + H * D;                // [H][V]
@@ -163,12 +165,6 @@ __global__ __launch_bounds__(256) void talking_rows_kernel(const T* __restrict__
   for (int h = t; h < H; h += 256) {
     ms[h] = -INFINITY;
     ls[h] = 0.f;
-  }
-  if (STORE) {
-    T* kd = keys + ((size_t)slot * a.p.ring + pos % a.p.ring) * nk;
-    T* vd = values + ((size_t)slot * a.p.ring + pos % a.p.ring) * nv;
-    for (int c = t; c < nk; c += 256) kd[c] = row[H * D + c];
-    for (int c = t; c < nv; c += 256) vd[c] = row[H * D + nk + c];
   }
   __syncthreads();
   auto score = [&](int h, int k0) {
@@ -215,6 +211,447 @@ __global__ __launch_bounds__(256) void talking_rows_kernel(const T* __restrict__
   for (int o = t; o < H * V; o += 256) store_one(out + (size_t)(s.row0 + i) * a.out_stride + o, acc[o]);   // (its own)
 }
 
+// ---------------------------------------------------------------- a step
+// One row a slot, two launches.  talking_scores: a wave 64 keys of one key head: the scores of its query heads, left in memory,
+// their largest and the sum of exponentials under it; the row's own key and value go into the ring.  talking_mix: a block VEC
+// columns of a value head, a thread a key: all heads' weights of that key, mixed for up to eight heads, times the value.
+constexpr int STEP_HEADS = 8;
+struct StepWork {   // floats a slot: scores [heads][chunk], then (largest, sum) [heads][pieces of 64 keys]
+  int pieces;
+  size_t stats, words;
+  __host__ __device__ StepWork(int heads, int chunk) : pieces((chunk + 63) / 64), stats((size_t)heads * chunk), words(stats + (size_t)heads * 2 * pieces) {}
+};
+template <typename T>
+__device__ __forceinline__ float weight_exp(float x) {
+  if constexpr (sizeof(T) == 2) return __expf(x);
+  else return expf(x);
+}
+
+template <typename T, int VEC>
+__global__ __launch_bounds__(64) void talking_scores_kernel(const T* __restrict__ x, T* __restrict__ keys, T* __restrict__ values,
+                                                            const int* __restrict__ spans, float* __restrict__ work, TalkShape a) {
+  extern __shared__ __align__(16) float qs[];   // [each][dim]
+  const int g = blockIdx.y, slot = blockIdx.z, k0 = blockIdx.x * 64, lane = threadIdx.x;
+  const Span s = span_of(spans, slot, a.p.rows);
+  const int pos = s.start, lo = pos / a.chunk * a.chunk, count = pos - lo + 1;
+  if (s.rows == 0 || k0 >= count) return;
+  const int H = a.p.heads, G = a.p.kv_heads, D = a.p.dim, V = a.p.vdim, each = H / G;
+  const T* row = x + (size_t)s.row0 * a.p.stride;
+  const T* own = row + H * D + g * D;
+  T* ring = keys + (size_t)slot * a.p.ring * G * D + g * D;
+  for (int c = lane; c < each * D; c += 64) qs[c] = load_one(row + g * each * D + c);
+  if (k0 == 0) {
+    const T* v = row + (H + G) * D + g * V;
+    T* vd = values + ((size_t)slot * a.p.ring + pos % a.p.ring) * G * V + g * V;
+    for (int c = lane; c < D; c += 64) ring[(size_t)(pos % a.p.ring) * G * D + c] = own[c];
+    for (int c = lane; c < V; c += 64) vd[c] = v[c];
+  }
+  __syncthreads();
+  const StepWork w(H, a.chunk);
+  float* mine = work + slot * w.words;
+  const int j = k0 + lane, p = lo + min(j, count - 1);
+  const T* kr = p == pos ? own : ring + (size_t)(p % a.p.ring) * G * D;
+  for (int e0 = 0; e0 < each; e0 += 4) {
+    float dot[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+    for (int c = 0; c < D; c += VEC) {
+      float f[VEC];
+      load_vec<VEC>(kr + c, f);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const float* q = qs + min(e0 + e, each - 1) * D + c;
+#pragma unroll
+        for (int n = 0; n < VEC; ++n) dot[e] = fmaf(f[n], q[n], dot[e]);
+      }
+    }
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      if (e0 + e >= each) continue;
+      const int h = g * each + e0 + e;
+      const float v = j < count ? dot[e] : -INFINITY, top = wave_max(v), sum = wave_sum(weight_exp<T>(v - top));
+      if (j < count) mine[(size_t)h * a.chunk + j] = v;
+      if (lane == 0) {
+        float* st = mine + w.stats + ((size_t)h * w.pieces + blockIdx.x) * 2;
+        st[0] = top;
+        st[1] = sum;
+      }
+    }
+  }
+}
+
+template <typename T, int VEC>
+__global__ __launch_bounds__(1024) void talking_mix_kernel(const T* __restrict__ x, const T* __restrict__ values, const bf16_t* __restrict__ talk,
+                                                           const int* __restrict__ spans, const float* __restrict__ work, T* __restrict__ out,
+                                                           TalkShape a) {
+  extern __shared__ __align__(16) float lds[];
+  __shared__ float red[16][STEP_HEADS * VEC];
+  const int slot = blockIdx.z, t = threadIdx.x, lane = t & 63, wave = t >> 6, waves = blockDim.x >> 6;
+  const Span s = span_of(spans, slot, a.p.rows);
+  if (s.rows == 0) return;
+  const int H = a.p.heads, G = a.p.kv_heads, D = a.p.dim, V = a.p.vdim, each = H / G, octets = (each + STEP_HEADS - 1) / STEP_HEADS;
+  const int g = blockIdx.y / octets, e0 = blockIdx.y % octets * STEP_HEADS, n = min(STEP_HEADS, each - e0), c = blockIdx.x * VEC;
+  const int pos = s.start, lo = pos / a.chunk * a.chunk, count = pos - lo + 1, live = (count + 63) / 64;
+  const StepWork w(H, a.chunk);
+  const float* mine = work + slot * w.words;
+  float* by = lds;                         // [H][8]: what the octet's heads take of a head, over its sum
+  float* top = by + H * STEP_HEADS;        // [H]
+  for (int h = t; h < H; h += blockDim.x) {
+    const float* st = mine + w.stats + (size_t)h * w.pieces * 2;
+    float m = -INFINITY, l = 0.f;
+    for (int i = 0; i < live; ++i) m = fmaxf(m, st[2 * i]);
+    for (int i = 0; i < live; ++i) l = fmaf(st[2 * i + 1], expf(st[2 * i] - m), l);
+    top[h] = m;
+    for (int e = 0; e < STEP_HEADS; ++e) by[h * STEP_HEADS + e] = e < n ? bf16_to_f32(talk[(size_t)(g * each + e0 + e) * H + h]) / l : 0.f;
+  }
+  __syncthreads();
+  float acc[STEP_HEADS][VEC];
+#pragma unroll
+  for (int e = 0; e < STEP_HEADS; ++e)
+#pragma unroll
+    for (int k = 0; k < VEC; ++k) acc[e][k] = 0.f;
+  const T* own = x + (size_t)s.row0 * a.p.stride + (H + G) * D + g * V + c;
+  const T* ring = values + (size_t)slot * a.p.ring * G * V + g * V + c;
+  for (int j = t; j < count; j += blockDim.x) {
+    const int p = lo + j;
+    float f[VEC], mixed[STEP_HEADS];
+    load_vec<VEC>(p == pos ? own : ring + (size_t)(p % a.p.ring) * G * V, f);
+#pragma unroll
+    for (int e = 0; e < STEP_HEADS; ++e) mixed[e] = 0.f;
+#pragma unroll 4
+    for (int h = 0; h < H; ++h) {
+      const float weight = weight_exp<T>(mine[(size_t)h * a.chunk + j] - top[h]);
+#pragma unroll
+      for (int e = 0; e < STEP_HEADS; ++e) mixed[e] = fmaf(by[h * STEP_HEADS + e], weight, mixed[e]);
+    }
+#pragma unroll
+    for (int e = 0; e < STEP_HEADS; ++e)
+#pragma unroll
+      for (int k = 0; k < VEC; ++k) acc[e][k] = fmaf(mixed[e], f[k], acc[e][k]);
+  }
+#pragma unroll
+  for (int e = 0; e < STEP_HEADS; ++e)
+    if (e < n) {
+#pragma unroll
+      for (int k = 0; k < VEC; ++k) {
+        const float sum = wave_sum(acc[e][k]);
+        if (lane == 0) red[wave][e * VEC + k] = sum;
+      }
+    }
+  __syncthreads();
+  if (t < n * VEC) {
+    float sum = 0.f;
+    for (int i = 0; i < waves; ++i) sum += red[i][t];
+    store_one(out + (size_t)s.row0 * a.out_stride + (g * each + e0 + t / VEC) * V + c + t % VEC, sum);
+  }
+}
+
+// -------------------------------------------------------------- a prompt
+// Two launches.  talking_stats: a block 64 queries of one head, flash attention without values: the logarithm (base 2) of
+// each row's softmax denominator.  With it a weight is one exponential, and what a key adds needs no rescaling: talking_prompt,
+// a block 16 queries with all heads, walks the keys KT at a time.  A wave makes the weights of eight heads against 16 keys
+// (keys down the MFMA's rows, queries across), which lie in LDS a pair (query, key) at a time, heads side by side: one MFMA
+// operand of the heads' mixing, whose result goes back to LDS a head at a time, keys side by side: one operand of the
+// product with the values (transposed in LDS).  Two barriers a tile; keys and values of the next are on their way meanwhile.
+constexpr float LOG2E = 1.4426950408889634f;
+constexpr int STAT_KEYS = 64;
+
+// The row of key or value `p` (both packed rows' and rings' are whole 16-byte pieces).
+__device__ __forceinline__ const bf16_t* row_of(const bf16_t* __restrict__ own, const bf16_t* __restrict__ held, int p, int start, int stride,
+                                                int width, int ring) {
+  return p >= start ? own + (size_t)(p - start) * stride : held + (size_t)(p % ring) * width;
+}
+
+template <int KD>
+__global__ __launch_bounds__(256) void talking_stats_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ keys,
+                                                            const int* __restrict__ spans, float* __restrict__ stats, TalkShape a) {
+  constexpr int DP = KD * 32, KP = STAT_KEYS * DP / 8 / 256;
+  __shared__ __align__(16) bf16_t kt[2][STAT_KEYS][DP + 8];
+  const int head = blockIdx.x, slot = blockIdx.z, q0 = blockIdx.y * 64;
+  const Span s = span_of(spans, slot, a.p.rows);
+  if (q0 >= s.rows) return;
+  const int H = a.p.heads, D = a.p.dim, G = a.p.kv_heads, g = head / (H / G);
+  const int t = threadIdx.x, lane = t & 63, wave = t >> 6, l16 = lane & 15, quad = lane >> 4;
+  const int first = s.start + q0, last = s.start + min(q0 + 64, s.rows) - 1, from = first / a.chunk * a.chunk;
+  const bf16_t* own = x + (size_t)s.row0 * a.p.stride + H * D + g * D;
+  const bf16_t* held = keys + (size_t)slot * a.p.ring * G * D + g * D;
+  const int i = min(q0 + wave * 16 + l16, s.rows - 1), pos = s.start + i, lo = pos / a.chunk * a.chunk;
+  bf16x8 qf[KD];
+#pragma unroll
+  for (int d = 0; d < KD; ++d) {
+    const int c = d * 32 + quad * 8;
+    uint4 v = make_uint4(0, 0, 0, 0);
+    if (c < D) v = *reinterpret_cast<const uint4*>(x + (size_t)(s.row0 + i) * a.p.stride + head * D + c);
+    qf[d] = __builtin_bit_cast(bf16x8, v);
+  }
+  u32x4 kn[KP];
+  auto fetch = [&](int base) {
+#pragma unroll
+    for (int e = 0; e < KP; ++e) {
+      const int u = t + 256 * e, c = min((u % (DP / 8)) * 8, D - 8);   // (columns past a head's: q is zero there)
+      kn[e] = *reinterpret_cast<const u32x4*>(row_of(own, held, min(base + u / (DP / 8), last), s.start, a.p.stride, G * D, a.p.ring) + c);
+    }
+  };
+  fetch(from);
+  float m = -1e30f, l = 0.f;
+  int turn = 0;
+  for (int base = from; base <= last; base += STAT_KEYS, turn ^= 1) {
+#pragma unroll
+    for (int e = 0; e < KP; ++e) {
+      const int u = t + 256 * e;
+      *reinterpret_cast<u32x4*>(&kt[turn][u / (DP / 8)][(u % (DP / 8)) * 8]) = kn[e];
+    }
+    __syncthreads();
+    fetch(min(base + STAT_KEYS, last));
+    f32x4 sc[4];
+#pragma unroll
+    for (int k = 0; k < 4; ++k) {
+      sc[k] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int d = 0; d < KD; ++d)
+        sc[k] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8*>(&kt[turn][k * 16 + l16][d * 32 + quad * 8]), qf[d], sc[k], 0, 0, 0);
+    }
+    float top = -INFINITY;
+    const bool whole = base + STAT_KEYS - 1 <= first && base >= last / a.chunk * a.chunk;   // every row sees every key
+#pragma unroll
+    for (int k = 0; k < 4; ++k)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int p = base + k * 16 + quad * 4 + r;
+        const float v = sc[k][r] * LOG2E;
+        sc[k][r] = whole || (p <= pos && p >= lo) ? v : -INFINITY;
+        top = fmaxf(top, sc[k][r]);
+      }
+    if (__builtin_amdgcn_ballot_w64(top > m + 8.f) != 0) {
+      top = fmaxf(top, __shfl_xor(top, 16, 64));
+      top = fmaxf(top, __shfl_xor(top, 32, 64));
+      top = fmaxf(m, top);
+      l *= __builtin_amdgcn_exp2f(m - top);
+      m = top;
+    }
+#pragma unroll
+    for (int k = 0; k < 4; ++k)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) l += __builtin_amdgcn_exp2f(sc[k][r] - m);
+  }
+  l += __shfl_xor(l, 16, 64);
+  l += __shfl_xor(l, 32, 64);
+  if (quad == 0 && q0 + wave * 16 + l16 < s.rows) stats[(size_t)(s.row0 + i) * H + head] = m + log2f(l);
+}
+
+// NG groups of eight heads (H <= 8 NG), KD pieces of 32 key columns, VT tiles of 16 value columns a head; EACH query heads in a
+// row share a key head.
+template <int NG, int KD, int VT>
+struct Talking {
+  static constexpr int KT = 128 / NG, HP = 8 * NG, HN = (HP + 15) / 16;
+  static constexpr int PAIR = KT * HP + 8;            // a query's weights: [key][head]
+  static constexpr int MIX = HP * (KT + 8) + 8;       // a query's mixed weights: [head][key]
+  static size_t lds(int kv_width) { return ((size_t)16 * PAIR + (size_t)16 * MIX + (size_t)kv_width * (KT + 8)) * 2; }
+};
+
+template <int NG, int KD, int VT, int EACH>
+__global__ __launch_bounds__(512) void talking_prompt_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ keys,
+                                                             const bf16_t* __restrict__ values, const bf16_t* __restrict__ talk,
+                                                             const int* __restrict__ spans, const float* __restrict__ stats,
+                                                             bf16_t* __restrict__ out, TalkShape a) {
+  using S = Talking<NG, KD, VT>;
+  constexpr int KT = S::KT, HP = S::HP, SETS = 8 / EACH;
+  constexpr bool HOLD = KD <= 2 && NG * VT <= 16;     // the queries stay in registers
+  constexpr bool AHEAD = SETS * KD <= 8 && NG * VT <= 16;   // a tile's keys are fetched under the tile before
+  extern __shared__ __align__(16) bf16_t shared[];
+  bf16_t* pair = shared;
+  bf16_t* mix = pair + 16 * S::PAIR;
+  bf16_t* vt = mix + 16 * S::MIX;                     // [G * V][KT + 8]
+  const int slot = blockIdx.y, q0 = ((int)gridDim.x - 1 - (int)blockIdx.x) * 16;
+  const Span s = span_of(spans, slot, a.p.rows);
+  if (q0 >= s.rows) return;
+  const int H = a.p.heads, G = a.p.kv_heads, D = a.p.dim, V = a.p.vdim, each = H / G, nk = G * D, nv = G * V;
+  const int t = threadIdx.x, lane = t & 63, wave = __builtin_amdgcn_readfirstlane(t >> 6), l16 = lane & 15, quad = lane >> 4;
+  const int first = s.start + q0, last = s.start + min(q0 + 16, s.rows) - 1, from = first / a.chunk * a.chunk;
+  const bf16_t* own_k = x + (size_t)s.row0 * a.p.stride + H * D;
+  const bf16_t* own_v = own_k + nk;
+  const bf16_t* held_k = keys + (size_t)slot * a.p.ring * nk;
+  const bf16_t* held_v = values + (size_t)slot * a.p.ring * nv;
+  const int i = min(q0 + l16, s.rows - 1), pos = s.start + i, lo = pos / a.chunk * a.chunk;
+  const bf16_t* q_row = x + (size_t)(s.row0 + i) * a.p.stride;
+
+  // This wave's weights: heads h0 .. h0 + 7 against keys sub * 16 .. + 15 of a tile.
+  const int h0 = (wave % NG) * 8, sub = wave / NG;
+  auto query = [&](int e, int d, int off) {
+    const int c = d * 32 + quad * 8;
+    u32x4 v = *reinterpret_cast<const u32x4*>(q_row + min(h0 + e, H - 1) * D + min(c, D - 8) + off);
+    if (c >= D) v = u32x4{0, 0, 0, 0};
+    return __builtin_bit_cast(bf16x8, v);
+  };
+  bf16x8 qf[HOLD ? 8 : 1][HOLD ? KD : 1];
+  float lse[8];
+#pragma unroll
+  for (int e = 0; e < 8; ++e) {
+    lse[e] = h0 + e < H ? stats[(size_t)(s.row0 + i) * H + h0 + e] : INFINITY;   // (a head that is none: no weight)
+    if constexpr (HOLD) {
+#pragma unroll
+      for (int d = 0; d < KD; ++d) qf[e][d] = query(e, d, 0);
+    }
+  }
+  // The heads' mixing as the second operand: head l16 (+ 16 n) of the result down its columns.
+  bf16x8 tf[S::HN];
+#pragma unroll
+  for (int n = 0; n < S::HN; ++n) {
+    bf16_t w[8];
+#pragma unroll
+    for (int j = 0; j < 8; ++j) {
+      const int h = n * 16 + l16, g = quad * 8 + j;
+      w[j] = h < H && g < H ? talk[h * H + g] : (bf16_t)0;
+    }
+    tf[n] = __builtin_bit_cast(bf16x8, make_uint4(w[0] | (uint32_t)w[1] << 16, w[2] | (uint32_t)w[3] << 16, w[4] | (uint32_t)w[5] << 16, w[6] | (uint32_t)w[7] << 16));
+  }
+  f32x4 acc[NG][VT];
+#pragma unroll
+  for (int e = 0; e < NG; ++e)
+#pragma unroll
+    for (int v = 0; v < VT; ++v) acc[e][v] = f32x4{0.f, 0.f, 0.f, 0.f};
+
+  bf16x8 kf[AHEAD ? SETS : 1][KD];
+  u32x4 vn[4];   // the thread's first piece of a tile's values, on its way
+  const int v_cols = nv / 8, v_pieces = (KT / 4) * v_cols;
+  auto key_row = [&](int base) { return row_of(own_k, held_k, min(base + sub * 16 + l16, last), s.start, a.p.stride, nk, a.p.ring); };
+  auto fetch_keys = [&](const bf16_t* row, int u, bf16x8 (&to)[KD]) {
+    const bf16_t* at = row + min(h0 + u * EACH, H - 1) / each * D;
+#pragma unroll
+    for (int d = 0; d < KD; ++d) to[d] = __builtin_bit_cast(bf16x8, *reinterpret_cast<const u32x4*>(at + min(d * 32 + quad * 8, D - 8)));
+  };
+  auto fetch_ahead = [&](int base) {
+    if constexpr (AHEAD) {
+      const bf16_t* row = key_row(base);
+#pragma unroll
+      for (int u = 0; u < SETS; ++u) fetch_keys(row, u, kf[u]);
+    }
+  };
+  auto fetch_values = [&](int base, int piece, u32x4 (&v)[4]) {   // four keys of eight columns
+    const int k4 = piece / v_cols * 4, c = (piece % v_cols) * 8;
+#pragma unroll
+    for (int j = 0; j < 4; ++j)
+      v[j] = *reinterpret_cast<const u32x4*>(row_of(own_v, held_v, min(base + k4 + j, last), s.start, a.p.stride, nv, a.p.ring) + c);
+  };
+  auto lay_values = [&](int piece, const u32x4 (&v)[4]) {   // turned: a column's four keys side by side
+    const int k4 = piece / v_cols * 4, c = (piece % v_cols) * 8;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      *reinterpret_cast<uint2*>(vt + (c + 2 * j) * (KT + 8) + k4) =
+          make_uint2((v[0][j] & 0xffffu) | (v[1][j] << 16), (v[2][j] & 0xffffu) | (v[3][j] << 16));
+      *reinterpret_cast<uint2*>(vt + (c + 2 * j + 1) * (KT + 8) + k4) =
+          make_uint2((v[0][j] >> 16) | (v[1][j] & 0xffff0000u), (v[2][j] >> 16) | (v[3][j] & 0xffff0000u));
+    }
+  };
+  fetch_ahead(from);
+  if (t < v_pieces) fetch_values(from, t, vn);
+  for (int base = from; base <= last; base += KT) {
+    // ---- weights
+    f32x4 sc[8];
+    int off = 0;
+    if constexpr (!HOLD) asm volatile("" : "+v"(off));   // (queries that are read every time are not to be held all the same)
+    const bf16_t* row = nullptr;
+    if constexpr (!AHEAD) row = key_row(base);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      sc[e] = f32x4{0.f, 0.f, 0.f, 0.f};
+      if constexpr (!AHEAD) {
+        if (e % EACH == 0) fetch_keys(row, e / EACH, kf[0]);
+      }
+#pragma unroll
+      for (int d = 0; d < KD; ++d)
+        sc[e] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[AHEAD ? e / EACH : 0][d], HOLD ? qf[HOLD ? e : 0][HOLD ? d : 0] : query(e, d, off), sc[e], 0, 0, 0);
+    }
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int j = sub * 16 + quad * 4 + r, p = base + j;
+      const bool seen = p <= pos && p >= lo;
+      float w[8];
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        w[e] = __builtin_amdgcn_exp2f(fmaf(sc[e][r], LOG2E, -lse[e]));
+        w[e] = seen ? w[e] : 0.f;
+      }
+      *reinterpret_cast<uint4*>(pair + l16 * S::PAIR + j * HP + h0) = pack8(w);
+    }
+    __syncthreads();   // the weights are there, and the last tile's products are done
+    fetch_ahead(min(base + KT, last));
+    // ---- values, turned, and the next ones on their way
+    if (t < v_pieces) lay_values(t, vn);
+    for (int piece = t + 512; piece < v_pieces; piece += 512) {
+      u32x4 v[4];
+      fetch_values(base, piece, v);
+      lay_values(piece, v);
+    }
+    if (t < v_pieces) fetch_values(min(base + KT, last), t, vn);
+    // ---- the heads mixed: 16 keys of one query at a time
+#pragma unroll 4
+    for (int u = wave; u < KT; u += 8) {   // KT / 16 pieces of each of 16 queries
+      const int qi = u / (KT / 16), j0 = u % (KT / 16) * 16;
+      uint4 v = *reinterpret_cast<const uint4*>(pair + qi * S::PAIR + (j0 + l16) * HP + (quad * 8 < HP ? quad * 8 : 0));
+      if (quad * 8 >= HP) v = make_uint4(0, 0, 0, 0);
+#pragma unroll
+      for (int n = 0; n < S::HN; ++n) {
+        const f32x4 zero = f32x4{0.f, 0.f, 0.f, 0.f};
+        const f32x4 m = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, v), tf[n], zero, 0, 0, 0);
+        if (n * 16 + l16 < HP)
+          *reinterpret_cast<uint2*>(mix + qi * S::MIX + (n * 16 + l16) * (KT + 8) + j0 + quad * 4) = make_uint2(pack_bf16(m[0], m[1]), pack_bf16(m[2], m[3]));
+      }
+    }
+    __syncthreads();
+    // ---- times the values: NG heads a wave
+#pragma unroll
+    for (int e = 0; e < NG; ++e) {
+      const int h = wave * NG + e;
+      if (h >= H) continue;
+      const int at = h / each * V;
+#pragma unroll
+      for (int k = 0; k < KT; k += 32) {
+        const bf16x8 pf = *reinterpret_cast<const bf16x8*>(mix + l16 * S::MIX + h * (KT + 8) + k + quad * 8);
+#pragma unroll
+        for (int v = 0; v < VT; ++v) {
+          if (v * 16 >= V) continue;
+          const bf16x8 vf = *reinterpret_cast<const bf16x8*>(vt + min(at + v * 16 + l16, nv - 1) * (KT + 8) + k + quad * 8);
+          acc[e][v] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pf, acc[e][v], 0, 0, 0);
+        }
+      }
+    }
+  }
+  if (q0 + l16 >= s.rows) return;
+#pragma unroll
+  for (int e = 0; e < NG; ++e) {
+    const int h = wave * NG + e;
+    if (h >= H) continue;
+#pragma unroll
+    for (int v = 0; v < VT; ++v) {
+      const int c = v * 16 + quad * 4;
+      if (c < V)
+        *reinterpret_cast<uint2*>(out + (size_t)(s.row0 + i) * a.out_stride + h * V + c) =
+            make_uint2(pack_bf16(acc[e][v][0], acc[e][v][1]), pack_bf16(acc[e][v][2], acc[e][v][3]));
+    }
+  }
+}
+
+template <int NG, int KD, int VT, int EACH>
+static int launch_talking_prompt(const bf16_t* x, const bf16_t* keys, const bf16_t* values, const bf16_t* talk, const int* spans,
+                                 const float* stats, bf16_t* out, const TalkShape& a, int slots, hipStream_t s) {
+  const size_t lds = Talking<NG, KD, VT>::lds(a.p.kv_heads * a.p.vdim);
+  static LdsOptIn opt;
+  const hipError_t e = opt.ensure(reinterpret_cast<const void*>(&talking_prompt_kernel<NG, KD, VT, EACH>), 160 * 1024);
+  if (e != hipSuccess) { set_error("%s", hipGetErrorString(e)); return (int)e; }
+  hipLaunchKernelGGL((talking_prompt_kernel<NG, KD, VT, EACH>), dim3((a.p.rows + 15) / 16, slots), dim3(512), lds, s, x, keys, values, talk, spans, stats,
+                     out, a);
+  IRON_LAUNCH_CHECK();
+}
+// The groups of heads a prompt's kernel takes these sizes in, 0 where it takes them not at all.
+static int talking_groups(int heads, int kv_heads, int dim, int vdim, int is_float) {
+  if (is_float || heads > 32 || dim % 8 || vdim % 8 || dim > 128 || vdim > 128) return 0;
+  for (int ng = heads <= 8 ? 1 : (heads <= 16 ? 2 : 4); ng <= 4; ng *= 2) {
+    const size_t kt = 128 / ng, lds = 32 * (kt * 8 * ng + 8) + 32 * (8 * ng * (kt + 8) + 8) + 2 * (size_t)kv_heads * vdim * (kt + 8);
+    if (lds <= 160 * 1024) return ng;
+  }
+  return 0;
+}
+
 }  // namespace iron
 
 using namespace iron;
@@ -252,10 +689,15 @@ extern "C" int iron_turned_heads(const void* x, void* y, const uint16_t* bias, c
   IRON_LAUNCH_CHECK();
 }
 
-extern "C" int iron_mha_talking(const void* x, void* keys, void* values, const uint16_t* talk, const int* spans, void* out, int slots, int rows,
-                                int stride, int heads, int kv_heads, int dim, int vdim, int chunk, int ring, int single, int is_float,
+extern "C" int64_t iron_mha_talking_workspace_bytes(int slots, int rows, int heads, int chunk, int single) {
+  return single ? (int64_t)slots * StepWork(heads, chunk).words * 4 : (int64_t)rows * heads * 4;
+}
+
+
+extern "C" int iron_mha_talking(const void* x, void* keys, void* values, const uint16_t* talk, const int* spans, void* out, void* workspace,
+                                int slots, int rows, int stride, int heads, int kv_heads, int dim, int vdim, int chunk, int ring, int single, int is_float,
                                 void* stream) {
-  IRON_REQUIRE(x && keys && values && talk && spans && out, "mha_talking: null operand");
+  IRON_REQUIRE(x && keys && values && talk && spans && out && workspace, "mha_talking: null operand");
   IRON_REQUIRE(((uintptr_t)spans & 15) == 0, "mha_talking: spans must be 16-byte aligned");
   IRON_REQUIRE(slots > 0 && slots <= 65535 && rows > 0, "mha_talking: slots (%d) and rows (%d) must be positive", slots, rows);
   IRON_REQUIRE(heads > 0 && kv_heads > 0 && heads % kv_heads == 0 && dim > 0 && vdim > 0, "mha_talking: kv_heads (%d) must divide heads (%d)",
@@ -265,23 +707,66 @@ extern "C" int iron_mha_talking(const void* x, void* keys, void* values, const u
   const TalkShape a{{rows, stride, heads, kv_heads, dim, vdim, ring}, chunk, heads * vdim};
   hipStream_t s = (hipStream_t)stream;
   const bool aligned = stride % 8 == 0 && dim % 8 == 0 && vdim % 8 == 0 && (((uintptr_t)x | (uintptr_t)keys | (uintptr_t)values) & 15) == 0;
-  const size_t lds = (size_t)talk_row_words(heads, dim, vdim) * 4;
-  IRON_REQUIRE(lds <= 160 * 1024, "mha_talking: %d heads of %d + %d need %zu bytes of LDS", heads, dim, vdim, lds);
-#define IRON_TALK_ROWS(T, VEC, STORE, ROWS)                                                                                              \
-  {                                                                                                                                      \
-    static LdsOptIn opt;                                                                                                                 \
-    const hipError_t e = opt.ensure(reinterpret_cast<const void*>(&talking_rows_kernel<T, VEC, STORE>), 160 * 1024);                     \
-    if (e != hipSuccess) { set_error("%s", hipGetErrorString(e)); return (int)e; }                                                       \
-    hipLaunchKernelGGL((talking_rows_kernel<T, VEC, STORE>), dim3(ROWS, slots), dim3(256), lds, s, (const T*)x, (T*)keys, (T*)values,   \
-                       talk, spans, (T*)out, a);                                                                                         \
+  IRON_REQUIRE(((uintptr_t)workspace & 3) == 0, "mha_talking: the workspace must be 4-byte aligned");
+  if (single) {   // the caller's spans have one row at most
+    const int each = heads / kv_heads, octets = (each + STEP_HEADS - 1) / STEP_HEADS, threads = chunk >= 1024 ? 1024 : (chunk + 63) / 64 * 64;
+    const size_t q_bytes = (size_t)each * dim * 4, m_bytes = (size_t)heads * (STEP_HEADS + 1) * 4;
+    IRON_REQUIRE(kv_heads * octets <= 65535 && q_bytes <= 64 * 1024 && m_bytes <= 48 * 1024, "mha_talking: %d heads of %d (%d key heads) in a step",
+                 heads, dim, kv_heads);
+    float* work = (float*)workspace;
+#define IRON_TALK_STEP(T, VEC)                                                                                                                \
+  {                                                                                                                                           \
+    hipLaunchKernelGGL((talking_scores_kernel<T, VEC>), dim3((chunk + 63) / 64, kv_heads, slots), dim3(64), q_bytes, s, (const T*)x, (T*)keys, \
+                       (T*)values, spans, work, a);                                                                                           \
+    hipLaunchKernelGGL((talking_mix_kernel<T, VEC>), dim3(vdim / VEC, kv_heads * octets, slots), dim3(threads), m_bytes, s, (const T*)x,       \
+                       (const T*)values, talk, spans, work, (T*)out, a);                                                                      \
   }
-  if (single) {   // the caller's spans have one row at most, which goes into the ring here
-    if (is_float) { if (aligned) IRON_TALK_ROWS(float, 8, true, 1) else IRON_TALK_ROWS(float, 1, true, 1) }
-    else { if (aligned) IRON_TALK_ROWS(bf16_t, 8, true, 1) else IRON_TALK_ROWS(bf16_t, 1, true, 1) }
+    if (is_float) { if (aligned) IRON_TALK_STEP(float, 8) else IRON_TALK_STEP(float, 1) }
+    else { if (aligned) IRON_TALK_STEP(bf16_t, 8) else IRON_TALK_STEP(bf16_t, 1) }
+#undef IRON_TALK_STEP
     IRON_LAUNCH_CHECK();
   }
-  if (is_float) { if (aligned) IRON_TALK_ROWS(float, 8, false, rows) else IRON_TALK_ROWS(float, 1, false, rows) }
-  else { if (aligned) IRON_TALK_ROWS(bf16_t, 8, false, rows) else IRON_TALK_ROWS(bf16_t, 1, false, rows) }
+  const size_t lds = (size_t)talk_row_words(heads, dim, vdim) * 4;
+  const int groups = aligned && ((uintptr_t)out & 7) == 0 ? talking_groups(heads, kv_heads, dim, vdim, is_float) : 0;
+  if (groups > 0) {
+    IRON_REQUIRE(rows <= 65535 * 64, "mha_talking: rows (%d) exceed the grid's y extent", rows);
+    const bf16_t *xb = (const bf16_t*)x, *kb = (const bf16_t*)keys, *vb = (const bf16_t*)values;
+    float* stats = (float*)workspace;
+    const dim3 grid(heads, (rows + 63) / 64, slots);
+    if (dim <= 64) hipLaunchKernelGGL((talking_stats_kernel<2>), grid, dim3(256), 0, s, xb, kb, spans, stats, a);
+    else hipLaunchKernelGGL((talking_stats_kernel<4>), grid, dim3(256), 0, s, xb, kb, spans, stats, a);
+    const bool fours = heads / kv_heads % 4 == 0;
+    int e;
+#define IRON_TALK(NG, KD, VT)                                                                                                \
+  e = fours ? launch_talking_prompt<NG, KD, VT, 4>(xb, kb, vb, talk, spans, stats, (bf16_t*)out, a, slots, s)                \
+            : launch_talking_prompt<NG, KD, VT, 1>(xb, kb, vb, talk, spans, stats, (bf16_t*)out, a, slots, s)
+#define IRON_TALKS(NG)                                       \
+  {                                                          \
+    if (dim <= 64 && vdim <= 64) IRON_TALK(NG, 2, 4);        \
+    else if (dim <= 64) IRON_TALK(NG, 2, 8);                 \
+    else if (vdim <= 64) IRON_TALK(NG, 4, 4);                \
+    else IRON_TALK(NG, 4, 8);                                \
+  }
+    if (groups == 1) IRON_TALKS(1)
+    else if (groups == 2) IRON_TALKS(2)
+    else IRON_TALKS(4)
+#undef IRON_TALKS
+#undef IRON_TALK
+    if (e != IRON_OK) return e;
+    launch_ring_store<bf16_t>(x, keys, values, spans, a.p, slots, s);
+    IRON_LAUNCH_CHECK();
+  }
+  IRON_REQUIRE(lds <= 160 * 1024, "mha_talking: %d heads of %d + %d need %zu bytes of LDS", heads, dim, vdim, lds);
+#define IRON_TALK_ROWS(T, VEC)                                                                                                          \
+  {                                                                                                                                     \
+    static LdsOptIn opt;                                                                                                                \
+    const hipError_t e = opt.ensure(reinterpret_cast<const void*>(&talking_rows_kernel<T, VEC>), 160 * 1024);                           \
+    if (e != hipSuccess) { set_error("%s", hipGetErrorString(e)); return (int)e; }                                                      \
+    hipLaunchKernelGGL((talking_rows_kernel<T, VEC>), dim3(rows, slots), dim3(256), lds, s, (const T*)x, (const T*)keys,                \
+                       (const T*)values, talk, spans, (T*)out, a);                                                                      \
+  }
+  if (is_float) { if (aligned) IRON_TALK_ROWS(float, 8) else IRON_TALK_ROWS(float, 1) }
+  else { if (aligned) IRON_TALK_ROWS(bf16_t, 8) else IRON_TALK_ROWS(bf16_t, 1) }
 #undef IRON_TALK_ROWS
   if (is_float) launch_ring_store<float>(x, keys, values, spans, a.p, slots, s);
   else launch_ring_store<bf16_t>(x, keys, values, spans, a.p, slots, s);

@@ -684,14 +684,16 @@ def turned_heads(x, y, bias, q_gain, k_gain, temp, spans, *, slots, rows, stride
                                   current_stream()), "iron_turned_heads")
 
 
-def mha_talking(x, keys, values, talk, spans, y, *, slots, rows, stride, heads, kv_heads, dim, vdim, chunk, ring, single=False):
+def mha_talking(x, keys, values, talk, spans, y, workspace, *, slots, rows, stride, heads, kv_heads, dim, vdim, chunk, ring, single=False):
     is_float = _act(x, rows * stride, "x")
     _same_kind(is_float, keys=keys, values=values, y=y)
     _act(keys, slots * ring * kv_heads * dim, "keys")
     _act(values, slots * ring * kv_heads * vdim, "values")
     _bf16(talk, heads * heads, "talk")
     _act(y, rows * heads * vdim, "y")
-    check(lib().iron_mha_talking(ptr(x), ptr(keys), ptr(values), ptr(talk), _spans(spans, slots), ptr(y), slots, rows, stride, heads, kv_heads,
+    need = int(lib().iron_mha_talking_workspace_bytes(slots, rows, heads, chunk, int(single)))
+    work = _work(workspace, need, "mha_talking: workspace")
+    check(lib().iron_mha_talking(ptr(x), ptr(keys), ptr(values), ptr(talk), _spans(spans, slots), ptr(y), work, slots, rows, stride, heads, kv_heads,
                                  dim, vdim, chunk, ring, int(single), int(is_float), current_stream()), "iron_mha_talking")
 
 

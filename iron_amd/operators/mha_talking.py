@@ -106,7 +106,14 @@ class TalkingMHA(Operator):
     keys = InOut(slots, chunk, kv_heads, dim, dtype=dtype)
     values = InOut(slots, chunk, kv_heads, vdim, dtype=dtype)
     y = Out(rows, width, dtype=dtype)
+    workspace_words: int = param(derive=lambda op: op._workspace_words(), repr=False)
+    workspace = Scratch(workspace_words, dtype=F32)
     valid = per_call(bounds=rows)
+
+    def _workspace_words(self) -> int:
+        from .._lib import lib
+
+        return int(lib().iron_mha_talking_workspace_bytes(self.slots, self.rows, self.heads, self.chunk, int(self.single))) // 4
 
     @classmethod
     def infer(cls, shapes, **kw):
@@ -128,6 +135,6 @@ class TalkingMHA(Operator):
         kw["ring"] = self.chunk
 
         def launch(t, words):
-            kernels.mha_talking(t["x"], t["keys"], t["values"], t["talk"], t["spans"], t["y"], **kw)
+            kernels.mha_talking(t["x"], t["keys"], t["values"], t["talk"], t["spans"], t["y"], t["workspace"], **kw)
 
         return Built("iron_mha_talking", launch)

@@ -146,7 +146,7 @@ def test_talking_attention_in_portions_and_steps(cuda, dtype, case, quiet):
         for n in sizes:
             op = TalkingMHA(slots=2, rows=n + 3, stride=x.shape[1], heads=H, kv_heads=G, dim=D, vdim=V, chunk=C, single=n == 1, dtype=dtype)
             out = ran(op, x=np.concatenate([np.full((3, x.shape[1]), 9.0), x[at : at + n]]), talk=talk, spans=table((1, 3, n, at), slots=2),
-                      keys=keys, values=values)
+                      keys=keys, values=values, workspace=True)
             keys, values = out["keys"], out["values"]
             assert (out["y"][:3] == 7).all()   # the sequence is not the batch's first rows
             assert (keys[0] == 5).all() and (values[0] == 5).all()
@@ -178,7 +178,7 @@ def test_talking_attention_over_several_requests(cuda, dtype, case, single):
             keys[slot, j % C], values[slot, j % C] = k[j], v[j]
         x[row : row + n] = packed(q, k, v)[start:]
     op = TalkingMHA(slots=6, rows=rows, stride=stride, heads=H, kv_heads=G, dim=D, vdim=V, chunk=C, single=single, dtype=dtype)
-    y = ran(op, x=x, talk=talk, spans=table(*parts, slots=6), keys=keys, values=values)["y"]
+    y = ran(op, x=x, talk=talk, spans=table(*parts, slots=6), keys=keys, values=values, workspace=True)["y"]
     for slot, row, n, _ in parts:
         assert np.abs(y[row : row + n] - want[slot]).max() <= (3e-5 if dtype is F32 else 2e-2) * np.abs(want[slot]).max(), slot
     idle = np.setdiff1d(np.arange(rows), np.concatenate([np.arange(r, r + n) for _, r, n, _ in parts]))
