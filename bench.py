@@ -709,8 +709,9 @@ def pegilix_state_bytes(config) -> int:
     return state
 
 
-def batched_served(torch, model_class, config, weights, steps, prompts, state_bytes):
-    """A batched model's prompts and replayed decode steps, every slot busy."""
+def batched_served(torch, model_class, config, weights, steps, prompts, state_bytes, weight_bytes=None):
+    """A batched model's prompts and replayed decode steps, every slot busy.  ``weight_bytes`` of weights a step reads; None: all but
+    the embedding."""
     from iron_amd.lm.batched import Entry
 
     model = model_class(config, weights)
@@ -728,7 +729,8 @@ def batched_served(torch, model_class, config, weights, steps, prompts, state_by
     first["prompt_tok_s"] = {n: round(v * config.slots, 1) for n, v in first["prompt_tok_s"].items()}
     first["launches_per_step"] = model.decode_step.launches_per_replay
     first["launches_per_portion"] = model.prompt_chunk.launches_per_call
-    weight_bytes = 2 * sum(int(np.prod(t.shape)) for n, t in weights.items() if n != "embed")
+    if weight_bytes is None:
+        weight_bytes = 2 * sum(int(np.prod(t.shape)) for n, t in weights.items() if n != "embed")
     bytes_step = weight_bytes + config.slots * state_bytes
     first |= {"decode_tok_s": round(1e3 * config.slots / first["decode_ms"], 1), "decode_GBps": round(bytes_step / first["decode_ms"] / 1e6, 1),
               "frac_hbm": round(bytes_step / first["decode_ms"] / 1e6 / HBM_PEAK_GBS, 4), "bytes_per_step": int(bytes_step)}
@@ -864,6 +866,77 @@ def bench_pufuzen(torch, dev, steps, widths, batch=8, prompts=(512, 2048)):
             "data": "synthetic", "dtype": "bf16", "sizes": rows}
 
 
+# The matrix memories of Tilarax layers at PEGILIX_SIZES' widths: (heads, key width, value width); the experts of its feed-forwards: (all, chosen)
+TILARAX_MEMORIES = {2048: (8, 128, 256), 3072: (12, 128, 256), 4096: (8, 256, 512)}
+TILARAX_EXPERTS = (16, 4)
+
+
+def tilarax_config(width, slots=1, chunk=2048):
+    """A Tilarax of ``width``'s sizes: chunked attention and matrix memories in turn, the first feed-forward dense, the others
+    experts of which a token's chosen ones are as wide together."""
+    from iron_amd.applications.tilarax import TilaraxConfig
+
+    H, G, D, F, layers, vocab = PEGILIX_SIZES[width]
+    heads, dim, vdim = TILARAX_MEMORIES[width]
+    every, top = TILARAX_EXPERTS
+    experts = {"kind": "moe", "expert": {"ff": F // top}, "router": {"experts": every, "top": top}}
+    attention = {"type": "attention", "mlp": experts, "mixer": {"heads": H, "kv_heads": G, "dim": D, "vdim": D, "mask": {"size": PEGILIX_WINDOW},
+                                                                 "rot": {"base": 10000.0, "dims": D}, "scale": D**-0.5, "v_mix": True}}
+    memory = {"type": "mlstm", "mlp": experts, "mixer": {"heads": heads, "dim": dim, "vdim": vdim, "gate_cap": 15.0}}
+    listed = [attention, memory] * (layers // 2)
+    listed[0] = {**attention, "mlp": {"ff": F, "kind": "dense"}}
+    return TilaraxConfig(vocab_size=vocab, hidden_size=width, layers=tuple(listed), eps=1e-5, max_seq_len=4096, prefill_chunk=chunk, slots=slots)
+
+
+def tilarax_step_bytes(config, weights, keys) -> tuple[int, int]:
+    """Bytes of weights a decode step of ``config.slots`` rows reads (of the experts, as many as that many draws meet on average), and
+    of states and keys a slot, ``keys`` of them in its chunk."""
+    every, top = TILARAX_EXPERTS
+    met = every * (1 - (1 - top / every) ** config.slots)
+    read = 2 * sum(int(np.prod(t.shape)) * (met / every if ".mlp.e" in n else 1) for n, t in weights.items())
+    state = 0
+    for spec in config.layers:
+        m = spec["mixer"]
+        state += keys * m["kv_heads"] * (m["dim"] + m["vdim"]) * 2 if spec["type"] == "attention" else 8 * m["heads"] * m["dim"] * (m["vdim"] + 1)
+    return int(read), state
+
+
+def bench_tilarax(torch, dev, steps, widths, batch=8, prompts=(512, 2048, 1920)):
+    """Prompt and decode throughput of Tilarax layers at a few widths, one sequence (decode deep in a chunk, behind the last of the
+    prompts) and a batch of ``batch``, beside a Pegilix of the same width, layers, vocabulary and feed-forward a token meets; random
+    weights, bf16."""
+    import dataclasses
+
+    from iron_amd.applications import pegilix, tilarax
+
+    rows = []
+    for width in widths:
+        row = {"width": width, "layers": PEGILIX_SIZES[width][4]}
+        for name, module, cls, config, kw in (("tilarax", tilarax, tilarax.Tilarax, tilarax_config(width), {}),
+                                              ("pegilix", pegilix, pegilix.Pegilix, pegilix_config(width), dict(bias_rows=32, rank=64))):
+            weights = random_weights(torch, module.shapes(config, **kw), dev)
+            row[f"{name}_params"] = sum(int(np.prod(t.shape)) for t in weights.values())
+            for n, t in weights.items():
+                if n.endswith(".dwa"):   # mostly the layer's own result
+                    t[:-1] *= 0.05
+            for slots, lengths in ((1, prompts), (batch, (512,))):
+                if not slots:
+                    continue
+                sized = dataclasses.replace(config, slots=slots)
+                if name == "tilarax":
+                    read, state = tilarax_step_bytes(sized, weights, lengths[-1] % PEGILIX_WINDOW)
+                else:
+                    read, state = None, pegilix_state_bytes(config)
+                row[name if slots == 1 else f"{name}_batch_{slots}"] = batched_served(torch, cls, sized, weights, steps, lengths, state, read)
+            del weights
+            torch.cuda.empty_cache()
+        rows.append(row)
+        print(json.dumps(row), file=sys.stderr, flush=True)
+    return {"what": f"prompt (ms, tok/s) and greedy decode steps as HIP-graph replays; chunks and windows of {PEGILIX_WINDOW}; frac_hbm: weights "
+                    "a step meets, states and keys over the time a step takes",
+            "data": "synthetic", "dtype": "bf16", "sizes": rows}
+
+
 class _AfterPrompt:
     """A single-sequence model's captured decode step behind a prompt of ``n`` tokens."""
 
@@ -983,9 +1056,11 @@ def main():
                     help="time only Pegilix layers at a few widths beside a Llama of equal size, and exit")
     ap.add_argument("--pufuzen", action="store_true",
                     help="time only Pufuzen layers at a few widths beside a Pegilix of equal size, and exit")
+    ap.add_argument("--tilarax", action="store_true",
+                    help="time only Tilarax layers at a few widths beside a Pegilix of equal size, and exit")
     ap.add_argument("--widths", type=int, nargs="+", default=sorted(PEGILIX_SIZES), choices=sorted(PEGILIX_SIZES),
-                    help="the widths --pegilix and --pufuzen time")
-    ap.add_argument("--batch", type=int, default=8, help="sequences of --pegilix's and --pufuzen's batch (0: one sequence only)")
+                    help="the widths --pegilix, --pufuzen and --tilarax time")
+    ap.add_argument("--batch", type=int, default=8, help="sequences of --pegilix's, --pufuzen's and --tilarax's batch (0: one sequence only)")
     args = ap.parse_args()
     if args.gpus != 1:
         print("bench.py: this build is a one-GPU hot path; --gpus must be 1 "
@@ -1021,6 +1096,9 @@ def main():
         return 0
     if args.pufuzen:
         print(json.dumps(bench_pufuzen(torch, dev, args.steps, args.widths, args.batch)))
+        return 0
+    if args.tilarax:
+        print(json.dumps(bench_tilarax(torch, dev, args.steps, args.widths, args.batch)))
         return 0
     if args.prompt_probe:
         prompt_probe(torch, dev)

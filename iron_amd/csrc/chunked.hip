@@ -37,14 +37,6 @@ __device__ __forceinline__ float widened(bf16_t v) { return bf16_to_f32(v); }
 __device__ __forceinline__ float widened(float v) { return v; }
 __device__ __forceinline__ float pick4(const f32x4& v, int i) { return i < 2 ? (i == 0 ? v[0] : v[1]) : (i == 2 ? v[2] : v[3]); }
 
-// A barrier for what the block exchanges through LDS: waits for its LDS traffic, not (as __syncthreads does)
-// for the loads from memory in flight.
-__device__ __forceinline__ void block_barrier_lds() {
-  __builtin_amdgcn_fence(__ATOMIC_RELEASE, "workgroup", "local");
-  __builtin_amdgcn_s_barrier();
-  __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "workgroup", "local");
-}
-
 // ---------------------------------------------------------------- time mixing
 // Workspace of a chunk and head: r exp(L before it) frags, k exp(L_end - L) frags transposed (both 16 a
 // row tile), exp(L_end), and the 16 x 16 matrix's frag.

@@ -44,17 +44,18 @@ __device__ __forceinline__ void choose(float* __restrict__ z, int n, int top, in
   if (lane < top) shares[lane] = mine / total;
 }
 
-template <typename T, int VEC>
-__global__ __launch_bounds__(256) void router_kernel(const T* __restrict__ h, const bf16_t* __restrict__ w, const bf16_t* __restrict__ bias,
+template <typename T, int VEC, int NW>
+__global__ __launch_bounds__(NW * 64) void router_kernel(const T* __restrict__ h, const bf16_t* __restrict__ w, const bf16_t* __restrict__ bias,
                                                      int* __restrict__ ids, float* __restrict__ shares, int rows, int cols, int experts,
                                                      int top, const int* __restrict__ valid) {
   __shared__ float z[ROUTER_MAX];
   const int row = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   if (row >= bound_or(valid, rows)) return;
   const T* hr = h + (size_t)row * cols;
-  for (int e = wave; e < experts; e += 4) {
+  for (int e = wave; e < experts; e += NW) {
     const bf16_t* wr = w + (size_t)e * cols;
     float sum = 0.f;
+#pragma unroll 4
     for (int c = lane * VEC; c < cols; c += 64 * VEC) {
       float a[VEC], b[VEC];
       load_vec<VEC>(hr + c, a);
@@ -92,7 +93,7 @@ __global__ __launch_bounds__(256) void expert_pairs_kernel(const T* __restrict__
     gr[p] = gate + at;
     ur[p] = up + at;
   }
-#pragma unroll 2
+#pragma unroll 4
   for (int c = lane * VEC; c < cols; c += 64 * VEC) {
     float x[VEC], b[PER][VEC], d[PER][VEC];
     load_vec<VEC>(hr + c, x);
@@ -116,29 +117,34 @@ __global__ __launch_bounds__(256) void expert_pairs_kernel(const T* __restrict__
   }
 }
 
-// y[row] = sum over its experts of share * down_e a[pair].
+// y[row] = sum over its experts of share * down_e a[pair]: a block PER rows of down, a wave every fourth of the experts.
 template <typename T, int VEC, int PER>
 __global__ __launch_bounds__(256) void expert_sums_kernel(const T* __restrict__ a, const bf16_t* __restrict__ down, const int* __restrict__ ids,
                                                           const float* __restrict__ shares, T* __restrict__ y, int rows, int cols, int ff,
                                                           int experts, int top, const int* __restrict__ valid) {
-  const int row = blockIdx.y, lane = threadIdx.x & 63, c0 = (blockIdx.x * 4 + (threadIdx.x >> 6)) * PER;
-  if (row >= bound_or(valid, rows) || c0 >= cols) return;
+  __shared__ float red[4][PER];
+  const int row = blockIdx.y, lane = threadIdx.x & 63, wave = threadIdx.x >> 6, c0 = blockIdx.x * PER;
+  if (row >= bound_or(valid, rows)) return;
   float sum[PER];
 #pragma unroll
   for (int p = 0; p < PER; ++p) sum[p] = 0.f;
-  for (int k = 0; k < top; ++k) {
+  for (int k = wave; k < top; k += 4) {
     const int pair = row * top + k, e = min(max(ids[pair], 0), experts - 1);
     const float share = shares[pair];
     const T* ar = a + (size_t)pair * ff;
+    const bf16_t* dr[PER];
     float part[PER];
 #pragma unroll
-    for (int p = 0; p < PER; ++p) part[p] = 0.f;
-#pragma unroll 2
+    for (int p = 0; p < PER; ++p) {
+      part[p] = 0.f;
+      dr[p] = down + ((size_t)e * cols + min(c0 + p, cols - 1)) * ff;
+    }
+#pragma unroll 4
     for (int f = lane * VEC; f < ff; f += 64 * VEC) {
       float x[VEC], b[PER][VEC];
-      load_vec<VEC>(ar + f, x);
 #pragma unroll
-      for (int p = 0; p < PER; ++p) load_vec<VEC>(down + ((size_t)e * cols + min(c0 + p, cols - 1)) * ff + f, b[p]);
+      for (int p = 0; p < PER; ++p) load_vec<VEC>(dr[p] + f, b[p]);
+      load_vec<VEC>(ar + f, x);
 #pragma unroll
       for (int p = 0; p < PER; ++p)
 #pragma unroll
@@ -150,8 +156,11 @@ __global__ __launch_bounds__(256) void expert_sums_kernel(const T* __restrict__ 
 #pragma unroll
   for (int p = 0; p < PER; ++p) {
     const float v = wave_sum(sum[p]);
-    if (lane == 0 && c0 + p < cols) store_one(y + (size_t)row * cols + c0 + p, v);
+    if (lane == 0) red[wave][p] = v;
   }
+  __syncthreads();
+  const int p = threadIdx.x;
+  if (p < PER && c0 + p < cols) store_one(y + (size_t)row * cols + c0 + p, red[0][p] + red[1][p] + red[2][p] + red[3][p]);
 }
 
 // ------------------------------------------------------------- many rows
@@ -237,10 +246,18 @@ extern "C" int iron_router(const void* h, const uint16_t* w, const uint16_t* bia
                rows, cols, experts, ROUTER_MAX);
   IRON_REQUIRE(top > 0 && top <= experts && top <= 64, "router: top (%d) from 1 to the experts (%d), 64 at most", top, experts);
   const bool vec = cols % 8 == 0 && (((uintptr_t)h | (uintptr_t)w) & 15) == 0;
-#define IRON_ROUTER(T, VEC) \
-  hipLaunchKernelGGL((router_kernel<T, VEC>), dim3(rows), dim3(256), 0, (hipStream_t)stream, (const T*)h, w, bias, ids, shares, rows, cols, experts, top, valid)
-  if (is_float) { if (vec) IRON_ROUTER(float, 8); else IRON_ROUTER(float, 1); }
-  else { if (vec) IRON_ROUTER(bf16_t, 8); else IRON_ROUTER(bf16_t, 1); }
+  // Few rows: a wave an expert, so that a row's weights are all on their way at once.
+#define IRON_ROUTER(T, VEC)                                                                                                                \
+  {                                                                                                                                        \
+    if (rows < 256)                                                                                                                        \
+      hipLaunchKernelGGL((router_kernel<T, VEC, 16>), dim3(rows), dim3(1024), 0, (hipStream_t)stream, (const T*)h, w, bias, ids, shares,   \
+                         rows, cols, experts, top, valid);                                                                                 \
+    else                                                                                                                                   \
+      hipLaunchKernelGGL((router_kernel<T, VEC, 4>), dim3(rows), dim3(256), 0, (hipStream_t)stream, (const T*)h, w, bias, ids, shares,     \
+                         rows, cols, experts, top, valid);                                                                                 \
+  }
+  if (is_float) { if (vec) IRON_ROUTER(float, 8) else IRON_ROUTER(float, 1) }
+  else { if (vec) IRON_ROUTER(bf16_t, 8) else IRON_ROUTER(bf16_t, 1) }
 #undef IRON_ROUTER
   IRON_LAUNCH_CHECK();
 }
@@ -281,7 +298,7 @@ extern "C" int iron_experts(const void* h, const uint16_t* gate, const uint16_t*
   {                                                                                                                                           \
     hipLaunchKernelGGL((expert_pairs_kernel<T, VEC, 1>), dim3((ff + 3) / 4, rows * top), dim3(256), 0, s, (const T*)h, gate, up, ids,         \
                        (T*)workspace, rows, cols, ff, experts, top, activation, valid);                                                       \
-    hipLaunchKernelGGL((expert_sums_kernel<T, VEC, 2>), dim3((cols + 7) / 8, rows), dim3(256), 0, s, (const T*)workspace, down, ids, shares, \
+    hipLaunchKernelGGL((expert_sums_kernel<T, VEC, 2>), dim3((cols + 1) / 2, rows), dim3(256), 0, s, (const T*)workspace, down, ids, shares, \
                        (T*)y, rows, cols, ff, experts, top, valid);                                                                           \
   }
   if (is_float) { if (vec) IRON_PAIRS(float, 8) else IRON_PAIRS(float, 1) }

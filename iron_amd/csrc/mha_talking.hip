@@ -214,12 +214,12 @@ __global__ __launch_bounds__(256) void talking_rows_kernel(const T* __restrict__
 // ---------------------------------------------------------------- a step
 // One row a slot, two launches.  talking_scores: a wave 64 keys of one key head: the scores of its query heads, left in memory,
 // their largest and the sum of exponentials under it; the row's own key and value go into the ring.  talking_mix: a block VEC
-// columns of a value head, a thread a key: all heads' weights of that key, mixed for up to eight heads, times the value.
-constexpr int STEP_HEADS = 8;
+// columns of a value head, a thread a key: all heads' weights of that key, mixed for up to HEADS heads, times the value.
 struct StepWork {   // floats a slot: scores [heads][chunk], then (largest, sum) [heads][pieces of 64 keys]
   int pieces;
   size_t stats, words;
-  __host__ __device__ StepWork(int heads, int chunk) : pieces((chunk + 63) / 64), stats((size_t)heads * chunk), words(stats + (size_t)heads * 2 * pieces) {}
+  __host__ __device__ StepWork(int heads, int chunk)
+      : pieces((chunk + 63) / 64), stats(((size_t)heads * chunk + 1) & ~(size_t)1), words(stats + (size_t)heads * 2 * pieces) {}
 };
 template <typename T>
 __device__ __forceinline__ float weight_exp(float x) {
@@ -239,6 +239,12 @@ __global__ __launch_bounds__(64) void talking_scores_kernel(const T* __restrict_
   const T* row = x + (size_t)s.row0 * a.p.stride;
   const T* own = row + H * D + g * D;
   T* ring = keys + (size_t)slot * a.p.ring * G * D + g * D;
+  const int j = k0 + lane, p = lo + min(j, count - 1);
+  const T* kr = p == pos ? own : ring + (size_t)(p - lo) * G * D;
+  constexpr int FIRST = 8;   // pieces of the key asked for ahead of the queries
+  float kf[FIRST][VEC];
+#pragma unroll
+  for (int u = 0; u < FIRST; ++u) load_vec<VEC>(kr + min(u * VEC, D - VEC), kf[u]);
   for (int c = lane; c < each * D; c += 64) qs[c] = load_one(row + g * each * D + c);
   if (k0 == 0) {
     const T* v = row + (H + G) * D + g * V;
@@ -249,20 +255,24 @@ __global__ __launch_bounds__(64) void talking_scores_kernel(const T* __restrict_
   __syncthreads();
   const StepWork w(H, a.chunk);
   float* mine = work + slot * w.words;
-  const int j = k0 + lane, p = lo + min(j, count - 1);
-  const T* kr = p == pos ? own : ring + (size_t)(p % a.p.ring) * G * D;
   for (int e0 = 0; e0 < each; e0 += 4) {
     float dot[4] = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll 4
-    for (int c = 0; c < D; c += VEC) {
-      float f[VEC];
-      load_vec<VEC>(kr + c, f);
+    auto add = [&](int c, const float (&f)[VEC]) {
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
         const float* q = qs + min(e0 + e, each - 1) * D + c;
 #pragma unroll
         for (int n = 0; n < VEC; ++n) dot[e] = fmaf(f[n], q[n], dot[e]);
       }
+    };
+#pragma unroll
+    for (int u = 0; u < FIRST; ++u)
+      if (u * VEC < D) add(u * VEC, kf[u]);
+#pragma unroll 8
+    for (int c = FIRST * VEC; c < D; c += VEC) {
+      float f[VEC];
+      load_vec<VEC>(kr + c, f);
+      add(c, f);
     }
 #pragma unroll
     for (int e = 0; e < 4; ++e) {
@@ -279,57 +289,78 @@ __global__ __launch_bounds__(64) void talking_scores_kernel(const T* __restrict_
   }
 }
 
-template <typename T, int VEC>
+template <typename T, int VEC, int HEADS>
 __global__ __launch_bounds__(1024) void talking_mix_kernel(const T* __restrict__ x, const T* __restrict__ values, const bf16_t* __restrict__ talk,
                                                            const int* __restrict__ spans, const float* __restrict__ work, T* __restrict__ out,
                                                            TalkShape a) {
   extern __shared__ __align__(16) float lds[];
-  __shared__ float red[16][STEP_HEADS * VEC];
+  __shared__ float red[16][HEADS * VEC];
   const int slot = blockIdx.z, t = threadIdx.x, lane = t & 63, wave = t >> 6, waves = blockDim.x >> 6;
   const Span s = span_of(spans, slot, a.p.rows);
   if (s.rows == 0) return;
-  const int H = a.p.heads, G = a.p.kv_heads, D = a.p.dim, V = a.p.vdim, each = H / G, octets = (each + STEP_HEADS - 1) / STEP_HEADS;
-  const int g = blockIdx.y / octets, e0 = blockIdx.y % octets * STEP_HEADS, n = min(STEP_HEADS, each - e0), c = blockIdx.x * VEC;
+  const int H = a.p.heads, G = a.p.kv_heads, D = a.p.dim, V = a.p.vdim, each = H / G, sets = (each + HEADS - 1) / HEADS;
+  const int g = blockIdx.y / sets, e0 = blockIdx.y % sets * HEADS, n = min(HEADS, each - e0), c = blockIdx.x * VEC;
   const int pos = s.start, lo = pos / a.chunk * a.chunk, count = pos - lo + 1, live = (count + 63) / 64;
   const StepWork w(H, a.chunk);
   const float* mine = work + slot * w.words;
-  float* by = lds;                         // [H][8]: what the octet's heads take of a head, over its sum
-  float* top = by + H * STEP_HEADS;        // [H]
-  for (int h = t; h < H; h += blockDim.x) {
-    const float* st = mine + w.stats + (size_t)h * w.pieces * 2;
-    float m = -INFINITY, l = 0.f;
-    for (int i = 0; i < live; ++i) m = fmaxf(m, st[2 * i]);
-    for (int i = 0; i < live; ++i) l = fmaf(st[2 * i + 1], expf(st[2 * i] - m), l);
-    top[h] = m;
-    for (int e = 0; e < STEP_HEADS; ++e) by[h * STEP_HEADS + e] = e < n ? bf16_to_f32(talk[(size_t)(g * each + e0 + e) * H + h]) / l : 0.f;
-  }
-  __syncthreads();
-  float acc[STEP_HEADS][VEC];
-#pragma unroll
-  for (int e = 0; e < STEP_HEADS; ++e)
-#pragma unroll
-    for (int k = 0; k < VEC; ++k) acc[e][k] = 0.f;
+  float* by = lds;                         // [H][HEADS]: what the block's heads take of a head, over its sum
+  float* top = by + H * HEADS;        // [H]
   const T* own = x + (size_t)s.row0 * a.p.stride + (H + G) * D + g * V + c;
   const T* ring = values + (size_t)slot * a.p.ring * G * V + g * V + c;
+  // A key's value and the scores of its first heads: the thread's first key's are asked for ahead of the statistics.
+  constexpr int AT_ONCE = 32;
+  float f[VEC], raw[AT_ONCE];
+  auto fetch_value = [&](int j) { load_vec<VEC>(lo + j == pos ? own : ring + (size_t)j * G * V, f); };
+  auto fetch_scores = [&](int j, int h0) {
+#pragma unroll
+    for (int u = 0; u < AT_ONCE; ++u) raw[u] = mine[(size_t)min(h0 + u, H - 1) * a.chunk + j];
+  };
+  if (t < count) {
+    fetch_value(t);
+    fetch_scores(t, 0);
+  }
+  for (int h = wave; h < H; h += waves) {
+    const float2* st = reinterpret_cast<const float2*>(mine + w.stats) + (size_t)h * w.pieces;
+    const float mix = lane < n ? bf16_to_f32(talk[(size_t)(g * each + e0 + lane) * H + h]) : 0.f;
+    float m = -INFINITY, l = 0.f;
+    for (int i = lane; i < live; i += 64) {
+      const float2 v = st[i];
+      const float higher = fmaxf(m, v.x);
+      l = l * expf(m - higher) + v.y * expf(v.x - higher);   // (each piece has a key: its largest is finite)
+      m = higher;
+    }
+    const float most = wave_max(m), sum = wave_sum(m > -INFINITY ? l * expf(m - most) : 0.f);
+    if (lane == 0) top[h] = most;
+    if (lane < HEADS) by[h * HEADS + lane] = mix / sum;
+  }
+  __syncthreads();
+  float acc[HEADS][VEC];
+#pragma unroll
+  for (int e = 0; e < HEADS; ++e)
+#pragma unroll
+    for (int k = 0; k < VEC; ++k) acc[e][k] = 0.f;
   for (int j = t; j < count; j += blockDim.x) {
-    const int p = lo + j;
-    float f[VEC], mixed[STEP_HEADS];
-    load_vec<VEC>(p == pos ? own : ring + (size_t)(p % a.p.ring) * G * V, f);
+    float mixed[HEADS];
 #pragma unroll
-    for (int e = 0; e < STEP_HEADS; ++e) mixed[e] = 0.f;
-#pragma unroll 4
-    for (int h = 0; h < H; ++h) {
-      const float weight = weight_exp<T>(mine[(size_t)h * a.chunk + j] - top[h]);
+    for (int e = 0; e < HEADS; ++e) mixed[e] = 0.f;
+    if (j != t) fetch_value(j);
+    for (int h0 = 0; h0 < H; h0 += AT_ONCE) {
+      if (j != t || h0 > 0) fetch_scores(j, h0);
 #pragma unroll
-      for (int e = 0; e < STEP_HEADS; ++e) mixed[e] = fmaf(by[h * STEP_HEADS + e], weight, mixed[e]);
+      for (int u = 0; u < AT_ONCE; ++u) {
+        if (h0 + u >= H) continue;
+        const float weight = weight_exp<T>(raw[u] - top[h0 + u]);
+#pragma unroll
+        for (int e = 0; e < HEADS; ++e) mixed[e] = fmaf(by[(h0 + u) * HEADS + e], weight, mixed[e]);
+      }
     }
 #pragma unroll
-    for (int e = 0; e < STEP_HEADS; ++e)
+    for (int e = 0; e < HEADS; ++e)
 #pragma unroll
       for (int k = 0; k < VEC; ++k) acc[e][k] = fmaf(mixed[e], f[k], acc[e][k]);
   }
 #pragma unroll
-  for (int e = 0; e < STEP_HEADS; ++e)
+  for (int e = 0; e < HEADS; ++e)
     if (e < n) {
 #pragma unroll
       for (int k = 0; k < VEC; ++k) {
@@ -355,10 +386,11 @@ __global__ __launch_bounds__(1024) void talking_mix_kernel(const T* __restrict__
 constexpr float LOG2E = 1.4426950408889634f;
 constexpr int STAT_KEYS = 64;
 
-// The row of key or value `p` (both packed rows' and rings' are whole 16-byte pieces).
+// The row of key or value `p`, of the chunk that starts at `from` or later: positions ahead of the span are that chunk's, in the
+// ring's rows from its first on.
 __device__ __forceinline__ const bf16_t* row_of(const bf16_t* __restrict__ own, const bf16_t* __restrict__ held, int p, int start, int stride,
-                                                int width, int ring) {
-  return p >= start ? own + (size_t)(p - start) * stride : held + (size_t)(p % ring) * width;
+                                                int width, int from) {
+  return p >= start ? own + (size_t)(p - start) * stride : held + (size_t)(p - from) * width;
 }
 
 template <int KD>
@@ -388,7 +420,7 @@ __global__ __launch_bounds__(256) void talking_stats_kernel(const bf16_t* __rest
 #pragma unroll
     for (int e = 0; e < KP; ++e) {
       const int u = t + 256 * e, c = min((u % (DP / 8)) * 8, D - 8);   // (columns past a head's: q is zero there)
-      kn[e] = *reinterpret_cast<const u32x4*>(row_of(own, held, min(base + u / (DP / 8), last), s.start, a.p.stride, G * D, a.p.ring) + c);
+      kn[e] = *reinterpret_cast<const u32x4*>(row_of(own, held, min(base + u / (DP / 8), last), s.start, a.p.stride, G * D, from) + c);
     }
   };
   fetch(from);
@@ -400,7 +432,7 @@ __global__ __launch_bounds__(256) void talking_stats_kernel(const bf16_t* __rest
       const int u = t + 256 * e;
       *reinterpret_cast<u32x4*>(&kt[turn][u / (DP / 8)][(u % (DP / 8)) * 8]) = kn[e];
     }
-    __syncthreads();
+    block_barrier_lds();
     fetch(min(base + STAT_KEYS, last));
     f32x4 sc[4];
 #pragma unroll
@@ -512,8 +544,8 @@ __global__ __launch_bounds__(512) void talking_prompt_kernel(const bf16_t* __res
 
   bf16x8 kf[AHEAD ? SETS : 1][KD];
   u32x4 vn[4];   // the thread's first piece of a tile's values, on its way
-  const int v_cols = nv / 8, v_pieces = (KT / 4) * v_cols;
-  auto key_row = [&](int base) { return row_of(own_k, held_k, min(base + sub * 16 + l16, last), s.start, a.p.stride, nk, a.p.ring); };
+  const int v_pieces = (KT / 4) * (nv / 8);   // a column group's keys over neighbouring lanes, for the turned stores' banks
+  auto key_row = [&](int base) { return row_of(own_k, held_k, min(base + sub * 16 + l16, last), s.start, a.p.stride, nk, from); };
   auto fetch_keys = [&](const bf16_t* row, int u, bf16x8 (&to)[KD]) {
     const bf16_t* at = row + min(h0 + u * EACH, H - 1) / each * D;
 #pragma unroll
@@ -527,13 +559,13 @@ __global__ __launch_bounds__(512) void talking_prompt_kernel(const bf16_t* __res
     }
   };
   auto fetch_values = [&](int base, int piece, u32x4 (&v)[4]) {   // four keys of eight columns
-    const int k4 = piece / v_cols * 4, c = (piece % v_cols) * 8;
+    const int k4 = piece % (KT / 4) * 4, c = piece / (KT / 4) * 8;
 #pragma unroll
     for (int j = 0; j < 4; ++j)
-      v[j] = *reinterpret_cast<const u32x4*>(row_of(own_v, held_v, min(base + k4 + j, last), s.start, a.p.stride, nv, a.p.ring) + c);
+      v[j] = *reinterpret_cast<const u32x4*>(row_of(own_v, held_v, min(base + k4 + j, last), s.start, a.p.stride, nv, from) + c);
   };
   auto lay_values = [&](int piece, const u32x4 (&v)[4]) {   // turned: a column's four keys side by side
-    const int k4 = piece / v_cols * 4, c = (piece % v_cols) * 8;
+    const int k4 = piece % (KT / 4) * 4, c = piece / (KT / 4) * 8;
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
       *reinterpret_cast<uint2*>(vt + (c + 2 * j) * (KT + 8) + k4) =
@@ -573,7 +605,7 @@ __global__ __launch_bounds__(512) void talking_prompt_kernel(const bf16_t* __res
       }
       *reinterpret_cast<uint4*>(pair + l16 * S::PAIR + j * HP + h0) = pack8(w);
     }
-    __syncthreads();   // the weights are there, and the last tile's products are done
+    block_barrier_lds();   // the weights are there, and the last tile's products are done
     fetch_ahead(min(base + KT, last));
     // ---- values, turned, and the next ones on their way
     if (t < v_pieces) lay_values(t, vn);
@@ -584,9 +616,9 @@ __global__ __launch_bounds__(512) void talking_prompt_kernel(const bf16_t* __res
     }
     if (t < v_pieces) fetch_values(min(base + KT, last), t, vn);
     // ---- the heads mixed: 16 keys of one query at a time
-#pragma unroll 4
-    for (int u = wave; u < KT; u += 8) {   // KT / 16 pieces of each of 16 queries
-      const int qi = u / (KT / 16), j0 = u % (KT / 16) * 16;
+#pragma unroll
+    for (int n8 = 0; n8 < KT / 8; ++n8) {   // KT / 16 pieces of each of 16 queries
+      const int u = n8 * 8 + wave, qi = u / (KT / 16), j0 = u % (KT / 16) * 16;
       uint4 v = *reinterpret_cast<const uint4*>(pair + qi * S::PAIR + (j0 + l16) * HP + (quad * 8 < HP ? quad * 8 : 0));
       if (quad * 8 >= HP) v = make_uint4(0, 0, 0, 0);
 #pragma unroll
@@ -597,7 +629,7 @@ __global__ __launch_bounds__(512) void talking_prompt_kernel(const bf16_t* __res
           *reinterpret_cast<uint2*>(mix + qi * S::MIX + (n * 16 + l16) * (KT + 8) + j0 + quad * 4) = make_uint2(pack_bf16(m[0], m[1]), pack_bf16(m[2], m[3]));
       }
     }
-    __syncthreads();
+    block_barrier_lds();
     // ---- times the values: NG heads a wave
 #pragma unroll
     for (int e = 0; e < NG; ++e) {
@@ -707,22 +739,27 @@ extern "C" int iron_mha_talking(const void* x, void* keys, void* values, const u
   const TalkShape a{{rows, stride, heads, kv_heads, dim, vdim, ring}, chunk, heads * vdim};
   hipStream_t s = (hipStream_t)stream;
   const bool aligned = stride % 8 == 0 && dim % 8 == 0 && vdim % 8 == 0 && (((uintptr_t)x | (uintptr_t)keys | (uintptr_t)values) & 15) == 0;
-  IRON_REQUIRE(((uintptr_t)workspace & 3) == 0, "mha_talking: the workspace must be 4-byte aligned");
+  IRON_REQUIRE(((uintptr_t)workspace & 7) == 0, "mha_talking: the workspace must be 8-byte aligned");
   if (single) {   // the caller's spans have one row at most
-    const int each = heads / kv_heads, octets = (each + STEP_HEADS - 1) / STEP_HEADS, threads = chunk >= 1024 ? 1024 : (chunk + 63) / 64 * 64;
-    const size_t q_bytes = (size_t)each * dim * 4, m_bytes = (size_t)heads * (STEP_HEADS + 1) * 4;
-    IRON_REQUIRE(kv_heads * octets <= 65535 && q_bytes <= 64 * 1024 && m_bytes <= 48 * 1024, "mha_talking: %d heads of %d (%d key heads) in a step",
+    const int each = heads / kv_heads, at_once = each == 1 ? 1 : (each <= 4 ? 4 : 8), sets = (each + at_once - 1) / at_once, threads = chunk >= 1024 ? 1024 : (chunk + 63) / 64 * 64;
+    const size_t q_bytes = (size_t)each * dim * 4, m_bytes = (size_t)heads * (at_once + 1) * 4;
+    IRON_REQUIRE(kv_heads * sets <= 65535 && q_bytes <= 64 * 1024 && m_bytes <= 48 * 1024, "mha_talking: %d heads of %d (%d key heads) in a step",
                  heads, dim, kv_heads);
     float* work = (float*)workspace;
+#define IRON_TALK_MIX(T, VEC, HEADS)                                                                                                         \
+  hipLaunchKernelGGL((talking_mix_kernel<T, VEC, HEADS>), dim3(vdim / VEC, kv_heads * sets, slots), dim3(threads), m_bytes, s, (const T*)x, \
+                     (const T*)values, talk, spans, work, (T*)out, a)
 #define IRON_TALK_STEP(T, VEC)                                                                                                                \
   {                                                                                                                                           \
     hipLaunchKernelGGL((talking_scores_kernel<T, VEC>), dim3((chunk + 63) / 64, kv_heads, slots), dim3(64), q_bytes, s, (const T*)x, (T*)keys, \
                        (T*)values, spans, work, a);                                                                                           \
-    hipLaunchKernelGGL((talking_mix_kernel<T, VEC>), dim3(vdim / VEC, kv_heads * octets, slots), dim3(threads), m_bytes, s, (const T*)x,       \
-                       (const T*)values, talk, spans, work, (T*)out, a);                                                                      \
+    if (at_once == 1) IRON_TALK_MIX(T, VEC, 1);                                                                                               \
+    else if (at_once == 4) IRON_TALK_MIX(T, VEC, 4);                                                                                          \
+    else IRON_TALK_MIX(T, VEC, 8);                                                                                                            \
   }
     if (is_float) { if (aligned) IRON_TALK_STEP(float, 8) else IRON_TALK_STEP(float, 1) }
     else { if (aligned) IRON_TALK_STEP(bf16_t, 8) else IRON_TALK_STEP(bf16_t, 1) }
+#undef IRON_TALK_MIX
 #undef IRON_TALK_STEP
     IRON_LAUNCH_CHECK();
   }

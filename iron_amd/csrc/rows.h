@@ -74,4 +74,12 @@ __device__ __forceinline__ int first_chunk(const int* __restrict__ spans, int sl
 }
 __host__ __device__ inline long chunks_of(int rows, int slots, int chunk) { return (rows + chunk - 1) / chunk + slots; }
 
+// A barrier for what the block exchanges through LDS: waits for its LDS traffic, not (as __syncthreads does)
+// for the loads from memory in flight.
+__device__ __forceinline__ void block_barrier_lds() {
+  __builtin_amdgcn_fence(__ATOMIC_RELEASE, "workgroup", "local");
+  __builtin_amdgcn_s_barrier();
+  __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "workgroup", "local");
+}
+
 }  // namespace iron
