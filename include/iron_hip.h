@@ -527,8 +527,8 @@ int iron_turned_heads(const void* x, void* y, const uint16_t* bias, const uint16
 /* Attention of such rows within chunks of `chunk` positions: softmax a head over the chunk's positions up to the row's own,
  * the heads' weights mixed by talk (heads, heads), each head's mixed weights applied to its own values.  Position p's key
  * and value live in row p % ring of the slot's ring, ring = chunk.  single: every span is one row at most.  workspace: of
- * that many bytes, 8-byte aligned. */
-int64_t iron_mha_talking_workspace_bytes(int slots, int rows, int heads, int chunk, int single);
+ * that many bytes, 16-byte aligned. */
+int64_t iron_mha_talking_workspace_bytes(int slots, int rows, int heads, int vdim, int chunk, int single);
 int iron_mha_talking(const void* x, void* keys, void* values, const uint16_t* talk, const int* spans, void* out,
                      void* workspace, int slots, int rows, int stride, int heads, int kv_heads, int dim, int vdim, int chunk, int ring, int single,
                      int is_float, void* stream);

@@ -94,7 +94,7 @@ SIGNATURES = {
     "iron_stream_depth_rows": (c_int, [_P] * 6 + [c_int, c_int, _P, c_int, c_int, c_float, c_float, c_int, _P, _P]),
     "iron_activation": (c_int, [_P, _P, c_int, c_int, c_int, c_int, _P, _P]),
     "iron_turned_heads": (c_int, [_P] * 9 + [c_int, c_int, _P] + [c_int] * 9 + [c_float, c_float, c_int, _P, _P]),
-    "iron_mha_talking_workspace_bytes": (c_int64, [c_int] * 5),
+    "iron_mha_talking_workspace_bytes": (c_int64, [c_int] * 6),
     "iron_mha_talking": (c_int, [_P] * 7 + [c_int] * 11 + [_P]),
     "iron_matrix_memory": (c_int, [_P] * 7 + [c_int] * 8 + [c_float, c_int, _P]),
     "iron_matrix_memory_workspace_bytes": (c_int64, [c_int] * 4),

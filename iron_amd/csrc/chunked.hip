@@ -279,6 +279,7 @@ __global__ __launch_bounds__(TOPS_THREADS) void memory_tops_kernel(const T* __re
     }
     __syncthreads();   // (two sets: the next turn's writers do not meet this one's readers)
     const int n = min(AT_ONCE, count - base / CHUNK);
+#pragma unroll 8
     for (int c = 0; c < n; ++c) {
       if (t == 0) starts[(size_t)(first + base / CHUNK + c) * heads + head] = m;
       m = fmaxf(sums[turn][c] + m, most[turn][c]);

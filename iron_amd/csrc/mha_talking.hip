@@ -212,14 +212,15 @@ __global__ __launch_bounds__(256) void talking_rows_kernel(const T* __restrict__
 }
 
 // ---------------------------------------------------------------- a step
-// One row a slot, two launches.  talking_scores: a wave 64 keys of one key head: the scores of its query heads, left in memory,
-// their largest and the sum of exponentials under it; the row's own key and value go into the ring.  talking_mix: a block VEC
-// columns of a value head, a thread a key: all heads' weights of that key, mixed for up to HEADS heads, times the value.
-struct StepWork {   // floats a slot: scores [heads][chunk], then (largest, sum) [heads][pieces of 64 keys]
+// One row a slot, three launches.  talking_scores: a wave 64 keys of one key head: the scores of its query heads, left in memory,
+// their largest and the sum of exponentials under it; the row's own key and value go into the ring.  talking_mix: the heads'
+// weights from all scores, mixed.  talking_values: times the values.
+struct StepWork {   // floats a slot: scores [heads][chunk], (largest, sum) [heads][pieces of 64 keys], mixed weights [heads][chunk]
   int pieces;
-  size_t stats, words;
+  size_t stats, mixed, words;
   __host__ __device__ StepWork(int heads, int chunk)
-      : pieces((chunk + 63) / 64), stats(((size_t)heads * chunk + 1) & ~(size_t)1), words(stats + (size_t)heads * 2 * pieces) {}
+      : pieces((chunk + 63) / 64), stats(((size_t)heads * chunk + 1) & ~(size_t)1), mixed(stats + (size_t)heads * 2 * pieces),
+        words((mixed + (size_t)heads * chunk + 1) & ~(size_t)1) {}
 };
 template <typename T>
 __device__ __forceinline__ float weight_exp(float x) {
@@ -289,75 +290,87 @@ __global__ __launch_bounds__(64) void talking_scores_kernel(const T* __restrict_
   }
 }
 
+// The weights of 64 keys for HEADS heads a wave: a key a lane.
+template <typename T, int HEADS>
+__global__ __launch_bounds__(64) void talking_mix_kernel(const bf16_t* __restrict__ talk, const int* __restrict__ spans, float* __restrict__ work,
+                                                         TalkShape a) {
+  extern __shared__ __align__(16) float by[];   // [H][HEADS]: what the wave's heads take of a head, over its sum; [H]: its largest score
+  const int slot = blockIdx.z, h0 = blockIdx.y * HEADS, k0 = blockIdx.x * 64, lane = threadIdx.x, H = a.p.heads;
+  const Span s = span_of(spans, slot, a.p.rows);
+  const int count = s.start - s.start / a.chunk * a.chunk + 1, live = (count + 63) / 64;
+  if (s.rows == 0 || k0 >= count) return;
+  const StepWork w(H, a.chunk);
+  float* mine = work + slot * w.words;
+  const int j = min(k0 + lane, count - 1);
+  constexpr int AT_ONCE = 32;   // scores asked for together, the first ahead of the statistics
+  float raw[AT_ONCE];
+  auto fetch = [&](int first) {
+#pragma unroll
+    for (int u = 0; u < AT_ONCE; ++u) raw[u] = mine[(size_t)min(first + u, H - 1) * a.chunk + j];
+  };
+  fetch(0);
+  for (int h = lane; h < H; h += 64) {
+    const float2* st = reinterpret_cast<const float2*>(mine + w.stats) + (size_t)h * w.pieces;
+    float m = -INFINITY, l = 0.f;
+#pragma unroll 8
+    for (int i = 0; i < live; ++i) {
+      const float2 v = st[i];
+      const float higher = fmaxf(m, v.x);
+      l = l * expf(m - higher) + v.y * expf(v.x - higher);   // (each piece has a key: its largest is finite)
+      m = higher;
+    }
+    by[H * HEADS + h] = m;
+#pragma unroll
+    for (int e = 0; e < HEADS; ++e) by[h * HEADS + e] = bf16_to_f32(talk[(size_t)min(h0 + e, H - 1) * H + h]) / l;
+  }
+  __syncthreads();
+  float mixed[HEADS];
+#pragma unroll
+  for (int e = 0; e < HEADS; ++e) mixed[e] = 0.f;
+  for (int first = 0; first < H; first += AT_ONCE) {
+    if (first > 0) fetch(first);
+#pragma unroll
+    for (int u = 0; u < AT_ONCE; ++u) {
+      if (first + u >= H) continue;
+      const float weight = weight_exp<T>(raw[u] - by[H * HEADS + first + u]);
+#pragma unroll
+      for (int e = 0; e < HEADS; ++e) mixed[e] = fmaf(by[(first + u) * HEADS + e], weight, mixed[e]);
+    }
+  }
+#pragma unroll
+  for (int e = 0; e < HEADS; ++e)
+    if (h0 + e < H && k0 + lane < count) mine[w.mixed + (size_t)(h0 + e) * a.chunk + j] = mixed[e];
+}
+
+// VEC columns of a value head for HEADS of its query heads a block, a thread a key.
 template <typename T, int VEC, int HEADS>
-__global__ __launch_bounds__(1024) void talking_mix_kernel(const T* __restrict__ x, const T* __restrict__ values, const bf16_t* __restrict__ talk,
-                                                           const int* __restrict__ spans, const float* __restrict__ work, T* __restrict__ out,
-                                                           TalkShape a) {
-  extern __shared__ __align__(16) float lds[];
+__global__ __launch_bounds__(1024) void talking_values_kernel(const T* __restrict__ x, const T* __restrict__ values, const int* __restrict__ spans,
+                                                              const float* __restrict__ work, T* __restrict__ out, TalkShape a) {
   __shared__ float red[16][HEADS * VEC];
   const int slot = blockIdx.z, t = threadIdx.x, lane = t & 63, wave = t >> 6, waves = blockDim.x >> 6;
   const Span s = span_of(spans, slot, a.p.rows);
   if (s.rows == 0) return;
   const int H = a.p.heads, G = a.p.kv_heads, D = a.p.dim, V = a.p.vdim, each = H / G, sets = (each + HEADS - 1) / HEADS;
   const int g = blockIdx.y / sets, e0 = blockIdx.y % sets * HEADS, n = min(HEADS, each - e0), c = blockIdx.x * VEC;
-  const int pos = s.start, lo = pos / a.chunk * a.chunk, count = pos - lo + 1, live = (count + 63) / 64;
+  const int pos = s.start, lo = pos / a.chunk * a.chunk, count = pos - lo + 1;
   const StepWork w(H, a.chunk);
-  const float* mine = work + slot * w.words;
-  float* by = lds;                         // [H][HEADS]: what the block's heads take of a head, over its sum
-  float* top = by + H * HEADS;        // [H]
+  const float* mixed = work + slot * w.words + w.mixed;
   const T* own = x + (size_t)s.row0 * a.p.stride + (H + G) * D + g * V + c;
   const T* ring = values + (size_t)slot * a.p.ring * G * V + g * V + c;
-  // A key's value and the scores of its first heads: the thread's first key's are asked for ahead of the statistics.
-  constexpr int AT_ONCE = 32;
-  float f[VEC], raw[AT_ONCE];
-  auto fetch_value = [&](int j) { load_vec<VEC>(lo + j == pos ? own : ring + (size_t)j * G * V, f); };
-  auto fetch_scores = [&](int j, int h0) {
-#pragma unroll
-    for (int u = 0; u < AT_ONCE; ++u) raw[u] = mine[(size_t)min(h0 + u, H - 1) * a.chunk + j];
-  };
-  if (t < count) {
-    fetch_value(t);
-    fetch_scores(t, 0);
-  }
-  for (int h = wave; h < H; h += waves) {
-    const float2* st = reinterpret_cast<const float2*>(mine + w.stats) + (size_t)h * w.pieces;
-    const float mix = lane < n ? bf16_to_f32(talk[(size_t)(g * each + e0 + lane) * H + h]) : 0.f;
-    float m = -INFINITY, l = 0.f;
-    for (int i = lane; i < live; i += 64) {
-      const float2 v = st[i];
-      const float higher = fmaxf(m, v.x);
-      l = l * expf(m - higher) + v.y * expf(v.x - higher);   // (each piece has a key: its largest is finite)
-      m = higher;
-    }
-    const float most = wave_max(m), sum = wave_sum(m > -INFINITY ? l * expf(m - most) : 0.f);
-    if (lane == 0) top[h] = most;
-    if (lane < HEADS) by[h * HEADS + lane] = mix / sum;
-  }
-  __syncthreads();
   float acc[HEADS][VEC];
 #pragma unroll
   for (int e = 0; e < HEADS; ++e)
 #pragma unroll
     for (int k = 0; k < VEC; ++k) acc[e][k] = 0.f;
   for (int j = t; j < count; j += blockDim.x) {
-    float mixed[HEADS];
+    float f[VEC], by[HEADS];
+    load_vec<VEC>(lo + j == pos ? own : ring + (size_t)j * G * V, f);
 #pragma unroll
-    for (int e = 0; e < HEADS; ++e) mixed[e] = 0.f;
-    if (j != t) fetch_value(j);
-    for (int h0 = 0; h0 < H; h0 += AT_ONCE) {
-      if (j != t || h0 > 0) fetch_scores(j, h0);
-#pragma unroll
-      for (int u = 0; u < AT_ONCE; ++u) {
-        if (h0 + u >= H) continue;
-        const float weight = weight_exp<T>(raw[u] - top[h0 + u]);
-#pragma unroll
-        for (int e = 0; e < HEADS; ++e) mixed[e] = fmaf(by[(h0 + u) * HEADS + e], weight, mixed[e]);
-      }
-    }
+    for (int e = 0; e < HEADS; ++e) by[e] = mixed[(size_t)(g * each + min(e0 + e, each - 1)) * a.chunk + j];
 #pragma unroll
     for (int e = 0; e < HEADS; ++e)
 #pragma unroll
-      for (int k = 0; k < VEC; ++k) acc[e][k] = fmaf(mixed[e], f[k], acc[e][k]);
+      for (int k = 0; k < VEC; ++k) acc[e][k] = fmaf(by[e], f[k], acc[e][k]);
   }
 #pragma unroll
   for (int e = 0; e < HEADS; ++e)
@@ -383,14 +396,30 @@ __global__ __launch_bounds__(1024) void talking_mix_kernel(const T* __restrict__
 // (keys down the MFMA's rows, queries across), which lie in LDS a pair (query, key) at a time, heads side by side: one MFMA
 // operand of the heads' mixing, whose result goes back to LDS a head at a time, keys side by side: one operand of the
 // product with the values (transposed in LDS).  Two barriers a tile; keys and values of the next are on their way meanwhile.
+// A row's keys are dealt to blocks PART at a time; where that makes more than one, float32 sums are left and a last launch adds
+// them.
+struct PromptWork {   // floats: each row's statistics, then the parts' sums [part][row][heads * vdim]
+  int least, parts;   // the fewest keys of a part, and how many parts that makes of a row's at most
+  size_t sums, words;
+  __host__ __device__ PromptWork(int rows, int heads, int vdim, int chunk) {
+    least = ((chunk + 7) / 8 + 127) / 128 * 128;   // (whole tiles of any size)
+    parts = (chunk + 15 + least - 1) / least;      // of sixteen rows that begin at a chunk's last
+    sums = ((size_t)rows * heads + 3) & ~(size_t)3;
+    words = sums + (parts > 1 ? (size_t)parts * rows * heads * vdim : 0);
+  }
+  // A long span has blocks enough with fewer parts, and less to add.
+  __device__ int part(const Span& s) const { return s.rows >= 1024 && least < 512 ? 512 : least; }
+};
 constexpr float LOG2E = 1.4426950408889634f;
 constexpr int STAT_KEYS = 64;
 
 // The row of key or value `p`, of the chunk that starts at `from` or later: positions ahead of the span are that chunk's, in the
-// ring's rows from its first on.
+// ring's rows from its first on.  (Rows and their lengths are below 2^24.)
 __device__ __forceinline__ const bf16_t* row_of(const bf16_t* __restrict__ own, const bf16_t* __restrict__ held, int p, int start, int stride,
                                                 int width, int from) {
-  return p >= start ? own + (size_t)(p - start) * stride : held + (size_t)(p - from) * width;
+  const bool mine = p >= start;
+  const unsigned at = __umul24(mine ? p - start : p - from, mine ? stride : width);
+  return (mine ? own : held) + at;
 }
 
 template <int KD>
@@ -483,47 +512,48 @@ struct Talking {
 template <int NG, int KD, int VT, int EACH>
 __global__ __launch_bounds__(512) void talking_prompt_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ keys,
                                                              const bf16_t* __restrict__ values, const bf16_t* __restrict__ talk,
-                                                             const int* __restrict__ spans, const float* __restrict__ stats,
+                                                             const int* __restrict__ spans, float* __restrict__ stats,
                                                              bf16_t* __restrict__ out, TalkShape a) {
   using S = Talking<NG, KD, VT>;
-  constexpr int KT = S::KT, HP = S::HP, SETS = 8 / EACH;
-  constexpr bool HOLD = KD <= 2 && NG * VT <= 16;     // the queries stay in registers
-  constexpr bool AHEAD = SETS * KD <= 8 && NG * VT <= 16;   // a tile's keys are fetched under the tile before
+  // A wave's weights: HU heads against KU * 16 keys, its queries in registers throughout.  A set of heads shares its key head.
+  constexpr int KT = S::KT, HP = S::HP, HU = KD <= 2 ? 8 : 4, KU = 8 / HU, SETS = HU / EACH;
+  constexpr bool AHEAD = SETS * KU * KD <= 8 && NG * VT <= 16;   // a tile's keys are fetched under the tile before
   extern __shared__ __align__(16) bf16_t shared[];
   bf16_t* pair = shared;
   bf16_t* mix = pair + 16 * S::PAIR;
   bf16_t* vt = mix + 16 * S::MIX;                     // [G * V][KT + 8]
-  const int slot = blockIdx.y, q0 = ((int)gridDim.x - 1 - (int)blockIdx.x) * 16;
+  const int slot = blockIdx.z, q0 = ((int)gridDim.x - 1 - (int)blockIdx.x) * 16;
   const Span s = span_of(spans, slot, a.p.rows);
   if (q0 >= s.rows) return;
   const int H = a.p.heads, G = a.p.kv_heads, D = a.p.dim, V = a.p.vdim, each = H / G, nk = G * D, nv = G * V;
   const int t = threadIdx.x, lane = t & 63, wave = __builtin_amdgcn_readfirstlane(t >> 6), l16 = lane & 15, quad = lane >> 4;
-  const int first = s.start + q0, last = s.start + min(q0 + 16, s.rows) - 1, from = first / a.chunk * a.chunk;
+  const int first = s.start + q0, end = s.start + min(q0 + 16, s.rows) - 1, from = first / a.chunk * a.chunk;
+  const PromptWork work(a.p.rows, H, V, a.chunk);
+  const int part = work.part(s), begin = from + (int)blockIdx.y * part, last = min(end, begin + part - 1);
+  if (begin > end) return;
   const bf16_t* own_k = x + (size_t)s.row0 * a.p.stride + H * D;
   const bf16_t* own_v = own_k + nk;
   const bf16_t* held_k = keys + (size_t)slot * a.p.ring * nk;
   const bf16_t* held_v = values + (size_t)slot * a.p.ring * nv;
-  const int i = min(q0 + l16, s.rows - 1), pos = s.start + i, lo = pos / a.chunk * a.chunk;
+  const int i = min(q0 + l16, s.rows - 1), pos = s.start + i, lo = pos / a.chunk * a.chunk, end_lo = end / a.chunk * a.chunk;
   const bf16_t* q_row = x + (size_t)(s.row0 + i) * a.p.stride;
 
-  // This wave's weights: heads h0 .. h0 + 7 against keys sub * 16 .. + 15 of a tile.
-  const int h0 = (wave % NG) * 8, sub = wave / NG;
-  auto query = [&](int e, int d, int off) {
-    const int c = d * 32 + quad * 8;
-    u32x4 v = *reinterpret_cast<const u32x4*>(q_row + min(h0 + e, H - 1) * D + min(c, D - 8) + off);
-    if (c >= D) v = u32x4{0, 0, 0, 0};
-    return __builtin_bit_cast(bf16x8, v);
-  };
-  bf16x8 qf[HOLD ? 8 : 1][HOLD ? KD : 1];
-  float lse[8];
+  const int h0 = wave % (HP / HU) * HU, k0 = wave / (HP / HU) * KU * 16;   // the wave's first head, and its keys' first place in a tile
+  bf16x8 qf[HU][KD];
+  float lse[HU];
 #pragma unroll
-  for (int e = 0; e < 8; ++e) {
-    lse[e] = h0 + e < H ? stats[(size_t)(s.row0 + i) * H + h0 + e] : INFINITY;   // (a head that is none: no weight)
-    if constexpr (HOLD) {
+  for (int e = 0; e < HU; ++e) {
+    lse[e] = stats[(size_t)(s.row0 + i) * H + min(h0 + e, H - 1)];   // (no branch around a load: they go out together)
 #pragma unroll
-      for (int d = 0; d < KD; ++d) qf[e][d] = query(e, d, 0);
+    for (int d = 0; d < KD; ++d) {
+      const int c = d * 32 + quad * 8;
+      u32x4 v = *reinterpret_cast<const u32x4*>(q_row + min(h0 + e, H - 1) * D + min(c, D - 8));
+      if (c >= D) v = u32x4{0, 0, 0, 0};
+      qf[e][d] = __builtin_bit_cast(bf16x8, v);
     }
   }
+#pragma unroll
+  for (int e = 0; e < HU; ++e) lse[e] = h0 + e < H ? lse[e] : INFINITY;   // a head that is none: no weight
   // The heads' mixing as the second operand: head l16 (+ 16 n) of the result down its columns.
   bf16x8 tf[S::HN];
 #pragma unroll
@@ -532,8 +562,11 @@ __global__ __launch_bounds__(512) void talking_prompt_kernel(const bf16_t* __res
 #pragma unroll
     for (int j = 0; j < 8; ++j) {
       const int h = n * 16 + l16, g = quad * 8 + j;
-      w[j] = h < H && g < H ? talk[h * H + g] : (bf16_t)0;
+      w[j] = talk[min(h, H - 1) * H + min(g, H - 1)];
     }
+#pragma unroll
+    for (int j = 0; j < 8; ++j)
+      if (n * 16 + l16 >= H || quad * 8 + j >= H) w[j] = 0;
     tf[n] = __builtin_bit_cast(bf16x8, make_uint4(w[0] | (uint32_t)w[1] << 16, w[2] | (uint32_t)w[3] << 16, w[4] | (uint32_t)w[5] << 16, w[6] | (uint32_t)w[7] << 16));
   }
   f32x4 acc[NG][VT];
@@ -542,20 +575,21 @@ __global__ __launch_bounds__(512) void talking_prompt_kernel(const bf16_t* __res
 #pragma unroll
     for (int v = 0; v < VT; ++v) acc[e][v] = f32x4{0.f, 0.f, 0.f, 0.f};
 
-  bf16x8 kf[AHEAD ? SETS : 1][KD];
+  bf16x8 kf[AHEAD ? SETS : 1][KU][KD];
   u32x4 vn[4];   // the thread's first piece of a tile's values, on its way
   const int v_pieces = (KT / 4) * (nv / 8);   // a column group's keys over neighbouring lanes, for the turned stores' banks
-  auto key_row = [&](int base) { return row_of(own_k, held_k, min(base + sub * 16 + l16, last), s.start, a.p.stride, nk, from); };
-  auto fetch_keys = [&](const bf16_t* row, int u, bf16x8 (&to)[KD]) {
-    const bf16_t* at = row + min(h0 + u * EACH, H - 1) / each * D;
+  auto fetch_keys = [&](int base, int set, bf16x8 (&to)[KU][KD]) {
 #pragma unroll
-    for (int d = 0; d < KD; ++d) to[d] = __builtin_bit_cast(bf16x8, *reinterpret_cast<const u32x4*>(at + min(d * 32 + quad * 8, D - 8)));
+    for (int u = 0; u < KU; ++u) {
+      const bf16_t* at = row_of(own_k, held_k, min(base + k0 + u * 16 + l16, last), s.start, a.p.stride, nk, from) + min(h0 + set * EACH, H - 1) / each * D;
+#pragma unroll
+      for (int d = 0; d < KD; ++d) to[u][d] = __builtin_bit_cast(bf16x8, *reinterpret_cast<const u32x4*>(at + min(d * 32 + quad * 8, D - 8)));
+    }
   };
   auto fetch_ahead = [&](int base) {
     if constexpr (AHEAD) {
-      const bf16_t* row = key_row(base);
 #pragma unroll
-      for (int u = 0; u < SETS; ++u) fetch_keys(row, u, kf[u]);
+      for (int set = 0; set < SETS; ++set) fetch_keys(base, set, kf[set]);
     }
   };
   auto fetch_values = [&](int base, int piece, u32x4 (&v)[4]) {   // four keys of eight columns
@@ -574,37 +608,40 @@ __global__ __launch_bounds__(512) void talking_prompt_kernel(const bf16_t* __res
           make_uint2((v[0][j] >> 16) | (v[1][j] & 0xffff0000u), (v[2][j] >> 16) | (v[3][j] & 0xffff0000u));
     }
   };
-  fetch_ahead(from);
-  if (t < v_pieces) fetch_values(from, t, vn);
-  for (int base = from; base <= last; base += KT) {
+  fetch_ahead(begin);
+  if (t < v_pieces) fetch_values(begin, t, vn);
+  for (int base = begin; base <= last; base += KT) {
     // ---- weights
-    f32x4 sc[8];
-    int off = 0;
-    if constexpr (!HOLD) asm volatile("" : "+v"(off));   // (queries that are read every time are not to be held all the same)
-    const bf16_t* row = nullptr;
-    if constexpr (!AHEAD) row = key_row(base);
+    f32x4 sc[HU][KU];
 #pragma unroll
-    for (int e = 0; e < 8; ++e) {
-      sc[e] = f32x4{0.f, 0.f, 0.f, 0.f};
+    for (int e = 0; e < HU; ++e) {
       if constexpr (!AHEAD) {
-        if (e % EACH == 0) fetch_keys(row, e / EACH, kf[0]);
+        if (e % EACH == 0) fetch_keys(base, e / EACH, kf[0]);
       }
 #pragma unroll
-      for (int d = 0; d < KD; ++d)
-        sc[e] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[AHEAD ? e / EACH : 0][d], HOLD ? qf[HOLD ? e : 0][HOLD ? d : 0] : query(e, d, off), sc[e], 0, 0, 0);
-    }
+      for (int u = 0; u < KU; ++u) {
+        sc[e][u] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const int j = sub * 16 + quad * 4 + r, p = base + j;
-      const bool seen = p <= pos && p >= lo;
-      float w[8];
-#pragma unroll
-      for (int e = 0; e < 8; ++e) {
-        w[e] = __builtin_amdgcn_exp2f(fmaf(sc[e][r], LOG2E, -lse[e]));
-        w[e] = seen ? w[e] : 0.f;
+        for (int d = 0; d < KD; ++d) sc[e][u] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[AHEAD ? e / EACH : 0][u][d], qf[e][d], sc[e][u], 0, 0, 0);
       }
-      *reinterpret_cast<uint4*>(pair + l16 * S::PAIR + j * HP + h0) = pack8(w);
     }
+    const bool whole = base + KT - 1 <= first && base >= end_lo;   // every query sees every key
+#pragma unroll
+    for (int u = 0; u < KU; ++u)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int j = k0 + u * 16 + quad * 4 + r, p = base + j;
+        const bool seen = whole || (p <= pos && p >= lo);
+        uint32_t w[HU / 2];
+#pragma unroll
+        for (int e = 0; e < HU; e += 2) {
+          const uint32_t two = pack_bf16(__builtin_amdgcn_exp2f(fmaf(sc[e][u][r], LOG2E, -lse[e])), __builtin_amdgcn_exp2f(fmaf(sc[e + 1][u][r], LOG2E, -lse[e + 1])));
+          w[e / 2] = seen ? two : 0;
+        }
+        bf16_t* to = pair + l16 * S::PAIR + j * HP + h0;
+        if constexpr (HU == 8) *reinterpret_cast<u32x4*>(to) = u32x4{w[0], w[1], w[2], w[3]};
+        else *reinterpret_cast<uint2*>(to) = make_uint2(w[0], w[1]);
+      }
     block_barrier_lds();   // the weights are there, and the last tile's products are done
     fetch_ahead(min(base + KT, last));
     // ---- values, turned, and the next ones on their way
@@ -631,19 +668,38 @@ __global__ __launch_bounds__(512) void talking_prompt_kernel(const bf16_t* __res
     }
     block_barrier_lds();
     // ---- times the values: NG heads a wave
+    auto weights = [&](int h, int k) { return *reinterpret_cast<const bf16x8*>(mix + l16 * S::MIX + h * (KT + 8) + k + quad * 8); };
+    auto value = [&](int at, int v, int k) {
+      return *reinterpret_cast<const bf16x8*>(vt + min(at + v * 16 + l16, nv - 1) * (KT + 8) + k + quad * 8);
+    };
+    if constexpr (EACH == 4) {   // the wave's heads share their values
+      if (wave * NG < H) {
+        const int at = wave * NG / each * V;
 #pragma unroll
-    for (int e = 0; e < NG; ++e) {
-      const int h = wave * NG + e;
-      if (h >= H) continue;
-      const int at = h / each * V;
+        for (int k = 0; k < KT; k += 32) {
+          bf16x8 pf[NG];
 #pragma unroll
-      for (int k = 0; k < KT; k += 32) {
-        const bf16x8 pf = *reinterpret_cast<const bf16x8*>(mix + l16 * S::MIX + h * (KT + 8) + k + quad * 8);
+          for (int e = 0; e < NG; ++e) pf[e] = weights(min(wave * NG + e, H - 1), k);
 #pragma unroll
-        for (int v = 0; v < VT; ++v) {
-          if (v * 16 >= V) continue;
-          const bf16x8 vf = *reinterpret_cast<const bf16x8*>(vt + min(at + v * 16 + l16, nv - 1) * (KT + 8) + k + quad * 8);
-          acc[e][v] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pf, acc[e][v], 0, 0, 0);
+          for (int v = 0; v < VT; ++v) {
+            if (v * 16 >= V) continue;
+            const bf16x8 vf = value(at, v, k);
+#pragma unroll
+            for (int e = 0; e < NG; ++e) acc[e][v] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pf[e], acc[e][v], 0, 0, 0);
+          }
+        }
+      }
+    } else {
+#pragma unroll
+      for (int e = 0; e < NG; ++e) {
+        const int h = wave * NG + e;
+        if (h >= H) continue;
+#pragma unroll
+        for (int k = 0; k < KT; k += 32) {
+          const bf16x8 pf = weights(h, k);
+#pragma unroll
+          for (int v = 0; v < VT; ++v)
+            if (v * 16 < V) acc[e][v] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(value(h / each * V, v, k), pf, acc[e][v], 0, 0, 0);
         }
       }
     }
@@ -656,22 +712,52 @@ __global__ __launch_bounds__(512) void talking_prompt_kernel(const bf16_t* __res
 #pragma unroll
     for (int v = 0; v < VT; ++v) {
       const int c = v * 16 + quad * 4;
-      if (c < V)
+      if (c >= V) continue;
+      if (end - from < part)
         *reinterpret_cast<uint2*>(out + (size_t)(s.row0 + i) * a.out_stride + h * V + c) =
             make_uint2(pack_bf16(acc[e][v][0], acc[e][v][1]), pack_bf16(acc[e][v][2], acc[e][v][3]));
+      else
+        *reinterpret_cast<float4*>(stats + work.sums + ((size_t)blockIdx.y * a.p.rows + s.row0 + i) * H * V + h * V + c) =
+            make_float4(acc[e][v][0], acc[e][v][1], acc[e][v][2], acc[e][v][3]);
     }
   }
 }
 
+// A row whose keys went to several blocks: their sums, added in the parts' order.
+__global__ __launch_bounds__(256) void talking_sums_kernel(const float* __restrict__ stats, const int* __restrict__ spans, bf16_t* __restrict__ out,
+                                                           int slots, TalkShape a) {
+  const int row = blockIdx.y, c = (blockIdx.x * 256 + threadIdx.x) * 4, slot = slot_of_row(spans, slots, a.p.rows, row);
+  if (slot < 0) return;
+  const Span s = span_of(spans, slot, a.p.rows);
+  const int wide = a.p.heads * a.p.vdim, q0 = (row - s.row0) / 16 * 16;
+  const int from = (s.start + q0) / a.chunk * a.chunk, end = s.start + min(q0 + 16, s.rows) - 1;
+  const PromptWork work(a.p.rows, a.p.heads, a.p.vdim, a.chunk);
+  const int parts = (end - from) / work.part(s) + 1;
+  if (parts < 2 || c >= wide) return;
+  const float* at = stats + work.sums + (size_t)row * wide + c;
+  float4 sum = make_float4(0.f, 0.f, 0.f, 0.f);
+#pragma unroll 4
+  for (int p = 0; p < parts; ++p) {
+    const float4 v = *reinterpret_cast<const float4*>(at + (size_t)p * a.p.rows * wide);
+    sum.x += v.x;
+    sum.y += v.y;
+    sum.z += v.z;
+    sum.w += v.w;
+  }
+  *reinterpret_cast<uint2*>(out + (size_t)row * a.out_stride + c) = make_uint2(pack_bf16(sum.x, sum.y), pack_bf16(sum.z, sum.w));
+}
+
 template <int NG, int KD, int VT, int EACH>
 static int launch_talking_prompt(const bf16_t* x, const bf16_t* keys, const bf16_t* values, const bf16_t* talk, const int* spans,
-                                 const float* stats, bf16_t* out, const TalkShape& a, int slots, hipStream_t s) {
+                                 float* stats, bf16_t* out, const TalkShape& a, int slots, hipStream_t s) {
   const size_t lds = Talking<NG, KD, VT>::lds(a.p.kv_heads * a.p.vdim);
+  const int parts = PromptWork(a.p.rows, a.p.heads, a.p.vdim, a.chunk).parts;
   static LdsOptIn opt;
   const hipError_t e = opt.ensure(reinterpret_cast<const void*>(&talking_prompt_kernel<NG, KD, VT, EACH>), 160 * 1024);
   if (e != hipSuccess) { set_error("%s", hipGetErrorString(e)); return (int)e; }
-  hipLaunchKernelGGL((talking_prompt_kernel<NG, KD, VT, EACH>), dim3((a.p.rows + 15) / 16, slots), dim3(512), lds, s, x, keys, values, talk, spans, stats,
-                     out, a);
+  hipLaunchKernelGGL((talking_prompt_kernel<NG, KD, VT, EACH>), dim3((a.p.rows + 15) / 16, parts, slots), dim3(512), lds, s, x, keys, values, talk, spans,
+                     stats, out, a);
+  if (parts > 1) hipLaunchKernelGGL(talking_sums_kernel, dim3((a.out_stride + 1023) / 1024, a.p.rows), dim3(256), 0, s, stats, spans, out, slots, a);
   IRON_LAUNCH_CHECK();
 }
 // The groups of heads a prompt's kernel takes these sizes in, 0 where it takes them not at all.
@@ -721,8 +807,8 @@ extern "C" int iron_turned_heads(const void* x, void* y, const uint16_t* bias, c
   IRON_LAUNCH_CHECK();
 }
 
-extern "C" int64_t iron_mha_talking_workspace_bytes(int slots, int rows, int heads, int chunk, int single) {
-  return single ? (int64_t)slots * StepWork(heads, chunk).words * 4 : (int64_t)rows * heads * 4;
+extern "C" int64_t iron_mha_talking_workspace_bytes(int slots, int rows, int heads, int vdim, int chunk, int single) {
+  return 4 * (int64_t)(single ? slots * StepWork(heads, chunk).words : PromptWork(rows, heads, vdim, chunk).words);
 }
 
 
@@ -739,34 +825,38 @@ extern "C" int iron_mha_talking(const void* x, void* keys, void* values, const u
   const TalkShape a{{rows, stride, heads, kv_heads, dim, vdim, ring}, chunk, heads * vdim};
   hipStream_t s = (hipStream_t)stream;
   const bool aligned = stride % 8 == 0 && dim % 8 == 0 && vdim % 8 == 0 && (((uintptr_t)x | (uintptr_t)keys | (uintptr_t)values) & 15) == 0;
-  IRON_REQUIRE(((uintptr_t)workspace & 7) == 0, "mha_talking: the workspace must be 8-byte aligned");
+  IRON_REQUIRE(((uintptr_t)workspace & 15) == 0, "mha_talking: the workspace must be 16-byte aligned");
   if (single) {   // the caller's spans have one row at most
     const int each = heads / kv_heads, at_once = each == 1 ? 1 : (each <= 4 ? 4 : 8), sets = (each + at_once - 1) / at_once, threads = chunk >= 1024 ? 1024 : (chunk + 63) / 64 * 64;
-    const size_t q_bytes = (size_t)each * dim * 4, m_bytes = (size_t)heads * (at_once + 1) * 4;
-    IRON_REQUIRE(kv_heads * sets <= 65535 && q_bytes <= 64 * 1024 && m_bytes <= 48 * 1024, "mha_talking: %d heads of %d (%d key heads) in a step",
+    const size_t q_bytes = (size_t)each * dim * 4;
+    IRON_REQUIRE(kv_heads * sets <= 65535 && q_bytes <= 64 * 1024 && heads <= 1024, "mha_talking: %d heads of %d (%d key heads) in a step",
                  heads, dim, kv_heads);
     float* work = (float*)workspace;
-#define IRON_TALK_MIX(T, VEC, HEADS)                                                                                                         \
-  hipLaunchKernelGGL((talking_mix_kernel<T, VEC, HEADS>), dim3(vdim / VEC, kv_heads * sets, slots), dim3(threads), m_bytes, s, (const T*)x, \
-                     (const T*)values, talk, spans, work, (T*)out, a)
+    constexpr int MIXED = 8;
+#define IRON_TALK_VALUES(T, VEC, HEADS)                                                                                                     \
+  hipLaunchKernelGGL((talking_values_kernel<T, VEC, HEADS>), dim3(vdim / VEC, kv_heads * sets, slots), dim3(threads), 0, s, (const T*)x,    \
+                     (const T*)values, spans, work, (T*)out, a)
 #define IRON_TALK_STEP(T, VEC)                                                                                                                \
   {                                                                                                                                           \
     hipLaunchKernelGGL((talking_scores_kernel<T, VEC>), dim3((chunk + 63) / 64, kv_heads, slots), dim3(64), q_bytes, s, (const T*)x, (T*)keys, \
                        (T*)values, spans, work, a);                                                                                           \
-    if (at_once == 1) IRON_TALK_MIX(T, VEC, 1);                                                                                               \
-    else if (at_once == 4) IRON_TALK_MIX(T, VEC, 4);                                                                                          \
-    else IRON_TALK_MIX(T, VEC, 8);                                                                                                            \
+    hipLaunchKernelGGL((talking_mix_kernel<T, MIXED>), dim3((chunk + 63) / 64, (heads + MIXED - 1) / MIXED, slots), dim3(64),                 \
+                       (size_t)heads * (MIXED + 1) * 4, s, talk, spans, work, a);                                                             \
+    if (at_once == 1) IRON_TALK_VALUES(T, VEC, 1);                                                                                            \
+    else if (at_once == 4) IRON_TALK_VALUES(T, VEC, 4);                                                                                       \
+    else IRON_TALK_VALUES(T, VEC, 8);                                                                                                         \
   }
     if (is_float) { if (aligned) IRON_TALK_STEP(float, 8) else IRON_TALK_STEP(float, 1) }
     else { if (aligned) IRON_TALK_STEP(bf16_t, 8) else IRON_TALK_STEP(bf16_t, 1) }
-#undef IRON_TALK_MIX
+#undef IRON_TALK_VALUES
 #undef IRON_TALK_STEP
     IRON_LAUNCH_CHECK();
   }
   const size_t lds = (size_t)talk_row_words(heads, dim, vdim) * 4;
   const int groups = aligned && ((uintptr_t)out & 7) == 0 ? talking_groups(heads, kv_heads, dim, vdim, is_float) : 0;
   if (groups > 0) {
-    IRON_REQUIRE(rows <= 65535 * 64, "mha_talking: rows (%d) exceed the grid's y extent", rows);
+    IRON_REQUIRE(rows <= 65535 && stride < (1 << 24) && (long)rows * stride < (1L << 31) && (long)chunk * kv_heads * (dim > vdim ? dim : vdim) < (1L << 31) && chunk < (1 << 24),
+                 "mha_talking: %d rows of %d, chunks of %d: a row's place takes 32 bits", rows, stride, chunk);
     const bf16_t *xb = (const bf16_t*)x, *kb = (const bf16_t*)keys, *vb = (const bf16_t*)values;
     float* stats = (float*)workspace;
     const dim3 grid(heads, (rows + 63) / 64, slots);

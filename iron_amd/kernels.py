@@ -691,7 +691,7 @@ def mha_talking(x, keys, values, talk, spans, y, workspace, *, slots, rows, stri
     _act(values, slots * ring * kv_heads * vdim, "values")
     _bf16(talk, heads * heads, "talk")
     _act(y, rows * heads * vdim, "y")
-    need = int(lib().iron_mha_talking_workspace_bytes(slots, rows, heads, chunk, int(single)))
+    need = int(lib().iron_mha_talking_workspace_bytes(slots, rows, heads, vdim, chunk, int(single)))
     work = _work(workspace, need, "mha_talking: workspace")
     check(lib().iron_mha_talking(ptr(x), ptr(keys), ptr(values), ptr(talk), _spans(spans, slots), ptr(y), work, slots, rows, stride, heads, kv_heads,
                                  dim, vdim, chunk, ring, int(single), int(is_float), current_stream()), "iron_mha_talking")

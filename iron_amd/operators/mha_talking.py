@@ -113,7 +113,7 @@ class TalkingMHA(Operator):
     def _workspace_words(self) -> int:
         from .._lib import lib
 
-        return int(lib().iron_mha_talking_workspace_bytes(self.slots, self.rows, self.heads, self.chunk, int(self.single))) // 4
+        return int(lib().iron_mha_talking_workspace_bytes(self.slots, self.rows, self.heads, self.vdim, self.chunk, int(self.single))) // 4
 
     @classmethod
     def infer(cls, shapes, **kw):

@@ -102,7 +102,7 @@ def test_turned_heads(cuda, dtype, H, G, D, V, turned):
 
 # heads, key/value heads, dim, vdim, chunk
 SIZES = [(6, 2, 32, 48, 37), (4, 4, 64, 24, 20), (3, 1, 11, 7, 13), (1, 1, 12, 7, 1), (16, 4, 64, 64, 96), (32, 4, 32, 64, 160), (2, 2, 40, 48, 70),
-         (24, 8, 128, 128, 300), (32, 8, 64, 64, 128), (8, 2, 96, 64, 65), (5, 5, 72, 16, 100), (12, 3, 128, 112, 64), (40, 8, 32, 32, 50)]
+         (24, 8, 128, 128, 300), (32, 8, 64, 64, 128), (8, 2, 96, 64, 65), (5, 5, 72, 16, 100), (12, 3, 128, 112, 64), (40, 8, 32, 32, 50), (32, 8, 128, 128, 600), (8, 8, 16, 8, 1050)]
 
 
 def talking_case(rng, H, G, D, V, C, T, quiet=False):
@@ -136,7 +136,7 @@ def packed(q, k, v):
 def test_talking_attention_in_portions_and_steps(cuda, dtype, case, quiet):
     H, G, D, V, C = case
     rng = np.random.default_rng(D + H)
-    T = 190 if C < 190 else 340
+    T = 190 if C < 190 else C + 40
     q, k, v, talk = talking_case(rng, *case, T, quiet)
     x, want = packed(q, k, v), plain_talking(q, k, v, talk, C)
     limit = (3e-5 if dtype is F32 else 2e-2) * np.abs(want).max()
