@@ -2,10 +2,11 @@
 // ones, and the shares' sum of what they make of the row, down (act(gate h) * (up h)).
 //
 //   router:   float32 logits, a row a block
-//   pairs:    a (row, chosen expert) at a time, the weights' rows dealt to waves (few rows; either type)
+//   pairs:    a (row, chosen expert) at a time, or all of an expert's at once, the weights' rows dealt to waves (few rows; either type)
 //   grouped:  pairs dealt to their experts, each expert's padded to whole row tiles, two grouped products and a row's sum (bf16)
 #include "../../include/iron_hip.h"
 #include "grouped.h"
+#include "row_products.h"
 #include "rows.h"
 
 namespace iron {
@@ -74,47 +75,108 @@ __device__ __forceinline__ float act_exact(int kind, float g) {
   return kind == 3 ? fmaxf(g, 0.f) : (kind == 1 ? g / (1.f + expf(-g)) : gelu_tanh_f32(g));
 }
 
-// a[pair] = act(gate_e h) * (up_e h): a wave PER rows of each matrix.
-template <typename T, int VEC, int PER>
+// VEC elements of a row and of a weight's row, and their product: bf16 pairs as they were loaded, or floats.
+template <typename T, int VEC>
+struct Run {
+  float f[VEC];
+  template <typename U>
+  __device__ __forceinline__ void load(const U* __restrict__ p) { load_vec<VEC>(p, f); }
+  template <typename U>
+  __device__ __forceinline__ void stream(const U* __restrict__ p) { load_vec<VEC>(p, f); }
+};
+template <>
+struct Run<bf16_t, 8> {
+  uint4 v;
+  __device__ __forceinline__ void load(const bf16_t* __restrict__ p) { v = *reinterpret_cast<const uint4*>(p); }
+  __device__ __forceinline__ void stream(const bf16_t* __restrict__ p) { v = load_stream(reinterpret_cast<const uint4*>(p)); }
+};
+template <typename T, int VEC>
+__device__ __forceinline__ float add_product(const Run<T, VEC>& a, const Run<T, VEC>& b, float sum) {
+  if constexpr (sizeof(T) == 2 && VEC == 8) {
+    const uint4 x[1] = {a.v}, y[1] = {b.v};
+    return sum + dot_row<1>(x, y);
+  } else {
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) sum = fmaf(a.f[j], b.f[j], sum);
+    return sum;
+  }
+}
+
+// a[pair] = act(gate_e h) * (up_e h): a wave a row of each matrix.
+template <typename T, int VEC>
 __global__ __launch_bounds__(256) void expert_pairs_kernel(const T* __restrict__ h, const bf16_t* __restrict__ gate, const bf16_t* __restrict__ up,
                                                            const int* __restrict__ ids, T* __restrict__ a, int rows, int cols, int ff, int experts,
                                                            int top, int kind, const int* __restrict__ valid) {
-  const int pair = blockIdx.y, lane = threadIdx.x & 63, f0 = (blockIdx.x * 4 + (threadIdx.x >> 6)) * PER;
-  if (pair / top >= bound_or(valid, rows) || f0 >= ff) return;
-  const int e = min(max(ids[pair], 0), experts - 1);
+  const int pair = blockIdx.y, lane = threadIdx.x & 63, f = blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (pair / top >= bound_or(valid, rows) || f >= ff) return;
+  const size_t at = ((size_t)min(max(ids[pair], 0), experts - 1) * ff + f) * cols;
   const T* hr = h + (size_t)(pair / top) * cols;
-  float g[PER], u[PER];
-#pragma unroll
-  for (int p = 0; p < PER; ++p) g[p] = u[p] = 0.f;
-  const bf16_t *gr[PER], *ur[PER];
-#pragma unroll
-  for (int p = 0; p < PER; ++p) {
-    const size_t at = ((size_t)e * ff + min(f0 + p, ff - 1)) * cols;
-    gr[p] = gate + at;
-    ur[p] = up + at;
-  }
+  float g = 0.f, u = 0.f;
 #pragma unroll 4
   for (int c = lane * VEC; c < cols; c += 64 * VEC) {
-    float x[VEC], b[PER][VEC], d[PER][VEC];
-    load_vec<VEC>(hr + c, x);
+    Run<T, VEC> x, b, d;
+    b.stream(gate + at + c);
+    d.stream(up + at + c);
+    x.load(hr + c);
+    g = add_product(b, x, g);
+    u = add_product(d, x, u);
+  }
+  g = wave_sum(g);
+  u = wave_sum(u);
+  if (lane == 0) store_one(a + (size_t)pair * ff + f, act_exact(kind, g) * u);
+}
+
+// The same, a block one expert: its weights' rows meet all of its pairs, four at a time (several rows of a step).
+constexpr int SHARED_PAIRS = 4096;
+template <typename T, int VEC, int N>
+__device__ __forceinline__ void expert_rows(const T* __restrict__ h, const bf16_t* __restrict__ gr, const bf16_t* __restrict__ ur,
+                                            const int* __restrict__ list, T* __restrict__ a, int f, int cols, int ff, int top, int kind) {
+  const int lane = threadIdx.x & 63;
+  const T* hr[N];
+  float g[N], u[N];
 #pragma unroll
-    for (int p = 0; p < PER; ++p) {
-      load_vec<VEC>(gr[p] + c, b[p]);
-      load_vec<VEC>(ur[p] + c, d[p]);
+  for (int p = 0; p < N; ++p) {
+    hr[p] = h + (size_t)(__builtin_amdgcn_readfirstlane(list[p]) / top) * cols;
+    g[p] = u[p] = 0.f;
+  }
+#pragma unroll 2
+  for (int c = lane * VEC; c < cols; c += 64 * VEC) {
+    Run<T, VEC> x[N], b, d;
+    b.load(gr + c);
+    d.load(ur + c);
+#pragma unroll
+    for (int p = 0; p < N; ++p) x[p].load(hr[p] + c);
+#pragma unroll
+    for (int p = 0; p < N; ++p) {
+      g[p] = add_product(b, x[p], g[p]);
+      u[p] = add_product(d, x[p], u[p]);
     }
-#pragma unroll
-    for (int p = 0; p < PER; ++p)
-#pragma unroll
-      for (int j = 0; j < VEC; ++j) {
-        g[p] = fmaf(x[j], b[p][j], g[p]);
-        u[p] = fmaf(x[j], d[p][j], u[p]);
-      }
   }
 #pragma unroll
-  for (int p = 0; p < PER; ++p) {
+  for (int p = 0; p < N; ++p) {
     const float gs = wave_sum(g[p]), us = wave_sum(u[p]);
-    if (lane == 0 && f0 + p < ff) store_one(a + (size_t)pair * ff + f0 + p, act_exact(kind, gs) * us);
+    if (lane == 0) store_one(a + (size_t)list[p] * ff + f, act_exact(kind, gs) * us);
   }
+}
+template <typename T, int VEC>
+__global__ __launch_bounds__(256) void expert_shared_kernel(const T* __restrict__ h, const bf16_t* __restrict__ gate, const bf16_t* __restrict__ up,
+                                                            const int* __restrict__ ids, T* __restrict__ a, int rows, int cols, int ff,
+                                                            int experts, int top, int kind, const int* __restrict__ valid) {
+  __shared__ int list[SHARED_PAIRS], held;
+  const int e = blockIdx.y, f = blockIdx.x * 4 + (threadIdx.x >> 6), pairs = bound_or(valid, rows) * top;
+  if (threadIdx.x == 0) held = 0;
+  __syncthreads();
+  for (int p = threadIdx.x; p < pairs; p += 256)
+    if (min(max(ids[p], 0), experts - 1) == e) list[atomicAdd(&held, 1)] = p;
+  __syncthreads();
+  const int n = held;
+  if (n == 0 || f >= ff) return;
+  const size_t at = ((size_t)e * ff + f) * cols;
+  int p = 0;
+  for (; p + 4 <= n; p += 4) expert_rows<T, VEC, 4>(h, gate + at, up + at, list + p, a, f, cols, ff, top, kind);
+  if (n - p == 3) expert_rows<T, VEC, 3>(h, gate + at, up + at, list + p, a, f, cols, ff, top, kind);
+  else if (n - p == 2) expert_rows<T, VEC, 2>(h, gate + at, up + at, list + p, a, f, cols, ff, top, kind);
+  else if (n - p == 1) expert_rows<T, VEC, 1>(h, gate + at, up + at, list + p, a, f, cols, ff, top, kind);
 }
 
 // y[row] = sum over its experts of share * down_e a[pair]: a block PER rows of down, a wave every fourth of the experts.
@@ -141,14 +203,12 @@ __global__ __launch_bounds__(256) void expert_sums_kernel(const T* __restrict__ 
     }
 #pragma unroll 4
     for (int f = lane * VEC; f < ff; f += 64 * VEC) {
-      float x[VEC], b[PER][VEC];
+      Run<T, VEC> x, b[PER];
 #pragma unroll
-      for (int p = 0; p < PER; ++p) load_vec<VEC>(dr[p] + f, b[p]);
-      load_vec<VEC>(ar + f, x);
+      for (int p = 0; p < PER; ++p) b[p].load(dr[p] + f);
+      x.load(ar + f);
 #pragma unroll
-      for (int p = 0; p < PER; ++p)
-#pragma unroll
-        for (int j = 0; j < VEC; ++j) part[p] = fmaf(x[j], b[p][j], part[p]);
+      for (int p = 0; p < PER; ++p) part[p] = add_product(b[p], x, part[p]);
     }
 #pragma unroll
     for (int p = 0; p < PER; ++p) sum[p] = fmaf(share, part[p], sum[p]);
@@ -296,8 +356,12 @@ extern "C" int iron_experts(const void* h, const uint16_t* gate, const uint16_t*
                    (((uintptr_t)h | (uintptr_t)gate | (uintptr_t)up | (uintptr_t)down | (uintptr_t)workspace | (uintptr_t)y) & 15) == 0;
 #define IRON_PAIRS(T, VEC)                                                                                                                    \
   {                                                                                                                                           \
-    hipLaunchKernelGGL((expert_pairs_kernel<T, VEC, 1>), dim3((ff + 3) / 4, rows * top), dim3(256), 0, s, (const T*)h, gate, up, ids,         \
-                       (T*)workspace, rows, cols, ff, experts, top, activation, valid);                                                       \
+    if (rows > 1 && rows * top <= SHARED_PAIRS && experts <= 65535)                                                                           \
+      hipLaunchKernelGGL((expert_shared_kernel<T, VEC>), dim3((ff + 3) / 4, experts), dim3(256), 0, s, (const T*)h, gate, up, ids,            \
+                         (T*)workspace, rows, cols, ff, experts, top, activation, valid);                                                     \
+    else                                                                                                                                      \
+      hipLaunchKernelGGL((expert_pairs_kernel<T, VEC>), dim3((ff + 3) / 4, rows * top), dim3(256), 0, s, (const T*)h, gate, up, ids,          \
+                         (T*)workspace, rows, cols, ff, experts, top, activation, valid);                                                     \
     hipLaunchKernelGGL((expert_sums_kernel<T, VEC, 2>), dim3((cols + 1) / 2, rows), dim3(256), 0, s, (const T*)workspace, down, ids, shares, \
                        (T*)y, rows, cols, ff, experts, top, valid);                                                                           \
   }
