@@ -407,8 +407,8 @@ struct PromptWork {   // floats: each row's statistics, then the parts' sums [pa
     sums = ((size_t)rows * heads + 3) & ~(size_t)3;
     words = sums + (parts > 1 ? (size_t)parts * rows * heads * vdim : 0);
   }
-  // A long span has blocks enough with fewer parts, and less to add.
-  __device__ int part(const Span& s) const { return s.rows >= 1024 && least < 512 ? 512 : least; }
+  // Where there are blocks enough, longer parts: a block takes as long to begin as for half a dozen tiles of keys.
+  __device__ int part(const Span& s, int slots) const { return max(least, s.rows >= 1024 ? 512 : (s.rows * slots >= 1024 ? 256 : 128)); }
 };
 constexpr float LOG2E = 1.4426950408889634f;
 constexpr int STAT_KEYS = 64;
@@ -424,12 +424,14 @@ __device__ __forceinline__ const bf16_t* row_of(const bf16_t* __restrict__ own, 
 
 template <int KD>
 __global__ __launch_bounds__(256) void talking_stats_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ keys,
-                                                            const int* __restrict__ spans, float* __restrict__ stats, TalkShape a) {
+                                                            const int* __restrict__ spans, float* __restrict__ stats, int slots,
+                                                            TalkShape a) {
   constexpr int DP = KD * 32, KP = STAT_KEYS * DP / 8 / 256;
   __shared__ __align__(16) bf16_t kt[2][STAT_KEYS][DP + 8];
-  const int head = blockIdx.x, slot = blockIdx.z, q0 = blockIdx.y * 64;
+  const int head = blockIdx.x;
+  int slot, q0;
+  if (!tile_of(spans, slots, a.p.rows, 64, blockIdx.y, slot, q0)) return;
   const Span s = span_of(spans, slot, a.p.rows);
-  if (q0 >= s.rows) return;
   const int H = a.p.heads, D = a.p.dim, G = a.p.kv_heads, g = head / (H / G);
   const int t = threadIdx.x, lane = t & 63, wave = t >> 6, l16 = lane & 15, quad = lane >> 4;
   const int first = s.start + q0, last = s.start + min(q0 + 64, s.rows) - 1, from = first / a.chunk * a.chunk;
@@ -513,7 +515,7 @@ template <int NG, int KD, int VT, int EACH>
 __global__ __launch_bounds__(512) void talking_prompt_kernel(const bf16_t* __restrict__ x, const bf16_t* __restrict__ keys,
                                                              const bf16_t* __restrict__ values, const bf16_t* __restrict__ talk,
                                                              const int* __restrict__ spans, float* __restrict__ stats,
-                                                             bf16_t* __restrict__ out, TalkShape a) {
+                                                             bf16_t* __restrict__ out, int slots, TalkShape a) {
   using S = Talking<NG, KD, VT>;
   // A wave's weights: HU heads against KU * 16 keys, its queries in registers throughout.  A set of heads shares its key head.
   constexpr int KT = S::KT, HP = S::HP, HU = KD <= 2 ? 8 : 4, KU = 8 / HU, SETS = HU / EACH;
@@ -522,14 +524,14 @@ __global__ __launch_bounds__(512) void talking_prompt_kernel(const bf16_t* __res
   bf16_t* pair = shared;
   bf16_t* mix = pair + 16 * S::PAIR;
   bf16_t* vt = mix + 16 * S::MIX;                     // [G * V][KT + 8]
-  const int slot = blockIdx.z, q0 = ((int)gridDim.x - 1 - (int)blockIdx.x) * 16;
+  int slot, q0;
+  if (!tile_of(spans, slots, a.p.rows, 16, (int)gridDim.x - 1 - (int)blockIdx.x, slot, q0)) return;
   const Span s = span_of(spans, slot, a.p.rows);
-  if (q0 >= s.rows) return;
   const int H = a.p.heads, G = a.p.kv_heads, D = a.p.dim, V = a.p.vdim, each = H / G, nk = G * D, nv = G * V;
   const int t = threadIdx.x, lane = t & 63, wave = __builtin_amdgcn_readfirstlane(t >> 6), l16 = lane & 15, quad = lane >> 4;
   const int first = s.start + q0, end = s.start + min(q0 + 16, s.rows) - 1, from = first / a.chunk * a.chunk;
   const PromptWork work(a.p.rows, H, V, a.chunk);
-  const int part = work.part(s), begin = from + (int)blockIdx.y * part, last = min(end, begin + part - 1);
+  const int part = work.part(s, slots), begin = from + (int)blockIdx.y * part, last = min(end, begin + part - 1);
   if (begin > end) return;
   const bf16_t* own_k = x + (size_t)s.row0 * a.p.stride + H * D;
   const bf16_t* own_v = own_k + nk;
@@ -732,7 +734,7 @@ __global__ __launch_bounds__(256) void talking_sums_kernel(const float* __restri
   const int wide = a.p.heads * a.p.vdim, q0 = (row - s.row0) / 16 * 16;
   const int from = (s.start + q0) / a.chunk * a.chunk, end = s.start + min(q0 + 16, s.rows) - 1;
   const PromptWork work(a.p.rows, a.p.heads, a.p.vdim, a.chunk);
-  const int parts = (end - from) / work.part(s) + 1;
+  const int parts = (end - from) / work.part(s, slots) + 1;
   if (parts < 2 || c >= wide) return;
   const float* at = stats + work.sums + (size_t)row * wide + c;
   float4 sum = make_float4(0.f, 0.f, 0.f, 0.f);
@@ -755,8 +757,8 @@ static int launch_talking_prompt(const bf16_t* x, const bf16_t* keys, const bf16
   static LdsOptIn opt;
   const hipError_t e = opt.ensure(reinterpret_cast<const void*>(&talking_prompt_kernel<NG, KD, VT, EACH>), 160 * 1024);
   if (e != hipSuccess) { set_error("%s", hipGetErrorString(e)); return (int)e; }
-  hipLaunchKernelGGL((talking_prompt_kernel<NG, KD, VT, EACH>), dim3((a.p.rows + 15) / 16, parts, slots), dim3(512), lds, s, x, keys, values, talk, spans,
-                     stats, out, a);
+  hipLaunchKernelGGL((talking_prompt_kernel<NG, KD, VT, EACH>), dim3((a.p.rows + 15) / 16 + slots - 1, parts), dim3(512), lds, s, x, keys, values, talk,
+                     spans, stats, out, slots, a);
   if (parts > 1) hipLaunchKernelGGL(talking_sums_kernel, dim3((a.out_stride + 1023) / 1024, a.p.rows), dim3(256), 0, s, stats, spans, out, slots, a);
   IRON_LAUNCH_CHECK();
 }
@@ -859,9 +861,9 @@ extern "C" int iron_mha_talking(const void* x, void* keys, void* values, const u
                  "mha_talking: %d rows of %d, chunks of %d: a row's place takes 32 bits", rows, stride, chunk);
     const bf16_t *xb = (const bf16_t*)x, *kb = (const bf16_t*)keys, *vb = (const bf16_t*)values;
     float* stats = (float*)workspace;
-    const dim3 grid(heads, (rows + 63) / 64, slots);
-    if (dim <= 64) hipLaunchKernelGGL((talking_stats_kernel<2>), grid, dim3(256), 0, s, xb, kb, spans, stats, a);
-    else hipLaunchKernelGGL((talking_stats_kernel<4>), grid, dim3(256), 0, s, xb, kb, spans, stats, a);
+    const dim3 grid(heads, (rows + 63) / 64 + slots - 1);
+    if (dim <= 64) hipLaunchKernelGGL((talking_stats_kernel<2>), grid, dim3(256), 0, s, xb, kb, spans, stats, slots, a);
+    else hipLaunchKernelGGL((talking_stats_kernel<4>), grid, dim3(256), 0, s, xb, kb, spans, stats, slots, a);
     const bool fours = heads / kv_heads % 4 == 0;
     int e;
 #define IRON_TALK(NG, KD, VT)                                                                                                \

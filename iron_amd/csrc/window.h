@@ -48,4 +48,29 @@ __device__ __forceinline__ int slot_of_row(const int* __restrict__ spans, int sl
   return -1;
 }
 
+// The spans cut into tiles of `size` rows, one span's after the other's in the order of the slots: the slot of tile `index` and its
+// first row within the span.  False past the last.
+__device__ __forceinline__ bool tile_of(const int* __restrict__ spans, int slots, int rows, int size, int index, int& slot, int& first) {
+  const int lane = (int)threadIdx.x & 63;
+  for (int f = 0; f < slots; f += 64) {
+    int n = 0;
+    if (f + lane < slots) n = (span_of(spans, f + lane, rows).rows + size - 1) / size;
+    int sum = n;
+#pragma unroll
+    for (int d = 1; d < 64; d <<= 1) {
+      const int v = __shfl_up(sum, d, 64);
+      if (lane >= d) sum += v;
+    }
+    const unsigned long long past = __builtin_amdgcn_ballot_w64(index < sum);
+    if (past != 0) {
+      const int at = __builtin_ctzll(past);
+      slot = __builtin_amdgcn_readfirstlane(f + at);
+      first = __builtin_amdgcn_readfirstlane((index - (__shfl(sum, at, 64) - __shfl(n, at, 64))) * size);
+      return true;
+    }
+    index -= __shfl(sum, 63, 64);
+  }
+  return false;
+}
+
 }  // namespace iron
