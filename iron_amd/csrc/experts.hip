@@ -107,23 +107,24 @@ template <typename T, int VEC>
 __global__ __launch_bounds__(256) void expert_pairs_kernel(const T* __restrict__ h, const bf16_t* __restrict__ gate, const bf16_t* __restrict__ up,
                                                            const int* __restrict__ ids, T* __restrict__ a, int rows, int cols, int ff, int experts,
                                                            int top, int kind, const int* __restrict__ valid) {
-  const int pair = blockIdx.y, lane = threadIdx.x & 63, f = blockIdx.x * 4 + (threadIdx.x >> 6);
-  if (pair / top >= bound_or(valid, rows) || f >= ff) return;
-  const size_t at = ((size_t)min(max(ids[pair], 0), experts - 1) * ff + f) * cols;
-  const T* hr = h + (size_t)(pair / top) * cols;
-  float g = 0.f, u = 0.f;
+  const int lane = threadIdx.x & 63, f = blockIdx.x * 4 + (threadIdx.x >> 6), pairs = f < ff ? bound_or(valid, rows) * top : 0;
+  for (int pair = blockIdx.y; pair < pairs; pair += gridDim.y) {
+    const size_t at = ((size_t)min(max(ids[pair], 0), experts - 1) * ff + f) * cols;
+    const T* hr = h + (size_t)(pair / top) * cols;
+    float g = 0.f, u = 0.f;
 #pragma unroll 4
-  for (int c = lane * VEC; c < cols; c += 64 * VEC) {
-    Run<T, VEC> x, b, d;
-    b.stream(gate + at + c);
-    d.stream(up + at + c);
-    x.load(hr + c);
-    g = add_product(b, x, g);
-    u = add_product(d, x, u);
+    for (int c = lane * VEC; c < cols; c += 64 * VEC) {
+      Run<T, VEC> x, b, d;
+      b.stream(gate + at + c);
+      d.stream(up + at + c);
+      x.load(hr + c);
+      g = add_product(b, x, g);
+      u = add_product(d, x, u);
+    }
+    g = wave_sum(g);
+    u = wave_sum(u);
+    if (lane == 0) store_one(a + (size_t)pair * ff + f, act_exact(kind, g) * u);
   }
-  g = wave_sum(g);
-  u = wave_sum(u);
-  if (lane == 0) store_one(a + (size_t)pair * ff + f, act_exact(kind, g) * u);
 }
 
 // The same, a block one expert: its weights' rows meet all of its pairs, four at a time (several rows of a step).
@@ -351,7 +352,8 @@ extern "C" int iron_experts(const void* h, const uint16_t* gate, const uint16_t*
     hipLaunchKernelGGL(expert_gather_kernel, dim3((cols + 2047) / 2048, rows), dim3(256), 0, s, outs, place, shares, (bf16_t*)y, rows, cols, top, valid);
     IRON_LAUNCH_CHECK();
   }
-  IRON_REQUIRE((long)rows * top <= 65535, "experts: %d rows of %d experts exceed the grid's y extent", rows, top);
+  IRON_REQUIRE(rows <= 65535 && (long)rows * top <= (1 << 30), "experts: %d rows of %d experts exceed the grid's y extent", rows, top);
+  const int pairs_y = rows * top < 65535 ? rows * top : 65535;
   const bool vec = cols % 8 == 0 && ff % 8 == 0 &&
                    (((uintptr_t)h | (uintptr_t)gate | (uintptr_t)up | (uintptr_t)down | (uintptr_t)workspace | (uintptr_t)y) & 15) == 0;
 #define IRON_PAIRS(T, VEC)                                                                                                                    \
@@ -360,7 +362,7 @@ extern "C" int iron_experts(const void* h, const uint16_t* gate, const uint16_t*
       hipLaunchKernelGGL((expert_shared_kernel<T, VEC>), dim3((ff + 3) / 4, experts), dim3(256), 0, s, (const T*)h, gate, up, ids,            \
                          (T*)workspace, rows, cols, ff, experts, top, activation, valid);                                                     \
     else                                                                                                                                      \
-      hipLaunchKernelGGL((expert_pairs_kernel<T, VEC>), dim3((ff + 3) / 4, rows * top), dim3(256), 0, s, (const T*)h, gate, up, ids,          \
+      hipLaunchKernelGGL((expert_pairs_kernel<T, VEC>), dim3((ff + 3) / 4, pairs_y), dim3(256), 0, s, (const T*)h, gate, up, ids,          \
                          (T*)workspace, rows, cols, ff, experts, top, activation, valid);                                                     \
     hipLaunchKernelGGL((expert_sums_kernel<T, VEC, 2>), dim3((cols + 1) / 2, rows), dim3(256), 0, s, (const T*)workspace, down, ids, shares, \
                        (T*)y, rows, cols, ff, experts, top, valid);                                                                           \

@@ -84,7 +84,7 @@ def test_norms_around_one_and_activations(cuda, dtype, cols):
 
 
 @BOTH
-@pytest.mark.parametrize("H,G,D,V,turned", [(6, 2, 32, 48, 16), (3, 1, 11, 7, 6), (2, 2, 128, 64, 128), (4, 2, 96, 200, 0), (8, 4, 8, 16, 2)])
+@pytest.mark.parametrize("H,G,D,V,turned", [(6, 2, 32, 48, 16), (3, 1, 11, 7, 6), (2, 2, 128, 64, 128), (6, 2, 88, 200, 0), (8, 4, 8, 16, 2)])
 def test_turned_heads(cuda, dtype, H, G, D, V, turned):
     rng = np.random.default_rng(D)
     stride, first_at = (H + G) * D + G * V, 24
@@ -102,7 +102,7 @@ def test_turned_heads(cuda, dtype, H, G, D, V, turned):
 
 # heads, key/value heads, dim, vdim, chunk
 SIZES = [(6, 2, 32, 48, 37), (4, 4, 64, 24, 20), (3, 1, 11, 7, 13), (1, 1, 12, 7, 1), (16, 4, 64, 64, 96), (32, 4, 32, 64, 160), (2, 2, 40, 48, 70),
-         (24, 8, 128, 128, 300), (32, 8, 64, 64, 128), (8, 2, 96, 64, 65), (5, 5, 72, 16, 100), (12, 3, 128, 112, 64), (40, 8, 32, 32, 50), (32, 8, 128, 128, 600), (8, 8, 16, 8, 1050)]
+         (24, 8, 128, 128, 300), (32, 8, 64, 64, 128), (8, 2, 88, 48, 65), (5, 5, 72, 16, 100), (12, 3, 128, 112, 64), (40, 8, 32, 32, 50), (32, 8, 128, 128, 600), (8, 8, 16, 8, 1050)]
 
 
 def talking_case(rng, H, G, D, V, C, T, quiet=False):
@@ -221,7 +221,7 @@ def test_a_matrix_memory(cuda, dtype, chunked, H, D, V):
 @TOKENS
 def test_the_memory_goes_on_where_a_portion_ends(cuda, chunked):
     rng = np.random.default_rng(7)
-    H, D, V, T = 2, 32, 48, 200
+    H, D, V, T = 2, 40, 48, 200
     op = memory_op(1, T, H, D, V, F32)
     whole = memory_inputs(rng, op, table((0, 0, T, 0)))
     whole["x"][90, op.i_at] = 60.0   # a gate that stands out
@@ -262,7 +262,7 @@ def test_memory_gates(cuda, dtype, H, V):
 
 
 @BOTH
-@pytest.mark.parametrize("rows,cols,experts,top", [(5, 128, 12, 3), (300, 96, 7, 7), (1, 60, 1, 1), (9, 37, 130, 11), (4, 2048, 64, 8)])
+@pytest.mark.parametrize("rows,cols,experts,top", [(5, 128, 13, 3), (300, 96, 7, 7), (1, 60, 1, 1), (9, 37, 130, 11), (4, 2048, 64, 8)])
 def test_a_router(cuda, dtype, rows, cols, experts, top):
     rng = np.random.default_rng(cols)
     given = dict(h=bf(rng, rows, cols), weight=bf(rng, experts, cols, scale=2 / np.sqrt(cols)), bias=bf(rng, experts))
@@ -276,8 +276,8 @@ def test_a_router(cuda, dtype, rows, cols, experts, top):
 
 
 @BOTH
-@pytest.mark.parametrize("rows,cols,ff,experts,top", [(5, 128, 96, 12, 3), (300, 96, 64, 7, 2), (1, 60, 21, 1, 1), (9, 37, 10, 5, 5), (200, 256, 128, 16, 4),
-                                                      (700, 192, 320, 3, 1), (130, 320, 96, 40, 3), (1000, 64, 72, 6, 2)])
+@pytest.mark.parametrize("rows,cols,ff,experts,top", [(5, 128, 80, 11, 2), (300, 96, 64, 7, 2), (1, 60, 21, 1, 1), (9, 37, 10, 5, 5), (200, 256, 128, 16, 4),
+                                                      (700, 192, 320, 3, 1), (130, 256, 104, 40, 3), (1000, 64, 72, 6, 2), (1100, 24, 9, 64, 60)])
 def test_routed_feed_forwards(cuda, dtype, rows, cols, ff, experts, top):
     rng = np.random.default_rng(ff)
     ids = np.stack([rng.permutation(experts)[:top] for _ in range(rows)]).astype(np.int32)
