@@ -384,10 +384,10 @@ int iron_gemm_few_bf16(const uint16_t* A, const uint16_t* B, const uint16_t* B2,
  * that starts at position 0 reads none, so a slot needs no clearing between sequences.
  * `is_float`: void* activations are float instead of bf16 (a model that runs in 32 bits throughout). */
 
-/* x[i] = table[ids[i]] widened to float, for i < *valid (or rows); ids outside the table are skipped.  also (may be
+/* x[i] = scale * table[ids[i]] in float, for i < *valid (or rows); ids outside the table are skipped.  also (may be
  * NULL): the same rows once more. */
 int iron_stream_embed(const uint16_t* table, const int* ids, float* x, float* also, int rows, int table_rows, int cols,
-                      const int* valid, void* stream);
+                      float scale, const int* valid, void* stream);
 /* The stream's rows: with y, x += rmsnorm(y + y_bias) * (unit + back_gain) in place (y_bias may be NULL); with h,
  * h = rmsnorm(x) * (unit + gain) of the rows as they then stand.  Float throughout, h rounded once. */
 int iron_stream_rows(float* x, const void* y, const uint16_t* y_bias, const uint16_t* back_gain, const uint16_t* gain, void* h,
@@ -403,6 +403,15 @@ int iron_stream_depth_rows(float* x, const void* y, const uint16_t* y_bias, cons
 int iron_stream_gated_rows(float* x, const void* y, const uint16_t* y_bias, const void* gate, const uint16_t* gate_bias,
                            int gate_stride, int gate_at, const uint16_t* gain, void* h, int rows, int cols, float eps,
                            int is_float, const int* valid, void* stream);
+/* The stream's rows: with y, x += y + y2 in place (y2 may be NULL); with h, each of the `groups` equal parts of a row as it
+ * then stands over its own root mean square, times (unit + gain).  Float throughout, h rounded once. */
+int iron_stream_groups(float* x, const void* y, const void* y2, const uint16_t* gain, void* h, int rows, int cols, int groups,
+                       float eps, float unit, int is_float, const int* valid, void* stream);
+/* Columns at .. + cols of y (rows of width) = act(g) * u, g and u the columns gate_at .. and gate_at + cols .. of x (rows of
+ * stride).  kind: 0 the limited gate, g' sigmoid(1.702 g') (u' + 1) with g' = min(g, limit), u' = u within [-limit, limit]; 1
+ * SiLU, 2 GELU (tanh form), 3 ReLU. */
+int iron_gated_columns(const void* x, void* y, int rows, int cols, int stride, int gate_at, int width, int at, int kind,
+                       float limit, int is_float, const int* valid, void* stream);
 /* y = a N(z) + b N(z^2) + c N(z^3) + e, z columns at .. of x (rows, stride) plus bias (may be NULL), powers element
  * by element, N over a row's root mean square; coefficients {a, b, c, e}.  y (rows, cols); float, rounded once. */
 int iron_poly_norm(const void* x, const uint16_t* bias, const uint16_t* coefficients, void* y, int rows, int cols,
@@ -456,7 +465,8 @@ int iron_time_mix_chunked(const void* r, const void* k, const void* v, const flo
 int64_t iron_delta_rule_workspace_bytes(int slots, int rows, int heads);
 int iron_delta_rule_chunked(const float* x, float* state, const int* spans, float* o, void* workspace, int slots, int rows,
                             int heads, int kv_heads, int dim, int vdim, void* stream);
-/* out = o / rms(o, one head) * gain * silu(gate) * scale; gain (dim) if gain_shared, else (heads * dim). */
+/* out = o / rms(o, one head) * gain * silu(gate) * scale; gain (dim) if gain_shared, else (heads * dim).  gate NULL: that
+ * factor is 1. */
 int iron_head_gate(const float* o, const void* gate, const uint16_t* gain, void* out, int rows, int heads, int dim,
                    int gate_stride, int gate_at, int gain_shared, int out_stride, int out_at, float eps, float scale,
                    int is_float, const int* valid, void* stream);
@@ -547,15 +557,49 @@ int iron_matrix_memory_chunked(const void* x, const uint16_t* i_bias, const uint
 /* y = o / (max(|n . q|, exp(-m)) + floor), RMS-normed a head, times gain (heads * dim) and sigmoid(gate). */
 int iron_memory_gate(const float* o, const void* gate, const uint16_t* gain, void* y, int rows, int heads, int dim,
                      int gate_stride, int gate_at, float floor, float eps, int is_float, const int* valid, void* stream);
-/* A row's `top` experts by the largest of its logits w h + bias (float), and their shares, a softmax over the chosen logits. */
-int iron_router(const void* h, const uint16_t* w, const uint16_t* bias, int* ids, float* shares, int rows, int cols,
-                int experts, int top, int is_float, const int* valid, void* stream);
+/* A row's `top` experts by the largest of its logits w h + bias (float; bias may be NULL), and their shares, a softmax over the
+ * chosen logits; or (scored) by the largest of the logits' softmax plus correction (may be NULL), and their shares, the softmax's
+ * over their sum + 1e-20. */
+int iron_router(const void* h, const uint16_t* w, const uint16_t* bias, const uint16_t* correction, int scored, int* ids,
+                float* shares, int rows, int cols, int experts, int top, int is_float, const int* valid, void* stream);
 /* y = sum over a row's experts e of share * down_e (act(gate_e h) * (up_e h)); gate and up (experts, ff, cols), down
- * (experts, cols, ff).  activation: 1 SiLU, 2 GELU (tanh form), 3 ReLU. */
+ * (experts, cols, ff).  With identity > 0, ids from `experts` on stand for h itself.  activation: 1 SiLU, 2 GELU (tanh form),
+ * 3 ReLU. */
 int64_t iron_experts_workspace_bytes(int rows, int cols, int ff, int experts, int top, int is_float);
 int iron_experts(const void* h, const uint16_t* gate, const uint16_t* up, const uint16_t* down, const int* ids,
-                 const float* shares, void* y, void* workspace, int rows, int cols, int ff, int experts, int top,
+                 const float* shares, void* y, void* workspace, int rows, int cols, int ff, int experts, int identity, int top,
                  int activation, int is_float, const int* valid, void* stream);
+/* HGRN2: per head S <- diag(f) S + (1 - f) v^T, then o = S^T silu(q), f = lower + (1 - lower) sigmoid(z + f_bias).  x: rows
+ * [q | z | v | ..]; f_bias, lower (heads * dim); state (slots, heads, dim, vdim); o (rows, heads * vdim), float.  dim <= 256. */
+int iron_hgrn2(const void* x, const uint16_t* f_bias, const uint16_t* lower, float* state, const int* spans, float* o, int slots,
+               int rows, int stride, int heads, int dim, int vdim, int is_float, void* stream);
+/* The same sixteen tokens at a time, with a workspace of that many bytes, 16-byte aligned. */
+int64_t iron_hgrn2_workspace_bytes(int slots, int rows, int heads, int dim);
+int iron_hgrn2_chunked(const void* x, const uint16_t* f_bias, const uint16_t* lower, float* state, const int* spans, float* o,
+                       void* workspace, int slots, int rows, int stride, int heads, int dim, int vdim, int is_float,
+                       void* stream);
+/* One token a slot, bf16, in one launch: iron_hgrn2, iron_head_gate without a gate (gains (vdim) shared by the heads) into columns
+ * out_at .. of out, and beside it iron_gated_columns of the same rows into those from gated_at (cols 0: none).  vdim a power
+ * of two from 16. */
+int iron_decode_hgrn2_bf16(const uint16_t* x, const uint16_t* f_bias, const uint16_t* lower, const uint16_t* norm, float* state,
+                           const int* spans, uint16_t* out, int slots, int rows, int stride, int heads, int dim, int vdim,
+                           int out_stride, int out_at, float eps, int cols, int gate_at, int gated_at, int kind, float limit,
+                           void* stream);
+/* Rows [q heads | k heads | v heads | ..] of a packed projection made ready to be attended: q and k RMS-normed a head with
+ * q_gain / k_gain (dim), columns i and i + turned / 2 of the first `turned` turned together by their position's row of angles
+ * (cos and sin side by side, multiplied in as they are); v, with value_norm, over its root mean square a head.  q (rows, heads *
+ * dim); position p's key and value in row p of keys (slots, kv_heads, context, dim) and values (.., vdim). */
+int iron_cached_heads(const void* x, void* q, void* keys, void* values, const uint16_t* q_gain, const uint16_t* k_gain,
+                      const float* angles, const int* spans, int slots, int rows, int stride, int heads, int kv_heads, int dim,
+                      int vdim, int context, int turned, int angle_rows, int value_norm, float eps, int is_float,
+                      const int* valid, void* stream);
+/* Causal attention over such caches, the rows' own keys in them already: score = q . k * scale, with cap > 0 cap *
+ * tanh(score / cap); softmax, with `sink` one more in its denominator; the values' sums in columns out_at .. of y (rows of
+ * out_stride).  single: no span has more than one row.  workspace: of that many bytes (it may be none), 16-byte aligned. */
+int64_t iron_mha_global_workspace_bytes(int slots, int heads, int kv_heads, int vdim, int context, int single);
+int iron_mha_global(const void* q, const void* keys, const void* values, const int* spans, void* y, void* workspace, int slots,
+                    int rows, int heads, int kv_heads, int dim, int vdim, int context, float scale, float cap, int sink,
+                    int out_stride, int out_at, int single, int is_float, void* stream);
 
 /* One row's product with its input made and its output taken in the same launch, bf16; each computes what the entry
  * points above and iron_gemv_bf16 compute in turn.

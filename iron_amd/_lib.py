@@ -89,9 +89,18 @@ SIGNATURES = {
     "iron_sample_advance_bf16": (c_int, [_P, c_int, _P, c_int, _P, c_int, _P, _P, _P, c_int, _P, _P, _P, c_int, _P,
                                          c_int, _P]),
     "iron_gemm_few_bf16": (c_int, [_P, _P, _P, _P, c_int, c_int, c_int, c_int, _P]),
-    "iron_stream_embed": (c_int, [_P, _P, _P, _P, c_int, c_int, c_int, _P, _P]),
+    "iron_stream_embed": (c_int, [_P, _P, _P, _P, c_int, c_int, c_int, c_float, _P, _P]),
     "iron_stream_rows": (c_int, [_P] * 6 + [c_int, c_int, c_float, c_float, c_int, _P, _P]),
     "iron_stream_depth_rows": (c_int, [_P] * 6 + [c_int, c_int, _P, c_int, c_int, c_float, c_float, c_int, _P, _P]),
+    "iron_stream_groups": (c_int, [_P] * 5 + [c_int] * 3 + [c_float, c_float, c_int, _P, _P]),
+    "iron_gated_columns": (c_int, [_P, _P] + [c_int] * 7 + [c_float, c_int, _P, _P]),
+    "iron_hgrn2": (c_int, [_P] * 6 + [c_int] * 7 + [_P]),
+    "iron_hgrn2_workspace_bytes": (c_int64, [c_int] * 4),
+    "iron_hgrn2_chunked": (c_int, [_P] * 7 + [c_int] * 7 + [_P]),
+    "iron_decode_hgrn2_bf16": (c_int, [_P] * 7 + [c_int] * 8 + [c_float] + [c_int] * 4 + [c_float, _P]),
+    "iron_cached_heads": (c_int, [_P] * 8 + [c_int] * 11 + [c_float, c_int, _P, _P]),
+    "iron_mha_global_workspace_bytes": (c_int64, [c_int] * 6),
+    "iron_mha_global": (c_int, [_P] * 6 + [c_int] * 7 + [c_float, c_float] + [c_int] * 5 + [_P]),
     "iron_activation": (c_int, [_P, _P, c_int, c_int, c_int, c_int, _P, _P]),
     "iron_turned_heads": (c_int, [_P] * 9 + [c_int, c_int, _P] + [c_int] * 9 + [c_float, c_float, c_int, _P, _P]),
     "iron_mha_talking_workspace_bytes": (c_int64, [c_int] * 6),
@@ -100,9 +109,9 @@ SIGNATURES = {
     "iron_matrix_memory_workspace_bytes": (c_int64, [c_int] * 4),
     "iron_matrix_memory_chunked": (c_int, [_P] * 8 + [c_int] * 8 + [c_float, c_int, _P]),
     "iron_memory_gate": (c_int, [_P] * 4 + [c_int] * 5 + [c_float, c_float, c_int, _P, _P]),
-    "iron_router": (c_int, [_P] * 5 + [c_int] * 5 + [_P, _P]),
+    "iron_router": (c_int, [_P] * 4 + [c_int, _P, _P] + [c_int] * 5 + [_P, _P]),
     "iron_experts_workspace_bytes": (c_int64, [c_int] * 6),
-    "iron_experts": (c_int, [_P] * 8 + [c_int] * 7 + [_P, _P]),
+    "iron_experts": (c_int, [_P] * 8 + [c_int] * 8 + [_P, _P]),
     "iron_span_tails": (c_int, [_P, _P, _P, c_int, c_int, c_int, _P]),
     "iron_softcap": (c_int, [_P, _P, _P, c_int, c_int, c_int, c_float, c_float, c_int, _P]),
     "iron_stream_gated_rows": (c_int, [_P] * 5 + [c_int, c_int, _P, _P, c_int, c_int, c_float, c_int, _P, _P]),

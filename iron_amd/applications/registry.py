@@ -9,6 +9,7 @@ from .gemma4 import Gemma4
 from .granite import Granite
 from .llama import Llama
 from .pegilix import Pegilix
+from .pudinex import Pudinex
 from .pufuzen import Pufuzen
 from .tilarax import Tilarax
 
@@ -19,6 +20,7 @@ ARCHITECTURES = {
     "Gemma4ForCausalLM": Gemma4,
     "Gemma4ForConditionalGeneration": Gemma4,
     "Pegilix": Pegilix,
+    "Pudinex": Pudinex,
     "Pufuzen": Pufuzen,
     "Tilarax": Tilarax,
 }

@@ -317,7 +317,7 @@ def plan(recording, tensor: Callable[[Any], Any], word: Callable[[Any], Any],
         if _name(s) == "StreamNorm":
             g = steps[j + 1] if j + 1 < len(steps) else None
             h = s.outputs["y"]
-            if not (g is not None and s.op.rows == 1 and s.op.dtype is bfloat16 and s.op.cols % 8 == 0 and s.op.cols <= 16384 and bare(s)
+            if not (g is not None and s.op.rows == 1 and s.op.groups == 1 and s.op.dtype is bfloat16 and s.op.cols % 8 == 0 and s.op.cols <= 16384 and bare(s)
                     and gemv_row(g, h) and once(h)):
                 return None
             args = dict(W=tensor(g.inputs["A"]), x=tensor(s.inputs["x"]).reshape(-1), gain=tensor(s.inputs["weight"]),
@@ -723,7 +723,7 @@ def plan(recording, tensor: Callable[[Any], Any], word: Callable[[Any], Any],
             # a block's output into the stream and the next block's norm out of it: one pass over the row
             nm = steps[i + 1]
             if (_same_view(nm.inputs["x"], s.outputs["x"]) and nm.op.dtype is s.op.dtype
-                    and (nm.op.epsilon, nm.op.unit) == (s.op.epsilon, s.op.unit)
+                    and (nm.op.epsilon, nm.op.unit, nm.op.groups) == (s.op.epsilon, s.op.unit, 1)
                     and (nm.op.rows, nm.op.cols) == (s.op.rows, s.op.cols) and nm.values.get("valid") == s.values.get("valid")
                     and set(nm.values) <= {"valid"} and set(s.values) <= {"valid"}):
                 args = dict(x=tensor(s.inputs["x"]), y=tensor(s.inputs["y"]), back_gain=tensor(s.inputs["weight"]),
@@ -740,7 +740,7 @@ def plan(recording, tensor: Callable[[Any], Any], word: Callable[[Any], Any],
             # a block's gated output into the stream and the next block's norm out of it: one pass over the row
             nm = steps[i + 1]
             if (_same_view(nm.inputs["x"], s.outputs["x"]) and nm.op.dtype is s.op.dtype and (nm.op.rows, nm.op.cols) == (s.op.rows, s.op.cols)
-                    and nm.values.get("valid") == s.values.get("valid") and set(nm.values) <= {"valid"} and set(s.values) <= {"valid"}):
+                    and nm.op.groups == 1 and nm.values.get("valid") == s.values.get("valid") and set(nm.values) <= {"valid"} and set(s.values) <= {"valid"}):
                 args = dict(x=tensor(s.inputs["x"]), y=tensor(s.inputs["y"]), gate=tensor(s.inputs["gate"]), gate_bias=tensor(s.inputs["gate_bias"]),
                             h=tensor(nm.outputs["y"]), gain=tensor(nm.inputs["weight"]))
                 if "y_bias" in s.inputs:

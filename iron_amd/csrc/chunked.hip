@@ -1,4 +1,4 @@
-// Time mixing, the delta rule and the matrix memory over a prompt's portion, sixteen tokens at a time on float32 MFMAs.
+// Time mixing, the delta rule, the matrix memory and HGRN2 over a prompt's portion, sixteen tokens at a time on float32 MFMAs.
 //
 // Within a chunk of 16 tokens everything that does not touch the state depends on the chunk alone, so a
 // first launch computes it for all chunks at once: what earlier tokens of the chunk leave of themselves
@@ -14,6 +14,7 @@
 // Decays enter as exponentials of differences of running sums of logarithms, later minus earlier: never
 // above 1, however strong the decay.
 #include "../../include/iron_hip.h"
+#include "hgrn2.h"
 #include "matrix_memory.h"
 #include "rows.h"
 
@@ -234,6 +235,80 @@ __global__ __launch_bounds__(256) void time_mix_walk_kernel(const T* __restrict_
       const int i = (wave * NT + n) * 16 + quad * 4 + j;
       if (i < dim && col < cols) sp[(size_t)i * cols + col] = S[n][j];
     }
+}
+
+// ---------------------------------------------------------------------- HGRN2
+// The same walk, read behind the write: queries enter as q exp(L), L with the token's own decay in it, keys are what the gates
+// leave, and the 16 x 16 matrix has its diagonal, undecayed.
+template <typename T>
+__global__ __launch_bounds__(256) void hgrn2_chunks_kernel(const T* __restrict__ x, FadeGates g, const int* __restrict__ spans,
+                                                           float* __restrict__ work, int rows, int slots, int stride, int heads, int dim) {
+  extern __shared__ __align__(16) float lds[];
+  const int head = blockIdx.y, slot = blockIdx.z, base = blockIdx.x * CHUNK;
+  const Span s = span_of(spans, slot, rows);
+  if (base >= s.rows) return;
+  const int n = min(CHUNK, s.rows - base), tiles = (dim + 15) / 16, wide = tiles * 16, pitch = wide + 4, t = threadIdx.x;
+  float* qs = lds;                       // [16][pitch]
+  float* ks = qs + CHUNK * pitch;
+  float* ls = ks + CHUNK * pitch;        // the sum up to and with token i
+  float* am = ls + CHUNK * pitch;        // [16][17]
+  const T* row = x + (size_t)(s.row0 + base) * stride + head * dim;
+  for (int e = t; e < CHUNK * wide; e += 256) {
+    const int i = e / wide, c = e - i * wide;
+    float q = 0.f, k = 0.f, l = 0.f;   // past the last token: nothing read or written, nothing fades
+    if (i < n && c < dim) {
+      const T* at = row + (size_t)i * stride + c;
+      const Fade f = fade_of(load_one(at + heads * dim), bf16_to_f32(g.bias[head * dim + c]), bf16_to_f32(g.lower[head * dim + c]));
+      q = silu_read(load_one(at));
+      k = f.write;
+      l = log_fade(f);
+    }
+    qs[i * pitch + c] = q;
+    ks[i * pitch + c] = k;
+    ls[i * pitch + c] = l;
+  }
+  for (int e = t; e < CHUNK * 17; e += 256) am[e] = 0.f;
+  __syncthreads();
+  for (int c = t; c < wide; c += 256) {
+    float sum = 0.f;
+#pragma unroll
+    for (int i = 0; i < CHUNK; ++i) {
+      sum += ls[i * pitch + c];
+      ls[i * pitch + c] = sum;
+    }
+  }
+  __syncthreads();
+  float* out = work + ((size_t)(first_chunk(spans, slots, slot, rows, CHUNK) + blockIdx.x) * heads + head) * mix_words(tiles);
+  const float* end = ls + (CHUNK - 1) * pitch;
+  for (int e = t; e < tiles * 64; e += 256) {
+    const int tile = e >> 6, lane = e & 63, l16 = lane & 15, quad = lane >> 4, c = tile * 16 + l16;
+    const float4 q = *reinterpret_cast<const float4*>(qs + l16 * pitch + tile * 16 + quad * 4), l = *reinterpret_cast<const float4*>(ls + l16 * pitch + tile * 16 + quad * 4);
+    float f[4];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) f[j] = ks[(quad * 4 + j) * pitch + c] * decay_exp<T>(end[c] - ls[(quad * 4 + j) * pitch + c]);
+    reinterpret_cast<float4*>(out)[e] = make_float4(q.x * decay_exp<T>(l.x), q.y * decay_exp<T>(l.y), q.z * decay_exp<T>(l.z), q.w * decay_exp<T>(l.w));
+    reinterpret_cast<float4*>(out + tiles * 256)[e] = make_float4(f[0], f[1], f[2], f[3]);
+  }
+  for (int c = t; c < wide; c += 256) out[tiles * 512 + c] = decay_exp<T>(end[c]);
+  // Pairs (i, j), j <= i: 64 at a time, four threads a pair.
+  for (int p = t >> 2; p < CHUNK * (CHUNK + 1) / 2; p += 64) {
+    int i = 0, j = p;
+    while (j > i) j -= ++i;
+    float sum = 0.f;
+    for (int c = (t & 3) * 4; c < wide; c += 16) {
+      const float4 q = *reinterpret_cast<const float4*>(qs + i * pitch + c), k = *reinterpret_cast<const float4*>(ks + j * pitch + c);
+      const float4 a = *reinterpret_cast<const float4*>(ls + i * pitch + c), b = *reinterpret_cast<const float4*>(ls + j * pitch + c);
+      sum = fmaf(q.x * k.x, decay_exp<T>(a.x - b.x), sum);
+      sum = fmaf(q.y * k.y, decay_exp<T>(a.y - b.y), sum);
+      sum = fmaf(q.z * k.z, decay_exp<T>(a.z - b.z), sum);
+      sum = fmaf(q.w * k.w, decay_exp<T>(a.w - b.w), sum);
+    }
+    sum += IRON_DPP(0.f, sum, 0xB1, 0xF);
+    sum += IRON_DPP(0.f, sum, 0x4E, 0xF);
+    if ((t & 3) == 0) am[i * 17 + j] = sum;
+  }
+  __syncthreads();
+  out[tiles * 528 + t] = am[((t >> 2) & 15) * 17 + (t >> 6) * 4 + (t & 3)];
 }
 
 // ----------------------------------------------------------- the matrix memory
@@ -626,6 +701,39 @@ extern "C" int iron_time_mix_chunked(const void* r, const void* k, const void* v
   else { IRON_MIX(bf16_t) }
 #undef IRON_MIX
 #undef IRON_MIX_WALK
+  IRON_LAUNCH_CHECK();
+}
+
+extern "C" int64_t iron_hgrn2_workspace_bytes(int slots, int rows, int heads, int dim) {
+  return chunks_of(rows, slots, CHUNK) * heads * (int64_t)mix_words((dim + 15) / 16) * 4;
+}
+
+extern "C" int iron_hgrn2_chunked(const void* x, const uint16_t* f_bias, const uint16_t* lower, float* state, const int* spans, float* o, void* workspace,
+                                  int slots, int rows, int stride, int heads, int dim, int vdim, int is_float, void* stream) {
+  IRON_REQUIRE(x && f_bias && lower && state && o && workspace, "hgrn2_chunked: null operand");
+  IRON_CHUNKED_REQUIRE("hgrn2_chunked");
+  IRON_REQUIRE(heads > 0 && heads <= 65535 && dim > 0 && dim <= 256 && vdim > 0, "hgrn2_chunked: heads (%d) and vdim (%d) positive, dim (%d) from 1 to 256",
+               heads, vdim, dim);
+  IRON_REQUIRE(stride >= heads * (2 * dim + vdim), "hgrn2_chunked: a row of %d holds no q, f and v of %d heads", stride, heads);
+  IRON_REQUIRE(((uintptr_t)workspace & 15) == 0, "hgrn2_chunked: the workspace must be 16-byte aligned");
+  IRON_REQUIRE((long)rows * stride < (1L << 28) && (long)rows * heads * vdim < (1L << 28), "hgrn2_chunked: the batch's rows are addressed with 32-bit offsets");
+  hipStream_t s = (hipStream_t)stream;
+  const int tiles = (dim + 15) / 16, pitch = tiles * 16 + 4;
+  const size_t lds = ((size_t)3 * CHUNK * pitch + CHUNK * 17) * 4;
+  const dim3 all((rows + CHUNK - 1) / CHUNK, heads, slots), walk(heads, (vdim + 15) / 16, slots);
+  float* work = (float*)workspace;
+  const FadeGates g{f_bias, lower};
+  const WalkShape shape{rows, slots, heads, dim, vdim, stride, heads * vdim};
+#define IRON_FADE_WALK(T, NT, DEPTH)   hipLaunchKernelGGL((time_mix_walk_kernel<T, NT, DEPTH>), walk, dim3(256), 0, s, (const T*)x + 2 * heads * dim, state, spans, work, o, shape)
+#define IRON_FADE(T)                                                                                                                        \
+  hipLaunchKernelGGL((hgrn2_chunks_kernel<T>), all, dim3(256), lds, s, (const T*)x, g, spans, work, rows, slots, stride, heads, dim);      \
+  if (tiles <= 4) IRON_FADE_WALK(T, 1, 6);                                                                                                  \
+  else if (tiles <= 8) IRON_FADE_WALK(T, 2, 4);                                                                                             \
+  else IRON_FADE_WALK(T, 4, 2);
+  if (is_float) { IRON_FADE(float) }
+  else { IRON_FADE(bf16_t) }
+#undef IRON_FADE
+#undef IRON_FADE_WALK
   IRON_LAUNCH_CHECK();
 }
 

@@ -3,6 +3,7 @@
 //   decode_parallel: low-rank decay, time-mixing step, head norm and gate (a block a head)
 //                    beside sliding-window attention with its distance bias (a block a query head)
 //   decode_delta:    short convolution, unit q and k, gated delta rule, head norm and gate
+//   decode_hgrn2:    forget gate, fading memory, head norm (a block a head) beside a feed-forward's gated columns
 //
 // bf16 rows, float32 inside.  A block is 16 waves.  A head's state (dim rows of `wide` columns, wide a power
 // of two from 16 to 256) is read once, four columns a thread, and kept in registers until it is replaced;
@@ -10,7 +11,7 @@
 // shuffles, across the waves through LDS.  Blocks of one slot read states that none of them replaces:
 // rings with a row to spare (see the prompt kernels, whose layouts these are).
 #include "../../include/iron_hip.h"
-#include "rows.h"
+#include "hgrn2.h"
 
 namespace iron {
 
@@ -495,6 +496,83 @@ __global__ __launch_bounds__(DM_THREADS) void decode_delta_kernel(DeltaStep a, c
   finish_head(sh.o, vdim, HeadOut{row + a.gate_at + head * vdim, a.norm, a.out + ((size_t)s.row0 * a.heads + head) * vdim, a.eps, 1.f}, sh.part[3]);
 }
 
+// ---------------------------------------------------------------------- HGRN2
+struct FadeStep {
+  const bf16_t* x;                        // (slots, stride): q, f, v
+  FadeGates g;
+  const bf16_t* norm;                     // (vdim)
+  float* state;                           // (slots, heads, dim, vdim)
+  bf16_t* out;                            // (slots, out_stride), from out_at
+  int stride, heads, dim, vdim, out_stride, out_at;
+  float eps;
+  int cols, gate_at, gated_at, kind;      // gated columns of the same rows: how many, where from, where to
+  float limit;
+};
+struct FadeShared {
+  float q[256], keep[256], write[256], v[256];
+  float sums[DM_WAVES][256];
+  float part[DM_WAVES];
+};
+
+template <int NR>
+__global__ __launch_bounds__(DM_THREADS) void decode_hgrn2_kernel(FadeStep a, const int* __restrict__ spans, int rows) {
+  __shared__ __align__(16) FadeShared sh;
+  const int slot = blockIdx.y, head = blockIdx.x, t = threadIdx.x;
+  const Span s = span_of(spans, slot, rows);
+  if (s.rows == 0) return;
+  const bf16_t* row = a.x + (size_t)s.row0 * a.stride;
+  bf16_t* to = a.out + (size_t)s.row0 * a.out_stride;
+  if (head >= a.heads) {
+    const int c = (head - a.heads) * DM_THREADS + t;
+    if (c < a.cols)
+      to[a.gated_at + c] = f32_to_bf16(gated_value(a.kind, a.limit, bf16_to_f32(row[a.gate_at + c]), bf16_to_f32(row[a.gate_at + a.cols + c])));
+    return;
+  }
+  const int lane = t & 63, wave = t >> 6, dim = a.dim, vdim = a.vdim;
+  const StateTiles tile(vdim);
+  float* sp = a.state + ((size_t)slot * a.heads + head) * dim * vdim;
+  float4 S[NR];
+#pragma unroll
+  for (int n = 0; n < NR; ++n) {
+    const int i = tile.row + n * tile.stride;
+    S[n] = (s.start > 0 && i < dim) ? *reinterpret_cast<const float4*>(sp + (size_t)i * vdim + tile.col) : make_float4(0.f, 0.f, 0.f, 0.f);
+  }
+  const float gain = t < vdim ? bf16_to_f32(a.norm[t]) : 0.f;
+  if (t < dim) {
+    const int c = head * dim + t;
+    const Fade f = fade_of(bf16_to_f32(row[a.heads * dim + c]), bf16_to_f32(a.g.bias[c]), bf16_to_f32(a.g.lower[c]));
+    sh.q[t] = silu_read(bf16_to_f32(row[c]));
+    sh.keep[t] = f.keep;
+    sh.write[t] = f.write;
+  } else if (t >= 512 && t < 512 + vdim) {
+    sh.v[t - 512] = bf16_to_f32(row[2 * a.heads * dim + head * vdim + t - 512]);
+  }
+  __syncthreads();
+  const float4 v = *reinterpret_cast<const float4*>(&sh.v[tile.col]);
+  float4 o = make_float4(0.f, 0.f, 0.f, 0.f);
+#pragma unroll
+  for (int n = 0; n < NR; ++n) {
+    const int i = tile.row + n * tile.stride;
+    if (i < dim) {
+      const float q = sh.q[i], k = sh.write[i], w = sh.keep[i];
+      S[n].x = fmaf(w, S[n].x, k * v.x); S[n].y = fmaf(w, S[n].y, k * v.y);
+      S[n].z = fmaf(w, S[n].z, k * v.z); S[n].w = fmaf(w, S[n].w, k * v.w);
+      o.x = fmaf(q, S[n].x, o.x); o.y = fmaf(q, S[n].y, o.y); o.z = fmaf(q, S[n].z, o.z); o.w = fmaf(q, S[n].w, o.w);
+      *reinterpret_cast<float4*>(sp + (size_t)i * vdim + tile.col) = S[n];
+    }
+  }
+  tile.fold(o);
+  if (lane < tile.quads) *reinterpret_cast<float4*>(&sh.sums[wave][tile.col]) = o;
+  __syncthreads();
+  float sum = 0.f;
+  if (t < vdim) {
+#pragma unroll
+    for (int w = 0; w < DM_WAVES; ++w) sum += sh.sums[w][t];
+  }
+  const float inv = 1.0f / sqrtf(dm_block_sum(sum * sum, sh.part) / (float)vdim + a.eps);
+  if (t < vdim) to[a.out_at + head * vdim + t] = f32_to_bf16(sum * inv * gain);
+}
+
 static bool whole_columns(int n) { return n >= 16 && n <= 256 && (n & (n - 1)) == 0; }
 static int rows_a_thread(int dim, int wide) {   // the power of two that covers dim over the block's rows
   const int stride = DM_THREADS / (wide / 4);
@@ -577,5 +655,35 @@ extern "C" int iron_decode_delta_bf16(const uint16_t* x, const uint16_t* taps_w,
     default: IRON_DELTA_STEP(16)
   }
 #undef IRON_DELTA_STEP
+  IRON_LAUNCH_CHECK();
+}
+
+extern "C" int iron_decode_hgrn2_bf16(const uint16_t* x, const uint16_t* f_bias, const uint16_t* lower, const uint16_t* norm, float* state,
+                                      const int* spans, uint16_t* out, int slots, int rows, int stride, int heads, int dim, int vdim, int out_stride,
+                                      int out_at, float eps, int cols, int gate_at, int gated_at, int kind, float limit, void* stream) {
+  IRON_REQUIRE(x && f_bias && lower && norm && state && spans && out, "decode_hgrn2: null operand");
+  IRON_REQUIRE(((uintptr_t)spans & 15) == 0 && ((uintptr_t)state & 15) == 0, "decode_hgrn2: spans and state must be 16-byte aligned");
+  IRON_REQUIRE(slots > 0 && slots <= 65535 && rows > 0, "decode_hgrn2: slots (%d) and rows (%d) must be positive", slots, rows);
+  IRON_REQUIRE(heads > 0 && dim > 0 && dim <= 256 && whole_columns(vdim), "decode_hgrn2: dim (%d) up to 256, vdim (%d) a power of two from 16 to 256", dim, vdim);
+  IRON_REQUIRE(stride >= heads * (2 * dim + vdim) && out_at >= 0 && out_at + heads * vdim <= out_stride,
+               "decode_hgrn2: rows of %d and %d for %d heads of %d and %d", stride, out_stride, heads, dim, vdim);
+  IRON_REQUIRE(cols >= 0 && (cols == 0 || (gate_at >= 0 && gate_at + 2 * cols <= stride && gated_at >= 0 && gated_at + cols <= out_stride)),
+               "decode_hgrn2: twice %d gated columns from %d, into those from %d", cols, gate_at, gated_at);
+  IRON_REQUIRE(kind >= 0 && kind <= 3, "decode_hgrn2: kind (%d) is 0 to 3", kind);
+  const FadeStep a{x, FadeGates{f_bias, lower}, norm, state, out, stride, heads, dim, vdim, out_stride, out_at, eps, cols, gate_at, gated_at, kind, limit};
+  const dim3 grid(heads + (cols + DM_THREADS - 1) / DM_THREADS, slots);
+#define IRON_FADE_STEP(NR)                                                                                           \
+  {                                                                                                                  \
+    hipLaunchKernelGGL((decode_hgrn2_kernel<NR>), grid, dim3(DM_THREADS), 0, (hipStream_t)stream, a, spans, rows);   \
+    break;                                                                                                           \
+  }
+  switch (rows_a_thread(dim, vdim)) {
+    case 1: IRON_FADE_STEP(1)
+    case 2: IRON_FADE_STEP(2)
+    case 4: IRON_FADE_STEP(4)
+    case 8: IRON_FADE_STEP(8)
+    default: IRON_FADE_STEP(16)
+  }
+#undef IRON_FADE_STEP
   IRON_LAUNCH_CHECK();
 }

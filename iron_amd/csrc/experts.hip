@@ -1,5 +1,6 @@
 // A feed-forward of routed experts: each row's `top` experts by its router's logits, shares by a softmax over the chosen
-// ones, and the shares' sum of what they make of the row, down (act(gate h) * (up h)).
+// ones -- or by a softmax over all, chosen by scores with corrections and shared by those without -- and the shares' sum of
+// what they make of the row, down (act(gate h) * (up h)).  Ids behind the experts' last are identities: they hand on the row.
 //
 //   router:   float32 logits, a row a block
 //   pairs:    a (row, chosen expert) at a time, or all of an expert's at once, the weights' rows dealt to waves (few rows; either type)
@@ -45,11 +46,55 @@ __device__ __forceinline__ void choose(float* __restrict__ z, int n, int top, in
   if (lane < top) shares[lane] = mine / total;
 }
 
+// The `top` largest of the n scores (a softmax over the logits z) plus corrections by one wave, in order, the first of equal ones
+// first; their shares, the scores over their sum.  z and by: LDS.
+__device__ __forceinline__ void choose_scored(float* __restrict__ z, float* __restrict__ by, const bf16_t* __restrict__ correction, int n, int top,
+                                              int* __restrict__ ids, float* __restrict__ shares) {
+  const int lane = threadIdx.x & 63;
+  float most = -INFINITY, total = 0.f;
+  for (int i = lane; i < n; i += 64) most = fmaxf(most, z[i]);
+  most = wave_max(most);
+  for (int i = lane; i < n; i += 64) total += expf(z[i] - most);
+  total = wave_sum(total);
+  for (int i = lane; i < n; i += 64) {   // (a lane reads what it wrote)
+    z[i] = expf(z[i] - most) / total;
+    by[i] = z[i] + (correction != nullptr ? bf16_to_f32(correction[i]) : 0.f);
+  }
+  float sum = 0.f, mine = 0.f;
+  for (int k = 0; k < top; ++k) {
+    float best = -INFINITY, score = 0.f;
+    int at = n;
+    for (int i = lane; i < n; i += 64)
+      if (by[i] > best) {
+        best = by[i];
+        score = z[i];
+        at = i;
+      }
+    const float largest = wave_max(best);
+    int id = n, from = 0;
+    for (unsigned long long left = __builtin_amdgcn_ballot_w64(best == largest && at < n); left != 0; left &= left - 1) {
+      const int l = __builtin_ctzll(left), other = __shfl(at, l, 64);
+      if (other < id) {
+        id = other;
+        from = l;
+      }
+    }
+    score = __shfl(score, from, 64);
+    if (id >= n) id = 0;   // (none that is a number: the first)
+    sum += score;
+    if (lane == k) mine = score;
+    if (lane == 0) ids[k] = id;
+    if (lane == (id & 63)) by[id] = -INFINITY;
+  }
+  if (lane < top) shares[lane] = mine / (sum + 1e-20f);
+}
+
 template <typename T, int VEC, int NW>
 __global__ __launch_bounds__(NW * 64) void router_kernel(const T* __restrict__ h, const bf16_t* __restrict__ w, const bf16_t* __restrict__ bias,
-                                                     int* __restrict__ ids, float* __restrict__ shares, int rows, int cols, int experts,
-                                                     int top, const int* __restrict__ valid) {
-  __shared__ float z[ROUTER_MAX];
+                                                     const bf16_t* __restrict__ correction, int scored, int* __restrict__ ids,
+                                                     float* __restrict__ shares, int rows, int cols, int experts, int top,
+                                                     const int* __restrict__ valid) {
+  __shared__ float z[ROUTER_MAX], by[ROUTER_MAX];
   const int row = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   if (row >= bound_or(valid, rows)) return;
   const T* hr = h + (size_t)row * cols;
@@ -65,15 +110,20 @@ __global__ __launch_bounds__(NW * 64) void router_kernel(const T* __restrict__ h
       for (int j = 0; j < VEC; ++j) sum = fmaf(a[j], b[j], sum);
     }
     sum = wave_sum(sum);
-    if (lane == 0) z[e] = sum + bf16_to_f32(bias[e]);
+    if (lane == 0) z[e] = sum + (bias != nullptr ? bf16_to_f32(bias[e]) : 0.f);
   }
   __syncthreads();
-  if (wave == 0) choose(z, experts, top, ids + (size_t)row * top, shares + (size_t)row * top);
+  if (wave != 0) return;
+  if (scored) choose_scored(z, by, correction, experts, top, ids + (size_t)row * top, shares + (size_t)row * top);
+  else choose(z, experts, top, ids + (size_t)row * top, shares + (size_t)row * top);
 }
 
 __device__ __forceinline__ float act_exact(int kind, float g) {
   return kind == 3 ? fmaxf(g, 0.f) : (kind == 1 ? g / (1.f + expf(-g)) : gelu_tanh_f32(g));
 }
+
+// The expert an id names, -1 for one of the identities behind the last.
+__device__ __forceinline__ int expert_of(int id, int experts, int identity) { return identity > 0 && id >= experts ? -1 : min(max(id, 0), experts - 1); }
 
 // VEC elements of a row and of a weight's row, and their product: bf16 pairs as they were loaded, or floats.
 template <typename T, int VEC>
@@ -106,10 +156,12 @@ __device__ __forceinline__ float add_product(const Run<T, VEC>& a, const Run<T, 
 template <typename T, int VEC>
 __global__ __launch_bounds__(256) void expert_pairs_kernel(const T* __restrict__ h, const bf16_t* __restrict__ gate, const bf16_t* __restrict__ up,
                                                            const int* __restrict__ ids, T* __restrict__ a, int rows, int cols, int ff, int experts,
-                                                           int top, int kind, const int* __restrict__ valid) {
+                                                           int identity, int top, int kind, const int* __restrict__ valid) {
   const int lane = threadIdx.x & 63, f = blockIdx.x * 4 + (threadIdx.x >> 6), pairs = f < ff ? bound_or(valid, rows) * top : 0;
   for (int pair = blockIdx.y; pair < pairs; pair += gridDim.y) {
-    const size_t at = ((size_t)min(max(ids[pair], 0), experts - 1) * ff + f) * cols;
+    const int e = expert_of(ids[pair], experts, identity);
+    if (e < 0) continue;
+    const size_t at = ((size_t)e * ff + f) * cols;
     const T* hr = h + (size_t)(pair / top) * cols;
     float g = 0.f, u = 0.f;
 #pragma unroll 4
@@ -162,13 +214,13 @@ __device__ __forceinline__ void expert_rows(const T* __restrict__ h, const bf16_
 template <typename T, int VEC>
 __global__ __launch_bounds__(256) void expert_shared_kernel(const T* __restrict__ h, const bf16_t* __restrict__ gate, const bf16_t* __restrict__ up,
                                                             const int* __restrict__ ids, T* __restrict__ a, int rows, int cols, int ff,
-                                                            int experts, int top, int kind, const int* __restrict__ valid) {
+                                                            int experts, int identity, int top, int kind, const int* __restrict__ valid) {
   __shared__ int list[SHARED_PAIRS], held;
   const int e = blockIdx.y, f = blockIdx.x * 4 + (threadIdx.x >> 6), pairs = bound_or(valid, rows) * top;
   if (threadIdx.x == 0) held = 0;
   __syncthreads();
   for (int p = threadIdx.x; p < pairs; p += 256)
-    if (min(max(ids[p], 0), experts - 1) == e) list[atomicAdd(&held, 1)] = p;
+    if (expert_of(ids[p], experts, identity) == e) list[atomicAdd(&held, 1)] = p;
   __syncthreads();
   const int n = held;
   if (n == 0 || f >= ff) return;
@@ -183,8 +235,8 @@ __global__ __launch_bounds__(256) void expert_shared_kernel(const T* __restrict_
 // y[row] = sum over its experts of share * down_e a[pair]: a block PER rows of down, a wave every fourth of the experts.
 template <typename T, int VEC, int PER>
 __global__ __launch_bounds__(256) void expert_sums_kernel(const T* __restrict__ a, const bf16_t* __restrict__ down, const int* __restrict__ ids,
-                                                          const float* __restrict__ shares, T* __restrict__ y, int rows, int cols, int ff,
-                                                          int experts, int top, const int* __restrict__ valid) {
+                                                          const float* __restrict__ shares, const T* __restrict__ h, T* __restrict__ y, int rows,
+                                                          int cols, int ff, int experts, int identity, int top, const int* __restrict__ valid) {
   __shared__ float red[4][PER];
   const int row = blockIdx.y, lane = threadIdx.x & 63, wave = threadIdx.x >> 6, c0 = blockIdx.x * PER;
   if (row >= bound_or(valid, rows)) return;
@@ -192,8 +244,14 @@ __global__ __launch_bounds__(256) void expert_sums_kernel(const T* __restrict__ 
 #pragma unroll
   for (int p = 0; p < PER; ++p) sum[p] = 0.f;
   for (int k = wave; k < top; k += 4) {
-    const int pair = row * top + k, e = min(max(ids[pair], 0), experts - 1);
+    const int pair = row * top + k, e = expert_of(ids[pair], experts, identity);
     const float share = shares[pair];
+    if (e < 0) {
+      if (lane == 0)
+#pragma unroll
+        for (int p = 0; p < PER; ++p) sum[p] = fmaf(share, load_one(h + (size_t)row * cols + min(c0 + p, cols - 1)), sum[p]);
+      continue;
+    }
     const T* ar = a + (size_t)pair * ff;
     const bf16_t* dr[PER];
     float part[PER];
@@ -243,14 +301,17 @@ struct GroupedPlan {
 
 // One block: how many pairs each expert has, where its tiles begin, and every pair's place.
 __global__ __launch_bounds__(1024) void expert_plan_kernel(const int* __restrict__ ids, int* __restrict__ count, int* __restrict__ which,
-                                                           int* __restrict__ place, int* __restrict__ rows_of, int rows, int experts, int top,
-                                                           int most, const int* __restrict__ valid) {
+                                                           int* __restrict__ place, int* __restrict__ rows_of, int rows, int experts, int identity,
+                                                           int top, int most, const int* __restrict__ valid) {
   __shared__ int held[ROUTER_MAX], first[ROUTER_MAX], scan[2][ROUTER_MAX];
   const int t = threadIdx.x, pairs = bound_or(valid, rows) * top;
   held[t] = 0;
   for (int i = t; i < most * 128; i += 1024) rows_of[i] = 0;   // a tile's places past its expert's pairs
   __syncthreads();
-  for (int p = t; p < pairs; p += 1024) atomicAdd(&held[min(max(ids[p], 0), experts - 1)], 1);
+  for (int p = t; p < pairs; p += 1024) {
+    const int e = expert_of(ids[p], experts, identity);
+    if (e >= 0) atomicAdd(&held[e], 1);
+  }
   __syncthreads();
   const int tiles = (held[t] + 127) / 128;
   scan[0][t] = tiles;
@@ -267,7 +328,10 @@ __global__ __launch_bounds__(1024) void expert_plan_kernel(const int* __restrict
   if (t == 0) *count = min(scan[at][ROUTER_MAX - 1], most);
   __syncthreads();
   for (int p = t; p < pairs; p += 1024) {
-    const int to = min(atomicAdd(&first[min(max(ids[p], 0), experts - 1)], 1), most * 128 - 1);
+    const int e = expert_of(ids[p], experts, identity);
+    place[p] = -1;
+    if (e < 0) continue;
+    const int to = min(atomicAdd(&first[e], 1), most * 128 - 1);
     place[p] = to;
     rows_of[to] = p / top;
   }
@@ -275,8 +339,8 @@ __global__ __launch_bounds__(1024) void expert_plan_kernel(const int* __restrict
 
 // y[row] = sum over its pairs of share * what the pair's expert left.
 __global__ __launch_bounds__(256) void expert_gather_kernel(const bf16_t* __restrict__ outs, const int* __restrict__ place,
-                                                            const float* __restrict__ shares, bf16_t* __restrict__ y, int rows, int cols,
-                                                            int top, const int* __restrict__ valid) {
+                                                            const float* __restrict__ shares, const bf16_t* __restrict__ h, bf16_t* __restrict__ y,
+                                                            int rows, int cols, int top, const int* __restrict__ valid) {
   const int row = blockIdx.y, c = (blockIdx.x * 256 + threadIdx.x) * 8;
   if (row >= bound_or(valid, rows) || c >= cols) return;
   float sum[8];
@@ -285,7 +349,8 @@ __global__ __launch_bounds__(256) void expert_gather_kernel(const bf16_t* __rest
 #pragma unroll 4
   for (int k = 0; k < top; ++k) {
     float f[8];
-    load_vec<8>(outs + (size_t)place[row * top + k] * cols + c, f);
+    const int from = place[row * top + k];
+    load_vec<8>((from < 0 ? h + (size_t)row * cols : outs + (size_t)from * cols) + c, f);
     const float share = shares[row * top + k];
 #pragma unroll
     for (int j = 0; j < 8; ++j) sum[j] = fmaf(share, f[j], sum[j]);
@@ -300,9 +365,9 @@ static bool grouped_pays(int rows, int cols, int ff, int is_float) { return !is_
 
 using namespace iron;
 
-extern "C" int iron_router(const void* h, const uint16_t* w, const uint16_t* bias, int* ids, float* shares, int rows, int cols, int experts,
-                           int top, int is_float, const int* valid, void* stream) {
-  IRON_REQUIRE(h && w && bias && ids && shares, "router: null operand");
+extern "C" int iron_router(const void* h, const uint16_t* w, const uint16_t* bias, const uint16_t* correction, int scored, int* ids, float* shares,
+                           int rows, int cols, int experts, int top, int is_float, const int* valid, void* stream) {
+  IRON_REQUIRE(h && w && ids && shares && (scored || correction == nullptr), "router: null operand, or corrections of no scores");
   IRON_REQUIRE(rows > 0 && cols > 0 && experts > 0 && experts <= ROUTER_MAX, "router: rows (%d), cols (%d) positive, experts (%d) from 1 to %d",
                rows, cols, experts, ROUTER_MAX);
   IRON_REQUIRE(top > 0 && top <= experts && top <= 64, "router: top (%d) from 1 to the experts (%d), 64 at most", top, experts);
@@ -311,10 +376,10 @@ extern "C" int iron_router(const void* h, const uint16_t* w, const uint16_t* bia
 #define IRON_ROUTER(T, VEC)                                                                                                                \
   {                                                                                                                                        \
     if (rows < 256)                                                                                                                        \
-      hipLaunchKernelGGL((router_kernel<T, VEC, 16>), dim3(rows), dim3(1024), 0, (hipStream_t)stream, (const T*)h, w, bias, ids, shares,   \
+      hipLaunchKernelGGL((router_kernel<T, VEC, 16>), dim3(rows), dim3(1024), 0, (hipStream_t)stream, (const T*)h, w, bias, correction, scored, ids, shares,   \
                          rows, cols, experts, top, valid);                                                                                 \
     else                                                                                                                                   \
-      hipLaunchKernelGGL((router_kernel<T, VEC, 4>), dim3(rows), dim3(256), 0, (hipStream_t)stream, (const T*)h, w, bias, ids, shares,     \
+      hipLaunchKernelGGL((router_kernel<T, VEC, 4>), dim3(rows), dim3(256), 0, (hipStream_t)stream, (const T*)h, w, bias, correction, scored, ids, shares,     \
                          rows, cols, experts, top, valid);                                                                                 \
   }
   if (is_float) { if (vec) IRON_ROUTER(float, 8) else IRON_ROUTER(float, 1) }
@@ -329,11 +394,11 @@ extern "C" int64_t iron_experts_workspace_bytes(int rows, int cols, int ff, int 
 }
 
 extern "C" int iron_experts(const void* h, const uint16_t* gate, const uint16_t* up, const uint16_t* down, const int* ids, const float* shares,
-                            void* y, void* workspace, int rows, int cols, int ff, int experts, int top, int activation, int is_float,
+                            void* y, void* workspace, int rows, int cols, int ff, int experts, int identity, int top, int activation, int is_float,
                             const int* valid, void* stream) {
   IRON_REQUIRE(h && gate && up && down && ids && shares && y && workspace, "experts: null operand");
-  IRON_REQUIRE(rows > 0 && cols > 0 && ff > 0 && experts > 0 && top > 0 && top <= experts, "experts: sizes must be positive, top (%d) of %d experts",
-               top, experts);
+  IRON_REQUIRE(rows > 0 && cols > 0 && ff > 0 && experts > 0 && identity >= 0 && top > 0 && top <= experts + identity,
+               "experts: sizes must be positive, top (%d) of %d experts and %d identities", top, experts, identity);
   IRON_REQUIRE(activation >= 1 && activation <= 3, "experts: activation (%d) is 1 (SiLU), 2 (GELU, tanh form) or 3 (ReLU)", activation);
   hipStream_t s = (hipStream_t)stream;
   if (grouped_pays(rows, cols, ff, is_float)) {
@@ -346,10 +411,10 @@ extern "C" int iron_experts(const void* h, const uint16_t* gate, const uint16_t*
     int *count = (int*)w, *which = (int*)(w + p.which), *place = (int*)(w + p.place), *rows_of = (int*)(w + p.rows);
     const GroupedTiles g{count, which, p.most};
     bf16_t *acts = (bf16_t*)(w + p.acts), *outs = (bf16_t*)(w + p.outs);
-    hipLaunchKernelGGL(expert_plan_kernel, dim3(1), dim3(1024), 0, s, ids, count, which, place, rows_of, rows, experts, top, p.most, valid);
+    hipLaunchKernelGGL(expert_plan_kernel, dim3(1), dim3(1024), 0, s, ids, count, which, place, rows_of, rows, experts, identity, top, p.most, valid);
     if (int e = launch_grouped_pair((const bf16_t*)h, gate, up, acts, ff, cols, g, rows_of, activation, s)) return e;
     if (int e = launch_grouped(acts, down, outs, cols, ff, g, s)) return e;
-    hipLaunchKernelGGL(expert_gather_kernel, dim3((cols + 2047) / 2048, rows), dim3(256), 0, s, outs, place, shares, (bf16_t*)y, rows, cols, top, valid);
+    hipLaunchKernelGGL(expert_gather_kernel, dim3((cols + 2047) / 2048, rows), dim3(256), 0, s, outs, place, shares, (const bf16_t*)h, (bf16_t*)y, rows, cols, top, valid);
     IRON_LAUNCH_CHECK();
   }
   IRON_REQUIRE(rows <= 65535 && (long)rows * top <= (1 << 30), "experts: %d rows of %d experts exceed the grid's y extent", rows, top);
@@ -360,12 +425,12 @@ extern "C" int iron_experts(const void* h, const uint16_t* gate, const uint16_t*
   {                                                                                                                                           \
     if (rows > 1 && rows * top <= SHARED_PAIRS && experts <= 65535)                                                                           \
       hipLaunchKernelGGL((expert_shared_kernel<T, VEC>), dim3((ff + 3) / 4, experts), dim3(256), 0, s, (const T*)h, gate, up, ids,            \
-                         (T*)workspace, rows, cols, ff, experts, top, activation, valid);                                                     \
+                         (T*)workspace, rows, cols, ff, experts, identity, top, activation, valid);                                                     \
     else                                                                                                                                      \
       hipLaunchKernelGGL((expert_pairs_kernel<T, VEC>), dim3((ff + 3) / 4, pairs_y), dim3(256), 0, s, (const T*)h, gate, up, ids,          \
-                         (T*)workspace, rows, cols, ff, experts, top, activation, valid);                                                     \
+                         (T*)workspace, rows, cols, ff, experts, identity, top, activation, valid);                                                     \
     hipLaunchKernelGGL((expert_sums_kernel<T, VEC, 2>), dim3((cols + 1) / 2, rows), dim3(256), 0, s, (const T*)workspace, down, ids, shares, \
-                       (T*)y, rows, cols, ff, experts, top, valid);                                                                           \
+                       (const T*)h, (T*)y, rows, cols, ff, experts, identity, top, valid);                                                                           \
   }
   if (is_float) { if (vec) IRON_PAIRS(float, 8) else IRON_PAIRS(float, 1) }
   else { if (vec) IRON_PAIRS(bf16_t, 8) else IRON_PAIRS(bf16_t, 1) }

@@ -403,7 +403,7 @@ __global__ __launch_bounds__(256) void delta_rule_kernel(const float* __restrict
 }
 
 // ------------------------------------------------------- per-head norm, gate
-// out = (o / rms(o)) * gain * silu(gate) * scale, the mean over one head's columns.
+// out = (o / rms(o)) * gain * silu(gate) * scale, the mean over one head's columns; without a gate, that factor is 1.
 // LANES lanes to a head's row of up to 4 LANES columns, four a lane where VEC (else one of every LANES).
 template <typename T, int LANES, bool VEC>
 __global__ __launch_bounds__(256) void head_gate_kernel(const float* __restrict__ o, const T* __restrict__ gate,
@@ -423,7 +423,9 @@ __global__ __launch_bounds__(256) void head_gate_kernel(const float* __restrict_
   if (VEC && c0 < dim) {
     const float4 v = *reinterpret_cast<const float4*>(src + c0);
     f[0] = v.x; f[1] = v.y; f[2] = v.z; f[3] = v.w;
-    if constexpr (sizeof(T) == 2) {
+    if (gate == nullptr) {
+      z[0] = z[1] = z[2] = z[3] = 0.f;
+    } else if constexpr (sizeof(T) == 2) {
       const uint2 w = *reinterpret_cast<const uint2*>(gr + c0);
       z[0] = bf16_lo(w.x); z[1] = bf16_hi(w.x); z[2] = bf16_lo(w.y); z[3] = bf16_hi(w.y);
     } else {
@@ -437,7 +439,7 @@ __global__ __launch_bounds__(256) void head_gate_kernel(const float* __restrict_
     for (int e = 0; e < 4; ++e)
       if (lane + LANES * e < dim) {
         f[e] = src[lane + LANES * e];
-        z[e] = load_one(gr + lane + LANES * e);
+        z[e] = gate != nullptr ? load_one(gr + lane + LANES * e) : 0.f;
         g[e] = bf16_to_f32(wr[lane + LANES * e]);
       }
   }
@@ -446,16 +448,17 @@ __global__ __launch_bounds__(256) void head_gate_kernel(const float* __restrict_
 #pragma unroll
   for (int mask = 1; mask < LANES; mask <<= 1) ss += __shfl_xor(ss, mask, 64);
   const float inv = 1.0f / sqrtf(ss / (float)dim + eps);
+  auto through = [&](float v) { return gate != nullptr ? v * sigmoid_exact(v) : 1.f; };
   if (VEC) {
     if (c0 >= dim) return;
 #pragma unroll
-    for (int e = 0; e < 4; ++e) f[e] = f[e] * inv * g[e] * (z[e] * sigmoid_exact(z[e])) * scale;
+    for (int e = 0; e < 4; ++e) f[e] = f[e] * inv * g[e] * through(z[e]) * scale;
     if constexpr (sizeof(T) == 2) *reinterpret_cast<uint2*>(to + c0) = make_uint2(pack_bf16(f[0], f[1]), pack_bf16(f[2], f[3]));
     else *reinterpret_cast<float4*>(to + c0) = make_float4(f[0], f[1], f[2], f[3]);
   } else {
 #pragma unroll
     for (int e = 0; e < 4; ++e)
-      if (lane + LANES * e < dim) store_one(to + lane + LANES * e, f[e] * inv * g[e] * (z[e] * sigmoid_exact(z[e])) * scale);
+      if (lane + LANES * e < dim) store_one(to + lane + LANES * e, f[e] * inv * g[e] * through(z[e]) * scale);
   }
 }
 
@@ -587,10 +590,10 @@ extern "C" int iron_delta_rule(const float* x, float* state, const int* spans, f
 extern "C" int iron_head_gate(const float* o, const void* gate, const uint16_t* gain, void* out, int rows, int heads, int dim,
                               int gate_stride, int gate_at, int gain_shared, int out_stride, int out_at, float eps,
                               float scale, int is_float, const int* valid, void* stream) {
-  IRON_REQUIRE(o && gate && gain && out, "head_gate: null operand");
+  IRON_REQUIRE(o && gain && out, "head_gate: null operand");
   IRON_REQUIRE(rows > 0 && heads > 0 && dim > 0 && dim <= 256, "head_gate: rows (%d), heads (%d) positive, dim (%d) from 1 to 256",
                rows, heads, dim);
-  IRON_REQUIRE(gate_at >= 0 && gate_at + heads * dim <= gate_stride && out_at >= 0 && out_at + heads * dim <= out_stride,
+  IRON_REQUIRE((gate == nullptr || (gate_at >= 0 && gate_at + heads * dim <= gate_stride)) && out_at >= 0 && out_at + heads * dim <= out_stride,
                "head_gate: %d columns from %d of a gate row of %d, from %d of an output row of %d", heads * dim, gate_at,
                gate_stride, out_at, out_stride);
   const long items = (long)rows * heads;

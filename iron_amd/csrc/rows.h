@@ -45,6 +45,17 @@ __device__ __forceinline__ void store_one(T* __restrict__ p, float v) {
   store_vec<1>(p, f);
 }
 
+// act(g) * u.  kind: 0 the limited gate, min(g, limit) through x sigmoid(1.702 x), times one more than u held within the limit;
+// 1 SiLU; 2 GELU (tanh form); 3 ReLU.
+__device__ __forceinline__ float gated_value(int kind, float limit, float g, float u) {
+  if (kind == 0) {
+    g = fminf(g, limit);
+    u = fminf(fmaxf(u, -limit), limit);
+    return g / (1.f + expf(-1.702f * g)) * (u + 1.f);
+  }
+  return (kind == 3 ? fmaxf(g, 0.f) : (kind == 1 ? g / (1.f + expf(-g)) : gelu_tanh_f32(g))) * u;
+}
+
 // One sequence's part of a batch of rows: `rows` rows from `row0` on are its tokens at positions
 // `start`, `start + 1`, ...  The table has an entry a slot; an idle slot's has no rows.  Held inside
 // the batch here, so that no table can lead a kernel outside its buffers.

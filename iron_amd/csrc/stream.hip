@@ -1,6 +1,6 @@
 // A decoder's residual stream held in float32: rows gathered from a bf16 table into it, a row or its RMS
 // norm out of it, a block's normed or gated output added to it, a weighted sum of what it was after every layer in its
-// place, and the head's scale and soft cap.  One rounding, to the activation type, where a row leaves the stream;
+// place, plain sums into it with a norm by groups behind them, and the head's scale and soft cap.  One rounding, to the activation type, where a row leaves the stream;
 // bandwidth bound, a block a row.
 #include "../../include/iron_hip.h"
 #include "rows.h"
@@ -10,7 +10,7 @@ namespace iron {
 template <int VEC>
 __global__ __launch_bounds__(256) void stream_embed_kernel(const bf16_t* __restrict__ table, const int* __restrict__ ids,
                                                            float* __restrict__ x, float* __restrict__ also, int rows,
-                                                           int table_rows, int cols, const int* __restrict__ valid) {
+                                                           int table_rows, int cols, float scale, const int* __restrict__ valid) {
   const int row = blockIdx.x;
   if (row >= bound_or(valid, rows)) return;
   const int id = ids[row];
@@ -18,6 +18,8 @@ __global__ __launch_bounds__(256) void stream_embed_kernel(const bf16_t* __restr
   for (int c = threadIdx.x * VEC; c < cols; c += 256 * VEC) {
     float f[VEC];
     load_vec<VEC>(table + (size_t)id * cols + c, f);
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) f[j] *= scale;
     store_vec<VEC>(x + (size_t)row * cols + c, f);
     if (also != nullptr) store_vec<VEC>(also + (size_t)row * cols + c, f);
   }
@@ -237,6 +239,84 @@ __global__ __launch_bounds__(256) void stream_rows_kernel(float* __restrict__ x,
   }
 }
 
+// x += y + y2 (each may be missing), in place; then h = the row, each of its `groups` equal parts over its own root mean
+// square, times the gains.  A wave takes whole parts, and holds its first CH pieces of one between the passes.
+template <typename T, int VEC, int CH>
+__global__ __launch_bounds__(256) void stream_groups_kernel(float* __restrict__ x, const T* __restrict__ y, const T* __restrict__ y2,
+                                                            const bf16_t* __restrict__ w, T* __restrict__ h, int rows, int cols, int groups,
+                                                            float eps, float unit, const int* __restrict__ valid) {
+  const long item = (long)blockIdx.x * 4 + (threadIdx.x >> 6);
+  const int row = (int)(item / groups), first = (threadIdx.x & 63) * VEC, part = cols / groups;
+  if (row >= bound_or(valid, rows)) return;
+  const size_t at = (size_t)row * cols + (item - (long)row * groups) * part;
+  constexpr int STEP = 64 * VEC;
+  auto load = [&](int c, float (&f)[VEC]) {   // what the stream's element becomes
+    load_vec<VEC>(x + at + c, f);
+    float a[VEC], b[VEC];
+    if (y != nullptr) {
+      load_vec<VEC>(y + at + c, a);
+      if (y2 != nullptr) load_vec<VEC>(y2 + at + c, b);
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) f[j] += y2 != nullptr ? a[j] + b[j] : a[j];
+    }
+  };
+  float held[CH][VEC], ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < CH; ++i)
+    if (first + i * STEP < part) load(first + i * STEP, held[i]);
+#pragma unroll
+  for (int i = 0; i < CH; ++i)
+    if (first + i * STEP < part) {
+      if (y != nullptr) store_vec<VEC>(x + at + first + i * STEP, held[i]);
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) ss = fmaf(held[i][j], held[i][j], ss);
+    }
+  for (int c = first + CH * STEP; c < part; c += STEP) {
+    float f[VEC];
+    load(c, f);
+    if (y != nullptr) store_vec<VEC>(x + at + c, f);
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) ss = fmaf(f[j], f[j], ss);
+  }
+  if (h == nullptr) return;
+  const float inv = 1.0f / sqrtf(wave_sum(ss) / (float)part + eps);
+  const bf16_t* gain = w + (at - (size_t)row * cols);
+#pragma unroll
+  for (int i = 0; i < CH; ++i)
+    if (first + i * STEP < part) {
+      float g[VEC];
+      load_vec<VEC>(gain + first + i * STEP, g);
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) held[i][j] = held[i][j] * inv * (unit + g[j]);
+      store_vec<VEC>(h + at + first + i * STEP, held[i]);
+    }
+  for (int c = first + CH * STEP; c < part; c += STEP) {   // this thread's own stores, if it made any
+    float f[VEC], g[VEC];
+    load_vec<VEC>(x + at + c, f);
+    load_vec<VEC>(gain + c, g);
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) f[j] = f[j] * inv * (unit + g[j]);
+    store_vec<VEC>(h + at + c, f);
+  }
+}
+
+// Of rows [.. gate | up ..]: act(gate) * up into columns of rows of another length.
+template <typename T, int VEC>
+__global__ __launch_bounds__(256) void gated_columns_kernel(const T* __restrict__ x, T* __restrict__ y, int rows, int cols, int stride, int gate_at,
+                                                            int width, int at, int kind, float limit, const int* __restrict__ valid) {
+  const int pieces = cols / VEC;
+  const long item = (long)blockIdx.x * 256 + threadIdx.x;
+  const int row = (int)(item / pieces), c = (int)(item - (long)row * pieces) * VEC;
+  if (row >= bound_or(valid, rows)) return;
+  const T* g = x + (size_t)row * stride + gate_at + c;
+  float f[VEC], u[VEC];
+  load_vec<VEC>(g, f);
+  load_vec<VEC>(g + cols, u);
+#pragma unroll
+  for (int j = 0; j < VEC; ++j) f[j] = gated_value(kind, limit, f[j], u[j]);
+  store_vec<VEC>(y + (size_t)row * width + at + c, f);
+}
+
 // The last row of every span, gathered: out[slot] = x[row0 + rows - 1] (an idle slot's row is left).
 __global__ __launch_bounds__(256) void span_tails_kernel(const float* __restrict__ x, const int* __restrict__ spans,
                                                          float* __restrict__ out, int rows, int cols) {
@@ -354,14 +434,14 @@ static unsigned few_blocks(long n) {
 using namespace iron;
 
 extern "C" int iron_stream_embed(const uint16_t* table, const int* ids, float* x, float* also, int rows, int table_rows, int cols,
-                                 const int* valid, void* stream) {
+                                 float scale, const int* valid, void* stream) {
   IRON_REQUIRE(table && ids && x, "stream_embed: null operand");
   IRON_REQUIRE(rows > 0 && table_rows > 0 && cols > 0, "stream_embed: rows (%d), table_rows (%d), cols (%d) must be positive",
                rows, table_rows, cols);
   if (cols % 8 == 0 && (((uintptr_t)table | (uintptr_t)x | (uintptr_t)also) & 15) == 0)
-    hipLaunchKernelGGL((stream_embed_kernel<8>), dim3(rows), dim3(256), 0, (hipStream_t)stream, table, ids, x, also, rows, table_rows, cols, valid);
+    hipLaunchKernelGGL((stream_embed_kernel<8>), dim3(rows), dim3(256), 0, (hipStream_t)stream, table, ids, x, also, rows, table_rows, cols, scale, valid);
   else
-    hipLaunchKernelGGL((stream_embed_kernel<1>), dim3(rows), dim3(256), 0, (hipStream_t)stream, table, ids, x, also, rows, table_rows, cols, valid);
+    hipLaunchKernelGGL((stream_embed_kernel<1>), dim3(rows), dim3(256), 0, (hipStream_t)stream, table, ids, x, also, rows, table_rows, cols, scale, valid);
   IRON_LAUNCH_CHECK();
 }
 
@@ -424,6 +504,51 @@ extern "C" int iron_stream_gated_rows(float* x, const void* y, const uint16_t* y
   if (is_float) { IRON_STREAM_GATED(float) }
   IRON_STREAM_GATED(bf16_t)
 #undef IRON_STREAM_GATED
+}
+
+extern "C" int iron_stream_groups(float* x, const void* y, const void* y2, const uint16_t* gain, void* h, int rows, int cols, int groups, float eps,
+                                  float unit, int is_float, const int* valid, void* stream) {
+  IRON_REQUIRE(x && (h || y), "stream_groups: null operand");
+  IRON_REQUIRE((y != nullptr || y2 == nullptr) && (h == nullptr) == (gain == nullptr), "stream_groups: a second row behind a first, gains for a norm");
+  IRON_REQUIRE(rows > 0 && cols > 0 && groups > 0 && cols % groups == 0, "stream_groups: rows (%d) positive, cols (%d) in equal groups (%d)", rows, cols, groups);
+  const int part = cols / groups;
+  const long blocks = ((long)rows * groups + 3) / 4;
+  IRON_REQUIRE(blocks < (1L << 31), "stream_groups: %d rows of %d groups exceed the grid", rows, groups);
+  hipStream_t s = (hipStream_t)stream;
+  const bool vec = part % 8 == 0 && (((uintptr_t)x | (uintptr_t)y | (uintptr_t)y2 | (uintptr_t)gain | (uintptr_t)h) & 15) == 0;
+#define IRON_GROUPS(T, VEC, CH) \
+  hipLaunchKernelGGL((stream_groups_kernel<T, VEC, CH>), dim3((unsigned)blocks), dim3(256), 0, s, x, (const T*)y, (const T*)y2, gain, (T*)h, rows, cols, groups, eps, unit, valid)
+#define IRON_GROUPSS(T)                            \
+  {                                                \
+    if (vec && part <= 512) IRON_GROUPS(T, 8, 1);  \
+    else if (vec) IRON_GROUPS(T, 8, 4);            \
+    else IRON_GROUPS(T, 1, 4);                     \
+  }
+  if (is_float) IRON_GROUPSS(float)
+  else IRON_GROUPSS(bf16_t)
+#undef IRON_GROUPSS
+#undef IRON_GROUPS
+  IRON_LAUNCH_CHECK();
+}
+
+extern "C" int iron_gated_columns(const void* x, void* y, int rows, int cols, int stride, int gate_at, int width, int at, int kind, float limit,
+                                  int is_float, const int* valid, void* stream) {
+  IRON_REQUIRE(x && y, "gated_columns: null operand");
+  IRON_REQUIRE(rows > 0 && cols > 0, "gated_columns: rows (%d) and cols (%d) must be positive", rows, cols);
+  IRON_REQUIRE(gate_at >= 0 && gate_at + 2 * cols <= stride && at >= 0 && at + cols <= width,
+               "gated_columns: twice %d columns from %d of a row of %d, into those from %d of %d", cols, gate_at, stride, at, width);
+  IRON_REQUIRE(kind >= 0 && kind <= 3 && (kind != 0 || limit > 0.f),
+               "gated_columns: kind (%d) is 0 (a limit above 0), 1 (SiLU), 2 (GELU, tanh form) or 3 (ReLU)", kind);
+  const bool vec = cols % 8 == 0 && stride % 8 == 0 && gate_at % 8 == 0 && width % 8 == 0 && at % 8 == 0 && (((uintptr_t)x | (uintptr_t)y) & 15) == 0;
+  const long blocks = ((long)rows * (vec ? cols / 8 : cols) + 255) / 256;
+  IRON_REQUIRE(blocks < (1L << 31), "gated_columns: %d rows of %d exceed the grid", rows, cols);
+#define IRON_COLUMNS(T, VEC)                                                                                                               \
+  hipLaunchKernelGGL((gated_columns_kernel<T, VEC>), dim3((unsigned)blocks), dim3(256), 0, (hipStream_t)stream, (const T*)x, (T*)y, rows, cols, \
+                     stride, gate_at, width, at, kind, limit, valid)
+  if (is_float) { if (vec) IRON_COLUMNS(float, 8); else IRON_COLUMNS(float, 1); }
+  else { if (vec) IRON_COLUMNS(bf16_t, 8); else IRON_COLUMNS(bf16_t, 1); }
+#undef IRON_COLUMNS
+  IRON_LAUNCH_CHECK();
 }
 
 extern "C" int iron_span_tails(const float* x, const int* spans, float* out, int slots, int rows, int cols, void* stream) {

@@ -609,14 +609,14 @@ def _spans(t, slots):
     return ptr(t)
 
 
-def stream_embed(table, ids, x, *, rows, table_rows, cols, also=None, valid=None):
+def stream_embed(table, ids, x, *, rows, table_rows, cols, scale=1.0, also=None, valid=None):
     _bf16(table, table_rows * cols, "table")
     _numel(_dev(ids, "ids", torch.int32), rows, "ids")
     _f32(x, rows * cols, "x")
     if also is not None:
         _f32(also, rows * cols, "also")
-    check(lib().iron_stream_embed(ptr(table), ptr(ids), ptr(x), ptr(also), rows, table_rows, cols, ptr(_word(valid, "valid")),
-                                  current_stream()), "iron_stream_embed")
+    check(lib().iron_stream_embed(ptr(table), ptr(ids), ptr(x), ptr(also), rows, table_rows, cols, float(scale),
+                                  ptr(_word(valid, "valid")), current_stream()), "iron_stream_embed")
 
 
 def _added(x, y, y_bias, back_gain, h, rows, cols):
@@ -656,6 +656,87 @@ def stream_depth_rows(x, *, rows, cols, eps=0.0, unit=0.0, y=None, y_bias=None, 
     check(lib().iron_stream_depth_rows(ptr(x), ptr(y), ptr(y_bias), ptr(back_gain), ptr(planes), ptr(weights), plane_rows, index, ptr(h),
                                        rows, cols, float(eps), float(unit), int(is_float), ptr(_word(valid, "valid")), current_stream()),
           "iron_stream_depth_rows")
+
+
+def stream_groups(x, *, rows, cols, groups=1, eps=0.0, unit=0.0, y=None, y2=None, h=None, gain=None, valid=None):
+    """``x += y + y2`` (with ``y``; ``y2`` may be missing) and ``h``, the norm by ``groups`` of a row times ``unit + gain`` (with
+    ``h``), one launch."""
+    is_float = _added(x, y, None, None, h, rows, cols)
+    if y2 is not None:
+        _same_kind(is_float, y2=y2)
+        _act(y2, rows * cols, "y2")
+    if h is not None:
+        _bf16(gain, cols, "the gain of h")
+    check(lib().iron_stream_groups(ptr(x), ptr(y), ptr(y2), ptr(gain), ptr(h), rows, cols, groups, float(eps), float(unit), int(is_float),
+                                   ptr(_word(valid, "valid")), current_stream()), "iron_stream_groups")
+
+
+COLUMN_GATES = {"limited": 0, **GATES}   # by the C ABI's number
+
+
+def gated_columns(x, y, *, rows, cols, stride, gate_at, width, at, kind, limit=0.0, valid=None):
+    is_float = _act(x, rows * stride, "x")
+    _same_kind(is_float, y=y)
+    _act(y, rows * width, "y")
+    check(lib().iron_gated_columns(ptr(x), ptr(y), rows, cols, stride, gate_at, width, at, COLUMN_GATES[kind], float(limit), int(is_float),
+                                   ptr(_word(valid, "valid")), current_stream()), "iron_gated_columns")
+
+
+def hgrn2(x, f_bias, lower, state, spans, o, *, slots, rows, stride, heads, dim, vdim, workspace=None):
+    """The recurrence token by token, or with ``workspace`` sixteen tokens at a time."""
+    is_float = _act(x, rows * stride, "x")
+    _bf16(f_bias, heads * dim, "f_bias")
+    _bf16(lower, heads * dim, "lower")
+    _f32(state, slots * heads * dim * vdim, "state")
+    _f32(o, rows * heads * vdim, "o")
+    sizes = (slots, rows, stride, heads, dim, vdim, int(is_float), current_stream())
+    if workspace is not None:
+        work = _work(workspace, int(lib().iron_hgrn2_workspace_bytes(slots, rows, heads, dim)), "hgrn2: workspace")
+        check(lib().iron_hgrn2_chunked(ptr(x), ptr(f_bias), ptr(lower), ptr(state), _spans(spans, slots), ptr(o), work, *sizes), "iron_hgrn2_chunked")
+        return
+    check(lib().iron_hgrn2(ptr(x), ptr(f_bias), ptr(lower), ptr(state), _spans(spans, slots), ptr(o), *sizes), "iron_hgrn2")
+
+
+def decode_hgrn2(x, f_bias, lower, norm, state, spans, out, *, slots, rows, stride, heads, dim, vdim, out_stride, out_at, eps, cols=0, gate_at=0,
+                 gated_at=0, kind="limited", limit=0.0):
+    """A decode step's forget gate, fading memory and head norm beside a feed-forward's gated columns."""
+    _bf16(x, rows * stride, "x")
+    _bf16(f_bias, heads * dim, "f_bias")
+    _bf16(lower, heads * dim, "lower")
+    _bf16(norm, vdim, "norm")
+    _f32(state, slots * heads * dim * vdim, "state")
+    _bf16(out, rows * out_stride, "out")
+    check(lib().iron_decode_hgrn2_bf16(ptr(x), ptr(f_bias), ptr(lower), ptr(norm), ptr(state), _spans(spans, slots), ptr(out), slots, rows, stride,
+                                       heads, dim, vdim, out_stride, out_at, float(eps), cols, gate_at, gated_at, COLUMN_GATES[kind], float(limit),
+                                       current_stream()), "iron_decode_hgrn2_bf16")
+
+
+def cached_heads(x, q, keys, values, q_gain, k_gain, spans, *, slots, rows, stride, heads, kv_heads, dim, vdim, context, eps, turned=0,
+                 angle_rows=1, angles=None, value_norm=False, valid=None):
+    is_float = _act(x, rows * stride, "x")
+    _same_kind(is_float, q=q, keys=keys, values=values)
+    _act(q, rows * heads * dim, "q")
+    _act(keys, slots * kv_heads * context * dim, "keys")
+    _act(values, slots * kv_heads * context * vdim, "values")
+    _bf16(q_gain, dim, "q_gain")
+    _bf16(k_gain, dim, "k_gain")
+    check(lib().iron_cached_heads(ptr(x), ptr(q), ptr(keys), ptr(values), ptr(q_gain), ptr(k_gain), _turned(angles, angle_rows, turned),
+                                  _spans(spans, slots), slots, rows, stride, heads, kv_heads, dim, vdim, context, turned, angle_rows,
+                                  int(value_norm), float(eps), int(is_float), ptr(_word(valid, "valid")), current_stream()), "iron_cached_heads")
+
+
+def mha_global(q, keys, values, spans, y, *, slots, rows, heads, kv_heads, dim, vdim, context, scale, cap=0.0, sink=False, out_stride, out_at=0,
+               single=False, workspace=None):
+    is_float = _act(q, rows * heads * dim, "q")
+    _same_kind(is_float, keys=keys, values=values, y=y)
+    _act(keys, slots * kv_heads * context * dim, "keys")
+    _act(values, slots * kv_heads * context * vdim, "values")
+    _act(y, rows * out_stride, "y")
+    need = int(lib().iron_mha_global_workspace_bytes(slots, heads, kv_heads, vdim, context, int(single)))
+    work = _work(workspace, need, "mha_global: workspace") if need else None
+    check(lib().iron_mha_global(ptr(q), ptr(keys), ptr(values), _spans(spans, slots), ptr(y), work, slots, rows, heads, kv_heads, dim, vdim,
+                                context, float(scale), float(cap), int(sink), out_stride, out_at, int(single), int(is_float), current_stream()),
+          "iron_mha_global")
 
 
 def activation(x, y, *, rows, cols, kind, valid=None):
@@ -725,17 +806,19 @@ def memory_gate(o, gate, gain, y, *, rows, heads, dim, gate_stride, gate_at, flo
                                  int(is_float), ptr(_word(valid, "valid")), current_stream()), "iron_memory_gate")
 
 
-def router(h, w, bias, ids, shares, *, rows, cols, experts, top, valid=None):
+def router(h, w, bias, ids, shares, *, rows, cols, experts, top, correction=None, scored=False, valid=None):
     is_float = _act(h, rows * cols, "h")
     _bf16(w, experts * cols, "w")
-    _bf16(bias, experts, "bias")
+    for t, name in ((bias, "bias"), (correction, "correction")):
+        if t is not None:
+            _bf16(t, experts, name)
     _numel(_dev(ids, "ids", torch.int32), rows * top, "ids")
     _f32(shares, rows * top, "shares")
-    check(lib().iron_router(ptr(h), ptr(w), ptr(bias), ptr(ids), ptr(shares), rows, cols, experts, top, int(is_float),
+    check(lib().iron_router(ptr(h), ptr(w), ptr(bias), ptr(correction), int(scored), ptr(ids), ptr(shares), rows, cols, experts, top, int(is_float),
                             ptr(_word(valid, "valid")), current_stream()), "iron_router")
 
 
-def experts(h, gate, up, down, ids, shares, y, workspace, *, rows, cols, ff, experts, top, activation, valid=None):
+def experts(h, gate, up, down, ids, shares, y, workspace, *, rows, cols, ff, experts, top, activation, identity=0, valid=None):
     is_float = _act(h, rows * cols, "h")
     for t, name in ((gate, "gate"), (up, "up"), (down, "down")):
         _bf16(t, experts * ff * cols, name)
@@ -745,8 +828,8 @@ def experts(h, gate, up, down, ids, shares, y, workspace, *, rows, cols, ff, exp
     _act(y, rows * cols, "y")
     need = int(lib().iron_experts_workspace_bytes(rows, cols, ff, experts, top, int(is_float)))
     check(lib().iron_experts(ptr(h), ptr(gate), ptr(up), ptr(down), ptr(ids), ptr(shares), ptr(y), _work(workspace, need, "experts: workspace"),
-                             rows, cols, ff, experts, top, GATES[activation], int(is_float), ptr(_word(valid, "valid")), current_stream()),
-          "iron_experts")
+                             rows, cols, ff, experts, identity, top, GATES[activation], int(is_float), ptr(_word(valid, "valid")),
+                             current_stream()), "iron_experts")
 
 
 def stream_gated_rows(x, y, gate, gate_bias, *, rows, cols, eps=0.0, gate_stride, gate_at, y_bias=None, h=None, gain=None, valid=None):
@@ -887,10 +970,11 @@ def delta_rule(x, state, spans, o, *, slots, rows, heads, kv_heads, dim, vdim, w
 def head_gate(o, gate, gain, out, *, rows, heads, dim, gate_stride, gate_at, gain_shared, out_stride, out_at, eps, scale,
               valid=None):
     _f32(o, rows * heads * dim, "o")
-    is_float = _act(gate, rows * gate_stride, "gate")
+    is_float = _act(out, rows * out_stride, "out")
     _bf16(gain, dim if gain_shared else heads * dim, "gain")
-    _same_kind(is_float, out=out)
-    _act(out, rows * out_stride, "out")
+    if gate is not None:
+        _same_kind(is_float, gate=gate)
+        _act(gate, rows * gate_stride, "gate")
     check(lib().iron_head_gate(ptr(o), ptr(gate), ptr(gain), ptr(out), rows, heads, dim, gate_stride, gate_at,
                                int(gain_shared), out_stride, out_at, float(eps), float(scale), int(is_float),
                                ptr(_word(valid, "valid")), current_stream()), "iron_head_gate")

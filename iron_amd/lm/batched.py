@@ -345,7 +345,7 @@ class StreamDecoder(Decoder):
 
     def __init__(self, c, layer):
         super().__init__(c, layer)
-        self.norm = StreamRMSNorm(c.hidden_size, c.eps, c.activations, c.norm_unit)
+        self.norm = StreamRMSNorm(c.hidden_size, c.eps, c.activations, c.norm_unit, c.norm_groups)
 
 
 class BatchedLM(CausalLM):
@@ -354,8 +354,8 @@ class BatchedLM(CausalLM):
 
     The config is a ``LayerListConfig``: it adds to a decoder's ``slots`` (sequences served at once),
     ``activations`` (bf16, or float32 for a model in 32 bits throughout), ``order`` (layer indices in running
-    order), ``norm_unit`` (what the final norm's gains are stored around), ``looks_back`` (layers read the stream behind every
-    earlier one), ``logit_scale``, ``logit_softcap`` and ``key_room`` (keys a portion's layers may attend in all)."""
+    order), ``norm_unit`` (what the final norm's gains are stored around), ``norm_groups`` (parts of a row it norms by themselves),
+    ``embed_scale``, ``looks_back`` (layers read the stream behind every earlier one), ``logit_scale``, ``logit_softcap`` and ``key_room`` (keys a portion's layers may attend in all)."""
 
     decoder_class = StreamDecoder
     session_class = SlotSession
@@ -385,7 +385,7 @@ class BatchedLM(CausalLM):
         x = call.bound(self.residual[:count])
         ids = call.bound(ids) if call.prompt else self.token
         first = [] if self.planes is None else [call.bound(self.planes[0][:count])]
-        StreamEmbed.step(self.model.embed_tokens.weight, ids, x, *first, twice=bool(first))
+        StreamEmbed.step(self.model.embed_tokens.weight, ids, x, *first, twice=bool(first), scale=c.embed_scale)
         for index, states in self.runs:
             x = self.layers[index](x, call, states)
         last = SpanTails.step(x, self.spans) if call.prompt else x

@@ -1,5 +1,5 @@
 """The numbers that define a decoder (``DecoderConfig``) and the rotary table they imply
-(``rope_angles``).
+(``rope_angles``; ``yarn`` stretches it).
 
 Fields carry the names of a Hugging Face ``config.json`` wherever that file has the notion, so a
 config can be read from and written to one; the interface follows iron/lm/config.py:23-42,184-267.
@@ -9,6 +9,7 @@ from __future__ import annotations
 
 import dataclasses
 import json
+import math
 from collections.abc import Callable
 from pathlib import Path
 
@@ -41,6 +42,18 @@ def rope_angles(head_dim: int, context_length: int, rope_theta: float = 500000.0
     phase = (position[:, None] * frequency[None, :]).astype(np.float64)
     table = np.stack((np.cos(phase), np.sin(phase)), axis=-1)
     return table.reshape(context_length, -1)[:, :head_dim].astype(np.float32)
+
+
+def yarn(dims: int, base: float, *, factor: float, original: float, fast: float, slow: float) -> tuple[RopeScaling, float]:
+    """YaRN for ``rope_angles`` of ``dims`` columns: the scaling of its frequencies, and what the table is multiplied by.  Pairs
+    that turn at least ``fast`` times over ``original`` positions keep their frequency, those that turn at most ``slow`` times
+    have it divided by ``factor``, and between them a ramp over the pairs blends the two."""
+    def pair(turns: float) -> float:
+        return dims * math.log(original / (2 * math.pi * turns)) / (2 * math.log(base))
+
+    low, high = max(math.floor(pair(fast)), 0), min(math.ceil(pair(slow)), dims - 1)
+    ramp = np.clip((np.arange(dims // 2) - low) / max(high - low, 0.001), 0, 1)
+    return lambda f: f / factor * ramp + f * (1 - ramp), 0.1 * math.log(factor) + 1
 
 
 def _required(field: dataclasses.Field) -> bool:
@@ -192,6 +205,8 @@ class LayerListConfig(ConfigFile):
     logit_softcap = None
     logit_scale = 1.0
     norm_unit = 0.0        # what the norms' weights are stored around: 1 where a gain is 1 + its weight
+    norm_groups = 1        # equal parts of a row that are normed by themselves
+    embed_scale = 1.0      # what embedding rows are multiplied by
     looks_back = False     # whether layers read the stream behind every earlier one
     key_room = None        # keys, of all requests together, that a portion may attend; None: any number
 

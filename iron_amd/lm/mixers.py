@@ -1,8 +1,8 @@
 """Token mixers over a batch of rows told apart by spans, and the layer that runs them around a float32
 residual stream: sliding-window attention with a learned distance bias, time mixing with a
 data-dependent decay, both side by side, the gated delta rule, a gated recurrence element by element,
-latent attention, attention within chunks whose heads mix their weights, and a matrix memory; feed-forwards that go
-with them.
+latent attention, attention within chunks whose heads mix their weights, a matrix memory, attention over everything before under
+a soft cap and a sink, and a memory that fades by its one forget gate; feed-forwards that go with them.
 
 A module holds weights; what a run of it carries from token to token is a ``states()`` mapping the
 caller makes once per run, so that a layer run several times in a row has a state for each pass.
@@ -18,12 +18,14 @@ import numpy as np
 from .. import functional as F
 from ..common import graph as iron
 from ..operators.experts import Experts, Router
+from ..operators.mha_global import CachedHeads, GlobalMHA
 from ..operators.mha_latent import EVERYTHING, LatentMHA, LatentRows
 from ..operators.mha_talking import TalkingMHA, TurnedHeads
 from ..operators.mha_window import WindowMHA
 from ..operators.recurrent import (
     DeltaRule,
     HeadGate,
+    Hgrn2,
     LowRankDecay,
     MatrixMemory,
     MemoryGate,
@@ -32,7 +34,17 @@ from ..operators.recurrent import (
     TimeMix,
     TokenShift,
 )
-from ..operators.stream import Activation, DepthAverage, PolyNorm, StreamAdd, StreamCast, StreamGatedAdd, StreamNorm
+from ..operators.stream import (
+    Activation,
+    DepthAverage,
+    GatedColumns,
+    PolyNorm,
+    StreamAdd,
+    StreamCast,
+    StreamGatedAdd,
+    StreamNorm,
+    StreamSum,
+)
 from .blocks import Linear
 
 
@@ -56,14 +68,15 @@ def distance_buckets(count: int, rows: int, bias_max: float) -> np.ndarray:
 
 class StreamRMSNorm(iron.Graph):
     """An RMS norm at the stream's edge: ``body`` takes a normed row out of it, ``add`` a block's output
-    into it.  Gains are ``unit`` (0, or 1 where they are stored around zero) plus the weight."""
+    into it.  Gains are ``unit`` (0, or 1 where they are stored around zero) plus the weight.  ``groups``: the row is normed in
+    that many equal parts, each by itself (out of the stream only)."""
 
-    def __init__(self, width: int, eps: float, dtype, unit: float = 0.0):
-        self.constants = dict(epsilon=eps, unit=unit, dtype=dtype)
+    def __init__(self, width: int, eps: float, dtype, unit: float = 0.0, groups: int = 1):
+        self.constants, self.groups = dict(epsilon=eps, unit=unit, dtype=dtype), groups
         self.weight = iron.param(width)
 
     def body(self, stream):
-        return StreamNorm.step(stream, self.weight, **self.constants)
+        return StreamNorm.step(stream, self.weight, groups=self.groups, **self.constants)
 
     def add(self, stream, y, y_bias=None):
         return StreamAdd.step(stream, y, self.weight, y_bias=y_bias, **self.constants)
@@ -140,7 +153,7 @@ class TimeMixing(iron.Graph):
         r, k, v, g, z = (as_rows(x, h.shape[0]) for x in (r, k, v, g, z))
         decay = LowRankDecay.step(z, self.w2, self.w0, dtype=self.dtype)
         o = TimeMix.step(r, k, v, decay, self.u, state["memory"], call.spans, dtype=self.dtype)[1]
-        return HeadGate.step(o, g, self.norm, heads=self.heads, width=width, at=at, epsilon=self.eps, scale=self.out_scale,
+        return HeadGate.step(o, self.norm, gate=g, heads=self.heads, width=width, at=at, epsilon=self.eps, scale=self.out_scale,
                              dtype=self.dtype)
 
 
@@ -196,7 +209,7 @@ class DeltaMixer(iron.Graph):
         _, y = ShortConv.step(x, self.conv, self.a_log, self.dt_bias, state["inputs"], call.spans, dim=self.dim, vdim=self.vdim,
                               b_at=self.b_at, a_at=self.a_at, dtype=self.dtype, **sizes)
         _, o = DeltaRule.step(y, state["memory"], call.spans, **sizes)
-        return self.out(HeadGate.step(o, x, self.norm, heads=self.heads, gate_at=self.gate_at, epsilon=self.eps,
+        return self.out(HeadGate.step(o, self.norm, gate=x, heads=self.heads, gate_at=self.gate_at, epsilon=self.eps,
                                       dtype=self.dtype))
 
 
@@ -403,19 +416,23 @@ class ActivatedMLP(iron.Graph):
 
 
 class ExpertsMLP(iron.Graph):
-    """Gated feed-forwards of which a router chooses ``top`` a row.  The experts' matrices are stacked."""
+    """Gated feed-forwards of which a router chooses ``top`` a row.  The experts' matrices are stacked.  ``scored``: the choice and
+    the shares are by the softmax over all of the router's logits, the choice by its scores plus corrections; else by biased
+    logits and a softmax over the chosen.  ``identity``: the router's last ones, that many, hand on the row itself."""
 
-    def __init__(self, width, *, inner, experts, top, activation, dtype):
-        self.top, self.kind, self.dtype = top, activation, dtype
-        self.router = iron.param(experts, width)
-        self.router_bias = iron.param(experts)
+    def __init__(self, width, *, inner, experts, top, activation, dtype, scored=False, identity=0):
+        self.top, self.kind, self.dtype, self.scored, self.identity = top, activation, dtype, scored, identity
+        self.router = iron.param(experts + identity, width)
+        self.router_bias = None if scored else iron.param(experts)
+        self.correction = iron.param(experts + identity) if scored else None
         self.gate = iron.param(experts * inner, width)
         self.up = iron.param(experts * inner, width)
         self.down = iron.param(experts * width, inner)
 
     def body(self, h):
-        ids, shares = Router.step(h, self.router, self.router_bias, top=self.top, dtype=self.dtype)
-        return Experts.step(h, self.gate, self.up, self.down, ids, shares, activation=self.kind, dtype=self.dtype)
+        ids, shares = Router.step(h, self.router, bias=self.router_bias, correction=self.correction, scored=self.scored, top=self.top,
+                                  dtype=self.dtype)
+        return Experts.step(h, self.gate, self.up, self.down, ids, shares, activation=self.kind, identity=self.identity, dtype=self.dtype)
 
 
 class PostNormLayer(iron.Graph):
@@ -436,3 +453,73 @@ class PostNormLayer(iron.Graph):
         if self.mlp is not None:
             x = self.norm2.add(x, as_rows(self.mlp(StreamCast.step(x, dtype=self.dtype)), x.shape[0]))
         return DepthAverage.step(x, call.planes, self.depth)[0]
+
+
+# ---- layers whose mixer and feed-forward read one norm of the stream side by side: one projection into both, one out of both
+
+
+class GlobalAttention(iron.Graph):
+    """Grouped-query attention over everything before: q and k normed a head, turned by ``angles`` in halves, values over their
+    root mean square (``value_norm``), scores times ``scale`` under a soft ``cap`` (0: none), ``sink`` one more in the softmax's
+    denominator.  Its columns of a packed projection's row are (q, k, v); fills the first ``out_width`` columns of a ``width``-column row."""
+
+    def __init__(self, *, heads, kv_heads, dim, vdim, scale, eps, context, dtype, angles=None, cap=0.0, sink=False, value_norm=False):
+        self.heads, self.kv_heads, self.dim, self.vdim = heads, kv_heads, dim, vdim
+        self.scale, self.cap, self.sink, self.value_norm = scale, cap, sink, value_norm
+        self.eps, self.context, self.dtype, self.angles = eps, context, dtype, angles
+        self.own, self.out_width = heads * dim + kv_heads * (dim + vdim), heads * vdim
+        self.q_norm = iron.param(dim)
+        self.k_norm = iron.param(dim)
+
+    def states(self, slots: int) -> dict:
+        # A key head's positions one after the other: a step reads them as one run.
+        return {"keys": iron.state((slots, self.kv_heads, self.context, self.dim), self.dtype),
+                "values": iron.state((slots, self.kv_heads, self.context, self.vdim), self.dtype)}
+
+    def body(self, x, call, state, width):
+        keys, values, q = CachedHeads.step(x, self.q_norm, self.k_norm, call.spans, state["keys"], state["values"], angles=self.angles,
+                                           heads=self.heads, value_norm=self.value_norm, epsilon=self.eps, dtype=self.dtype)
+        return GlobalMHA.step(q, keys, values, call.spans, width=width, scale=self.scale, cap=self.cap, sink=self.sink,
+                              single=not call.prompt, dtype=self.dtype)
+
+
+class FadingMemory(iron.Graph):
+    """HGRN2: a matrix a head that a forget gate a channel fades and, by what it leaves, writes, each head normed.  Its columns of
+    a packed projection's row are (q, forget gate, v); fills the first ``out_width`` columns of a ``width``-column row."""
+
+    def __init__(self, *, heads, dim, vdim, eps, dtype):
+        self.heads, self.dim, self.vdim, self.eps, self.dtype = heads, dim, vdim, eps, dtype
+        self.own, self.out_width = heads * (2 * dim + vdim), heads * vdim
+        self.f_bias = iron.param(heads * dim)
+        self.lower = iron.param(heads * dim)
+        self.norm = iron.param(vdim)
+
+    def states(self, slots: int) -> dict:
+        return {"memory": iron.state((slots, self.heads, self.dim, self.vdim), np.float32)}
+
+    def body(self, x, call, state, width):
+        _, o = Hgrn2.step(x, self.f_bias, self.lower, state["memory"], call.spans, dtype=self.dtype)
+        return HeadGate.step(o, self.norm, heads=self.heads, width=width, epsilon=self.eps, dtype=self.dtype)
+
+
+class SideBySideLayer(iron.Graph):
+    """``h = norm(x); x += mixer(h) + ff(h)`` around a float32 stream.  ``proj`` packs the mixer's columns and those of a gated
+    feed-forward of ``inner`` (gate, up; ``kind`` and ``limit`` as GatedColumns has them); ``out`` is the output projections of
+    both side by side; ``routed`` a feed-forward of experts beside them (or None)."""
+
+    def __init__(self, width, mixer, *, inner=0, kind="silu", limit=0.0, routed=None, eps, groups, dtype, precision):
+        self.mixer, self.routed, self.inner, self.kind, self.limit, self.dtype = mixer, routed, inner, kind, limit, dtype
+        self.norm1 = StreamRMSNorm(width, eps, dtype, groups=groups)
+        self.proj = Linear(width, mixer.own + 2 * inner, precision=precision)
+        self.out = Linear(mixer.out_width + inner, width, precision=precision)
+        self.rope = None
+
+    def body(self, x, call, state):
+        rows, h = x.shape[0], self.norm1(x)
+        packed = as_rows(self.proj(h), rows)
+        made = self.mixer(packed, call, state, self.out.in_features)
+        if self.inner:
+            made = GatedColumns.step(packed, made, cols=self.inner, gate_at=self.mixer.own, at=self.mixer.out_width, kind=self.kind,
+                                     limit=self.limit, dtype=self.dtype)
+        beside = {"also": as_rows(self.routed(h), rows)} if self.routed is not None else {}
+        return StreamSum.step(x, as_rows(self.out(made), rows), dtype=self.dtype, **beside)

@@ -15,25 +15,32 @@ F32 = np.float32
 
 class Router(Operator):
     """The ``top`` experts with the largest ``weight h + bias`` (float32) of each row, and their shares: a softmax over the
-    chosen logits alone."""
+    chosen logits alone.  ``scored``: those with the largest softmax score (over all logits) plus ``correction``, and their
+    shares, the scores over their sum."""
 
     rows: int = param()
     cols: int = param()
     experts: int = param()
     top: int = param()
+    scored: bool = param(default=False, repr=False)
+    biased: bool = param(default=True, repr=False)
+    corrected: bool = param(default=False, repr=False)
     dtype: Any = param(default=bfloat16, repr=False)
     h = In(rows, cols, dtype=dtype)
     weight = In(experts, cols)
-    bias = In(experts)
+    bias = In(experts, when=biased)
+    correction = In(experts, when=corrected)
     ids = Out(rows, top, dtype=np.int32)
     shares = Out(rows, top, dtype=F32)
     valid = per_call(bounds=rows)
 
     @classmethod
     def infer(cls, shapes, **kw):
-        return dict(rows=shapes["h"][0], cols=shapes["h"][1], experts=shapes["weight"][0], **kw)
+        return dict(rows=shapes["h"][0], cols=shapes["h"][1], experts=shapes["weight"][0], biased="bias" in shapes, corrected="correction" in shapes, **kw)
 
     def validate(self):
+        if self.corrected and not self.scored:
+            raise ValueError("Router: corrections are of scores")
         if not 1 <= self.top <= min(self.experts, 64) or self.experts > 1024:
             raise ValueError(f"Router: top ({self.top}) from 1 to the experts ({self.experts}), 64 at most of 1024")
 
@@ -43,16 +50,17 @@ class Router(Operator):
     def build(self) -> Built:
         from .. import kernels
 
-        kw = dict(rows=self.rows, cols=self.cols, experts=self.experts, top=self.top)
+        kw = dict(rows=self.rows, cols=self.cols, experts=self.experts, top=self.top, scored=self.scored)
 
         def launch(t, words):
-            kernels.router(t["h"], t["weight"], t["bias"], t["ids"], t["shares"], valid=words.get("valid"), **kw)
+            kernels.router(t["h"], t["weight"], t.get("bias"), t["ids"], t["shares"], correction=t.get("correction"), valid=words.get("valid"), **kw)
 
         return Built("iron_router", launch)
 
 
 class Experts(Operator):
-    """``sum over a row's experts e of share * down_e (act(gate_e h) * (up_e h))``; the experts' matrices are stacked."""
+    """``sum over a row's experts e of share * down_e (act(gate_e h) * (up_e h))``; the experts' matrices are stacked.
+    ``identity``: that many ids behind the experts' last stand for ``h`` itself."""
 
     rows: int = param()
     cols: int = param()
@@ -60,6 +68,7 @@ class Experts(Operator):
     top: int = param()
     ff: int = param()
     activation: str = param()
+    identity: int = param(default=0)
     stacked: int = param(derive=lambda op: op.experts * op.ff, repr=False)
     tall: int = param(derive=lambda op: op.experts * op.cols, repr=False)
     dtype: Any = param(default=bfloat16, repr=False)
@@ -86,6 +95,10 @@ class Experts(Operator):
         tall, ff = shapes["down"]
         return dict(rows=rows, cols=cols, experts=tall // cols, ff=ff, top=shapes["ids"][1], **kw)
 
+    def validate(self):
+        if self.identity < 0 or not 1 <= self.top <= self.experts + self.identity:
+            raise ValueError(f"Experts: top ({self.top}) from 1 to {self.experts} experts and {self.identity} identities")
+
     def ops(self) -> int:
         return 6 * self.rows * self.top * self.cols * self.ff
 
@@ -95,7 +108,7 @@ class Experts(Operator):
     def build(self) -> Built:
         from .. import kernels
 
-        kw = {n: getattr(self, n) for n in ("rows", "cols", "ff", "experts", "top", "activation")}
+        kw = {n: getattr(self, n) for n in ("rows", "cols", "ff", "experts", "identity", "top", "activation")}
 
         def launch(t, words):
             kernels.experts(t["h"], t["gate"], t["up"], t["down"], t["ids"], t["shares"], t["y"], t["workspace"], valid=words.get("valid"), **kw)

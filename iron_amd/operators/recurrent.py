@@ -283,13 +283,15 @@ class DeltaRule(_DeltaShape):
 
 class HeadGate(Operator):
     """``o / rms(o) * gain * silu(gate) * scale`` a head, into columns ``at ..`` of a row of ``width``.  The
-    gate is columns ``gate_at ..`` of its row; ``gain`` is one head's (shared by all) or every column's."""
+    gate is columns ``gate_at ..`` of its row (not ``gated``: there is no such factor); ``gain`` is one head's (shared by
+    all) or every column's."""
 
     rows: int = param()
     heads: int = param()
     dim: int = param()
     o_width: int = param(derive=lambda op: op.heads * op.dim, repr=False)
-    gate_width: int = param()
+    gated: bool = param(default=True, repr=False)
+    gate_width: int = param(default=0)
     gate_at: int = param(default=0, array=True)
     gains: int = param()
     width: int = param()
@@ -298,7 +300,7 @@ class HeadGate(Operator):
     scale: float = param(default=1.0, array=True)
     dtype: Any = param(default=bfloat16, repr=False)
     o = In(rows, o_width, dtype=F32)
-    gate = In(rows, gate_width, dtype=dtype)
+    gate = In(rows, gate_width, dtype=dtype, when=gated)
     gain = In(gains)
     y = Out(rows, width, dtype=dtype)
     valid = per_call(bounds=rows)
@@ -306,8 +308,8 @@ class HeadGate(Operator):
     @classmethod
     def infer(cls, shapes, **kw):
         dim = shapes["o"][1] // kw["heads"]
-        return {"rows": shapes["o"][0], "dim": dim, "gate_width": shapes["gate"][1], "gains": shapes["gain"][0],
-                "width": shapes["o"][1], **kw}
+        gate = {"gate_width": shapes["gate"][1]} if "gate" in shapes else {"gated": False}
+        return {"rows": shapes["o"][0], "dim": dim, "gains": shapes["gain"][0], "width": shapes["o"][1], **gate, **kw}
 
     def validate(self):
         if self.gains not in (self.dim, self.o_width):
@@ -324,9 +326,58 @@ class HeadGate(Operator):
                   eps=float(self.epsilon), scale=float(self.scale))
 
         def launch(t, words):
-            kernels.head_gate(t["o"], t["gate"], t["gain"], t["y"], valid=words.get("valid"), **kw)
+            kernels.head_gate(t["o"], t.get("gate"), t["gain"], t["y"], valid=words.get("valid"), **kw)
 
         return Built("iron_head_gate", launch)
+
+
+class Hgrn2(_Spanned):
+    """HGRN2: per head ``S <- diag(f) S + (1 - f) v^T``, then ``o = S^T silu(q)``, with the forget gate ``f = lower + (1 - lower)
+    sigmoid(z + f_bias)`` a channel.  Rows ``[q | z | v | ..]``."""
+
+    slots: int = param()
+    rows: int = param()
+    stride: int = param()
+    heads: int = param()
+    dim: int = param()
+    vdim: int = param()
+    channels: int = param(derive=lambda op: op.heads * op.dim, repr=False)
+    width: int = param(derive=lambda op: op.heads * op.vdim, repr=False)
+    dtype: Any = param(default=bfloat16, repr=False)
+    x = In(rows, stride, dtype=dtype)
+    f_bias = In(channels)
+    lower = In(channels)
+    state = InOut(slots, heads, dim, vdim, dtype=F32)
+    spans = In(slots, 4, dtype=np.int32)
+    o = Out(rows, width, dtype=F32)
+    chunked: bool = param(default=lambda op: op.rows > op.CHUNKED_ROWS * op.slots, array=True, repr=False)
+    workspace_words: int = param(derive=lambda op: op._workspace_words(), repr=False)
+    workspace = Scratch(workspace_words, dtype=F32, when=chunked)
+    valid = per_call(bounds=rows)
+
+    def _workspace_words(self) -> int:
+        from .._lib import lib
+
+        return int(lib().iron_hgrn2_workspace_bytes(self.slots, self.rows, self.heads, self.dim)) // 4
+
+    @classmethod
+    def infer(cls, shapes, **kw):
+        slots, heads, dim, vdim = shapes["state"]
+        return dict(slots=slots, rows=shapes["x"][0], stride=shapes["x"][1], heads=heads, dim=dim, vdim=vdim, **kw)
+
+    def validate(self):
+        if not (1 <= self.dim <= 256 and self.heads * (2 * self.dim + self.vdim) <= self.stride):
+            raise ValueError(f"Hgrn2: dim ({self.dim}) from 1 to 256; {self.heads} heads of {self.dim} and {self.vdim} in a row of {self.stride}")
+
+    def build(self) -> Built:
+        from .. import kernels
+
+        kw = {n: getattr(self, n) for n in ("slots", "rows", "stride", "heads", "dim", "vdim")}
+
+        def launch(t, words):
+            kernels.hgrn2(t["x"], t["f_bias"], t["lower"], t["state"], t["spans"], t["o"], workspace=t.get("workspace"), **kw)
+
+        return Built("iron_hgrn2", launch)
 
 
 class MatrixMemory(_Spanned):

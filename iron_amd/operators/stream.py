@@ -1,5 +1,5 @@
 """The float32 residual stream of a decoder: rows into it, rows or their norms out of it, blocks' outputs added to it,
-averages over what it was behind earlier layers, and the head's scale and soft cap.  ``dtype`` is what the rows that leave the stream are rounded to: bf16, or
+averages over what it was behind earlier layers, a feed-forward's gated columns, and the head's scale and soft cap.  ``dtype`` is what the rows that leave the stream are rounded to: bf16, or
 float32 in a model that runs in 32 bits throughout.  The stream is updated in place.
 """
 
@@ -18,12 +18,13 @@ F32 = np.float32
 
 
 class StreamEmbed(Operator):
-    """``x[i] = table[ids[i]]``, widened: a decoder's embedding rows as its stream's first values.  ``twice``: into a second
-    place as well."""
+    """``x[i] = scale * table[ids[i]]`` in float32: a decoder's embedding rows as its stream's first values.  ``twice``: into a
+    second place as well."""
 
     rows: int = param()
     table_rows: int = param(array=True)
     cols: int = param()
+    scale: float = param(default=1.0, array=True)
     twice: bool = param(default=False, repr=False)
     table = In(table_rows, cols)
     ids = In(rows, dtype=np.int32)
@@ -41,20 +42,22 @@ class StreamEmbed(Operator):
     def build(self) -> Built:
         from .. import kernels
 
-        rows, table_rows, cols = self.rows, self.table_rows, self.cols
+        rows, table_rows, cols, scale = self.rows, self.table_rows, self.cols, float(self.scale)
 
         def launch(t, words):
-            kernels.stream_embed(t["table"], t["ids"].reshape(-1), t["x"], rows=rows, table_rows=table_rows, cols=cols,
+            kernels.stream_embed(t["table"], t["ids"].reshape(-1), t["x"], rows=rows, table_rows=table_rows, cols=cols, scale=scale,
                                  also=t.get("also"), valid=words.get("valid"))
 
         return Built("iron_stream_embed", launch)
 
 
 class StreamNorm(Operator):
-    """``y = dtype(x / rms(x) * (unit + weight))`` of a float32 row: one rounding, where it leaves the stream."""
+    """``y = dtype(x / rms(x) * (unit + weight))`` of a float32 row: one rounding, where it leaves the stream.  ``groups``: each
+    of a row's that many equal parts over its own root mean square."""
 
     rows: int = param()
     cols: int = param()
+    groups: int = param(default=1)
     epsilon: float = param(array=True)
     unit: float = param(default=0.0, array=True)
     dtype: Any = param(default=bfloat16, repr=False)
@@ -67,6 +70,10 @@ class StreamNorm(Operator):
     def infer(cls, shapes, **kw):
         return dict(rows=shapes["x"][0], cols=shapes["x"][1], **kw)
 
+    def validate(self):
+        if self.groups < 1 or self.cols % self.groups:
+            raise ValueError(f"StreamNorm: {self.cols} columns in {self.groups} equal groups")
+
     def tolerance(self):
         return Tolerance.relative(1e-2, 1e-2, note="float32, rounded once")
 
@@ -74,11 +81,89 @@ class StreamNorm(Operator):
         from .. import kernels
 
         kw = dict(rows=self.rows, cols=self.cols, eps=float(self.epsilon), unit=float(self.unit))
+        grouped = self.groups > 1
 
         def launch(t, words):
-            kernels.stream_rows(t["x"], h=t["y"], gain=t["weight"], valid=words.get("valid"), **kw)
+            given = dict(h=t["y"], gain=t["weight"], valid=words.get("valid"), **kw)
+            if grouped:
+                kernels.stream_groups(t["x"], groups=self.groups, **given)
+            else:
+                kernels.stream_rows(t["x"], **given)
 
-        return Built("iron_stream_rows", launch)
+        return Built("iron_stream_groups" if grouped else "iron_stream_rows", launch)
+
+
+class StreamSum(Operator):
+    """``x += y + also`` in float32: what blocks side by side made of one row joins the stream (``also`` may be missing)."""
+
+    rows: int = param()
+    cols: int = param()
+    two: bool = param(default=False, repr=False)
+    dtype: Any = param(default=bfloat16, repr=False)
+    x = InOut(rows, cols, dtype=F32)
+    y = In(rows, cols, dtype=dtype)
+    also = In(rows, cols, dtype=dtype, when=two)
+    valid = per_call(bounds=rows)
+
+    @classmethod
+    def infer(cls, shapes, **kw):
+        return dict(rows=shapes["x"][0], cols=shapes["x"][1], two="also" in shapes, **kw)
+
+    def tolerance(self):
+        return Tolerance.relative(1e-5, 1e-5, note="float32")
+
+    def build(self) -> Built:
+        from .. import kernels
+
+        kw = dict(rows=self.rows, cols=self.cols)
+
+        def launch(t, words):
+            kernels.stream_groups(t["x"], y=t["y"], y2=t.get("also"), valid=words.get("valid"), **kw)
+
+        return Built("iron_stream_groups", launch)
+
+
+class GatedColumns(Operator):
+    """``act(gate) * up`` of columns ``gate_at ..`` and ``gate_at + cols ..`` of a projection's row, into columns ``at ..`` of
+    ``y`` (whose other columns are left alone).  ``kind`` ``limited``: ``g sigmoid(1.702 g) (u + 1)``, g the gate held to at most
+    ``limit``, u within it on both sides; else an activation's name."""
+
+    rows: int = param()
+    cols: int = param()
+    stride: int = param()
+    width: int = param()
+    gate_at: int = param(default=0, array=True)
+    at: int = param(default=0, array=True)
+    kind: str = param()
+    limit: float = param(default=0.0, array=True)
+    dtype: Any = param(default=bfloat16, repr=False)
+    x = In(rows, stride, dtype=dtype)
+    y = InOut(rows, width, dtype=dtype)
+    valid = per_call(bounds=rows)
+
+    @classmethod
+    def infer(cls, shapes, **kw):
+        return dict(rows=shapes["x"][0], stride=shapes["x"][1], width=shapes["y"][1], **kw)
+
+    def validate(self):
+        if not (0 <= self.gate_at <= self.stride - 2 * self.cols and 0 <= self.at <= self.width - self.cols):
+            raise ValueError(f"GatedColumns: twice {self.cols} columns from {self.gate_at} of {self.stride}, into those from {self.at} of {self.width}")
+        if self.kind == "limited" and not self.limit > 0:
+            raise ValueError(f"GatedColumns: a limit ({self.limit}) above 0")
+
+    def tolerance(self):
+        return Tolerance.relative(1e-2, 1e-2, note="float32, rounded once")
+
+    def build(self) -> Built:
+        from .. import kernels
+
+        kw = {n: getattr(self, n) for n in ("rows", "cols", "stride", "gate_at", "width", "at", "kind")}
+        kw["limit"] = float(self.limit)
+
+        def launch(t, words):
+            kernels.gated_columns(t["x"], t["y"], valid=words.get("valid"), **kw)
+
+        return Built("iron_gated_columns", launch)
 
 
 class StreamAdd(Operator):

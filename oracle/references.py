@@ -160,7 +160,7 @@ def _spans(spans):
 
 
 def stream_embed(op, table, ids):
-    rows = np.asarray(table, np.float32)[np.clip(np.asarray(ids).reshape(-1), 0, op.table_rows - 1)]
+    rows = np.asarray(table, np.float32)[np.clip(np.asarray(ids).reshape(-1), 0, op.table_rows - 1)] * np.float32(op.scale)
     return (rows, rows) if op.twice else rows
 
 
@@ -170,7 +170,9 @@ def _unit_rms(x, eps):
 
 
 def stream_norm(op, x, weight):
-    return _out(op, _unit_rms(x, op.epsilon) * (op.unit + np.asarray(weight, np.float64)))
+    x = np.reshape(x, (op.rows, op.cols))
+    parts = _unit_rms(np.reshape(x, (op.rows, op.groups, -1)), op.epsilon).reshape(x.shape)
+    return _out(op, parts * (op.unit + np.asarray(weight, np.float64)))
 
 
 def stream_add(op, x, y, weight, *, y_bias=None):
@@ -335,8 +337,15 @@ def activation(op, x):
     return _out(op, _act_of(op.kind, np.asarray(x, np.float64)))
 
 
-def router(op, h, weight, bias):
-    z = np.asarray(h, np.float64) @ np.asarray(weight, np.float64).T + bias
+def router(op, h, weight, *, bias=None, correction=None):
+    z = np.asarray(h, np.float64) @ np.asarray(weight, np.float64).T + (0 if bias is None else bias)
+    if op.scored:
+        e = np.exp(z - z.max(1, keepdims=True))
+        e = e / e.sum(1, keepdims=True)
+        by = e + (0 if correction is None else np.asarray(correction, np.float64))
+        ids = np.argsort(-by, axis=1, kind="stable")[:, : op.top]
+        e = np.take_along_axis(e, ids, 1)
+        return ids.astype(np.int32), (e / (e.sum(1, keepdims=True) + 1e-20)).astype(np.float32)
     ids = np.argsort(-z, axis=1, kind="stable")[:, : op.top]
     chosen = np.take_along_axis(z, ids, 1)
     e = np.exp(chosen - chosen.max(1, keepdims=True))
@@ -349,8 +358,86 @@ def experts(op, h, gate, up, down, ids, shares):
     down = np.reshape(np.asarray(down, np.float64), (op.experts, op.cols, op.ff))
     for r in range(op.rows):
         for e, share in zip(np.asarray(ids)[r], np.asarray(shares, np.float64)[r]):
+            if e >= op.experts:   # an identity
+                y[r] += share * h[r]
+                continue
             a = _out(op, _act_of(op.activation, gate[e] @ h[r]) * (up[e] @ h[r]))
             y[r] += share * (down[e] @ np.asarray(a, np.float64))
+    return _out(op, y)
+
+
+def stream_sum(op, x, y, *, also=None):
+    return np.asarray(np.asarray(x, np.float64) + y + (0 if also is None else np.asarray(also, np.float64)), np.float32)
+
+
+def gated_columns(op, x, y):
+    y = np.array(y)
+    g, u = (np.asarray(x, np.float64)[:, at : at + op.cols] for at in (op.gate_at, op.gate_at + op.cols))
+    if op.kind == "limited":
+        g, u = np.minimum(g, op.limit), np.clip(u, -op.limit, op.limit)
+        made = g * _sigmoid(1.702 * g) * (u + 1)
+    else:
+        made = _act_of(op.kind, g) * u
+    y[:, op.at : op.at + op.cols] = made
+    return _out(op, y)
+
+
+def hgrn2(op, x, f_bias, lower, state, spans):
+    H, D, V = op.heads, op.dim, op.vdim
+    state, o = np.array(state), np.zeros((op.rows, H, V), np.float32)
+    x, lower = np.asarray(x, np.float64), np.asarray(lower, np.float64)
+    q = (x[:, : H * D] * _sigmoid(x[:, : H * D])).reshape(-1, H, D)
+    f = (lower + (1 - lower) * _sigmoid(x[:, H * D : 2 * H * D] + f_bias)).reshape(-1, H, D)
+    v = x[:, 2 * H * D : H * (2 * D + V)].reshape(-1, H, V)
+    for s, row, n, start in _spans(spans):
+        S = np.asarray(state[s], np.float64) if start else np.zeros((H, D, V))
+        for t in range(row, row + n):
+            S = f[t][:, :, None] * S + (1 - f[t])[:, :, None] * v[t][:, None, :]
+            o[t] = np.einsum("hdv,hd->hv", S, q[t])
+        state[s] = S
+    return state, o.reshape(op.rows, -1)
+
+
+def _turn_halves(x, angles, n):
+    """Columns i and i + n / 2 of x (..., width) turned together by a row of cosines and sines side by side."""
+    x = np.array(x)
+    u, v, c, s = x[..., : n // 2].copy(), x[..., n // 2 : n].copy(), angles[..., 0:n:2], angles[..., 1:n:2]
+    x[..., : n // 2], x[..., n // 2 : n] = u * c - v * s, v * c + u * s
+    return x
+
+
+def cached_heads(op, x, q_gain, k_gain, spans, keys, values, *, angles=None):
+    H, G, D, V = op.heads, op.kv_heads, op.dim, op.vdim
+    keys, values, q = np.array(keys), np.array(values), np.zeros((op.rows, op.inner), np.float32)
+    for s, row, n, start in _spans(spans):
+        own, at = np.asarray(x, np.float64)[row : row + n], np.arange(start, start + n)
+        made = []
+        for heads, gain in ((own[:, : H * D].reshape(n, H, D), q_gain), (own[:, H * D : (H + G) * D].reshape(n, G, D), k_gain)):
+            heads = _unit_rms(heads, op.epsilon) * gain
+            if op.turned:
+                heads = _turn_halves(heads, np.asarray(angles, np.float64)[start : start + n, None], op.turned)
+            made.append(heads)
+        v = own[:, (H + G) * D : (H + G) * D + G * V].reshape(n, G, V)
+        v = _unit_rms(v, op.epsilon) if op.value_norm else v
+        q[row : row + n] = made[0].reshape(n, -1)
+        keys[s][:, at], values[s][:, at] = _out(op, made[1]).swapaxes(0, 1), _out(op, v).swapaxes(0, 1)
+    return keys, values, _out(op, q)
+
+
+def global_mha(op, q, keys, values, spans):
+    H, G, D, V = op.heads, op.kv_heads, op.dim, op.vdim
+    y, group = np.zeros((op.rows, op.width), np.float32), np.arange(H) // (H // G)
+    q = np.asarray(q, np.float64).reshape(op.rows, H, D)
+    for s, row, n, start in _spans(spans):
+        for i in range(n):
+            k, v = (np.asarray(c[s][:, : start + i + 1], np.float64)[group] for c in (keys, values))
+            score = np.einsum("hd,hjd->hj", q[row + i], k) * op.scale
+            if op.cap:
+                score = op.cap * np.tanh(score / op.cap)
+            top = np.maximum(score.max(1, keepdims=True), 0)
+            e = np.exp(score - top)
+            p = e / (e.sum(1, keepdims=True) + (np.exp(-top) if op.sink else 0))
+            y[row + i, op.at : op.at + H * V] = np.einsum("hj,hjv->hv", p, v).reshape(-1)
     return _out(op, y)
 
 
@@ -448,13 +535,13 @@ def delta_rule(op, x, state, spans):
     return state, o.reshape(op.rows, -1)
 
 
-def head_gate(op, o, gate, gain):
+def head_gate(op, o, gain, *, gate=None):
     H, D = op.heads, op.dim
-    z = np.asarray(gate, np.float64)[:, op.gate_at : op.gate_at + H * D]
+    z = None if gate is None else np.asarray(gate, np.float64)[:, op.gate_at : op.gate_at + H * D]
     gains = np.asarray(gain, np.float64) if op.gains == op.o_width else np.tile(np.asarray(gain, np.float64), H)
     y = np.zeros((op.rows, op.width), np.float32)
     y[:, op.at : op.at + H * D] = (_unit_rms(np.reshape(o, (-1, H, D)), op.epsilon).reshape(op.rows, -1) * gains
-                                   * z / (1 + np.exp(-z)) * op.scale)
+                                   * (1 if z is None else z / (1 + np.exp(-z))) * op.scale)
     return _out(op, y)
 
 
@@ -504,6 +591,7 @@ def install() -> None:
         SampleSlots=sample_slots, StreamGatedAdd=stream_gated_add, PolyNorm=poly_norm, MinGRU=min_gru, LatentRows=latent_rows,
         LatentMHA=latent_mha, DepthAverage=depth_average, StreamCast=stream_cast, TurnedHeads=turned_heads, TalkingMHA=talking_mha,
         MatrixMemory=matrix_memory, MemoryGate=memory_gate, Activation=activation, Router=router, Experts=experts,
+        StreamSum=stream_sum, GatedColumns=gated_columns, Hgrn2=hgrn2, CachedHeads=cached_heads, GlobalMHA=global_mha,
         # The host's draw, for iron_amd.lm.generation.Sampler's checks.
         sample_ref=ops.sample_ref, sample_weights=ops.sample_weights,
     )
