@@ -579,11 +579,12 @@ int iron_hgrn2_chunked(const void* x, const uint16_t* f_bias, const uint16_t* lo
                        void* workspace, int slots, int rows, int stride, int heads, int dim, int vdim, int is_float,
                        void* stream);
 /* One token a slot, bf16, in one launch: iron_hgrn2, iron_head_gate without a gate (gains (vdim) shared by the heads) into columns
- * out_at .. of out, and beside it iron_gated_columns of the same rows into those from gated_at (cols 0: none).  vdim a power
- * of two from 16. */
+ * out_at .. of out, and beside it iron_gated_columns of the same rows into those from gated_at (cols 0: none), and, for one slot, iron_router's
+ * scored choice from its logits z (NULL: none).  vdim a power of two from 16. */
 int iron_decode_hgrn2_bf16(const uint16_t* x, const uint16_t* f_bias, const uint16_t* lower, const uint16_t* norm, float* state,
                            const int* spans, uint16_t* out, int slots, int rows, int stride, int heads, int dim, int vdim,
                            int out_stride, int out_at, float eps, int cols, int gate_at, int gated_at, int kind, float limit,
+                           const float* z, const uint16_t* correction, int logits, int top, int* ids, float* shares,
                            void* stream);
 /* Rows [q heads | k heads | v heads | ..] of a packed projection made ready to be attended: q and k RMS-normed a head with
  * q_gain / k_gain (dim), columns i and i + turned / 2 of the first `turned` turned together by their position's row of angles
@@ -593,6 +594,14 @@ int iron_cached_heads(const void* x, void* q, void* keys, void* values, const ui
                       const float* angles, const int* spans, int slots, int rows, int stride, int heads, int kv_heads, int dim,
                       int vdim, int context, int turned, int angle_rows, int value_norm, float eps, int is_float,
                       const int* valid, void* stream);
+/* One token a slot, bf16, in one launch: iron_cached_heads, and beside it iron_gated_columns of the same rows into columns
+ * gated_at .. of out (cols 0: none), and, for one slot, iron_router's scored choice from its logits z (NULL: none). */
+int iron_decode_heads_global_bf16(const uint16_t* x, uint16_t* q, uint16_t* keys, uint16_t* values, const uint16_t* q_gain,
+                                  const uint16_t* k_gain, const float* angles, const int* spans, int slots, int rows, int stride,
+                                  int heads, int kv_heads, int dim, int vdim, int context, int turned, int angle_rows,
+                                  int value_norm, float eps, uint16_t* out, int out_stride, int cols, int gate_at, int gated_at,
+                                  int kind, float limit, const float* z, const uint16_t* correction, int logits, int top, int* ids,
+                                  float* shares, void* stream);
 /* Causal attention over such caches, the rows' own keys in them already: score = q . k * scale, with cap > 0 cap *
  * tanh(score / cap); softmax, with `sink` one more in its denominator; the values' sums in columns out_at .. of y (rows of
  * out_stride).  single: no span has more than one row.  workspace: of that many bytes (it may be none), 16-byte aligned. */
@@ -612,6 +621,16 @@ int iron_stream_product_bf16(int input, const void* x, const uint16_t* gain, con
                              float* state, const int* spans, float eps, float unit, const uint16_t* W, int M,
                              int K, uint16_t* y, float* stream_row, const uint16_t* y_bias, const uint16_t* gate, const uint16_t* gate_bias,
                              void* stream);
+/* norm_product: y = W (M, K) times h, the float row x normed in `groups` parts (iron_stream_groups); h (may be NULL) as well, and
+ * with a router (logits, K) its logits in float to z.  product_sum: the stream's row += W (M, K) times x, plus also (may be NULL). */
+int iron_norm_product_bf16(const float* x, const uint16_t* gain, int groups, float eps, float unit, const uint16_t* W, int M, int K,
+                           uint16_t* y, uint16_t* h, const uint16_t* router, int logits, float* z, void* stream);
+int iron_product_sum_bf16(const uint16_t* x, const uint16_t* W, int M, int K, const uint16_t* also, float* stream_row, void* stream);
+/* One row through its experts (iron_experts; h, gate .. activation as there) and, in the launch that sums them, out (cols, inner)
+ * times made: the stream's row += both, each rounded.  workspace: 2 top ff bytes.  Two launches. */
+int iron_experts_tail_bf16(const uint16_t* h, const uint16_t* gate, const uint16_t* up, const uint16_t* down, const int* ids, const float* shares,
+                           const uint16_t* out, const uint16_t* made, float* stream_row, void* workspace, int cols, int ff, int inner,
+                           int experts, int identity, int top, int activation, void* stream);
 int iron_latent_query_bf16(const uint16_t* x, const uint16_t* q_gain, const uint16_t* c_gain, const float* angles,
                            const int* spans, const uint16_t* W, uint16_t* q, uint16_t* latents, uint16_t* shared_keys,
                            int M, int stride, int q_rank, int rank, int rot, int turned, int angle_rows, int ring,

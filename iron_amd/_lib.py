@@ -97,7 +97,11 @@ SIGNATURES = {
     "iron_hgrn2": (c_int, [_P] * 6 + [c_int] * 7 + [_P]),
     "iron_hgrn2_workspace_bytes": (c_int64, [c_int] * 4),
     "iron_hgrn2_chunked": (c_int, [_P] * 7 + [c_int] * 7 + [_P]),
-    "iron_decode_hgrn2_bf16": (c_int, [_P] * 7 + [c_int] * 8 + [c_float] + [c_int] * 4 + [c_float, _P]),
+    "iron_decode_hgrn2_bf16": (c_int, [_P] * 7 + [c_int] * 8 + [c_float] + [c_int] * 4 + [c_float, _P, _P, c_int, c_int, _P, _P, _P]),
+    "iron_decode_heads_global_bf16": (c_int, [_P] * 8 + [c_int] * 11 + [c_float, _P] + [c_int] * 5 + [c_float, _P, _P, c_int, c_int, _P, _P, _P]),
+    "iron_norm_product_bf16": (c_int, [_P, _P, c_int, c_float, c_float, _P, c_int, c_int, _P, _P, _P, c_int, _P, _P]),
+    "iron_product_sum_bf16": (c_int, [_P, _P, c_int, c_int, _P, _P, _P]),
+    "iron_experts_tail_bf16": (c_int, [_P] * 10 + [c_int] * 7 + [_P]),
     "iron_cached_heads": (c_int, [_P] * 8 + [c_int] * 11 + [c_float, c_int, _P, _P]),
     "iron_mha_global_workspace_bytes": (c_int64, [c_int] * 6),
     "iron_mha_global": (c_int, [_P] * 6 + [c_int] * 7 + [c_float, c_float] + [c_int] * 5 + [_P]),

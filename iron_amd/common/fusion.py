@@ -33,10 +33,17 @@ in a batched decoder's decode step (bf16; a float32 stream, layers with a state)
   StreamNorm, GEMV (one slot, as the rest here)          => iron_stream_product_bf16 (input 1)
   [MinGRU / PolyNorm,] GEMV, StreamGatedAdd              => iron_stream_product_bf16 (input 0 / 3 / 4)
   LatentRows, GEMV (the queries)                         => iron_latent_query_bf16
+  StreamNorm (groups), GEMV                              => iron_norm_product_bf16
+  Hgrn2, HeadGate [, GatedColumns] (any slots)           => iron_decode_hgrn2_bf16
+  CachedHeads, GlobalMHA [, GatedColumns] (any slots)    => iron_decode_heads_global_bf16, iron_mha_global
+  ... either behind StreamNorm, GEMV, Router             => iron_norm_product_bf16 with the logits; the choice beside the mixer
+  GEMV, StreamSum                                        => iron_product_sum_bf16
+  Experts, GEMV, StreamSum                               => iron_experts_tail_bf16
 
 and in either,
 
   StreamAdd, StreamNorm                                  => iron_stream_rows
+  StreamSum, StreamNorm                                  => iron_stream_groups
   [StreamAdd,] [DepthAverage,] [StreamCast] (two of them) => iron_stream_depth_rows
   StreamGatedAdd, StreamNorm                             => iron_stream_gated_rows
   RMSNorm, ElementwiseAdd (a sandwich layer's residual)  => iron_rmsnorm_add_bf16
@@ -384,6 +391,123 @@ def plan(recording, tensor: Callable[[Any], Any], word: Callable[[Any], Any],
             args["h"] = tensor(cast.outputs["y"])
         return Fused("stream_depth_rows", j, at - j, lambda a=args, kw=kw: kernels.stream_depth_rows(**a, **kw))
 
+    def step_mixer_at(j):
+        """``(steps, launch)`` where a decode step's mixer with what it needs ahead and behind, and a feed-forward's gated columns
+        beside it (if there are any), start at step ``j``; ``launch(**choice)`` runs them, a router's choice beside -- or None."""
+        first, second = steps[j : j + 2] if j + 1 < len(steps) else (None, None)
+        if first is None or first.op.dtype is not bfloat16 or first.values or second.values:
+            return None
+        o = first.op
+        if _name(first) == "Hgrn2" and _name(second) == "HeadGate":
+            ok = (o.rows == o.slots and 16 <= o.vdim <= 256 and o.vdim & (o.vdim - 1) == 0 and not second.op.gated and second.op.gains == o.vdim
+                  and second.op.dtype is bfloat16 and second.op.scale == 1.0 and _same(second.inputs["o"], first.outputs["o"])
+                  and once(first.outputs["o"]))
+        elif _name(first) == "CachedHeads" and _name(second) == "GlobalMHA":
+            ok = (o.rows == o.slots and second.op.single and not any(n % 8 for n in (o.dim, o.vdim, o.stride)) and max(o.dim, o.vdim) <= 256
+                  and _same(second.inputs["q"], first.outputs["q"]) and second.op.dtype is bfloat16)
+        else:
+            return None
+        if not ok:
+            return None
+        made, count = second.outputs["y"], 2
+        columns = steps[j + 2] if j + 2 < len(steps) and _name(steps[j + 2]) == "GatedColumns" else None
+        if (columns is not None and not columns.values and columns.op.dtype is bfloat16 and _same(columns.inputs["x"], first.inputs["x"])
+                and _same(columns.inputs["y"], made)):
+            count, c = 3, columns.op
+            beside = dict(cols=c.cols, gate_at=c.gate_at, gated_at=c.at, kind=c.kind, limit=float(c.limit))
+        else:
+            beside = {}
+        if _name(first) == "Hgrn2":
+            args = {n: tensor(first.inputs[n]) for n in ("x", "f_bias", "lower", "state", "spans")}
+            args |= dict(norm=tensor(second.inputs["gain"]), out=tensor(made))
+            kw = {n: getattr(o, n) for n in ("slots", "rows", "stride", "heads", "dim", "vdim")}
+            kw |= dict(out_stride=second.op.width, out_at=second.op.at, eps=float(second.op.epsilon), **beside)
+            return count, 1, lambda **choice: kernels.decode_hgrn2(**args, **kw, **choice)
+        heads = {n: tensor(first.inputs[n]) for n in ("x", "q_gain", "k_gain", "spans", "keys", "values", "angles") if n in first.inputs}
+        heads |= dict(q=tensor(first.outputs["q"]), out=tensor(made))
+        kw = {n: getattr(o, n) for n in ("slots", "rows", "stride", "heads", "kv_heads", "dim", "vdim", "context", "turned", "angle_rows", "value_norm")}
+        kw |= dict(eps=float(o.epsilon), out_stride=second.op.width, **beside)
+        m = second.op
+        attend = dict(q=heads["q"], keys=heads["keys"], values=heads["values"], spans=heads["spans"], y=heads["out"],
+                      workspace=tensor(second.outputs["workspace"]))
+        attend |= {n: getattr(m, n) for n in ("slots", "rows", "heads", "kv_heads", "dim", "vdim", "context", "sink")}
+        attend |= dict(scale=float(m.scale), cap=float(m.cap), out_stride=m.width, out_at=m.at, single=True)
+
+        def launch(**choice):
+            kernels.decode_heads_global(**heads, **kw, **choice)
+            kernels.mha_global(**attend)
+
+        return count, 3, launch
+
+    def step_mixer(j):
+        found = step_mixer_at(j)
+        return None if found is None else Fused("step_mixer", j, found[0], found[2], launches=found[1])
+
+    def norm_product_at(j):
+        """The launch for a single row's grouped norm and the product of it -- with a router's logits and, beside the mixer behind
+        it, the router's choice, where they follow -- or None."""
+        s = steps[j]
+        g = steps[j + 1] if j + 1 < len(steps) else None
+        h, o = s.outputs["y"], s.op
+        if not (g is not None and o.rows == 1 and o.dtype is bfloat16 and o.cols % (8 * o.groups) == 0 and o.cols <= 16384 and o.groups <= 256
+                and bare(s) and gemv_row(g, h)):
+            return None
+        args = dict(W=tensor(g.inputs["A"]), x=tensor(s.inputs["x"]).reshape(-1), gain=tensor(s.inputs["weight"]),
+                    y=tensor(g.outputs["C"]).reshape(-1))
+        kw = dict(M=g.op.M, K=g.op.K, groups=o.groups, eps=float(o.epsilon), unit=float(o.unit))
+        if once(h):
+            return Fused("norm_product", j, 2, lambda: kernels.norm_product(**args, **kw))
+        args["h"] = tensor(h).reshape(-1)
+        r = steps[j + 2] if j + 2 < len(steps) and _name(steps[j + 2]) == "Router" else None
+        if (r is not None and scratch is not None and bare(r) and r.op.scored and not r.op.biased and r.op.dtype is bfloat16 and _same(r.inputs["h"], h)
+                and (mixer := step_mixer_at(j + 3)) is not None):
+            need = 4 * r.op.experts
+            z = scratch(j, need)
+            logits = dict(router=tensor(r.inputs["weight"]), z=z, logits=r.op.experts)
+            choice = dict(z=z, logits=r.op.experts, top=r.op.top, ids=tensor(r.outputs["ids"]).reshape(-1), shares=tensor(r.outputs["shares"]).reshape(-1))
+            if "correction" in r.inputs:
+                choice["correction"] = tensor(r.inputs["correction"])
+            count, launches, run = mixer
+
+            def launch():
+                kernels.norm_product(**args, **kw, **logits)
+                run(**choice)
+
+            return Fused("norm_product_router_mixer", j, 3 + count, launch, launches=1 + launches, scratch_bytes=need)
+        return Fused("norm_product", j, 2, lambda: kernels.norm_product(**args, **kw))
+
+    def stream_end(j):
+        """``(product, sum)`` where step ``j`` is one row's product and the next adds it to the stream -- or None."""
+        g, add = steps[j : j + 2] if j + 1 < len(steps) else (None, None)
+        if not (g is not None and gemv_row(g) and g.op.K % 8 == 0 and g.op.K <= 16384 and _name(add) == "StreamSum" and add.op.rows == 1
+                and add.op.dtype is bfloat16 and bare(add) and _same(add.inputs["y"], g.outputs["C"]) and once(g.outputs["C"])):
+            return None
+        return g, add
+
+    def product_sum_at(j):
+        if (end := stream_end(j)) is None:
+            return None
+        g, add = end
+        args = dict(x=tensor(g.inputs["B"]).reshape(-1), W=tensor(g.inputs["A"]), stream=tensor(add.inputs["x"]).reshape(-1))
+        if "also" in add.inputs:
+            args["also"] = tensor(add.inputs["also"]).reshape(-1)
+        return Fused("product_sum", j, 2, lambda: kernels.product_sum(**args, M=g.op.M, K=g.op.K))
+
+    def experts_tail_at(j):
+        """The launches for one row's experts, and the product and the sum that join the stream with them -- or None."""
+        s = steps[j]
+        o, y, end = s.op, s.outputs["y"], stream_end(j + 1)
+        if not (end and o.rows == 1 and o.dtype is bfloat16 and bare(s) and once(y) and "also" in end[1].inputs and _same(end[1].inputs["also"], y)
+                and not any(n % 8 for n in (o.cols, o.ff)) and o.top <= 64 and end[0].op.K // 8 + o.top * o.ff // 8 <= 4096):
+            return None
+        g, add = end
+        args = {n: tensor(s.inputs[n]) for n in ("gate", "up", "down")}
+        args |= {n: tensor(s.inputs[n]).reshape(-1) for n in ("h", "ids", "shares")}
+        args |= dict(out=tensor(g.inputs["A"]), made=tensor(g.inputs["B"]).reshape(-1), stream=tensor(add.inputs["x"]).reshape(-1),
+                     workspace=tensor(s.outputs["workspace"]))
+        kw = dict(cols=o.cols, ff=o.ff, inner=g.op.K, experts=o.experts, identity=o.identity, top=o.top, activation=o.activation)
+        return Fused("experts_tail", j, 3, lambda: kernels.experts_tail(**args, **kw), launches=2)
+
     def latent_query_at(j):
         """The launch for a single slot's latents and the product of its queries -- or None."""
         s = steps[j]
@@ -719,6 +843,25 @@ def plan(recording, tensor: Callable[[Any], Any], word: Callable[[Any], Any],
                 got = Fused("gemv_act_mul", i, 3, lambda a=args, kw=kw: kernels.gemv_fused(**a, **kw))
         elif _name(s) in ("StreamAdd", "DepthAverage") and (got := depth_rows_at(i)) is not None:
             pass
+        elif _name(s) == "StreamNorm" and (s.op.groups > 1 or (i + 2 < len(steps) and _name(steps[i + 2]) == "Router")):
+            got = norm_product_at(i)
+        elif _name(s) in ("Hgrn2", "CachedHeads"):
+            got = step_mixer(i)
+        elif _name(s) == "Experts":
+            got = experts_tail_at(i)
+        elif gemv_row(s) and (got := product_sum_at(i)) is not None:
+            pass
+        elif _name(s) == "StreamSum" and i + 1 < len(steps) and _name(steps[i + 1]) == "StreamNorm":
+            # what blocks made joins the stream, and the next blocks' norm leaves it: one pass over the row
+            nm = steps[i + 1]
+            if (_same_view(nm.inputs["x"], s.outputs["x"]) and nm.op.dtype is s.op.dtype and (nm.op.rows, nm.op.cols) == (s.op.rows, s.op.cols)
+                    and nm.values.get("valid") == s.values.get("valid") and set(nm.values) <= {"valid"} and set(s.values) <= {"valid"}):
+                args = dict(x=tensor(s.inputs["x"]), y=tensor(s.inputs["y"]), h=tensor(nm.outputs["y"]), gain=tensor(nm.inputs["weight"]))
+                if "also" in s.inputs:
+                    args["y2"] = tensor(s.inputs["also"])
+                kw = dict(rows=s.op.rows, cols=s.op.cols, groups=nm.op.groups, eps=float(nm.op.epsilon), unit=float(nm.op.unit),
+                          valid=word(s.values.get("valid")))
+                got = Fused("stream_sum_norm", i, 2, lambda a=args, kw=kw: kernels.stream_groups(**a, **kw))
         elif _name(s) == "StreamAdd" and i + 1 < len(steps) and _name(steps[i + 1]) == "StreamNorm":
             # a block's output into the stream and the next block's norm out of it: one pass over the row
             nm = steps[i + 1]

@@ -3,7 +3,8 @@
 //   decode_parallel: low-rank decay, time-mixing step, head norm and gate (a block a head)
 //                    beside sliding-window attention with its distance bias (a block a query head)
 //   decode_delta:    short convolution, unit q and k, gated delta rule, head norm and gate
-//   decode_hgrn2:    forget gate, fading memory, head norm (a block a head) beside a feed-forward's gated columns
+//   decode_hgrn2:    forget gate, fading memory, head norm (a block a head) beside a feed-forward's gated columns and a router's
+//                    choice
 //
 // bf16 rows, float32 inside.  A block is 16 waves.  A head's state (dim rows of `wide` columns, wide a power
 // of two from 16 to 256) is read once, four columns a thread, and kept in registers until it is replaced;
@@ -12,6 +13,7 @@
 // rings with a row to spare (see the prompt kernels, whose layouts these are).
 #include "../../include/iron_hip.h"
 #include "hgrn2.h"
+#include "router.h"
 
 namespace iron {
 
@@ -507,18 +509,28 @@ struct FadeStep {
   float eps;
   int cols, gate_at, gated_at, kind;      // gated columns of the same rows: how many, where from, where to
   float limit;
+  RouterChoice choice;                    // of slot 0's logits
 };
 struct FadeShared {
   float q[256], keep[256], write[256], v[256];
   float sums[DM_WAVES][256];
   float part[DM_WAVES];
 };
+union FadeOrChoice {
+  FadeShared fade;
+  float choice[2][ROUTER_MAX];
+};
 
 template <int NR>
 __global__ __launch_bounds__(DM_THREADS) void decode_hgrn2_kernel(FadeStep a, const int* __restrict__ spans, int rows) {
-  __shared__ __align__(16) FadeShared sh;
+  __shared__ __align__(16) FadeOrChoice lds;
+  FadeShared& sh = lds.fade;
   const int slot = blockIdx.y, head = blockIdx.x, t = threadIdx.x;
   const Span s = span_of(spans, slot, rows);
+  if (a.choice.z != nullptr && blockIdx.x == gridDim.x - 1) {   // (whether the slot has a row or not, as the router by itself)
+    choose_row(a.choice, lds.choice[0], lds.choice[1]);
+    return;
+  }
   if (s.rows == 0) return;
   const bf16_t* row = a.x + (size_t)s.row0 * a.stride;
   bf16_t* to = a.out + (size_t)s.row0 * a.out_stride;
@@ -660,8 +672,10 @@ extern "C" int iron_decode_delta_bf16(const uint16_t* x, const uint16_t* taps_w,
 
 extern "C" int iron_decode_hgrn2_bf16(const uint16_t* x, const uint16_t* f_bias, const uint16_t* lower, const uint16_t* norm, float* state,
                                       const int* spans, uint16_t* out, int slots, int rows, int stride, int heads, int dim, int vdim, int out_stride,
-                                      int out_at, float eps, int cols, int gate_at, int gated_at, int kind, float limit, void* stream) {
+                                      int out_at, float eps, int cols, int gate_at, int gated_at, int kind, float limit, const float* z,
+                                      const uint16_t* correction, int logits, int top, int* ids, float* shares, void* stream) {
   IRON_REQUIRE(x && f_bias && lower && norm && state && spans && out, "decode_hgrn2: null operand");
+  IRON_ROUTER_CHOICE_REQUIRE("decode_hgrn2");
   IRON_REQUIRE(((uintptr_t)spans & 15) == 0 && ((uintptr_t)state & 15) == 0, "decode_hgrn2: spans and state must be 16-byte aligned");
   IRON_REQUIRE(slots > 0 && slots <= 65535 && rows > 0, "decode_hgrn2: slots (%d) and rows (%d) must be positive", slots, rows);
   IRON_REQUIRE(heads > 0 && dim > 0 && dim <= 256 && whole_columns(vdim), "decode_hgrn2: dim (%d) up to 256, vdim (%d) a power of two from 16 to 256", dim, vdim);
@@ -670,8 +684,9 @@ extern "C" int iron_decode_hgrn2_bf16(const uint16_t* x, const uint16_t* f_bias,
   IRON_REQUIRE(cols >= 0 && (cols == 0 || (gate_at >= 0 && gate_at + 2 * cols <= stride && gated_at >= 0 && gated_at + cols <= out_stride)),
                "decode_hgrn2: twice %d gated columns from %d, into those from %d", cols, gate_at, gated_at);
   IRON_REQUIRE(kind >= 0 && kind <= 3, "decode_hgrn2: kind (%d) is 0 to 3", kind);
-  const FadeStep a{x, FadeGates{f_bias, lower}, norm, state, out, stride, heads, dim, vdim, out_stride, out_at, eps, cols, gate_at, gated_at, kind, limit};
-  const dim3 grid(heads + (cols + DM_THREADS - 1) / DM_THREADS, slots);
+  const FadeStep a{x, FadeGates{f_bias, lower}, norm, state, out, stride, heads, dim, vdim, out_stride, out_at, eps, cols, gate_at, gated_at, kind, limit,
+                   RouterChoice{z, correction, logits, top, ids, shares}};
+  const dim3 grid(heads + (cols + DM_THREADS - 1) / DM_THREADS + (z != nullptr), slots);
 #define IRON_FADE_STEP(NR)                                                                                           \
   {                                                                                                                  \
     hipLaunchKernelGGL((decode_hgrn2_kernel<NR>), grid, dim3(DM_THREADS), 0, (hipStream_t)stream, a, spans, rows);   \

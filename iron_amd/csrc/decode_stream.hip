@@ -1,9 +1,9 @@
 // One row of a decoder around a float32 stream: a product with what makes its input ahead of it and what takes its
 // output behind it, in one launch.
 //
-//   input:   a bf16 row; the stream's row, or a bf16 row, RMS-normed; a gated recurrence's step; an activation
-//            over the normed powers of a row
-//   output:  a bf16 row; or, through a sigmoid gate, the stream
+//   input:   a bf16 row; the stream's row (whole or in groups), or a bf16 row, RMS-normed; a gated recurrence's step; an
+//            activation over the normed powers of a row
+//   output:  a bf16 row; or, through a sigmoid gate or as it is, the stream
 //
 // Every block makes the whole input for its own few rows of the weight (L2 serves it) while those are on their way
 // from memory.  What a launch replaces, no other block of it reads: a recurrence has two states, by a position's
@@ -12,11 +12,14 @@
 #include "../../include/iron_hip.h"
 #include "latent.h"
 #include "row_products.h"
+#include "rows.h"
 
 namespace iron {
 
-enum { IN_ROW = 0, IN_STREAM_NORM = 1, IN_ROW_NORM = 2, IN_GRU = 3, IN_POLY = 4 };
-enum { OUT_ROW = 0, OUT_GATED = 1, OUT_LATENT = 2 };   // OUT_LATENT: a row, and the last block a position's latent
+enum { IN_ROW = 0, IN_STREAM_NORM = 1, IN_ROW_NORM = 2, IN_GRU = 3, IN_POLY = 4, IN_STREAM_GROUPS = 5 };
+// OUT_LATENT: a row, and the last block a position's latent.  OUT_LOGITS: a row, and a router's logits in float behind it.
+enum { OUT_ROW = 0, OUT_GATED = 1, OUT_LATENT = 2, OUT_ADD = 3, OUT_LOGITS = 4 };
+constexpr int MOST_GROUPS = 256;
 
 struct StreamIn {
   const void* x;              // float (the stream) or bf16
@@ -26,11 +29,16 @@ struct StreamIn {
   const int* spans;           // IN_GRU, OUT_LATENT
   float eps;
   float unit;                 // added to a norm's gains
+  int groups;                 // IN_STREAM_GROUPS
+  bf16_t* made;               // ... where the first block leaves the input it made, for later launches (may be NULL)
 };
 struct StreamOut {
   bf16_t* y;
   float* stream;
-  const bf16_t *y_bias, *gate, *gate_bias;
+  const bf16_t *y_bias, *gate, *gate_bias;   // OUT_ADD: y_bias is a second row that joins the stream
+  const bf16_t* router;       // OUT_LOGITS: `logits` more rows of a weight, and where their products go
+  float* z;
+  int logits;
   // OUT_LATENT
   const bf16_t *row, *c_gain;
   const float* angles;
@@ -46,7 +54,8 @@ __device__ __forceinline__ float4 load_bounded_floats(__amdgpu_buffer_rsrc_t run
 // This thread's CH pieces of the product's input: asked for, and then made.
 template <int CH, int IN>
 struct Made {
-  static constexpr int ROWS = IN == IN_GRU ? 5 : (IN == IN_ROW ? 1 : 2), FLOATS = IN == IN_STREAM_NORM || IN == IN_GRU ? 2 : 1;
+  static constexpr bool STREAM = IN == IN_STREAM_NORM || IN == IN_STREAM_GROUPS;
+  static constexpr int ROWS = IN == IN_GRU ? 5 : (IN == IN_ROW ? 1 : 2), FLOATS = STREAM || IN == IN_GRU ? 2 : 1;
   uint4 v[ROWS][CH];
   float4 f[FLOATS][CH];
   int4 span;
@@ -54,7 +63,7 @@ struct Made {
   __device__ __forceinline__ void issue(const StreamIn& in, int K) {
     const bf16_t* x = reinterpret_cast<const bf16_t*>(in.x);
     const bf16_t* from[5] = {x, nullptr, nullptr, nullptr, nullptr};
-    if (IN == IN_STREAM_NORM) from[0] = in.gain;
+    if (STREAM) from[0] = in.gain;
     if (IN == IN_ROW_NORM) from[1] = in.gain;
     if (IN == IN_POLY) from[1] = in.b0;
     if (IN == IN_GRU) {
@@ -63,8 +72,8 @@ struct Made {
       from[3] = in.b0;
       from[4] = in.b1;
     }
-    constexpr int N = IN == IN_STREAM_NORM ? 1 : ROWS;
-    if (IN == IN_STREAM_NORM) {
+    constexpr int N = STREAM ? 1 : ROWS;
+    if (STREAM) {
       const __amdgpu_buffer_rsrc_t run = bounded_bytes(in.x, 4 * K);
 #pragma unroll
       for (int i = 0; i < CH; ++i)
@@ -87,10 +96,46 @@ struct Made {
     }
   }
 
-  __device__ __forceinline__ void finish(const StreamIn& in, int K, float (*part)[4], uint4 (&out)[CH]) {
+  // sums, inverses (IN_STREAM_GROUPS): LDS, a float a 16-byte piece of the row and one a group.
+  __device__ __forceinline__ void finish(const StreamIn& in, int K, float (*part)[4], uint4 (&out)[CH], float* sums = nullptr,
+                                         float* inverses = nullptr) {
     if (IN == IN_ROW) {
 #pragma unroll
       for (int i = 0; i < CH; ++i) out[i] = v[0][i];
+      return;
+    }
+    if (IN == IN_STREAM_GROUPS) {
+      float x[CH][8];
+      const int pieces = K / 8 / in.groups, lane = threadIdx.x & 63;
+#pragma unroll
+      for (int i = 0; i < CH; ++i) {
+        const float4 a = f[0][i], b = f[FLOATS - 1][i];
+        x[i][0] = a.x; x[i][1] = a.y; x[i][2] = a.z; x[i][3] = a.w;
+        x[i][4] = b.x; x[i][5] = b.y; x[i][6] = b.z; x[i][7] = b.w;
+        float sum = 0.f;
+#pragma unroll
+        for (int j = 0; j < 8; ++j) sum = fmaf(x[i][j], x[i][j], sum);
+        sums[threadIdx.x + 256 * i] = sum;
+      }
+      block_barrier_lds();
+      for (int g = threadIdx.x >> 6; g < in.groups; g += 4) {   // a wave a group
+        float sum = 0.f;
+        for (int c = lane; c < pieces; c += 64) sum += sums[g * pieces + c];
+        sum = wave_sum(sum);
+        if (lane == 0) inverses[g] = 1.0f / sqrtf(sum / (float)(pieces * 8) + in.eps);
+      }
+      block_barrier_lds();
+#pragma unroll
+      for (int i = 0; i < CH; ++i) {
+        float g[8];
+        const int c = threadIdx.x + 256 * i;
+        const float inv = inverses[min(c / pieces, in.groups - 1)];
+        unpack8(v[0][i], g);
+#pragma unroll
+        for (int j = 0; j < 8; ++j) x[i][j] = x[i][j] * inv * (in.unit + g[j]);
+        out[i] = pack8(x[i]);
+        if (blockIdx.x == 0 && in.made != nullptr && c < (K >> 3)) reinterpret_cast<uint4*>(in.made)[c] = out[i];
+      }
       return;
     }
     if (IN == IN_STREAM_NORM || IN == IN_ROW_NORM) {
@@ -188,6 +233,7 @@ struct Made {
 template <int RPW, int CH, int IN, int OUT>
 __global__ __launch_bounds__(256) void stream_product_kernel(const bf16_t* __restrict__ W, StreamIn in, StreamOut out, int M, int K) {
   __shared__ float part[3][4], sums[4][RPW];
+  __shared__ float piece_sums[IN == IN_STREAM_GROUPS ? CH * 256 : 1], inverses[IN == IN_STREAM_GROUPS ? MOST_GROUPS : 1];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, row0 = blockIdx.x * RPW;
   if (OUT == OUT_LATENT && row0 >= M) {   // the one block behind the product's
     const int4 span = *reinterpret_cast<const int4*>(in.spans);
@@ -200,10 +246,19 @@ __global__ __launch_bounds__(256) void stream_product_kernel(const bf16_t* __res
   made.issue(in, K);
   uint4 w[RPW][CH];
 #pragma unroll
-  for (int r = 0; r < RPW; ++r) load_row<CH>(W + (size_t)min(row0 + r, M - 1) * K, K, w[r]);
+  for (int r = 0; r < RPW; ++r) {
+    const int row = row0 + r;
+    const bf16_t* from = OUT == OUT_LOGITS && row >= M ? out.router + (size_t)min(row - M, out.logits - 1) * K : W + (size_t)min(row, M - 1) * K;
+    load_row<CH>(from, K, w[r]);
+  }
   // What the output's threads need at the end, asked for by all of them ahead of the wait.
   float held = 0.f;
   bf16_t yb = 0, gate = 0, gb = 0;
+  if (OUT == OUT_ADD) {
+    const int row = min(row0 + min((int)threadIdx.x, RPW - 1), M - 1);
+    held = out.stream[row];
+    if (out.y_bias != nullptr) yb = out.y_bias[row];
+  }
   if (OUT == OUT_GATED) {
     const int row = min(row0 + min((int)threadIdx.x, RPW - 1), M - 1);
     held = out.stream[row];
@@ -212,7 +267,7 @@ __global__ __launch_bounds__(256) void stream_product_kernel(const bf16_t* __res
     if (out.y_bias != nullptr) yb = out.y_bias[row];
   }
   uint4 x[CH];
-  made.finish(in, K, part, x);
+  made.finish(in, K, part, x, piece_sums, inverses);
 #pragma unroll
   for (int r = 0; r < RPW; ++r) {
     const float a = wave_sum(dot_row<CH>(w[r], x));
@@ -220,8 +275,16 @@ __global__ __launch_bounds__(256) void stream_product_kernel(const bf16_t* __res
   }
   __syncthreads();
   const int r = threadIdx.x, row = row0 + r;
-  if (r >= RPW || row >= M) return;
-  const float v = round_bf16(sums[0][r] + sums[1][r] + sums[2][r] + sums[3][r]);
+  if (r >= RPW || row >= (OUT == OUT_LOGITS ? M + out.logits : M)) return;
+  const float whole = sums[0][r] + sums[1][r] + sums[2][r] + sums[3][r], v = round_bf16(whole);
+  if (OUT == OUT_LOGITS && row >= M) {
+    out.z[row - M] = whole;
+    return;
+  }
+  if (OUT == OUT_ADD) {
+    out.stream[row] = held + (out.y_bias != nullptr ? v + bf16_to_f32(yb) : v);
+    return;
+  }
   if (OUT == OUT_GATED) out.stream[row] = held + (v + bf16_to_f32(yb)) * (1.0f / (1.0f + expf(-(bf16_to_f32(gate) + bf16_to_f32(gb)))));
   else out.y[row] = f32_to_bf16(v);
 }
@@ -231,13 +294,13 @@ static int launch_stream_product(const bf16_t* W, const StreamIn& in, const Stre
   const int ch = K <= 2048 ? 1 : (K <= 4096 ? 2 : (K <= 8192 ? 4 : 8));
 #define IRON_PRODUCT(RPW, CH)                                                                                                     \
   {                                                                                                                               \
-    const int blocks = (M + RPW - 1) / RPW + (OUT == OUT_LATENT ? 1 : 0);                                                         \
+    const int rows = OUT == OUT_LOGITS ? M + out.logits : M, blocks = (rows + RPW - 1) / RPW + (OUT == OUT_LATENT ? 1 : 0);                                                         \
     hipLaunchKernelGGL((stream_product_kernel<RPW, CH, IN, OUT>), dim3(blocks), dim3(256), 0, s, W, in, out, M, K);               \
     IRON_LAUNCH_CHECK();                                                                                                          \
   }
   // Rows a block takes (measured): more where the input is long in the making and the matrix is tall.
-  constexpr bool MADE = IN == IN_STREAM_NORM || IN == IN_GRU;
-  if (ch == 1 && IN == IN_STREAM_NORM && M >= 8192) IRON_PRODUCT(8, 1)
+  constexpr bool NORM = IN == IN_STREAM_NORM || IN == IN_STREAM_GROUPS, MADE = NORM || IN == IN_GRU;
+  if (ch == 1 && NORM && M >= 8192) IRON_PRODUCT(8, 1)
   if (ch == 1 && IN == IN_GRU) IRON_PRODUCT(4, 1)
   if (ch == 1 && M > 2048) IRON_PRODUCT(2, 1)
   if (ch == 1) IRON_PRODUCT(1, 1)
@@ -265,7 +328,7 @@ extern "C" int iron_stream_product_bf16(int input, const void* x, const uint16_t
   IRON_REQUIRE(stream_row == nullptr || input != IN_STREAM_NORM, "stream_product: the stream is an input or the output");
   IRON_REQUIRE((((uintptr_t)x | (uintptr_t)W | (uintptr_t)b0 | (uintptr_t)b1 | (uintptr_t)state | (uintptr_t)spans |
                  (input == IN_POLY ? 0 : (uintptr_t)gain)) & 15) == 0, "stream_product: operands must be 16-byte aligned");
-  const StreamIn in{x, gain, b0, b1, state, spans, eps, unit};
+  const StreamIn in{x, gain, b0, b1, state, spans, eps, unit, 1, nullptr};
   StreamOut out{};
   out.y = y;
   out.stream = stream_row;
@@ -285,6 +348,35 @@ extern "C" int iron_stream_product_bf16(int input, const void* x, const uint16_t
   IRON_REQUIRE(false, "stream_product: input %d is served into a row only", input);
 }
 
+extern "C" int iron_norm_product_bf16(const float* x, const uint16_t* gain, int groups, float eps, float unit, const uint16_t* W, int M, int K,
+                                      uint16_t* y, uint16_t* h, const uint16_t* router, int logits, float* z, void* stream) {
+  IRON_REQUIRE(x && gain && W && y && (router == nullptr || z), "norm_product: null operand");
+  IRON_REQUIRE(M > 0 && K > 0 && K % 8 == 0 && K <= 8 * 2048, "norm_product: M (%d) positive, K (%d) a multiple of 8 up to %d", M, K, 8 * 2048);
+  IRON_REQUIRE(groups > 0 && groups <= MOST_GROUPS && K % (8 * groups) == 0, "norm_product: K (%d) in equal groups (%d, up to %d) of whole 16-byte pieces", K,
+               groups, MOST_GROUPS);
+  IRON_REQUIRE(router == nullptr || logits > 0, "norm_product: logits (%d) must be positive", logits);
+  IRON_REQUIRE((((uintptr_t)x | (uintptr_t)gain | (uintptr_t)W | (uintptr_t)h | (uintptr_t)router) & 15) == 0, "norm_product: operands must be 16-byte aligned");
+  const StreamIn in{x, gain, nullptr, nullptr, nullptr, nullptr, eps, unit, groups, h};
+  StreamOut out{};
+  out.y = y;
+  out.router = router;
+  out.z = z;
+  out.logits = logits;
+  if (router != nullptr) return launch_stream_product<IN_STREAM_GROUPS, OUT_LOGITS>(W, in, out, M, K, (hipStream_t)stream);
+  return launch_stream_product<IN_STREAM_GROUPS, OUT_ROW>(W, in, out, M, K, (hipStream_t)stream);
+}
+
+extern "C" int iron_product_sum_bf16(const uint16_t* x, const uint16_t* W, int M, int K, const uint16_t* also, float* stream_row, void* stream) {
+  IRON_REQUIRE(x && W && stream_row, "product_sum: null operand");
+  IRON_REQUIRE(M > 0 && K > 0 && K % 8 == 0 && K <= 8 * 2048, "product_sum: M (%d) positive, K (%d) a multiple of 8 up to %d", M, K, 8 * 2048);
+  IRON_REQUIRE((((uintptr_t)x | (uintptr_t)W) & 15) == 0, "product_sum: operands must be 16-byte aligned");
+  const StreamIn in{x, nullptr, nullptr, nullptr, nullptr, nullptr, 0.f, 0.f, 1, nullptr};
+  StreamOut out{};
+  out.stream = stream_row;
+  out.y_bias = also;
+  return launch_stream_product<IN_ROW, OUT_ADD>(W, in, out, M, K, (hipStream_t)stream);
+}
+
 extern "C" int iron_latent_query_bf16(const uint16_t* x, const uint16_t* q_gain, const uint16_t* c_gain, const float* angles, const int* spans,
                                       const uint16_t* W, uint16_t* q, uint16_t* latents, uint16_t* shared_keys, int M, int stride, int q_rank,
                                       int rank, int rot, int turned, int angle_rows, int ring, float eps, void* stream) {
@@ -297,7 +389,7 @@ extern "C" int iron_latent_query_bf16(const uint16_t* x, const uint16_t* q_gain,
   IRON_REQUIRE(turned <= rot && (turned == 0 || (angles && angle_rows > 0)), "latent_query: %d of %d columns turn, by a table of %d rows", turned, rot, angle_rows);
   IRON_REQUIRE((((uintptr_t)x | (uintptr_t)q_gain | (uintptr_t)c_gain | (uintptr_t)spans | (uintptr_t)W | (uintptr_t)latents | (uintptr_t)shared_keys) & 15) == 0,
                "latent_query: operands must be 16-byte aligned");
-  const StreamIn in{x, q_gain, nullptr, nullptr, nullptr, spans, eps, 0.f};
+  const StreamIn in{x, q_gain, nullptr, nullptr, nullptr, spans, eps, 0.f, 1, nullptr};
   StreamOut out{};
   out.y = q;
   out.row = x;

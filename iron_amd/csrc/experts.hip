@@ -8,86 +8,9 @@
 #include "../../include/iron_hip.h"
 #include "grouped.h"
 #include "row_products.h"
-#include "rows.h"
+#include "router.h"
 
 namespace iron {
-
-constexpr int ROUTER_MAX = 1024;   // experts
-
-// The `top` largest of n logits in LDS by one wave, in order, the first of equal ones first; their shares.
-__device__ __forceinline__ void choose(float* __restrict__ z, int n, int top, int* __restrict__ ids, float* __restrict__ shares) {
-  const int lane = threadIdx.x & 63;
-  float first = 0.f, total = 0.f, mine = 0.f;
-  for (int k = 0; k < top; ++k) {
-    float best = -INFINITY;
-    int at = n;
-    for (int i = lane; i < n; i += 64)
-      if (z[i] > best) {
-        best = z[i];
-        at = i;
-      }
-    const float most = wave_max(best);
-    // (no logit above -inf, or none that is a number: the first expert)
-    const unsigned long long here = __builtin_amdgcn_ballot_w64(best == most && at < n);
-    int id = n;
-    for (unsigned long long left = here; left != 0; left &= left - 1) id = min(id, __shfl(at, __builtin_ctzll(left), 64));
-    if (id >= n) id = 0;
-    if (k == 0) first = most;
-    const float e = expf(most - first);
-    total += e;
-    if (lane == k) mine = e;
-    if (lane == 0) {
-      ids[k] = id;
-      z[id] = -INFINITY;
-    }
-    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
-    __builtin_amdgcn_wave_barrier();
-  }
-  if (lane < top) shares[lane] = mine / total;
-}
-
-// The `top` largest of the n scores (a softmax over the logits z) plus corrections by one wave, in order, the first of equal ones
-// first; their shares, the scores over their sum.  z and by: LDS.
-__device__ __forceinline__ void choose_scored(float* __restrict__ z, float* __restrict__ by, const bf16_t* __restrict__ correction, int n, int top,
-                                              int* __restrict__ ids, float* __restrict__ shares) {
-  const int lane = threadIdx.x & 63;
-  float most = -INFINITY, total = 0.f;
-  for (int i = lane; i < n; i += 64) most = fmaxf(most, z[i]);
-  most = wave_max(most);
-  for (int i = lane; i < n; i += 64) total += expf(z[i] - most);
-  total = wave_sum(total);
-  for (int i = lane; i < n; i += 64) {   // (a lane reads what it wrote)
-    z[i] = expf(z[i] - most) / total;
-    by[i] = z[i] + (correction != nullptr ? bf16_to_f32(correction[i]) : 0.f);
-  }
-  float sum = 0.f, mine = 0.f;
-  for (int k = 0; k < top; ++k) {
-    float best = -INFINITY, score = 0.f;
-    int at = n;
-    for (int i = lane; i < n; i += 64)
-      if (by[i] > best) {
-        best = by[i];
-        score = z[i];
-        at = i;
-      }
-    const float largest = wave_max(best);
-    int id = n, from = 0;
-    for (unsigned long long left = __builtin_amdgcn_ballot_w64(best == largest && at < n); left != 0; left &= left - 1) {
-      const int l = __builtin_ctzll(left), other = __shfl(at, l, 64);
-      if (other < id) {
-        id = other;
-        from = l;
-      }
-    }
-    score = __shfl(score, from, 64);
-    if (id >= n) id = 0;   // (none that is a number: the first)
-    sum += score;
-    if (lane == k) mine = score;
-    if (lane == 0) ids[k] = id;
-    if (lane == (id & 63)) by[id] = -INFINITY;
-  }
-  if (lane < top) shares[lane] = mine / (sum + 1e-20f);
-}
 
 template <typename T, int VEC, int NW>
 __global__ __launch_bounds__(NW * 64) void router_kernel(const T* __restrict__ h, const bf16_t* __restrict__ w, const bf16_t* __restrict__ bias,
@@ -121,9 +44,6 @@ __global__ __launch_bounds__(NW * 64) void router_kernel(const T* __restrict__ h
 __device__ __forceinline__ float act_exact(int kind, float g) {
   return kind == 3 ? fmaxf(g, 0.f) : (kind == 1 ? g / (1.f + expf(-g)) : gelu_tanh_f32(g));
 }
-
-// The expert an id names, -1 for one of the identities behind the last.
-__device__ __forceinline__ int expert_of(int id, int experts, int identity) { return identity > 0 && id >= experts ? -1 : min(max(id, 0), experts - 1); }
 
 // VEC elements of a row and of a weight's row, and their product: bf16 pairs as they were loaded, or floats.
 template <typename T, int VEC>
@@ -358,6 +278,52 @@ __global__ __launch_bounds__(256) void expert_gather_kernel(const bf16_t* __rest
   store_vec<8>(y + (size_t)row * cols + c, sum);
 }
 
+// One row: stream[c] += out_c . made + what its experts make of column c: a block a column, its row of `out` and its experts' rows of
+// down as one run of 16-byte pieces.
+constexpr int TAIL_EXPERTS = 64;
+template <int CH>
+__global__ __launch_bounds__(256) void expert_tail_kernel(const bf16_t* __restrict__ out, const bf16_t* __restrict__ made, int inner,
+                                                          const bf16_t* __restrict__ down, const bf16_t* __restrict__ acts,
+                                                          const int* __restrict__ ids, const float* __restrict__ shares,
+                                                          const bf16_t* __restrict__ h, float* __restrict__ stream, int cols, int ff, int experts,
+                                                          int identity, int top) {
+  __shared__ float red[2][4];
+  const int c = blockIdx.x, t = threadIdx.x, lane = t & 63, wave = t >> 6, first = inner / 8, each = ff / 8, pieces = first + top * each;
+  const float held = stream[c], own = bf16_to_f32(h[c]);
+  const float share_own = lane < top ? shares[lane] : 0.f;
+  const int id_own = lane < top ? expert_of(ids[lane], experts, identity) : 0;
+  uint4 w[CH], x[CH];
+  float by[CH];
+#pragma unroll
+  for (int i = 0; i < CH; ++i) {
+    const int p = min(t + 256 * i, pieces - 1), k = p < first ? 0 : (p - first) / each, e = __shfl(id_own, k, 64);
+    const int at = p < first ? p : (p - first) - k * each;
+    const float share = __shfl(share_own, k, 64);
+    by[i] = p < first ? 1.f : share;
+    if (t + 256 * i >= pieces || (p >= first && e < 0)) by[i] = 0.f;
+    w[i] = load_stream(reinterpret_cast<const uint4*>(p < first ? out + (size_t)c * inner : down + ((size_t)max(e, 0) * cols + c) * ff) + at);
+    x[i] = reinterpret_cast<const uint4*>(p < first ? made : acts + (size_t)k * ff)[at];
+  }
+  float mixed = 0.f, routed = 0.f;
+#pragma unroll
+  for (int i = 0; i < CH; ++i) {
+    const uint4 a[1] = {w[i]}, b[1] = {x[i]};
+    const float part = by[i] == 0.f ? 0.f : dot_row<1>(a, b);   // (an identity's activated row is nobody's)
+    if (t + 256 * i < first) mixed += part;
+    else routed = fmaf(by[i], part, routed);
+  }
+  if (wave == 0 && lane < top && id_own < 0) routed = fmaf(share_own, own, routed);
+  mixed = wave_sum(mixed);
+  routed = wave_sum(routed);
+  if (lane == 0) {
+    red[0][wave] = mixed;
+    red[1][wave] = routed;
+  }
+  __syncthreads();
+  if (t == 0)
+    stream[c] = held + (round_bf16(red[0][0] + red[0][1] + red[0][2] + red[0][3]) + round_bf16(red[1][0] + red[1][1] + red[1][2] + red[1][3]));
+}
+
 // Rows from which a portion's pairs are grouped.
 static bool grouped_pays(int rows, int cols, int ff, int is_float) { return !is_float && rows >= 64 && cols % 64 == 0 && ff % 64 == 0; }
 
@@ -435,5 +401,31 @@ extern "C" int iron_experts(const void* h, const uint16_t* gate, const uint16_t*
   if (is_float) { if (vec) IRON_PAIRS(float, 8) else IRON_PAIRS(float, 1) }
   else { if (vec) IRON_PAIRS(bf16_t, 8) else IRON_PAIRS(bf16_t, 1) }
 #undef IRON_PAIRS
+  IRON_LAUNCH_CHECK();
+}
+
+extern "C" int iron_experts_tail_bf16(const uint16_t* h, const uint16_t* gate, const uint16_t* up, const uint16_t* down, const int* ids, const float* shares,
+                                      const uint16_t* out, const uint16_t* made, float* stream_row, void* workspace, int cols, int ff, int inner,
+                                      int experts, int identity, int top, int activation, void* stream) {
+  IRON_REQUIRE(h && gate && up && down && ids && shares && out && made && stream_row && workspace, "experts_tail: null operand");
+  IRON_REQUIRE(cols > 0 && ff > 0 && inner > 0 && experts > 0 && identity >= 0 && top > 0 && top <= experts + identity && top <= TAIL_EXPERTS,
+               "experts_tail: sizes must be positive, top (%d) of %d experts and %d identities, at most %d", top, experts, identity, TAIL_EXPERTS);
+  IRON_REQUIRE(activation >= 1 && activation <= 3, "experts_tail: activation (%d) is 1 (SiLU), 2 (GELU, tanh form) or 3 (ReLU)", activation);
+  IRON_REQUIRE(cols % 8 == 0 && ff % 8 == 0 && inner % 8 == 0 &&
+                   (((uintptr_t)h | (uintptr_t)gate | (uintptr_t)up | (uintptr_t)down | (uintptr_t)out | (uintptr_t)made | (uintptr_t)workspace) & 15) == 0,
+               "experts_tail: rows (%d, %d, %d) of whole 16-byte pieces, 16-byte aligned", cols, ff, inner);
+  const int pieces = inner / 8 + top * (ff / 8);
+  IRON_REQUIRE(pieces <= 16 * 256, "experts_tail: a column's weights (%d) exceed %d pieces", pieces, 16 * 256);
+  hipStream_t s = (hipStream_t)stream;
+  bf16_t* acts = (bf16_t*)workspace;
+  hipLaunchKernelGGL((expert_pairs_kernel<bf16_t, 8>), dim3((ff + 3) / 4, top), dim3(256), 0, s, h, gate, up, ids, acts, 1, cols, ff, experts, identity, top,
+                     activation, nullptr);
+#define IRON_TAIL(CH) \
+  hipLaunchKernelGGL((expert_tail_kernel<CH>), dim3(cols), dim3(256), 0, s, out, made, inner, down, acts, ids, shares, h, stream_row, cols, ff, experts, identity, top)
+  if (pieces <= 512) IRON_TAIL(2);
+  else if (pieces <= 1024) IRON_TAIL(4);
+  else if (pieces <= 2048) IRON_TAIL(8);
+  else IRON_TAIL(16);
+#undef IRON_TAIL
   IRON_LAUNCH_CHECK();
 }

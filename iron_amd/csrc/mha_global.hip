@@ -14,6 +14,7 @@
 // Scores behind a cap are bounded.  Where their exponentials cannot leave a float's range either way (SCORES_FIXED) they are taken
 // as they are: no largest score is looked for and nothing is rescaled.
 #include "../../include/iron_hip.h"
+#include "router.h"
 #include "window.h"
 
 namespace iron {
@@ -33,21 +34,16 @@ struct CacheIn {
   const float* angles;                   // [angle_rows][turned]: cos and sin side by side
 };
 
-// LANES lanes a head, 8 consecutive columns each (VEC), or a wave a head, column by column.
+// LANES lanes a head, 8 consecutive columns each (VEC), or a wave a head, column by column.  A row's heads from unit `first` on,
+// every `step`-th set of as many as the block takes at once.
 template <typename T, int LANES, bool VEC>
-__global__ __launch_bounds__(256) void cached_heads_kernel(const T* __restrict__ x, T* __restrict__ q, T* __restrict__ keys,
-                                                           T* __restrict__ values, const int* __restrict__ spans, CacheIn in, CacheShape a,
-                                                           const int* __restrict__ valid) {
-  const int row = blockIdx.x;
-  if (row >= bound_or(valid, a.rows)) return;
-  const int slot = slot_of_row(spans, a.slots, a.rows, row);
-  if (slot < 0) return;
-  const Span s = span_of(spans, slot, a.rows);
+__device__ __forceinline__ void cached_row(const T* __restrict__ x, T* __restrict__ q, T* __restrict__ keys, T* __restrict__ values, const CacheIn& in,
+                                           const CacheShape& a, const Span& s, int slot, int row, int first, int step) {
   const int pos = s.start + row - s.row0, half = a.turned / 2;
   if (pos >= a.context) return;
   const float* turn = in.angles + (size_t)min(pos, a.angle_rows - 1) * a.turned;
   const int lane = threadIdx.x % LANES, qk = a.heads + a.kv_heads, units = qk + a.kv_heads;
-  for (int u = threadIdx.x / LANES; u < units; u += 256 / LANES) {
+  for (int u = first + threadIdx.x / LANES; u < units; u += step) {
     const bool value = u >= qk, query = u < a.heads;
     const int at = value ? qk * a.dim + (u - qk) * a.vdim : u * a.dim, n = value ? a.vdim : a.dim;
     const T* xr = x + (size_t)row * a.stride + at;
@@ -110,6 +106,47 @@ __global__ __launch_bounds__(256) void cached_heads_kernel(const T* __restrict__
       for (int c = lane; c < n; c += LANES) store_one(to + c, made(c, load_one(xr + c)));
     }
   }
+}
+
+template <typename T, int LANES, bool VEC>
+__global__ __launch_bounds__(256) void cached_heads_kernel(const T* __restrict__ x, T* __restrict__ q, T* __restrict__ keys,
+                                                           T* __restrict__ values, const int* __restrict__ spans, CacheIn in, CacheShape a,
+                                                           const int* __restrict__ valid) {
+  const int row = blockIdx.x;
+  if (row >= bound_or(valid, a.rows)) return;
+  const int slot = slot_of_row(spans, a.slots, a.rows, row);
+  if (slot < 0) return;
+  cached_row<T, LANES, VEC>(x, q, keys, values, in, a, span_of(spans, slot, a.rows), slot, row, blockIdx.y * (256 / LANES), gridDim.y * (256 / LANES));
+}
+
+// One row a slot, bf16: its heads dealt to the first blocks, beside them a feed-forward's gated columns of the row, and a router's
+// choice for slot 0.
+struct StepColumns {
+  bf16_t* out;                            // the rows the columns go to
+  int out_stride, cols, gate_at, gated_at, kind;
+  float limit;
+};
+template <int LANES>
+__global__ __launch_bounds__(256) void decode_heads_kernel(const bf16_t* __restrict__ x, bf16_t* __restrict__ q, bf16_t* __restrict__ keys,
+                                                           bf16_t* __restrict__ values, const int* __restrict__ spans, CacheIn in, CacheShape a,
+                                                           StepColumns g, RouterChoice choice) {
+  constexpr int AT_ONCE = 256 / LANES;
+  __shared__ float lds[2][ROUTER_MAX];
+  const int slot = blockIdx.y, head_blocks = (a.heads + 2 * a.kv_heads + AT_ONCE - 1) / AT_ONCE, block = blockIdx.x;
+  const Span s = span_of(spans, slot, a.rows);
+  if (choice.z != nullptr && block == (int)gridDim.x - 1) {   // (whether the slot has a row or not, as the router by itself)
+    choose_row(choice, lds[0], lds[1]);
+    return;
+  }
+  if (s.rows == 0) return;
+  if (block < head_blocks) {
+    cached_row<bf16_t, LANES, true>(x, q, keys, values, in, a, s, slot, s.row0, block * AT_ONCE, 1 << 30);
+    return;
+  }
+  const int c = (block - head_blocks) * 256 + threadIdx.x;
+  const bf16_t* row = x + (size_t)s.row0 * a.stride + g.gate_at;
+  if (c < g.cols)
+    g.out[(size_t)s.row0 * g.out_stride + g.gated_at + c] = f32_to_bf16(gated_value(g.kind, g.limit, bf16_to_f32(row[c]), bf16_to_f32(row[g.cols + c])));
 }
 
 // ------------------------------------------------------------ row by row
@@ -678,7 +715,7 @@ extern "C" int iron_cached_heads(const void* x, void* q, void* keys, void* value
   const bool vec = dim % 8 == 0 && vdim % 8 == 0 && stride % 8 == 0 && wide <= 512 &&
                    (((uintptr_t)x | (uintptr_t)q | (uintptr_t)keys | (uintptr_t)values | (uintptr_t)q_gain | (uintptr_t)k_gain) & 15) == 0;
 #define IRON_HEADS(T, LANES, VEC)                                                                                                          \
-  hipLaunchKernelGGL((cached_heads_kernel<T, LANES, VEC>), dim3(rows), dim3(256), 0, (hipStream_t)stream, (const T*)x, (T*)q, (T*)keys, \
+  hipLaunchKernelGGL((cached_heads_kernel<T, LANES, VEC>), dim3(rows, rows < 256 ? (heads + 2 * kv_heads + 256 / LANES - 1) / (256 / LANES) : 1), dim3(256), 0, (hipStream_t)stream, (const T*)x, (T*)q, (T*)keys, \
                      (T*)values, spans, in, a, valid)
 #define IRON_HEADSS(T)                              \
   {                                                 \
@@ -692,6 +729,41 @@ extern "C" int iron_cached_heads(const void* x, void* q, void* keys, void* value
   else IRON_HEADSS(bf16_t)
 #undef IRON_HEADSS
 #undef IRON_HEADS
+  IRON_LAUNCH_CHECK();
+}
+
+extern "C" int iron_decode_heads_global_bf16(const uint16_t* x, uint16_t* q, uint16_t* keys, uint16_t* values, const uint16_t* q_gain,
+                                             const uint16_t* k_gain, const float* angles, const int* spans, int slots, int rows, int stride,
+                                             int heads, int kv_heads, int dim, int vdim, int context, int turned, int angle_rows, int value_norm,
+                                             float eps, uint16_t* out, int out_stride, int cols, int gate_at, int gated_at, int kind, float limit,
+                                             const float* z, const uint16_t* correction, int logits, int top, int* ids, float* shares,
+                                             void* stream) {
+  IRON_REQUIRE(x && q && keys && values && q_gain && k_gain && spans && (turned == 0 || angles), "decode_heads_global: null operand");
+  IRON_REQUIRE(((uintptr_t)spans & 15) == 0 && ((uintptr_t)angles & 7) == 0, "decode_heads_global: spans must be 16-byte aligned");
+  IRON_REQUIRE(slots > 0 && slots <= 65535 && rows > 0 && heads > 0 && kv_heads > 0 && dim > 0 && vdim > 0 && context > 0,
+               "decode_heads_global: sizes must be positive");
+  IRON_REQUIRE(turned >= 0 && turned % 2 == 0 && turned <= dim && angle_rows > 0, "decode_heads_global: %d of %d columns turn, in pairs", turned, dim);
+  IRON_REQUIRE(stride >= heads * dim + kv_heads * (dim + vdim), "decode_heads_global: a row of %d holds no q, k and v of %d heads", stride, heads);
+  const int wide = dim > vdim ? dim : vdim;
+  IRON_REQUIRE(dim % 8 == 0 && vdim % 8 == 0 && stride % 8 == 0 && wide <= 256 &&
+                   (((uintptr_t)x | (uintptr_t)q | (uintptr_t)keys | (uintptr_t)values | (uintptr_t)q_gain | (uintptr_t)k_gain) & 15) == 0,
+               "decode_heads_global: heads of whole 16-byte pieces up to 256 columns");
+  IRON_REQUIRE(cols >= 0 && (cols == 0 || (out && gate_at >= 0 && gate_at + 2 * cols <= stride && gated_at >= 0 && gated_at + cols <= out_stride)),
+               "decode_heads_global: twice %d gated columns from %d, into those from %d", cols, gate_at, gated_at);
+  IRON_REQUIRE(kind >= 0 && kind <= 3, "decode_heads_global: kind (%d) is 0 to 3", kind);
+  IRON_ROUTER_CHOICE_REQUIRE("decode_heads_global");
+  const CacheIn in{q_gain, k_gain, angles};
+  const CacheShape a{rows, stride, slots, heads, kv_heads, dim, vdim, context, turned, angle_rows, value_norm, eps};
+  const StepColumns g{out, out_stride, cols, gate_at, gated_at, kind, limit};
+  const RouterChoice choice{z, correction, logits, top, ids, shares};
+#define IRON_STEP_HEADS(LANES)                                                                                                                    \
+  hipLaunchKernelGGL((decode_heads_kernel<LANES>),                                                                                                \
+                     dim3((heads + 2 * kv_heads + 256 / LANES - 1) / (256 / LANES) + (cols + 255) / 256 + (z != nullptr), slots), dim3(256), 0,    \
+                     (hipStream_t)stream, x, q, keys, values, spans, in, a, g, choice)
+  if (wide <= 64) IRON_STEP_HEADS(8);
+  else if (wide <= 128) IRON_STEP_HEADS(16);
+  else IRON_STEP_HEADS(32);
+#undef IRON_STEP_HEADS
   IRON_LAUNCH_CHECK();
 }
 

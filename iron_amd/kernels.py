@@ -697,9 +697,21 @@ def hgrn2(x, f_bias, lower, state, spans, o, *, slots, rows, stride, heads, dim,
     check(lib().iron_hgrn2(ptr(x), ptr(f_bias), ptr(lower), ptr(state), _spans(spans, slots), ptr(o), *sizes), "iron_hgrn2")
 
 
+def _choice(z, correction, logits, top, ids, shares):
+    """A router's choice beside a step's mixer: the C ABI's arguments for it."""
+    if z is None:
+        return None, None, 0, 0, None, None
+    _f32(z, logits, "z")
+    if correction is not None:
+        _bf16(correction, logits, "correction")
+    _numel(_dev(ids, "ids", torch.int32), top, "ids")
+    _f32(shares, top, "shares")
+    return ptr(z), ptr(correction), logits, top, ptr(ids), ptr(shares)
+
+
 def decode_hgrn2(x, f_bias, lower, norm, state, spans, out, *, slots, rows, stride, heads, dim, vdim, out_stride, out_at, eps, cols=0, gate_at=0,
-                 gated_at=0, kind="limited", limit=0.0):
-    """A decode step's forget gate, fading memory and head norm beside a feed-forward's gated columns."""
+                 gated_at=0, kind="limited", limit=0.0, z=None, correction=None, logits=0, top=0, ids=None, shares=None):
+    """A decode step's forget gate, fading memory and head norm beside a feed-forward's gated columns and a router's choice."""
     _bf16(x, rows * stride, "x")
     _bf16(f_bias, heads * dim, "f_bias")
     _bf16(lower, heads * dim, "lower")
@@ -708,7 +720,66 @@ def decode_hgrn2(x, f_bias, lower, norm, state, spans, out, *, slots, rows, stri
     _bf16(out, rows * out_stride, "out")
     check(lib().iron_decode_hgrn2_bf16(ptr(x), ptr(f_bias), ptr(lower), ptr(norm), ptr(state), _spans(spans, slots), ptr(out), slots, rows, stride,
                                        heads, dim, vdim, out_stride, out_at, float(eps), cols, gate_at, gated_at, COLUMN_GATES[kind], float(limit),
-                                       current_stream()), "iron_decode_hgrn2_bf16")
+                                       *_choice(z, correction, logits, top, ids, shares), current_stream()), "iron_decode_hgrn2_bf16")
+
+
+def decode_heads_global(x, q, keys, values, q_gain, k_gain, spans, *, slots, rows, stride, heads, kv_heads, dim, vdim, context, eps, turned=0,
+                        angle_rows=1, angles=None, value_norm=False, out=None, out_stride=0, cols=0, gate_at=0, gated_at=0, kind="limited", limit=0.0,
+                        z=None, correction=None, logits=0, top=0, ids=None, shares=None):
+    """A decode step's heads into their caches beside a feed-forward's gated columns and a router's choice."""
+    _bf16(x, rows * stride, "x")
+    _bf16(q, rows * heads * dim, "q")
+    _bf16(keys, slots * kv_heads * context * dim, "keys")
+    _bf16(values, slots * kv_heads * context * vdim, "values")
+    _bf16(q_gain, dim, "q_gain")
+    _bf16(k_gain, dim, "k_gain")
+    if cols:
+        _bf16(out, rows * out_stride, "out")
+    check(lib().iron_decode_heads_global_bf16(ptr(x), ptr(q), ptr(keys), ptr(values), ptr(q_gain), ptr(k_gain), _turned(angles, angle_rows, turned),
+                                              _spans(spans, slots), slots, rows, stride, heads, kv_heads, dim, vdim, context, turned, angle_rows,
+                                              int(value_norm), float(eps), ptr(out), out_stride, cols, gate_at, gated_at, COLUMN_GATES[kind],
+                                              float(limit), *_choice(z, correction, logits, top, ids, shares), current_stream()),
+          "iron_decode_heads_global_bf16")
+
+
+def norm_product(x, gain, W, y, *, M, K, groups, eps, unit=0.0, h=None, router=None, z=None, logits=0):
+    """One row: the stream's, normed in groups, through ``W``; the normed row to ``h`` too, and with ``router`` its logits to ``z``."""
+    _f32(x, K, "x")
+    _bf16(gain, K, "gain")
+    _bf16(W, M * K, "W")
+    _bf16(y, M, "y")
+    if h is not None:
+        _bf16(h, K, "h")
+    if router is not None:
+        _bf16(router, logits * K, "router")
+        _f32(z, logits, "z")
+    check(lib().iron_norm_product_bf16(ptr(x), ptr(gain), groups, float(eps), float(unit), ptr(W), M, K, ptr(y), ptr(h), ptr(router), logits, ptr(z),
+                                       current_stream()), "iron_norm_product_bf16")
+
+
+def product_sum(x, W, stream, *, M, K, also=None):
+    """One row: ``stream += W x + also``."""
+    _bf16(x, K, "x")
+    _bf16(W, M * K, "W")
+    _f32(stream, M, "stream")
+    if also is not None:
+        _bf16(also, M, "also")
+    check(lib().iron_product_sum_bf16(ptr(x), ptr(W), M, K, ptr(also), ptr(stream), current_stream()), "iron_product_sum_bf16")
+
+
+def experts_tail(h, gate, up, down, ids, shares, out, made, stream, workspace, *, cols, ff, inner, experts, top, activation, identity=0):
+    """One row: its experts, and with their sums ``out`` times ``made``, both onto the stream's row."""
+    _bf16(h, cols, "h")
+    for t, name in ((gate, "gate"), (up, "up"), (down, "down")):
+        _bf16(t, experts * ff * cols, name)
+    _numel(_dev(ids, "ids", torch.int32), top, "ids")
+    _f32(shares, top, "shares")
+    _bf16(out, cols * inner, "out")
+    _bf16(made, inner, "made")
+    _f32(stream, cols, "stream")
+    check(lib().iron_experts_tail_bf16(ptr(h), ptr(gate), ptr(up), ptr(down), ptr(ids), ptr(shares), ptr(out), ptr(made), ptr(stream),
+                                       _work(workspace, 2 * top * ff, "experts_tail: workspace"), cols, ff, inner, experts, identity, top,
+                                       GATES[activation], current_stream()), "iron_experts_tail_bf16")
 
 
 def cached_heads(x, q, keys, values, q_gain, k_gain, spans, *, slots, rows, stride, heads, kv_heads, dim, vdim, context, eps, turned=0,

@@ -430,8 +430,12 @@ class ExpertsMLP(iron.Graph):
         self.down = iron.param(experts * width, inner)
 
     def body(self, h):
-        ids, shares = Router.step(h, self.router, bias=self.router_bias, correction=self.correction, scored=self.scored, top=self.top,
-                                  dtype=self.dtype)
+        return self.apply(h, *self.choose(h))
+
+    def choose(self, h):
+        return Router.step(h, self.router, bias=self.router_bias, correction=self.correction, scored=self.scored, top=self.top, dtype=self.dtype)
+
+    def apply(self, h, ids, shares):
         return Experts.step(h, self.gate, self.up, self.down, ids, shares, activation=self.kind, identity=self.identity, dtype=self.dtype)
 
 
@@ -517,9 +521,10 @@ class SideBySideLayer(iron.Graph):
     def body(self, x, call, state):
         rows, h = x.shape[0], self.norm1(x)
         packed = as_rows(self.proj(h), rows)
+        chosen = self.routed.choose(h) if self.routed is not None else None   # (what a decode step makes in one launch, side by side)
         made = self.mixer(packed, call, state, self.out.in_features)
         if self.inner:
             made = GatedColumns.step(packed, made, cols=self.inner, gate_at=self.mixer.own, at=self.mixer.out_width, kind=self.kind,
                                      limit=self.limit, dtype=self.dtype)
-        beside = {"also": as_rows(self.routed(h), rows)} if self.routed is not None else {}
+        beside = {"also": as_rows(self.routed.apply(h, *chosen), rows)} if chosen is not None else {}
         return StreamSum.step(x, as_rows(self.out(made), rows), dtype=self.dtype, **beside)
