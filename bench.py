@@ -937,6 +937,78 @@ def bench_tilarax(torch, dev, steps, widths, batch=8, prompts=(512, 2048, 1920))
             "data": "synthetic", "dtype": "bf16", "sizes": rows}
 
 
+# The heads of 128 columns that keep a fading memory at PEGILIX_SIZES' widths, and the experts of PUDINEX layers: (all, identities, chosen)
+PUDINEX_MEMORY = 128
+PUDINEX_EXPERTS = (16, 2, 4)
+
+
+def pudinex_config(width, slots=1, chunk=2048):
+    """A Pudinex of ``width``'s sizes: attention and fading memories in turn, the first feed-forward dense, the others experts and
+    a shared one, of which what a token meets (its chosen experts, none an identity) is as wide."""
+    from iron_amd.applications.pudinex import PudinexConfig
+
+    H, G, D, F, layers, vocab = PEGILIX_SIZES[width]
+    every, identity, top = PUDINEX_EXPERTS
+    experts = {"kind": "moe", "expert": {"ff": F // 2 // top}, "router": {"experts": every, "identity": identity, "top": top}, "shared": {"ff": F // 2}}
+    attention = {"type": "attention", "mlp": experts, "mixer": {
+        "heads": H, "kv_heads": G, "dim": D, "vdim": D, "scale": D**-0.5, "softcap": 30.0,
+        "rot": {"base": 10000.0, "dims": D, "scaling": {"factor": 4.0, "original": 1024, "fast": 32.0, "slow": 1.0}}}}
+    memory = {"type": "hgrn2", "mlp": experts, "mixer": {"heads": width // PUDINEX_MEMORY, "dim": PUDINEX_MEMORY, "vdim": PUDINEX_MEMORY}}
+    listed = [attention, memory] * (layers // 2)
+    listed[0] = {**attention, "mlp": {"ff": F, "kind": "dense", "limit": 7.0}}
+    return PudinexConfig(vocab_size=vocab, hidden_size=width, layers=tuple(listed), eps=1e-5, norm_groups=4, embed_scale=float(width) ** 0.5,
+                         max_seq_len=4096, prefill_chunk=chunk, slots=slots)
+
+
+def pudinex_step_bytes(config, weights, keys) -> tuple[int, int]:
+    """Bytes of weights a decode step of ``config.slots`` rows reads (of the experts, as many as that many draws among them and the
+    identities meet on average), and of states and keys a slot, ``keys`` positions in its cache."""
+    every, identity, top = PUDINEX_EXPERTS
+    met = 1 - (1 - top / (every + identity)) ** config.slots
+    read = 2 * sum(int(np.prod(t.shape)) * (met if ".mlp.e" in n else 1) for n, t in weights.items() if n != "embed")
+    state = 0
+    for spec in config.layers:
+        m = spec["mixer"]
+        state += keys * m["kv_heads"] * (m["dim"] + m["vdim"]) * 2 if spec["type"] == "attention" else 8 * m["heads"] * m["dim"] * m["vdim"]
+    return int(read), state
+
+
+def bench_pudinex(torch, dev, steps, widths, batch=8, prompts=(512, 2048, 1920)):
+    """Prompt and decode throughput of Pudinex layers at a few widths, one sequence (decode behind the last of the prompts) and a
+    batch of ``batch``, beside a Tilarax of the same width, layers, vocabulary and feed-forward a token meets; random weights, bf16."""
+    import dataclasses
+
+    from iron_amd.applications import pudinex, tilarax
+
+    rows = []
+    for width in widths:
+        row = {"width": width, "layers": PEGILIX_SIZES[width][4]}
+        for name, module, cls, config, step_bytes in (("pudinex", pudinex, pudinex.Pudinex, pudinex_config(width), pudinex_step_bytes),
+                                                      ("tilarax", tilarax, tilarax.Tilarax, tilarax_config(width), tilarax_step_bytes)):
+            weights = random_weights(torch, module.shapes(config), dev)
+            row[f"{name}_params"] = sum(int(np.prod(t.shape)) for t in weights.values())
+            for n, t in weights.items():
+                if n.endswith(".dwa"):   # mostly the layer's own result
+                    t[:-1] *= 0.05
+                elif n.endswith(".lower"):
+                    t.copy_(torch.rand_like(t, dtype=torch.float32).mul_(0.9))
+                elif n.endswith(".correction"):
+                    t.sub_(1.0).mul_(0.1)
+            for slots, lengths in ((1, prompts), (batch, (512,))):
+                if not slots:
+                    continue
+                sized = dataclasses.replace(config, slots=slots)
+                read, state = step_bytes(sized, weights, lengths[-1] if name == "pudinex" else lengths[-1] % PEGILIX_WINDOW)
+                row[name if slots == 1 else f"{name}_batch_{slots}"] = batched_served(torch, cls, sized, weights, steps, lengths, state, read)
+            del weights
+            torch.cuda.empty_cache()
+        rows.append(row)
+        print(json.dumps(row), file=sys.stderr, flush=True)
+    return {"what": "prompt (ms, tok/s) and greedy decode steps as HIP-graph replays; Pudinex attends everything before, Tilarax chunks of "
+                    f"{PEGILIX_WINDOW}; frac_hbm: weights a step meets, states and keys over the time a step takes",
+            "data": "synthetic", "dtype": "bf16", "sizes": rows}
+
+
 class _AfterPrompt:
     """A single-sequence model's captured decode step behind a prompt of ``n`` tokens."""
 
@@ -1058,9 +1130,11 @@ def main():
                     help="time only Pufuzen layers at a few widths beside a Pegilix of equal size, and exit")
     ap.add_argument("--tilarax", action="store_true",
                     help="time only Tilarax layers at a few widths beside a Pegilix of equal size, and exit")
+    ap.add_argument("--pudinex", action="store_true",
+                    help="time only Pudinex layers at a few widths beside a Tilarax of equal size, and exit")
     ap.add_argument("--widths", type=int, nargs="+", default=sorted(PEGILIX_SIZES), choices=sorted(PEGILIX_SIZES),
-                    help="the widths --pegilix, --pufuzen and --tilarax time")
-    ap.add_argument("--batch", type=int, default=8, help="sequences of --pegilix's, --pufuzen's and --tilarax's batch (0: one sequence only)")
+                    help="the widths --pegilix, --pufuzen, --tilarax and --pudinex time")
+    ap.add_argument("--batch", type=int, default=8, help="sequences of the batch of --pegilix, --pufuzen, --tilarax and --pudinex (0: one sequence only)")
     args = ap.parse_args()
     if args.gpus != 1:
         print("bench.py: this build is a one-GPU hot path; --gpus must be 1 "
@@ -1099,6 +1173,9 @@ def main():
         return 0
     if args.tilarax:
         print(json.dumps(bench_tilarax(torch, dev, args.steps, args.widths, args.batch)))
+        return 0
+    if args.pudinex:
+        print(json.dumps(bench_pudinex(torch, dev, args.steps, args.widths, args.batch)))
         return 0
     if args.prompt_probe:
         prompt_probe(torch, dev)

@@ -145,6 +145,7 @@ struct WalkShape {
   int rows, slots, heads, dim, vdim;
   int v_stride, o_stride;                // lengths of the rows v lies in (vdim columns a head) and of the readings' rows
 };
+
 template <typename T, int NT, int DEPTH, bool COUNTED = false>
 __global__ __launch_bounds__(256) void time_mix_walk_kernel(const T* __restrict__ v, float* __restrict__ state,
                                                             const int* __restrict__ spans, const float* __restrict__ work,
@@ -238,9 +239,16 @@ __global__ __launch_bounds__(256) void time_mix_walk_kernel(const T* __restrict_
 }
 
 // ---------------------------------------------------------------------- HGRN2
-// The same walk, read behind the write: queries enter as q exp(L), L with the token's own decay in it, keys are what the gates
-// leave, and the 16 x 16 matrix has its diagonal, undecayed.
+// The same walk, read behind the write: queries enter as q 2^L, L the running sum of the gates' logarithms with the token's own in it,
+// keys are what the gates leave, and the 16 x 16 matrix has its diagonal, undecayed.
 template <typename T>
+__device__ __forceinline__ float decay_exp2(float x) {
+  if constexpr (sizeof(T) == 2) return __builtin_amdgcn_exp2f(x);
+  else return exp2f(x);
+}
+
+// VEC: rows and gains of whole 16-byte pieces, eight columns of a token a thread at a time; else one.
+template <typename T, int VEC>
 __global__ __launch_bounds__(256) void hgrn2_chunks_kernel(const T* __restrict__ x, FadeGates g, const int* __restrict__ spans,
                                                            float* __restrict__ work, int rows, int slots, int stride, int heads, int dim) {
   extern __shared__ __align__(16) float lds[];
@@ -253,28 +261,42 @@ __global__ __launch_bounds__(256) void hgrn2_chunks_kernel(const T* __restrict__
   float* ls = ks + CHUNK * pitch;        // the sum up to and with token i
   float* am = ls + CHUNK * pitch;        // [16][17]
   const T* row = x + (size_t)(s.row0 + base) * stride + head * dim;
-  for (int e = t; e < CHUNK * wide; e += 256) {
-    const int i = e / wide, c = e - i * wide;
-    float q = 0.f, k = 0.f, l = 0.f;   // past the last token: nothing read or written, nothing fades
-    if (i < n && c < dim) {
-      const T* at = row + (size_t)i * stride + c;
-      const Fade f = fade_of(load_one(at + heads * dim), bf16_to_f32(g.bias[head * dim + c]), bf16_to_f32(g.lower[head * dim + c]));
-      q = silu_read(load_one(at));
-      k = f.write;
-      l = log_fade(f);
+  const int pieces = wide / VEC;
+  for (int e = t; e < CHUNK * pieces; e += 256) {
+    const int i = e / pieces, c = (e - i * pieces) * VEC;
+    float q[VEC], z[VEC], bias[VEC], lower[VEC];
+    const bool in = i < n && c < dim;
+    if (in) {
+      load_vec<VEC>(row + (size_t)i * stride + c, q);
+      load_vec<VEC>(row + (size_t)i * stride + heads * dim + c, z);
+      load_vec<VEC>(g.bias + head * dim + c, bias);
+      load_vec<VEC>(g.lower + head * dim + c, lower);
     }
-    qs[i * pitch + c] = q;
-    ks[i * pitch + c] = k;
-    ls[i * pitch + c] = l;
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) {
+      if (in) {
+        const Fade f = fade_of<T>(z[j], bias[j], lower[j]);
+        q[j] = silu_read<T>(q[j]);
+        z[j] = f.write;
+        bias[j] = log2_fade<T>(f);
+      } else {   // past the last token: nothing read or written, nothing fades
+        q[j] = z[j] = bias[j] = 0.f;
+      }
+    }
+    store_vec<VEC>(qs + i * pitch + c, q);
+    store_vec<VEC>(ks + i * pitch + c, z);
+    store_vec<VEC>(ls + i * pitch + c, bias);
   }
   for (int e = t; e < CHUNK * 17; e += 256) am[e] = 0.f;
   __syncthreads();
   for (int c = t; c < wide; c += 256) {
-    float sum = 0.f;
+    float v[CHUNK];
 #pragma unroll
-    for (int i = 0; i < CHUNK; ++i) {
-      sum += ls[i * pitch + c];
-      ls[i * pitch + c] = sum;
+    for (int i = 0; i < CHUNK; ++i) v[i] = ls[i * pitch + c];
+#pragma unroll
+    for (int i = 1; i < CHUNK; ++i) {
+      v[i] += v[i - 1];
+      ls[i * pitch + c] = v[i];
     }
   }
   __syncthreads();
@@ -285,23 +307,24 @@ __global__ __launch_bounds__(256) void hgrn2_chunks_kernel(const T* __restrict__
     const float4 q = *reinterpret_cast<const float4*>(qs + l16 * pitch + tile * 16 + quad * 4), l = *reinterpret_cast<const float4*>(ls + l16 * pitch + tile * 16 + quad * 4);
     float f[4];
 #pragma unroll
-    for (int j = 0; j < 4; ++j) f[j] = ks[(quad * 4 + j) * pitch + c] * decay_exp<T>(end[c] - ls[(quad * 4 + j) * pitch + c]);
-    reinterpret_cast<float4*>(out)[e] = make_float4(q.x * decay_exp<T>(l.x), q.y * decay_exp<T>(l.y), q.z * decay_exp<T>(l.z), q.w * decay_exp<T>(l.w));
+    for (int j = 0; j < 4; ++j) f[j] = ks[(quad * 4 + j) * pitch + c] * decay_exp2<T>(end[c] - ls[(quad * 4 + j) * pitch + c]);
+    reinterpret_cast<float4*>(out)[e] = make_float4(q.x * decay_exp2<T>(l.x), q.y * decay_exp2<T>(l.y), q.z * decay_exp2<T>(l.z), q.w * decay_exp2<T>(l.w));
     reinterpret_cast<float4*>(out + tiles * 256)[e] = make_float4(f[0], f[1], f[2], f[3]);
   }
-  for (int c = t; c < wide; c += 256) out[tiles * 512 + c] = decay_exp<T>(end[c]);
+  for (int c = t; c < wide; c += 256) out[tiles * 512 + c] = decay_exp2<T>(end[c]);
   // Pairs (i, j), j <= i: 64 at a time, four threads a pair.
   for (int p = t >> 2; p < CHUNK * (CHUNK + 1) / 2; p += 64) {
     int i = 0, j = p;
     while (j > i) j -= ++i;
     float sum = 0.f;
+#pragma unroll 2
     for (int c = (t & 3) * 4; c < wide; c += 16) {
       const float4 q = *reinterpret_cast<const float4*>(qs + i * pitch + c), k = *reinterpret_cast<const float4*>(ks + j * pitch + c);
       const float4 a = *reinterpret_cast<const float4*>(ls + i * pitch + c), b = *reinterpret_cast<const float4*>(ls + j * pitch + c);
-      sum = fmaf(q.x * k.x, decay_exp<T>(a.x - b.x), sum);
-      sum = fmaf(q.y * k.y, decay_exp<T>(a.y - b.y), sum);
-      sum = fmaf(q.z * k.z, decay_exp<T>(a.z - b.z), sum);
-      sum = fmaf(q.w * k.w, decay_exp<T>(a.w - b.w), sum);
+      sum = fmaf(q.x * k.x, decay_exp2<T>(a.x - b.x), sum);
+      sum = fmaf(q.y * k.y, decay_exp2<T>(a.y - b.y), sum);
+      sum = fmaf(q.z * k.z, decay_exp2<T>(a.z - b.z), sum);
+      sum = fmaf(q.w * k.w, decay_exp2<T>(a.w - b.w), sum);
     }
     sum += IRON_DPP(0.f, sum, 0xB1, 0xF);
     sum += IRON_DPP(0.f, sum, 0x4E, 0xF);
@@ -723,10 +746,13 @@ extern "C" int iron_hgrn2_chunked(const void* x, const uint16_t* f_bias, const u
   const dim3 all((rows + CHUNK - 1) / CHUNK, heads, slots), walk(heads, (vdim + 15) / 16, slots);
   float* work = (float*)workspace;
   const FadeGates g{f_bias, lower};
+  const bool vec = dim % 8 == 0 && stride % 8 == 0 && (((uintptr_t)x | (uintptr_t)f_bias | (uintptr_t)lower) & 15) == 0;
   const WalkShape shape{rows, slots, heads, dim, vdim, stride, heads * vdim};
-#define IRON_FADE_WALK(T, NT, DEPTH)   hipLaunchKernelGGL((time_mix_walk_kernel<T, NT, DEPTH>), walk, dim3(256), 0, s, (const T*)x + 2 * heads * dim, state, spans, work, o, shape)
+#define IRON_FADE_WALK(T, NT, DEPTH) \
+  hipLaunchKernelGGL((time_mix_walk_kernel<T, NT, DEPTH>), walk, dim3(256), 0, s, (const T*)x + 2 * heads * dim, state, spans, work, o, shape)
 #define IRON_FADE(T)                                                                                                                        \
-  hipLaunchKernelGGL((hgrn2_chunks_kernel<T>), all, dim3(256), lds, s, (const T*)x, g, spans, work, rows, slots, stride, heads, dim);      \
+  if (vec) hipLaunchKernelGGL((hgrn2_chunks_kernel<T, 8>), all, dim3(256), lds, s, (const T*)x, g, spans, work, rows, slots, stride, heads, dim); \
+  else hipLaunchKernelGGL((hgrn2_chunks_kernel<T, 1>), all, dim3(256), lds, s, (const T*)x, g, spans, work, rows, slots, stride, heads, dim); \
   if (tiles <= 4) IRON_FADE_WALK(T, 1, 6);                                                                                                  \
   else if (tiles <= 8) IRON_FADE_WALK(T, 2, 4);                                                                                             \
   else IRON_FADE_WALK(T, 4, 2);

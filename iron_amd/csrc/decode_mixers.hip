@@ -552,8 +552,8 @@ __global__ __launch_bounds__(DM_THREADS) void decode_hgrn2_kernel(FadeStep a, co
   const float gain = t < vdim ? bf16_to_f32(a.norm[t]) : 0.f;
   if (t < dim) {
     const int c = head * dim + t;
-    const Fade f = fade_of(bf16_to_f32(row[a.heads * dim + c]), bf16_to_f32(a.g.bias[c]), bf16_to_f32(a.g.lower[c]));
-    sh.q[t] = silu_read(bf16_to_f32(row[c]));
+    const Fade f = fade_of<bf16_t>(bf16_to_f32(row[a.heads * dim + c]), bf16_to_f32(a.g.bias[c]), bf16_to_f32(a.g.lower[c]));
+    sh.q[t] = silu_read<bf16_t>(bf16_to_f32(row[c]));
     sh.keep[t] = f.keep;
     sh.write[t] = f.write;
   } else if (t >= 512 && t < 512 + vdim) {

@@ -21,19 +21,33 @@ __global__ __launch_bounds__(NW * 64) void router_kernel(const T* __restrict__ h
   const int row = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   if (row >= bound_or(valid, rows)) return;
   const T* hr = h + (size_t)row * cols;
-  for (int e = wave; e < experts; e += NW) {
-    const bf16_t* wr = w + (size_t)e * cols;
-    float sum = 0.f;
+  constexpr int AT_ONCE = NW >= 16 ? 2 : 4;   // experts whose weights meet a piece of the row
+  for (int e0 = wave; e0 < experts; e0 += NW * AT_ONCE) {
+    float sum[AT_ONCE];
+    const bf16_t* wr[AT_ONCE];
+#pragma unroll
+    for (int k = 0; k < AT_ONCE; ++k) {
+      sum[k] = 0.f;
+      wr[k] = w + (size_t)min(e0 + k * NW, experts - 1) * cols;
+    }
 #pragma unroll 4
     for (int c = lane * VEC; c < cols; c += 64 * VEC) {
-      float a[VEC], b[VEC];
+      float a[VEC];
       load_vec<VEC>(hr + c, a);
-      load_vec<VEC>(wr + c, b);
 #pragma unroll
-      for (int j = 0; j < VEC; ++j) sum = fmaf(a[j], b[j], sum);
+      for (int k = 0; k < AT_ONCE; ++k) {
+        float b[VEC];
+        load_vec<VEC>(wr[k] + c, b);
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) sum[k] = fmaf(a[j], b[j], sum[k]);
+      }
     }
-    sum = wave_sum(sum);
-    if (lane == 0) z[e] = sum + (bias != nullptr ? bf16_to_f32(bias[e]) : 0.f);
+#pragma unroll
+    for (int k = 0; k < AT_ONCE; ++k) {
+      const float total = wave_sum(sum[k]);
+      const int e = e0 + k * NW;
+      if (lane == 0 && e < experts) z[e] = total + (bias != nullptr ? bf16_to_f32(bias[e]) : 0.f);
+    }
   }
   __syncthreads();
   if (wave != 0) return;
@@ -422,10 +436,17 @@ extern "C" int iron_experts_tail_bf16(const uint16_t* h, const uint16_t* gate, c
                      activation, nullptr);
 #define IRON_TAIL(CH) \
   hipLaunchKernelGGL((expert_tail_kernel<CH>), dim3(cols), dim3(256), 0, s, out, made, inner, down, acts, ids, shares, h, stream_row, cols, ff, experts, identity, top)
-  if (pieces <= 512) IRON_TAIL(2);
-  else if (pieces <= 1024) IRON_TAIL(4);
-  else if (pieces <= 2048) IRON_TAIL(8);
-  else IRON_TAIL(16);
+  switch ((pieces + 255) / 256) {
+    case 1: case 2: IRON_TAIL(2); break;
+    case 3: IRON_TAIL(3); break;
+    case 4: IRON_TAIL(4); break;
+    case 5: IRON_TAIL(5); break;
+    case 6: IRON_TAIL(6); break;
+    case 7: case 8: IRON_TAIL(8); break;
+    case 9: case 10: IRON_TAIL(10); break;
+    case 11: case 12: IRON_TAIL(12); break;
+    default: IRON_TAIL(16);
+  }
 #undef IRON_TAIL
   IRON_LAUNCH_CHECK();
 }

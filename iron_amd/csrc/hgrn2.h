@@ -14,13 +14,25 @@ struct FadeGates {
 struct Fade {
   float keep, write;
 };
+// (T: the rows' type; the hardware's exponential, reciprocal and logarithm, an ulp or two off, where they are bf16)
+template <typename T>
+__device__ __forceinline__ float logistic(float z) {
+  if constexpr (sizeof(T) == 2) return __builtin_amdgcn_rcpf(1.f + __expf(-z));
+  else return 1.f / (1.f + expf(-z));
+}
+template <typename T>
 __device__ __forceinline__ Fade fade_of(float z, float bias, float lower) {
   z += bias;
   const float rest = 1.f - lower;
-  return Fade{lower + rest / (1.f + expf(-z)), rest / (1.f + expf(z))};
+  return Fade{lower + rest * logistic<T>(z), rest * logistic<T>(-z)};
 }
-// log f, finite: a gate that has closed altogether counts as one that is as good as closed.
-__device__ __forceinline__ float log_fade(const Fade& f) { return f.keep > 0.5f ? log1pf(-f.write) : logf(fmaxf(f.keep, 1e-37f)); }
-__device__ __forceinline__ float silu_read(float q) { return q / (1.f + expf(-q)); }
+// log2 f, finite: a gate that has closed altogether counts as one that is as good as closed.
+template <typename T>
+__device__ __forceinline__ float log2_fade(const Fade& f) {
+  if constexpr (sizeof(T) == 2) return __builtin_amdgcn_logf(fmaxf(f.keep, 1e-37f));
+  else return f.keep > 0.5f ? log1pf(-f.write) * 1.4426950408889634f : log2f(fmaxf(f.keep, 1e-37f));
+}
+template <typename T>
+__device__ __forceinline__ float silu_read(float q) { return q * logistic<T>(q); }
 
 }  // namespace iron

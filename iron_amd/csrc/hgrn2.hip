@@ -50,8 +50,8 @@ __global__ __launch_bounds__(256) void hgrn2_kernel(const T* __restrict__ x, Fad
     for (int e = 0; e < NI; ++e) {
       const int i = ig * NI + e;
       const bool in = i < dim && base + tok < s.rows;   // past the last row: the state stays
-      const Fade f = fade_of(zn[e], bias[e], lower[e]);
-      qs[tok][i] = silu_read(qn[e]);
+      const Fade f = fade_of<T>(zn[e], bias[e], lower[e]);
+      qs[tok][i] = silu_read<T>(qn[e]);
       fs[tok][i] = in ? f.keep : 1.f;
       ws[tok][i] = in ? f.write : 0.f;
     }
