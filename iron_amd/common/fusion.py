@@ -479,7 +479,7 @@ def plan(recording, tensor: Callable[[Any], Any], word: Callable[[Any], Any],
     def stream_end(j):
         """``(product, sum)`` where step ``j`` is one row's product and the next adds it to the stream -- or None."""
         g, add = steps[j : j + 2] if j + 1 < len(steps) else (None, None)
-        if not (g is not None and gemv_row(g) and g.op.K % 8 == 0 and g.op.K <= 16384 and _name(add) == "StreamSum" and add.op.rows == 1
+        if not (g is not None and gemv_row(g) and g.op.K % 8 == 0 and g.op.K <= 32768 and _name(add) == "StreamSum" and add.op.rows == 1
                 and add.op.dtype is bfloat16 and bare(add) and _same(add.inputs["y"], g.outputs["C"]) and once(g.outputs["C"])):
             return None
         return g, add

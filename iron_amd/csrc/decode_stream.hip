@@ -307,6 +307,9 @@ static int launch_stream_product(const bf16_t* W, const StreamIn& in, const Stre
   if (ch == 2 && MADE) IRON_PRODUCT(4, 2)
   if (ch == 2) IRON_PRODUCT(2, 2)
   if (ch == 4) IRON_PRODUCT(4, 4)
+  if constexpr (OUT == OUT_ADD) {
+    if (K > 8 * 2048) IRON_PRODUCT(1, 16)
+  }
   IRON_PRODUCT(2, 8)
 #undef IRON_PRODUCT
 }
@@ -368,7 +371,7 @@ extern "C" int iron_norm_product_bf16(const float* x, const uint16_t* gain, int 
 
 extern "C" int iron_product_sum_bf16(const uint16_t* x, const uint16_t* W, int M, int K, const uint16_t* also, float* stream_row, void* stream) {
   IRON_REQUIRE(x && W && stream_row, "product_sum: null operand");
-  IRON_REQUIRE(M > 0 && K > 0 && K % 8 == 0 && K <= 8 * 2048, "product_sum: M (%d) positive, K (%d) a multiple of 8 up to %d", M, K, 8 * 2048);
+  IRON_REQUIRE(M > 0 && K > 0 && K % 8 == 0 && K <= 16 * 2048, "product_sum: M (%d) positive, K (%d) a multiple of 8 up to %d", M, K, 16 * 2048);
   IRON_REQUIRE((((uintptr_t)x | (uintptr_t)W) & 15) == 0, "product_sum: operands must be 16-byte aligned");
   const StreamIn in{x, nullptr, nullptr, nullptr, nullptr, nullptr, 0.f, 0.f, 1, nullptr};
   StreamOut out{};

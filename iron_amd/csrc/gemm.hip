@@ -361,6 +361,17 @@ __device__ __forceinline__ void tile_of_block(int bid, int tiles_m, int tiles_n,
   }
 }
 
+// The same under a row bound read on the device: an order that is not patched is that of the live tile rows alone, or the few
+// there are would be a few XCDs'.  False: the block has none.
+__device__ __forceinline__ bool live_tile(int bid, int tiles_m, int tiles_n, int patched, int live_m, int& tm, int& tn) {
+  if (!patched) {
+    tiles_m = min(tiles_m, live_m);
+    if (bid >= tiles_m * tiles_n) return false;
+  }
+  tile_of_block(bid, tiles_m, tiles_n, patched, tm, tn);
+  return true;
+}
+
 // 64 x 64 tiles, B as (N,K), for problems -- or row bounds -- whose 128 x 128 tiles would leave CUs
 // idle (k/v projections, short chunks): the direct-to-LDS pipeline of the 128 x 128 kernel below
 // (buffer loads, XOR-swizzled chunks) with a wave owning one 32x32x16 MFMA tile.  A stage is four
@@ -388,7 +399,7 @@ __device__ __forceinline__ void gemm_nt64_body(const bf16_t* __restrict__ A, con
   const int Mv = bound_or(valid, M);
 
   int tm, tn;
-  tile_of_block(blockIdx.x, tiles_m, tiles_n, patched, tm, tn);
+  if (!live_tile(blockIdx.x, tiles_m, tiles_n, patched, (Mv + NT_BM - 1) / NT_BM, tm, tn)) return;
   const int m0 = tm * NT_BM, n0 = tn * NT_BN;
   if (m0 >= Mv) return;
 
@@ -558,12 +569,12 @@ __device__ __forceinline__ void gemm_nt16_body(const bf16_t* __restrict__ A, con
   const int Mv = bound_or(valid, M);
 
   int tm, tn;
-  tile_of_block(blockIdx.x, tiles_m, tiles_n, patched, tm, tn);
-  if constexpr (!QKV) {
-    if (qkv.tile_plus1 > 0) {
-      tm = (qkv.tile_plus1 - 1) / tiles_n;
-      tn = (qkv.tile_plus1 - 1) % tiles_n;
-    }
+  const bool given = !QKV && qkv.tile_plus1 > 0;
+  if (given) {
+    tm = (qkv.tile_plus1 - 1) / tiles_n;
+    tn = (qkv.tile_plus1 - 1) % tiles_n;
+  } else if (!live_tile(blockIdx.x, tiles_m, tiles_n, patched, (Mv + NT_BM - 1) / NT_BM, tm, tn)) {
+    return;
   }
   const int m0 = tm * NT_BM;
   if (m0 >= Mv) return;
@@ -1330,7 +1341,7 @@ __device__ __forceinline__ void gemm_nt256_body(const bf16_t* __restrict__ A, co
   const int Mv = bound_or(valid, M);
 
   int tm, tn;
-  tile_of_block(blockIdx.x, tiles_m, tiles_n, patched, tm, tn);
+  if (!live_tile(blockIdx.x, tiles_m, tiles_n, patched, (Mv + BIG_BM - 1) / BIG_BM, tm, tn)) return;
   const int m0 = tm * BIG_BM, n0 = tn * BIG_BN;
   if (m0 >= Mv) return;
 
@@ -1827,7 +1838,9 @@ __device__ __forceinline__ void gemm_nt16_pair_body(const bf16_t* __restrict__ A
   const int Mv = bound_or(valid, M);
 
   int tm = tiles_m, tn = tiles_n;
-  if constexpr (!GROUPED) tile_of_block(blockIdx.x, tiles_m, tiles_n, patched, tm, tn);
+  if constexpr (!GROUPED) {
+    if (!live_tile(blockIdx.x, tiles_m, tiles_n, patched, (Mv + NT_BM - 1) / NT_BM, tm, tn)) return;
+  }
   const int m0 = tm * NT_BM;
   if (m0 >= Mv) return;
   const int n0 = tn * NT_BN;

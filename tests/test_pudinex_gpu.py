@@ -96,7 +96,7 @@ def test_a_normed_row_s_product_and_logits(cuda, K_, M, groups, logits):
 
 
 @pytest.mark.parametrize("two", [False, True])
-@pytest.mark.parametrize("K_,M", [(384, 100), (2048, 2049), (10240, 33), (16384, 7)])
+@pytest.mark.parametrize("K_,M", [(384, 100), (2048, 2049), (10240, 33), (16384, 7), (18432, 50), (32768, 3)])
 def test_a_product_joins_the_stream(cuda, K_, M, two):
     rng = np.random.default_rng(M)
     x, W, stream, also = bf(rng, K_), bf(rng, M, K_, scale=K_**-0.5), rng.standard_normal(M).astype(F32), bf(rng, M)
