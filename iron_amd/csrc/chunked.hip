@@ -193,24 +193,44 @@ __global__ __launch_bounds__(256) void time_mix_walk_kernel(const T* __restrict_
       else x.v[j] = __builtin_bit_cast(float, __builtin_amdgcn_raw_buffer_load_b32(vb, v_at + j * row_v, c * CHUNK * row_v, 0));
     }
   };
+  // A chunk's sums of the four waves' parts: asked for ahead of the next chunk's products, and used behind them.
+  float part[4];
+  auto ask = [&](int c) {   // wave w finishes rows quad * 4 + w
+#pragma unroll
+    for (int w = 0; w < 4; ++w) part[w] = reinterpret_cast<const float*>(&os[c & 1][w][lane])[wave];
+  };
+  auto finish = [&](int c) {
+    const float sum = part[0] + part[1] + part[2] + part[3];
+    __builtin_amdgcn_raw_buffer_store_b32(__builtin_bit_cast(unsigned, sum), ob, o_at, c * CHUNK * a.o_stride * 4, 0);
+  };
   auto run = [&](const MixOperands<T, NT>& x, int c) {
-    f32x4 vf, out = f32x4{0.f, 0.f, 0.f, 0.f};
+    if (c > 0) ask(c - 1);
+    f32x4 vf, next[NT], out[2] = {f32x4{0.f, 0.f, 0.f, 0.f}, f32x4{0.f, 0.f, 0.f, 0.f}};
 #pragma unroll
     for (int j = 0; j < 4; ++j) vf[j] = COUNTED && col == vdim ? 1.f : widened(x.v[j]);
+    float r[NT][4], k[NT][4];
 #pragma unroll
     for (int n = 0; n < NT; ++n) {
-      out = product16(f32x4{x.r[n].x, x.r[n].y, x.r[n].z, x.r[n].w}, S[n], out);   // S of a tile past the last stays 0
-      S[n] *= f32x4{x.w[n].x, x.w[n].y, x.w[n].z, x.w[n].w};
-      const bool in = wave * NT + n < tiles;
-      S[n] = product16(f32x4{in ? x.k[n].x : 0.f, in ? x.k[n].y : 0.f, in ? x.k[n].z : 0.f, in ? x.k[n].w : 0.f}, vf, S[n]);
+      const bool in = wave * NT + n < tiles;   // S of a tile past the last stays 0
+      r[n][0] = x.r[n].x; r[n][1] = x.r[n].y; r[n][2] = x.r[n].z; r[n][3] = x.r[n].w;
+      k[n][0] = in ? x.k[n].x : 0.f; k[n][1] = in ? x.k[n].y : 0.f; k[n][2] = in ? x.k[n].z : 0.f; k[n][3] = in ? x.k[n].w : 0.f;
+      next[n] = S[n] * f32x4{x.w[n].x, x.w[n].y, x.w[n].z, x.w[n].w};
     }
-    out = mfma4(x.a, pick4(vf, wave), out);
-    os[c & 1][wave][lane] = make_float4(out[0], out[1], out[2], out[3]);
-    block_barrier_lds();
-    float sum = 0.f;   // wave w finishes rows quad * 4 + w
+    out[1] = mfma4(x.a, pick4(vf, wave), out[1]);
+    // Chains side by side: a product waits for the one before it in its own chain, not for its neighbours.
 #pragma unroll
-    for (int w = 0; w < 4; ++w) sum += reinterpret_cast<const float*>(&os[c & 1][w][lane])[wave];
-    __builtin_amdgcn_raw_buffer_store_b32(__builtin_bit_cast(unsigned, sum), ob, o_at, c * CHUNK * a.o_stride * 4, 0);
+    for (int j = 0; j < 4; ++j)
+#pragma unroll
+      for (int n = 0; n < NT; ++n) {
+        out[n & 1] = mfma4(r[n][j], S[n][j], out[n & 1]);
+        next[n] = mfma4(k[n][j], vf[j], next[n]);
+      }
+#pragma unroll
+    for (int n = 0; n < NT; ++n) S[n] = next[n];
+    const f32x4 both = out[0] + out[1];
+    if (c > 0) finish(c - 1);
+    os[c & 1][wave][lane] = make_float4(both[0], both[1], both[2], both[3]);
+    block_barrier_lds();   // (the other buffer's readers are behind it, too)
   };
 #pragma unroll
   for (int d = 0; d < DEPTH; ++d) {
@@ -229,6 +249,8 @@ __global__ __launch_bounds__(256) void time_mix_walk_kernel(const T* __restrict_
 #pragma unroll
   for (int d = 0; d < DEPTH; ++d)
     if (c + d < count) run(ops[d], c + d);
+  ask(count - 1);
+  finish(count - 1);
 #pragma unroll
   for (int n = 0; n < NT; ++n)
 #pragma unroll
