@@ -44,6 +44,21 @@ __device__ __forceinline__ void choose(float* __restrict__ z, int n, int top, in
 __device__ __forceinline__ void choose_scored(float* __restrict__ z, float* __restrict__ by, const bf16_t* __restrict__ correction, int n, int top,
                                               int* __restrict__ ids, float* __restrict__ shares) {
   const int lane = threadIdx.x & 63;
+  if (n <= 64) {   // a logit a lane
+    const float logit = lane < n ? z[lane] : -INFINITY, e = expf(logit - wave_max(logit)), score = e / wave_sum(e);
+    float key = lane < n ? score + (correction != nullptr ? bf16_to_f32(correction[lane]) : 0.f) : -INFINITY, sum = 0.f, mine = 0.f;
+    for (int k = 0; k < top; ++k) {
+      const unsigned long long here = __builtin_amdgcn_ballot_w64(key == wave_max(key) && key > -INFINITY);
+      const int id = here != 0 ? __builtin_ctzll(here) : 0;   // (none that is a number: the first)
+      const float chosen = __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, score), id));
+      sum += chosen;
+      if (lane == k) mine = chosen;
+      if (lane == 0) ids[k] = id;
+      if (lane == id) key = -INFINITY;
+    }
+    if (lane < top) shares[lane] = mine / (sum + 1e-20f);
+    return;
+  }
   float most = -INFINITY, total = 0.f;
   for (int i = lane; i < n; i += 64) most = fmaxf(most, z[i]);
   most = wave_max(most);

@@ -15,7 +15,7 @@ from iron_amd.lm import Sampler, rope_angles, write_safetensors
 from iron_amd.lm.batched import BatchedOnHost, Entry
 from iron_amd.lm.config import yarn
 from tests.pudinex_plain import clamped_gate, frequencies, group_norm, hgrn2, over_rms, routed, sigmoid, silu, sunk_weights, turned
-from tests.pudinex_support import MODELS, Plain, attention, built, dense, document, experts, far_off, memory, weights_of
+from tests.pudinex_support import MODELS, Plain, attention, built, dense, document, far_off, memory, weights_of
 
 oracle.install()
 
